@@ -14,7 +14,10 @@ CSRC = os.path.join(HERE, "csrc")
 LIBDIR = os.path.join(HERE, "lib")
 LIB = os.path.join(LIBDIR, "libchatts_amd.so")
 SOURCES = ["api.hip", "ts_frontend.hip", "gemv.hip", "gemm.hip", "gemm_ring.hip", "gemm_f16q.hip", "gemm_fp8.hip", "elementwise.hip", "sampler.hip", "attention.hip", "tp.hip", "decoder.hip"]
-FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function"]
+# no packed float32 instructions (v_pk_add / mul / fma_f32): the compiler forms them from ordinary float code and some of their forms
+# have given wrong results on this hardware
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", *NO_PACKED_FP32]
 # per-file extra flags (none at the moment)
 EXTRA_FLAGS = {}
 
@@ -42,7 +45,7 @@ def _digest():
 # options table, error strings, geometry choices, handle bookkeeping - everything the C-ABI does before a kernel is enqueued.  GPU ASan
 # needs xnack+ code objects, which this pool refuses; -fno-gpu-sanitize keeps the device code as shipped.
 ASAN_FLAGS = ["--offload-arch=gfx950", "-O1", "-g", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-fsanitize=address",
-              "-fno-gpu-sanitize", "-shared-libsan", "-fno-omit-frame-pointer"]
+              "-fno-gpu-sanitize", "-shared-libsan", "-fno-omit-frame-pointer", *NO_PACKED_FP32]
 ASAN_LIBDIR = os.path.join(HERE, "lib_asan")
 ASAN_LIB = os.path.join(ASAN_LIBDIR, "libchatts_amd_asan.so")
 
