@@ -10,7 +10,7 @@ from . import build as _build
 _LIB = None
 
 OK, E_BADARG, E_SHAPE, E_COUNT_MISMATCH, E_LAUNCH, E_WORKSPACE = 0, -1, -2, -3, -4, -5
-EPI_NONE, EPI_GELU, EPI_RESID, EPI_SWIGLU = 0, 1, 2, 3
+EPI_NONE, EPI_GELU, EPI_RESID, EPI_SWIGLU, EPI_RELU2 = 0, 1, 2, 3, 4
 
 c_void_p, c_int, c_int32, c_int64, c_float, c_size_t, c_uint32 = (
     C.c_void_p, C.c_int, C.c_int32, C.c_int64, C.c_float, C.c_size_t, C.c_uint32)
@@ -29,7 +29,7 @@ class TsWeights(C.Structure):
                 ("b", c_void_p * 8)]
 
 
-ABI_VERSION = 9            # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
+ABI_VERSION = 10           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
 W8_FP8, W8_INT8 = 0, 1     # ChattsLinearArgs.w8_format
 
 
@@ -42,7 +42,7 @@ class LinearArgs(C.Structure):
                 ("c_hi", c_void_p), ("c_lo", c_void_p), ("ld_cplanes", c_int),
                 ("post_norm_w", c_void_p), ("post_norm_eps", c_float), ("post_hi", c_void_p), ("post_lo", c_void_p), ("ld_post", c_int),
                 ("w4", c_void_p), ("w4_sz", c_void_p), ("ldw4", c_int), ("w4_group", c_int),
-                ("w8_format", c_int), ("tp_reduce", c_void_p), ("w_tiled", c_void_p), ("planes_tiled", c_int)]
+                ("w8_format", c_int), ("tp_reduce", c_void_p), ("w_tiled", c_void_p), ("planes_tiled", c_int), ("exact_f32", c_int)]
 
 
 class LinearFp8Args(C.Structure):
@@ -110,6 +110,64 @@ class DecoderBuffers(C.Structure):
                 ("planes_hi", c_void_p), ("planes_lo", c_void_p), ("planes2_hi", c_void_p), ("planes2_lo", c_void_p),
                 ("tp_pair_logit", c_void_p), ("tp_pair_token", c_void_p), ("logits_full", c_void_p),
                 ("kv_block_table", c_void_p), ("kv_block_size", c_int), ("kv_table_stride", c_int), ("kv_pool_blocks", c_int)]
+
+
+class Operand(C.Structure):
+    _fields_ = [("f32", c_void_p), ("hi", c_void_p), ("lo", c_void_p), ("ld", c_int)]
+
+
+class ResidualNormArgs(C.Structure):
+    _fields_ = [("x", c_void_p), ("y", c_void_p), ("post_w", c_void_p), ("add", c_void_p), ("pre_w", c_void_p), ("out", Operand),
+                ("t", c_int), ("width", c_int), ("ldx", c_int), ("ldy", c_int), ("eps", c_float)]
+
+
+class HeadLinearArgs(C.Structure):
+    _fields_ = [("a", c_void_p), ("w", c_void_p), ("out", Operand)] + [(n, c_int) for n in ("m", "heads", "n", "k", "lda", "a_head", "out_head", "exact")]
+
+
+class DeltaArgs(C.Structure):
+    """ChattsDeltaArgs: gated delta rule with a decay per head and key channel (csrc/delta.hip)"""
+    _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_a", "off_g", "off_b", "conv_ch", "heads",
+                                                             "kv_heads", "dim", "vdim", "taps", "rank_a", "rank_g")] +
+                [("conv_w", c_void_p), ("a2", c_void_p), ("g2", c_void_p), ("ld_a2", c_int), ("ld_g2", c_int), ("dt_bias", c_void_p),
+                 ("neg_a", c_void_p), ("norm_w", c_void_p), ("eps", c_float), ("state", c_void_p), ("ring", c_void_p), ("rows", c_void_p),
+                 ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int)] +
+                [(n, c_void_p) for n in ("q", "k", "v", "g", "gate", "beta", "o", "dt")] + [("ld_dt", c_int), ("ld_gate", c_int), ("out", Operand)])
+
+
+class LatentArgs(C.Structure):
+    """ChattsLatentArgs: attention over a paged latent cache (csrc/latent.hip)"""
+    _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_qr", "off_c", "off_kr", "heads", "dim", "rot", "rank", "vdim",
+                                                             "rank_p", "rot_p")] +
+                [("scale", c_float), ("eps", c_float), ("c_norm", c_void_p), ("cos_tab", c_void_p), ("sin_tab", c_void_p), ("cache", c_void_p),
+                 ("cache_f32", c_int), ("table", c_void_p), ("table_stride", c_int), ("log_block", c_int), ("rows", c_void_p), ("n_rows", c_int),
+                 ("q", Operand), ("o", c_void_p), ("n_splits", c_int), ("partial", c_void_p)])
+
+
+MIX_LATENT, MIX_DELTA = 1, 2
+
+
+class MixLayer(C.Structure):
+    _fields_ = ([("kind", c_int)] + [(n, c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "in_t", "out", "out_t", "up", "up_t", "down",
+                                                             "down_t")] +
+                [(n, c_int) for n in ("in_n", "out_k", "ff")] + [("uk", c_void_p), ("uv", c_void_p)] +
+                [(n, c_int) for n in ("dim_p", "vdim_p", "out_head", "dt_n", "gate_n")] + [("latent", LatentArgs), ("delta", DeltaArgs)])
+
+
+class MixRun(C.Structure):
+    _fields_ = [("layer", c_int), ("add", c_void_p), ("cache", c_void_p), ("state", c_void_p), ("ring", c_void_p)]
+
+
+class MixConfig(C.Structure):
+    _fields_ = ([(n, c_int) for n in ("width", "width_p", "n_layers", "n_runs", "exact", "t_max", "max_slots", "max_ctx")] +
+                [("vocab", c_int64), ("vocab_p", c_int64), ("eps", c_float), ("block_size", c_int), ("table_stride", c_int)])
+
+
+class MixBuffers(C.Structure):
+    _fields_ = ([(n, c_void_p) for n in ("embed", "head", "head_t", "final_norm", "x", "y", "proj", "a_f32", "b_f32", "a_hi", "a_lo", "b_hi", "b_lo",
+                                         "q_f32", "o_lat", "partial", "q_hi", "q_lo")] + [("partial_elems", c_size_t)] +
+                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dout", "ddt", "rows", "spans", "table", "logits", "workspace")] +
+                [("workspace_bytes", c_size_t)])
 
 
 # name -> (restype, argtypes); this table IS the list of symbols include/chatts_amd.h declares
@@ -192,6 +250,21 @@ SIGNATURES = {
     "chatts_decoder_set_tp": (c_int, [c_void_p, c_void_p]),
     "chatts_decoder_select_tokens": (c_int, [c_void_p, c_void_p, c_int, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                                              c_void_p, c_int, C.POINTER(SamplingArgs), c_void_p]),
+    # mixed-layer decoders (delta.hip, latent.hip, mixdec.hip)
+    "chatts_residual_norm": (c_int, [C.POINTER(ResidualNormArgs), c_void_p]),
+    "chatts_head_linear": (c_int, [C.POINTER(HeadLinearArgs), c_void_p]),
+    "chatts_delta_decode": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
+    "chatts_delta_prep": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
+    "chatts_delta_scan": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
+    "chatts_delta_out": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
+    "chatts_latent_prep": (c_int, [C.POINTER(LatentArgs), c_void_p]),
+    "chatts_latent_attend": (c_int, [C.POINTER(LatentArgs), c_void_p]),
+    "chatts_mixdec_create": (c_void_p, [C.POINTER(MixConfig), C.POINTER(MixLayer), C.POINTER(MixRun), C.POINTER(MixBuffers)]),
+    "chatts_mixdec_destroy": (None, [c_void_p]),
+    "chatts_mixdec_workspace": (c_size_t, [C.POINTER(MixConfig), C.POINTER(MixLayer)]),
+    "chatts_mixdec_forward": (c_int, [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
+    "chatts_mixdec_logits": (c_int, [c_void_p, c_void_p, c_int, c_void_p, c_void_p]),
+    "chatts_mixdec_decode": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
     # tensor-parallel exchange (tp.hip)
     "chatts_tp_buffer_bytes": (c_size_t, [c_int, c_int64]),
     "chatts_tp_buffer_bytes_bulk": (c_size_t, [c_int, c_int64, c_int64]),

@@ -154,6 +154,36 @@ struct RopeFuse {
 // `row` = this head's 128 floats of the qkv buffer (q is written back there)
 __device__ __forceinline__ void rope_kv_head(float a, float b, int h, int pos, int lane, float* row, const RopeFuse& r);
 
+// ---- the operand of a following projection: float32 and / or bf16 hi / lo planes (ChattsOperand) ----
+__device__ __forceinline__ void store_operand(const ChattsOperand& o, size_t row, int col, float v) {
+#pragma clang fp contract(off)      // lo is the split of the ROUNDED float32 value
+  const size_t at = row * o.ld + col;
+  if (o.f32) o.f32[at] = v;
+  if (o.hi) {
+    const __bf16 h = (__bf16)v;
+    o.hi[at] = __builtin_bit_cast(uint16_t, h);
+    if (o.lo) o.lo[at] = __builtin_bit_cast(uint16_t, (__bf16)(v - (float)h));
+  }
+}
+__device__ __forceinline__ void store_operand4(const ChattsOperand& o, size_t row, int col, const float (&v)[4]) {
+#pragma clang fp contract(off)
+  typedef __bf16 bf16x4_t __attribute__((ext_vector_type(4)));
+  const size_t at = row * o.ld + col;
+  if (o.f32) *reinterpret_cast<f32x4*>(o.f32 + at) = (f32x4){v[0], v[1], v[2], v[3]};
+  if (o.hi) {
+    bf16x4_t hv, lv;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const __bf16 h = (__bf16)v[j];
+      hv[j] = h;
+      lv[j] = (__bf16)(v[j] - (float)h);
+    }
+    *reinterpret_cast<bf16x4_t*>(o.hi + at) = hv;
+    if (o.lo) *reinterpret_cast<bf16x4_t*>(o.lo + at) = lv;
+  }
+}
+__device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
+
 inline hipStream_t as_stream(chatts_stream_t s) { return reinterpret_cast<hipStream_t>(s); }
 
 // ---- stage ranges for traces (api.hip): roctx push / pop around the host-side enqueue of a stage, resolved with dlopen at first use

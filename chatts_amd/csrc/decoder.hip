@@ -11,6 +11,7 @@
 
 namespace chatts {
 int launch_gemv(const ChattsLinearArgs* a, hipStream_t s);
+int launch_gemm_f32(const ChattsLinearArgs* a, hipStream_t s);
 int launch_gemm(const ChattsLinearArgs* a, hipStream_t s, const RopeFuse* rope = nullptr, bool* rope_done = nullptr);
 int attention_decode_batched_impl(const float* qkv_raw, int batch, int n_q, int n_kv, const float* q_norm_w, const float* k_norm_w,
                                   float norm_eps, const float* cos_tab, const float* sin_tab, int pos, const int32_t* pos_dev,
@@ -69,7 +70,7 @@ static int linear_impl(const ChattsLinearArgs* a, chatts_stream_t stream, const 
     CHATTS_REQUIRE(a->a_hi && a->a_lo && a->ld_planes >= a->k && a->ld_planes % 8 == 0 && ((uintptr_t)a->a_hi % 16) == 0 &&
                        ((uintptr_t)a->a_lo % 16) == 0 && a->m > 1 && !a->norm_w,
                    CHATTS_E_SHAPE, "linear: pre-split A needs both planes, ld_planes >= K and %% 8, 16-byte alignment, M > 1");
-  CHATTS_REQUIRE(a->epilogue >= CHATTS_EPI_NONE && a->epilogue <= CHATTS_EPI_SWIGLU, CHATTS_E_BADARG,
+  CHATTS_REQUIRE(a->epilogue >= CHATTS_EPI_NONE && a->epilogue <= CHATTS_EPI_RELU2, CHATTS_E_BADARG,
                  "linear: epilogue %d", a->epilogue);
   CHATTS_REQUIRE(a->epilogue != CHATTS_EPI_RESID || a->resid, CHATTS_E_BADARG, "linear: EPI_RESID without resid");
   CHATTS_REQUIRE(a->k % 32 == 0, CHATTS_E_SHAPE, "linear: K=%d must be a multiple of 32 (pad the weight)", a->k);
@@ -93,7 +94,12 @@ static int linear_impl(const ChattsLinearArgs* a, chatts_stream_t stream, const 
                        (a->epilogue == CHATTS_EPI_NONE || a->epilogue == CHATTS_EPI_RESID) && !cplanes,
                    CHATTS_E_BADARG, "linear: post-norm planes need M > 1, float32 c, EPI_NONE / EPI_RESID, both planes, ld_post >= N");
   if (a->tp_reduce) CHATTS_REQUIRE(a->m == 1, CHATTS_E_BADARG, "linear: tp_reduce is available for M == 1 (the decode GEMV) only");
-  if (a->m == 1 && a->epilogue != CHATTS_EPI_GELU) return launch_gemv(a, as_stream(stream));
+  if (a->m == 1 && a->epilogue != CHATTS_EPI_GELU) return launch_gemv(a, as_stream(stream));      // (products and sums in float32 already)
+  if (a->exact_f32) {
+    CHATTS_REQUIRE(a->a && a->c && !cplanes && !a->post_norm_w && !a->norm_w && !a->w8, CHATTS_E_BADARG,
+                   "linear: exact_f32 takes a float32 A and C and bf16 weights, without fused norms or planes");
+    return launch_gemm_f32(a, as_stream(stream));
+  }
   CHATTS_REQUIRE(a->norm_w == nullptr, CHATTS_E_BADARG, "linear: fused RMSNorm is only available for M == 1");
   return launch_gemm(a, as_stream(stream), rope, rope_done);
 }

@@ -1,0 +1,405 @@
+// delta.hip - the gated delta rule with a decay per head and key channel, with its short convolutions, norms and gates.
+//   S <- g * S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q          S [dim, vdim] per head, float32
+// Kernels:
+//  * delta_decode_kernel: one token per sequence, everything of a (sequence, head) in one workgroup: convolutions from the ring of
+//    earlier inputs, unit norms, the low-rank decay and gate products, the state update (state in registers between its two passes) and the
+//    normed, gated read-out.  One launch instead of five, the state is read and written once.
+//  * delta_prep_kernel / delta_scan_kernel / delta_out_kernel: several tokens per sequence.  prep does what is parallel over tokens; scan
+//    walks the tokens with the state in registers - a column of S belongs to 16 lanes of a wave, so the two sums over key channels are
+//    DPP row reductions and columns never talk to each other; out norms and gates.
+// The ring of convolution inputs is indexed by position modulo taps: the current token's entry is never one that the same step reads, so
+// heads that share a q / k head need no ordering, and a sequence that starts over in a used slot reads none of the old entries.
+#include "common.h"
+
+namespace chatts {
+
+__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+
+// ---- one token per sequence -----------------------------------------------------------------------------------------------------
+// thread (tx, ty): 4 consecutive value columns tx * 4, key rows ty + TY * r.
+template <int NT, int NR>
+__global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int TX) {
+  extern __shared__ float sm[];
+  const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
+  const int pos = p.rows[row].pos, slot = p.rows[row].slot;
+  if (pos < 0) return;
+  const int dim = p.dim, vdim = p.vdim, v4 = (vdim + 3) & ~3;
+  const int group = p.heads / p.kv_heads, hk = h / group;
+  float* red = sm;                      // NT * 4
+  float* su = red + NT * 4;             // (red and su are read as float4)
+  float* sv = su + v4;
+  float* sgate = sv + v4;
+  float* sq = sgate + v4;
+  float* sk = sq + dim;
+  float* sg = sk + dim;
+  float* sa = sg + dim;
+  float* sgi = sa + p.rank_a;
+  float* scratch = sgi + p.rank_g;      // NT / 64
+  const int tx = tid & (TX - 1), ty = tid / TX, TY = NT / TX;
+  const bool live = tx * 4 < v4;
+  float* S = p.state + ((size_t)slot * p.heads + h) * dim * v4;
+  const int stride = TY * v4;
+  float* Sp = S + (size_t)ty * v4 + tx * 4;
+  f32x4 s[NR];
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    s[r] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    if (pos > 0 && live && ty + TY * r < dim) s[r] = *reinterpret_cast<const f32x4*>(Sp + (size_t)r * stride);
+  }
+  const float* pr = p.proj + (size_t)row * p.ld_proj;
+  float* ring = p.ring + (size_t)slot * p.taps * p.conv_ch;
+  for (int i = tid; i < 2 * dim + vdim; i += NT) {
+    int ch;
+    bool owner = true;
+    if (i < dim) { ch = p.off_q + hk * dim + i; owner = h == hk * group; }
+    else if (i < 2 * dim) { ch = p.off_k + hk * dim + i - dim; owner = h == hk * group; }
+    else ch = p.off_v + h * vdim + i - 2 * dim;
+    const float cur = pr[ch];
+    float acc = 0.f;
+    for (int j = 0; j < p.taps - 1; ++j) {
+      const int q = pos - (p.taps - 1 - j);
+      if (q >= 0) acc += p.conv_w[(size_t)j * p.conv_ch + ch] * ring[(size_t)(q % p.taps) * p.conv_ch + ch];
+    }
+    acc += p.conv_w[(size_t)(p.taps - 1) * p.conv_ch + ch] * cur;
+    if (owner) ring[(size_t)(pos % p.taps) * p.conv_ch + ch] = cur;
+    acc *= sigmoid_f(acc);
+    if (i < dim) sq[i] = acc;
+    else if (i < 2 * dim) sk[i - dim] = acc;
+    else sv[i - 2 * dim] = acc;
+  }
+  for (int i = tid; i < p.rank_a; i += NT) sa[i] = pr[p.off_a + i];
+  for (int i = tid; i < p.rank_g; i += NT) sgi[i] = pr[p.off_g + i];
+  __syncthreads();
+  float qs = 0.f, ks = 0.f;      // every wave forms both norms
+  for (int i = tid & 63; i < dim; i += 64) { qs += sq[i] * sq[i]; ks += sk[i] * sk[i]; }
+  qs = wave_sum(qs);
+  ks = wave_sum(ks);
+  const float qn = rsqrtf((float)dim) / sqrtf(qs + 1e-6f), kn = 1.0f / sqrtf(ks + 1e-6f);
+  const float na = p.neg_a[h];
+  for (int i = tid; i < dim + vdim; i += NT) {
+    const bool dec = i < dim;
+    const int o = dec ? h * dim + i : h * vdim + i - dim;
+    const uint16_t* w = dec ? p.a2 + (size_t)o * p.ld_a2 : p.g2 + (size_t)o * p.ld_g2;
+    const float* x = dec ? sa : sgi;
+    const int rank = dec ? p.rank_a : p.rank_g;
+    float acc = 0.f;
+    for (int c = 0; c < rank; c += 8) {
+      const u32x4 wv = *reinterpret_cast<const u32x4*>(w + c);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        acc += bf16_lo(wv[j]) * x[c + 2 * j];
+        acc += bf16_hi(wv[j]) * x[c + 2 * j + 1];
+      }
+    }
+    if (dec) sg[i] = expf(na * softplus_f(acc + p.dt_bias[o]));
+    else sgate[i - dim] = sigmoid_f(acc);
+  }
+  const float beta = sigmoid_f(pr[p.off_b + h]);
+  __syncthreads();
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    const int i = ty + TY * r;
+    if (i < dim) {
+      const float g = sg[i], k = sk[i] * kn;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { s[r][j] *= g; acc[j] += s[r][j] * k; }
+    }
+  }
+  *reinterpret_cast<f32x4*>(red + tid * 4) = acc;
+  __syncthreads();
+  for (int j = tid; j < v4; j += NT) {
+    float t = 0.f;
+    for (int y = 0; y < TY; ++y) t += red[(y * TX + (j >> 2)) * 4 + (j & 3)];
+    su[j] = j < vdim ? beta * (sv[j] - t) : 0.f;
+  }
+  __syncthreads();
+  acc = (f32x4){0.f, 0.f, 0.f, 0.f};
+  if (live) {
+    const f32x4 u = *reinterpret_cast<const f32x4*>(su + tx * 4);
+#pragma unroll
+    for (int r = 0; r < NR; ++r) {
+      const int i = ty + TY * r;
+      if (i < dim) {
+        const float k = sk[i] * kn, q = sq[i] * qn;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { s[r][j] += k * u[j]; acc[j] += s[r][j] * q; }
+        *reinterpret_cast<f32x4*>(Sp + (size_t)r * stride) = s[r];
+      }
+    }
+  }
+  *reinterpret_cast<f32x4*>(red + tid * 4) = acc;
+  __syncthreads();
+  float o = 0.f;
+  if (tid < vdim)
+    for (int y = 0; y < TY; ++y) o += red[(y * TX + (tid >> 2)) * 4 + (tid & 3)];
+  const float ss = block_sum<NT / 64>(tid < vdim ? o * o : 0.f, scratch);
+  if (tid < vdim)
+    store_operand(p.out, row, h * vdim + tid, o * (1.0f / sqrtf(ss / (float)vdim + p.eps)) * p.norm_w[tid] * sgate[tid]);
+}
+
+// ---- several tokens: what is parallel over tokens -------------------------------------------------------------------------------
+// convolution + silu of channel ch of row r; earlier tokens come from the segment's own rows or from the ring
+__device__ __forceinline__ float conv_silu(const ChattsDeltaArgs& p, int row, const ChattsRow& R, int ch) {
+  float acc = 0.f;
+  const float* ring = p.ring + (size_t)R.slot * p.taps * p.conv_ch;
+  for (int j = 0; j < p.taps; ++j) {
+    const int lag = p.taps - 1 - j, q = R.pos - lag;
+    if (q < 0) continue;
+    const float x = row - lag >= R.first ? p.proj[(size_t)(row - lag) * p.ld_proj + ch] : ring[(size_t)(q % p.taps) * p.conv_ch + ch];
+    acc += p.conv_w[(size_t)j * p.conv_ch + ch] * x;
+  }
+  return acc * sigmoid_f(acc);
+}
+
+// a wave takes one item of a row at a time: a q or k head, 64 channels of v, 64 decays
+__global__ __launch_bounds__(256) void delta_prep_kernel(ChattsDeltaArgs p) {
+  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = blockIdx.y * 4 + (threadIdx.x >> 6), waves = gridDim.y * 4;
+  const ChattsRow R = p.rows[row];
+  if (R.pos < 0) return;
+  const int dim = p.dim, nv = p.heads * p.vdim, ng = p.heads * dim;
+  const int vchunks = (nv + 63) / 64, gchunks = (ng + 63) / 64, bchunks = (p.heads + 63) / 64;
+  const int items = 2 * p.kv_heads + vchunks + gchunks + bchunks;
+  for (int it = wave; it < items; it += waves) {
+    int e = it;
+    if (e < 2 * p.kv_heads) {
+      const bool isq = e < p.kv_heads;
+      const int hk = isq ? e : e - p.kv_heads, base = (isq ? p.off_q : p.off_k) + hk * dim;
+      float v[4], ss = 0.f;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        const int i = c * 64 + lane;
+        v[c] = i < dim ? conv_silu(p, row, R, base + i) : 0.f;
+        ss += v[c] * v[c];
+      }
+      ss = wave_sum(ss);
+      const float f = (isq ? rsqrtf((float)dim) : 1.0f) / sqrtf(ss + 1e-6f);
+      float* dst = (isq ? p.q : p.k) + ((size_t)row * p.kv_heads + hk) * dim;
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        if (c * 64 + lane < dim) dst[c * 64 + lane] = v[c] * f;
+      continue;
+    }
+    e -= 2 * p.kv_heads;
+    if (e < vchunks) {
+      const int i = e * 64 + lane;
+      if (i < nv) p.v[(size_t)row * nv + i] = conv_silu(p, row, R, p.off_v + i);
+      continue;
+    }
+    e -= vchunks;
+    if (e < gchunks) {
+      const int i = e * 64 + lane;
+      if (i < ng) p.g[(size_t)row * ng + i] = expf(p.neg_a[i / dim] * softplus_f(p.dt[(size_t)row * p.ld_dt + i] + p.dt_bias[i]));
+      continue;
+    }
+    e -= gchunks;
+    const int i = e * 64 + lane;
+    if (i < p.heads) p.beta[(size_t)row * p.heads + i] = sigmoid_f(p.proj[(size_t)row * p.ld_proj + p.off_b + i]);
+  }
+}
+
+// ---- the recurrence over a span: grid (heads * column blocks, spans), 4 waves x 4 columns ---------------------------------------------
+// Lane l of a row of 16 holds key channels (c * 16 + l) * 4 .. + 3 (c < NC) of its column.
+template <int NC>
+__global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int colblocks) {
+  constexpr int D = NC * 64, kScanT = NC <= 2 ? 16 : 8;      // tokens staged together
+  __shared__ __attribute__((aligned(16))) float sk[2][kScanT][D], sq[2][kScanT][D], sg[2][kScanT][D];
+  __shared__ float sv[2][kScanT][16], so[kScanT][16], sb[2][kScanT];
+  const ChattsSpan sp = p.spans[blockIdx.y];
+  if (sp.t < 1) return;
+  const int h = blockIdx.x / colblocks, cb = blockIdx.x - h * colblocks, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int dim = p.dim, vdim = p.vdim, v4 = (vdim + 3) & ~3, hk = h / (p.heads / p.kv_heads);
+  const int l16 = lane & 15, cl = wave * 4 + (lane >> 4), col = cb * 16 + cl;
+  const bool live = col < vdim;
+  float* S = p.state + ((size_t)sp.slot * p.heads + h) * dim * v4;
+  float s[NC][4];
+#pragma unroll
+  for (int c = 0; c < NC; ++c)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = (c * 16 + l16) * 4 + j;
+      s[c][j] = sp.pos0 > 0 && live && i < dim ? S[(size_t)i * v4 + col] : 0.f;
+    }
+  const int qrow = p.kv_heads * dim, grow = p.heads * dim, vrow = p.heads * vdim;
+  constexpr int PER = kScanT * D / 256;      // values of one of k / q / g per thread and stage
+  float rk[PER], rq[PER], rg[PER], rv, rb;
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int e = 0; e < PER; ++e) {
+      const int at = e * 256 + tid, t = t0 + at / D, i = at % D;
+      const bool ok = t < sp.t && i < dim;
+      const size_t r = sp.row0 + t;
+      rk[e] = ok ? p.k[r * qrow + hk * dim + i] : 0.f;
+      rq[e] = ok ? p.q[r * qrow + hk * dim + i] : 0.f;
+      rg[e] = ok ? p.g[r * grow + h * dim + i] : 1.f;
+    }
+    const int t = t0 + (tid >> 4), c = cb * 16 + (tid & 15);
+    rv = tid < kScanT * 16 && t < sp.t && c < vdim ? p.v[(size_t)(sp.row0 + t) * vrow + h * vdim + c] : 0.f;
+    rb = tid < kScanT && t0 + tid < sp.t ? p.beta[(size_t)(sp.row0 + t0 + tid) * p.heads + h] : 0.f;
+  };
+  auto stage = [&](int b) {
+#pragma unroll
+    for (int e = 0; e < PER; ++e) {
+      const int at = e * 256 + tid, t = at / D, i = at % D;
+      sk[b][t][i] = rk[e];
+      sq[b][t][i] = rq[e];
+      sg[b][t][i] = rg[e];
+    }
+    if (tid < kScanT * 16) sv[b][tid >> 4][tid & 15] = rv;
+    if (tid < kScanT) sb[b][tid] = rb;
+  };
+  fetch(0);
+  stage(0);
+  __syncthreads();
+  int b = 0;
+  for (int t0 = 0; t0 < sp.t; t0 += kScanT, b ^= 1) {
+    if (t0 + kScanT < sp.t) fetch(t0 + kScanT);
+    const int n = sp.t - t0 < kScanT ? sp.t - t0 : kScanT;
+    for (int t = 0; t < n; ++t) {
+      f32x4 k[NC], q[NC], g[NC];
+#pragma unroll
+      for (int c = 0; c < NC; ++c) {
+        const int i = (c * 16 + l16) * 4;
+        k[c] = *reinterpret_cast<const f32x4*>(&sk[b][t][i]);
+        g[c] = *reinterpret_cast<const f32x4*>(&sg[b][t][i]);
+        q[c] = *reinterpret_cast<const f32x4*>(&sq[b][t][i]);
+      }
+      const float beta = sb[b][t], v = sv[b][t][cl];
+      float d0 = 0.f, d1 = 0.f;
+#pragma unroll
+      for (int c = 0; c < NC; ++c) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s[c][j] *= g[c][j];
+        d0 += s[c][0] * k[c][0]; d1 += s[c][1] * k[c][1];
+        d0 += s[c][2] * k[c][2]; d1 += s[c][3] * k[c][3];
+      }
+      const float u = beta * (v - row16_sum(d0 + d1));
+      float o0 = 0.f, o1 = 0.f;
+#pragma unroll
+      for (int c = 0; c < NC; ++c) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s[c][j] += k[c][j] * u;
+        o0 += s[c][0] * q[c][0]; o1 += s[c][1] * q[c][1];
+        o0 += s[c][2] * q[c][2]; o1 += s[c][3] * q[c][3];
+      }
+      const float o = row16_sum(o0 + o1);
+      if (l16 == 0) so[t][cl] = o;
+    }
+    if (t0 + kScanT < sp.t) stage(b ^ 1);
+    __syncthreads();
+    const int t = tid >> 4, c = cb * 16 + (tid & 15);
+    if (t < n && c < vdim) p.o[(size_t)(sp.row0 + t0 + t) * vrow + h * vdim + c] = so[t][tid & 15];
+    __syncthreads();
+  }
+  if (live)
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int i = (c * 16 + l16) * 4 + j;
+        if (i < dim) S[(size_t)i * v4 + col] = s[c][j];
+      }
+}
+
+// ---- norm + gate of the read-outs; the last `taps` rows of a span enter the ring (prep has read the old entries by now) -----------
+__global__ __launch_bounds__(256) void delta_out_kernel(ChattsDeltaArgs p) {
+  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = blockIdx.y * 4 + (threadIdx.x >> 6), waves = gridDim.y * 4;
+  const ChattsRow R = p.rows[row];
+  if (R.pos < 0) return;
+  const int vdim = p.vdim, vrow = p.heads * vdim;
+  for (int h = wave; h < p.heads; h += waves) {
+    float v[4], ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int i = c * 64 + lane;
+      v[c] = i < vdim ? p.o[(size_t)row * vrow + h * vdim + i] : 0.f;
+      ss += v[c] * v[c];
+    }
+    ss = wave_sum(ss);
+    const float f = 1.0f / sqrtf(ss / (float)vdim + p.eps);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int i = c * 64 + lane;
+      if (i < vdim) store_operand(p.out, row, h * vdim + i, v[c] * f * p.norm_w[i] * sigmoid_f(p.gate[(size_t)row * p.ld_gate + h * vdim + i]));
+    }
+  }
+  if (R.rest < p.taps) {
+    float* ring = p.ring + ((size_t)R.slot * p.taps + R.pos % p.taps) * p.conv_ch;
+    for (int i = blockIdx.y * 256 + threadIdx.x; i < p.conv_ch; i += gridDim.y * 256) ring[i] = p.proj[(size_t)row * p.ld_proj + i];
+  }
+}
+
+static int check_delta(const ChattsDeltaArgs* a, const char* who) {
+  CHATTS_REQUIRE(a && a->proj && a->rows && a->state && a->ring && a->conv_w && a->dt_bias && a->neg_a && a->norm_w, CHATTS_E_BADARG, "%s: null pointer", who);
+  CHATTS_REQUIRE(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->taps >= 1, CHATTS_E_SHAPE, "%s: heads %d / %d, taps %d", who,
+                 a->heads, a->kv_heads, a->taps);
+  CHATTS_REQUIRE(a->dim >= 1 && a->dim <= 256 && a->vdim >= 1 && a->vdim <= 256, CHATTS_E_SHAPE, "%s: head sizes %d x %d (at most 256 x 256)", who,
+                 a->dim, a->vdim);
+  CHATTS_REQUIRE(a->rank_a % 8 == 0 && a->rank_g % 8 == 0 && a->ld_a2 % 8 == 0 && a->ld_g2 % 8 == 0, CHATTS_E_SHAPE, "%s: ranks must be multiples of 8", who);
+  CHATTS_REQUIRE(a->ld_proj % 4 == 0 && a->conv_ch <= a->ld_proj && a->off_v + a->heads * a->vdim <= a->conv_ch &&
+                     a->off_q + a->kv_heads * a->dim <= a->conv_ch && a->off_k + a->kv_heads * a->dim <= a->conv_ch, CHATTS_E_SHAPE, "%s: column blocks", who);
+  return CHATTS_OK;
+}
+
+}  // namespace chatts
+
+using namespace chatts;
+
+extern "C" int chatts_delta_decode(const ChattsDeltaArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_delta(a, "delta_decode")) return rc;
+  CHATTS_REQUIRE(a->a2 && a->g2 && (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim, CHATTS_E_BADARG, "delta_decode: null pointer");
+  if (a->n_rows == 0) return CHATTS_OK;
+  const int v4 = (a->vdim + 3) & ~3;
+  int TX = 1;
+  while (TX * 4 < v4) TX *= 2;
+  auto rows_for = [&](int nt) { return (a->dim + nt / TX - 1) / (nt / TX); };
+  const int nt = rows_for(256) > 32 ? 512 : 256, nr = rows_for(nt);
+  const size_t lds = (size_t)(3 * a->dim + 3 * v4 + a->rank_a + a->rank_g + nt * 4 + 16 + 16) * sizeof(float);
+  CHATTS_REQUIRE(lds <= 64 * 1024, CHATTS_E_SHAPE, "delta_decode: ranks %d / %d too large", a->rank_a, a->rank_g);
+  const dim3 g(a->heads, a->n_rows);
+  hipStream_t s = as_stream(stream);
+  if (nt == 512) hipLaunchKernelGGL((delta_decode_kernel<512, 32>), g, dim3(512), lds, s, *a, TX);
+  else if (nr <= 4) hipLaunchKernelGGL((delta_decode_kernel<256, 4>), g, dim3(256), lds, s, *a, TX);
+  else if (nr <= 8) hipLaunchKernelGGL((delta_decode_kernel<256, 8>), g, dim3(256), lds, s, *a, TX);
+  else if (nr <= 16) hipLaunchKernelGGL((delta_decode_kernel<256, 16>), g, dim3(256), lds, s, *a, TX);
+  else hipLaunchKernelGGL((delta_decode_kernel<256, 32>), g, dim3(256), lds, s, *a, TX);
+  CHATTS_CHECK_LAUNCH("delta_decode");
+  return CHATTS_OK;
+}
+
+extern "C" int chatts_delta_prep(const ChattsDeltaArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_delta(a, "delta_prep")) return rc;
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->dt, CHATTS_E_BADARG, "delta_prep: null scratch");
+  if (a->n_rows == 0) return CHATTS_OK;
+  const int items = 2 * a->kv_heads + (a->heads * a->vdim + 63) / 64 + (a->heads * a->dim + 63) / 64 + 1;
+  const int y = (items + 15) / 16;
+  hipLaunchKernelGGL(delta_prep_kernel, dim3(a->n_rows, y), dim3(256), 0, as_stream(stream), *a);
+  CHATTS_CHECK_LAUNCH("delta_prep");
+  return CHATTS_OK;
+}
+
+extern "C" int chatts_delta_scan(const ChattsDeltaArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_delta(a, "delta_scan")) return rc;
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->o && a->spans, CHATTS_E_BADARG, "delta_scan: null scratch");
+  if (a->n_spans == 0) return CHATTS_OK;
+  const int cb = (a->vdim + 15) / 16;
+  const dim3 g(a->heads * cb, a->n_spans), b(256);
+  hipStream_t s = as_stream(stream);
+  switch ((a->dim + 63) / 64) {
+    case 1: hipLaunchKernelGGL(delta_scan_kernel<1>, g, b, 0, s, *a, cb); break;
+    case 2: hipLaunchKernelGGL(delta_scan_kernel<2>, g, b, 0, s, *a, cb); break;
+    case 3: hipLaunchKernelGGL(delta_scan_kernel<3>, g, b, 0, s, *a, cb); break;
+    default: hipLaunchKernelGGL(delta_scan_kernel<4>, g, b, 0, s, *a, cb); break;
+  }
+  CHATTS_CHECK_LAUNCH("delta_scan");
+  return CHATTS_OK;
+}
+
+extern "C" int chatts_delta_out(const ChattsDeltaArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_delta(a, "delta_out")) return rc;
+  CHATTS_REQUIRE(a->o && a->gate && (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim, CHATTS_E_BADARG, "delta_out: null pointer");
+  if (a->n_rows == 0) return CHATTS_OK;
+  hipLaunchKernelGGL(delta_out_kernel, dim3(a->n_rows, (a->heads + 15) / 16), dim3(256), 0, as_stream(stream), *a);
+  CHATTS_CHECK_LAUNCH("delta_out");
+  return CHATTS_OK;
+}

@@ -46,6 +46,80 @@ __global__ __launch_bounds__(256) void rmsnorm_kernel(const float* __restrict__ 
   }
 }
 
+// ---- residual update of a sublayer with a norm after it, and the norm before the next one, in one pass over the row ----
+//   x += y / rms(y) * post_w   (post_w NULL: x += y; y NULL: x unchanged);  x += add;  out = x / rms(x) * pre_w
+// Rows are `width` wide inside padded rows; the padding of x and out is written as zero.  A thread keeps its columns in registers.
+template <int NV>
+__global__ __launch_bounds__(256) void residual_norm_kernel(ChattsResidualNormArgs p, int padded) {
+  __shared__ float red[4];
+  const size_t row = blockIdx.x;
+  f32x4 xv[NV];
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 4;
+    xv[i] = c < padded ? *reinterpret_cast<const f32x4*>(p.x + row * p.ldx + c) : zero;
+  }
+  if (p.y) {
+    f32x4 yv[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (i * 256 + threadIdx.x) * 4;
+      yv[i] = c < padded ? *reinterpret_cast<const f32x4*>(p.y + row * p.ldy + c) : zero;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) if (c + j < p.width) ss += yv[i][j] * yv[i][j];
+    }
+    if (p.post_w) {
+      ss = block_sum<4>(ss, red);
+      const float r = 1.0f / sqrtf(ss / (float)p.width + p.eps);
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (i * 256 + threadIdx.x) * 4;
+        if (c < padded) {
+          const f32x4 w = *reinterpret_cast<const f32x4*>(p.post_w + c);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) yv[i][j] = yv[i][j] * r * w[j];
+        }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) xv[i][j] += yv[i][j];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 4;
+    if (c >= padded) continue;
+    if (p.add) {
+      const f32x4 a = *reinterpret_cast<const f32x4*>(p.add + c);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) xv[i][j] += a[j];
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (c + j >= p.width) xv[i][j] = 0.f;
+      ss += xv[i][j] * xv[i][j];
+    }
+    if (p.y || p.add) *reinterpret_cast<f32x4*>(p.x + row * p.ldx + c) = xv[i];
+  }
+  if (!p.pre_w) return;
+  ss = block_sum<4>(ss, red);
+  const float r = 1.0f / sqrtf(ss / (float)p.width + p.eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 4;
+    if (c >= padded) continue;
+    const f32x4 w = *reinterpret_cast<const f32x4*>(p.pre_w + c);
+    float v[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = c + j < p.width ? xv[i][j] * r * w[j] : 0.f;
+    store_operand4(p.out, row, c, v);
+  }
+}
+
 // ---- RoPE + KV write: one wave per (token, head); lane l owns dims (l, l+64) = a rotate-half pair ----
 // q/k heads: optional RMSNorm over the 128 dims (Qwen3 q_norm/k_norm), then
 //   out[l]    = x[l]    * cos[l] - x[l+64] * sin[l]
@@ -412,5 +486,33 @@ extern "C" int chatts_residual_add(float* x, const float* delta, int64_t n, chat
   if (blocks > 2048) blocks = 2048;
   hipLaunchKernelGGL(residual_add_kernel, dim3((unsigned)blocks), dim3(256), 0, as_stream(stream), x, delta, n / 4);
   CHATTS_CHECK_LAUNCH("residual_add");
+  return CHATTS_OK;
+}
+
+extern "C" int chatts_residual_norm(const ChattsResidualNormArgs* a, chatts_stream_t stream) {
+  CHATTS_REQUIRE(a && a->x && a->t >= 0 && a->width > 0, CHATTS_E_BADARG, "residual_norm: bad arguments");
+  if (a->t == 0) return CHATTS_OK;
+  const int padded = (a->width + 3) / 4 * 4;
+  CHATTS_REQUIRE(a->ldx >= padded && a->ldx % 4 == 0 && (!a->y || (a->ldy >= padded && a->ldy % 4 == 0)), CHATTS_E_SHAPE,
+                 "residual_norm: row strides %d / %d for a width of %d", a->ldx, a->ldy, a->width);
+  CHATTS_REQUIRE(!a->pre_w || ((a->out.f32 || a->out.hi) && a->out.ld >= padded && a->out.ld % 4 == 0), CHATTS_E_BADARG, "residual_norm: no output");
+  CHATTS_REQUIRE((((uintptr_t)a->x | (uintptr_t)a->y | (uintptr_t)a->post_w | (uintptr_t)a->add | (uintptr_t)a->pre_w | (uintptr_t)a->out.f32) % 16) == 0 &&
+                     (((uintptr_t)a->out.hi | (uintptr_t)a->out.lo) % 8) == 0, CHATTS_E_SHAPE, "residual_norm: pointers must be aligned (16 bytes, planes 8)");
+  // the weights are read in fours: their buffers are padded to the row stride of x
+  int pad = a->ldx;
+  if (a->y && a->ldy < pad) pad = a->ldy;
+  if (a->pre_w && a->out.ld < pad) pad = a->out.ld;
+  const int lim = (a->width + 63) / 64 * 64;
+  if (pad > lim) pad = lim;
+  const dim3 g(a->t), b(256);
+  hipStream_t s = as_stream(stream);
+  if (pad <= 1024) hipLaunchKernelGGL(residual_norm_kernel<1>, g, b, 0, s, *a, pad);
+  else if (pad <= 4096) hipLaunchKernelGGL(residual_norm_kernel<4>, g, b, 0, s, *a, pad);
+  else if (pad <= 8192) hipLaunchKernelGGL(residual_norm_kernel<8>, g, b, 0, s, *a, pad);
+  else {
+    CHATTS_REQUIRE(pad <= 16384, CHATTS_E_SHAPE, "residual_norm: width %d > 16384", a->width);
+    hipLaunchKernelGGL(residual_norm_kernel<16>, g, b, 0, s, *a, pad);
+  }
+  CHATTS_CHECK_LAUNCH("residual_norm");
   return CHATTS_OK;
 }

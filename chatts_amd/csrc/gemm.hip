@@ -90,6 +90,7 @@ __device__ __forceinline__ void gemm_store(const GemmParams& p, const f32x4 (&ac
         if (row >= p.m) continue;
         float v = acc[i][j][r] * sc + b;
         if (p.epilogue == CHATTS_EPI_GELU) v = gelu_erf_f(v);
+        if (p.epilogue == CHATTS_EPI_RELU2) v = relu2_f(v);
         if (p.epilogue == CHATTS_EPI_RESID) v = p.resid[(size_t)row * p.ldc + col] + v;
         if (p.c_hi) store_planes(p.c_hi, p.c_lo, (size_t)row * p.ldcp + col, v);
         else p.c[(size_t)row * p.ldc + col] = v;
@@ -494,6 +495,7 @@ __global__ __launch_bounds__(256) void splitk_epilogue_kernel(const float* __res
   if (scale) v *= scale[col];
   if (bias) v += bias[col];
   if (epilogue == CHATTS_EPI_GELU) v = gelu_erf_f(v);
+  if (epilogue == CHATTS_EPI_RELU2) v = relu2_f(v);
   if (epilogue == CHATTS_EPI_RESID) v = resid[(size_t)row * ldc + col] + v;
   if (c_hi) store_planes(c_hi, c_lo, (size_t)row * ldcp + col, v);
   else c[(size_t)row * ldc + col] = v;
@@ -528,6 +530,7 @@ __global__ __launch_bounds__(256) void splitk_epilogue_v4_kernel(const float* __
     if (scale) v[j] *= sc[j];
     if (bias) v[j] += bb[j];
     if (epilogue == CHATTS_EPI_GELU) v[j] = gelu_erf_f(v[j]);
+    if (epilogue == CHATTS_EPI_RELU2) v[j] = relu2_f(v[j]);
     if (epilogue == CHATTS_EPI_RESID) v[j] = rr[j] + v[j];
   }
   if (c_hi) {

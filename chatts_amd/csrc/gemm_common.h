@@ -37,6 +37,7 @@ __device__ __forceinline__ void store_planes(uint16_t* hi, uint16_t* lo, size_t 
 }
 
 __device__ __forceinline__ float gelu_erf_f(float x) { return 0.5f * x * (1.0f + erff(x * 0.70710678118654752440f)); }
+__device__ __forceinline__ float relu2_f(float x) { const float r = fmaxf(x, 0.f); return r * r; }      // the square of relu
 __device__ __forceinline__ float silu_g(float x) { return x / (1.0f + expf(-x)); }
 
 constexpr int kRingPanel = 256;      // W rows per panel of the prefill kernel

@@ -21,7 +21,7 @@ namespace chatts {
 
 // EPI_RESID of a row-parallel projection under tensor parallelism (ChattsLinearArgs.tp_reduce): the sum over the ranks is formed
 // inside the launch.  Internal template value, not part of the C-ABI's epilogue enum.
-constexpr int kEpiResidTp = 4;
+constexpr int kEpiResidTp = 16;
 
 struct GemvParams {
   const uint16_t* w;
@@ -120,6 +120,7 @@ __device__ __forceinline__ void gemv_epilogue(const GemvParams& p, int task, int
         float v = acc[r];
         if (p.bias) v += p.bias[row];
         if (EPI == CHATTS_EPI_RESID) v = p.resid[row] + v;
+        if (EPI == CHATTS_EPI_RELU2) { v = fmaxf(v, 0.f); v *= v; }
         p.out[row] = v;
       }
     }
@@ -577,6 +578,7 @@ static void launch_ldsx(const GemvParams& p, int epi, bool norm, int blocks, int
     case CHATTS_EPI_RESID: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_RESID>(p, norm, blocks, threads, lds, s); break;
     case kEpiResidTp: hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, kEpiResidTp, false>), dim3(blocks), dim3(threads), lds, s, p); break;
     case CHATTS_EPI_SWIGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_SWIGLU>(p, norm, blocks, threads, lds, s); break;
+    case CHATTS_EPI_RELU2: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_RELU2>(p, norm, blocks, threads, lds, s); break;
     default: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_NONE>(p, norm, blocks, threads, lds, s); break;
   }
 }
@@ -673,6 +675,7 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
                    (long long)tp_capacity(a->tp_reduce));
     epilogue = kEpiResidTp;
   }
+  CHATTS_REQUIRE(a->epilogue != CHATTS_EPI_RELU2 || (!a->w4 && !a->w8), CHATTS_E_BADARG, "gemv: EPI_RELU2 takes bf16 weights");
   const int swiglu = a->epilogue == CHATTS_EPI_SWIGLU;
   const int units = swiglu ? a->n / 2 : a->n;
   const int nchunks = (a->k + 511) / 512;
@@ -787,6 +790,10 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
         case CHATTS_EPI_SWIGLU:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_SWIGLU, true>), g, b, lds, s, p);
           else hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_SWIGLU, false>), g, b, lds, s, p);
+          break;
+        case CHATTS_EPI_RELU2:
+          if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_RELU2, true>), g, b, lds, s, p);
+          else hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_RELU2, false>), g, b, lds, s, p);
           break;
         default:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_NONE, true>), g, b, lds, s, p);

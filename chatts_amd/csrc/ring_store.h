@@ -6,7 +6,7 @@
 namespace chatts {
 
 // modes of the branch-free epilogue (selected once per unit)
-enum { kStRaw = 0, kStNone, kStGelu, kStResid, kStSwiglu };
+enum { kStRaw = 0, kStNone, kStGelu, kStResid, kStSwiglu, kStRelu2 };
 
 __device__ __forceinline__ void ring_wait_vmcnt(int n) {      // wave-uniform n: at most n of this wave's loads outstanding
 #define CHATTS_VM(N) case N: asm volatile("s_waitcnt vmcnt(" #N ")" ::: "memory"); break;
@@ -126,6 +126,7 @@ __device__ __forceinline__ void ring_store(const GemmParams& p, const f32x4 (&ac
           for (int r = 0; r < 4; ++r) {
             v[r] = acc[i][j][r] + b4[j][r];
             if constexpr (MODE == kStGelu) v[r] = gelu_erf_f(v[r]);
+            if constexpr (MODE == kStRelu2) v[r] = relu2_f(v[r]);
             if constexpr (MODE == kStResid) v[r] = rs[j][r] + v[r];
           }
           if (tok < p.m && fb < p.n) put((size_t)tok * p.ldc, (size_t)tok * p.ldcp, fb, v);

@@ -107,6 +107,10 @@ class Engine:
 
     def _encode(self, r):
         import torch
+        if isinstance(r.prompt, (list, tuple)):         # token ids
+            if r.timeseries:
+                raise ValueError("time series need a text prompt")
+            return [int(t) for t in r.prompt], None, []
         text, encs, lens = self.processor.splice(r.prompt, [np.asarray(s, dtype=np.float64) for s in r.timeseries])
         ids = self.processor.tokenizer.encode(text)
         ser = torch.from_numpy(self.processor.pad_stack(encs)) if encs else None

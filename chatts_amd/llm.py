@@ -31,7 +31,7 @@ class RequestOutput:
         self.prompt, self.prompt_token_ids, self.outputs = prompt, prompt_token_ids, outputs
 
 
-def _load_checkpoint_tokenizer(path):
+def _load_checkpoint_tokenizer(path, required=True):
     """The HF tokenizer stored in a checkpoint directory (demo/demo_vllm.py builds prompts with it).  A directory written
     by ChatTSConfig.save_pretrained for the synthetic-weight tests marks itself with `synthetic_tokenizer` in config.json."""
     import json
@@ -39,6 +39,8 @@ def _load_checkpoint_tokenizer(path):
         if json.load(f).get("synthetic_tokenizer"):
             return None
     has_files = any(os.path.exists(os.path.join(path, f)) for f in ("tokenizer.json", "vocab.json", "tokenizer.model"))
+    if not has_files and not required:
+        return None
     if not has_files:
         raise ValueError(f"{path} holds no tokenizer files (tokenizer.json / vocab.json): pass tokenizer=... explicitly; "
                          "the synthetic stand-in tokenizer would feed meaningless ids to real weights")
@@ -54,10 +56,10 @@ def _build_llm(model, kw):
 class LLM:
     def __init__(self, model, tensor_parallel_size=1, max_model_len=6000, limit_mm_per_prompt=None,
                  trust_remote_code=True, gpu_memory_utilization=None, seed=0, tokenizer=None, comm=None,
-                 max_num_seqs=1, block_size=None, num_gpu_blocks_override=None, **kw):
-        from .config import PRESETS, ChatTSConfig, preset
-        from .modeling import ChatTSForCausalLM
-        from .processing import ChatTSProcessor
+                 max_num_seqs=1, block_size=None, num_gpu_blocks_override=None, dtype=None, **kw):
+        from .config import PRESETS, preset
+        from .processing import ChatTSProcessor, TextProcessor
+        from .registry import load_config, model_class
         from .tp import Comm, LocalComm
         self._tp_group = None
         if tensor_parallel_size > 1 and comm is None and "WORLD_SIZE" not in os.environ:
@@ -69,7 +71,7 @@ class LLM:
                 args = dict(tensor_parallel_size=tensor_parallel_size, max_model_len=max_model_len,
                             limit_mm_per_prompt=limit_mm_per_prompt, trust_remote_code=trust_remote_code,
                             gpu_memory_utilization=gpu_memory_utilization, seed=seed, tokenizer=tokenizer,
-                            max_num_seqs=max_num_seqs, block_size=block_size, num_gpu_blocks_override=num_gpu_blocks_override, **kw)
+                            max_num_seqs=max_num_seqs, block_size=block_size, num_gpu_blocks_override=num_gpu_blocks_override, dtype=dtype, **kw)
                 group, inner = TpGroup.launch(tensor_parallel_size, _build_llm, (model, args))
                 self.__dict__.update(inner.__dict__)
                 self._tp_group = group
@@ -85,18 +87,29 @@ class LLM:
         # max_num_seqs x max_model_len / block_size oversubscribes the slots (requests then wait for blocks at admission)
         mk = dict(comm=comm, max_ctx=max_model_len, max_prefill_tokens=min(2048, max_model_len),
                   max_batch=max(1, int(max_num_seqs)), kv_block_size=block_size, kv_pool_blocks=num_gpu_blocks_override)
-        if isinstance(model, ChatTSConfig):
-            self.model = ChatTSForCausalLM.from_synthetic(model, seed=seed, **mk)
-        elif isinstance(model, str) and model in PRESETS:
-            self.model = ChatTSForCausalLM.from_synthetic(preset(model), seed=seed, **mk)
+        # the design's own class serves it: a configuration object, a preset name or a checkpoint directory (chatts_amd/registry.py)
+        path = None
+        if isinstance(model, str) and model in PRESETS:
+            model = preset(model)
         elif isinstance(model, str) and os.path.isdir(model):
-            self.model = ChatTSForCausalLM.from_pretrained(model, **mk)
-            if tokenizer is None:           # real weights need the checkpoint's own tokenizer, never the synthetic stand-in
-                tokenizer = _load_checkpoint_tokenizer(model)
+            path, model = model, load_config(model)
+        elif isinstance(model, str) or not hasattr(model, "to_dict"):
+            raise ValueError(f"model must be a checkpoint directory, a configuration object or one of {sorted(PRESETS)}")
+        cls, text_only = model_class(model), not hasattr(model, "ts")
+        if text_only and dtype is not None:
+            mk["dtype"] = dtype
+        if path is None:
+            self.model = cls.from_synthetic(model, seed=seed, **mk)
         else:
-            raise ValueError(f"model must be a checkpoint directory, a ChatTSConfig or one of {sorted(PRESETS)}")
+            self.model = cls.from_pretrained(path, **mk)
+            if tokenizer is None:           # real weights need the checkpoint's own tokenizer, never the synthetic stand-in
+                tokenizer = _load_checkpoint_tokenizer(path, required=not text_only)
         self.config = self.model.config
-        self.processor = ChatTSProcessor.from_pretrained(self.config, tokenizer=tokenizer)
+        if text_only:
+            from .tokenizer import TokenIdTokenizer
+            self.processor = TextProcessor(tokenizer or TokenIdTokenizer())
+        else:
+            self.processor = ChatTSProcessor.from_pretrained(self.config, tokenizer=tokenizer)
         self.limit = (limit_mm_per_prompt or {}).get("timeseries", 50)      # chatts_vllm.py:220 caps at 50
 
     def get_tokenizer(self):
@@ -118,16 +131,23 @@ class LLM:
         if self._tp_group is not None:      # spawned followers run the same call now; all ranks meet inside the exchange kernels
             self._tp_group.call("generate", prompts, sampling_params)
         sp = sampling_params or SamplingParams()
-        self.model.set_sampling(sp.temperature or 0.0, max(int(sp.top_k or 0), 0), sp.top_p,
-                                self._seed if sp.seed is None else sp.seed)
         if isinstance(prompts, (str, dict)):
             prompts = [prompts]
+        self.model.set_sampling(sp.temperature or 0.0, max(int(sp.top_k or 0), 0), sp.top_p,
+                                self._seed if sp.seed is None else sp.seed)
         import torch
         reqs, metas = [], []
         for req in prompts:
             if isinstance(req, str):
                 req = {"prompt": req}
             series = list((req.get("multi_modal_data") or {}).get("timeseries", []))
+            if "prompt_token_ids" in req:       # (vLLM's TokensPrompt)
+                if series:
+                    raise ValueError("time series need a text prompt")
+                ids = [int(t) for t in req["prompt_token_ids"]]
+                reqs.append((ids, None, []))
+                metas.append((req.get("prompt"), ids))
+                continue
             if len(series) > self.limit:
                 raise ValueError(f"At most {self.limit} timeseries may be provided in one prompt, got {len(series)}")
             text, encs, lens = self.processor.splice(req["prompt"], [np.asarray(s, dtype=np.float64) for s in series])

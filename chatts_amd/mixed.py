@@ -1,0 +1,509 @@
+"""MixedDecoder - a served model whose layers each name their mixer, run by csrc/mixdec.hip.
+
+A layer is norm1 -> mixer -> norm1b -> residual, then optionally norm2 -> squared-relu feed-forward -> norm2b -> residual.  Mixers:
+  LatentMixer   attention over a paged cache of one latent + one rotated key part per token (csrc/latent.hip)
+  DeltaMixer    gated delta rule: a float32 state and a ring of convolution inputs per slot (csrc/delta.hip)
+A design (chatts_amd/fobolix.py) says in which order layers run (config.runs(): a layer may run several times, every run has its own pages or
+state) and maps its tensor names onto LayerWeights.
+
+Everything is padded once, at load: widths and feed-forwards to multiples of 64, the stacked input projections block by block, heads to
+what the kernels tile by.  Padding is zero weights, so activations never need clearing.
+
+Slots, pages, sampling, scheduling and generation are SlotModel's.  A recurrent state is a function of the whole prefix and is not kept per
+position, so prefixes are not reused between requests.
+"""
+import ctypes as C
+import glob
+import os
+from dataclasses import dataclass
+from types import SimpleNamespace
+from typing import Any, Optional
+
+import torch
+
+from . import _lib
+from .kv_blocks import BlockPool
+from .rotary import rotary_tables
+from .slot_model import SlotModel
+from .tp import LocalComm
+
+
+@dataclass
+class LatentMixer:
+    heads: int
+    dim: int
+    rot: int
+    vdim: int
+    rank: int
+    scale: float
+    rot_base: float
+    rot_scaling: Optional[dict]
+    q: Any          # [heads * (dim + rot), width], head by head
+    dkv: Any        # [rank + rot, width]
+    c_norm: Any
+    uk: Any         # [heads * dim, rank]
+    uv: Any         # [heads * vdim, rank]
+    o: Any          # [width, heads * vdim]
+
+
+@dataclass
+class DeltaMixer:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+    q: Any
+    k: Any
+    v: Any
+    q_conv: Any     # [channels, taps]
+    k_conv: Any
+    v_conv: Any
+    b: Any
+    a_log: Any
+    a1: Any
+    a2: Any
+    dt_bias: Any
+    g1: Any
+    g2: Any
+    norm: Any
+    o: Any
+
+
+@dataclass
+class LayerWeights:
+    mixer: Any
+    norm1: Any
+    norm1b: Any
+    norm2: Any = None
+    norm2b: Any = None
+    up: Any = None
+    down: Any = None
+
+
+def _up(n, m):
+    return (int(n) + m - 1) // m * m
+
+
+def _pad(t, rows, cols):
+    out = torch.zeros((rows, cols), dtype=t.dtype, device=t.device)
+    out[:t.shape[0], :t.shape[1]] = t
+    return out
+
+
+class MixedDecoder(SlotModel):
+    step_is_idempotent = False       # a decode step advances recurrent states
+
+    def __init__(self, config, device="cuda", comm=None, max_ctx=2048, max_prefill_tokens=2048, use_graph=True, max_batch=1, kv_block_size=None,
+                 kv_pool_blocks=None, dtype="bfloat16", prefill_tiled_weights=None, weight_format="bf16", **unused):
+        """dtype "bfloat16": bf16 hi / lo operand planes and a bf16 latent cache; "float32": every product and sum in 32-bit (checks)."""
+        if not torch.cuda.is_available():
+            raise RuntimeError("chatts_amd needs a ROCm GPU: there is no CPU fallback for the model")
+        if dtype not in ("bfloat16", "float32"):
+            raise ValueError("dtype must be 'bfloat16' or 'float32'")
+        if weight_format != "bf16":
+            raise ValueError(f"{type(config).__name__} is served with bf16 weights, not {weight_format!r}")
+        self.comm = comm or LocalComm()
+        if self.comm.world != 1:
+            raise ValueError("decoders of mixed layers run on one GPU (tensor_parallel_size 1)")
+        self.lib = _lib.load()
+        self.config, self.device = config, torch.device(device)
+        self.dtype, self.exact = dtype, dtype == "float32"
+        self.max_batch = max(1, int(max_batch))
+        self.kv_block_size = int(kv_block_size or 64)
+        if self.kv_block_size < 64 or self.kv_block_size & (self.kv_block_size - 1):
+            raise ValueError(f"kv_block_size={kv_block_size} must be a power of two >= 64")
+        self.max_ctx = _up(max_ctx, self.kv_block_size)
+        self.t_max = int(max(min(max_prefill_tokens, self.max_ctx * self.max_batch), self.max_batch))
+        self._kv_pool_blocks = None if kv_pool_blocks is None else int(kv_pool_blocks)
+        self.use_graph, self._graph, self._graph_batched, self._tp = use_graph, None, None, None
+        if prefill_tiled_weights is None:
+            prefill_tiled_weights = self.t_max >= 96 and os.environ.get("CHATTS_TILED_WEIGHTS", "1") != "0"
+        self.tiled = bool(prefill_tiled_weights) and not self.exact
+        self.plan = SimpleNamespace(world=1, rank=0, vocab=config.vocab_size, v0=0)
+        self.enable_prefix_caching = False
+        self._slot_idents = [[] for _ in range(self.max_batch)]
+        self._slot_seen = [0] * self.max_batch
+        self._kv_replaced = {}
+        self.prefix_stats = {"requests": 0, "hits": 0, "tokens_reused": 0, "tokens_prefilled": 0}
+        self._decoder, self._keep, self.loaded = None, [], set()
+
+    # ---- weights -------------------------------------------------------------------------------------------------------------
+    def layer_weights(self, sd, i):
+        raise NotImplementedError
+
+    def model_weights(self, sd):
+        raise NotImplementedError
+
+    @classmethod
+    def from_pretrained(cls, path, config=None, torch_dtype=None, device_map=None, trust_remote_code=None, **kw):
+        from safetensors import safe_open
+        from .registry import load_config
+        if torch_dtype is not None and "dtype" not in kw:
+            kw["dtype"] = str(torch_dtype).replace("torch.", "")
+        m = cls(config or load_config(path), **kw)
+
+        def pairs():
+            for f in sorted(glob.glob(os.path.join(path, "*.safetensors"))):
+                with safe_open(f, framework="pt", device="cpu") as h:
+                    for k in h.keys():
+                        yield k, h.get_tensor(k)
+        m.load_weights(pairs())
+        return m
+
+    @classmethod
+    def from_synthetic(cls, config, seed=0, rank_a=None, rank_g=None, **kw):
+        """random weights of the configuration's shapes, made on the device (speed measurements)"""
+        m = cls(config, **kw)
+        gen = torch.Generator(device=m.device).manual_seed(seed)
+        big = max((l["mixer"].get("dim", 64) for l in config.layers), default=64)
+        sd = {}
+        for name, shape in config.tensor_shapes(rank_a or big, rank_g or big).items():
+            t = torch.randn(shape, generator=gen, device=m.device)
+            if len(shape) == 2 and not name.endswith(".conv") and name != "embed":
+                t *= shape[1] ** -0.5
+            if name.endswith(("norm", "norm1", "norm2", "norm1b", "norm2b")):
+                t = 1.0 + 0.1 * t
+            if name.endswith("dt_bias"):
+                t = 0.5 * t - 3.0
+            sd[name] = t.to(torch.bfloat16)
+        m.load_weights(sd.items())
+        return m
+
+    def load_weights(self, weights):
+        """consume (name, tensor) pairs; returns the set of names taken"""
+        sd = {n: t.to(self.device) for n, t in weights}
+        want = self.config.tensor_shapes()
+        missing = sorted(set(want) - set(sd))
+        if missing:
+            raise ValueError(f"checkpoint lacks {missing[:5]}{' ...' if len(missing) > 5 else ''}")
+        for n, shape in want.items():
+            if any(s is not None and s != g for s, g in zip(shape, sd[n].shape)) or len(shape) != sd[n].dim():
+                raise ValueError(f"{n}: shape {tuple(sd[n].shape)}, the configuration says {shape}")
+        self._build(sd)
+        self.loaded = set(want)
+        return self.loaded
+
+    def _dev(self, t):
+        t = t.contiguous()
+        self._keep.append(t)
+        return t.data_ptr()
+
+    def _f32(self, t, n=None):
+        t = t.to(torch.float32).reshape(-1)
+        if n is not None and n > t.numel():
+            t = torch.cat([t, torch.zeros(n - t.numel(), dtype=torch.float32, device=self.device)])
+        return self._dev(t)
+
+    def _mat(self, t, rows=None, cols=None, tile=False):
+        """bf16 matrix, zero padded -> (pointer, pointer of its tiled copy or None)"""
+        t = t.to(torch.bfloat16)
+        t = _pad(t, rows or t.shape[0], cols or t.shape[1]).contiguous()
+        p, pt = self._dev(t), None
+        if tile and self.tiled:
+            out = torch.empty(int(self.lib.chatts_tile_bf16_elems(t.shape[0], t.shape[1])), dtype=torch.bfloat16, device=self.device)
+            _lib.check(self.lib.chatts_tile_bf16(p, t.shape[0], t.shape[1], t.shape[1], out.data_ptr(), _lib.stream_ptr()))
+            pt = self._dev(out)
+        return p, pt
+
+    def _stack(self, blocks):
+        """stacked input projection: (name, [rows, width], padded rows) -> (matrix, {name: first row})"""
+        off, at = {}, 0
+        for name, t, rows in blocks:
+            off[name] = at
+            at += rows
+        out = torch.zeros((_up(at, 64), self._wp), dtype=torch.bfloat16, device=self.device)
+        for name, t, rows in blocks:
+            out[off[name]:off[name] + t.shape[0], :t.shape[1]] = t.to(torch.bfloat16)
+        return out, off
+
+    def _latent_layer(self, L, m):
+        H, W = m.heads, self.config.hidden_size
+        dim_p, rank_p, rot_p, vdim_p = _up(m.dim, 32), _up(m.rank, 32), _up(m.rot, 32), _up(m.vdim, 16)
+        q = m.q.view(H, m.dim + m.rot, W)
+        un = torch.zeros((H, dim_p, W), dtype=q.dtype, device=self.device)
+        un[:, :m.dim] = q[:, :m.dim]
+        w, off = self._stack([("q", un.view(H * dim_p, W), H * dim_p), ("qr", q[:, m.dim:].reshape(H * m.rot, W), _up(H * m.rot, 64)),
+                              ("c", m.dkv[:m.rank], _up(m.rank, 64)), ("kr", m.dkv[m.rank:], _up(m.rot, 64))])
+        L.kind, L.in_n = _lib.MIX_LATENT, w.shape[0]
+        L.w_in, L.in_t = self._mat(w, tile=True)
+        o = torch.zeros((W, H, vdim_p), dtype=m.o.dtype, device=self.device)
+        o[:, :, :m.vdim] = m.o.view(W, H, m.vdim)
+        L.out_k, L.out_head, L.dim_p, L.vdim_p = _up(H * vdim_p, 64), vdim_p, dim_p, vdim_p
+        L.out, L.out_t = self._mat(o.view(W, H * vdim_p), self._wp, L.out_k, tile=True)
+        uk = torch.zeros((H, rank_p, dim_p), dtype=torch.bfloat16, device=self.device)
+        uk[:, :m.rank, :m.dim] = m.uk.view(H, m.dim, m.rank).transpose(1, 2).to(torch.bfloat16)
+        uv = torch.zeros((H, vdim_p, rank_p), dtype=torch.bfloat16, device=self.device)
+        uv[:, :m.vdim, :m.rank] = m.uv.view(H, m.vdim, m.rank).to(torch.bfloat16)
+        L.uk, L.uv = self._dev(uk), self._dev(uv)
+        cos, sin = rotary_tables(m.rot, m.rot_base, self.max_ctx, m.rot_scaling, self.device)
+        L.latent = _lib.LatentArgs(off_q=off["q"], off_qr=off["qr"], off_c=off["c"], off_kr=off["kr"], heads=H, dim=m.dim, rot=m.rot, rank=m.rank,
+                                   vdim=m.vdim, rank_p=rank_p, rot_p=rot_p, scale=m.scale, c_norm=self._f32(m.c_norm), cos_tab=self._dev(cos),
+                                   sin_tab=self._dev(sin))
+        self._lat_q, self._lat_o = max(self._lat_q, H * (rank_p + rot_p)), max(self._lat_o, H * rank_p)
+
+    def _delta_layer(self, L, m):
+        qk, v, ra, rg = m.kv_heads * m.dim, m.heads * m.vdim, m.a1.shape[0], m.g1.shape[0]
+        ra_p, rg_p = _up(ra, 64), _up(rg, 64)
+        w, off = self._stack([("q", m.q, _up(qk, 64)), ("k", m.k, _up(qk, 64)), ("v", m.v, _up(v, 64)), ("a", m.a1, ra_p), ("g", m.g1, rg_p),
+                              ("b", m.b, _up(m.heads, 64))])
+        L.kind, L.in_n = _lib.MIX_DELTA, w.shape[0]
+        L.w_in, L.in_t = self._mat(w, tile=True)
+        L.out_k, L.out_head = _up(v, 64), m.vdim
+        L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
+        L.dt_n, L.gate_n = _up(m.heads * m.dim, 16), _up(v, 16)
+        conv = torch.zeros((m.taps, off["a"]), dtype=torch.float32, device=self.device)
+        for n, t in (("q", m.q_conv), ("k", m.k_conv), ("v", m.v_conv)):
+            conv[:, off[n]:off[n] + t.shape[0]] = t.to(torch.float32).t()
+        L.delta = _lib.DeltaArgs(off_q=off["q"], off_k=off["k"], off_v=off["v"], off_a=off["a"], off_g=off["g"], off_b=off["b"], conv_ch=off["a"],
+                                 heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, taps=m.taps, rank_a=ra_p, rank_g=rg_p,
+                                 conv_w=self._dev(conv), a2=self._mat(m.a2, L.dt_n, ra_p)[0], g2=self._mat(m.g2, L.gate_n, rg_p)[0], ld_a2=ra_p, ld_g2=rg_p,
+                                 dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32))), norm_w=self._f32(m.norm))
+
+    def _build(self, sd):
+        cfg, lib, dev = self.config, self.lib, self.device
+        W, self._wp = cfg.hidden_size, _up(cfg.hidden_size, 64)
+        Wp, V, Vp, MB, T = self._wp, cfg.vocab_size, _up(cfg.vocab_size, 64), self.max_batch, self.t_max
+        self.vocab_p = Vp
+        self._lat_q = self._lat_o = 1
+        mixers, arr = [], (_lib.MixLayer * len(cfg.layers))()
+        for i in range(len(cfg.layers)):
+            lw, L = self.layer_weights(sd, i), arr[i]
+            L.norm1, L.norm1b = self._f32(lw.norm1, Wp), self._f32(lw.norm1b, Wp)
+            (self._latent_layer if isinstance(lw.mixer, LatentMixer) else self._delta_layer)(L, lw.mixer)
+            if lw.up is not None:
+                L.norm2, L.norm2b, L.ff = self._f32(lw.norm2, Wp), self._f32(lw.norm2b, Wp), _up(lw.up.shape[0], 64)
+                L.up, L.up_t = self._mat(lw.up, L.ff, Wp, tile=True)
+                L.down, L.down_t = self._mat(lw.down, Wp, L.ff, tile=True)
+            mixers.append(lw.mixer)
+        mw = self.model_weights(sd)
+        f32 = dict(dtype=torch.float32, device=dev)
+        # every run's pages / states
+        bps = self.max_ctx // self.kv_block_size
+        nblk = MB * bps if self._kv_pool_blocks is None else self._kv_pool_blocks
+        if nblk < 1 or nblk > MB * bps:
+            raise ValueError(f"kv_pool_blocks={nblk} must lie in 1..{MB * bps} (max_batch x max_ctx / kv_block_size)")
+        self._kv = BlockPool(nblk, self.kv_block_size, MB, bps)
+        self._kv_dynamic = nblk < MB * bps
+        cache_dtype = torch.float32 if self.exact else torch.bfloat16
+        order = cfg.runs()
+        runs = (_lib.MixRun * len(order))()
+        self.cache_bytes = self.state_bytes = 0
+        for r, (i, opens) in enumerate(order):
+            runs[r].layer = i
+            if opens is not None:
+                runs[r].add = self._f32(mw["steps"][opens], Wp)
+            if isinstance(mixers[i], LatentMixer):
+                a = arr[i].latent
+                t = torch.zeros((nblk, self.kv_block_size, a.rank_p + a.rot_p), dtype=cache_dtype, device=dev)
+                runs[r].cache = self._dev(t)
+                self.cache_bytes += t.numel() * t.element_size()
+            else:
+                a = arr[i].delta
+                s = torch.zeros((MB, a.heads, a.dim, _up(a.vdim, 4)), **f32)
+                ring = torch.zeros((MB, a.taps, a.conv_ch), **f32)
+                runs[r].state, runs[r].ring = self._dev(s), self._dev(ring)
+                self.state_bytes += 4 * (s.numel() + ring.numel())
+        head, head_t = self._mat(mw["head"], Vp, Wp, tile=True)
+        embed = self._mat(mw["embed"], V, Wp)[0]
+        kmax = max([Wp] + [max(L.out_k, L.ff) for L in arr])
+        deltas = [L for L in arr if L.kind == _lib.MIX_DELTA]
+        most = lambda f: max([f(L) for L in deltas], default=1)
+        mc = _lib.MixConfig(width=W, width_p=Wp, n_layers=len(arr), n_runs=len(order), exact=int(self.exact), t_max=T, max_slots=MB, max_ctx=self.max_ctx,
+                            vocab=V, vocab_p=Vp, eps=cfg.rms_norm_eps, block_size=self.kv_block_size, table_stride=bps)
+        ws = int(lib.chatts_mixdec_workspace(C.byref(mc), arr))
+        rows = T + 1                                     # (kernels may read one row past the last)
+        bf = dict(dtype=torch.bfloat16, device=dev)
+        self.buf = B = {
+            "x": torch.zeros((rows, Wp), **f32), "y": torch.zeros((rows, Wp), **f32), "proj": torch.zeros((rows, max(L.in_n for L in arr)), **f32),
+            "a_f32": torch.zeros((rows, Wp), **f32), "b_f32": torch.zeros((rows, kmax), **f32),
+            "a_planes": torch.zeros((2, rows, Wp), **bf), "b_planes": torch.zeros((2, rows, kmax), **bf),
+            "q_f32": torch.zeros((rows, self._lat_q) if self.exact else (1, 1), **f32),
+            "q_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, self._lat_q), **bf),
+            "o_lat": torch.zeros((rows, self._lat_o), **f32), "partial": torch.zeros(max(64, MB) * 8 * self._lat_o + 65536, **f32),
+            "dq": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
+            "dk": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
+            "dv": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
+            "dg": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.dim)), **f32),
+            "dgate": torch.zeros((rows, most(lambda L: L.gate_n)), **f32), "dbeta": torch.zeros((rows, most(lambda L: L.delta.heads)), **f32),
+            "dout": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32), "ddt": torch.zeros((rows, most(lambda L: L.dt_n)), **f32),
+            "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 4), dtype=torch.int32, device=dev),
+            "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
+            "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),
+            "pos_all": torch.full((MB,), -1, dtype=torch.int32, device=dev), "step_all": torch.zeros(MB, dtype=torch.int32, device=dev),
+            "token_all": torch.zeros(MB, dtype=torch.int64, device=dev), "token_logit_all": torch.zeros(MB, **f32),
+            "out_tokens_all": torch.zeros((MB, self.max_ctx + 8), dtype=torch.int64, device=dev),
+        }
+        B["pos"], B["step"], B["token"], B["out_tokens"] = B["pos_all"][:1], B["step_all"][:1], B["token_all"][:1], B["out_tokens_all"][0]
+        P = _lib.ptr
+        mb = _lib.MixBuffers(embed=embed, head=head, head_t=head_t, final_norm=self._f32(mw["final_norm"], Wp), x=P(B["x"]), y=P(B["y"]), proj=P(B["proj"]),
+                             a_f32=P(B["a_f32"]), b_f32=P(B["b_f32"]), a_hi=P(B["a_planes"][0]), a_lo=P(B["a_planes"][1]), b_hi=P(B["b_planes"][0]),
+                             b_lo=P(B["b_planes"][1]), q_f32=P(B["q_f32"]), o_lat=P(B["o_lat"]), partial=P(B["partial"]), q_hi=P(B["q_planes"][0]),
+                             q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
+                             logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
+                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dout", "ddt")})
+        h = lib.chatts_mixdec_create(C.byref(mc), arr, runs, C.byref(mb))
+        if not h:
+            raise _lib.ChattsError(-1, lib.chatts_last_error().decode())
+        self._decoder, self._layer_arr, self._mix_config = C.c_void_p(h), arr, mc
+        if not self._kv_dynamic:
+            for s in range(MB):
+                self._kv.reserve(s, self.max_ctx)
+                self._kv.retire(s)
+                self._push_kv_row(s)
+
+    def __del__(self):
+        try:
+            if self._decoder:
+                self.lib.chatts_mixdec_destroy(self._decoder)
+        except Exception:
+            pass
+
+    # ---- the step ------------------------------------------------------------------------------------------------------------
+    def _forward(self, ids, segs):
+        """ids: all tokens of the batch; segs: (first row, tokens, first position, slot), slots distinct"""
+        B, T = self.buf, len(ids)
+        if T > self.t_max:
+            raise ValueError(f"{T} tokens exceed max_prefill_tokens={self.t_max}")
+        V = self.config.vocab_size
+        if min(ids) < 0 or max(ids) >= V:
+            raise ValueError(f"token ids must lie in 0..{V - 1}")
+        B["ids"][:T].copy_(torch.tensor(ids, dtype=torch.int64))
+        meta = torch.empty((T, 4), dtype=torch.int32)
+        for row, t, pos0, slot in segs:
+            r = torch.arange(t, dtype=torch.int32)
+            meta[row:row + t, 0], meta[row:row + t, 1], meta[row:row + t, 2], meta[row:row + t, 3] = slot, pos0 + r, row, t - 1 - r
+        B["rows"][:T].copy_(meta)
+        single = all(s[1] == 1 for s in segs)
+        if not single:
+            B["spans"][:len(segs)].copy_(torch.tensor([(r, t, p, s) for r, t, p, s in segs], dtype=torch.int32))
+        _lib.check(self.lib.chatts_mixdec_forward(self._decoder, _lib.ptr(B["ids"]), T, len(segs), int(single), _lib.stream_ptr()))
+
+    def _logits(self, index):
+        """logits of rows `index` of the last forward -> [n, vocab_p] float32"""
+        out = torch.empty((len(index), self.vocab_p), dtype=torch.float32, device=self.device)
+        idx = torch.tensor(index, dtype=torch.int32, device=self.device)
+        for a in range(0, len(index), 256):
+            n = min(256, len(index) - a, self.t_max)
+            _lib.check(self.lib.chatts_mixdec_logits(self._decoder, idx[a:].data_ptr(), n, out[a:].data_ptr(), _lib.stream_ptr()))
+        return out
+
+    def _run_segments(self, ids, segs, index):
+        self._forward(ids, segs)
+        return self._logits(index)[:, :self.config.vocab_size] if index else None
+
+    def _select(self, logits, slot, n, sampling, pos):
+        """tokens of rows slot .. slot + n from `logits` [n, vocab_p]: appended to out_tokens, step (and position, when pos) advanced"""
+        B, lib, st, V = self.buf, self.lib, _lib.stream_ptr(), self.config.vocab_size
+        out, stride = B["out_tokens_all"][slot:].data_ptr(), B["out_tokens_all"].shape[1]
+        at = lambda k: B[k][slot:].data_ptr()
+        posp, limit = (at("pos_all"), self.max_ctx - 1) if pos else (None, 0)
+        if sampling is None:
+            _lib.check(lib.chatts_argmax_batched_ws(logits.data_ptr(), n, self.vocab_p, V, 0, at("token_all"), at("token_logit_all"), out, stride, at("step_all"),
+                                                    posp, limit, B["ws"].data_ptr(), B["ws"].numel(), st))
+        else:
+            _lib.check(lib.chatts_sample_batched(logits.data_ptr(), n, self.vocab_p, V, 0, C.byref(sampling), at("token_all"), at("token_logit_all"), out, stride,
+                                                 at("step_all"), posp, limit, st))
+
+    def _batched_step_eager(self):
+        B = self.buf
+        _lib.check(self.lib.chatts_mixdec_decode(self._decoder, self.max_batch, _lib.ptr(B["token_all"]), _lib.ptr(B["pos_all"]), _lib.ptr(B["logits_all"]),
+                                                 _lib.stream_ptr()))
+        self._select(B["logits_all"], 0, self.max_batch, getattr(self, "_sampling", None), True)
+
+    def decode_step(self):
+        self.batched_step()
+
+    def _install_sampling(self, args):
+        pass                                             # (_select reads self._sampling when the step is enqueued or captured)
+
+    # ---- admission -----------------------------------------------------------------------------------------------------------
+    def request_tokens(self, ids, series=None, lengths=None):
+        return len(ids)
+
+    def _request_idents(self, ids, series, lengths):
+        return None
+
+    def admit_begin(self, slot, ids, series=None, lengths=None, max_new_tokens=1):
+        if series is not None and len(series):
+            raise ValueError(f"{self.config.name} takes token ids only, no time series")
+        ids = [int(t) for t in ids]
+        T = len(ids)
+        if T < 1:
+            raise ValueError("an empty prompt")
+        if T + max_new_tokens > self.max_ctx:
+            raise ValueError(f"prompt ({T}) + max_new_tokens ({max_new_tokens}) exceeds max_ctx={self.max_ctx}")
+        if min(ids) < 0 or max(ids) >= self.config.vocab_size:
+            raise ValueError(f"token ids must lie in 0..{self.config.vocab_size - 1}")
+        self.reserve_kv(slot, T + max_new_tokens)
+        self.prefix_stats["requests"] += 1
+        self.prefix_stats["tokens_prefilled"] += T
+        return {"slot": slot, "ids": ids, "T": T, "done": 0}
+
+    def admit_step(self, st, max_rows=None):
+        slot, T, a = st["slot"], st["T"], st["done"]
+        end = T if max_rows is None else min(T, a + max(int(max_rows), 1))
+        while a < end:
+            n = min(self.t_max, end - a)
+            self._forward(st["ids"][a:a + n], [(0, n, a, slot)])
+            a += n
+        st["done"] = a
+        if a < T:
+            return False
+        self._first_token(slot, n - 1, T)
+        return True
+
+    def _first_token(self, slot, row, T):
+        B = self.buf
+        lg = self._logits([row])
+        B["pos_all"][slot] = T
+        B["step_all"][slot] = 0
+        sa = getattr(self, "_sampling", None)
+        if getattr(self, "_sampling_key", None) == "rows":
+            sa = self._rows_args(slot)
+        elif sa is not None:                             # (a later step draws with (seed, slot, step): fold the slot into this one's seed)
+            sa = _lib.SamplingArgs(temperature=sa.temperature, top_k=sa.top_k, top_p=sa.top_p, seed=(sa.seed ^ (0x51ED27 * (slot + 1))) & 0xFFFFFFFF,
+                                   n_kept=None, kept_mass=None)
+        self._select(lg, slot, 1, sa, False)
+
+    def _admit_packed(self, items):
+        """several prompts in one ragged pass (plan_pack has checked that they fit t_max)"""
+        states = []
+        try:
+            for it in items:
+                states.append(self.admit_begin(*it))
+        except Exception:
+            for st in states:                            # nothing ran yet: others may take these reservations
+                self._kv.retire(st["slot"])
+            raise
+        ids, segs = [], []
+        for st in states:
+            segs.append((len(ids), st["T"], 0, st["slot"]))
+            ids += st["ids"]
+        self._forward(ids, segs)
+        self.prefix_stats["packed_prefills"] = self.prefix_stats.get("packed_prefills", 0) + 1
+        for row, t, _, slot in segs:
+            self._first_token(slot, row + t - 1, t)
+        return [st["T"] for st in states]
+
+    def _prefill_request(self, ids, series, lengths, max_new_tokens):
+        return self._admit(0, ids, series, lengths, max_new_tokens)
+
+    # ---- call surface --------------------------------------------------------------------------------------------------------
+    @torch.no_grad()
+    def generate(self, input_ids=None, attention_mask=None, max_new_tokens=64, max_length=None, eos_token_id=None, do_sample=False, temperature=None,
+                 top_k=None, top_p=None, seed=0, **kw):
+        """like the other models' generate(): LongTensor [B, T_in + new], rows right-padded with pad_token_id"""
+        if do_sample:
+            self.set_sampling(1.0 if temperature is None else temperature, 50 if top_k is None else top_k, 1.0 if top_p is None else top_p, seed)
+        else:
+            self.set_sampling(0.0)
+        ids = input_ids if isinstance(input_ids, torch.Tensor) else torch.tensor(input_ids)
+        ids = (ids[None] if ids.dim() == 1 else ids).cpu()
+        mask = attention_mask.cpu() if attention_mask is not None else torch.ones_like(ids)
+        reqs = [(ids[b][mask[b].bool()].tolist(), None, None) for b in range(ids.shape[0])]
+        budget = max_new_tokens if max_length is None else max(1, max_length - max(len(r[0]) for r in reqs))
+        outs = self.generate_batch(reqs, budget, self.config.eos_token_id if eos_token_id is None else eos_token_id)
+        rows = [ids[b].tolist() + outs[b] for b in range(ids.shape[0])]
+        n = max(len(r) for r in rows)
+        return torch.tensor([r + [self.config.pad_token_id] * (n - len(r)) for r in rows], dtype=torch.long)

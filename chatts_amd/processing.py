@@ -55,6 +55,22 @@ def hf_prefix(series, mean, factor):
             f"min={np.min(x):.4f}|left={x[0]:.4f}|right={x[-1]:.4f}]" + PLACEHOLDER)
 
 
+class TextProcessor:
+    """The processor of text-only designs: prompts without series."""
+
+    def __init__(self, tokenizer):
+        self.tokenizer = tokenizer
+
+    def splice(self, prompt, series_list):
+        if len(series_list):
+            raise ValueError("this model takes no time series")
+        return prompt, [], []
+
+    @staticmethod
+    def pad_stack(encs):
+        return np.zeros((0, 0, 1), dtype=np.float32)
+
+
 class BatchFeature(dict):
     """dict with ``.to(device)`` like transformers.BatchFeature (callers also do {k: v.to(0)})."""
 

@@ -153,12 +153,15 @@ def create_app(engine_thread, tokenizer, served_model_name="chatts", limit_times
                 prompt, series = render_chat(body.get("messages") or [])
             else:
                 prompt = body.get("prompt")
-                if isinstance(prompt, list):
+                tokens = isinstance(prompt, list) and bool(prompt) and all(isinstance(t, int) for t in prompt)      # token ids
+                if isinstance(prompt, list) and not tokens:
                     prompt = prompt[0]
                 series = [[float(v) for v in s] for s in ((body.get("multi_modal_data") or {}).get("timeseries") or [])]
-                if not isinstance(prompt, str):
-                    raise ValueError("prompt must be a string")
-                if prompt.count("<ts><ts/>") != len(series):
+                if not isinstance(prompt, str) and not tokens:
+                    raise ValueError("prompt must be a string or a list of token ids")
+                if tokens and series:
+                    raise ValueError("time series need a text prompt")
+                if not tokens and prompt.count("<ts><ts/>") != len(series):
                     raise ValueError(f"prompt holds {prompt.count('<ts><ts/>')} <ts><ts/> placeholders but {len(series)} timeseries")
             if len(series) > limit_timeseries:
                 raise ValueError(f"At most {limit_timeseries} timeseries may be provided in one prompt, got {len(series)}")
@@ -266,7 +269,7 @@ def build_server(model, tensor_parallel_size=1, max_model_len=6000, max_num_seqs
 
 def main():
     ap = argparse.ArgumentParser(description="OpenAI-compatible ChatTS server on the MI355X-native engine")
-    ap.add_argument("--model", required=True, help="checkpoint directory or a preset name (chatts-14b, chatts-8b: synthetic weights)")
+    ap.add_argument("--model", required=True, help="checkpoint directory (its config.json names the design) or a preset name (chatts-14b, chatts-8b: synthetic weights)")
     ap.add_argument("--served-model-name", default="chatts")
     ap.add_argument("--host", default="0.0.0.0")
     ap.add_argument("--port", type=int, default=12345)

@@ -16,6 +16,22 @@ _SPECIAL = re.compile(r"(<\|im_start\|>|<\|im_end\|>|<\|endoftext\|>|<ts/>|<ts>)
 _PRE = re.compile(r"'s|'t|'re|'ve|'m|'ll|'d| ?[^\W\d_]+|\d| ?[^\s\w]+|_|\s+(?!\S)|\s+", re.UNICODE)
 
 
+class TokenIdTokenizer:
+    """For checkpoints without tokenizer files whose users speak token ids: the text form of a sequence is its ids, space separated."""
+    padding_side = "left"
+    pad_token_id = 0
+    eos_token_id = None
+
+    def encode(self, text, **kw):
+        try:
+            return [int(t) for t in text.split()]
+        except ValueError:
+            raise ValueError("this checkpoint has no tokenizer files: give token ids (a list, or their decimal numbers separated by spaces)")
+
+    def decode(self, ids, **kw):
+        return " ".join(str(int(t)) for t in ids)
+
+
 class SyntheticTokenizer:
     padding_side = "left"
 

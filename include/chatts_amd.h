@@ -49,8 +49,10 @@ const char* chatts_last_error(void);
  *     chatts_linear_f16q, ChattsLayerWeights.*16 / *_q8 / *_q8e, chatts_decoder_set_prefill_f16q: an opt-in, parity-grade, SLOWER prefill mode - DESIGN.md section 14);
  *     the tensor-parallel exchange's release form per communicator (chatts_tp_cross_device / chatts_tp_set_cross_device /
  *     chatts_tp_set_bulk_release / chatts_tp_bulk_release); tiled prefill weights (chatts_tile_bf16, ChattsLinearArgs.w_tiled /
- *     planes_tiled, ChattsLayerWeights.*_t). */
-#define CHATTS_ABI_VERSION 9
+ *     planes_tiled, ChattsLayerWeights.*_t);
+ * 10: decoders of mixed layers chatts_mixdec_* with their kernels (chatts_residual_norm, chatts_delta_*, chatts_latent_*, chatts_head_linear),
+ *     CHATTS_EPI_RELU2, ChattsLinearArgs.exact_f32. */
+#define CHATTS_ABI_VERSION 10
 int chatts_abi_version(void);
 /* Number of CUs of the current device (grid sizing), or <0. */
 int chatts_device_cus(void);
@@ -149,6 +151,7 @@ int chatts_ts_encode(const float* series, const int32_t* row_off, const int32_t*
 #define CHATTS_EPI_RESID 2    /* C = resid + acc (+bias); C may alias resid                         */
 #define CHATTS_EPI_SWIGLU 3   /* W rows are gate/up interleaved in blocks of 16 rows;               */
                               /* C[M,N/2] = silu(gate) * up            (Qwen2MLP.forward)           */
+#define CHATTS_EPI_RELU2 4    /* C = max(acc + bias, 0)^2              (bf16 weights)               */
 
 typedef struct ChattsLinearArgs {
   const float* a;          /* [M, lda] */
@@ -218,6 +221,9 @@ typedef struct ChattsLinearArgs {
    * the prefill kernel refuses them). */
   const chatts_bf16* w_tiled;
   int planes_tiled;
+  /* optional: every product and sum in float32 (M > 1: the float32 matrix pipe on the widened weights, gemm_f32.hip; M == 1: the GEMV as
+   * always).  Needs float32 `a` and `c`, bf16 `w`; no planes, no fused norm.  For 32-bit runs of a model, not a fast path. */
+  int exact_f32;
 } ChattsLinearArgs;
 #define CHATTS_W8_FP8 0
 #define CHATTS_W8_INT8 1
@@ -736,6 +742,170 @@ int chatts_decoder_logits(ChattsDecoder*, int row, chatts_stream_t stream);
 int chatts_decoder_decode_step(ChattsDecoder*, int32_t* pos_dev, int32_t* step_dev,
                                int64_t* token_dev, float* token_logit_dev, int64_t* out_tokens,
                                int n_splits, chatts_stream_t stream);
+
+
+/* ---------------------------------------------------------------------------------------------
+ * Decoders of MIXED layers: every layer names its mixer (latent attention over a paged latent cache, or a gated delta rule with a
+ * recurrent state), a range of layers may run several times per token (each pass with its own cache / state), norms stand before AND
+ * after each sublayer.  No reference twin (the reference serves Qwen2 / Qwen3 only).  The mechanisms are separate entry points with their
+ * constants as parameters; chatts_mixdec_* composes them.
+ *
+ * Rows of a step: one ChattsRow per token row.  pos < 0 marks a parked row (nothing is read or written for it).
+ * ------------------------------------------------------------------------------------------- */
+typedef struct ChattsRow { int32_t slot, pos, first, rest; } ChattsRow;   /* cache / state slot; position in its sequence; first row of
+                                                                           * its segment in this step; rows of the segment after this one */
+typedef struct ChattsSpan { int32_t row0, t, pos0, slot; } ChattsSpan;    /* a segment: t rows from row0 at positions pos0 .. */
+typedef struct ChattsOperand {   /* where the input of a following projection is written: float32 and / or bf16 hi / lo planes */
+  float* f32;
+  chatts_bf16* hi;
+  chatts_bf16* lo;
+  int ld;
+} ChattsOperand;
+
+typedef struct ChattsResidualNormArgs {
+  float* x;                /* [T, ldx] residual stream, updated in place */
+  const float* y;          /* [T, ldy] a sublayer's output, or NULL */
+  const float* post_w;     /* norm weight of y (padded with zeros to the row stride), NULL: y is added as it is */
+  const float* add;        /* a vector added to every row after that, or NULL */
+  const float* pre_w;      /* norm weight of the next sublayer, NULL: no output */
+  ChattsOperand out;
+  int t, width, ldx, ldy;
+  float eps;
+} ChattsResidualNormArgs;
+int chatts_residual_norm(const ChattsResidualNormArgs* args, chatts_stream_t stream);
+
+/* C[m, h, :] = W[h] . A[m, h, :] for every head h: a float32 [M, lda] (+ h * a_head), w bf16 [H, n, k], result float32 and / or planes at
+ * out (+ h * out_head columns).  k % 32 == 0 (zero padded weights; A is read to k), n % 16 == 0.  exact: float32 products and sums. */
+typedef struct ChattsHeadLinearArgs {
+  const float* a;
+  const chatts_bf16* w;
+  ChattsOperand out;
+  int m, heads, n, k, lda, a_head, out_head, exact;
+} ChattsHeadLinearArgs;
+int chatts_head_linear(const ChattsHeadLinearArgs* args, chatts_stream_t stream);
+
+/* ---- gated delta rule with one decay per head and key channel (delta.hip) ----
+ * Input: rows of one projection with the blocks q [kv_heads * dim], k, v [heads * vdim] (the first `conv_ch` columns, each block at its own
+ * offset), the low-rank inputs of the decay and of the output gate, and beta's logits.
+ *   q, k, v pass a causal convolution over `taps` tokens per channel, then silu; q and k become unit vectors per head (eps 1e-6 inside the
+ *   root), q times dim^-1/2;  g = exp(neg_a[h] * softplus(A2 a + dt_bias));  beta = sigmoid(b)
+ *   S <- g * S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+ *   out = o / rms(o) * norm_w * sigmoid(G2 gin)
+ * State per slot: S [heads, dim, vdim4] float32 (vdim4 = vdim rounded up to 4) and the convolution's inputs as a ring over positions
+ * [taps, conv_ch] float32.  A row at position 0 starts from zero whatever the slot holds. */
+typedef struct ChattsDeltaArgs {
+  const float* proj;
+  int ld_proj, off_q, off_k, off_v, off_a, off_g, off_b, conv_ch;
+  int heads, kv_heads, dim, vdim, taps, rank_a, rank_g;      /* ranks padded to multiples of 8 (zero weights) */
+  const float* conv_w;       /* [taps, conv_ch] */
+  const chatts_bf16* a2;     /* [heads * dim, ld_a2] */
+  const chatts_bf16* g2;     /* [heads * vdim, ld_g2] */
+  int ld_a2, ld_g2;
+  const float* dt_bias;      /* [heads * dim] */
+  const float* neg_a;        /* [heads] = -exp(A_log) */
+  const float* norm_w;       /* [vdim] */
+  float eps;
+  float* state;
+  float* ring;
+  const ChattsRow* rows;
+  int n_rows;
+  const ChattsSpan* spans;   /* device; chatts_delta_scan only */
+  int n_spans;
+  /* scratch of the several-token form: q / k [T, kv_heads * dim], v / o [T, heads * vdim], g [T, heads * dim] (in: A2 a, out: decay),
+   * gate [T, heads * vdim] (G2 gin), beta [T, heads]; row strides = the widths, except ld_dt / ld_gate */
+  float *q, *k, *v, *g, *gate, *beta, *o;
+  const float* dt;
+  int ld_dt, ld_gate;
+  ChattsOperand out;
+} ChattsDeltaArgs;
+int chatts_delta_decode(const ChattsDeltaArgs* args, chatts_stream_t stream);   /* every row is a segment of one token: one launch */
+int chatts_delta_prep(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* several tokens: convolutions, norms, decays ... */
+int chatts_delta_scan(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* ... the recurrence over every span ... */
+int chatts_delta_out(const ChattsDeltaArgs* args, chatts_stream_t stream);      /* ... norm and gate of the read-outs, ring update */
+
+/* ---- latent attention (latent.hip) ----
+ * Cache row of a token: [latent c, padded to rank_p | rotated key part, padded to rot_p] (both multiples of 32; cw = rank_p + rot_p), bf16 or
+ * float32, in pages of 2^log_block tokens found through the slot's row of the block table. */
+typedef struct ChattsLatentArgs {
+  float* proj;               /* [T, ld_proj]: unrotated and rotated query parts, latent [rank], key part [rot] */
+  int ld_proj, off_q, off_qr, off_c, off_kr;         /* unrotated parts [heads, dim_p] (dim_p: the layer's), rotated parts [heads, rot] */
+  int heads, dim, rot, rank, vdim, rank_p, rot_p;
+  float scale, eps;
+  const float* c_norm;       /* [rank] */
+  const float* cos_tab;      /* [positions, rot / 2], magnitude included */
+  const float* sin_tab;
+  void* cache;
+  int cache_f32;             /* 1: float32 pages, 0: bf16 */
+  const int32_t* table;      /* [slots, table_stride] */
+  int table_stride, log_block;
+  const ChattsRow* rows;
+  int n_rows;
+  ChattsOperand q;           /* absorbed queries [T, heads * cw]: [W_uk^T q_unrotated | rotated part] per head */
+  float* o;                  /* [T, heads * rank_p]: the weighted latents */
+  int n_splits;              /* decode: key ranges per sequence, merged afterwards */
+  float* partial;            /* [T, heads, n_splits, rank_p + 2] when n_splits > 1 */
+} ChattsLatentArgs;
+int chatts_latent_prep(const ChattsLatentArgs* args, chatts_stream_t stream);        /* rotation, latent norm, cache write */
+int chatts_latent_attend(const ChattsLatentArgs* args, chatts_stream_t stream);      /* absorbed form: all heads share the cached rows */
+
+/* ---- the composed decoder (mixdec.hip) ---- */
+#define CHATTS_MIX_LATENT 1
+#define CHATTS_MIX_DELTA 2
+typedef struct ChattsMixLayer {
+  int kind;                                          /* CHATTS_MIX_* */
+  const float *norm1, *norm1b, *norm2, *norm2b;      /* before / after the mixer, before / after the feed-forward; padded with zeros to width_p */
+  const chatts_bf16 *in, *in_t;                      /* the mixer's input projections, stacked: [in_n, width_p] (+ chatts_tile_bf16 copy) */
+  const chatts_bf16 *out, *out_t;                    /* [width_p, out_k] */
+  const chatts_bf16 *up, *up_t, *down, *down_t;      /* squared-relu feed-forward [ff, width_p], [width_p, ff]; up == NULL: none */
+  int in_n, out_k, ff;
+  const chatts_bf16 *uk, *uv;                        /* latent: W_uk^T per head [heads, rank_p, dim_p], W_uv per head [heads, vdim_p, rank_p] */
+  int dim_p, vdim_p, out_head;                       /* out_head: columns between heads in the input of `out` */
+  int dt_n, gate_n;                                  /* delta: rows of a2 / g2, padded to 16 */
+  ChattsLatentArgs latent;                           /* sizes, offsets and weights; the rest is filled in per step */
+  ChattsDeltaArgs delta;
+} ChattsMixLayer;
+typedef struct ChattsMixRun {      /* one pass through a layer */
+  int layer;
+  const float* add;                /* vector added to the residual stream before it, or NULL */
+  void* cache;                     /* latent: this run's pages */
+  float* state;                    /* delta: this run's states and convolution rings */
+  float* ring;
+} ChattsMixRun;
+typedef struct ChattsMixConfig {
+  int width, width_p, n_layers, n_runs, exact, t_max, max_slots, max_ctx;
+  int64_t vocab, vocab_p;
+  float eps;
+  int block_size, table_stride;
+} ChattsMixConfig;
+typedef struct ChattsMixBuffers {
+  const chatts_bf16 *embed, *head, *head_t;          /* [vocab, width_p], [vocab_p, width_p] */
+  const float* final_norm;
+  float *x, *y, *proj;                               /* [t_max, width_p] x 2, [t_max, max in_n] */
+  float *a_f32, *b_f32;                              /* operand buffers [t_max, widest] */
+  chatts_bf16 *a_hi, *a_lo, *b_hi, *b_lo;
+  float *q_f32, *o_lat, *partial;                    /* latent: [t_max, heads * cw] (32-bit runs), [t_max, heads * rank_p], splits */
+  chatts_bf16 *q_hi, *q_lo;
+  size_t partial_elems;
+  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dout, *ddt;
+  ChattsRow* rows;                                   /* device, [t_max] */
+  ChattsSpan* spans;                                 /* device, [max_slots] */
+  int32_t* table;                                    /* device, [max_slots, table_stride] */
+  float* logits;                                     /* [>= rows asked for, vocab_p] */
+  void* workspace;
+  size_t workspace_bytes;
+} ChattsMixBuffers;
+typedef struct ChattsMixDecoder ChattsMixDecoder;
+ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, const ChattsMixLayer* layers, const ChattsMixRun* runs, const ChattsMixBuffers* b);
+void chatts_mixdec_destroy(ChattsMixDecoder* d);
+size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const ChattsMixLayer* layers);
+/* x[0 .. t) = the residual stream of t rows described by buffers.rows / .spans (n_spans segments), embedded from `tokens` (device).  single:
+ * every segment is one row (decode kernels, no spans read). */
+int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, int n_spans, int single, chatts_stream_t stream);
+/* logits[i] = head . norm(x[index[i]]) for n rows (index: device, NULL = rows 0 .. n) */
+int chatts_mixdec_logits(ChattsMixDecoder* d, const int32_t* index, int n, float* logits, chatts_stream_t stream);
+/* decode: rows of slots 0 .. batch at pos[slot] (< 0: parked) with token[slot]; logits of all rows; nothing is selected here */
+int chatts_mixdec_decode(ChattsMixDecoder* d, int batch, const int64_t* token, const int32_t* pos, float* logits, chatts_stream_t stream);
+
 
 #ifdef __cplusplus
 }
