@@ -75,6 +75,7 @@ class Engine:
         self.slots = [None] * self.nslots
         self.produced = [0] * self.nslots
         self.active_key = None
+        self.check_ids = getattr(model, "check_ids", lambda ids: None)      # a prompt the model cannot take fails alone, at its own encoding
         self.mixed = hasattr(model, "set_slot_sampling")   # per-slot sampling settings on the device: no sampling groups
         self._since_sync = 0
         self._rid = 0
@@ -110,9 +111,12 @@ class Engine:
         if isinstance(r.prompt, (list, tuple)):         # token ids
             if r.timeseries:
                 raise ValueError("time series need a text prompt")
-            return [int(t) for t in r.prompt], None, []
+            ids = [int(t) for t in r.prompt]
+            self.check_ids(ids)
+            return ids, None, []
         text, encs, lens = self.processor.splice(r.prompt, [np.asarray(s, dtype=np.float64) for s in r.timeseries])
         ids = self.processor.tokenizer.encode(text)
+        self.check_ids(ids)
         ser = torch.from_numpy(self.processor.pad_stack(encs)) if encs else None
         return ids, ser, lens
 

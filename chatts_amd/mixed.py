@@ -365,9 +365,7 @@ class MixedDecoder(SlotModel):
         B, T = self.buf, len(ids)
         if T > self.t_max:
             raise ValueError(f"{T} tokens exceed max_prefill_tokens={self.t_max}")
-        V = self.config.vocab_size
-        if min(ids) < 0 or max(ids) >= V:
-            raise ValueError(f"token ids must lie in 0..{V - 1}")
+        self.check_ids(ids)
         B["ids"][:T].copy_(torch.tensor(ids, dtype=torch.int64))
         meta = torch.empty((T, 4), dtype=torch.int32)
         for row, t, pos0, slot in segs:
@@ -421,6 +419,12 @@ class MixedDecoder(SlotModel):
     def request_tokens(self, ids, series=None, lengths=None):
         return len(ids)
 
+    def check_ids(self, ids):
+        if not len(ids):
+            raise ValueError("an empty prompt")
+        if min(ids) < 0 or max(ids) >= self.config.vocab_size:
+            raise ValueError(f"token ids must lie in 0..{self.config.vocab_size - 1}")
+
     def _request_idents(self, ids, series, lengths):
         return None
 
@@ -428,13 +432,10 @@ class MixedDecoder(SlotModel):
         if series is not None and len(series):
             raise ValueError(f"{self.config.name} takes token ids only, no time series")
         ids = [int(t) for t in ids]
+        self.check_ids(ids)
         T = len(ids)
-        if T < 1:
-            raise ValueError("an empty prompt")
         if T + max_new_tokens > self.max_ctx:
             raise ValueError(f"prompt ({T}) + max_new_tokens ({max_new_tokens}) exceeds max_ctx={self.max_ctx}")
-        if min(ids) < 0 or max(ids) >= self.config.vocab_size:
-            raise ValueError(f"token ids must lie in 0..{self.config.vocab_size - 1}")
         self.reserve_kv(slot, T + max_new_tokens)
         self.prefix_stats["requests"] += 1
         self.prefix_stats["tokens_prefilled"] += T

@@ -21,6 +21,9 @@ from . import _lib
 class SlotModel:
     step_is_idempotent = True        # a decode step repeated from the same positions and tokens changes nothing (pure KV caches)
 
+    def check_ids(self, ids):
+        """raise ValueError for a prompt the model cannot take (before it shares a pass with others)"""
+
     # ---- one ragged batch: any number of new tokens per slot --------------------------------------------------------------
     def step_tokens(self, entries):
         """entries: list of (slot, new token ids, wanted places among them), slots distinct.  Runs all tokens as one batch on top of what
