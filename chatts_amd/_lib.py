@@ -132,16 +132,27 @@ class DeltaArgs(C.Structure):
                 [("conv_w", c_void_p), ("a2", c_void_p), ("g2", c_void_p), ("ld_a2", c_int), ("ld_g2", c_int), ("dt_bias", c_void_p),
                  ("neg_a", c_void_p), ("norm_w", c_void_p), ("eps", c_float), ("state", c_void_p), ("ring", c_void_p), ("rows", c_void_p),
                  ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int)] +
-                [(n, c_void_p) for n in ("q", "k", "v", "g", "gate", "beta", "o", "dt")] + [("ld_dt", c_int), ("ld_gate", c_int), ("out", Operand)])
+                [(n, c_void_p) for n in ("q", "k", "v", "g", "gate", "beta", "kq", "o", "dt")] + [("ld_dt", c_int), ("ld_gate", c_int), ("out", Operand)])
 
 
 class LatentArgs(C.Structure):
     """ChattsLatentArgs: attention over a paged latent cache (csrc/latent.hip)"""
     _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_qr", "off_c", "off_kr", "heads", "dim", "rot", "rank", "vdim",
-                                                             "rank_p", "rot_p")] +
+                                                             "rank_p", "rot_p", "dim_p")] +
                 [("scale", c_float), ("eps", c_float), ("c_norm", c_void_p), ("cos_tab", c_void_p), ("sin_tab", c_void_p), ("cache", c_void_p),
                  ("cache_f32", c_int), ("table", c_void_p), ("table_stride", c_int), ("log_block", c_int), ("rows", c_void_p), ("n_rows", c_int),
-                 ("q", Operand), ("o", c_void_p), ("n_splits", c_int), ("partial", c_void_p)])
+                 ("q", Operand), ("o", c_void_p), ("n_splits", c_int), ("partial", c_void_p), ("qx", c_void_p)])
+
+
+class Span(C.Structure):
+    _fields_ = [(n, c_int32) for n in ("row0", "t", "pos0", "slot", "base")]
+
+
+class LatentExpandArgs(C.Structure):
+    _fields_ = ([("latent", C.POINTER(LatentArgs)), ("spans", C.POINTER(Span)), ("spans_dev", c_void_p)] +
+                [(n, c_int) for n in ("n_spans", "vdim_p", "out_head", "max_rows")] +
+                [(n, c_void_p) for n in ("uk", "uv", "cbuf", "krbuf", "zero", "k_hi", "k_lo", "v_hi", "v_lo")] +
+                [("out", Operand), ("workspace", c_void_p), ("workspace_bytes", c_size_t)])
 
 
 MIX_LATENT, MIX_DELTA = 1, 2
@@ -150,7 +161,7 @@ MIX_LATENT, MIX_DELTA = 1, 2
 class MixLayer(C.Structure):
     _fields_ = ([("kind", c_int)] + [(n, c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "in_t", "out", "out_t", "up", "up_t", "down",
                                                              "down_t")] +
-                [(n, c_int) for n in ("in_n", "out_k", "ff")] + [("uk", c_void_p), ("uv", c_void_p)] +
+                [(n, c_int) for n in ("in_n", "out_k", "ff")] + [("uk", c_void_p), ("uv", c_void_p), ("ukx", c_void_p), ("uvx", c_void_p)] +
                 [(n, c_int) for n in ("dim_p", "vdim_p", "out_head", "dt_n", "gate_n")] + [("latent", LatentArgs), ("delta", DeltaArgs)])
 
 
@@ -159,14 +170,15 @@ class MixRun(C.Structure):
 
 
 class MixConfig(C.Structure):
-    _fields_ = ([(n, c_int) for n in ("width", "width_p", "n_layers", "n_runs", "exact", "t_max", "max_slots", "max_ctx")] +
+    _fields_ = ([(n, c_int) for n in ("width", "width_p", "n_layers", "n_runs", "exact", "t_max", "max_slots", "max_ctx", "expand_rows")] +
                 [("vocab", c_int64), ("vocab_p", c_int64), ("eps", c_float), ("block_size", c_int), ("table_stride", c_int)])
 
 
 class MixBuffers(C.Structure):
     _fields_ = ([(n, c_void_p) for n in ("embed", "head", "head_t", "final_norm", "x", "y", "proj", "a_f32", "b_f32", "a_hi", "a_lo", "b_hi", "b_lo",
                                          "q_f32", "o_lat", "partial", "q_hi", "q_lo")] + [("partial_elems", c_size_t)] +
-                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dout", "ddt", "rows", "spans", "table", "logits", "workspace")] +
+                [(n, c_void_p) for n in ("qx", "cbuf", "krbuf", "kx_hi", "kx_lo", "vx_hi", "vx_lo", "zero")] +
+                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dkq", "dout", "ddt", "rows", "spans", "table", "logits", "workspace")] +
                 [("workspace_bytes", c_size_t)])
 
 
@@ -262,7 +274,10 @@ SIGNATURES = {
     "chatts_mixdec_create": (c_void_p, [C.POINTER(MixConfig), C.POINTER(MixLayer), C.POINTER(MixRun), C.POINTER(MixBuffers)]),
     "chatts_mixdec_destroy": (None, [c_void_p]),
     "chatts_mixdec_workspace": (c_size_t, [C.POINTER(MixConfig), C.POINTER(MixLayer)]),
-    "chatts_mixdec_forward": (c_int, [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
+    "chatts_latent_can_expand": (c_int, [c_int, c_int, c_int, c_int]),
+    "chatts_latent_expanded": (c_int, [C.POINTER(LatentExpandArgs), c_void_p]),
+    "chatts_mixdec_forward": (c_int, [c_void_p, c_void_p, c_int, C.POINTER(Span), c_int, c_int, c_void_p]),
+    "chatts_mixdec_plan": (c_int, [c_void_p, C.POINTER(Span), c_int]),
     "chatts_mixdec_logits": (c_int, [c_void_p, c_void_p, c_int, c_void_p, c_void_p]),
     "chatts_mixdec_decode": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p]),
     # tensor-parallel exchange (tp.hip)

@@ -9,11 +9,11 @@
 //    DPP row reductions and columns never talk to each other; out norms and gates.
 // The ring of convolution inputs is indexed by position modulo taps: the current token's entry is never one that the same step reads, so
 // heads that share a q / k head need no ordering, and a sequence that starts over in a used slot reads none of the old entries.
+#include <type_traits>
+
 #include "common.h"
 
 namespace chatts {
-
-__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
 // ---- one token per sequence -----------------------------------------------------------------------------------------------------
 // thread (tx, ty): 4 consecutive value columns tx * 4, key rows ty + TY * r.
@@ -91,7 +91,7 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
         acc += bf16_hi(wv[j]) * x[c + 2 * j + 1];
       }
     }
-    if (dec) sg[i] = expf(na * softplus_f(acc + p.dt_bias[o]));
+    if (dec) sg[i] = exp_hw(na * softplus_f(acc + p.dt_bias[o]));
     else sgate[i - dim] = sigmoid_f(acc);
   }
   const float beta = sigmoid_f(pr[p.off_b + h]);
@@ -139,72 +139,164 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
 }
 
 // ---- several tokens: what is parallel over tokens -------------------------------------------------------------------------------
-// convolution + silu of channel ch of row r; earlier tokens come from the segment's own rows or from the ring
-__device__ __forceinline__ float conv_silu(const ChattsDeltaArgs& p, int row, const ChattsRow& R, int ch) {
-  float acc = 0.f;
-  const float* ring = p.ring + (size_t)R.slot * p.taps * p.conv_ch;
-  for (int j = 0; j < p.taps; ++j) {
-    const int lag = p.taps - 1 - j, q = R.pos - lag;
-    if (q < 0) continue;
-    const float x = row - lag >= R.first ? p.proj[(size_t)(row - lag) * p.ld_proj + ch] : ring[(size_t)(q % p.taps) * p.conv_ch + ch];
-    acc += p.conv_w[(size_t)j * p.conv_ch + ch] * x;
+constexpr int kPrepRows = 4;      // consecutive rows of a wave: the convolution's window slides in registers
+
+// convolution + silu of channel ch for rows row0 .. row0 + kPrepRows.  Tokens before a row's segment come from the ring.
+template <int TAPS>      // 0: any number of taps
+__device__ __forceinline__ void conv_rows(const ChattsDeltaArgs& p, int row0, const ChattsRow (&R)[kPrepRows], int ch, float (&y)[kPrepRows]) {
+  if constexpr (TAPS > 0) {
+    float x[kPrepRows + TAPS - 1], w[TAPS];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = p.conv_w[(size_t)j * p.conv_ch + ch];
+#pragma unroll
+    for (int j = 0; j < kPrepRows + TAPS - 1; ++j) {
+      int r = row0 + j - (TAPS - 1);
+      r = r < 0 ? 0 : (r > p.n_rows - 1 ? p.n_rows - 1 : r);
+      x[j] = p.proj[(size_t)r * p.ld_proj + ch];
+    }
+#pragma unroll
+    for (int i = 0; i < kPrepRows; ++i) {
+      float acc = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        const int lag = TAPS - 1 - j;
+        float v = x[i + j];
+        if (row0 + i - lag < R[i].first) {      // (uniform over the wave)
+          const int q = R[i].pos - lag;
+          v = q < 0 ? 0.f : p.ring[((size_t)R[i].slot * TAPS + q % TAPS) * p.conv_ch + ch];
+        }
+        acc += w[j] * v;
+      }
+      y[i] = acc * sigmoid_f(acc);
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < kPrepRows; ++i) {
+      float acc = 0.f;
+      for (int j = 0; j < p.taps; ++j) {
+        const int lag = p.taps - 1 - j, q = R[i].pos - lag, r = row0 + i - lag;
+        if (q < 0) continue;
+        acc += p.conv_w[(size_t)j * p.conv_ch + ch] * (r >= R[i].first ? p.proj[(size_t)r * p.ld_proj + ch]
+                                                                       : p.ring[((size_t)R[i].slot * p.taps + q % p.taps) * p.conv_ch + ch]);
+      }
+      y[i] = acc * sigmoid_f(acc);
+    }
   }
-  return acc * sigmoid_f(acc);
 }
 
-// a wave takes one item of a row at a time: a q or k head, 64 channels of v, 64 decays
+// a wave takes one item of kPrepRows rows at a time: a q / k head, 64 channels of v, 64 decays, 64 betas
+template <int TAPS, int NCH>      // NCH: 64-channel pieces of a q / k head
 __global__ __launch_bounds__(256) void delta_prep_kernel(ChattsDeltaArgs p) {
-  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = blockIdx.y * 4 + (threadIdx.x >> 6), waves = gridDim.y * 4;
-  const ChattsRow R = p.rows[row];
-  if (R.pos < 0) return;
+  const int row0 = blockIdx.x * kPrepRows, lane = threadIdx.x & 63, wave = blockIdx.y * 4 + (threadIdx.x >> 6), waves = gridDim.y * 4;
+  ChattsRow R[kPrepRows];
+  bool live[kPrepRows];
+#pragma unroll
+  for (int i = 0; i < kPrepRows; ++i) {
+    R[i] = p.rows[row0 + i < p.n_rows ? row0 + i : p.n_rows - 1];
+    live[i] = row0 + i < p.n_rows && R[i].pos >= 0;
+    if (!live[i]) R[i] = ChattsRow{0, 0, row0 + i < p.n_rows ? row0 + i : p.n_rows - 1, 0};
+  }
   const int dim = p.dim, nv = p.heads * p.vdim, ng = p.heads * dim;
   const int vchunks = (nv + 63) / 64, gchunks = (ng + 63) / 64, bchunks = (p.heads + 63) / 64;
-  const int items = 2 * p.kv_heads + vchunks + gchunks + bchunks;
+  const int items = p.kv_heads + vchunks + gchunks + bchunks;
   for (int it = wave; it < items; it += waves) {
     int e = it;
-    if (e < 2 * p.kv_heads) {
-      const bool isq = e < p.kv_heads;
-      const int hk = isq ? e : e - p.kv_heads, base = (isq ? p.off_q : p.off_k) + hk * dim;
-      float v[4], ss = 0.f;
+    if (e < p.kv_heads) {
+      float q[NCH][kPrepRows], k[NCH][kPrepRows], qs[kPrepRows], ks[kPrepRows], qk[kPrepRows];
 #pragma unroll
-      for (int c = 0; c < 4; ++c) {
-        const int i = c * 64 + lane;
-        v[c] = i < dim ? conv_silu(p, row, R, base + i) : 0.f;
-        ss += v[c] * v[c];
+      for (int i = 0; i < kPrepRows; ++i) qs[i] = ks[i] = qk[i] = 0.f;
+#pragma unroll
+      for (int c = 0; c < NCH; ++c) {
+        const int ch = c * 64 + lane;
+        const bool ok = ch < dim;
+        conv_rows<TAPS>(p, row0, R, p.off_q + e * dim + (ok ? ch : 0), q[c]);
+        conv_rows<TAPS>(p, row0, R, p.off_k + e * dim + (ok ? ch : 0), k[c]);
+#pragma unroll
+        for (int i = 0; i < kPrepRows; ++i) {
+          if (!ok) q[c][i] = k[c][i] = 0.f;
+          qs[i] += q[c][i] * q[c][i];
+          ks[i] += k[c][i] * k[c][i];
+          qk[i] += q[c][i] * k[c][i];
+        }
       }
-      ss = wave_sum(ss);
-      const float f = (isq ? rsqrtf((float)dim) : 1.0f) / sqrtf(ss + 1e-6f);
-      float* dst = (isq ? p.q : p.k) + ((size_t)row * p.kv_heads + hk) * dim;
+      const float qscale = rsqrtf((float)dim);
 #pragma unroll
-      for (int c = 0; c < 4; ++c)
-        if (c * 64 + lane < dim) dst[c * 64 + lane] = v[c] * f;
+      for (int i = 0; i < kPrepRows; ++i) {
+        const float fq = qscale / sqrtf(wave_sum(qs[i]) + 1e-6f), fk = 1.0f / sqrtf(wave_sum(ks[i]) + 1e-6f), d = wave_sum(qk[i]);
+        if (!live[i]) continue;
+        const size_t at = (size_t)(row0 + i) * p.kv_heads + e;
+#pragma unroll
+        for (int c = 0; c < NCH; ++c) {
+          const int ch = c * 64 + lane;
+          if (ch < dim) {
+            p.q[at * dim + ch] = q[c][i] * fq;
+            p.k[at * dim + ch] = k[c][i] * fk;
+          }
+        }
+        if (lane == 0) p.kq[at] = d * fq * fk;
+      }
       continue;
     }
-    e -= 2 * p.kv_heads;
+    e -= p.kv_heads;
     if (e < vchunks) {
-      const int i = e * 64 + lane;
-      if (i < nv) p.v[(size_t)row * nv + i] = conv_silu(p, row, R, p.off_v + i);
+      const int ch = e * 64 + lane;
+      if (ch >= nv) continue;
+      float y[kPrepRows];
+      conv_rows<TAPS>(p, row0, R, p.off_v + ch, y);
+#pragma unroll
+      for (int i = 0; i < kPrepRows; ++i)
+        if (live[i]) p.v[(size_t)(row0 + i) * nv + ch] = y[i];
       continue;
     }
     e -= vchunks;
     if (e < gchunks) {
-      const int i = e * 64 + lane;
-      if (i < ng) p.g[(size_t)row * ng + i] = expf(p.neg_a[i / dim] * softplus_f(p.dt[(size_t)row * p.ld_dt + i] + p.dt_bias[i]));
+      const int ch = e * 64 + lane;
+      if (ch >= ng) continue;
+      const float na = p.neg_a[ch / dim], bias = p.dt_bias[ch];
+      float x[kPrepRows];
+#pragma unroll
+      for (int i = 0; i < kPrepRows; ++i) x[i] = live[i] ? p.dt[(size_t)(row0 + i) * p.ld_dt + ch] : 0.f;
+#pragma unroll
+      for (int i = 0; i < kPrepRows; ++i)
+        if (live[i]) p.g[(size_t)(row0 + i) * ng + ch] = exp_hw(na * softplus_f(x[i] + bias));
       continue;
     }
     e -= gchunks;
-    const int i = e * 64 + lane;
-    if (i < p.heads) p.beta[(size_t)row * p.heads + i] = sigmoid_f(p.proj[(size_t)row * p.ld_proj + p.off_b + i]);
+    const int ch = e * 64 + lane;
+    if (ch < p.heads)
+#pragma unroll
+      for (int i = 0; i < kPrepRows; ++i)
+        if (live[i]) p.beta[(size_t)(row0 + i) * p.heads + ch] = sigmoid_f(p.proj[(size_t)(row0 + i) * p.ld_proj + p.off_b + ch]);
   }
 }
 
+template <int TAPS>
+static void launch_prep(const ChattsDeltaArgs* a, hipStream_t s) {
+  const int items = a->kv_heads + (a->heads * a->vdim + 63) / 64 + (a->heads * a->dim + 63) / 64 + (a->heads + 63) / 64;
+  const dim3 g((a->n_rows + kPrepRows - 1) / kPrepRows, (items + 7) / 8), b(256);
+  if (a->dim <= 64) hipLaunchKernelGGL((delta_prep_kernel<TAPS, 1>), g, b, 0, s, *a);
+  else if (a->dim <= 128) hipLaunchKernelGGL((delta_prep_kernel<TAPS, 2>), g, b, 0, s, *a);
+  else hipLaunchKernelGGL((delta_prep_kernel<TAPS, 4>), g, b, 0, s, *a);
+}
+
 // ---- the recurrence over a span: grid (heads * column blocks, spans), 4 waves x 4 columns ---------------------------------------------
-// Lane l of a row of 16 holds key channels (c * 16 + l) * 4 .. + 3 (c < NC) of its column.
+// Lane l of a row of 16 holds key channels (c * 16 + l) * 4 .. + 3 (c < NC) of its column.  Both sums over key channels are taken on the
+// decayed state before the update, S^T k for u and S^T q for the read-out (o = S^T q + (k . q) u with the k . q of prep): their reductions
+// are independent of each other and only the first is on the token-to-token path.  Tokens are staged in LDS kT at a time and walked
+// fully unrolled, the next token's operands requested while the current one is computed; beta, k . q and v of the kT tokens sit in the
+// lanes of a row and are broadcast from there.  Rows past the end of the span are staged as k = q = 0, g = 1, beta = 0: they change nothing.
+template <int T, int N, typename F>
+__device__ __forceinline__ void unroll_tokens(F&& f) {
+  if constexpr (T < N) {
+    f(std::integral_constant<int, T>{});
+    unroll_tokens<T + 1, N>(f);
+  }
+}
 template <int NC>
 __global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int colblocks) {
-  constexpr int D = NC * 64, kScanT = NC <= 2 ? 16 : 8;      // tokens staged together
-  __shared__ __attribute__((aligned(16))) float sk[2][kScanT][D], sq[2][kScanT][D], sg[2][kScanT][D];
-  __shared__ float sv[2][kScanT][16], so[kScanT][16], sb[2][kScanT];
+  constexpr int D = NC * 64, kT = NC <= 2 ? 16 : 8;
+  __shared__ __attribute__((aligned(16))) float sk[2][kT][D], sq[2][kT][D], sg[2][kT][D];
+  __shared__ float so[kT][17];
   const ChattsSpan sp = p.spans[blockIdx.y];
   if (sp.t < 1) return;
   const int h = blockIdx.x / colblocks, cb = blockIdx.x - h * colblocks, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -212,7 +304,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int 
   const int l16 = lane & 15, cl = wave * 4 + (lane >> 4), col = cb * 16 + cl;
   const bool live = col < vdim;
   float* S = p.state + ((size_t)sp.slot * p.heads + h) * dim * v4;
-  float s[NC][4];
+  f32x4 s[NC];
 #pragma unroll
   for (int c = 0; c < NC; ++c)
 #pragma unroll
@@ -221,74 +313,93 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int 
       s[c][j] = sp.pos0 > 0 && live && i < dim ? S[(size_t)i * v4 + col] : 0.f;
     }
   const int qrow = p.kv_heads * dim, grow = p.heads * dim, vrow = p.heads * vdim;
-  constexpr int PER = kScanT * D / 256;      // values of one of k / q / g per thread and stage
-  float rk[PER], rq[PER], rg[PER], rv, rb;
+  constexpr int PER = kT * D / 256, TS = 256 / D;      // values of one of k / q / g per thread and stage, tokens between them
+  const int fi = tid % D, ft = tid / D;
+  const bool fok = fi < dim;
+  const float* gk = p.k + (size_t)sp.row0 * qrow + hk * dim + (fok ? fi : 0);
+  const float* gq = p.q + (size_t)sp.row0 * qrow + hk * dim + (fok ? fi : 0);
+  const float* gg = p.g + (size_t)sp.row0 * grow + h * dim + (fok ? fi : 0);
+  const float* gv = p.v + (size_t)sp.row0 * vrow + h * vdim + (live ? col : 0);
+  const float* gb = p.beta + (size_t)sp.row0 * p.heads + h;
+  const float* gc = p.kq + (size_t)sp.row0 * p.kv_heads + hk;
+  float rk[PER], rq[PER], rg[PER], nv, nb, nc;      // the next stage; v, beta, k . q of token l16
   auto fetch = [&](int t0) {
 #pragma unroll
     for (int e = 0; e < PER; ++e) {
-      const int at = e * 256 + tid, t = t0 + at / D, i = at % D;
-      const bool ok = t < sp.t && i < dim;
-      const size_t r = sp.row0 + t;
-      rk[e] = ok ? p.k[r * qrow + hk * dim + i] : 0.f;
-      rq[e] = ok ? p.q[r * qrow + hk * dim + i] : 0.f;
-      rg[e] = ok ? p.g[r * grow + h * dim + i] : 1.f;
+      int t = t0 + ft + e * TS;
+      const bool ok = fok && t < sp.t;
+      if (t > sp.t - 1) t = sp.t - 1;
+      rk[e] = gk[(size_t)t * qrow];
+      rq[e] = gq[(size_t)t * qrow];
+      rg[e] = gg[(size_t)t * grow];
+      if (!ok) { rk[e] = rq[e] = 0.f; rg[e] = 1.f; }
     }
-    const int t = t0 + (tid >> 4), c = cb * 16 + (tid & 15);
-    rv = tid < kScanT * 16 && t < sp.t && c < vdim ? p.v[(size_t)(sp.row0 + t) * vrow + h * vdim + c] : 0.f;
-    rb = tid < kScanT && t0 + tid < sp.t ? p.beta[(size_t)(sp.row0 + t0 + tid) * p.heads + h] : 0.f;
+    int t = t0 + (l16 & (kT - 1));
+    const bool ok = t < sp.t;
+    if (!ok) t = sp.t - 1;
+    nv = gv[(size_t)t * vrow];
+    nb = gb[(size_t)t * p.heads];
+    nc = gc[(size_t)t * p.kv_heads];
+    if (!ok) nb = 0.f;
   };
   auto stage = [&](int b) {
 #pragma unroll
     for (int e = 0; e < PER; ++e) {
-      const int at = e * 256 + tid, t = at / D, i = at % D;
-      sk[b][t][i] = rk[e];
-      sq[b][t][i] = rq[e];
-      sg[b][t][i] = rg[e];
+      const int t = ft + e * TS;
+      sk[b][t][fi] = rk[e];
+      sq[b][t][fi] = rq[e];
+      sg[b][t][fi] = rg[e];
     }
-    if (tid < kScanT * 16) sv[b][tid >> 4][tid & 15] = rv;
-    if (tid < kScanT) sb[b][tid] = rb;
+  };
+  struct Ops { f32x4 k[NC], q[NC], g[NC]; };
+  auto read = [&](int b, int t, Ops& o) __attribute__((always_inline)) {
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int i = (c * 16 + l16) * 4;
+      o.g[c] = *reinterpret_cast<const f32x4*>(&sg[b][t][i]);
+      o.k[c] = *reinterpret_cast<const f32x4*>(&sk[b][t][i]);
+      o.q[c] = *reinterpret_cast<const f32x4*>(&sq[b][t][i]);
+    }
   };
   fetch(0);
   stage(0);
   __syncthreads();
   int b = 0;
-  for (int t0 = 0; t0 < sp.t; t0 += kScanT, b ^= 1) {
-    if (t0 + kScanT < sp.t) fetch(t0 + kScanT);
-    const int n = sp.t - t0 < kScanT ? sp.t - t0 : kScanT;
-    for (int t = 0; t < n; ++t) {
-      f32x4 k[NC], q[NC], g[NC];
-#pragma unroll
-      for (int c = 0; c < NC; ++c) {
-        const int i = (c * 16 + l16) * 4;
-        k[c] = *reinterpret_cast<const f32x4*>(&sk[b][t][i]);
-        g[c] = *reinterpret_cast<const f32x4*>(&sg[b][t][i]);
-        q[c] = *reinterpret_cast<const f32x4*>(&sq[b][t][i]);
-      }
-      const float beta = sb[b][t], v = sv[b][t][cl];
-      float d0 = 0.f, d1 = 0.f;
-#pragma unroll
-      for (int c = 0; c < NC; ++c) {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) s[c][j] *= g[c][j];
-        d0 += s[c][0] * k[c][0]; d1 += s[c][1] * k[c][1];
-        d0 += s[c][2] * k[c][2]; d1 += s[c][3] * k[c][3];
-      }
-      const float u = beta * (v - row16_sum(d0 + d1));
-      float o0 = 0.f, o1 = 0.f;
+  for (int t0 = 0; t0 < sp.t; t0 += kT, b ^= 1) {
+    const float beta = nb, bv = nb * nv, kq = nc;      // of token l16
+    float keep = 0.f;
+    Ops ops[2];
+    read(b, 0, ops[0]);
+    const bool more = t0 + kT < sp.t;
+    if (more) fetch(t0 + kT);
+    unroll_tokens<0, kT>([&](auto tc) __attribute__((always_inline)) {
+      constexpr int t = decltype(tc)::value;
+      if constexpr (t + 1 < kT) read(b, t + 1, ops[(t + 1) & 1]);
+      const Ops& o = ops[t & 1];
+      float d[2] = {0.f, 0.f}, e[2] = {0.f, 0.f};
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) s[c][j] += k[c][j] * u;
-        o0 += s[c][0] * q[c][0]; o1 += s[c][1] * q[c][1];
-        o0 += s[c][2] * q[c][2]; o1 += s[c][3] * q[c][3];
+        for (int j = 0; j < 4; ++j) s[c][j] *= o.g[c][j];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) d[j & 1] += s[c][j] * o.k[c][j];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) e[j & 1] += s[c][j] * o.q[c][j];
       }
-      const float o = row16_sum(o0 + o1);
-      if (l16 == 0) so[t][cl] = o;
-    }
-    if (t0 + kScanT < sp.t) stage(b ^ 1);
+      const float dd = row16_sum(d[0] + d[1]), ee = row16_sum(e[0] + e[1]);
+      const float u = row_bcast<t>(bv) - row_bcast<t>(beta) * dd;      // beta (v - S^T k)
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) s[c][j] += o.k[c][j] * u;
+      const float out = ee + row_bcast<t>(kq) * u;
+      keep = l16 == t ? out : keep;
+    });
+    if (l16 < kT) so[l16][cl] = keep;
+    if (more) stage(b ^ 1);
     __syncthreads();
     const int t = tid >> 4, c = cb * 16 + (tid & 15);
-    if (t < n && c < vdim) p.o[(size_t)(sp.row0 + t0 + t) * vrow + h * vdim + c] = so[t][tid & 15];
+    if (t < kT && t0 + t < sp.t && c < vdim) p.o[(size_t)(sp.row0 + t0 + t) * vrow + h * vdim + c] = so[t][tid & 15];
     __syncthreads();
   }
   if (live)
@@ -369,18 +480,21 @@ extern "C" int chatts_delta_decode(const ChattsDeltaArgs* a, chatts_stream_t str
 
 extern "C" int chatts_delta_prep(const ChattsDeltaArgs* a, chatts_stream_t stream) {
   if (const int rc = check_delta(a, "delta_prep")) return rc;
-  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->dt, CHATTS_E_BADARG, "delta_prep: null scratch");
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->kq && a->dt, CHATTS_E_BADARG, "delta_prep: null scratch");
   if (a->n_rows == 0) return CHATTS_OK;
-  const int items = 2 * a->kv_heads + (a->heads * a->vdim + 63) / 64 + (a->heads * a->dim + 63) / 64 + 1;
-  const int y = (items + 15) / 16;
-  hipLaunchKernelGGL(delta_prep_kernel, dim3(a->n_rows, y), dim3(256), 0, as_stream(stream), *a);
+  switch (a->taps) {
+    case 2: launch_prep<2>(a, as_stream(stream)); break;
+    case 3: launch_prep<3>(a, as_stream(stream)); break;
+    case 4: launch_prep<4>(a, as_stream(stream)); break;
+    default: launch_prep<0>(a, as_stream(stream)); break;
+  }
   CHATTS_CHECK_LAUNCH("delta_prep");
   return CHATTS_OK;
 }
 
 extern "C" int chatts_delta_scan(const ChattsDeltaArgs* a, chatts_stream_t stream) {
   if (const int rc = check_delta(a, "delta_scan")) return rc;
-  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->o && a->spans, CHATTS_E_BADARG, "delta_scan: null scratch");
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->kq && a->o && a->spans, CHATTS_E_BADARG, "delta_scan: null scratch");
   if (a->n_spans == 0) return CHATTS_OK;
   const int cb = (a->vdim + 15) / 16;
   const dim3 g(a->heads * cb, a->n_spans), b(256);
@@ -388,7 +502,6 @@ extern "C" int chatts_delta_scan(const ChattsDeltaArgs* a, chatts_stream_t strea
   switch ((a->dim + 63) / 64) {
     case 1: hipLaunchKernelGGL(delta_scan_kernel<1>, g, b, 0, s, *a, cb); break;
     case 2: hipLaunchKernelGGL(delta_scan_kernel<2>, g, b, 0, s, *a, cb); break;
-    case 3: hipLaunchKernelGGL(delta_scan_kernel<3>, g, b, 0, s, *a, cb); break;
     default: hipLaunchKernelGGL(delta_scan_kernel<4>, g, b, 0, s, *a, cb); break;
   }
   CHATTS_CHECK_LAUNCH("delta_scan");

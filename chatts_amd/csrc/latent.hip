@@ -7,8 +7,10 @@
 //   * latent_prep_kernel: rotation of the query parts, norm of the latent, rotation of the key part, cache write
 //   * head_linear_kernel: W_uk^T on the queries, W_uv on the weighted latents (a product per head)
 //   * latent_attend_kernel: one (row, head) per workgroup on the vector units, float32 or bf16 cache: the 32-bit runs and odd sizes
-//   * latent_decode_kernel: 16 heads of a row per workgroup on the matrix pipe over every n_splits-th key tile, bf16 cache, partials merged by
-//     latent_merge_kernel
+//   * latent_decode_kernel: 16 heads of a row per workgroup on the matrix pipe, bf16 cache, the keys spread over waves and workgroups, partials
+//     merged by latent_merge_kernel
+// The expanded form (first half of each line) does fewer products per key once many queries share it: prompts take it
+//   * latent_gather_kernel, two projections (keys; values, transposed by exchanging the operands) and latent_prefill_kernel, a flash loop
 #include "gemm_common.h"
 
 namespace chatts {
@@ -42,7 +44,15 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(ChattsLatentArgs p) {
   const int half = p.rot >> 1;
   const float* ct = p.cos_tab + (size_t)R.pos * half;
   const float* st = p.sin_tab + (size_t)R.pos * half;
-  for (int e = tid; e < p.heads * p.rot_p; e += 256) {      // the rotated part of every head's absorbed query, padding included
+  if (p.qx)                                                  // expanded form: the unrotated part as it is
+    for (int e = tid; e < p.heads * (p.dim_p >> 2); e += 256) {
+      const int h = e / (p.dim_p >> 2), c = (e - h * (p.dim_p >> 2)) * 4;
+      const f32x4 v = *reinterpret_cast<const f32x4*>(pr + p.off_q + h * p.dim_p + c);
+      typedef __bf16 bf16x4_t __attribute__((ext_vector_type(4)));
+      *reinterpret_cast<bf16x4_t*>(p.qx + (size_t)row * p.heads * (p.dim_p + p.rot_p) + h * (p.dim_p + p.rot_p) + c) =
+          (bf16x4_t){(__bf16)v.x, (__bf16)v.y, (__bf16)v.z, (__bf16)v.w};
+    }
+  for (int e = tid; e < p.heads * p.rot_p; e += 256) {      // the rotated part of every head's query, padding included
     const int h = e / p.rot_p, i = e - h * p.rot_p;
     float v = 0.f;
     if (i < p.rot) {
@@ -51,7 +61,8 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(ChattsLatentArgs p) {
       const float u = q[f], w = q[f + half];
       v = i < half ? u * ct[f] - w * st[f] : w * ct[f] + u * st[f];
     }
-    store_operand(p.q, row, h * cw + p.rank_p + i, v);
+    if (p.q.f32 || p.q.hi) store_operand(p.q, row, h * cw + p.rank_p + i, v);
+    if (p.qx) p.qx[(size_t)row * p.heads * (p.dim_p + p.rot_p) + h * (p.dim_p + p.rot_p) + p.dim_p + i] = to_cache<uint16_t>(v);
   }
   float ss = 0.f;
   for (int i = tid; i < p.rank; i += 256) { const float v = pr[p.off_c + i]; ss += v * v; }
@@ -131,151 +142,362 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(ChattsLatentArgs p) 
   }
 }
 
-// ---- absorbed attention on the matrix pipe: grid (head tiles, rows, splits), 16 heads x 64 keys per step ----
-// S = Q K^T: wave w takes keys 16 w .. + 15 of the tile; the scores meet in LDS, 16 lanes per head do the online softmax; O += P C: wave w
-// takes latent columns [w, w + 1) * rank_p / 4, its B fragments gathered from the same LDS rows (8 keys of one column per lane).  Q enters
-// as bf16 hi + lo, P too: only the cache's own rounding to bf16 is left.
-constexpr int kLdP = 72;
-template <int NT>      // 16-column fragments of the latent per wave (rank_p <= 64 NT)
-__global__ __launch_bounds__(256) void latent_decode_kernel(ChattsLatentArgs p) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int ht = blockIdx.x, row = blockIdx.y, split = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int cw = p.rank_p + p.rot_p, ldk = cw + 8, cv = cw >> 3;
+// ---- absorbed attention on the matrix pipe: grid (splits, rows, head tiles), 16 heads per workgroup -------------------------------------
+// A wave works alone on tiles of 32 keys (every 4 n_splits-th), which LDS-DMA brings into its own LDS region: S^T = K Q^T reads rows of it as A
+// fragments, so a lane ends up with 8 scores of one head (column = lane & 15); O^T = C^T P^T reads it transposed, and its B fragment IS the
+// 8 probabilities of the lane.  K slot 8 g + j of that product means key 4 g + j (j < 4) or 16 + 4 g + j - 4, on both sides.  No barrier until
+// the four waves' sums are merged at the end; while one wave waits for its tile the other three compute.
+// 16-byte chunk c of row r lies at position c ^ (r & swizzle): neither way of reading meets the same banks in every row.
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) s16x4* lds_s16x4;
+
+static __host__ __device__ inline int latent_wave_bytes(int rank_p, int cw) { return 64 * (cw > rank_p + 16 ? cw : rank_p + 16); }
+
+template <int NF, int NK, bool FULL>      // rank_p <= 16 NF, cw <= 32 NK; FULL: equal
+__global__ __launch_bounds__(256, 1) void latent_decode_kernel(ChattsLatentArgs p) {
+  extern __shared__ __attribute__((aligned(1024))) char smem[];
+  __shared__ float stat[2][4][16];
+  const int split = blockIdx.x, row = blockIdx.y, ht = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int cw = p.rank_p + p.rot_p, cv = cw >> 3, nf = FULL ? NF : p.rank_p >> 4, nk = FULL ? NK : cw >> 5, sw = (cv & 7) == 0 ? 7 : 3;
   const ChattsRow R = p.rows[row];
-  uint16_t* kt = reinterpret_cast<uint16_t*>(smem);          // [64][ldk]
-  uint16_t* qh = kt + 64 * ldk;                              // [16][ldk]
-  uint16_t* ql = qh + 16 * ldk;
-  uint16_t* ph = ql + 16 * ldk;                              // [16][kLdP]
-  uint16_t* pl = ph + 16 * kLdP;
-  float* ss = reinterpret_cast<float*>(pl + 16 * kLdP);      // [16][68]
-  float* sal = ss + 16 * 68;                                 // [16] rescale factors
-  const int n = R.pos + 1, ntiles = (n + 63) >> 6;
   if (R.pos < 0) return;
-  for (int e = tid; e < 16 * cv; e += 256) {
-    const int r = e / cv, c = (e - r * cv) * 8;
-    int h = ht * 16 + r;
+  const int n = R.pos + 1, ntiles = (n + 31) >> 5, fr = lane & 15, fg = lane >> 4;
+  char* kt = smem + wave * latent_wave_bytes(p.rank_p, cw);
+  bf16x8_t q[NK];
+  {
+    int h = ht * 16 + fr;
     if (h >= p.heads) h = p.heads - 1;
-    const size_t at = (size_t)row * p.q.ld + (size_t)h * cw + c;
-    *reinterpret_cast<u32x4*>(qh + r * ldk + c) = *reinterpret_cast<const u32x4*>(p.q.hi + at);
-    *reinterpret_cast<u32x4*>(ql + r * ldk + c) = *reinterpret_cast<const u32x4*>(p.q.lo + at);
+    const uint16_t* src = p.q.hi + (size_t)row * p.q.ld + (size_t)h * cw + fg * 8;
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      if (k < nk) q[k] = *reinterpret_cast<const bf16x8_t*>(src + k * 32);
   }
   const uint16_t* cache = reinterpret_cast<const uint16_t*>(p.cache);
-  float m = -INFINITY, l = 0.f;      // of head tid >> 4
-  f32x4 acc[NT];
+  float m = -INFINITY, l = 0.f;      // of head fr; l: this lane's keys only
+  f32x4 acc[NF];
 #pragma unroll
-  for (int i = 0; i < NT; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  const int nf = p.rank_p >> 4, fr = lane & 15, fg = lane >> 4;
-  for (int t = split; t < ntiles; t += p.n_splits) {
-    const uint16_t* tile = cache + latent_row(p, R.slot, t * 64, cw);
-    const int lim = n - t * 64 < 64 ? n - t * 64 : 64;
-    for (int e = tid; e < 64 * cv; e += 256) {
-      const int r = e / cv, c = (e - r * cv) * 8;
-      // rows past the last key: zeros, so that 0 * row stays 0 whatever an unused cache row holds
-      u32x4 v = {0u, 0u, 0u, 0u};
-      if (r < lim) v = *reinterpret_cast<const u32x4*>(tile + (size_t)r * cw + c);
-      *reinterpret_cast<u32x4*>(kt + r * ldk + c) = v;
-    }
-    __syncthreads();
-    f32x4 sacc = {0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < cw; k += 32) {
-      const bf16x8_t b = *reinterpret_cast<const bf16x8_t*>(kt + (wave * 16 + fr) * ldk + k + fg * 8);
-      const bf16x8_t a0 = *reinterpret_cast<const bf16x8_t*>(qh + fr * ldk + k + fg * 8);
-      const bf16x8_t a1 = *reinterpret_cast<const bf16x8_t*>(ql + fr * ldk + k + fg * 8);
-      sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0, b, sacc, 0, 0, 0);
-      sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a1, b, sacc, 0, 0, 0);
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) ss[(fg * 4 + r) * 68 + wave * 16 + fr] = sacc[r];
-    __syncthreads();
+  for (int i = 0; i < NF; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const int step = p.n_splits * 4, pieces = cw >> 4;      // 1 KB pieces of a tile
+  // chunk `lane` of piece 0: row, column; a piece later it is 64 chunks further
+  const int r0 = lane / cv, c0 = lane - r0 * cv, dr = 64 / cv, dc = 64 - dr * cv;
+  for (int t = split * 4 + wave; t < ntiles; t += step) {
+    const uint16_t* tile = cache + latent_row(p, R.slot, t * 32, cw);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // the previous tile has been read
     {
-      const int h = tid >> 4, c = tid & 15;
-      float v[4], mx = -INFINITY;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int key = j * 16 + c;
-        v[j] = key < lim ? ss[h * 68 + key] * p.scale : -INFINITY;
-        mx = fmaxf(mx, v[j]);
+      int r = r0, c = c0;
+      for (int i = 0; i < pieces; ++i) {
+        __builtin_amdgcn_global_load_lds((gptr_t)(tile + (size_t)r * cw + ((c ^ (r & sw)) << 3)), (lptr_t)(kt + i * 1024), 16, 0, 0);
+        r += dr;
+        c += dc;
+        if (c >= cv) { c -= cv; ++r; }
       }
-      const float mn = fmaxf(m, row16_max(mx)), alpha = expf(m - mn);
-      float sum = 0.f;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float e = expf(v[j] - mn);
-        sum += e;
-        uint16_t hi, lo;
-        split_bf16x2(e, hi, lo);
-        ph[h * kLdP + j * 16 + c] = hi;
-        pl[h * kLdP + j * 16 + c] = lo;
-      }
-      l = l * alpha + row16_sum(sum);
-      m = mn;
-      if (c == 0) sal[h] = alpha;
     }
-    __syncthreads();
-    float al[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) al[r] = sal[fg * 4 + r];
-    bf16x8_t a[2][2];
-#pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      a[k][0] = *reinterpret_cast<const bf16x8_t*>(ph + fr * kLdP + k * 32 + fg * 8);
-      a[k][1] = *reinterpret_cast<const bf16x8_t*>(pl + fr * kLdP + k * 32 + fg * 8);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    const int lim = n - t * 32;
+    if (lim < 32) {      // keys past the last one become zeros, whatever an unused cache row holds
+      for (int e = lim * cv + lane; e < 32 * cv; e += 64) *reinterpret_cast<u32x4*>(kt + e * 16) = (u32x4){0u, 0u, 0u, 0u};
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     }
+    f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    {
+      const char* a0 = kt + fr * cw * 2;
+      const char* a1 = kt + (16 + fr) * cw * 2;
+      const int x = fr & sw;      // (16 is a multiple of the swizzle's period)
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int f = wave + 4 * i;
-      if (f < nf) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) acc[i][r] *= al[r];
-#pragma unroll
-        for (int k = 0; k < 2; ++k) {
-          union { uint16_t u[8]; bf16x8_t v; } b;
-#pragma unroll
-          for (int j = 0; j < 8; ++j) b.u[j] = kt[(k * 32 + fg * 8 + j) * ldk + f * 16 + fr];
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[k][0], b.v, acc[i], 0, 0, 0);
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[k][1], b.v, acc[i], 0, 0, 0);
+      for (int k = 0; k < NK; ++k)
+        if (k < nk) {
+          const int c = ((k * 4 + fg) ^ x) << 4;
+          s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a0 + c), q[k], s[0], 0, 0, 0);
+          s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a1 + c), q[k], s[1], 0, 0, 0);
+          if (k % 6 == 5) asm volatile("" ::: "memory");      // (keeps the reads in flight within the registers)
         }
-      }
     }
-    __syncthreads();
+    float v[8], mx = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int key = (j >> 2) * 16 + fg * 4 + (j & 3);
+      v[j] = key < lim ? s[j >> 2][j & 3] * p.scale : -INFINITY;
+      mx = fmaxf(mx, v[j]);
+    }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx), alpha = exp_hw(m - mn);
+    m = mn;
+    bf16x8_t ph, pl;
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float e = exp_hw(v[j] - mn);
+      sum += e;
+      ph[j] = (__bf16)e;
+      pl[j] = (__bf16)(e - (float)ph[j]);
+    }
+    l = l * alpha + sum;
+    if (__any(alpha != 1.0f)) {
+#pragma unroll
+      for (int i = 0; i < NF; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[i][r] *= alpha;
+    }
+    {
+      // transposing reads: lane -> row 4 g + (fr >> 2) (and + 16), 4 columns (fr & 3) * 4 of the fragment's 16: chunk 2 i + (fr >> 1 & 1), half fr & 1
+      const int tr = fg * 4 + (fr >> 2), x = tr & sw, cb = (fr >> 1) & 1;
+      const char* t0 = kt + tr * cw * 2 + (fr & 1) * 8;
+#pragma unroll
+      for (int i = 0; i < NF; ++i)
+        if (i < nf) {
+          const int c = ((2 * i + cb) ^ x) << 4;
+          union { s16x4 h[2]; bf16x8_t v; } a;
+          a.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(t0 + c));
+          a.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(t0 + 32 * cw + c));
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, ph, acc[i], 0, 0, 0);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pl, acc[i], 0, 0, 0);
+          if (i % 8 == 7) asm volatile("" ::: "memory");
+        }
+    }
   }
-  // write out: C layout col = lane & 15 (latent column), row = 4 * (lane >> 4) + r (head)
-  if ((tid & 15) == 0) { ss[tid >> 4] = m; ss[16 + (tid >> 4)] = l; }
+  // merge of the four waves: O^T (lane: 4 consecutive latent columns of its head) into the wave's LDS tile as [16 heads][rank_p + 16] floats
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (fg == 0) { stat[0][wave][fr] = m; stat[1][wave][fr] = l; }
+  const int ldk = p.rank_p + 16, wf = latent_wave_bytes(p.rank_p, cw) >> 2;
+  float* ot = reinterpret_cast<float*>(kt);
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+#pragma unroll
+  for (int i = 0; i < NF; ++i)
+    if (i < nf) *reinterpret_cast<f32x4*>(ot + fr * ldk + i * 16 + fg * 4) = acc[i];
   __syncthreads();
-#pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int hh = fg * 4 + r, h = ht * 16 + hh;
+  const int c4 = p.rank_p >> 2;
+  for (int e = tid; e < 16 * c4; e += 256) {
+    const int hh = e / c4, c = (e - hh * c4) * 4, h = ht * 16 + hh;
     if (h >= p.heads) continue;
-    const float ll = ss[16 + hh];
+    float M = -INFINITY, L = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) M = fmaxf(M, stat[0][w][hh]);
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float mw = stat[0][w][hh];
+      if (mw == -INFINITY) continue;      // a wave without a tile
+      const float f = exp_hw(mw - M);
+      L += f * stat[1][w][hh];
+      const f32x4 x = *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem) + (size_t)w * wf + hh * ldk + c);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] += f * x[r];
+    }
     if (p.n_splits == 1) {
-      float* o = p.o + ((size_t)row * p.heads + h) * p.rank_p;
 #pragma unroll
-      for (int i = 0; i < NT; ++i)
-        if (wave + 4 * i < nf) o[(wave + 4 * i) * 16 + fr] = acc[i][r] / ll;
+      for (int r = 0; r < 4; ++r) o[r] /= L;
+      *reinterpret_cast<f32x4*>(p.o + ((size_t)row * p.heads + h) * p.rank_p + c) = o;
     } else {
-      float* o = p.partial + (((size_t)row * p.heads + h) * p.n_splits + split) * (p.rank_p + 2);
-#pragma unroll
-      for (int i = 0; i < NT; ++i)
-        if (wave + 4 * i < nf) o[(wave + 4 * i) * 16 + fr] = acc[i][r];
-      if (wave == 0 && fr == 0) { o[p.rank_p] = ss[hh]; o[p.rank_p + 1] = ll; }
+      float* dst = p.partial + (((size_t)row * p.heads + h) * p.n_splits + split) * (p.rank_p + 4);
+      *reinterpret_cast<f32x4*>(dst + c) = o;
+      if (c == 0) { dst[p.rank_p] = M; dst[p.rank_p + 1] = L; }
     }
   }
 }
 
 // merge of the splits: one workgroup per (head, row)
-__global__ __launch_bounds__(256) void latent_merge_kernel(ChattsLatentArgs p) {
-  const int h = blockIdx.x, row = blockIdx.y;
+__global__ __launch_bounds__(128) void latent_merge_kernel(ChattsLatentArgs p) {
+  __shared__ float w[64];
+  const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, ld = p.rank_p + 4;
   if (p.rows[row].pos < 0) return;
-  const float* part = p.partial + ((size_t)row * p.heads + h) * p.n_splits * (p.rank_p + 2);
-  const int ld = p.rank_p + 2;
-  float M = -INFINITY;
-  for (int s = 0; s < p.n_splits; ++s) M = fmaxf(M, part[(size_t)s * ld + p.rank_p]);
-  float L = 0.f;
-  for (int s = 0; s < p.n_splits; ++s) L += expf(part[(size_t)s * ld + p.rank_p] - M) * part[(size_t)s * ld + p.rank_p + 1];
-  for (int c = threadIdx.x; c < p.rank_p; c += 256) {
-    float o = 0.f;
-    for (int s = 0; s < p.n_splits; ++s) o += expf(part[(size_t)s * ld + p.rank_p] - M) * part[(size_t)s * ld + c];
-    p.o[((size_t)row * p.heads + h) * p.rank_p + c] = o / L;
+  const float* part = p.partial + ((size_t)row * p.heads + h) * p.n_splits * ld;
+  if (tid < 64) {
+    const float m = tid < p.n_splits ? part[(size_t)tid * ld + p.rank_p] : -INFINITY, l = tid < p.n_splits ? part[(size_t)tid * ld + p.rank_p + 1] : 0.f;
+    const float M = wave_max(m), f = m == -INFINITY ? 0.f : exp_hw(m - M);
+    const float L = wave_sum(f * l);
+    w[tid] = f / L;
+  }
+  __syncthreads();
+  for (int c = tid * 4; c < p.rank_p; c += 512) {
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int s = 0; s < p.n_splits; ++s) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(part + (size_t)s * ld + c);
+      const float f = w[s];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] += f * x[r];
+    }
+    *reinterpret_cast<f32x4*>(p.o + ((size_t)row * p.heads + h) * p.rank_p + c) = o;
+  }
+}
+
+// ---- expanded form, for prompts: keys and values of every head are written out for the sequence, then ordinary flash attention ----------
+// gather: the latents and rotated key parts of each expanded span's sequence from its pages into consecutive rows (span.base ..), a whole
+// number of 64-row tiles per span, zeros past the last key.  grid (row groups of 16, spans)
+__global__ __launch_bounds__(256) void latent_gather_kernel(ChattsLatentArgs p, const ChattsSpan* __restrict__ spans, uint16_t* __restrict__ cbuf,
+                                                            uint16_t* __restrict__ krbuf) {
+  const ChattsSpan sp = spans[blockIdx.y];
+  if (sp.base < 0) return;
+  const int n = sp.pos0 + sp.t, rows = (n + 63) & ~63, cw = p.rank_p + p.rot_p, cv = cw >> 3;
+  const int j0 = blockIdx.x * 16;
+  if (j0 >= rows) return;
+  const uint16_t* src = reinterpret_cast<const uint16_t*>(p.cache) + (j0 < n ? latent_row(p, sp.slot, j0, cw) : 0);
+  for (int e = threadIdx.x; e < 16 * cv; e += 256) {
+    const int r = e / cv, c = (e - r * cv) * 8;
+    u32x4 v = {0u, 0u, 0u, 0u};
+    if (j0 + r < n) v = *reinterpret_cast<const u32x4*>(src + (size_t)r * cw + c);
+    const size_t at = (size_t)(sp.base + j0 + r);
+    if (c < p.rank_p) *reinterpret_cast<u32x4*>(cbuf + at * p.rank_p + c) = v;
+    else *reinterpret_cast<u32x4*>(krbuf + at * p.rot_p + c - p.rank_p) = v;
+  }
+}
+
+// grid (query tiles of 128, heads, spans), a wave owns 32 queries of one head, 64 keys per step: S^T = K Q^T, O^T = V^T P^T - the probabilities of
+// a lane are the B fragment of the second product (K slot 8 g + j = key 8 g + j: the rows of K are read in the order that makes it so).
+struct LatentPrefill {
+  const uint16_t* kx;      // [rows, ldk]: unrotated keys, head by head (dim_p each)
+  const uint16_t* kr;      // [rows, rot_p]
+  const uint16_t* vt;      // [heads * vdim_p, ldv]: values, transposed
+  const uint16_t* qx;      // [T, ldq]: [unrotated | rotated] per head (dim_p + rot_p)
+  int ldk, ldv, ldq, dim_p, rot_p, vdim_p, out_head;
+  float scale;
+  ChattsOperand out;
+};
+template <int NK, int NV, int OCC, bool FULL>      // dim_p + rot_p <= 32 NK, vdim_p <= 16 NV; FULL: equal
+__global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill p, const ChattsSpan* __restrict__ spans) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const ChattsSpan sp = spans[blockIdx.z];
+  const int qt0 = (gridDim.x - 1 - blockIdx.x) * 128, h = blockIdx.y;      // the longest key ranges first
+  if (sp.base < 0 || qt0 >= sp.t) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const int dq = FULL ? 32 * NK : p.dim_p + p.rot_p, vdim_p = FULL ? 16 * NV : p.vdim_p, ldl = dq + 8, nk = dq >> 5, nv = vdim_p >> 4;
+  constexpr int kLdV = 72;
+  uint16_t* ks = reinterpret_cast<uint16_t*>(smem);      // [64][ldl]
+  uint16_t* vs = ks + 64 * ldl;                          // [vdim_p][72]
+  const int qlast = qt0 + 127 < sp.t ? qt0 + 127 : sp.t - 1;
+  const int ntiles = (sp.pos0 + qlast + 64) >> 6;        // keys 0 .. pos0 + qlast
+  const int q0 = qt0 + wave * 32;
+  bf16x8_t q[2][NK];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    int r = q0 + u * 16 + fr;
+    if (r > sp.t - 1) r = sp.t - 1;
+    const uint16_t* src = p.qx + (size_t)(sp.row0 + r) * p.ldq + h * dq + fg * 8;
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      if (k < nk) q[u][k] = *reinterpret_cast<const bf16x8_t*>(src + k * 32);
+  }
+  f32x4 o[NV][2];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) o[i][0] = o[i][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
+  // staging: K rows in 16-byte pieces (64 rows x dq / 8), V^T rows (vdim_p x 8)
+  constexpr int KP = NK, VP = (NV + 1) / 2;
+  u32x4 rk[KP], rv[VP];
+  const int kc = dq >> 3, dc = p.dim_p >> 3;
+  auto fetch = [&](int t) {
+    const size_t base = (size_t)sp.base + t * 64;
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int e = i * 256 + tid;
+      if (e < 64 * kc) {
+        const int r = e / kc, c = e - r * kc;
+        rk[i] = c < dc ? *reinterpret_cast<const u32x4*>(p.kx + (base + r) * p.ldk + h * p.dim_p + c * 8)
+                       : *reinterpret_cast<const u32x4*>(p.kr + (base + r) * p.rot_p + (c - dc) * 8);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int e = i * 256 + tid;
+      if (e < vdim_p * 8) rv[i] = *reinterpret_cast<const u32x4*>(p.vt + (size_t)(h * vdim_p + (e >> 3)) * p.ldv + base + (e & 7) * 8);
+    }
+  };
+  fetch(0);
+  for (int t = 0; t < ntiles; ++t) {
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int e = i * 256 + tid;
+      if (e < 64 * kc) *reinterpret_cast<u32x4*>(ks + (e / kc) * ldl + (e % kc) * 8) = rk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int e = i * 256 + tid;
+      if (e < vdim_p * 8) *reinterpret_cast<u32x4*>(vs + (e >> 3) * kLdV + (e & 7) * 8) = rv[i];
+    }
+    __syncthreads();
+    if (t + 1 < ntiles) fetch(t + 1);
+    if (t * 64 > sp.pos0 + q0 + 31) continue;      // (uniform per wave) nothing visible to this wave's queries
+    f32x4 s[4][2];      // [32-key group * 2 + half][query block]
+#pragma unroll
+    for (int a = 0; a < 4; ++a) s[a][0] = s[a][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const uint16_t* kb = ks + (8 * (fr >> 2) + (fr & 3)) * ldl + fg * 8;
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      if (k < nk) {
+#pragma unroll
+        for (int a = 0; a < 4; ++a) {
+          const bf16x8_t kv = *reinterpret_cast<const bf16x8_t*>(kb + ((a >> 1) * 32 + (a & 1) * 4) * ldl + k * 32);
+          s[a][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kv, q[0][k], s[a][0], 0, 0, 0);
+          s[a][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kv, q[1][k], s[a][1], 0, 0, 0);
+        }
+        asm volatile("" ::: "memory");
+      }
+    bf16x8_t pf[2][2];      // [32-key group][query block]
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int qpos = sp.pos0 + q0 + u * 16 + fr;
+      const bool edge = t * 64 + 63 > sp.pos0 + q0 + u * 16;      // (uniform) some key of the tile is in the future of some query
+      float mx = -INFINITY;
+#pragma unroll
+      for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          float v = s[a][u][r] * p.scale;
+          if (edge && t * 64 + (a >> 1) * 32 + fg * 8 + (a & 1) * 4 + r > qpos) v = -INFINITY;
+          s[a][u][r] = v;
+          mx = fmaxf(mx, v);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m[u], mx), safe = mn == -INFINITY ? 0.f : mn, alpha = exp_hw(m[u] - safe);
+      m[u] = mn;
+      float sum = 0.f;
+#pragma unroll
+      for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = exp_hw(s[a][u][r] - safe);
+          sum += e;
+          pf[a >> 1][u][(a & 1) * 4 + r] = (__bf16)e;
+        }
+      l[u] = l[u] * alpha + sum;
+      if (__any(alpha != 1.0f)) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o[i][u][r] *= alpha;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if (i < nv) {
+#pragma unroll
+        for (int g = 0; g < 2; ++g) {
+          const bf16x8_t vv = *reinterpret_cast<const bf16x8_t*>(vs + (i * 16 + fr) * kLdV + g * 32 + fg * 8);
+          o[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pf[g][0], o[i][0], 0, 0, 0);
+          o[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pf[g][1], o[i][1], 0, 0, 0);
+        }
+        if (i % 2 == 1) asm volatile("" ::: "memory");      // (keeps the reads in flight within the registers)
+      }
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int r = q0 + u * 16 + fr;
+    float L = l[u];
+    L += __shfl_xor(L, 16, 64);
+    L += __shfl_xor(L, 32, 64);
+    if (r >= sp.t) continue;
+    const float inv = 1.0f / L;
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if (i < nv) {
+        const float v[4] = {o[i][u][0] * inv, o[i][u][1] * inv, o[i][u][2] * inv, o[i][u][3] * inv};
+        store_operand4(p.out, sp.row0 + r, h * p.out_head + i * 16 + fg * 4, v);
+      }
   }
 }
 
@@ -319,20 +541,23 @@ static int check_latent(const ChattsLatentArgs* a, const char* who) {
   return CHATTS_OK;
 }
 
-template <int NT>
-static int launch_latent_decode(const ChattsLatentArgs* a, hipStream_t s) {
-  const int cw = a->rank_p + a->rot_p;
-  const size_t lds = (size_t)(64 + 32) * (cw + 8) * 2 + 2 * 16 * kLdP * 2 + (16 * 68 + 16) * 4;
-  CHATTS_REQUIRE(lds <= 160 * 1024, CHATTS_E_SHAPE, "latent_attend: a cache row of %d elements does not fit", cw);
+template <int NF, int NK, bool FULL>
+static int launch_latent_decode_t(const ChattsLatentArgs* a, hipStream_t s) {
+  const size_t lds = (size_t)4 * latent_wave_bytes(a->rank_p, a->rank_p + a->rot_p);
   static bool configured = false;
   if (!configured) {
-    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NT>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NF, NK, FULL>), hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024);
     CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "latent_attend: cannot reserve LDS: %s", hipGetErrorString(e));
     configured = true;
   }
-  hipLaunchKernelGGL(latent_decode_kernel<NT>, dim3((a->heads + 15) / 16, a->n_rows, a->n_splits), dim3(256), lds, s, *a);
+  hipLaunchKernelGGL((latent_decode_kernel<NF, NK, FULL>), dim3(a->n_splits, a->n_rows, (a->heads + 15) / 16), dim3(256), lds, s, *a);
   CHATTS_CHECK_LAUNCH("latent_decode");
   return CHATTS_OK;
+}
+
+template <int NF, int NK>
+static int launch_latent_decode(const ChattsLatentArgs* a, hipStream_t s) {
+  return a->rank_p == 16 * NF && a->rank_p + a->rot_p == 32 * NK ? launch_latent_decode_t<NF, NK, true>(a, s) : launch_latent_decode_t<NF, NK, false>(a, s);
 }
 
 static int latent_attend_impl(const ChattsLatentArgs* a, hipStream_t s) {
@@ -340,8 +565,13 @@ static int latent_attend_impl(const ChattsLatentArgs* a, hipStream_t s) {
   CHATTS_REQUIRE(a->o && (a->q.f32 || a->q.hi), CHATTS_E_BADARG, "latent_attend: null pointer");
   if (a->n_rows == 0) return CHATTS_OK;
   const int cw = a->rank_p + a->rot_p;
-  const bool matrix = !a->cache_f32 && a->q.hi && a->q.lo && (size_t)(64 + 32) * (cw + 8) * 2 + 2 * 16 * kLdP * 2 + (16 * 68 + 16) * 4 <= 160 * 1024;
-  if (!matrix) {
+  CHATTS_REQUIRE(a->n_splits >= 1 && a->n_splits <= 64 && (a->n_splits == 1 || a->partial), CHATTS_E_BADARG, "latent_attend: %d splits", a->n_splits);
+  int rc;
+  if (!a->cache_f32 && a->q.hi && a->rank_p <= 64 && cw <= 128) rc = launch_latent_decode<4, 4>(a, s);
+  else if (!a->cache_f32 && a->q.hi && a->rank_p <= 128 && cw <= 192) rc = launch_latent_decode<8, 6>(a, s);
+  else if (!a->cache_f32 && a->q.hi && a->rank_p <= 256 && cw <= 384) rc = launch_latent_decode<16, 12>(a, s);
+  else if (!a->cache_f32 && a->q.hi && a->rank_p <= 512 && cw <= 576) rc = launch_latent_decode<32, 18>(a, s);
+  else {
     const size_t lds = (size_t)(cw + 64) * sizeof(float);
     const dim3 g(a->heads, a->n_rows);
     if (a->cache_f32) hipLaunchKernelGGL(latent_attend_kernel<float>, g, dim3(256), lds, s, *a);
@@ -349,18 +579,31 @@ static int latent_attend_impl(const ChattsLatentArgs* a, hipStream_t s) {
     CHATTS_CHECK_LAUNCH("latent_attend");
     return CHATTS_OK;
   }
-  CHATTS_REQUIRE(a->n_splits >= 1 && (a->n_splits == 1 || a->partial), CHATTS_E_BADARG, "latent_attend: %d splits without a buffer", a->n_splits);
-  int rc;
-  if (a->rank_p <= 128) rc = launch_latent_decode<2>(a, s);
-  else if (a->rank_p <= 256) rc = launch_latent_decode<4>(a, s);
-  else if (a->rank_p <= 512) rc = launch_latent_decode<8>(a, s);
-  else rc = launch_latent_decode<16>(a, s);
   if (rc) return rc;
   if (a->n_splits > 1) {
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(a->heads, a->n_rows), dim3(256), 0, s, *a);
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(a->heads, a->n_rows), dim3(128), 0, s, *a);
     CHATTS_CHECK_LAUNCH("latent_merge");
   }
   return CHATTS_OK;
+}
+
+template <int NK, int NV, int OCC, bool FULL>
+static int launch_latent_prefill_t(const LatentPrefill& p, const ChattsSpan* spans, int n_spans, int heads, int longest, hipStream_t s) {
+  const size_t lds = (size_t)(64 * (p.dim_p + p.rot_p + 8) + p.vdim_p * 72) * 2;
+  static bool configured = false;
+  if (!configured) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_prefill_kernel<NK, NV, OCC, FULL>), hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
+    CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "latent_expanded: cannot reserve LDS: %s", hipGetErrorString(e));
+    configured = true;
+  }
+  hipLaunchKernelGGL((latent_prefill_kernel<NK, NV, OCC, FULL>), dim3((longest + 127) / 128, heads, n_spans), dim3(256), lds, s, p, spans);
+  CHATTS_CHECK_LAUNCH("latent_prefill");
+  return CHATTS_OK;
+}
+template <int NK, int NV, int OCC>
+static int launch_latent_prefill(const LatentPrefill& p, const ChattsSpan* spans, int n_spans, int heads, int longest, hipStream_t s) {
+  return p.dim_p + p.rot_p == 32 * NK && p.vdim_p == 16 * NV ? launch_latent_prefill_t<NK, NV, OCC, true>(p, spans, n_spans, heads, longest, s)
+                                                             : launch_latent_prefill_t<NK, NV, OCC, false>(p, spans, n_spans, heads, longest, s);
 }
 
 }  // namespace chatts
@@ -369,7 +612,8 @@ using namespace chatts;
 
 extern "C" int chatts_latent_prep(const ChattsLatentArgs* a, chatts_stream_t stream) {
   if (const int rc = check_latent(a, "latent_prep")) return rc;
-  CHATTS_REQUIRE(a->proj && a->c_norm && (a->rot == 0 || (a->cos_tab && a->sin_tab)) && (a->q.f32 || a->q.hi), CHATTS_E_BADARG, "latent_prep: null pointer");
+  CHATTS_REQUIRE(a->proj && a->c_norm && (a->rot == 0 || (a->cos_tab && a->sin_tab)) && (a->q.f32 || a->q.hi || a->qx), CHATTS_E_BADARG, "latent_prep: null pointer");
+  CHATTS_REQUIRE(!a->qx || (a->dim_p % 4 == 0 && a->off_q % 4 == 0 && a->ld_proj % 4 == 0), CHATTS_E_SHAPE, "latent_prep: query columns");
   if (a->n_rows == 0) return CHATTS_OK;
   if (a->cache_f32) hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(a->n_rows), dim3(256), 0, as_stream(stream), *a);
   else hipLaunchKernelGGL(latent_prep_kernel<uint16_t>, dim3(a->n_rows), dim3(256), 0, as_stream(stream), *a);
@@ -393,4 +637,50 @@ extern "C" int chatts_head_linear(const ChattsHeadLinearArgs* a, chatts_stream_t
   hipLaunchKernelGGL(head_linear_kernel, dim3((a->n / 16 + 3) / 4, (a->m + 15) / 16, a->heads), dim3(256), 0, as_stream(stream), *a);
   CHATTS_CHECK_LAUNCH("head_linear");
   return CHATTS_OK;
+}
+
+extern "C" int chatts_latent_can_expand(int dim_p, int rot_p, int vdim_p, int rank_p) {
+  return rank_p % 64 == 0 && dim_p % 32 == 0 && rot_p % 32 == 0 && vdim_p % 16 == 0 && dim_p + rot_p <= 384 && vdim_p <= 256;
+}
+
+extern "C" int chatts_latent_expanded(const ChattsLatentExpandArgs* x, chatts_stream_t stream) {
+  CHATTS_REQUIRE(x && x->latent && x->spans && x->spans_dev && x->cbuf && x->krbuf && x->zero && x->k_hi && x->k_lo && x->v_hi && x->v_lo && x->uk && x->uv &&
+                     x->latent->qx, CHATTS_E_BADARG, "latent_expanded: null pointer");
+  const ChattsLatentArgs* a = x->latent;
+  if (const int rc = check_latent(a, "latent_expanded")) return rc;
+  CHATTS_REQUIRE(!a->cache_f32 && chatts_latent_can_expand(a->dim_p, a->rot_p, x->vdim_p, a->rank_p), CHATTS_E_SHAPE, "latent_expanded: head sizes %d + %d / %d, latent %d",
+                 a->dim_p, a->rot_p, x->vdim_p, a->rank_p);
+  CHATTS_REQUIRE((x->out.f32 || x->out.hi) && x->out.ld >= (a->heads - 1) * x->out_head + x->vdim_p && x->out.ld % 4 == 0 && x->out_head % 4 == 0, CHATTS_E_SHAPE,
+                 "latent_expanded: output stride");
+  int rows = 0, longest = 0, longest_ctx = 0;
+  for (int i = 0; i < x->n_spans; ++i) {
+    const ChattsSpan& sp = x->spans[i];
+    if (sp.base < 0) continue;
+    CHATTS_REQUIRE(sp.base == rows && sp.t >= 1 && sp.pos0 >= 0, CHATTS_E_SHAPE, "latent_expanded: span %d starts at row %d, not %d", i, sp.base, rows);
+    rows += (sp.pos0 + sp.t + 63) & ~63;
+    if (sp.t > longest) longest = sp.t;
+    if (sp.pos0 + sp.t > longest_ctx) longest_ctx = sp.pos0 + sp.t;
+  }
+  if (rows == 0) return CHATTS_OK;
+  CHATTS_REQUIRE(rows <= x->max_rows, CHATTS_E_SHAPE, "latent_expanded: %d rows exceed the buffers (%d)", rows, x->max_rows);
+  hipStream_t s = as_stream(stream);
+  hipLaunchKernelGGL(latent_gather_kernel, dim3((((longest_ctx + 63) & ~63) + 15) / 16, x->n_spans), dim3(256), 0, s, *a, x->spans_dev, x->cbuf, x->krbuf);
+  CHATTS_CHECK_LAUNCH("latent_gather");
+  ChattsLinearArgs g{};      // keys: [rows, heads * dim_p] = latents . W_uk^T;  values, transposed: [heads * vdim_p, rows] = W_uv . latents^T
+  g.workspace = x->workspace; g.workspace_bytes = x->workspace_bytes;
+  g.a_hi = x->cbuf; g.a_lo = x->zero; g.ld_planes = a->rank_p; g.w = x->uk; g.ldw = a->rank_p;
+  g.m = rows; g.n = a->heads * a->dim_p; g.k = a->rank_p; g.ldc = g.n; g.c_hi = x->k_hi; g.c_lo = x->k_lo; g.ld_cplanes = g.n; g.epilogue = CHATTS_EPI_NONE;
+  int rc;
+  if ((rc = chatts_linear(&g, stream)) != 0) return rc;
+  g.a_hi = x->uv; g.w = x->cbuf;
+  g.m = a->heads * x->vdim_p; g.n = rows; g.ldc = rows; g.c_hi = x->v_hi; g.c_lo = x->v_lo; g.ld_cplanes = rows;
+  if ((rc = chatts_linear(&g, stream)) != 0) return rc;
+  LatentPrefill p{};
+  p.kx = x->k_hi; p.kr = x->krbuf; p.vt = x->v_hi; p.qx = a->qx;
+  p.ldk = a->heads * a->dim_p; p.ldv = rows; p.ldq = a->heads * (a->dim_p + a->rot_p);
+  p.dim_p = a->dim_p; p.rot_p = a->rot_p; p.vdim_p = x->vdim_p; p.out_head = x->out_head; p.scale = a->scale; p.out = x->out;
+  const int dq = a->dim_p + a->rot_p;
+  if (dq <= 96 && x->vdim_p <= 64) return launch_latent_prefill<3, 4, 2>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
+  if (dq <= 192 && x->vdim_p <= 128) return launch_latent_prefill<6, 8, 2>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
+  return launch_latent_prefill<12, 16, 1>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
 }

@@ -51,7 +51,22 @@ extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const Chatts
     if (l.kind == CHATTS_MIX_DELTA) { add(l.dt_n, l.delta.ld_a2); add(l.gate_n, l.delta.ld_g2); }
   }
   add((int)c->vocab_p, c->width_p);
-  size_t ws = argmax_scratch_bytes(c->max_slots > 1 ? c->max_slots : 1);
+  // keys and values written out from the latents: rows in whole tiles of 64
+  size_t ws = 0;
+  for (int i = 0; i < c->n_layers; ++i) {
+    const ChattsMixLayer& l = layers[i];
+    bool seen = l.kind != CHATTS_MIX_LATENT || !l.ukx;
+    for (int j = 0; j < i && !seen; ++j)
+      seen = layers[j].kind == CHATTS_MIX_LATENT && layers[j].ukx && layers[j].latent.heads == l.latent.heads && layers[j].dim_p == l.dim_p &&
+             layers[j].vdim_p == l.vdim_p && layers[j].latent.rank_p == l.latent.rank_p;
+    for (int n = 64; !seen && n <= c->expand_rows; n += 64) {
+      const size_t a = chatts_linear_workspace(n, l.latent.heads * l.dim_p, l.latent.rank_p), b = chatts_linear_workspace(l.latent.heads * l.vdim_p, n, l.latent.rank_p);
+      if (a > ws) ws = a;
+      if (b > ws) ws = b;
+    }
+  }
+  const size_t am = argmax_scratch_bytes(c->max_slots > 1 ? c->max_slots : 1);
+  if (am > ws) ws = am;
   for (int t = 2; t <= c->t_max; ++t)
     for (auto& s : shapes) {
       const size_t w = chatts_linear_workspace(t, s.first, s.second);
@@ -118,37 +133,100 @@ static ChattsOperand f32_out(float* p, int ld) {
   return o;
 }
 
-static int mix_latent(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, const ChattsOperand& out, chatts_stream_t s) {
-  StageRange stage("chatts.mix.latent");
-  ChattsLatentArgs a = l.latent;
+static ChattsOperand rows_from(ChattsOperand o, int row) {
+  const size_t at = (size_t)row * o.ld;
+  if (o.f32) o.f32 += at;
+  if (o.hi) o.hi += at;
+  if (o.lo) o.lo += at;
+  return o;
+}
+
+// absorbed attention for rows r0 .. r0 + n (a: prepared for the whole batch)
+static int mix_latent_absorbed(const ChattsMixDecoder* d, const ChattsMixLayer& l, ChattsLatentArgs a, int r0, int n, const ChattsOperand& out, chatts_stream_t s) {
   const int cw = a.rank_p + a.rot_p;
-  a.proj = d->b.proj; a.ld_proj = l.in_n;
-  a.cache = run.cache; a.cache_f32 = d->c.exact;
-  a.table = d->b.table; a.table_stride = d->c.table_stride; a.log_block = kv_log_block(d->c.block_size);
-  a.rows = d->b.rows; a.n_rows = t; a.eps = d->c.eps;
-  a.q = ChattsOperand{};
-  a.q.ld = a.heads * cw;
-  if (d->c.exact) a.q.f32 = d->b.q_f32;
-  else { a.q.hi = d->b.q_hi; a.q.lo = d->b.q_lo; }
-  a.o = d->b.o_lat;
+  a.rows += r0; a.n_rows = n;
+  a.q = rows_from(a.q, r0);
+  a.o = d->b.o_lat + (size_t)r0 * a.heads * a.rank_p;
   int rc;
-  if ((rc = chatts_latent_prep(&a, s)) != 0) return rc;
   ChattsHeadLinearArgs h{};
-  h.a = d->b.proj + a.off_q; h.lda = l.in_n; h.a_head = l.dim_p;
-  h.w = l.uk; h.m = t; h.heads = a.heads; h.n = a.rank_p; h.k = l.dim_p; h.out = a.q; h.out_head = cw; h.exact = d->c.exact;
+  h.a = a.proj + (size_t)r0 * a.ld_proj + a.off_q; h.lda = a.ld_proj; h.a_head = l.dim_p;
+  h.w = l.uk; h.m = n; h.heads = a.heads; h.n = a.rank_p; h.k = l.dim_p; h.out = a.q; h.out_head = cw; h.exact = d->c.exact;
   if ((rc = chatts_head_linear(&h, s)) != 0) return rc;
-  // few rows: the keys of a row are spread over workgroups until the chip has ~2 per CU
-  const int tiles = (a.heads + 15) / 16 * t;
-  int splits = tiles >= 512 ? 1 : 512 / tiles;
-  if (splits > 64) splits = 64;
-  const int most = (d->c.max_ctx + 63) / 64;
+  // few rows: the keys of a row are spread over workgroups (each takes 128 keys at a time) until there is about one per CU
+  const int tiles = (a.heads + 15) / 16 * n;
+  int splits = tiles >= 256 ? 1 : 256 / tiles;
+  const int most = (d->c.max_ctx + 127) / 128;
   if (splits > most) splits = most;
-  while (splits > 1 && (size_t)t * a.heads * splits * (a.rank_p + 2) > d->b.partial_elems) --splits;
+  if (splits > 64) splits = 64;
+  while (splits > 1 && (size_t)n * a.heads * splits * (a.rank_p + 4) > d->b.partial_elems) --splits;
   a.n_splits = splits; a.partial = d->b.partial;
   if ((rc = chatts_latent_attend(&a, s)) != 0) return rc;
-  h.a = d->b.o_lat; h.lda = a.heads * a.rank_p; h.a_head = a.rank_p;
-  h.w = l.uv; h.n = l.vdim_p; h.k = a.rank_p; h.out = out; h.out_head = l.out_head;
+  h.a = a.o; h.lda = a.heads * a.rank_p; h.a_head = a.rank_p;
+  h.w = l.uv; h.n = l.vdim_p; h.k = a.rank_p; h.out = rows_from(out, r0); h.out_head = l.out_head;
   return chatts_head_linear(&h, s);
+}
+
+static int mix_latent(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, const ChattsSpan* spans, int n_spans, bool single,
+                      const ChattsOperand& out, chatts_stream_t s) {
+  StageRange stage("chatts.mix.latent");
+  ChattsLatentArgs a = l.latent;
+  a.proj = d->b.proj; a.ld_proj = l.in_n; a.dim_p = l.dim_p;
+  a.cache = run.cache; a.cache_f32 = d->c.exact;
+  a.table = d->b.table; a.table_stride = d->c.table_stride; a.log_block = kv_log_block(d->c.block_size);
+  a.rows = d->b.rows; a.n_rows = t; a.eps = d->c.eps; a.n_splits = 1;
+  a.q = ChattsOperand{};
+  a.q.ld = a.heads * (a.rank_p + a.rot_p);
+  int expanded = 0;
+  if (!single && l.ukx)
+    for (int i = 0; i < n_spans; ++i) expanded += spans[i].base >= 0;
+  if (single || expanded < n_spans) {      // some rows run absorbed
+    if (d->c.exact) a.q.f32 = d->b.q_f32;
+    else { a.q.hi = d->b.q_hi; a.q.lo = d->b.q_lo; }
+  }
+  if (expanded) a.qx = d->b.qx;
+  int rc;
+  if ((rc = chatts_latent_prep(&a, s)) != 0) return rc;
+  if (expanded) {
+    ChattsLatentExpandArgs x{};
+    x.latent = &a; x.spans = spans; x.spans_dev = d->b.spans; x.n_spans = n_spans; x.vdim_p = l.vdim_p; x.out_head = l.out_head; x.max_rows = d->c.expand_rows;
+    x.uk = l.ukx; x.uv = l.uvx; x.cbuf = d->b.cbuf; x.krbuf = d->b.krbuf; x.zero = d->b.zero;
+    x.k_hi = d->b.kx_hi; x.k_lo = d->b.kx_lo; x.v_hi = d->b.vx_hi; x.v_lo = d->b.vx_lo;
+    x.out = out; x.workspace = d->b.workspace; x.workspace_bytes = d->b.workspace_bytes;
+    if ((rc = chatts_latent_expanded(&x, s)) != 0) return rc;
+    if (expanded == n_spans) return CHATTS_OK;
+  }
+  if (!expanded) return mix_latent_absorbed(d, l, a, 0, t, out, s);
+  for (int i = 0; i < n_spans;) {          // runs of neighbouring spans that are not expanded
+    if (spans[i].base >= 0) { ++i; continue; }
+    const int r0 = spans[i].row0;
+    int n = 0;
+    for (; i < n_spans && spans[i].base < 0; ++i) n += spans[i].t;
+    if ((rc = mix_latent_absorbed(d, l, a, r0, n, out, s)) != 0) return rc;
+  }
+  return CHATTS_OK;
+}
+
+// The absorbed form costs ~(2 rank + rot) products per query, key and head, the expanded one (dim + rot + vdim) plus rank (dim + vdim) per key and
+// head for writing keys and values out (two passes).  The absorbed kernel serves 16 heads of ONE query per workgroup and fetches the keys again
+// for every query: measured, a product costs about four times as much there.
+extern "C" int chatts_mixdec_plan(ChattsMixDecoder* d, ChattsSpan* spans, int n_spans) {
+  CHATTS_REQUIRE(d && spans && n_spans >= 0, CHATTS_E_BADARG, "mixdec_plan: null argument");
+  const ChattsMixLayer* l = nullptr;
+  for (const ChattsMixLayer& x : d->layers)
+    if (x.kind == CHATTS_MIX_LATENT && x.ukx) { l = &x; break; }
+  int rows = 0;
+  for (int i = 0; i < n_spans; ++i) {
+    ChattsSpan& sp = spans[i];
+    sp.base = -1;
+    if (!l || d->c.expand_rows <= 0 || sp.t < 8) continue;
+    const double own = 4.0 * sp.t * (2.0 * l->latent.rank_p + l->latent.rot_p);
+    const double exp = sp.t * (double)(l->dim_p + l->latent.rot_p + l->vdim_p) + 2.0 * l->latent.rank_p * (l->dim_p + l->vdim_p);
+    const int need = (sp.pos0 + sp.t + 63) & ~63;
+    if (own <= exp || rows + need > d->c.expand_rows) continue;
+    sp.base = rows;
+    rows += need;
+  }
+  return CHATTS_OK;
 }
 
 static int mix_delta(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, int n_spans, bool single, const ChattsOperand& out,
@@ -160,7 +238,7 @@ static int mix_delta(const ChattsMixDecoder* d, const ChattsMixLayer& l, const C
   a.rows = d->b.rows; a.n_rows = t; a.spans = d->b.spans; a.n_spans = n_spans;
   a.out = out;
   if (single) return chatts_delta_decode(&a, s);
-  a.q = d->b.dq; a.k = d->b.dk; a.v = d->b.dv; a.g = d->b.dg; a.gate = d->b.dgate; a.beta = d->b.dbeta; a.o = d->b.dout;
+  a.q = d->b.dq; a.k = d->b.dk; a.v = d->b.dv; a.g = d->b.dg; a.gate = d->b.dgate; a.beta = d->b.dbeta; a.kq = d->b.dkq; a.o = d->b.dout;
   a.dt = d->b.ddt; a.ld_dt = l.dt_n; a.ld_gate = l.gate_n;
   int rc;
   if ((rc = mix_linear(d, f32_out(d->b.proj + a.off_a, l.in_n), a.a2, nullptr, t, l.dt_n, a.ld_a2, CHATTS_EPI_NONE, f32_out(d->b.ddt, l.dt_n), s)) != 0) return rc;
@@ -178,8 +256,8 @@ static int mix_norm(const ChattsMixDecoder* d, int t, const float* y, const floa
   return chatts_residual_norm(&a, s);
 }
 
-extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, int n_spans, int single, chatts_stream_t s) {
-  CHATTS_REQUIRE(d && tokens, CHATTS_E_BADARG, "mixdec_forward: null argument");
+extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, const ChattsSpan* spans, int n_spans, int single, chatts_stream_t s) {
+  CHATTS_REQUIRE(d && tokens && (single || spans), CHATTS_E_BADARG, "mixdec_forward: null argument");
   const ChattsMixConfig& c = d->c;
   CHATTS_REQUIRE(t >= 1 && t <= c.t_max && (single || (n_spans >= 1 && n_spans <= c.max_slots)), CHATTS_E_SHAPE, "mixdec_forward: %d rows in %d segments", t, n_spans);
   StageRange stage(single ? "chatts.mix.decode" : "chatts.mix.prefill");
@@ -195,7 +273,7 @@ extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens,
     const float* next_norm = next ? d->layers[next->layer].norm1 : nullptr;
     if ((rc = mix_linear(d, A, l.in, l.in_t, t, l.in_n, c.width_p, CHATTS_EPI_NONE, f32_out(d->b.proj, l.in_n), s)) != 0) return rc;
     const ChattsOperand B = operand(d, true, t, l.out_k);
-    rc = l.kind == CHATTS_MIX_LATENT ? mix_latent(d, l, run, t, B, s) : mix_delta(d, l, run, t, n_spans, single != 0, B, s);
+    rc = l.kind == CHATTS_MIX_LATENT ? mix_latent(d, l, run, t, spans, n_spans, single != 0, B, s) : mix_delta(d, l, run, t, n_spans, single != 0, B, s);
     if (rc) return rc;
     if ((rc = mix_linear(d, B, l.out, l.out_t, t, c.width_p, l.out_k, CHATTS_EPI_NONE, Y, s)) != 0) return rc;
     if (!l.up) {
@@ -235,6 +313,6 @@ extern "C" int chatts_mixdec_decode(ChattsMixDecoder* d, int batch, const int64_
   CHATTS_REQUIRE(d && token && pos && batch >= 1 && batch <= d->c.max_slots, CHATTS_E_BADARG, "mixdec_decode: batch %d", batch);
   hipLaunchKernelGGL(rows_from_pos_kernel, dim3((batch + 255) / 256), dim3(256), 0, as_stream(s), d->b.rows, pos, batch);
   CHATTS_CHECK_LAUNCH("rows_from_pos");
-  if (const int rc = chatts_mixdec_forward(d, token, batch, 0, 1, s)) return rc;
+  if (const int rc = chatts_mixdec_forward(d, token, batch, nullptr, 0, 1, s)) return rc;
   return chatts_mixdec_logits(d, nullptr, batch, logits, s);
 }

@@ -219,7 +219,7 @@ class MixedDecoder(SlotModel):
 
     def _latent_layer(self, L, m):
         H, W = m.heads, self.config.hidden_size
-        dim_p, rank_p, rot_p, vdim_p = _up(m.dim, 32), _up(m.rank, 32), _up(m.rot, 32), _up(m.vdim, 16)
+        dim_p, rank_p, rot_p, vdim_p = _up(m.dim, 32), _up(m.rank, 64), _up(m.rot, 32), _up(m.vdim, 16)
         q = m.q.view(H, m.dim + m.rot, W)
         un = torch.zeros((H, dim_p, W), dtype=q.dtype, device=self.device)
         un[:, :m.dim] = q[:, :m.dim]
@@ -236,6 +236,9 @@ class MixedDecoder(SlotModel):
         uv = torch.zeros((H, vdim_p, rank_p), dtype=torch.bfloat16, device=self.device)
         uv[:, :m.vdim, :m.rank] = m.uv.view(H, m.vdim, m.rank).to(torch.bfloat16)
         L.uk, L.uv = self._dev(uk), self._dev(uv)
+        if self.expand_rows and self.lib.chatts_latent_can_expand(dim_p, rot_p, vdim_p, rank_p):      # prompts: keys and values written out
+            L.ukx, L.uvx = self._dev(uk.transpose(1, 2).reshape(H * dim_p, rank_p)), L.uv
+            self._exp = [max(a, b) for a, b in zip(self._exp, (rank_p, rot_p, H * dim_p, H * vdim_p, H * (dim_p + rot_p)))]
         cos, sin = rotary_tables(m.rot, m.rot_base, self.max_ctx, m.rot_scaling, self.device)
         L.latent = _lib.LatentArgs(off_q=off["q"], off_qr=off["qr"], off_c=off["c"], off_kr=off["kr"], heads=H, dim=m.dim, rot=m.rot, rank=m.rank,
                                    vdim=m.vdim, rank_p=rank_p, rot_p=rot_p, scale=m.scale, c_norm=self._f32(m.c_norm), cos_tab=self._dev(cos),
@@ -266,6 +269,8 @@ class MixedDecoder(SlotModel):
         Wp, V, Vp, MB, T = self._wp, cfg.vocab_size, _up(cfg.vocab_size, 64), self.max_batch, self.t_max
         self.vocab_p = Vp
         self._lat_q = self._lat_o = 1
+        self.expand_rows = 0 if self.exact else _up(min(self.max_ctx, max(8192, 2 * T)), 64) + 64 * MB
+        self._exp = [0] * 5                              # latent, rotated part, keys, values, queries of the expanded form: widest layer
         mixers, arr = [], (_lib.MixLayer * len(cfg.layers))()
         for i in range(len(cfg.layers)):
             lw, L = self.layer_weights(sd, i), arr[i]
@@ -310,10 +315,12 @@ class MixedDecoder(SlotModel):
         deltas = [L for L in arr if L.kind == _lib.MIX_DELTA]
         most = lambda f: max([f(L) for L in deltas], default=1)
         mc = _lib.MixConfig(width=W, width_p=Wp, n_layers=len(arr), n_runs=len(order), exact=int(self.exact), t_max=T, max_slots=MB, max_ctx=self.max_ctx,
+                            expand_rows=self.expand_rows if self._exp[0] else 0,
                             vocab=V, vocab_p=Vp, eps=cfg.rms_norm_eps, block_size=self.kv_block_size, table_stride=bps)
         ws = int(lib.chatts_mixdec_workspace(C.byref(mc), arr))
         rows = T + 1                                     # (kernels may read one row past the last)
         bf = dict(dtype=torch.bfloat16, device=dev)
+        xr = self.expand_rows if self._exp[0] else 0
         self.buf = B = {
             "x": torch.zeros((rows, Wp), **f32), "y": torch.zeros((rows, Wp), **f32), "proj": torch.zeros((rows, max(L.in_n for L in arr)), **f32),
             "a_f32": torch.zeros((rows, Wp), **f32), "b_f32": torch.zeros((rows, kmax), **f32),
@@ -321,13 +328,17 @@ class MixedDecoder(SlotModel):
             "q_f32": torch.zeros((rows, self._lat_q) if self.exact else (1, 1), **f32),
             "q_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, self._lat_q), **bf),
             "o_lat": torch.zeros((rows, self._lat_o), **f32), "partial": torch.zeros(max(64, MB) * 8 * self._lat_o + 65536, **f32),
+            "x_q": torch.zeros(rows * self._exp[4] + 16, **bf), "x_c": torch.zeros(xr * self._exp[0] + 16, **bf), "x_kr": torch.zeros(xr * self._exp[1] + 16, **bf),
+            "x_k": torch.zeros((2, xr * self._exp[2] + 16), **bf), "x_v": torch.zeros((2, xr * self._exp[3] + 16), **bf),
+            "x_zero": torch.zeros(max(xr, self._exp[3]) * self._exp[0] + 16, **bf),
             "dq": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
             "dk": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
             "dv": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
             "dg": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.dim)), **f32),
             "dgate": torch.zeros((rows, most(lambda L: L.gate_n)), **f32), "dbeta": torch.zeros((rows, most(lambda L: L.delta.heads)), **f32),
+            "dkq": torch.zeros((rows, most(lambda L: L.delta.kv_heads)), **f32),
             "dout": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32), "ddt": torch.zeros((rows, most(lambda L: L.dt_n)), **f32),
-            "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 4), dtype=torch.int32, device=dev),
+            "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
             "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),
             "pos_all": torch.full((MB,), -1, dtype=torch.int32, device=dev), "step_all": torch.zeros(MB, dtype=torch.int32, device=dev),
@@ -339,9 +350,10 @@ class MixedDecoder(SlotModel):
         mb = _lib.MixBuffers(embed=embed, head=head, head_t=head_t, final_norm=self._f32(mw["final_norm"], Wp), x=P(B["x"]), y=P(B["y"]), proj=P(B["proj"]),
                              a_f32=P(B["a_f32"]), b_f32=P(B["b_f32"]), a_hi=P(B["a_planes"][0]), a_lo=P(B["a_planes"][1]), b_hi=P(B["b_planes"][0]),
                              b_lo=P(B["b_planes"][1]), q_f32=P(B["q_f32"]), o_lat=P(B["o_lat"]), partial=P(B["partial"]), q_hi=P(B["q_planes"][0]),
-                             q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
+                             q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), qx=P(B["x_q"]), cbuf=P(B["x_c"]), krbuf=P(B["x_kr"]),
+                             kx_hi=P(B["x_k"][0]), kx_lo=P(B["x_k"][1]), vx_hi=P(B["x_v"][0]), vx_lo=P(B["x_v"][1]), zero=P(B["x_zero"]), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
                              logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
-                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dout", "ddt")})
+                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dkq", "dout", "ddt")})
         h = lib.chatts_mixdec_create(C.byref(mc), arr, runs, C.byref(mb))
         if not h:
             raise _lib.ChattsError(-1, lib.chatts_last_error().decode())
@@ -373,9 +385,11 @@ class MixedDecoder(SlotModel):
             meta[row:row + t, 0], meta[row:row + t, 1], meta[row:row + t, 2], meta[row:row + t, 3] = slot, pos0 + r, row, t - 1 - r
         B["rows"][:T].copy_(meta)
         single = all(s[1] == 1 for s in segs)
+        spans = (_lib.Span * len(segs))(*[_lib.Span(r, t, p, s, -1) for r, t, p, s in segs])
         if not single:
-            B["spans"][:len(segs)].copy_(torch.tensor([(r, t, p, s) for r, t, p, s in segs], dtype=torch.int32))
-        _lib.check(self.lib.chatts_mixdec_forward(self._decoder, _lib.ptr(B["ids"]), T, len(segs), int(single), _lib.stream_ptr()))
+            _lib.check(self.lib.chatts_mixdec_plan(self._decoder, spans, len(segs)))
+            B["spans"][:len(segs)].copy_(torch.frombuffer(spans, dtype=torch.int32).view(-1, 5))
+        _lib.check(self.lib.chatts_mixdec_forward(self._decoder, _lib.ptr(B["ids"]), T, spans, len(segs), int(single), _lib.stream_ptr()))
 
     def _logits(self, index):
         """logits of rows `index` of the last forward -> [n, vocab_p] float32"""

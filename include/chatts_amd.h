@@ -754,7 +754,8 @@ int chatts_decoder_decode_step(ChattsDecoder*, int32_t* pos_dev, int32_t* step_d
  * ------------------------------------------------------------------------------------------- */
 typedef struct ChattsRow { int32_t slot, pos, first, rest; } ChattsRow;   /* cache / state slot; position in its sequence; first row of
                                                                            * its segment in this step; rows of the segment after this one */
-typedef struct ChattsSpan { int32_t row0, t, pos0, slot; } ChattsSpan;    /* a segment: t rows from row0 at positions pos0 .. */
+typedef struct ChattsSpan { int32_t row0, t, pos0, slot, base; } ChattsSpan;   /* a segment: t rows from row0 at positions pos0 ..; base: first row of
+                                                                                 * its expanded keys (chatts_latent_expanded), < 0: not expanded */
 typedef struct ChattsOperand {   /* where the input of a following projection is written: float32 and / or bf16 hi / lo planes */
   float* f32;
   chatts_bf16* hi;
@@ -812,8 +813,8 @@ typedef struct ChattsDeltaArgs {
   const ChattsSpan* spans;   /* device; chatts_delta_scan only */
   int n_spans;
   /* scratch of the several-token form: q / k [T, kv_heads * dim], v / o [T, heads * vdim], g [T, heads * dim] (in: A2 a, out: decay),
-   * gate [T, heads * vdim] (G2 gin), beta [T, heads]; row strides = the widths, except ld_dt / ld_gate */
-  float *q, *k, *v, *g, *gate, *beta, *o;
+   * gate [T, heads * vdim] (G2 gin), beta [T, heads], kq [T, kv_heads] (k . q); row strides = the widths, except ld_dt / ld_gate */
+  float *q, *k, *v, *g, *gate, *beta, *kq, *o;
   const float* dt;
   int ld_dt, ld_gate;
   ChattsOperand out;
@@ -829,7 +830,7 @@ int chatts_delta_out(const ChattsDeltaArgs* args, chatts_stream_t stream);      
 typedef struct ChattsLatentArgs {
   float* proj;               /* [T, ld_proj]: unrotated and rotated query parts, latent [rank], key part [rot] */
   int ld_proj, off_q, off_qr, off_c, off_kr;         /* unrotated parts [heads, dim_p] (dim_p: the layer's), rotated parts [heads, rot] */
-  int heads, dim, rot, rank, vdim, rank_p, rot_p;
+  int heads, dim, rot, rank, vdim, rank_p, rot_p, dim_p;
   float scale, eps;
   const float* c_norm;       /* [rank] */
   const float* cos_tab;      /* [positions, rot / 2], magnitude included */
@@ -843,10 +844,29 @@ typedef struct ChattsLatentArgs {
   ChattsOperand q;           /* absorbed queries [T, heads * cw]: [W_uk^T q_unrotated | rotated part] per head */
   float* o;                  /* [T, heads * rank_p]: the weighted latents */
   int n_splits;              /* decode: key ranges per sequence, merged afterwards */
-  float* partial;            /* [T, heads, n_splits, rank_p + 2] when n_splits > 1 */
+  float* partial;            /* [T, heads, n_splits, rank_p + 4] when n_splits > 1 */
+  chatts_bf16* qx;           /* prep: also the expanded form's queries [T, heads * (dim_p + rot_p)], or NULL */
 } ChattsLatentArgs;
 int chatts_latent_prep(const ChattsLatentArgs* args, chatts_stream_t stream);        /* rotation, latent norm, cache write */
 int chatts_latent_attend(const ChattsLatentArgs* args, chatts_stream_t stream);      /* absorbed form: all heads share the cached rows */
+/* expanded form for spans of many tokens: keys and values of the spans' whole sequences are computed from the cached latents into scratch, then
+ * flash attention over them.  Spans with base >= 0, in order: base = rows of the spans before (each rounded up to 64). */
+typedef struct ChattsLatentExpandArgs {
+  const ChattsLatentArgs* latent;      /* as for chatts_latent_prep; qx written */
+  const ChattsSpan* spans;             /* host */
+  const ChattsSpan* spans_dev;
+  int n_spans, vdim_p, out_head, max_rows;
+  const chatts_bf16* uk;               /* [heads * dim_p, rank_p] */
+  const chatts_bf16* uv;               /* [heads * vdim_p, rank_p] */
+  chatts_bf16 *cbuf, *krbuf;           /* [max_rows, rank_p], [max_rows, rot_p] */
+  const chatts_bf16* zero;             /* zeros, [max(max_rows, heads * vdim_p), rank_p] */
+  chatts_bf16 *k_hi, *k_lo, *v_hi, *v_lo;   /* [max_rows, heads * dim_p], [heads * vdim_p, max_rows] */
+  ChattsOperand out;
+  void* workspace;
+  size_t workspace_bytes;
+} ChattsLatentExpandArgs;
+int chatts_latent_can_expand(int dim_p, int rot_p, int vdim_p, int rank_p);
+int chatts_latent_expanded(const ChattsLatentExpandArgs* args, chatts_stream_t stream);
 
 /* ---- the composed decoder (mixdec.hip) ---- */
 #define CHATTS_MIX_LATENT 1
@@ -859,6 +879,7 @@ typedef struct ChattsMixLayer {
   const chatts_bf16 *up, *up_t, *down, *down_t;      /* squared-relu feed-forward [ff, width_p], [width_p, ff]; up == NULL: none */
   int in_n, out_k, ff;
   const chatts_bf16 *uk, *uv;                        /* latent: W_uk^T per head [heads, rank_p, dim_p], W_uv per head [heads, vdim_p, rank_p] */
+  const chatts_bf16 *ukx, *uvx;                      /* latent, expanded form: [heads * dim_p, rank_p], [heads * vdim_p, rank_p]; NULL: never expanded */
   int dim_p, vdim_p, out_head;                       /* out_head: columns between heads in the input of `out` */
   int dt_n, gate_n;                                  /* delta: rows of a2 / g2, padded to 16 */
   ChattsLatentArgs latent;                           /* sizes, offsets and weights; the rest is filled in per step */
@@ -873,6 +894,7 @@ typedef struct ChattsMixRun {      /* one pass through a layer */
 } ChattsMixRun;
 typedef struct ChattsMixConfig {
   int width, width_p, n_layers, n_runs, exact, t_max, max_slots, max_ctx;
+  int expand_rows;                 /* rows of buffers.cbuf ..: keys that a step may expand; 0: latent attention always runs absorbed */
   int64_t vocab, vocab_p;
   float eps;
   int block_size, table_stride;
@@ -886,7 +908,9 @@ typedef struct ChattsMixBuffers {
   float *q_f32, *o_lat, *partial;                    /* latent: [t_max, heads * cw] (32-bit runs), [t_max, heads * rank_p], splits */
   chatts_bf16 *q_hi, *q_lo;
   size_t partial_elems;
-  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dout, *ddt;
+  chatts_bf16 *qx, *cbuf, *krbuf, *kx_hi, *kx_lo, *vx_hi, *vx_lo;   /* latent, expanded form (ChattsLatentExpandArgs) */
+  const chatts_bf16* zero;
+  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dkq, *dout, *ddt;
   ChattsRow* rows;                                   /* device, [t_max] */
   ChattsSpan* spans;                                 /* device, [max_slots] */
   int32_t* table;                                    /* device, [max_slots, table_stride] */
@@ -899,8 +923,11 @@ ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, const ChattsMix
 void chatts_mixdec_destroy(ChattsMixDecoder* d);
 size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const ChattsMixLayer* layers);
 /* x[0 .. t) = the residual stream of t rows described by buffers.rows / .spans (n_spans segments), embedded from `tokens` (device).  single:
- * every segment is one row (decode kernels, no spans read). */
-int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, int n_spans, int single, chatts_stream_t stream);
+ * every segment is one row (decode kernels, no spans read).
+ * spans: the host's copy of buffers.spans. */
+int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, const ChattsSpan* spans, int n_spans, int single, chatts_stream_t stream);
+/* which of the spans run expanded, and where (fills span.base; the caller then uploads them to buffers.spans) */
+int chatts_mixdec_plan(ChattsMixDecoder* d, ChattsSpan* spans, int n_spans);
 /* logits[i] = head . norm(x[index[i]]) for n rows (index: device, NULL = rows 0 .. n) */
 int chatts_mixdec_logits(ChattsMixDecoder* d, const int32_t* index, int n, float* logits, chatts_stream_t stream);
 /* decode: rows of slots 0 .. batch at pos[slot] (< 0: parked) with token[slot]; logits of all rows; nothing is selected here */

@@ -93,7 +93,7 @@ def test_reference_delta_rule_writes_before_it_reads():
 
 def test_struct_layouts_match_the_header(tmp_path):
     from chatts_amd import _lib
-    names = {"ChattsRow": 16, "ChattsSpan": 16, "ChattsOperand": C.sizeof(_lib.Operand), "ChattsResidualNormArgs": C.sizeof(_lib.ResidualNormArgs),
+    names = {"ChattsRow": 16, "ChattsSpan": C.sizeof(_lib.Span), "ChattsLatentExpandArgs": C.sizeof(_lib.LatentExpandArgs), "ChattsOperand": C.sizeof(_lib.Operand), "ChattsResidualNormArgs": C.sizeof(_lib.ResidualNormArgs),
              "ChattsHeadLinearArgs": C.sizeof(_lib.HeadLinearArgs), "ChattsDeltaArgs": C.sizeof(_lib.DeltaArgs), "ChattsLatentArgs": C.sizeof(_lib.LatentArgs),
              "ChattsMixLayer": C.sizeof(_lib.MixLayer), "ChattsMixRun": C.sizeof(_lib.MixRun), "ChattsMixConfig": C.sizeof(_lib.MixConfig),
              "ChattsMixBuffers": C.sizeof(_lib.MixBuffers), "ChattsLinearArgs": C.sizeof(_lib.LinearArgs)}
