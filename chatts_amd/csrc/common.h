@@ -195,7 +195,9 @@ __device__ __forceinline__ float softplus_f(float x) {
 }
 // lane N of each row of 16, to the whole row
 template <int N>
-__device__ __forceinline__ float row_bcast(float v) { return dpp_mov<0x150 + N>(v); }
+__device__ __forceinline__ float row_bcast(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x150 + N, 0xF, 0xF, true));      // (every lane is valid: folds into the user)
+}
 
 inline hipStream_t as_stream(chatts_stream_t s) { return reinterpret_cast<hipStream_t>(s); }
 

@@ -375,6 +375,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int 
     unroll_tokens<0, kT>([&](auto tc) __attribute__((always_inline)) {
       constexpr int t = decltype(tc)::value;
       if constexpr (t + 1 < kT) read(b, t + 1, ops[(t + 1) & 1]);
+      __builtin_amdgcn_sched_barrier(0);      // (a whole token of work between the request and its use)
       const Ops& o = ops[t & 1];
       float d[2] = {0.f, 0.f}, e[2] = {0.f, 0.f};
 #pragma unroll
@@ -387,13 +388,18 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int 
         for (int j = 0; j < 4; ++j) e[j & 1] += s[c][j] * o.q[c][j];
       }
       const float dd = row16_sum(d[0] + d[1]), ee = row16_sum(e[0] + e[1]);
-      const float u = row_bcast<t>(bv) - row_bcast<t>(beta) * dd;      // beta (v - S^T k)
+      float u;
+      {
+#pragma clang fp contract(off)
+        u = row_bcast<t>(bv) - row_bcast<t>(beta) * dd;      // beta (v - S^T k)
+      }
 #pragma unroll
       for (int c = 0; c < NC; ++c)
 #pragma unroll
         for (int j = 0; j < 4; ++j) s[c][j] += o.k[c][j] * u;
       const float out = ee + row_bcast<t>(kq) * u;
       keep = l16 == t ? out : keep;
+      __builtin_amdgcn_sched_barrier(0);
     });
     if (l16 < kT) so[l16][cl] = keep;
     if (more) stage(b ^ 1);
