@@ -7,11 +7,11 @@
 //   * latent_prep_kernel: rotation of the query parts, norm of the latent, rotation of the key part, cache write
 //   * head_linear_kernel: W_uk^T on the queries, W_uv on the weighted latents (a product per head)
 //   * latent_attend_kernel: one (row, head) per workgroup on the vector units, float32 or bf16 cache: the 32-bit runs and odd sizes
-//   * latent_decode_kernel: 16 heads of a row per workgroup on the matrix pipe, bf16 cache, the keys spread over waves and workgroups, partials
+//   * latent_decode_kernel: up to 32 heads of a row per workgroup on the matrix pipe, bf16 cache, the keys spread over workgroups, partials
 //     merged by latent_merge_kernel
 // The expanded form (first half of each line) does fewer products per key once many queries share it: prompts take it
 //   * latent_gather_kernel, two projections (keys; values, transposed by exchanging the operands) and latent_prefill_kernel, a flash loop
-#include "gemm_common.h"
+#include "ring_store.h"
 
 namespace chatts {
 
@@ -142,28 +142,69 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(ChattsLatentArgs p) 
   }
 }
 
-// ---- absorbed attention on the matrix pipe: grid (splits, rows, head tiles), 16 heads per workgroup -------------------------------------
-// A wave works alone on tiles of 32 keys (every 4 n_splits-th), which LDS-DMA brings into its own LDS region: S^T = K Q^T reads rows of it as A
-// fragments, so a lane ends up with 8 scores of one head (column = lane & 15); O^T = C^T P^T reads it transposed, and its B fragment IS the
-// 8 probabilities of the lane.  K slot 8 g + j of that product means key 4 g + j (j < 4) or 16 + 4 g + j - 4, on both sides.  No barrier until
-// the four waves' sums are merged at the end; while one wave waits for its tile the other three compute.
+// ---- absorbed attention on the matrix pipe: grid (splits, rows, head tiles / HT), HT x 16 heads per workgroup ----------------------------
+// Tiles of 32 keys pass through a ring of four in LDS, filled by two loader waves (LDS-DMA) and read by four compute waves; compute wave = (head
+// tile, slice of the latent columns).  S^T = K Q^T reads rows of the tile as A fragments, so a lane ends up with 8 scores of one head (column =
+// lane & 15); O^T = C^T P^T reads the tile transposed, and its B fragment IS the 8 probabilities of the lane.  K slot 8 g + j of that product means
+// key 4 g + j (j < 4) or 16 + 4 g + j - 4, on both sides.  The waves of a head tile compute the same scores (that is cheaper than handing them
+// round) and own different latent columns: nothing is merged inside a workgroup.
 // 16-byte chunk c of row r lies at position c ^ (r & swizzle): neither way of reading meets the same banks in every row.
 typedef short s16x4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) s16x4* lds_s16x4;
+constexpr int kLatStages = 4, kLatLoaders = 2, kLatThreads = 64 * (4 + kLatLoaders);
 
-static __host__ __device__ inline int latent_wave_bytes(int rank_p, int cw) { return 64 * (cw > rank_p + 16 ? cw : rank_p + 16); }
+// at most n (wave-uniform) of this wave's requests outstanding
+__device__ __forceinline__ void latent_wait(int n) {
+#define CHATTS_VM(N) case N: asm volatile("s_waitcnt vmcnt(" #N ")" ::: "memory"); break;
+#define CHATTS_VM4(A, B, C, D) CHATTS_VM(A) CHATTS_VM(B) CHATTS_VM(C) CHATTS_VM(D)
+  switch (n) {
+    CHATTS_VM4(1, 2, 3, 4) CHATTS_VM4(5, 6, 7, 8) CHATTS_VM4(9, 10, 11, 12) CHATTS_VM4(13, 14, 15, 16) CHATTS_VM4(17, 18, 20, 22) CHATTS_VM4(24, 26, 28, 30)
+    CHATTS_VM(32) CHATTS_VM(34) CHATTS_VM(36)
+    default: asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); break;
+  }
+#undef CHATTS_VM4
+#undef CHATTS_VM
+}
 
-template <int NF, int NK, bool FULL>      // rank_p <= 16 NF, cw <= 32 NK; FULL: equal
-__global__ __launch_bounds__(256, 1) void latent_decode_kernel(ChattsLatentArgs p) {
+template <int NF, int NK, int HT, bool FULL>      // rank_p <= 16 NF, cw <= 32 NK; FULL: equal
+__global__ __launch_bounds__(kLatThreads, 2) void latent_decode_kernel(ChattsLatentArgs p) {
   extern __shared__ __attribute__((aligned(1024))) char smem[];
-  __shared__ float stat[2][4][16];
-  const int split = blockIdx.x, row = blockIdx.y, ht = blockIdx.z, tid = threadIdx.x, lane = tid & 63;
+  constexpr int RS = 4 / HT, NFW = NF / RS;      // slices of the latent columns, fragments per wave
+  const int split = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int cw = p.rank_p + p.rot_p, cv = cw >> 3, nf = FULL ? NF : p.rank_p >> 4, nk = FULL ? NK : cw >> 5, sw = (cv & 7) == 0 ? 7 : 3;
+  const int cw = FULL ? 32 * NK : p.rank_p + p.rot_p, cv = cw >> 3, nf = FULL ? NF : p.rank_p >> 4, nk = FULL ? NK : cw >> 5, sw = (cv & 7) == 0 ? 7 : 3;
   const ChattsRow R = p.rows[row];
   if (R.pos < 0) return;
   const int n = R.pos + 1, ntiles = (n + 31) >> 5, fr = lane & 15, fg = lane >> 4;
-  char* kt = smem + wave * latent_wave_bytes(p.rank_p, cw);
+  const int count = split < ntiles ? (ntiles - split + p.n_splits - 1) / p.n_splits : 0;      // tiles split, split + n_splits, ...
+  const int stage = cw * 64;
+  if (wave >= 4) {
+    // ---- loader: every kLatLoaders-th of the cw / 16 pieces (64 chunks of 16 bytes) of a tile
+    const int L = wave - 4, pieces = cw >> 4, mine = (pieces - L + kLatLoaders - 1) / kLatLoaders;
+    const int e0 = L * 64 + lane, r0 = e0 / cv, c0 = e0 - r0 * cv, dr = kLatLoaders * 64 / cv, dc = kLatLoaders * 64 - dr * cv;
+    const char* cache = reinterpret_cast<const char*>(p.cache);
+    auto issue = [&](int k) {
+      const char* tile = cache + latent_row(p, R.slot, (split + k * p.n_splits) * 32, cw) * 2;
+      char* base = smem + (k & (kLatStages - 1)) * stage + L * 1024;
+      int r = r0, c = c0;
+      for (int i = 0; i < mine; ++i) {
+        __builtin_amdgcn_global_load_lds((gptr_t)(tile + (uint32_t)(r * cw + ((c ^ (r & sw)) << 3)) * 2), (lptr_t)(base + i * (kLatLoaders * 1024)), 16, 0, 0);
+        r += dr;
+        c += dc;
+        if (c >= cv) { c -= cv; ++r; }
+      }
+    };
+    for (int k = 0; k < kLatStages - 1 && k < count; ++k) issue(k);
+    for (int k = 0; k < count; ++k) {
+      const int later = count - 1 - k < kLatStages - 2 ? count - 1 - k : kLatStages - 2;
+      latent_wait(later * mine);                              // tile k has landed
+      __builtin_amdgcn_s_barrier();                           // ... and everyone has read tile k - 1
+      if (n - (split + k * p.n_splits) * 32 < 32) __builtin_amdgcn_s_barrier();
+      if (k + kLatStages - 1 < count) issue(k + kLatStages - 1);
+    }
+    return;
+  }
+  const int ht = blockIdx.z * HT + wave / RS, f0 = (wave % RS) * NFW;
   bf16x8_t q[NK];
   {
     int h = ht * 16 + fr;
@@ -173,45 +214,54 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(ChattsLatentArgs 
     for (int k = 0; k < NK; ++k)
       if (k < nk) q[k] = *reinterpret_cast<const bf16x8_t*>(src + k * 32);
   }
-  const uint16_t* cache = reinterpret_cast<const uint16_t*>(p.cache);
   float m = -INFINITY, l = 0.f;      // of head fr; l: this lane's keys only
-  f32x4 acc[NF];
+  f32x4 acc[NFW];
 #pragma unroll
-  for (int i = 0; i < NF; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  const int step = p.n_splits * 4, pieces = cw >> 4;      // 1 KB pieces of a tile
-  // chunk `lane` of piece 0: row, column; a piece later it is 64 chunks further
-  const int r0 = lane / cv, c0 = lane - r0 * cv, dr = 64 / cv, dc = 64 - dr * cv;
-  for (int t = split * 4 + wave; t < ntiles; t += step) {
-    const uint16_t* tile = cache + latent_row(p, R.slot, t * 32, cw);
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // the previous tile has been read
-    {
-      int r = r0, c = c0;
-      for (int i = 0; i < pieces; ++i) {
-        __builtin_amdgcn_global_load_lds((gptr_t)(tile + (size_t)r * cw + ((c ^ (r & sw)) << 3)), (lptr_t)(kt + i * 1024), 16, 0, 0);
-        r += dr;
-        c += dc;
-        if (c >= cv) { c -= cv; ++r; }
-      }
-    }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    const int lim = n - t * 32;
+  for (int i = 0; i < NFW; ++i) acc[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < count; ++k) {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // this wave has read tile k - 1
+    __builtin_amdgcn_s_barrier();                           // tile k is complete
+    char* kt = smem + (k & (kLatStages - 1)) * stage;
+    const int lim = n - (split + k * p.n_splits) * 32;
     if (lim < 32) {      // keys past the last one become zeros, whatever an unused cache row holds
-      for (int e = lim * cv + lane; e < 32 * cv; e += 64) *reinterpret_cast<u32x4*>(kt + e * 16) = (u32x4){0u, 0u, 0u, 0u};
+      for (int e = lim * cv + tid; e < 32 * cv; e += 256) *reinterpret_cast<u32x4*>(kt + e * 16) = (u32x4){0u, 0u, 0u, 0u};
       asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      __builtin_amdgcn_s_barrier();
     }
     f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
     {
       const char* a0 = kt + fr * cw * 2;
       const char* a1 = kt + (16 + fr) * cw * 2;
       const int x = fr & sw;      // (16 is a multiple of the swizzle's period)
+      // fragments of G K-steps are requested while those before are multiplied
+      constexpr int G = 3, NG = (NK + G - 1) / G;
+      bf16x8_t kf[2][G][2];
+      auto request = [&](int g, bf16x8_t (&dst)[G][2]) __attribute__((always_inline)) {
 #pragma unroll
-      for (int k = 0; k < NK; ++k)
-        if (k < nk) {
-          const int c = ((k * 4 + fg) ^ x) << 4;
-          s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a0 + c), q[k], s[0], 0, 0, 0);
-          s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a1 + c), q[k], s[1], 0, 0, 0);
-          if (k % 6 == 5) asm volatile("" ::: "memory");      // (keeps the reads in flight within the registers)
+        for (int u = 0; u < G; ++u) {
+          const int k2 = g * G + u;
+          if (k2 < NK && k2 < nk) {
+            const int c = ((k2 * 4 + fg) ^ x) << 4;
+            dst[u][0] = *reinterpret_cast<const bf16x8_t*>(a0 + c);
+            dst[u][1] = *reinterpret_cast<const bf16x8_t*>(a1 + c);
+          }
         }
+      };
+      request(0, kf[0]);
+#pragma unroll
+      for (int g = 0; g < NG; ++g) {
+        if (g + 1 < NG) request(g + 1, kf[(g + 1) & 1]);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int u = 0; u < G; ++u) {
+          const int k2 = g * G + u;
+          if (k2 < NK && k2 < nk) {
+            s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[g & 1][u][0], q[k2], s[0], 0, 0, 0);
+            s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[g & 1][u][1], q[k2], s[1], 0, 0, 0);
+          }
+        }
+        __builtin_amdgcn_sched_barrier(0);
+      }
     }
     float v[8], mx = -INFINITY;
 #pragma unroll
@@ -236,66 +286,55 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(ChattsLatentArgs 
     l = l * alpha + sum;
     if (__any(alpha != 1.0f)) {
 #pragma unroll
-      for (int i = 0; i < NF; ++i)
+      for (int i = 0; i < NFW; ++i)
 #pragma unroll
         for (int r = 0; r < 4; ++r) acc[i][r] *= alpha;
     }
     {
-      // transposing reads: lane -> row 4 g + (fr >> 2) (and + 16), 4 columns (fr & 3) * 4 of the fragment's 16: chunk 2 i + (fr >> 1 & 1), half fr & 1
+      // transposing reads: lane -> row 4 g + (fr >> 2) (and + 16), 4 columns (fr & 3) * 4 of the fragment's 16: chunk 2 f + (fr >> 1 & 1), half fr & 1
       const int tr = fg * 4 + (fr >> 2), x = tr & sw, cb = (fr >> 1) & 1;
       const char* t0 = kt + tr * cw * 2 + (fr & 1) * 8;
+      constexpr int G = NFW < 4 ? NFW : 4, NG = NFW / G;
+      union Tr { s16x4 h[2]; bf16x8_t v; };
+      Tr a[2][G];
+      auto request = [&](int g, Tr (&dst)[G]) __attribute__((always_inline)) {
 #pragma unroll
-      for (int i = 0; i < NF; ++i)
-        if (i < nf) {
-          const int c = ((2 * i + cb) ^ x) << 4;
-          union { s16x4 h[2]; bf16x8_t v; } a;
-          a.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(t0 + c));
-          a.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(t0 + 32 * cw + c));
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, ph, acc[i], 0, 0, 0);
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pl, acc[i], 0, 0, 0);
-          if (i % 8 == 7) asm volatile("" ::: "memory");
+        for (int u = 0; u < G; ++u) {
+          const int f = f0 + g * G + u;
+          if (FULL || f < nf) {
+            const int c = ((2 * f + cb) ^ x) << 4;
+            dst[u].h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(t0 + c));
+            dst[u].h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(t0 + 32 * cw + c));
+          }
         }
+      };
+      request(0, a[0]);
+#pragma unroll
+      for (int g = 0; g < NG; ++g) {
+        if (g + 1 < NG) request(g + 1, a[(g + 1) & 1]);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int u = 0; u < G; ++u)
+          if (FULL || f0 + g * G + u < nf) acc[g * G + u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[g & 1][u].v, ph, acc[g * G + u], 0, 0, 0);
+#pragma unroll
+        for (int u = 0; u < G; ++u)
+          if (FULL || f0 + g * G + u < nf) acc[g * G + u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[g & 1][u].v, pl, acc[g * G + u], 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0);
+      }
     }
   }
-  // merge of the four waves: O^T (lane: 4 consecutive latent columns of its head) into the wave's LDS tile as [16 heads][rank_p + 16] floats
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
-  if (fg == 0) { stat[0][wave][fr] = m; stat[1][wave][fr] = l; }
-  const int ldk = p.rank_p + 16, wf = latent_wave_bytes(p.rank_p, cw) >> 2;
-  float* ot = reinterpret_cast<float*>(kt);
-  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  const int h = ht * 16 + fr;
+  if (h >= p.heads) return;
+  // a lane: 4 consecutive latent columns of its head per fragment
+  const bool whole = p.n_splits == 1;
+  float* dst = whole ? p.o + ((size_t)row * p.heads + h) * p.rank_p : p.partial + (((size_t)row * p.heads + h) * p.n_splits + split) * (p.rank_p + 4);
+  const float f = whole ? 1.0f / l : 1.0f;
 #pragma unroll
-  for (int i = 0; i < NF; ++i)
-    if (i < nf) *reinterpret_cast<f32x4*>(ot + fr * ldk + i * 16 + fg * 4) = acc[i];
-  __syncthreads();
-  const int c4 = p.rank_p >> 2;
-  for (int e = tid; e < 16 * c4; e += 256) {
-    const int hh = e / c4, c = (e - hh * c4) * 4, h = ht * 16 + hh;
-    if (h >= p.heads) continue;
-    float M = -INFINITY, L = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) M = fmaxf(M, stat[0][w][hh]);
-    f32x4 o = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int w = 0; w < 4; ++w) {
-      const float mw = stat[0][w][hh];
-      if (mw == -INFINITY) continue;      // a wave without a tile
-      const float f = exp_hw(mw - M);
-      L += f * stat[1][w][hh];
-      const f32x4 x = *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem) + (size_t)w * wf + hh * ldk + c);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] += f * x[r];
-    }
-    if (p.n_splits == 1) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] /= L;
-      *reinterpret_cast<f32x4*>(p.o + ((size_t)row * p.heads + h) * p.rank_p + c) = o;
-    } else {
-      float* dst = p.partial + (((size_t)row * p.heads + h) * p.n_splits + split) * (p.rank_p + 4);
-      *reinterpret_cast<f32x4*>(dst + c) = o;
-      if (c == 0) { dst[p.rank_p] = M; dst[p.rank_p + 1] = L; }
-    }
-  }
+  for (int i = 0; i < NFW; ++i)
+    if (FULL || f0 + i < nf) *reinterpret_cast<f32x4*>(dst + (f0 + i) * 16 + fg * 4) = (f32x4){acc[i][0] * f, acc[i][1] * f, acc[i][2] * f, acc[i][3] * f};
+  if (!whole && f0 == 0 && fg == 0) { dst[p.rank_p] = m; dst[p.rank_p + 1] = l; }
 }
 
 // merge of the splits: one workgroup per (head, row)
@@ -541,23 +580,26 @@ static int check_latent(const ChattsLatentArgs* a, const char* who) {
   return CHATTS_OK;
 }
 
-template <int NF, int NK, bool FULL>
+template <int NF, int NK, int HT, bool FULL>
 static int launch_latent_decode_t(const ChattsLatentArgs* a, hipStream_t s) {
-  const size_t lds = (size_t)4 * latent_wave_bytes(a->rank_p, a->rank_p + a->rot_p);
   static bool configured = false;
   if (!configured) {
-    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NF, NK, FULL>), hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024);
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_kernel<NF, NK, HT, FULL>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                             kLatStages * 32 * NK * 64);
     CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "latent_attend: cannot reserve LDS: %s", hipGetErrorString(e));
     configured = true;
   }
-  hipLaunchKernelGGL((latent_decode_kernel<NF, NK, FULL>), dim3(a->n_splits, a->n_rows, (a->heads + 15) / 16), dim3(256), lds, s, *a);
+  const int tiles = (a->heads + 15) / 16;
+  hipLaunchKernelGGL((latent_decode_kernel<NF, NK, HT, FULL>), dim3(a->n_splits, a->n_rows, (tiles + HT - 1) / HT), dim3(kLatThreads),
+                     kLatStages * (a->rank_p + a->rot_p) * 64, s, *a);
   CHATTS_CHECK_LAUNCH("latent_decode");
   return CHATTS_OK;
 }
-
 template <int NF, int NK>
 static int launch_latent_decode(const ChattsLatentArgs* a, hipStream_t s) {
-  return a->rank_p == 16 * NF && a->rank_p + a->rot_p == 32 * NK ? launch_latent_decode_t<NF, NK, true>(a, s) : launch_latent_decode_t<NF, NK, false>(a, s);
+  const bool full = a->rank_p == 16 * NF && a->rank_p + a->rot_p == 32 * NK;
+  if (a->heads <= 16) return full ? launch_latent_decode_t<NF, NK, 1, true>(a, s) : launch_latent_decode_t<NF, NK, 1, false>(a, s);
+  return full ? launch_latent_decode_t<NF, NK, 2, true>(a, s) : launch_latent_decode_t<NF, NK, 2, false>(a, s);
 }
 
 static int latent_attend_impl(const ChattsLatentArgs* a, hipStream_t s) {

@@ -152,10 +152,10 @@ static int mix_latent_absorbed(const ChattsMixDecoder* d, const ChattsMixLayer& 
   h.a = a.proj + (size_t)r0 * a.ld_proj + a.off_q; h.lda = a.ld_proj; h.a_head = l.dim_p;
   h.w = l.uk; h.m = n; h.heads = a.heads; h.n = a.rank_p; h.k = l.dim_p; h.out = a.q; h.out_head = cw; h.exact = d->c.exact;
   if ((rc = chatts_head_linear(&h, s)) != 0) return rc;
-  // few rows: the keys of a row are spread over workgroups (each takes 128 keys at a time) until there is about one per CU
-  const int tiles = (a.heads + 15) / 16 * n;
-  int splits = tiles >= 256 ? 1 : 256 / tiles;
-  const int most = (d->c.max_ctx + 127) / 128;
+  // few rows: the keys of a row are spread over workgroups (32 at a time) until there is about one per CU
+  const int groups = (a.heads + 31) / 32 * n;
+  int splits = groups >= 256 ? 1 : 256 / groups;
+  const int most = (d->c.max_ctx + 63) / 64;
   if (splits > most) splits = most;
   if (splits > 64) splits = 64;
   while (splits > 1 && (size_t)n * a.heads * splits * (a.rank_p + 4) > d->b.partial_elems) --splits;
