@@ -156,6 +156,7 @@ class LatentExpandArgs(C.Structure):
 
 
 MIX_LATENT, MIX_DELTA = 1, 2
+EXPAND_PAD = 128           # CHATTS_LATENT_EXPAND_PAD
 
 
 class MixLayer(C.Structure):

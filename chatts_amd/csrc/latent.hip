@@ -384,8 +384,13 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(ChattsLatentArgs p, 
   }
 }
 
-// grid (query tiles of 128, heads, spans), a wave owns 32 queries of one head, 64 keys per step: S^T = K Q^T, O^T = V^T P^T - the probabilities of
-// a lane are the B fragment of the second product (K slot 8 g + j = key 8 g + j: the rows of K are read in the order that makes it so).
+// grid (heads, query tiles of 128, spans) - the heads of an XCD (workgroup id modulo 8) stay the same, so their keys and values stay in its L2, and every
+// XCD gets long and short query tiles alike -, a wave owns 32 queries of one head, 64 keys per step: S^T = K Q^T, O^T = V^T P^T - the probabilities of
+// a lane are the B fragment of the second product (K slot 8 g + j = key 8 g + j: the rows of K are staged in the order that makes it so).
+// Rows of the expanded keys and values are 256 bytes longer than their contents: at a power-of-two stride every row of a tile would lie in the
+// same L2 channel.
+constexpr int kExpandPad = CHATTS_LATENT_EXPAND_PAD;
+
 struct LatentPrefill {
   const uint16_t* kx;      // [rows, ldk]: unrotated keys, head by head (dim_p each)
   const uint16_t* kr;      // [rows, rot_p]
@@ -399,7 +404,7 @@ template <int NK, int NV, int OCC, bool FULL>      // dim_p + rot_p <= 32 NK, vd
 __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill p, const ChattsSpan* __restrict__ spans) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const ChattsSpan sp = spans[blockIdx.z];
-  const int qt0 = (gridDim.x - 1 - blockIdx.x) * 128, h = blockIdx.y;      // the longest key ranges first
+  const int qt0 = (gridDim.y - 1 - blockIdx.y) * 128, h = blockIdx.x;      // the longest key ranges first
   if (sp.base < 0 || qt0 >= sp.t) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, fg = lane >> 4;
   const int dq = FULL ? 32 * NK : p.dim_p + p.rot_p, vdim_p = FULL ? 16 * NV : p.vdim_p, ldl = dq + 8, nk = dq >> 5, nv = vdim_p >> 4;
@@ -423,6 +428,7 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
 #pragma unroll
   for (int i = 0; i < NV; ++i) o[i][0] = o[i][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
+  const float scale2 = p.scale * 1.44269504088896341f;      // scores in base 2
   // staging: K rows in 16-byte pieces (64 rows x dq / 8), V^T rows (vdim_p x 8)
   constexpr int KP = NK, VP = (NV + 1) / 2;
   u32x4 rk[KP], rv[VP];
@@ -432,7 +438,7 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
       const int e = i * 256 + tid;
-      if (e < 64 * kc) {
+      if (FULL || e < 64 * kc) {
         const int r = e / kc, c = e - r * kc;
         rk[i] = c < dc ? *reinterpret_cast<const u32x4*>(p.kx + (base + r) * p.ldk + h * p.dim_p + c * 8)
                        : *reinterpret_cast<const u32x4*>(p.kr + (base + r) * p.rot_p + (c - dc) * 8);
@@ -441,7 +447,7 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
 #pragma unroll
     for (int i = 0; i < VP; ++i) {
       const int e = i * 256 + tid;
-      if (e < vdim_p * 8) rv[i] = *reinterpret_cast<const u32x4*>(p.vt + (size_t)(h * vdim_p + (e >> 3)) * p.ldv + base + (e & 7) * 8);
+      if (FULL ? NV % 2 == 0 || e < vdim_p * 8 : e < vdim_p * 8) rv[i] = *reinterpret_cast<const u32x4*>(p.vt + (size_t)(h * vdim_p + (e >> 3)) * p.ldv + base + (e & 7) * 8);
     }
   };
   fetch(0);
@@ -450,12 +456,15 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
       const int e = i * 256 + tid;
-      if (e < 64 * kc) *reinterpret_cast<u32x4*>(ks + (e / kc) * ldl + (e % kc) * 8) = rk[i];
+      if (FULL || e < 64 * kc) {      // key 32 G + 8 g + 4 h + j -> row 32 G + 16 h + 4 g + j: the rows of a fragment lie next to each other
+        const int key = e / kc, r = (key & 35) | ((key & 4) << 2) | ((key & 24) >> 1);
+        *reinterpret_cast<u32x4*>(ks + r * ldl + (e - key * kc) * 8) = rk[i];
+      }
     }
 #pragma unroll
     for (int i = 0; i < VP; ++i) {
       const int e = i * 256 + tid;
-      if (e < vdim_p * 8) *reinterpret_cast<u32x4*>(vs + (e >> 3) * kLdV + (e & 7) * 8) = rv[i];
+      if (FULL ? NV % 2 == 0 || e < vdim_p * 8 : e < vdim_p * 8) *reinterpret_cast<u32x4*>(vs + (e >> 3) * kLdV + (e & 7) * 8) = rv[i];
     }
     __syncthreads();
     if (t + 1 < ntiles) fetch(t + 1);
@@ -463,18 +472,27 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
     f32x4 s[4][2];      // [32-key group * 2 + half][query block]
 #pragma unroll
     for (int a = 0; a < 4; ++a) s[a][0] = s[a][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const uint16_t* kb = ks + (8 * (fr >> 2) + (fr & 3)) * ldl + fg * 8;
+    const uint16_t* kb = ks + fr * ldl + fg * 8;
+    {
+      bf16x8_t kf[2][4];      // the next K-step's fragments are requested while this one's are multiplied
+      auto request = [&](int k, bf16x8_t (&dst)[4]) __attribute__((always_inline)) {
 #pragma unroll
-    for (int k = 0; k < NK; ++k)
-      if (k < nk) {
+        for (int a = 0; a < 4; ++a) dst[a] = *reinterpret_cast<const bf16x8_t*>(kb + a * 16 * ldl + k * 32);
+      };
+      request(0, kf[0]);
 #pragma unroll
-        for (int a = 0; a < 4; ++a) {
-          const bf16x8_t kv = *reinterpret_cast<const bf16x8_t*>(kb + ((a >> 1) * 32 + (a & 1) * 4) * ldl + k * 32);
-          s[a][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kv, q[0][k], s[a][0], 0, 0, 0);
-          s[a][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kv, q[1][k], s[a][1], 0, 0, 0);
+      for (int k = 0; k < NK; ++k)
+        if (k < nk) {
+          if (k + 1 < NK && k + 1 < nk) request(k + 1, kf[(k + 1) & 1]);
+          __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+          for (int a = 0; a < 4; ++a) {
+            s[a][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k & 1][a], q[0][k], s[a][0], 0, 0, 0);
+            s[a][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k & 1][a], q[1][k], s[a][1], 0, 0, 0);
+          }
+          __builtin_amdgcn_sched_barrier(0);
         }
-        asm volatile("" ::: "memory");
-      }
+    }
     bf16x8_t pf[2][2];      // [32-key group][query block]
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
@@ -485,21 +503,21 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
       for (int a = 0; a < 4; ++a)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          float v = s[a][u][r] * p.scale;
+          float v = s[a][u][r] * scale2;
           if (edge && t * 64 + (a >> 1) * 32 + fg * 8 + (a & 1) * 4 + r > qpos) v = -INFINITY;
           s[a][u][r] = v;
           mx = fmaxf(mx, v);
         }
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mn = fmaxf(m[u], mx), safe = mn == -INFINITY ? 0.f : mn, alpha = exp_hw(m[u] - safe);
+      const float mn = fmaxf(m[u], mx), safe = mn == -INFINITY ? 0.f : mn, alpha = __builtin_amdgcn_exp2f(m[u] - safe);
       m[u] = mn;
       float sum = 0.f;
 #pragma unroll
       for (int a = 0; a < 4; ++a)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float e = exp_hw(s[a][u][r] - safe);
+          const float e = __builtin_amdgcn_exp2f(s[a][u][r] - safe);
           sum += e;
           pf[a >> 1][u][(a & 1) * 4 + r] = (__bf16)e;
         }
@@ -511,17 +529,26 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
           for (int r = 0; r < 4; ++r) o[i][u][r] *= alpha;
       }
     }
+    {
+      bf16x8_t vf[2][2];
+      auto request = [&](int i, bf16x8_t (&dst)[2]) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < NV; ++i)
-      if (i < nv) {
+        for (int g = 0; g < 2; ++g) dst[g] = *reinterpret_cast<const bf16x8_t*>(vs + (i * 16 + fr) * kLdV + g * 32 + fg * 8);
+      };
+      request(0, vf[0]);
 #pragma unroll
-        for (int g = 0; g < 2; ++g) {
-          const bf16x8_t vv = *reinterpret_cast<const bf16x8_t*>(vs + (i * 16 + fr) * kLdV + g * 32 + fg * 8);
-          o[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pf[g][0], o[i][0], 0, 0, 0);
-          o[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pf[g][1], o[i][1], 0, 0, 0);
+      for (int i = 0; i < NV; ++i)
+        if (i < nv) {
+          if (i + 1 < NV && i + 1 < nv) request(i + 1, vf[(i + 1) & 1]);
+          __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+          for (int g = 0; g < 2; ++g) {
+            o[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i & 1][g], pf[g][0], o[i][0], 0, 0, 0);
+            o[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i & 1][g], pf[g][1], o[i][1], 0, 0, 0);
+          }
+          __builtin_amdgcn_sched_barrier(0);
         }
-        if (i % 2 == 1) asm volatile("" ::: "memory");      // (keeps the reads in flight within the registers)
-      }
+    }
   }
 #pragma unroll
   for (int u = 0; u < 2; ++u) {
@@ -638,7 +665,7 @@ static int launch_latent_prefill_t(const LatentPrefill& p, const ChattsSpan* spa
     CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "latent_expanded: cannot reserve LDS: %s", hipGetErrorString(e));
     configured = true;
   }
-  hipLaunchKernelGGL((latent_prefill_kernel<NK, NV, OCC, FULL>), dim3((longest + 127) / 128, heads, n_spans), dim3(256), lds, s, p, spans);
+  hipLaunchKernelGGL((latent_prefill_kernel<NK, NV, OCC, FULL>), dim3(heads, (longest + 127) / 128, n_spans), dim3(256), lds, s, p, spans);
   CHATTS_CHECK_LAUNCH("latent_prefill");
   return CHATTS_OK;
 }
@@ -711,18 +738,18 @@ extern "C" int chatts_latent_expanded(const ChattsLatentExpandArgs* x, chatts_st
   ChattsLinearArgs g{};      // keys: [rows, heads * dim_p] = latents . W_uk^T;  values, transposed: [heads * vdim_p, rows] = W_uv . latents^T
   g.workspace = x->workspace; g.workspace_bytes = x->workspace_bytes;
   g.a_hi = x->cbuf; g.a_lo = x->zero; g.ld_planes = a->rank_p; g.w = x->uk; g.ldw = a->rank_p;
-  g.m = rows; g.n = a->heads * a->dim_p; g.k = a->rank_p; g.ldc = g.n; g.c_hi = x->k_hi; g.c_lo = x->k_lo; g.ld_cplanes = g.n; g.epilogue = CHATTS_EPI_NONE;
+  g.m = rows; g.n = a->heads * a->dim_p; g.k = a->rank_p; g.ldc = g.n; g.c_hi = x->k_hi; g.c_lo = x->k_lo; g.ld_cplanes = g.n + kExpandPad; g.epilogue = CHATTS_EPI_NONE;
   int rc;
   if ((rc = chatts_linear(&g, stream)) != 0) return rc;
   g.a_hi = x->uv; g.w = x->cbuf;
-  g.m = a->heads * x->vdim_p; g.n = rows; g.ldc = rows; g.c_hi = x->v_hi; g.c_lo = x->v_lo; g.ld_cplanes = rows;
+  g.m = a->heads * x->vdim_p; g.n = rows; g.ldc = rows; g.c_hi = x->v_hi; g.c_lo = x->v_lo; g.ld_cplanes = rows + kExpandPad;
   if ((rc = chatts_linear(&g, stream)) != 0) return rc;
   LatentPrefill p{};
   p.kx = x->k_hi; p.kr = x->krbuf; p.vt = x->v_hi; p.qx = a->qx;
-  p.ldk = a->heads * a->dim_p; p.ldv = rows; p.ldq = a->heads * (a->dim_p + a->rot_p);
+  p.ldk = a->heads * a->dim_p + kExpandPad; p.ldv = rows + kExpandPad; p.ldq = a->heads * (a->dim_p + a->rot_p);
   p.dim_p = a->dim_p; p.rot_p = a->rot_p; p.vdim_p = x->vdim_p; p.out_head = x->out_head; p.scale = a->scale; p.out = x->out;
   const int dq = a->dim_p + a->rot_p;
   if (dq <= 96 && x->vdim_p <= 64) return launch_latent_prefill<3, 4, 2>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
-  if (dq <= 192 && x->vdim_p <= 128) return launch_latent_prefill<6, 8, 2>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
+  if (dq <= 192 && x->vdim_p <= 128) return launch_latent_prefill<6, 8, 1>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
   return launch_latent_prefill<12, 16, 1>(p, x->spans_dev, x->n_spans, a->heads, longest, s);
 }

@@ -329,7 +329,8 @@ class MixedDecoder(SlotModel):
             "q_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, self._lat_q), **bf),
             "o_lat": torch.zeros((rows, self._lat_o), **f32), "partial": torch.zeros(max(64, MB) * 8 * self._lat_o + 65536, **f32),
             "x_q": torch.zeros(rows * self._exp[4] + 16, **bf), "x_c": torch.zeros(xr * self._exp[0] + 16, **bf), "x_kr": torch.zeros(xr * self._exp[1] + 16, **bf),
-            "x_k": torch.zeros((2, xr * self._exp[2] + 16), **bf), "x_v": torch.zeros((2, xr * self._exp[3] + 16), **bf),
+            "x_k": torch.zeros((2, xr * (self._exp[2] + _lib.EXPAND_PAD) + 16), **bf),
+            "x_v": torch.zeros((2, self._exp[3] * (xr + _lib.EXPAND_PAD) + 16), **bf),
             "x_zero": torch.zeros(max(xr, self._exp[3]) * self._exp[0] + 16, **bf),
             "dq": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
             "dk": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),

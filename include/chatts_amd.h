@@ -860,11 +860,12 @@ typedef struct ChattsLatentExpandArgs {
   const chatts_bf16* uv;               /* [heads * vdim_p, rank_p] */
   chatts_bf16 *cbuf, *krbuf;           /* [max_rows, rank_p], [max_rows, rot_p] */
   const chatts_bf16* zero;             /* zeros, [max(max_rows, heads * vdim_p), rank_p] */
-  chatts_bf16 *k_hi, *k_lo, *v_hi, *v_lo;   /* [max_rows, heads * dim_p], [heads * vdim_p, max_rows] */
+  chatts_bf16 *k_hi, *k_lo, *v_hi, *v_lo;   /* [max_rows, heads * dim_p + pad], [heads * vdim_p, max_rows + pad], pad = CHATTS_LATENT_EXPAND_PAD */
   ChattsOperand out;
   void* workspace;
   size_t workspace_bytes;
 } ChattsLatentExpandArgs;
+#define CHATTS_LATENT_EXPAND_PAD 128
 int chatts_latent_can_expand(int dim_p, int rot_p, int vdim_p, int rank_p);
 int chatts_latent_expanded(const ChattsLatentExpandArgs* args, chatts_stream_t stream);
 

@@ -410,7 +410,7 @@ def test_latent_expanded(heads, dim, rot, vdim, rank):
     host = (_lib.Span * 3)(*[_lib.Span(*s, b) for s, b in zip(spans, bases)])
     dev = torch.tensor([list(s) + [b] for s, b in zip(spans, bases)], dtype=torch.int32, device=DEV)
     z = lambda *s: torch.zeros(*s, dtype=torch.bfloat16, device=DEV)
-    cb, kr, zero, kh, kl, vh, vl = z(at, m.rp), z(at, m.rotp), z(max(at, heads * vp), m.rp), z(at, heads * dp), z(at, heads * dp), z(heads * vp, at), z(heads * vp, at)
+    cb, kr, zero, kh, kl, vh, vl = z(at, m.rp), z(at, m.rotp), z(max(at, heads * vp), m.rp), z(at, heads * dp + 128), z(at, heads * dp + 128), z(heads * vp, at + 128), z(heads * vp, at + 128)
     ukd, uvd, qd = ukp.to(DEV), uvp.to(DEV), qx.reshape(T, -1).contiguous().to(DEV)
     out = torch.full((T, heads * (vp + 4)), 5.0, device=DEV)
     ws = torch.zeros(64 << 20, dtype=torch.uint8, device=DEV)
