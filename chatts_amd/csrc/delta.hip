@@ -4,7 +4,7 @@
 //  * delta_decode_kernel: one token per sequence, everything of a (sequence, head) in one workgroup: convolutions from the ring of
 //    earlier inputs, unit norms, the low-rank decay and gate products, the state update (state in registers between its two passes) and the
 //    normed, gated read-out.  One launch instead of five, the state is read and written once.
-//  * delta_prep_kernel / delta_scan_kernel / delta_out_kernel: several tokens per sequence.  prep does what is parallel over tokens; scan
+//  * delta_lowrank_kernel, delta_prep_*_kernel / delta_scan_kernel / delta_out_kernel: several tokens per sequence.  The first do what is parallel over tokens; scan
 //    walks the tokens with the state in registers - a column of S belongs to 16 lanes of a wave, so the two sums over key channels are
 //    DPP row reductions and columns never talk to each other; out norms and gates.
 // The ring of convolution inputs is indexed by position modulo taps: the current token's entry is never one that the same step reads, so
@@ -139,23 +139,21 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
 }
 
 // ---- several tokens: what is parallel over tokens -------------------------------------------------------------------------------
-constexpr int kPrepRows = 4;      // consecutive rows of a wave: the convolution's window slides in registers
-
-// convolution + silu of channel ch for rows row0 .. row0 + kPrepRows.  Tokens before a row's segment come from the ring.
-template <int TAPS>      // 0: any number of taps
-__device__ __forceinline__ void conv_rows(const ChattsDeltaArgs& p, int row0, const ChattsRow (&R)[kPrepRows], int ch, float (&y)[kPrepRows]) {
+// convolution + silu of channel ch for rows row0 .. row0 + ROWS: the window slides in registers.  Tokens before a row's segment come from the ring.
+template <int TAPS, int ROWS>      // TAPS 0: any number of taps
+__device__ __forceinline__ void conv_rows(const ChattsDeltaArgs& p, int row0, const ChattsRow (&R)[ROWS], int ch, float (&y)[ROWS]) {
   if constexpr (TAPS > 0) {
-    float x[kPrepRows + TAPS - 1], w[TAPS];
+    float x[ROWS + TAPS - 1], w[TAPS];
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) w[j] = p.conv_w[(size_t)j * p.conv_ch + ch];
 #pragma unroll
-    for (int j = 0; j < kPrepRows + TAPS - 1; ++j) {
+    for (int j = 0; j < ROWS + TAPS - 1; ++j) {
       int r = row0 + j - (TAPS - 1);
       r = r < 0 ? 0 : (r > p.n_rows - 1 ? p.n_rows - 1 : r);
       x[j] = p.proj[(size_t)r * p.ld_proj + ch];
     }
 #pragma unroll
-    for (int i = 0; i < kPrepRows; ++i) {
+    for (int i = 0; i < ROWS; ++i) {
       float acc = 0.f;
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) {
@@ -171,7 +169,7 @@ __device__ __forceinline__ void conv_rows(const ChattsDeltaArgs& p, int row0, co
     }
   } else {
 #pragma unroll
-    for (int i = 0; i < kPrepRows; ++i) {
+    for (int i = 0; i < ROWS; ++i) {
       float acc = 0.f;
       for (int j = 0; j < p.taps; ++j) {
         const int lag = p.taps - 1 - j, q = R[i].pos - lag, r = row0 + i - lag;
@@ -183,100 +181,168 @@ __device__ __forceinline__ void conv_rows(const ChattsDeltaArgs& p, int row0, co
     }
   }
 }
-
-// a wave takes one item of kPrepRows rows at a time: a q / k head, 64 channels of v, 64 decays, 64 betas
-template <int TAPS, int NCH>      // NCH: 64-channel pieces of a q / k head
-__global__ __launch_bounds__(256) void delta_prep_kernel(ChattsDeltaArgs p) {
-  const int row0 = blockIdx.x * kPrepRows, lane = threadIdx.x & 63, wave = blockIdx.y * 4 + (threadIdx.x >> 6), waves = gridDim.y * 4;
-  ChattsRow R[kPrepRows];
-  bool live[kPrepRows];
+template <int ROWS>
+__device__ __forceinline__ void prep_rows(const ChattsDeltaArgs& p, int row0, ChattsRow (&R)[ROWS], bool (&live)[ROWS]) {
 #pragma unroll
-  for (int i = 0; i < kPrepRows; ++i) {
-    R[i] = p.rows[row0 + i < p.n_rows ? row0 + i : p.n_rows - 1];
+  for (int i = 0; i < ROWS; ++i) {
+    const int r = row0 + i < p.n_rows ? row0 + i : p.n_rows - 1;
+    R[i] = p.rows[r];
     live[i] = row0 + i < p.n_rows && R[i].pos >= 0;
-    if (!live[i]) R[i] = ChattsRow{0, 0, row0 + i < p.n_rows ? row0 + i : p.n_rows - 1, 0};
+    if (!live[i]) R[i] = ChattsRow{0, 0, r, 0};
   }
-  const int dim = p.dim, nv = p.heads * p.vdim, ng = p.heads * dim;
-  const int vchunks = (nv + 63) / 64, gchunks = (ng + 63) / 64, bchunks = (p.heads + 63) / 64;
-  const int items = p.kv_heads + vchunks + gchunks + bchunks;
-  for (int it = wave; it < items; it += waves) {
-    int e = it;
-    if (e < p.kv_heads) {
-      float q[NCH][kPrepRows], k[NCH][kPrepRows], qs[kPrepRows], ks[kPrepRows], qk[kPrepRows];
+}
+
+// q / k heads: a wave = one head of four rows
+constexpr int kQkRows = 4, kVRows = 8;
+template <int TAPS, int NCH>      // NCH: 64-channel pieces of a head
+__global__ __launch_bounds__(256) void delta_prep_qk_kernel(ChattsDeltaArgs p) {
+  const int row0 = blockIdx.x * kQkRows, lane = threadIdx.x & 63, e = blockIdx.y * 4 + (threadIdx.x >> 6), dim = p.dim;
+  if (e >= p.kv_heads) return;
+  ChattsRow R[kQkRows];
+  bool live[kQkRows];
+  prep_rows(p, row0, R, live);
+  float q[NCH][kQkRows], k[NCH][kQkRows], qs[kQkRows], ks[kQkRows], qk[kQkRows];
 #pragma unroll
-      for (int i = 0; i < kPrepRows; ++i) qs[i] = ks[i] = qk[i] = 0.f;
+  for (int i = 0; i < kQkRows; ++i) qs[i] = ks[i] = qk[i] = 0.f;
 #pragma unroll
-      for (int c = 0; c < NCH; ++c) {
-        const int ch = c * 64 + lane;
-        const bool ok = ch < dim;
-        conv_rows<TAPS>(p, row0, R, p.off_q + e * dim + (ok ? ch : 0), q[c]);
-        conv_rows<TAPS>(p, row0, R, p.off_k + e * dim + (ok ? ch : 0), k[c]);
+  for (int c = 0; c < NCH; ++c) {
+    const int ch = c * 64 + lane;
+    const bool ok = ch < dim;
+    conv_rows<TAPS>(p, row0, R, p.off_q + e * dim + (ok ? ch : 0), q[c]);
+    conv_rows<TAPS>(p, row0, R, p.off_k + e * dim + (ok ? ch : 0), k[c]);
 #pragma unroll
-        for (int i = 0; i < kPrepRows; ++i) {
-          if (!ok) q[c][i] = k[c][i] = 0.f;
-          qs[i] += q[c][i] * q[c][i];
-          ks[i] += k[c][i] * k[c][i];
-          qk[i] += q[c][i] * k[c][i];
-        }
+    for (int i = 0; i < kQkRows; ++i) {
+      if (!ok) q[c][i] = k[c][i] = 0.f;
+      qs[i] += q[c][i] * q[c][i];
+      ks[i] += k[c][i] * k[c][i];
+      qk[i] += q[c][i] * k[c][i];
+    }
+  }
+  const float qscale = rsqrtf((float)dim);
+#pragma unroll
+  for (int i = 0; i < kQkRows; ++i) {
+    const float fq = qscale / sqrtf(wave_sum(qs[i]) + 1e-6f), fk = 1.0f / sqrtf(wave_sum(ks[i]) + 1e-6f), d = wave_sum(qk[i]);
+    if (!live[i]) continue;
+    const size_t at = (size_t)(row0 + i) * p.kv_heads + e;
+#pragma unroll
+    for (int c = 0; c < NCH; ++c) {
+      const int ch = c * 64 + lane;
+      if (ch < dim) {
+        p.q[at * dim + ch] = q[c][i] * fq;
+        p.k[at * dim + ch] = k[c][i] * fk;
       }
-      const float qscale = rsqrtf((float)dim);
-#pragma unroll
-      for (int i = 0; i < kPrepRows; ++i) {
-        const float fq = qscale / sqrtf(wave_sum(qs[i]) + 1e-6f), fk = 1.0f / sqrtf(wave_sum(ks[i]) + 1e-6f), d = wave_sum(qk[i]);
-        if (!live[i]) continue;
-        const size_t at = (size_t)(row0 + i) * p.kv_heads + e;
-#pragma unroll
-        for (int c = 0; c < NCH; ++c) {
-          const int ch = c * 64 + lane;
-          if (ch < dim) {
-            p.q[at * dim + ch] = q[c][i] * fq;
-            p.k[at * dim + ch] = k[c][i] * fk;
-          }
-        }
-        if (lane == 0) p.kq[at] = d * fq * fk;
-      }
-      continue;
     }
-    e -= p.kv_heads;
-    if (e < vchunks) {
-      const int ch = e * 64 + lane;
-      if (ch >= nv) continue;
-      float y[kPrepRows];
-      conv_rows<TAPS>(p, row0, R, p.off_v + ch, y);
-#pragma unroll
-      for (int i = 0; i < kPrepRows; ++i)
-        if (live[i]) p.v[(size_t)(row0 + i) * nv + ch] = y[i];
-      continue;
-    }
-    e -= vchunks;
-    if (e < gchunks) {
-      const int ch = e * 64 + lane;
-      if (ch >= ng) continue;
-      const float na = p.neg_a[ch / dim], bias = p.dt_bias[ch];
-      float x[kPrepRows];
-#pragma unroll
-      for (int i = 0; i < kPrepRows; ++i) x[i] = live[i] ? p.dt[(size_t)(row0 + i) * p.ld_dt + ch] : 0.f;
-#pragma unroll
-      for (int i = 0; i < kPrepRows; ++i)
-        if (live[i]) p.g[(size_t)(row0 + i) * ng + ch] = exp_hw(na * softplus_f(x[i] + bias));
-      continue;
-    }
-    e -= gchunks;
+    if (lane == 0) p.kq[at] = d * fq * fk;
+  }
+}
+
+// v and beta: a wave = 64 channels of eight rows
+template <int TAPS>
+__global__ __launch_bounds__(256) void delta_prep_v_kernel(ChattsDeltaArgs p) {
+  const int row0 = blockIdx.x * kVRows, lane = threadIdx.x & 63, e = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int nv = p.heads * p.vdim, vchunks = (nv + 63) / 64;
+  ChattsRow R[kVRows];
+  bool live[kVRows];
+  prep_rows(p, row0, R, live);
+  if (e < vchunks) {
     const int ch = e * 64 + lane;
-    if (ch < p.heads)
+    if (ch >= nv) return;
+    float y[kVRows];
+    conv_rows<TAPS>(p, row0, R, p.off_v + ch, y);
 #pragma unroll
-      for (int i = 0; i < kPrepRows; ++i)
-        if (live[i]) p.beta[(size_t)(row0 + i) * p.heads + ch] = sigmoid_f(p.proj[(size_t)(row0 + i) * p.ld_proj + p.off_b + ch]);
+    for (int i = 0; i < kVRows; ++i)
+      if (live[i]) p.v[(size_t)(row0 + i) * nv + ch] = y[i];
+    return;
+  }
+  const int h = (e - vchunks) * 64 + lane;
+  if (h < p.heads)
+#pragma unroll
+    for (int i = 0; i < kVRows; ++i)
+      if (live[i]) p.beta[(size_t)(row0 + i) * p.heads + h] = sigmoid_f(p.proj[(size_t)(row0 + i) * p.ld_proj + p.off_b + h]);
+}
+
+// The low-rank products with what follows them:  g = exp(neg_a[h] * softplus(A2 a + dt_bias)),  gate = sigmoid(G2 gin).  grid (row tiles of 16, blocks of
+// 512 outputs): a wave keeps its 16 rows of a (or gin) in registers, split into bf16 planes (three of them in 32-bit runs: exact), and walks 8
+// tiles of 16 outputs, the weights requested two tiles ahead.
+constexpr int kLrTiles = 8;
+template <int NP, int KMAX>      // planes, rank / 32
+__global__ __launch_bounds__(256) void delta_lowrank_kernel(ChattsDeltaArgs p, int ablocks) {
+  typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+  const bool dec = (int)blockIdx.y < ablocks;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, fr = lane & 15, fg = lane >> 4, m0 = blockIdx.x * 16;
+  const int n = dec ? p.heads * p.dim : p.heads * p.vdim, rank = dec ? p.rank_a : p.rank_g, ldw = dec ? p.ld_a2 : p.ld_g2;
+  const int n0 = (dec ? blockIdx.y : blockIdx.y - ablocks) * (64 * kLrTiles) + wave * (16 * kLrTiles);
+  if (n0 >= n) return;
+  const uint16_t* w = dec ? p.a2 : p.g2;
+  const int r = m0 + fr < p.n_rows ? m0 + fr : p.n_rows - 1;
+  const float* x = p.proj + (size_t)r * p.ld_proj + (dec ? p.off_a : p.off_g) + fg * 8;
+  f32x4 acc[kLrTiles];
+#pragma unroll
+  for (int t = 0; t < kLrTiles; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < rank; k0 += 32 * KMAX) {
+    bf16x8_t a[KMAX][NP];
+    int ko[KMAX];      // K offsets; past the rank: offset 0 and zeros in a
+#pragma unroll
+    for (int k = 0; k < KMAX; ++k) {
+      const bool ok = k0 + k * 32 < rank;
+      ko[k] = ok ? k0 + k * 32 : 0;
+      const f32x4 x0 = *reinterpret_cast<const f32x4*>(x + ko[k]), x1 = *reinterpret_cast<const f32x4*>(x + ko[k] + 4);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        float v = ok ? (j < 4 ? x0[j] : x1[j - 4]) : 0.f;
+#pragma unroll
+        for (int q = 0; q < NP; ++q) {
+          a[k][q][j] = (__bf16)v;
+          v -= (float)a[k][q][j];
+        }
+      }
+    }
+    bf16x8_t b[3][KMAX];
+    auto request = [&](int t, bf16x8_t (&dst)[KMAX]) __attribute__((always_inline)) {
+      int o = n0 + t * 16 + fr;
+      if (o > n - 1) o = n - 1;
+#pragma unroll
+      for (int k = 0; k < KMAX; ++k) dst[k] = *reinterpret_cast<const bf16x8_t*>(w + (size_t)o * ldw + ko[k] + fg * 8);
+    };
+    request(0, b[0]);
+    request(1, b[1]);
+#pragma unroll
+    for (int t = 0; t < kLrTiles; ++t) {
+      if (t + 2 < kLrTiles) request(t + 2, b[(t + 2) % 3]);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int k = 0; k < KMAX; ++k)
+#pragma unroll
+        for (int q = NP - 1; q >= 0; --q) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[k][q], b[t % 3][k], acc[t], 0, 0, 0);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+  }
+  const float inv_dim = 1.0f / (float)p.dim;
+#pragma unroll
+  for (int t = 0; t < kLrTiles; ++t) {
+    const int o = n0 + t * 16 + fr;
+    if (o < n) {
+      int h = dec ? (int)((float)o * inv_dim) : 0;      // o / dim: off by one at most (o < 2^24), set right below
+      if (dec) h += (o - h * p.dim >= p.dim) - (o < h * p.dim);
+      const float na = dec ? p.neg_a[h] : 0.f, bias = dec ? p.dt_bias[o] : 0.f;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int row = m0 + fg * 4 + q;
+        const float v = dec ? exp_hw(na * softplus_f(acc[t][q] + bias)) : sigmoid_f(acc[t][q]);
+        if (row < p.n_rows) (dec ? p.g : p.gate)[(size_t)row * n + o] = v;
+      }
+    }
   }
 }
 
 template <int TAPS>
 static void launch_prep(const ChattsDeltaArgs* a, hipStream_t s) {
-  const int items = a->kv_heads + (a->heads * a->vdim + 63) / 64 + (a->heads * a->dim + 63) / 64 + (a->heads + 63) / 64;
-  const dim3 g((a->n_rows + kPrepRows - 1) / kPrepRows, (items + 7) / 8), b(256);
-  if (a->dim <= 64) hipLaunchKernelGGL((delta_prep_kernel<TAPS, 1>), g, b, 0, s, *a);
-  else if (a->dim <= 128) hipLaunchKernelGGL((delta_prep_kernel<TAPS, 2>), g, b, 0, s, *a);
-  else hipLaunchKernelGGL((delta_prep_kernel<TAPS, 4>), g, b, 0, s, *a);
+  const dim3 g((a->n_rows + kQkRows - 1) / kQkRows, (a->kv_heads + 3) / 4), b(256);
+  if (a->dim <= 64) hipLaunchKernelGGL((delta_prep_qk_kernel<TAPS, 1>), g, b, 0, s, *a);
+  else if (a->dim <= 128) hipLaunchKernelGGL((delta_prep_qk_kernel<TAPS, 2>), g, b, 0, s, *a);
+  else hipLaunchKernelGGL((delta_prep_qk_kernel<TAPS, 4>), g, b, 0, s, *a);
+  const int items = (a->heads * a->vdim + 63) / 64 + (a->heads + 63) / 64;
+  hipLaunchKernelGGL(delta_prep_v_kernel<TAPS>, dim3((a->n_rows + kVRows - 1) / kVRows, (items + 3) / 4), b, 0, s, *a);
 }
 
 // ---- the recurrence over a span: grid (heads * column blocks, spans), 4 waves x 4 columns ---------------------------------------------
@@ -293,13 +359,14 @@ __device__ __forceinline__ void unroll_tokens(F&& f) {
   }
 }
 template <int NC>
-__global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p, int colblocks) {
+__global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p) {
   constexpr int D = NC * 64, kT = NC <= 2 ? 16 : 8;
   __shared__ __attribute__((aligned(16))) float sk[2][kT][D], sq[2][kT][D], sg[2][kT][D];
   __shared__ float so[kT][17];
   const ChattsSpan sp = p.spans[blockIdx.y];
   if (sp.t < 1) return;
-  const int h = blockIdx.x / colblocks, cb = blockIdx.x - h * colblocks, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  // (consecutive workgroups take consecutive heads: the column blocks of a head run on one XCD where heads % 8 == 0, its k / q / g in that L2)
+  const int cb = blockIdx.x / p.heads, h = blockIdx.x - cb * p.heads, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int dim = p.dim, vdim = p.vdim, v4 = (vdim + 3) & ~3, hk = h / (p.heads / p.kv_heads);
   const int l16 = lane & 15, cl = wave * 4 + (lane >> 4), col = cb * 16 + cl;
   const bool live = col < vdim;
@@ -437,7 +504,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(ChattsDeltaArgs p) {
 #pragma unroll
     for (int c = 0; c < 4; ++c) {
       const int i = c * 64 + lane;
-      if (i < vdim) store_operand(p.out, row, h * vdim + i, v[c] * f * p.norm_w[i] * sigmoid_f(p.gate[(size_t)row * p.ld_gate + h * vdim + i]));
+      if (i < vdim) store_operand(p.out, row, h * vdim + i, v[c] * f * p.norm_w[i] * p.gate[(size_t)row * vrow + h * vdim + i]);
     }
   }
   if (R.rest < p.taps) {
@@ -486,8 +553,15 @@ extern "C" int chatts_delta_decode(const ChattsDeltaArgs* a, chatts_stream_t str
 
 extern "C" int chatts_delta_prep(const ChattsDeltaArgs* a, chatts_stream_t stream) {
   if (const int rc = check_delta(a, "delta_prep")) return rc;
-  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->kq && a->dt, CHATTS_E_BADARG, "delta_prep: null scratch");
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->gate && a->beta && a->kq && a->a2 && a->g2, CHATTS_E_BADARG, "delta_prep: null scratch");
   if (a->n_rows == 0) return CHATTS_OK;
+  CHATTS_REQUIRE(a->rank_a % 32 == 0 && a->rank_g % 32 == 0 && ((uintptr_t)a->a2 % 16) == 0 && ((uintptr_t)a->g2 % 16) == 0 && a->off_a % 4 == 0 && a->off_g % 4 == 0,
+                 CHATTS_E_SHAPE, "delta_prep: ranks %d / %d must be padded to multiples of 32", a->rank_a, a->rank_g);
+  const int ablocks = (a->heads * a->dim + 64 * kLrTiles - 1) / (64 * kLrTiles), gblocks = (a->heads * a->vdim + 64 * kLrTiles - 1) / (64 * kLrTiles);
+  const dim3 g((a->n_rows + 15) / 16, ablocks + gblocks), b(256);
+  if (a->exact) hipLaunchKernelGGL((delta_lowrank_kernel<3, 4>), g, b, 0, as_stream(stream), *a, ablocks);
+  else hipLaunchKernelGGL((delta_lowrank_kernel<2, 4>), g, b, 0, as_stream(stream), *a, ablocks);
+  CHATTS_CHECK_LAUNCH("delta_lowrank");
   switch (a->taps) {
     case 2: launch_prep<2>(a, as_stream(stream)); break;
     case 3: launch_prep<3>(a, as_stream(stream)); break;
@@ -506,9 +580,9 @@ extern "C" int chatts_delta_scan(const ChattsDeltaArgs* a, chatts_stream_t strea
   const dim3 g(a->heads * cb, a->n_spans), b(256);
   hipStream_t s = as_stream(stream);
   switch ((a->dim + 63) / 64) {
-    case 1: hipLaunchKernelGGL(delta_scan_kernel<1>, g, b, 0, s, *a, cb); break;
-    case 2: hipLaunchKernelGGL(delta_scan_kernel<2>, g, b, 0, s, *a, cb); break;
-    default: hipLaunchKernelGGL(delta_scan_kernel<4>, g, b, 0, s, *a, cb); break;
+    case 1: hipLaunchKernelGGL(delta_scan_kernel<1>, g, b, 0, s, *a); break;
+    case 2: hipLaunchKernelGGL(delta_scan_kernel<2>, g, b, 0, s, *a); break;
+    default: hipLaunchKernelGGL(delta_scan_kernel<4>, g, b, 0, s, *a); break;
   }
   CHATTS_CHECK_LAUNCH("delta_scan");
   return CHATTS_OK;

@@ -48,7 +48,6 @@ extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const Chatts
     add(l.in_n, c->width_p);
     add(c->width_p, l.out_k);
     if (l.up) { add(l.ff, c->width_p); add(c->width_p, l.ff); }
-    if (l.kind == CHATTS_MIX_DELTA) { add(l.dt_n, l.delta.ld_a2); add(l.gate_n, l.delta.ld_g2); }
   }
   add((int)c->vocab_p, c->width_p);
   // keys and values written out from the latents: rows in whole tiles of 64
@@ -239,10 +238,8 @@ static int mix_delta(const ChattsMixDecoder* d, const ChattsMixLayer& l, const C
   a.out = out;
   if (single) return chatts_delta_decode(&a, s);
   a.q = d->b.dq; a.k = d->b.dk; a.v = d->b.dv; a.g = d->b.dg; a.gate = d->b.dgate; a.beta = d->b.dbeta; a.kq = d->b.dkq; a.o = d->b.dout;
-  a.dt = d->b.ddt; a.ld_dt = l.dt_n; a.ld_gate = l.gate_n;
+  a.exact = d->c.exact;
   int rc;
-  if ((rc = mix_linear(d, f32_out(d->b.proj + a.off_a, l.in_n), a.a2, nullptr, t, l.dt_n, a.ld_a2, CHATTS_EPI_NONE, f32_out(d->b.ddt, l.dt_n), s)) != 0) return rc;
-  if ((rc = mix_linear(d, f32_out(d->b.proj + a.off_g, l.in_n), a.g2, nullptr, t, l.gate_n, a.ld_g2, CHATTS_EPI_NONE, f32_out(d->b.dgate, l.gate_n), s)) != 0) return rc;
   if ((rc = chatts_delta_prep(&a, s)) != 0) return rc;
   if ((rc = chatts_delta_scan(&a, s)) != 0) return rc;
   return chatts_delta_out(&a, s);

@@ -254,13 +254,12 @@ class MixedDecoder(SlotModel):
         L.w_in, L.in_t = self._mat(w, tile=True)
         L.out_k, L.out_head = _up(v, 64), m.vdim
         L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
-        L.dt_n, L.gate_n = _up(m.heads * m.dim, 16), _up(v, 16)
         conv = torch.zeros((m.taps, off["a"]), dtype=torch.float32, device=self.device)
         for n, t in (("q", m.q_conv), ("k", m.k_conv), ("v", m.v_conv)):
             conv[:, off[n]:off[n] + t.shape[0]] = t.to(torch.float32).t()
         L.delta = _lib.DeltaArgs(off_q=off["q"], off_k=off["k"], off_v=off["v"], off_a=off["a"], off_g=off["g"], off_b=off["b"], conv_ch=off["a"],
                                  heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, taps=m.taps, rank_a=ra_p, rank_g=rg_p,
-                                 conv_w=self._dev(conv), a2=self._mat(m.a2, L.dt_n, ra_p)[0], g2=self._mat(m.g2, L.gate_n, rg_p)[0], ld_a2=ra_p, ld_g2=rg_p,
+                                 conv_w=self._dev(conv), a2=self._mat(m.a2, None, ra_p)[0], g2=self._mat(m.g2, None, rg_p)[0], ld_a2=ra_p, ld_g2=rg_p,
                                  dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32))), norm_w=self._f32(m.norm))
 
     def _build(self, sd):
@@ -336,9 +335,9 @@ class MixedDecoder(SlotModel):
             "dk": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
             "dv": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
             "dg": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.dim)), **f32),
-            "dgate": torch.zeros((rows, most(lambda L: L.gate_n)), **f32), "dbeta": torch.zeros((rows, most(lambda L: L.delta.heads)), **f32),
+            "dgate": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32), "dbeta": torch.zeros((rows, most(lambda L: L.delta.heads)), **f32),
             "dkq": torch.zeros((rows, most(lambda L: L.delta.kv_heads)), **f32),
-            "dout": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32), "ddt": torch.zeros((rows, most(lambda L: L.dt_n)), **f32),
+            "dout": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
             "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
             "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),
@@ -354,7 +353,7 @@ class MixedDecoder(SlotModel):
                              q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), qx=P(B["x_q"]), cbuf=P(B["x_c"]), krbuf=P(B["x_kr"]),
                              kx_hi=P(B["x_k"][0]), kx_lo=P(B["x_k"][1]), vx_hi=P(B["x_v"][0]), vx_lo=P(B["x_v"][1]), zero=P(B["x_zero"]), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
                              logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
-                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dkq", "dout", "ddt")})
+                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dkq", "dout")})
         h = lib.chatts_mixdec_create(C.byref(mc), arr, runs, C.byref(mb))
         if not h:
             raise _lib.ChattsError(-1, lib.chatts_last_error().decode())

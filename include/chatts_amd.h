@@ -812,15 +812,14 @@ typedef struct ChattsDeltaArgs {
   int n_rows;
   const ChattsSpan* spans;   /* device; chatts_delta_scan only */
   int n_spans;
-  /* scratch of the several-token form: q / k [T, kv_heads * dim], v / o [T, heads * vdim], g [T, heads * dim] (in: A2 a, out: decay),
-   * gate [T, heads * vdim] (G2 gin), beta [T, heads], kq [T, kv_heads] (k . q); row strides = the widths, except ld_dt / ld_gate */
+  /* scratch of the several-token form: q / k [T, kv_heads * dim], v / o [T, heads * vdim], g (decays) [T, heads * dim],
+   * gate [T, heads * vdim], beta [T, heads], kq (k . q) [T, kv_heads] */
   float *q, *k, *v, *g, *gate, *beta, *kq, *o;
-  const float* dt;
-  int ld_dt, ld_gate;
+  int exact;                 /* 32-bit runs: the low-rank products of the several-token form in true float32 */
   ChattsOperand out;
 } ChattsDeltaArgs;
 int chatts_delta_decode(const ChattsDeltaArgs* args, chatts_stream_t stream);   /* every row is a segment of one token: one launch */
-int chatts_delta_prep(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* several tokens: convolutions, norms, decays ... */
+int chatts_delta_prep(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* several tokens: convolutions, norms, decays, gates ... */
 int chatts_delta_scan(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* ... the recurrence over every span ... */
 int chatts_delta_out(const ChattsDeltaArgs* args, chatts_stream_t stream);      /* ... norm and gate of the read-outs, ring update */
 
@@ -882,7 +881,6 @@ typedef struct ChattsMixLayer {
   const chatts_bf16 *uk, *uv;                        /* latent: W_uk^T per head [heads, rank_p, dim_p], W_uv per head [heads, vdim_p, rank_p] */
   const chatts_bf16 *ukx, *uvx;                      /* latent, expanded form: [heads * dim_p, rank_p], [heads * vdim_p, rank_p]; NULL: never expanded */
   int dim_p, vdim_p, out_head;                       /* out_head: columns between heads in the input of `out` */
-  int dt_n, gate_n;                                  /* delta: rows of a2 / g2, padded to 16 */
   ChattsLatentArgs latent;                           /* sizes, offsets and weights; the rest is filled in per step */
   ChattsDeltaArgs delta;
 } ChattsMixLayer;
@@ -911,7 +909,7 @@ typedef struct ChattsMixBuffers {
   size_t partial_elems;
   chatts_bf16 *qx, *cbuf, *krbuf, *kx_hi, *kx_lo, *vx_hi, *vx_lo;   /* latent, expanded form (ChattsLatentExpandArgs) */
   const chatts_bf16* zero;
-  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dkq, *dout, *ddt;
+  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dkq, *dout;
   ChattsRow* rows;                                   /* device, [t_max] */
   ChattsSpan* spans;                                 /* device, [max_slots] */
   int32_t* table;                                    /* device, [max_slots, table_stride] */

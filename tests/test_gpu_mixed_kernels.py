@@ -129,9 +129,7 @@ class Delta:
         for n, t in self.conv.items():
             cw[:, self.off[n]:self.off[n] + t.shape[0]] = t.T
         pad = lambda t, c: torch.cat([t, torch.zeros(t.shape[0], c - t.shape[1], dtype=t.dtype)], 1)
-        self.dtn, self.gn = up(H * dim, 16), up(H * vd, 16)
-        rows = lambda t, n: torch.cat([t, torch.zeros(n - t.shape[0], t.shape[1], dtype=t.dtype)])
-        self.t = dict(cw=cw, a2=rows(pad(self.a2, self.rap), self.dtn), g2=rows(pad(self.g2, self.rgp), self.gn), dt=self.dt_bias, na=-torch.exp(self.a_log), nw=self.norm)
+        self.t = dict(cw=cw, a2=pad(self.a2, self.rap), g2=pad(self.g2, self.rgp), dt=self.dt_bias, na=-torch.exp(self.a_log), nw=self.norm)
         self.t = {k: v.contiguous().to(DEV) for k, v in self.t.items()}
         # used slots hold rubbish: a sequence that starts must not see it
         self.state = torch.randn(slots, H, dim, up(vd, 4), generator=g).to(DEV)
@@ -175,7 +173,7 @@ class Delta:
         return a
 
     def step(self, segs, forms):
-        """segs: list of (slot, pos0, x [t, ld]) -> list of [t, H * vd]; forms 'decode' (every t == 1) or 'scan'"""
+        """segs: list of (slot, pos0, x [t, ld]) -> list of [t, H * vd]; forms 'decode' (every t == 1), 'scan' or 'scan32'"""
         x = torch.cat([s[2] for s in segs]).to(DEV)
         rows, spans, at = [], [], 0
         for slot, pos0, xs in segs:
@@ -192,10 +190,9 @@ class Delta:
             H, KH, dim, vd = self.H, self.KH, self.dim, self.vd
             z = lambda n: torch.full((at, n), float("nan"), device=DEV)
             q, k, v, g, beta, kq, o = z(KH * dim), z(KH * dim), z(H * vd), z(H * dim), z(H), z(KH), z(H * vd)
-            dt = (x[:, self.off["a"]:self.off["a"] + self.rap] @ self.t["a2"].float().T).contiguous()
-            gate = (x[:, self.off["g"]:self.off["g"] + self.rgp] @ self.t["g2"].float().T).contiguous()
-            a.q, a.k, a.v, a.g, a.beta, a.kq, a.o = (t.data_ptr() for t in (q, k, v, g, beta, kq, o))
-            a.dt, a.gate, a.ld_dt, a.ld_gate = dt.data_ptr(), gate.data_ptr(), self.dtn, self.gn
+            gate = z(H * vd)
+            a.q, a.k, a.v, a.g, a.beta, a.kq, a.o, a.gate = (t.data_ptr() for t in (q, k, v, g, beta, kq, o, gate))
+            a.exact = int(forms == "scan32")
             for fn in ("chatts_delta_prep", "chatts_delta_scan", "chatts_delta_out"):
                 call(fn, a)
         res, at = [], 0
@@ -217,9 +214,10 @@ def test_delta_token_by_token_and_whole(shape):
     got = torch.cat([m.step([(1, t, x[t:t + 1])], "decode")[0] for t in range(T)])
     assert rel(got, want) < 2e-5
     assert rel(m.state[1, :, :, :m.vd], S) < 2e-5
-    got = m.step([(2, 0, x)], "scan")[0]
-    assert rel(got, want) < 2e-5
-    assert rel(m.state[2, :, :, :m.vd], S) < 2e-5
+    for form, tol in (("scan", 1e-4), ("scan32", 2e-5)):
+        got = m.step([(2, 0, x)], form)[0]
+        assert rel(got, want) < tol
+        assert rel(m.state[2, :, :, :m.vd], S) < tol
 
 
 @pytest.mark.parametrize("shape", SHAPES[:3])
@@ -244,7 +242,7 @@ def test_delta_portions_batches_and_reused_slots(shape):
             got[n_].append(r)
         at += c
     for n in got:
-        assert rel(torch.cat(got[n]), want[n]) < 2e-5, n
+        assert rel(torch.cat(got[n]), want[n]) < 1e-4, n
 
 
 def test_delta_parked_rows_touch_nothing():
