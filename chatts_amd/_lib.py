@@ -129,7 +129,7 @@ class DeltaArgs(C.Structure):
     """ChattsDeltaArgs: gated delta rule with a decay per head and key channel (csrc/delta.hip)"""
     _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_a", "off_g", "off_b", "conv_ch", "heads",
                                                              "kv_heads", "dim", "vdim", "taps", "rank_a", "rank_g")] +
-                [("conv_w", c_void_p), ("a2", c_void_p), ("g2", c_void_p), ("ld_a2", c_int), ("ld_g2", c_int), ("dt_bias", c_void_p),
+                [("conv_w", c_void_p), ("a2", c_void_p), ("g2", c_void_p), ("a2d", c_void_p), ("g2d", c_void_p), ("ld_a2", c_int), ("ld_g2", c_int), ("dt_bias", c_void_p),
                  ("neg_a", c_void_p), ("norm_w", c_void_p), ("eps", c_float), ("state", c_void_p), ("ring", c_void_p), ("rows", c_void_p),
                  ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int)] +
                 [(n, c_void_p) for n in ("q", "k", "v", "g", "gate", "beta", "kq", "o")] + [("exact", c_int), ("out", Operand)])

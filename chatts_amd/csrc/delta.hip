@@ -17,7 +17,9 @@ namespace chatts {
 
 // ---- one token per sequence -----------------------------------------------------------------------------------------------------
 // thread (tx, ty): 4 consecutive value columns tx * 4, key rows ty + TY * r.
-template <int NT, int NR>
+// Everything a workgroup reads is requested at once, the small inputs first (loads return in order) and the state last, so that the convolutions,
+// norms and gates are formed while the state is on its way.  No load is conditional: addresses are clamped and the values selected.
+template <int NT, int NR, int NU>      // NU: channels of q, k, v per thread
 __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int TX) {
   extern __shared__ float sm[];
   const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
@@ -40,61 +42,103 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
   float* S = p.state + ((size_t)slot * p.heads + h) * dim * v4;
   const int stride = TY * v4;
   float* Sp = S + (size_t)ty * v4 + tx * 4;
+  const float* pr = p.proj + (size_t)row * p.ld_proj;
+  float* ring = p.ring + (size_t)slot * p.taps * p.conv_ch;
+  const int total = 2 * dim + vdim;
+  auto channel = [&](int i) {
+    if (i < dim) return p.off_q + hk * dim + i;
+    if (i < 2 * dim) return p.off_k + hk * dim + i - dim;
+    return p.off_v + h * vdim + i - 2 * dim;
+  };
+  constexpr int kPast = 3;      // earlier tokens requested ahead; more taps take the loop below
+  float cur[NU], past[NU][kPast], cw[NU][kPast + 1];
+#pragma unroll
+  for (int u = 0; u < NU; ++u) {
+    const int i = u * NT + tid, ch = channel(i < total ? i : total - 1);
+    cur[u] = pr[ch];
+    cw[u][0] = p.conv_w[(size_t)(p.taps - 1) * p.conv_ch + ch];
+#pragma unroll
+    for (int g = 1; g <= kPast; ++g) {
+      const bool ok = g < p.taps && pos >= g;
+      past[u][g - 1] = ring[(size_t)((ok ? pos - g : pos) % p.taps) * p.conv_ch + ch];
+      cw[u][g] = p.conv_w[(size_t)(g < p.taps ? p.taps - 1 - g : 0) * p.conv_ch + ch];
+      if (!ok) cw[u][g] = 0.f;
+    }
+  }
+  const float beta_in = pr[p.off_b + h], na = p.neg_a[h];
+  constexpr int kW = 8;      // 8-value pieces of this thread's low-rank row requested ahead
+  const bool dec = tid < dim;
+  const int lr = tid < dim + vdim ? tid : dim + vdim - 1, lrow = dec ? h * dim + tid : h * vdim + (lr - dim < 0 ? 0 : lr - dim);
+  const int lrank = (dec ? p.rank_a : p.rank_g) >> 3, lrows = dec ? p.heads * dim : p.heads * vdim;
+  const uint16_t* lw = (dec ? p.a2d : p.g2d) + (size_t)lrow * 8;
+  u32x4 wv[kW];
+#pragma unroll
+  for (int c = 0; c < kW; ++c) wv[c] = *reinterpret_cast<const u32x4*>(lw + (size_t)(c < lrank ? c : 0) * lrows * 8);
+  const float lbias = dec ? p.dt_bias[lrow] : 0.f;
+  const float a_in = pr[p.off_a + (tid < p.rank_a ? tid : 0)], g_in = pr[p.off_g + (tid < p.rank_g ? tid : 0)];
   f32x4 s[NR];
 #pragma unroll
   for (int r = 0; r < NR; ++r) {
-    s[r] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    if (pos > 0 && live && ty + TY * r < dim) s[r] = *reinterpret_cast<const f32x4*>(Sp + (size_t)r * stride);
+    const int i = ty + TY * r < dim ? ty + TY * r : dim - 1;
+    s[r] = *reinterpret_cast<const f32x4*>(S + (size_t)i * v4 + (live ? tx * 4 : 0));
   }
-  const float* pr = p.proj + (size_t)row * p.ld_proj;
-  float* ring = p.ring + (size_t)slot * p.taps * p.conv_ch;
-  for (int i = tid; i < 2 * dim + vdim; i += NT) {
-    int ch;
-    bool owner = true;
-    if (i < dim) { ch = p.off_q + hk * dim + i; owner = h == hk * group; }
-    else if (i < 2 * dim) { ch = p.off_k + hk * dim + i - dim; owner = h == hk * group; }
-    else ch = p.off_v + h * vdim + i - 2 * dim;
-    const float cur = pr[ch];
+#pragma unroll
+  for (int u = 0; u < NU; ++u) {
+    const int i = u * NT + tid;
+    if (i >= total) continue;
+    const int ch = channel(i);
     float acc = 0.f;
-    for (int j = 0; j < p.taps - 1; ++j) {
-      const int q = pos - (p.taps - 1 - j);
-      if (q >= 0) acc += p.conv_w[(size_t)j * p.conv_ch + ch] * ring[(size_t)(q % p.taps) * p.conv_ch + ch];
-    }
-    acc += p.conv_w[(size_t)(p.taps - 1) * p.conv_ch + ch] * cur;
-    if (owner) ring[(size_t)(pos % p.taps) * p.conv_ch + ch] = cur;
+    for (int g = p.taps - 1; g > kPast; --g)
+      if (pos >= g) acc += p.conv_w[(size_t)(p.taps - 1 - g) * p.conv_ch + ch] * ring[(size_t)((pos - g) % p.taps) * p.conv_ch + ch];
+#pragma unroll
+    for (int g = kPast; g >= 1; --g)
+      if (cw[u][g] != 0.f) acc += cw[u][g] * past[u][g - 1];      // (an unused entry may hold anything)
+    acc += cw[u][0] * cur[u];
+    if (i >= 2 * dim || h == hk * group) ring[(size_t)(pos % p.taps) * p.conv_ch + ch] = cur[u];      // q / k: the first head of the group
     acc *= sigmoid_f(acc);
     if (i < dim) sq[i] = acc;
     else if (i < 2 * dim) sk[i - dim] = acc;
     else sv[i - 2 * dim] = acc;
   }
-  for (int i = tid; i < p.rank_a; i += NT) sa[i] = pr[p.off_a + i];
-  for (int i = tid; i < p.rank_g; i += NT) sgi[i] = pr[p.off_g + i];
+  if (tid < p.rank_a) sa[tid] = a_in;
+  if (tid < p.rank_g) sgi[tid] = g_in;
+  for (int i = tid + NT; i < p.rank_a; i += NT) sa[i] = pr[p.off_a + i];
+  for (int i = tid + NT; i < p.rank_g; i += NT) sgi[i] = pr[p.off_g + i];
   __syncthreads();
   float qs = 0.f, ks = 0.f;      // every wave forms both norms
   for (int i = tid & 63; i < dim; i += 64) { qs += sq[i] * sq[i]; ks += sk[i] * sk[i]; }
   qs = wave_sum(qs);
   ks = wave_sum(ks);
   const float qn = rsqrtf((float)dim) / sqrtf(qs + 1e-6f), kn = 1.0f / sqrtf(ks + 1e-6f);
-  const float na = p.neg_a[h];
-  for (int i = tid; i < dim + vdim; i += NT) {
-    const bool dec = i < dim;
-    const int o = dec ? h * dim + i : h * vdim + i - dim;
-    const uint16_t* w = dec ? p.a2 + (size_t)o * p.ld_a2 : p.g2 + (size_t)o * p.ld_g2;
-    const float* x = dec ? sa : sgi;
-    const int rank = dec ? p.rank_a : p.rank_g;
-    float acc = 0.f;
-    for (int c = 0; c < rank; c += 8) {
-      const u32x4 wv = *reinterpret_cast<const u32x4*>(w + c);
+  auto dot8 = [](const u32x4& w, const float* x, float acc) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        acc += bf16_lo(wv[j]) * x[c + 2 * j];
-        acc += bf16_hi(wv[j]) * x[c + 2 * j + 1];
-      }
+    for (int j = 0; j < 4; ++j) {
+      acc += bf16_lo(w[j]) * x[2 * j];
+      acc += bf16_hi(w[j]) * x[2 * j + 1];
     }
-    if (dec) sg[i] = exp_hw(na * softplus_f(acc + p.dt_bias[o]));
+    return acc;
+  };
+  for (int i = tid; i < dim + vdim; i += NT) {
+    const bool de = i < dim;
+    const int o = de ? h * dim + i : h * vdim + i - dim, rank8 = (de ? p.rank_a : p.rank_g) >> 3, rows = de ? p.heads * dim : p.heads * vdim;
+    const uint16_t* w = (de ? p.a2d : p.g2d) + (size_t)o * 8;
+    const float* x = de ? sa : sgi;
+    float acc = 0.f;
+    int c = 0;
+    if (i == tid) {
+#pragma unroll
+      for (int e = 0; e < kW; ++e)
+        if (e < rank8) acc = dot8(wv[e], x + e * 8, acc);
+      c = kW;
+    }
+    for (; c < rank8; ++c) acc = dot8(*reinterpret_cast<const u32x4*>(w + (size_t)c * rows * 8), x + c * 8, acc);
+    if (de) sg[i] = exp_hw(na * softplus_f(acc + (i == tid ? lbias : p.dt_bias[o])));
     else sgate[i - dim] = sigmoid_f(acc);
   }
-  const float beta = sigmoid_f(pr[p.off_b + h]);
+#pragma unroll
+  for (int r = 0; r < NR; ++r)
+    if (!(pos > 0 && live && ty + TY * r < dim)) s[r] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const float beta = sigmoid_f(beta_in);
   __syncthreads();
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -531,7 +575,7 @@ using namespace chatts;
 
 extern "C" int chatts_delta_decode(const ChattsDeltaArgs* a, chatts_stream_t stream) {
   if (const int rc = check_delta(a, "delta_decode")) return rc;
-  CHATTS_REQUIRE(a->a2 && a->g2 && (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim, CHATTS_E_BADARG, "delta_decode: null pointer");
+  CHATTS_REQUIRE(a->a2d && a->g2d && (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim, CHATTS_E_BADARG, "delta_decode: null pointer");
   if (a->n_rows == 0) return CHATTS_OK;
   const int v4 = (a->vdim + 3) & ~3;
   int TX = 1;
@@ -542,11 +586,19 @@ extern "C" int chatts_delta_decode(const ChattsDeltaArgs* a, chatts_stream_t str
   CHATTS_REQUIRE(lds <= 64 * 1024, CHATTS_E_SHAPE, "delta_decode: ranks %d / %d too large", a->rank_a, a->rank_g);
   const dim3 g(a->heads, a->n_rows);
   hipStream_t s = as_stream(stream);
-  if (nt == 512) hipLaunchKernelGGL((delta_decode_kernel<512, 32>), g, dim3(512), lds, s, *a, TX);
-  else if (nr <= 4) hipLaunchKernelGGL((delta_decode_kernel<256, 4>), g, dim3(256), lds, s, *a, TX);
-  else if (nr <= 8) hipLaunchKernelGGL((delta_decode_kernel<256, 8>), g, dim3(256), lds, s, *a, TX);
-  else if (nr <= 16) hipLaunchKernelGGL((delta_decode_kernel<256, 16>), g, dim3(256), lds, s, *a, TX);
-  else hipLaunchKernelGGL((delta_decode_kernel<256, 32>), g, dim3(256), lds, s, *a, TX);
+  const int nu = (2 * a->dim + a->vdim + nt - 1) / nt;
+#define CHATTS_DELTA_DECODE(NT, NR)                                                                                   \
+  do {                                                                                                                 \
+    if (nu <= 1) hipLaunchKernelGGL((delta_decode_kernel<NT, NR, 1>), g, dim3(NT), lds, s, *a, TX);                    \
+    else if (nu == 2) hipLaunchKernelGGL((delta_decode_kernel<NT, NR, 2>), g, dim3(NT), lds, s, *a, TX);               \
+    else hipLaunchKernelGGL((delta_decode_kernel<NT, NR, 3>), g, dim3(NT), lds, s, *a, TX);                            \
+  } while (0)
+  if (nt == 512) CHATTS_DELTA_DECODE(512, 32);
+  else if (nr <= 4) CHATTS_DELTA_DECODE(256, 4);
+  else if (nr <= 8) CHATTS_DELTA_DECODE(256, 8);
+  else if (nr <= 16) CHATTS_DELTA_DECODE(256, 16);
+  else CHATTS_DELTA_DECODE(256, 32);
+#undef CHATTS_DELTA_DECODE
   CHATTS_CHECK_LAUNCH("delta_decode");
   return CHATTS_OK;
 }

@@ -206,6 +206,11 @@ class MixedDecoder(SlotModel):
             pt = self._dev(out)
         return p, pt
 
+    def _pieces(self, t, cols):
+        """[rows, rank] -> [rank / 8, rows, 8]: what neighbouring threads read of neighbouring rows lies side by side"""
+        t = _pad(t.to(torch.bfloat16), t.shape[0], cols)
+        return self._dev(t.view(t.shape[0], cols // 8, 8).transpose(0, 1).contiguous())
+
     def _stack(self, blocks):
         """stacked input projection: (name, [rows, width], padded rows) -> (matrix, {name: first row})"""
         off, at = {}, 0
@@ -259,7 +264,8 @@ class MixedDecoder(SlotModel):
             conv[:, off[n]:off[n] + t.shape[0]] = t.to(torch.float32).t()
         L.delta = _lib.DeltaArgs(off_q=off["q"], off_k=off["k"], off_v=off["v"], off_a=off["a"], off_g=off["g"], off_b=off["b"], conv_ch=off["a"],
                                  heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, taps=m.taps, rank_a=ra_p, rank_g=rg_p,
-                                 conv_w=self._dev(conv), a2=self._mat(m.a2, None, ra_p)[0], g2=self._mat(m.g2, None, rg_p)[0], ld_a2=ra_p, ld_g2=rg_p,
+                                 conv_w=self._dev(conv), a2=self._mat(m.a2, None, ra_p)[0], g2=self._mat(m.g2, None, rg_p)[0],
+                                 a2d=self._pieces(m.a2, ra_p), g2d=self._pieces(m.g2, rg_p), ld_a2=ra_p, ld_g2=rg_p,
                                  dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32))), norm_w=self._f32(m.norm))
 
     def _build(self, sd):

@@ -801,6 +801,7 @@ typedef struct ChattsDeltaArgs {
   const float* conv_w;       /* [taps, conv_ch] */
   const chatts_bf16* a2;     /* [heads * dim, ld_a2] */
   const chatts_bf16* g2;     /* [heads * vdim, ld_g2] */
+  const chatts_bf16 *a2d, *g2d;   /* chatts_delta_decode: the same, as [rank / 8, rows, 8] (neighbouring rows side by side) */
   int ld_a2, ld_g2;
   const float* dt_bias;      /* [heads * dim] */
   const float* neg_a;        /* [heads] = -exp(A_log) */

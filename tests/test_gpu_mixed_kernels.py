@@ -130,6 +130,8 @@ class Delta:
             cw[:, self.off[n]:self.off[n] + t.shape[0]] = t.T
         pad = lambda t, c: torch.cat([t, torch.zeros(t.shape[0], c - t.shape[1], dtype=t.dtype)], 1)
         self.t = dict(cw=cw, a2=pad(self.a2, self.rap), g2=pad(self.g2, self.rgp), dt=self.dt_bias, na=-torch.exp(self.a_log), nw=self.norm)
+        for n in ("a2", "g2"):
+            self.t[n + "d"] = self.t[n].view(self.t[n].shape[0], -1, 8).transpose(0, 1)
         self.t = {k: v.contiguous().to(DEV) for k, v in self.t.items()}
         # used slots hold rubbish: a sequence that starts must not see it
         self.state = torch.randn(slots, H, dim, up(vd, 4), generator=g).to(DEV)
@@ -165,7 +167,7 @@ class Delta:
         t, T = self.t, x.shape[0]
         a = _lib.DeltaArgs(proj=x.data_ptr(), ld_proj=self.ld, off_q=self.off["q"], off_k=self.off["k"], off_v=self.off["v"], off_a=self.off["a"], off_g=self.off["g"],
                            off_b=self.off["b"], conv_ch=self.conv_ch, heads=self.H, kv_heads=self.KH, dim=self.dim, vdim=self.vd, taps=self.taps, rank_a=self.rap,
-                           rank_g=self.rgp, conv_w=t["cw"].data_ptr(), a2=t["a2"].data_ptr(), g2=t["g2"].data_ptr(), ld_a2=self.rap, ld_g2=self.rgp,
+                           rank_g=self.rgp, conv_w=t["cw"].data_ptr(), a2=t["a2"].data_ptr(), g2=t["g2"].data_ptr(), a2d=t["a2d"].data_ptr(), g2d=t["g2d"].data_ptr(), ld_a2=self.rap, ld_g2=self.rgp,
                            dt_bias=t["dt"].data_ptr(), neg_a=t["na"].data_ptr(), norm_w=t["nw"].data_ptr(), eps=self.eps, state=self.state.data_ptr(),
                            ring=self.ring.data_ptr(), rows=rows.data_ptr(), n_rows=T, out=operand(out, None, self.H * self.vd))
         if spans is not None:
