@@ -132,7 +132,7 @@ class DeltaArgs(C.Structure):
                 [("conv_w", c_void_p), ("a2", c_void_p), ("g2", c_void_p), ("a2d", c_void_p), ("g2d", c_void_p), ("ld_a2", c_int), ("ld_g2", c_int), ("dt_bias", c_void_p),
                  ("neg_a", c_void_p), ("norm_w", c_void_p), ("eps", c_float), ("state", c_void_p), ("ring", c_void_p), ("rows", c_void_p),
                  ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int)] +
-                [(n, c_void_p) for n in ("q", "k", "v", "g", "gate", "beta", "kq", "o")] + [("exact", c_int), ("out", Operand)])
+                [(n, c_void_p) for n in ("q", "k", "v", "g", "gate", "beta", "chunks", "o")] + [("exact", c_int), ("out", Operand)])
 
 
 class LatentArgs(C.Structure):
@@ -179,7 +179,7 @@ class MixBuffers(C.Structure):
     _fields_ = ([(n, c_void_p) for n in ("embed", "head", "head_t", "final_norm", "x", "y", "proj", "a_f32", "b_f32", "a_hi", "a_lo", "b_hi", "b_lo",
                                          "q_f32", "o_lat", "partial", "q_hi", "q_lo")] + [("partial_elems", c_size_t)] +
                 [(n, c_void_p) for n in ("qx", "cbuf", "krbuf", "kx_hi", "kx_lo", "vx_hi", "vx_lo", "zero")] +
-                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dkq", "dout", "rows", "spans", "table", "logits", "workspace")] +
+                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout", "rows", "spans", "table", "logits", "workspace")] +
                 [("workspace_bytes", c_size_t)])
 
 
@@ -269,6 +269,7 @@ SIGNATURES = {
     "chatts_delta_decode": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
     "chatts_delta_prep": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
     "chatts_delta_scan": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
+    "chatts_delta_chunk_floats": (C.c_int64, [c_int, c_int, c_int, c_int]),
     "chatts_delta_out": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
     "chatts_latent_prep": (c_int, [C.POINTER(LatentArgs), c_void_p]),
     "chatts_latent_attend": (c_int, [C.POINTER(LatentArgs), c_void_p]),

@@ -193,12 +193,6 @@ __device__ __forceinline__ float softplus_f(float x) {
   const float z = e * __builtin_amdgcn_rcpf(2.0f + e), z2 = z * z;
   return 2.0f * z * (1.0f + z2 * (1.0f / 3 + z2 * (1.0f / 5 + z2 * (1.0f / 7 + z2 * (1.0f / 9 + z2 * (1.0f / 11))))));
 }
-// lane N of each row of 16, to the whole row
-template <int N>
-__device__ __forceinline__ float row_bcast(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x150 + N, 0xF, 0xF, true));      // (every lane is valid: folds into the user)
-}
-
 inline hipStream_t as_stream(chatts_stream_t s) { return reinterpret_cast<hipStream_t>(s); }
 
 // ---- stage ranges for traces (api.hip): roctx push / pop around the host-side enqueue of a stage, resolved with dlopen at first use

@@ -4,13 +4,10 @@
 //  * delta_decode_kernel: one token per sequence, everything of a (sequence, head) in one workgroup: convolutions from the ring of
 //    earlier inputs, unit norms, the low-rank decay and gate products, the state update (state in registers between its two passes) and the
 //    normed, gated read-out.  One launch instead of five, the state is read and written once.
-//  * delta_lowrank_kernel, delta_prep_*_kernel / delta_scan_kernel / delta_out_kernel: several tokens per sequence.  The first do what is parallel over tokens; scan
-//    walks the tokens with the state in registers - a column of S belongs to 16 lanes of a wave, so the two sums over key channels are
-//    DPP row reductions and columns never talk to each other; out norms and gates.
+//  * delta_lowrank_kernel, delta_prep_*_kernel, delta_chunk_kernel / delta_scan_kernel / delta_out_kernel: several tokens per sequence.  The first do
+//    what is parallel over tokens or chunks of 16 tokens; scan passes the state from chunk to chunk on the float32 matrix pipe; out norms and gates.
 // The ring of convolution inputs is indexed by position modulo taps: the current token's entry is never one that the same step reads, so
 // heads that share a q / k head need no ordering, and a sequence that starts over in a used slot reads none of the old entries.
-#include <type_traits>
-
 #include "common.h"
 
 namespace chatts {
@@ -245,9 +242,9 @@ __global__ __launch_bounds__(256) void delta_prep_qk_kernel(ChattsDeltaArgs p) {
   ChattsRow R[kQkRows];
   bool live[kQkRows];
   prep_rows(p, row0, R, live);
-  float q[NCH][kQkRows], k[NCH][kQkRows], qs[kQkRows], ks[kQkRows], qk[kQkRows];
+  float q[NCH][kQkRows], k[NCH][kQkRows], qs[kQkRows], ks[kQkRows];
 #pragma unroll
-  for (int i = 0; i < kQkRows; ++i) qs[i] = ks[i] = qk[i] = 0.f;
+  for (int i = 0; i < kQkRows; ++i) qs[i] = ks[i] = 0.f;
 #pragma unroll
   for (int c = 0; c < NCH; ++c) {
     const int ch = c * 64 + lane;
@@ -259,13 +256,12 @@ __global__ __launch_bounds__(256) void delta_prep_qk_kernel(ChattsDeltaArgs p) {
       if (!ok) q[c][i] = k[c][i] = 0.f;
       qs[i] += q[c][i] * q[c][i];
       ks[i] += k[c][i] * k[c][i];
-      qk[i] += q[c][i] * k[c][i];
     }
   }
   const float qscale = rsqrtf((float)dim);
 #pragma unroll
   for (int i = 0; i < kQkRows; ++i) {
-    const float fq = qscale / sqrtf(wave_sum(qs[i]) + 1e-6f), fk = 1.0f / sqrtf(wave_sum(ks[i]) + 1e-6f), d = wave_sum(qk[i]);
+    const float fq = qscale / sqrtf(wave_sum(qs[i]) + 1e-6f), fk = 1.0f / sqrtf(wave_sum(ks[i]) + 1e-6f);
     if (!live[i]) continue;
     const size_t at = (size_t)(row0 + i) * p.kv_heads + e;
 #pragma unroll
@@ -276,7 +272,6 @@ __global__ __launch_bounds__(256) void delta_prep_qk_kernel(ChattsDeltaArgs p) {
         p.k[at * dim + ch] = k[c][i] * fk;
       }
     }
-    if (lane == 0) p.kq[at] = d * fq * fk;
   }
 }
 
@@ -389,143 +384,243 @@ static void launch_prep(const ChattsDeltaArgs* a, hipStream_t s) {
   hipLaunchKernelGGL(delta_prep_v_kernel<TAPS>, dim3((a->n_rows + kVRows - 1) / kVRows, (items + 3) / 4), b, 0, s, *a);
 }
 
-// ---- the recurrence over a span: grid (heads * column blocks, spans), 4 waves x 4 columns ---------------------------------------------
-// Lane l of a row of 16 holds key channels (c * 16 + l) * 4 .. + 3 (c < NC) of its column.  Both sums over key channels are taken on the
-// decayed state before the update, S^T k for u and S^T q for the read-out (o = S^T q + (k . q) u with the k . q of prep): their reductions
-// are independent of each other and only the first is on the token-to-token path.  Tokens are staged in LDS kT at a time and walked
-// fully unrolled, the next token's operands requested while the current one is computed; beta, k . q and v of the kT tokens sit in the
-// lanes of a row and are broadcast from there.  Rows past the end of the span are staged as k = q = 0, g = 1, beta = 0: they change nothing.
-template <int T, int N, typename F>
-__device__ __forceinline__ void unroll_tokens(F&& f) {
-  if constexpr (T < N) {
-    f(std::integral_constant<int, T>{});
-    unroll_tokens<T + 1, N>(f);
+// ---- the recurrence over a span, 16 tokens (a chunk) at a time -----------------------------------------------------------------------
+// Within a chunk that starts from state S, with G_t = g_0 .. g_t (products per key channel, g of the chunk's tokens) and D(s, t) = g_{s+1} .. g_t:
+//   u_t = beta_t (v_t - S^T (G_t k_t) - sum_{s < t} A_ts u_s),   A_ts = k_t . (D(s, t) k_s)
+//   o_t = S^T (G_t q_t) + sum_{s <= t} P_ts u_s,                 P_ts = q_t . (D(s, t) k_s)
+//   S  <- G_15 S + sum_s (D(s, 15) k_s) u_s^T
+// Every decay product runs forward in time (factors <= 1, nothing is divided: strong decays vanish instead of overflowing).  With
+// T = (I + diag(beta) A)^-1 diag(beta) the first line is u = T (v - S^T (G k)).  All of G k, G q, D(., 15) k, T, P and G_15 depend on the
+// inputs only: delta_chunk_kernel forms them for all chunks in parallel; delta_scan_kernel is left with small products that pass the state
+// along, on the float32 matrix pipe.  Rows past the end of a span count as k = q = 0, g = 1, beta = 0: they change nothing.
+//
+// A (chunk, head) holds, in floats, D = 64 NC channels:  G k [D / 16][64][4] | G q, the same | D(., 15) k [D / 16][64][4] | T [64][4] | P [64][4] | G_15 [D],
+// each in the order in which the 64 lanes of a wave read matrix fragments.  Chunk c of span i is number row0 / 16 + i + c.
+constexpr int kChunk = CHATTS_DELTA_CHUNK;
+static_assert(kChunk == 16, "a chunk is a matrix fragment");
+__host__ __device__ constexpr int chunk_floats(int nc) { return 64 * nc * (3 * kChunk + 1) + 512; }
+
+template <int NC>
+__global__ __launch_bounds__(256) void delta_chunk_kernel(ChattsDeltaArgs p) {
+  constexpr int D = NC * 64, D4 = D / 4;
+  __shared__ __attribute__((aligned(16))) float sk[kChunk][D], sq[kChunk][D], sg[kChunk][D];
+  __shared__ float sa[kChunk][kChunk + 1], sb[kChunk];
+  const int h = blockIdx.x, chunk = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  int row = -1, n = 0;      // first row and rows of this chunk
+  for (int i = 0; i < p.n_spans; ++i) {
+    const int r0 = p.spans[i].row0, t = p.spans[i].t, c = chunk - (r0 / kChunk + i);
+    if (c >= 0 && c * kChunk < t) { row = r0 + c * kChunk; n = t - c * kChunk; }
+  }
+  if (row < 0) return;
+  if (n > kChunk) n = kChunk;
+  const int dim = p.dim, hk = h / (p.heads / p.kv_heads), qrow = p.kv_heads * dim, grow = p.heads * dim;
+  float* out = p.chunks + ((size_t)chunk * p.heads + h) * chunk_floats(NC);
+#pragma unroll
+  for (int e = 0; e < kChunk * D / 256; ++e) {
+    const int j = e * 256 + tid, t = j / D, c = j % D;
+    const bool ok = t < n && c < dim;
+    const size_t r = row + (t < n ? t : 0);
+    const int cc = c < dim ? c : 0;
+    const float k = p.k[r * qrow + hk * dim + cc], q = p.q[r * qrow + hk * dim + cc], g = p.g[r * grow + h * dim + cc];
+    sk[t][c] = ok ? k : 0.f;
+    sq[t][c] = ok ? q : 0.f;
+    sg[t][c] = ok ? g : 1.f;
+  }
+  if (tid < kChunk) sb[tid] = tid < n ? p.beta[(size_t)(row + tid) * p.heads + h] : 0.f;
+  __syncthreads();
+  {
+    // A, P: thread = (token s, 1 / 16 of the channels), w = D(s, t) k_s walks forward in t
+    const int s = tid >> 4, l16 = tid & 15;
+    f32x4 w[NC];
+#pragma unroll
+    for (int c = 0; c < NC; ++c) w[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    float ka = 0.f, kp = 0.f;      // of token t = l16
+#pragma unroll 4
+    for (int t = 0; t < kChunk; ++t) {
+      float a = 0.f, b = 0.f;
+#pragma unroll
+      for (int c = 0; c < NC; ++c) {
+        const f32x4 g = *reinterpret_cast<const f32x4*>(&sg[t][c * 64 + l16 * 4]), k = *reinterpret_cast<const f32x4*>(&sk[t][c * 64 + l16 * 4]),
+                    q = *reinterpret_cast<const f32x4*>(&sq[t][c * 64 + l16 * 4]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          w[c][j] = t == s ? k[j] : w[c][j] * g[j];
+          a += k[j] * w[c][j];
+          b += q[j] * w[c][j];
+        }
+      }
+      a = row16_sum(a);
+      b = row16_sum(b);
+      ka = l16 == t ? a : ka;
+      kp = l16 == t ? b : kp;
+    }
+    sa[l16][s] = l16 > s ? ka : 0.f;
+    out[(3 * kChunk) * D + 256 + ((s >> 2) * 16 + l16) * 4 + (s & 3)] = l16 >= s ? kp : 0.f;      // P[t = l16][s]
+  }
+  // G k, G q and D(., 15) k of (token, 4 channels)
+  constexpr int PER = D4 * kChunk / 256;
+  f32x4 kt[PER];
+#pragma unroll
+  for (int e = 0; e < PER; ++e) {
+    const int ct = e * 4 + wave, t = lane & 15, c = ct * 16 + (lane >> 4) * 4;
+    f32x4 f = {1.f, 1.f, 1.f, 1.f}, b = {1.f, 1.f, 1.f, 1.f};
+#pragma unroll
+    for (int r = 0; r < kChunk; ++r) {
+      const f32x4 g = *reinterpret_cast<const f32x4*>(&sg[r][c]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        f[j] *= r <= t ? g[j] : 1.f;
+        b[j] *= r > t ? g[j] : 1.f;
+      }
+    }
+    const f32x4 k = *reinterpret_cast<const f32x4*>(&sk[t][c]), q = *reinterpret_cast<const f32x4*>(&sq[t][c]);
+    f32x4 gk, gq;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) { gk[j] = f[j] * k[j]; gq[j] = f[j] * q[j]; kt[e][j] = b[j] * k[j]; }
+    *reinterpret_cast<f32x4*>(out + ct * 256 + lane * 4) = gk;
+    *reinterpret_cast<f32x4*>(out + kChunk * D + ct * 256 + lane * 4) = gq;
+    if (t == kChunk - 1) *reinterpret_cast<f32x4*>(out + 3 * kChunk * D + 512 + c) = f;
+  }
+  __syncthreads();      // (sg is free, sa complete)
+#pragma unroll
+  for (int e = 0; e < PER; ++e)
+    *reinterpret_cast<f32x4*>(&sg[lane & 15][(e * 4 + wave) * 16 + (lane >> 4) * 4]) = kt[e];
+  if (tid < kChunk) {      // column tid of T, by forward substitution
+    float x[kChunk];
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) {
+      float v = t == tid ? 1.f : 0.f;
+#pragma unroll
+      for (int s = 0; s < t; ++s) v -= sa[t][s] * x[s];
+      x[t] = sb[t] * v;
+      out[(3 * kChunk) * D + ((tid >> 2) * 16 + t) * 4 + (tid & 3)] = x[t];
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int e = 0; e < PER; ++e) {      // transposed: lane = (4 tokens lane >> 4, channel lane & 15)
+    const int ct = e * 4 + wave;
+    f32x4 v;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = sg[(lane >> 4) * 4 + j][ct * 16 + (lane & 15)];
+    *reinterpret_cast<f32x4*>(out + 2 * kChunk * D + ct * 256 + lane * 4) = v;
   }
 }
+
+// grid (heads * column blocks of 16, spans), 4 waves: a wave holds NC tiles (16 channels x 16 columns) of the state as accumulators of the matrix
+// pipe, which are also the right-hand operands of S^T (G k) and S^T (G q) - K slot g of product r means channel 4 g + r of a tile, token 4 g + r in
+// the others, on both sides, so nothing is shuffled.  The waves' sums over channels meet in LDS once per chunk; u is formed by every wave.
 template <int NC>
-__global__ __launch_bounds__(256) void delta_scan_kernel(ChattsDeltaArgs p) {
-  constexpr int D = NC * 64, kT = NC <= 2 ? 16 : 8;
-  __shared__ __attribute__((aligned(16))) float sk[2][kT][D], sq[2][kT][D], sg[2][kT][D];
-  __shared__ float so[kT][17];
+__global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(ChattsDeltaArgs p) {
+  constexpr int D = NC * 64;
+  __shared__ f32x4 sd[2][4][64], so[2][4][64];
   const ChattsSpan sp = p.spans[blockIdx.y];
   if (sp.t < 1) return;
-  // (consecutive workgroups take consecutive heads: the column blocks of a head run on one XCD where heads % 8 == 0, its k / q / g in that L2)
-  const int cb = blockIdx.x / p.heads, h = blockIdx.x - cb * p.heads, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int dim = p.dim, vdim = p.vdim, v4 = (vdim + 3) & ~3, hk = h / (p.heads / p.kv_heads);
-  const int l16 = lane & 15, cl = wave * 4 + (lane >> 4), col = cb * 16 + cl;
+  // (consecutive workgroups take consecutive heads: the column blocks of a head run on one XCD where heads % 8 == 0, its operands in that L2)
+  const int cb = blockIdx.x / p.heads, h = blockIdx.x - cb * p.heads, tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int dim = p.dim, vdim = p.vdim, v4 = (vdim + 3) & ~3, fr = lane & 15, fg = lane >> 4, col = cb * 16 + fr;
   const bool live = col < vdim;
   float* S = p.state + ((size_t)sp.slot * p.heads + h) * dim * v4;
   f32x4 s[NC];
 #pragma unroll
   for (int c = 0; c < NC; ++c)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int i = (c * 16 + l16) * 4 + j;
-      s[c][j] = sp.pos0 > 0 && live && i < dim ? S[(size_t)i * v4 + col] : 0.f;
+    for (int r = 0; r < 4; ++r) {
+      const int i = (wave * NC + c) * 16 + fg * 4 + r;
+      s[c][r] = sp.pos0 > 0 && live && i < dim ? S[(size_t)i * v4 + col] : 0.f;
     }
-  const int qrow = p.kv_heads * dim, grow = p.heads * dim, vrow = p.heads * vdim;
-  constexpr int PER = kT * D / 256, TS = 256 / D;      // values of one of k / q / g per thread and stage, tokens between them
-  const int fi = tid % D, ft = tid / D;
-  const bool fok = fi < dim;
-  const float* gk = p.k + (size_t)sp.row0 * qrow + hk * dim + (fok ? fi : 0);
-  const float* gq = p.q + (size_t)sp.row0 * qrow + hk * dim + (fok ? fi : 0);
-  const float* gg = p.g + (size_t)sp.row0 * grow + h * dim + (fok ? fi : 0);
+  const int vrow = p.heads * vdim, nch = (sp.t + kChunk - 1) / kChunk;
+  const float* ops = p.chunks + ((size_t)(sp.row0 / kChunk + blockIdx.y) * p.heads + h) * chunk_floats(NC) + lane * 4;
+  const size_t step = (size_t)p.heads * chunk_floats(NC);
   const float* gv = p.v + (size_t)sp.row0 * vrow + h * vdim + (live ? col : 0);
-  const float* gb = p.beta + (size_t)sp.row0 * p.heads + h;
-  const float* gc = p.kq + (size_t)sp.row0 * p.kv_heads + hk;
-  float rk[PER], rq[PER], rg[PER], nv, nb, nc;      // the next stage; v, beta, k . q of token l16
-  auto fetch = [&](int t0) {
+  float* go = p.o + (size_t)sp.row0 * vrow + h * vdim + col;
+  struct Ops { f32x4 k[NC], q[NC], kt[NC], g[NC], t, v; float pw; };
+  auto fetch = [&](int c, Ops& o) __attribute__((always_inline)) {
+    if (c > nch - 1) c = nch - 1;
+    const float* b = ops + (size_t)c * step;
 #pragma unroll
-    for (int e = 0; e < PER; ++e) {
-      int t = t0 + ft + e * TS;
-      const bool ok = fok && t < sp.t;
+    for (int i = 0; i < NC; ++i) o.k[i] = *reinterpret_cast<const f32x4*>(b + (wave * NC + i) * 256);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      int t = c * kChunk + fg * 4 + r;
       if (t > sp.t - 1) t = sp.t - 1;
-      rk[e] = gk[(size_t)t * qrow];
-      rq[e] = gq[(size_t)t * qrow];
-      rg[e] = gg[(size_t)t * grow];
-      if (!ok) { rk[e] = rq[e] = 0.f; rg[e] = 1.f; }
+      o.v[r] = gv[(size_t)t * vrow];
     }
-    int t = t0 + (l16 & (kT - 1));
-    const bool ok = t < sp.t;
-    if (!ok) t = sp.t - 1;
-    nv = gv[(size_t)t * vrow];
-    nb = gb[(size_t)t * p.heads];
-    nc = gc[(size_t)t * p.kv_heads];
-    if (!ok) nb = 0.f;
-  };
-  auto stage = [&](int b) {
+    o.t = *reinterpret_cast<const f32x4*>(b + 3 * kChunk * D);
 #pragma unroll
-    for (int e = 0; e < PER; ++e) {
-      const int t = ft + e * TS;
-      sk[b][t][fi] = rk[e];
-      sq[b][t][fi] = rq[e];
-      sg[b][t][fi] = rg[e];
+    for (int i = 0; i < NC; ++i) {
+      o.q[i] = *reinterpret_cast<const f32x4*>(b + kChunk * D + (wave * NC + i) * 256);
+      o.kt[i] = *reinterpret_cast<const f32x4*>(b + 2 * kChunk * D + (wave * NC + i) * 256);
+      o.g[i] = *reinterpret_cast<const f32x4*>(b - lane * 4 + 3 * kChunk * D + 512 + (wave * NC + i) * 16 + fg * 4);
     }
+    o.pw = b[3 * kChunk * D + 256 + wave];
   };
-  struct Ops { f32x4 k[NC], q[NC], g[NC]; };
-  auto read = [&](int b, int t, Ops& o) __attribute__((always_inline)) {
+  f32x4 read_out = {0.f, 0.f, 0.f, 0.f};      // of the chunk before, this wave's channels and a quarter of its tokens' writes
+  auto emit = [&](int c, int b) __attribute__((always_inline)) {      // this wave: the chunk's tokens 4 g + wave
+    const float* x = reinterpret_cast<const float*>(&so[b][0][lane]) + wave;
+    const float v = (x[0] + x[256]) + (x[512] + x[768]);
+    const int t = c * kChunk + fg * 4 + wave;
+    if (live && t < sp.t) go[(size_t)t * vrow] = v;
+  };
+  auto meet = [&]() __attribute__((always_inline)) {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+  };
+  auto chunk = [&](int c, Ops& o, Ops& later) __attribute__((always_inline)) {
+    const int b = c & 1;
+    fetch(c + 2, later);
+    __builtin_amdgcn_sched_barrier(0);
+    f32x4 d = {0.f, 0.f, 0.f, 0.f}, e = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int c = 0; c < NC; ++c) {
-      const int i = (c * 16 + l16) * 4;
-      o.g[c] = *reinterpret_cast<const f32x4*>(&sg[b][t][i]);
-      o.k[c] = *reinterpret_cast<const f32x4*>(&sk[b][t][i]);
-      o.q[c] = *reinterpret_cast<const f32x4*>(&sq[b][t][i]);
+    for (int i = 0; i < NC; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) d = __builtin_amdgcn_mfma_f32_16x16x4f32(o.k[i][r], s[i][r], d, 0, 0, 0);
+    so[b][wave][lane] = read_out;
+    sd[b][wave][lane] = d;
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i][r], s[i][r], e, 0, 0, 0);
+    meet();
+    const f32x4 d0 = sd[b][0][lane], d1 = sd[b][1][lane], d2 = sd[b][2][lane], d3 = sd[b][3][lane];
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[i][r] *= o.g[i][r];
+    f32x4 u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float x = o.v[r] - ((d0[r] + d1[r]) + (d2[r] + d3[r]));
+      u = __builtin_amdgcn_mfma_f32_16x16x4f32(o.t[r], x, u, 0, 0, 0);
     }
+    if (c > 0) emit(c - 1, b);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int i = 0; i < NC; ++i) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kt[i][r], u[r], s[i], 0, 0, 0);
+    const float uw = wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3];
+    read_out = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pw, uw, e, 0, 0, 0);
   };
-  fetch(0);
-  stage(0);
-  __syncthreads();
-  int b = 0;
-  for (int t0 = 0; t0 < sp.t; t0 += kT, b ^= 1) {
-    const float beta = nb, bv = nb * nv, kq = nc;      // of token l16
-    float keep = 0.f;
-    Ops ops[2];
-    read(b, 0, ops[0]);
-    const bool more = t0 + kT < sp.t;
-    if (more) fetch(t0 + kT);
-    unroll_tokens<0, kT>([&](auto tc) __attribute__((always_inline)) {
-      constexpr int t = decltype(tc)::value;
-      if constexpr (t + 1 < kT) read(b, t + 1, ops[(t + 1) & 1]);
-      __builtin_amdgcn_sched_barrier(0);      // (a whole token of work between the request and its use)
-      const Ops& o = ops[t & 1];
-      float d[2] = {0.f, 0.f}, e[2] = {0.f, 0.f};
-#pragma unroll
-      for (int c = 0; c < NC; ++c) {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) s[c][j] *= o.g[c][j];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) d[j & 1] += s[c][j] * o.k[c][j];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) e[j & 1] += s[c][j] * o.q[c][j];
-      }
-      const float dd = row16_sum(d[0] + d[1]), ee = row16_sum(e[0] + e[1]);
-      float u;
-      {
-#pragma clang fp contract(off)
-        u = row_bcast<t>(bv) - row_bcast<t>(beta) * dd;      // beta (v - S^T k)
-      }
-#pragma unroll
-      for (int c = 0; c < NC; ++c)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) s[c][j] += o.k[c][j] * u;
-      const float out = ee + row_bcast<t>(kq) * u;
-      keep = l16 == t ? out : keep;
-      __builtin_amdgcn_sched_barrier(0);
-    });
-    if (l16 < kT) so[l16][cl] = keep;
-    if (more) stage(b ^ 1);
-    __syncthreads();
-    const int t = tid >> 4, c = cb * 16 + (tid & 15);
-    if (t < kT && t0 + t < sp.t && c < vdim) p.o[(size_t)(sp.row0 + t0 + t) * vrow + h * vdim + c] = so[t][tid & 15];
-    __syncthreads();
+  Ops ops3[3];
+  fetch(0, ops3[0]);
+  fetch(1, ops3[1]);
+  for (int c = 0; c < nch; c += 3) {
+    chunk(c, ops3[0], ops3[2]);
+    if (c + 1 < nch) chunk(c + 1, ops3[1], ops3[0]);
+    if (c + 2 < nch) chunk(c + 2, ops3[2], ops3[1]);
   }
+  so[nch & 1][wave][lane] = read_out;
+  meet();
+  emit(nch - 1, nch & 1);
   if (live)
 #pragma unroll
     for (int c = 0; c < NC; ++c)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int i = (c * 16 + l16) * 4 + j;
-        if (i < dim) S[(size_t)i * v4 + col] = s[c][j];
+      for (int r = 0; r < 4; ++r) {
+        const int i = (wave * NC + c) * 16 + fg * 4 + r;
+        if (i < dim) S[(size_t)i * v4 + col] = s[c][r];
       }
 }
 
@@ -605,7 +700,7 @@ extern "C" int chatts_delta_decode(const ChattsDeltaArgs* a, chatts_stream_t str
 
 extern "C" int chatts_delta_prep(const ChattsDeltaArgs* a, chatts_stream_t stream) {
   if (const int rc = check_delta(a, "delta_prep")) return rc;
-  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->gate && a->beta && a->kq && a->a2 && a->g2, CHATTS_E_BADARG, "delta_prep: null scratch");
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->gate && a->beta && a->a2 && a->g2, CHATTS_E_BADARG, "delta_prep: null scratch");
   if (a->n_rows == 0) return CHATTS_OK;
   CHATTS_REQUIRE(a->rank_a % 32 == 0 && a->rank_g % 32 == 0 && ((uintptr_t)a->a2 % 16) == 0 && ((uintptr_t)a->g2 % 16) == 0 && a->off_a % 4 == 0 && a->off_g % 4 == 0,
                  CHATTS_E_SHAPE, "delta_prep: ranks %d / %d must be padded to multiples of 32", a->rank_a, a->rank_g);
@@ -624,17 +719,26 @@ extern "C" int chatts_delta_prep(const ChattsDeltaArgs* a, chatts_stream_t strea
   return CHATTS_OK;
 }
 
+extern "C" int64_t chatts_delta_chunk_floats(int heads, int dim, int n_rows, int n_spans) {
+  return (int64_t)(n_rows / kChunk + n_spans) * heads * chunk_floats((dim + 63) / 64);
+}
+
+template <int NC>
+static void launch_scan(const ChattsDeltaArgs* a, hipStream_t s) {
+  hipLaunchKernelGGL(delta_chunk_kernel<NC>, dim3(a->heads, a->n_rows / kChunk + a->n_spans), dim3(256), 0, s, *a);
+  hipLaunchKernelGGL(delta_scan_kernel<NC>, dim3(a->heads * ((a->vdim + 15) / 16), a->n_spans), dim3(256), 0, s, *a);
+}
+
 extern "C" int chatts_delta_scan(const ChattsDeltaArgs* a, chatts_stream_t stream) {
   if (const int rc = check_delta(a, "delta_scan")) return rc;
-  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->kq && a->o && a->spans, CHATTS_E_BADARG, "delta_scan: null scratch");
+  CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->beta && a->chunks && a->o && a->spans, CHATTS_E_BADARG, "delta_scan: null scratch");
+  CHATTS_REQUIRE(((uintptr_t)a->chunks % 16) == 0, CHATTS_E_SHAPE, "delta_scan: alignment");
   if (a->n_spans == 0) return CHATTS_OK;
-  const int cb = (a->vdim + 15) / 16;
-  const dim3 g(a->heads * cb, a->n_spans), b(256);
-  hipStream_t s = as_stream(stream);
   switch ((a->dim + 63) / 64) {
-    case 1: hipLaunchKernelGGL(delta_scan_kernel<1>, g, b, 0, s, *a); break;
-    case 2: hipLaunchKernelGGL(delta_scan_kernel<2>, g, b, 0, s, *a); break;
-    default: hipLaunchKernelGGL(delta_scan_kernel<4>, g, b, 0, s, *a); break;
+    case 1: launch_scan<1>(a, as_stream(stream)); break;
+    case 2: launch_scan<2>(a, as_stream(stream)); break;
+    case 3: launch_scan<3>(a, as_stream(stream)); break;
+    default: launch_scan<4>(a, as_stream(stream)); break;
   }
   CHATTS_CHECK_LAUNCH("delta_scan");
   return CHATTS_OK;

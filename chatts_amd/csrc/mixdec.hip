@@ -237,7 +237,7 @@ static int mix_delta(const ChattsMixDecoder* d, const ChattsMixLayer& l, const C
   a.rows = d->b.rows; a.n_rows = t; a.spans = d->b.spans; a.n_spans = n_spans;
   a.out = out;
   if (single) return chatts_delta_decode(&a, s);
-  a.q = d->b.dq; a.k = d->b.dk; a.v = d->b.dv; a.g = d->b.dg; a.gate = d->b.dgate; a.beta = d->b.dbeta; a.kq = d->b.dkq; a.o = d->b.dout;
+  a.q = d->b.dq; a.k = d->b.dk; a.v = d->b.dv; a.g = d->b.dg; a.gate = d->b.dgate; a.beta = d->b.dbeta; a.chunks = d->b.dchunks; a.o = d->b.dout;
   a.exact = d->c.exact;
   int rc;
   if ((rc = chatts_delta_prep(&a, s)) != 0) return rc;
@@ -257,6 +257,14 @@ extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens,
   CHATTS_REQUIRE(d && tokens && (single || spans), CHATTS_E_BADARG, "mixdec_forward: null argument");
   const ChattsMixConfig& c = d->c;
   CHATTS_REQUIRE(t >= 1 && t <= c.t_max && (single || (n_spans >= 1 && n_spans <= c.max_slots)), CHATTS_E_SHAPE, "mixdec_forward: %d rows in %d segments", t, n_spans);
+  if (!single) {
+    int rows = 0;
+    for (int i = 0; i < n_spans; ++i) {
+      CHATTS_REQUIRE(spans[i].row0 == rows && spans[i].t >= 1, CHATTS_E_SHAPE, "mixdec_forward: segment %d starts at row %d, not %d", i, spans[i].row0, rows);
+      rows += spans[i].t;
+    }
+    CHATTS_REQUIRE(rows == t, CHATTS_E_SHAPE, "mixdec_forward: segments hold %d of %d rows", rows, t);
+  }
   StageRange stage(single ? "chatts.mix.decode" : "chatts.mix.prefill");
   int rc;
   if ((rc = chatts_embed_token_batched(tokens, t, d->b.embed, 0, c.vocab, c.width_p, d->b.x, s)) != 0) return rc;

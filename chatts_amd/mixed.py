@@ -342,7 +342,7 @@ class MixedDecoder(SlotModel):
             "dv": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
             "dg": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.dim)), **f32),
             "dgate": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32), "dbeta": torch.zeros((rows, most(lambda L: L.delta.heads)), **f32),
-            "dkq": torch.zeros((rows, most(lambda L: L.delta.kv_heads)), **f32),
+            "dchunks": torch.zeros(most(lambda L: int(lib.chatts_delta_chunk_floats(L.delta.heads, L.delta.dim, T, MB))), **f32),
             "dout": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
             "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
@@ -359,7 +359,7 @@ class MixedDecoder(SlotModel):
                              q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), qx=P(B["x_q"]), cbuf=P(B["x_c"]), krbuf=P(B["x_kr"]),
                              kx_hi=P(B["x_k"][0]), kx_lo=P(B["x_k"][1]), vx_hi=P(B["x_v"][0]), vx_lo=P(B["x_v"][1]), zero=P(B["x_zero"]), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
                              logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
-                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dkq", "dout")})
+                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout")})
         h = lib.chatts_mixdec_create(C.byref(mc), arr, runs, C.byref(mb))
         if not h:
             raise _lib.ChattsError(-1, lib.chatts_last_error().decode())

@@ -811,17 +811,19 @@ typedef struct ChattsDeltaArgs {
   float* ring;
   const ChattsRow* rows;
   int n_rows;
-  const ChattsSpan* spans;   /* device; chatts_delta_scan only */
+  const ChattsSpan* spans;   /* device; chatts_delta_scan only: spans cover rows 0 .. n_rows - 1 in order, without gaps */
   int n_spans;
   /* scratch of the several-token form: q / k [T, kv_heads * dim], v / o [T, heads * vdim], g (decays) [T, heads * dim],
-   * gate [T, heads * vdim], beta [T, heads], kq (k . q) [T, kv_heads] */
-  float *q, *k, *v, *g, *gate, *beta, *kq, *o;
+   * gate [T, heads * vdim], beta [T, heads], chunks: chatts_delta_chunk_floats() */
+  float *q, *k, *v, *g, *gate, *beta, *chunks, *o;
   int exact;                 /* 32-bit runs: the low-rank products of the several-token form in true float32 */
   ChattsOperand out;
 } ChattsDeltaArgs;
 int chatts_delta_decode(const ChattsDeltaArgs* args, chatts_stream_t stream);   /* every row is a segment of one token: one launch */
 int chatts_delta_prep(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* several tokens: convolutions, norms, decays, gates ... */
 int chatts_delta_scan(const ChattsDeltaArgs* args, chatts_stream_t stream);     /* ... the recurrence over every span ... */
+#define CHATTS_DELTA_CHUNK 16
+int64_t chatts_delta_chunk_floats(int heads, int dim, int n_rows, int n_spans);   /* size of `chunks` */
 int chatts_delta_out(const ChattsDeltaArgs* args, chatts_stream_t stream);      /* ... norm and gate of the read-outs, ring update */
 
 /* ---- latent attention (latent.hip) ----
@@ -910,7 +912,7 @@ typedef struct ChattsMixBuffers {
   size_t partial_elems;
   chatts_bf16 *qx, *cbuf, *krbuf, *kx_hi, *kx_lo, *vx_hi, *vx_lo;   /* latent, expanded form (ChattsLatentExpandArgs) */
   const chatts_bf16* zero;
-  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dkq, *dout;
+  float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dchunks, *dout;
   ChattsRow* rows;                                   /* device, [t_max] */
   ChattsSpan* spans;                                 /* device, [max_slots] */
   int32_t* table;                                    /* device, [max_slots, table_stride] */

@@ -191,9 +191,10 @@ class Delta:
         else:
             H, KH, dim, vd = self.H, self.KH, self.dim, self.vd
             z = lambda n: torch.full((at, n), float("nan"), device=DEV)
-            q, k, v, g, beta, kq, o = z(KH * dim), z(KH * dim), z(H * vd), z(H * dim), z(H), z(KH), z(H * vd)
+            q, k, v, g, beta, o = z(KH * dim), z(KH * dim), z(H * vd), z(H * dim), z(H), z(H * vd)
+            chunks = torch.full((int(_lib.load().chatts_delta_chunk_floats(H, dim, at, len(segs))),), float("nan"), device=DEV)
             gate = z(H * vd)
-            a.q, a.k, a.v, a.g, a.beta, a.kq, a.o, a.gate = (t.data_ptr() for t in (q, k, v, g, beta, kq, o, gate))
+            a.q, a.k, a.v, a.g, a.beta, a.chunks, a.o, a.gate = (t.data_ptr() for t in (q, k, v, g, beta, chunks, o, gate))
             a.exact = int(forms == "scan32")
             for fn in ("chatts_delta_prep", "chatts_delta_scan", "chatts_delta_out"):
                 call(fn, a)
