@@ -519,6 +519,7 @@ __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(Chatts
   // (consecutive workgroups take consecutive heads: the column blocks of a head run on one XCD where heads % 8 == 0, its operands in that L2)
   const int cb = blockIdx.x / p.heads, h = blockIdx.x - cb * p.heads, tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const float mine[4] = {wave == 0 ? 1.f : 0.f, wave == 1 ? 1.f : 0.f, wave == 2 ? 1.f : 0.f, wave == 3 ? 1.f : 0.f};
   const int dim = p.dim, vdim = p.vdim, v4 = (vdim + 3) & ~3, fr = lane & 15, fg = lane >> 4, col = cb * 16 + fr;
   const bool live = col < vdim;
   float* S = p.state + ((size_t)sp.slot * p.heads + h) * dim * v4;
@@ -530,90 +531,117 @@ __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(Chatts
       const int i = (wave * NC + c) * 16 + fg * 4 + r;
       s[c][r] = sp.pos0 > 0 && live && i < dim ? S[(size_t)i * v4 + col] : 0.f;
     }
-  const int vrow = p.heads * vdim, nch = (sp.t + kChunk - 1) / kChunk;
-  const float* ops = p.chunks + ((size_t)(sp.row0 / kChunk + blockIdx.y) * p.heads + h) * chunk_floats(NC) + lane * 4;
+  // addresses: a uniform base per chunk + constant 32-bit offsets of the lane
+  const int vrow = p.heads * vdim, t_all = __builtin_amdgcn_readfirstlane(sp.t), row0 = __builtin_amdgcn_readfirstlane(sp.row0), nch = (t_all + kChunk - 1) / kChunk;
+  const float* ops = p.chunks + ((size_t)(row0 / kChunk + blockIdx.y) * p.heads + h) * chunk_floats(NC);
   const size_t step = (size_t)p.heads * chunk_floats(NC);
-  const float* gv = p.v + (size_t)sp.row0 * vrow + h * vdim + (live ? col : 0);
-  float* go = p.o + (size_t)sp.row0 * vrow + h * vdim + col;
+  const float* gv = p.v + (size_t)row0 * vrow + h * vdim;
+  float* go = p.o + (ptrdiff_t)row0 * vrow + h * vdim;
+  const uint32_t lane16 = lane * 16, tile0 = wave * NC * 1024, gain0 = (wave * NC * 16 + fg * 4) * 4, p0 = lane16 + wave * 4;
+  const uint32_t v_last = ((uint32_t)(t_all - 1) * vrow + (live ? col : 0)) * 4;
+  uint32_t v_at[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) v_at[r] = ((uint32_t)(fg * 4 + r) * vrow + (live ? col : 0)) * 4;
+  const uint32_t o_at = ((uint32_t)(fg * 4 + wave) * vrow + col) * 4;
   struct Ops { f32x4 k[NC], q[NC], kt[NC], g[NC], t, v; float pw; };
+  auto at4 = [](const float* base, uint32_t off) __attribute__((always_inline)) { return *reinterpret_cast<const f32x4*>(reinterpret_cast<const char*>(base) + off); };
+  auto at1 = [](const float* base, uint32_t off) __attribute__((always_inline)) { return *reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + off); };
   auto fetch = [&](int c, Ops& o) __attribute__((always_inline)) {
     if (c > nch - 1) c = nch - 1;
     const float* b = ops + (size_t)c * step;
 #pragma unroll
-    for (int i = 0; i < NC; ++i) o.k[i] = *reinterpret_cast<const f32x4*>(b + (wave * NC + i) * 256);
+    for (int i = 0; i < NC; ++i) o.k[i] = at4(b + i * 256, tile0 + lane16);
+    const uint32_t skip = (uint32_t)c * kChunk * vrow * 4;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      int t = c * kChunk + fg * 4 + r;
-      if (t > sp.t - 1) t = sp.t - 1;
-      o.v[r] = gv[(size_t)t * vrow];
+      const uint32_t off = v_at[r] + skip;
+      o.v[r] = at1(gv, off < v_last ? off : v_last);
     }
-    o.t = *reinterpret_cast<const f32x4*>(b + 3 * kChunk * D);
+    o.t = at4(b + 3 * kChunk * D, lane16);
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
-      o.q[i] = *reinterpret_cast<const f32x4*>(b + kChunk * D + (wave * NC + i) * 256);
-      o.kt[i] = *reinterpret_cast<const f32x4*>(b + 2 * kChunk * D + (wave * NC + i) * 256);
-      o.g[i] = *reinterpret_cast<const f32x4*>(b - lane * 4 + 3 * kChunk * D + 512 + (wave * NC + i) * 16 + fg * 4);
+      o.q[i] = at4(b + kChunk * D + i * 256, tile0 + lane16);
+      o.kt[i] = at4(b + 2 * kChunk * D + i * 256, tile0 + lane16);
+      o.g[i] = at4(b + 3 * kChunk * D + 512 + i * 16, gain0);
     }
-    o.pw = b[3 * kChunk * D + 256 + wave];
+    o.pw = at1(b + 3 * kChunk * D + 256, p0);
   };
   f32x4 read_out = {0.f, 0.f, 0.f, 0.f};      // of the chunk before, this wave's channels and a quarter of its tokens' writes
-  auto emit = [&](int c, int b) __attribute__((always_inline)) {      // this wave: the chunk's tokens 4 g + wave
-    const float* x = reinterpret_cast<const float*>(&so[b][0][lane]) + wave;
-    const float v = (x[0] + x[256]) + (x[512] + x[768]);
-    const int t = c * kChunk + fg * 4 + wave;
-    if (live && t < sp.t) go[(size_t)t * vrow] = v;
+  // this wave writes the tokens 4 g + wave of a chunk
+  const int emit_from = live ? fg * 4 + wave : t_all;
+  auto collect = [&](int b, float (&x)[4]) __attribute__((always_inline)) {
+#pragma unroll
+    for (int w = 0; w < 4; ++w) x[w] = reinterpret_cast<const float*>(&so[b][w][lane])[wave];
+  };
+  auto emit = [&](int c, const float (&x)[4]) __attribute__((always_inline)) {
+    const int t0 = c * kChunk;
+    if (c >= 0 && emit_from < t_all - t0) *reinterpret_cast<float*>(reinterpret_cast<char*>(go + (ptrdiff_t)t0 * vrow) + o_at) = (x[0] + x[1]) + (x[2] + x[3]);
   };
   auto meet = [&]() __attribute__((always_inline)) {
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
   };
+  // S^T (G k) is the critical chain: it goes first, the products of S^T (G q) fill the waits of the exchange
+  constexpr int kBefore = 3;
   auto chunk = [&](int c, Ops& o, Ops& later) __attribute__((always_inline)) {
     const int b = c & 1;
     fetch(c + 2, later);
     __builtin_amdgcn_sched_barrier(0);
     f32x4 d = {0.f, 0.f, 0.f, 0.f}, e = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < NC; ++i)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) d = __builtin_amdgcn_mfma_f32_16x16x4f32(o.k[i][r], s[i][r], d, 0, 0, 0);
+    for (int i = 0; i < 4 * NC; ++i) d = __builtin_amdgcn_mfma_f32_16x16x4f32(o.k[i >> 2][i & 3], s[i >> 2][i & 3], d, 0, 0, 0);
     so[b][wave][lane] = read_out;
+    __builtin_amdgcn_sched_barrier(0);
+    e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[0][0], s[0][0], e, 0, 0, 0);
+    __builtin_amdgcn_sched_barrier(0);
     sd[b][wave][lane] = d;
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int i = 0; i < NC; ++i)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i][r], s[i][r], e, 0, 0, 0);
+    for (int i = 1; i < kBefore; ++i) e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i >> 2][i & 3], s[i >> 2][i & 3], e, 0, 0, 0);
+    __builtin_amdgcn_sched_barrier(0);
     meet();
     const f32x4 d0 = sd[b][0][lane], d1 = sd[b][1][lane], d2 = sd[b][2][lane], d3 = sd[b][3][lane];
+    float past[4];
+    collect(b, past);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int i = kBefore; i < 4 * NC; ++i) e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i >> 2][i & 3], s[i >> 2][i & 3], e, 0, 0, 0);
+    __builtin_amdgcn_sched_barrier(0);
+    f32x4 u = {0.f, 0.f, 0.f, 0.f}, x;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) x[r] = o.v[r] - ((d0[r] + d1[r]) + (d2[r] + d3[r]));
+#pragma unroll
+    for (int r = 0; r < 4; ++r) u = __builtin_amdgcn_mfma_f32_16x16x4f32(o.t[r], x[r], u, 0, 0, 0);
 #pragma unroll
     for (int i = 0; i < NC; ++i)
 #pragma unroll
       for (int r = 0; r < 4; ++r) s[i][r] *= o.g[i][r];
-    f32x4 u = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float x = o.v[r] - ((d0[r] + d1[r]) + (d2[r] + d3[r]));
-      u = __builtin_amdgcn_mfma_f32_16x16x4f32(o.t[r], x, u, 0, 0, 0);
-    }
-    if (c > 0) emit(c - 1, b);
+    emit(c - 1, past);
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
       for (int i = 0; i < NC; ++i) s[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.kt[i][r], u[r], s[i], 0, 0, 0);
-    const float uw = wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3];
+    const float uw = u[0] * mine[0] + u[1] * mine[1] + u[2] * mine[2] + u[3] * mine[3];      // = u[wave], without branches
     read_out = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pw, uw, e, 0, 0, 0);
   };
   Ops ops3[3];
   fetch(0, ops3[0]);
   fetch(1, ops3[1]);
-  for (int c = 0; c < nch; c += 3) {
+  int c = 0;
+  for (; c + 3 <= nch; c += 3) {
     chunk(c, ops3[0], ops3[2]);
-    if (c + 1 < nch) chunk(c + 1, ops3[1], ops3[0]);
-    if (c + 2 < nch) chunk(c + 2, ops3[2], ops3[1]);
+    chunk(c + 1, ops3[1], ops3[0]);
+    chunk(c + 2, ops3[2], ops3[1]);
   }
+  if (c < nch) chunk(c, ops3[0], ops3[2]);
+  if (c + 1 < nch) chunk(c + 1, ops3[1], ops3[0]);
   so[nch & 1][wave][lane] = read_out;
   meet();
-  emit(nch - 1, nch & 1);
+  float past[4];
+  collect(nch & 1, past);
+  emit(nch - 1, past);
   if (live)
 #pragma unroll
     for (int c = 0; c < NC; ++c)
