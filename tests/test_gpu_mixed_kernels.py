@@ -248,6 +248,27 @@ def test_delta_portions_batches_and_reused_slots(shape):
         assert rel(torch.cat(got[n]), want[n]) < 1e-4, n
 
 
+@pytest.mark.parametrize("a_log,dt,what", [(4.0, 3.0, "forgets at once"), (1.5, 1.0, "fades within a chunk"), (-6.0, -9.0, "keeps everything")])
+def test_delta_extreme_decays_and_repeated_keys(a_log, dt, what):
+    """decay products that vanish within a few tokens or stay at 1, and one key written over and over at full strength"""
+    m = Delta(2, 1, 48, 32, 2, 8, 8)
+    m.a_log, m.dt_bias = torch.tensor([a_log, a_log - 1]), m.dt_bias * 0.5 + 1.5 + dt
+    m.t["na"], m.t["dt"] = (-torch.exp(m.a_log)).to(DEV), m.dt_bias.to(DEV)
+    T = 70
+    x = m.inputs(T, 3)
+    k0, nk = m.off["k"], m.KH * m.dim
+    x[20:60, k0:k0 + nk] = x[20, k0:k0 + nk]
+    x[:, m.off["b"]:m.off["b"] + m.H] = 9.0
+    want, S = m.reference(x)
+    for cuts in ([T], [17, 2, 31, 20]):
+        got, at = [], 0
+        for c in cuts:
+            got += m.step([(1, at, x[at:at + c])], "scan32")
+            at += c
+        assert rel(torch.cat(got), want) < 5e-5, (what, cuts)
+        assert rel(m.state[1, :, :, :m.vd], S) < 5e-5, (what, cuts)
+
+
 def test_delta_parked_rows_touch_nothing():
     m = Delta(2, 2, 16, 16, 3, 8, 8)
     before = m.state.clone(), m.ring.clone()
