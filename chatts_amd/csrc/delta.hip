@@ -513,7 +513,8 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(ChattsDeltaArgs p) {
 template <int NC>
 __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(ChattsDeltaArgs p) {
   constexpr int D = NC * 64;
-  __shared__ f32x4 sd[2][4][64], so[2][4][64];
+  __shared__ f32x4 sd[2][4][64];
+  __shared__ float so[2][4][4][64];
   const ChattsSpan sp = p.spans[blockIdx.y];
   if (sp.t < 1) return;
   // (consecutive workgroups take consecutive heads: the column blocks of a head run on one XCD where heads % 8 == 0, its operands in that L2)
@@ -546,52 +547,66 @@ __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(Chatts
   struct Ops { f32x4 k[NC], q[NC], kt[NC], g[NC], t, v; float pw; };
   auto at4 = [](const float* base, uint32_t off) __attribute__((always_inline)) { return *reinterpret_cast<const f32x4*>(reinterpret_cast<const char*>(base) + off); };
   auto at1 = [](const float* base, uint32_t off) __attribute__((always_inline)) { return *reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + off); };
-  auto fetch = [&](int c, Ops& o) __attribute__((always_inline)) {
+  auto fetch_part = [&](int part, int c, Ops& o) __attribute__((always_inline)) {      // 0 .. kParts - 1
     if (c > nch - 1) c = nch - 1;
     const float* b = ops + (size_t)c * step;
+    if (part == 0)
 #pragma unroll
-    for (int i = 0; i < NC; ++i) o.k[i] = at4(b + i * 256, tile0 + lane16);
-    const uint32_t skip = (uint32_t)c * kChunk * vrow * 4;
+      for (int i = 0; i < NC; ++i) o.k[i] = at4(b + i * 256, tile0 + lane16);
+    if (part == 1) {
+      const uint32_t skip = (uint32_t)c * kChunk * vrow * 4;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const uint32_t off = v_at[r] + skip;
-      o.v[r] = at1(gv, off < v_last ? off : v_last);
+      for (int r = 0; r < 4; ++r) {
+        const uint32_t off = v_at[r] + skip;
+        o.v[r] = at1(gv, off < v_last ? off : v_last);
+      }
     }
-    o.t = at4(b + 3 * kChunk * D, lane16);
+    if (part == 2) {
+      o.t = at4(b + 3 * kChunk * D, lane16);
 #pragma unroll
-    for (int i = 0; i < NC; ++i) {
-      o.q[i] = at4(b + kChunk * D + i * 256, tile0 + lane16);
-      o.kt[i] = at4(b + 2 * kChunk * D + i * 256, tile0 + lane16);
-      o.g[i] = at4(b + 3 * kChunk * D + 512 + i * 16, gain0);
+      for (int i = 0; i < NC; ++i) o.q[i] = at4(b + kChunk * D + i * 256, tile0 + lane16);
     }
-    o.pw = at1(b + 3 * kChunk * D + 256, p0);
+    if (part == 3)
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        o.g[i] = at4(b + 3 * kChunk * D + 512 + i * 16, gain0);
+        o.kt[i] = at4(b + 2 * kChunk * D + i * 256, tile0 + lane16);
+      }
+    if (part == 4) o.pw = at1(b + 3 * kChunk * D + 256, p0);
+  };
+  constexpr int kParts = 5;
+  auto fetch = [&](int c, Ops& o) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < kParts; ++i) fetch_part(i, c, o);
   };
   f32x4 read_out = {0.f, 0.f, 0.f, 0.f};      // of the chunk before, this wave's channels and a quarter of its tokens' writes
   // this wave writes the tokens 4 g + wave of a chunk
   const int emit_from = live ? fg * 4 + wave : t_all;
   auto collect = [&](int b, float (&x)[4]) __attribute__((always_inline)) {
 #pragma unroll
-    for (int w = 0; w < 4; ++w) x[w] = reinterpret_cast<const float*>(&so[b][w][lane])[wave];
+    for (int w = 0; w < 4; ++w) x[w] = so[b][w][wave][lane];
   };
   auto emit = [&](int c, const float (&x)[4]) __attribute__((always_inline)) {
     const int t0 = c * kChunk;
     if (c >= 0 && emit_from < t_all - t0) *reinterpret_cast<float*>(reinterpret_cast<char*>(go + (ptrdiff_t)t0 * vrow) + o_at) = (x[0] + x[1]) + (x[2] + x[3]);
+  };
+  auto hand_over = [&](int b) __attribute__((always_inline)) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) so[b][wave][r][lane] = read_out[r];
   };
   auto meet = [&]() __attribute__((always_inline)) {
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
   };
-  // S^T (G k) is the critical chain: it goes first, the products of S^T (G q) fill the waits of the exchange
+  // S^T (G k) is the critical chain: it goes first; the products of S^T (G q) and the requests fill the waits of the exchange
   constexpr int kBefore = 3;
   auto chunk = [&](int c, Ops& o, Ops& later) __attribute__((always_inline)) {
     const int b = c & 1;
-    fetch(c + 2, later);
-    __builtin_amdgcn_sched_barrier(0);
     f32x4 d = {0.f, 0.f, 0.f, 0.f}, e = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < 4 * NC; ++i) d = __builtin_amdgcn_mfma_f32_16x16x4f32(o.k[i >> 2][i & 3], s[i >> 2][i & 3], d, 0, 0, 0);
-    so[b][wave][lane] = read_out;
+    hand_over(b);
     __builtin_amdgcn_sched_barrier(0);
     e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[0][0], s[0][0], e, 0, 0, 0);
     __builtin_amdgcn_sched_barrier(0);
@@ -606,8 +621,11 @@ __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(Chatts
     collect(b, past);
     __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int i = kBefore; i < 4 * NC; ++i) e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i >> 2][i & 3], s[i >> 2][i & 3], e, 0, 0, 0);
-    __builtin_amdgcn_sched_barrier(0);
+    for (int i = kBefore; i < 4 * NC || i - kBefore < kParts; ++i) {      // requests for the chunk after the next go between products
+      if (i < 4 * NC) e = __builtin_amdgcn_mfma_f32_16x16x4f32(o.q[i >> 2][i & 3], s[i >> 2][i & 3], e, 0, 0, 0);
+      if (i - kBefore < kParts) fetch_part(i - kBefore, c + 2, later);
+      __builtin_amdgcn_sched_barrier(0);
+    }
     f32x4 u = {0.f, 0.f, 0.f, 0.f}, x;
 #pragma unroll
     for (int r = 0; r < 4; ++r) x[r] = o.v[r] - ((d0[r] + d1[r]) + (d2[r] + d3[r]));
@@ -637,7 +655,7 @@ __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(Chatts
   }
   if (c < nch) chunk(c, ops3[0], ops3[2]);
   if (c + 1 < nch) chunk(c + 1, ops3[1], ops3[0]);
-  so[nch & 1][wave][lane] = read_out;
+  hand_over(nch & 1);
   meet();
   float past[4];
   collect(nch & 1, past);
