@@ -352,24 +352,38 @@ __global__ __launch_bounds__(256) void delta_lowrank_kernel(ChattsDeltaArgs p, i
 #pragma unroll
       for (int k = 0; k < KMAX; ++k)
 #pragma unroll
-        for (int q = NP - 1; q >= 0; --q) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[k][q], b[t % 3][k], acc[t], 0, 0, 0);
+        for (int q = NP - 1; q >= 0; --q) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b[t % 3][k], a[k][q], acc[t], 0, 0, 0);
       __builtin_amdgcn_sched_barrier(0);
     }
   }
+  // a lane: 4 consecutive outputs of row m0 + fr per tile
   const float inv_dim = 1.0f / (float)p.dim;
+  if (m0 + fr >= p.n_rows) return;
+  float* dst = (dec ? p.g : p.gate) + (size_t)(m0 + fr) * n;
+  const bool quads = (n & 3) == 0;
 #pragma unroll
   for (int t = 0; t < kLrTiles; ++t) {
-    const int o = n0 + t * 16 + fr;
-    if (o < n) {
-      int h = dec ? (int)((float)o * inv_dim) : 0;      // o / dim: off by one at most (o < 2^24), set right below
-      if (dec) h += (o - h * p.dim >= p.dim) - (o < h * p.dim);
-      const float na = dec ? p.neg_a[h] : 0.f, bias = dec ? p.dt_bias[o] : 0.f;
+    const int o0 = n0 + t * 16 + fg * 4;
+    if (o0 >= n) continue;
+    f32x4 v = acc[t];
+    if (dec) {
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        const int row = m0 + fg * 4 + q;
-        const float v = dec ? exp_hw(na * softplus_f(acc[t][q] + bias)) : sigmoid_f(acc[t][q]);
-        if (row < p.n_rows) (dec ? p.g : p.gate)[(size_t)row * n + o] = v;
+        const int o = o0 + q < n ? o0 + q : n - 1;
+        int h = (int)((float)o * inv_dim);      // o / dim: off by one at most (o < 2^24), set right below
+        h += (o - h * p.dim >= p.dim) - (o < h * p.dim);
+        v[q] = exp_hw(p.neg_a[h] * softplus_f(v[q] + p.dt_bias[o]));
       }
+    } else {
+#pragma unroll
+      for (int q = 0; q < 4; ++q) v[q] = sigmoid_f(v[q]);
+    }
+    if (quads) {
+      *reinterpret_cast<f32x4*>(dst + o0) = v;
+    } else {
+#pragma unroll
+      for (int q = 0; q < 4; ++q)
+        if (o0 + q < n) dst[o0 + q] = v[q];
     }
   }
 }
@@ -671,30 +685,48 @@ __global__ __launch_bounds__(256, NC <= 2 ? 2 : 1) void delta_scan_kernel(Chatts
 }
 
 // ---- norm + gate of the read-outs; the last `taps` rows of a span enter the ring (prep has read the old entries by now) -----------
-__global__ __launch_bounds__(256) void delta_out_kernel(ChattsDeltaArgs p) {
-  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = blockIdx.y * 4 + (threadIdx.x >> 6), waves = gridDim.y * 4;
+// A head belongs to G lanes (a power of two, 4 G >= vdim), 4 consecutive columns each.
+template <bool QUADS>      // vdim % 4 == 0
+__global__ __launch_bounds__(256) void delta_out_kernel(ChattsDeltaArgs p, int G) {
+  const int row = blockIdx.x, tid = threadIdx.x, per = 256 / G, i = (tid & (G - 1)) * 4;
   const ChattsRow R = p.rows[row];
   if (R.pos < 0) return;
   const int vdim = p.vdim, vrow = p.heads * vdim;
-  for (int h = wave; h < p.heads; h += waves) {
-    float v[4], ss = 0.f;
+  const float* o = p.o + (size_t)row * vrow;
+  const float* gate = p.gate + (size_t)row * vrow;
+  float w[4];
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-      const int i = c * 64 + lane;
-      v[c] = i < vdim ? p.o[(size_t)row * vrow + h * vdim + i] : 0.f;
-      ss += v[c] * v[c];
+  for (int j = 0; j < 4; ++j) w[j] = i + j < vdim ? p.norm_w[i + j] : 0.f;
+  for (int h = blockIdx.y * per + tid / G; h < p.heads; h += gridDim.y * per) {      // (h is the same in all lanes of a group)
+    float v[4] = {0.f, 0.f, 0.f, 0.f}, g[4] = {0.f, 0.f, 0.f, 0.f};
+    const int at = h * vdim + i;
+    if (QUADS) {
+      if (i < vdim) {
+        const f32x4 x = *reinterpret_cast<const f32x4*>(o + at), y = *reinterpret_cast<const f32x4*>(gate + at);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { v[j] = x[j]; g[j] = y[j]; }
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (i + j < vdim) { v[j] = o[at + j]; g[j] = gate[at + j]; }
     }
-    ss = wave_sum(ss);
+    float ss = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+    for (int x = 1; x < G; x <<= 1) ss += __shfl_xor(ss, x, 64);
     const float f = 1.0f / sqrtf(ss / (float)vdim + p.eps);
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-      const int i = c * 64 + lane;
-      if (i < vdim) store_operand(p.out, row, h * vdim + i, v[c] * f * p.norm_w[i] * p.gate[(size_t)row * vrow + h * vdim + i]);
+    for (int j = 0; j < 4; ++j) v[j] = v[j] * f * w[j] * g[j];
+    if (QUADS) {
+      if (i < vdim) store_operand4(p.out, row, at, v);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (i + j < vdim) store_operand(p.out, row, at + j, v[j]);
     }
   }
   if (R.rest < p.taps) {
     float* ring = p.ring + ((size_t)R.slot * p.taps + R.pos % p.taps) * p.conv_ch;
-    for (int i = blockIdx.y * 256 + threadIdx.x; i < p.conv_ch; i += gridDim.y * 256) ring[i] = p.proj[(size_t)row * p.ld_proj + i];
+    for (int c = blockIdx.y * 256 + tid; c < p.conv_ch; c += gridDim.y * 256) ring[c] = p.proj[(size_t)row * p.ld_proj + c];
   }
 }
 
@@ -794,7 +826,12 @@ extern "C" int chatts_delta_out(const ChattsDeltaArgs* a, chatts_stream_t stream
   if (const int rc = check_delta(a, "delta_out")) return rc;
   CHATTS_REQUIRE(a->o && a->gate && (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim, CHATTS_E_BADARG, "delta_out: null pointer");
   if (a->n_rows == 0) return CHATTS_OK;
-  hipLaunchKernelGGL(delta_out_kernel, dim3(a->n_rows, (a->heads + 15) / 16), dim3(256), 0, as_stream(stream), *a);
+  int lanes = 1;
+  while (lanes * 4 < a->vdim) lanes *= 2;
+  const int per = 256 / lanes;
+  const dim3 g(a->n_rows, (a->heads + 2 * per - 1) / (2 * per));
+  if (a->vdim % 4 == 0 && a->out.ld % 4 == 0) hipLaunchKernelGGL(delta_out_kernel<true>, g, dim3(256), 0, as_stream(stream), *a, lanes);
+  else hipLaunchKernelGGL(delta_out_kernel<false>, g, dim3(256), 0, as_stream(stream), *a, lanes);
   CHATTS_CHECK_LAUNCH("delta_out");
   return CHATTS_OK;
 }

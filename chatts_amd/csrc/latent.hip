@@ -570,14 +570,14 @@ __global__ __launch_bounds__(256, OCC) void latent_prefill_kernel(LatentPrefill 
 // ---- a product per head: wave = 16 rows x 16 columns, A split hi / lo in registers ----
 __global__ __launch_bounds__(256) void head_linear_kernel(ChattsHeadLinearArgs p) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = blockIdx.z;
-  const int n0 = (blockIdx.x * 4 + wave) * 16, m0 = blockIdx.y * 16;
+  const int n0 = (blockIdx.x * (blockDim.x >> 6) + wave) * 16, m0 = blockIdx.y * 16;
   if (n0 >= p.n) return;
   const int fr = lane & 15, fg = lane >> 4;
   const int r = m0 + fr < p.m ? m0 + fr : p.m - 1;
   const float* a = p.a + (size_t)r * p.lda + (size_t)h * p.a_head + fg * 8;
   const uint16_t* w = p.w + ((size_t)h * p.n + n0 + fr) * p.k + fg * 8;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 8
   for (int k = 0; k < p.k; k += 32) {
     const f32x4 x0 = *reinterpret_cast<const f32x4*>(a + k), x1 = *reinterpret_cast<const f32x4*>(a + k + 4);
     const bf16x8_t b = *reinterpret_cast<const bf16x8_t*>(w + k);
@@ -703,7 +703,8 @@ extern "C" int chatts_head_linear(const ChattsHeadLinearArgs* a, chatts_stream_t
     return launch_gemm_f32_batched(a->a, a->a_head, a->lda, a->w, (int64_t)a->n * a->k, a->k, a->out.f32, a->out_head, a->out.ld, a->m, a->n, a->k,
                                    a->heads, as_stream(stream));
   }
-  hipLaunchKernelGGL(head_linear_kernel, dim3((a->n / 16 + 3) / 4, (a->m + 15) / 16, a->heads), dim3(256), 0, as_stream(stream), *a);
+  const int waves = a->m <= 16 ? 1 : 4;      // one row tile: spread over as many CUs as there are column tiles
+  hipLaunchKernelGGL(head_linear_kernel, dim3((a->n / 16 + waves - 1) / waves, (a->m + 15) / 16, a->heads), dim3(64 * waves), 0, as_stream(stream), *a);
   CHATTS_CHECK_LAUNCH("head_linear");
   return CHATTS_OK;
 }
