@@ -186,12 +186,12 @@ __device__ __forceinline__ void store_operand4(const ChattsOperand& o, size_t ro
 __device__ __forceinline__ float exp_hw(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896341f); }
 __device__ __forceinline__ float sigmoid_f(float x) { return __builtin_amdgcn_rcpf(1.0f + exp_hw(-x)); }
 // log(1 + e^x): for a small e = e^x through log(1 + e) = 2 atanh(e / (2 + e)), which keeps the relative precision log(1 + e) would lose
-__device__ __forceinline__ float softplus_f(float x) {
-  if (x > 20.f) return x;
-  const float e = exp_hw(x);
-  if (e > 0.5f) return __builtin_amdgcn_logf(1.0f + e) * 0.69314718055994531f;
+__device__ __forceinline__ float softplus_f(float x) {      // (both forms are computed and selected: no branches in unrolled loops)
+  const float e = exp_hw(fminf(x, 20.f)), large = __builtin_amdgcn_logf(1.0f + e) * 0.69314718055994531f;
   const float z = e * __builtin_amdgcn_rcpf(2.0f + e), z2 = z * z;
-  return 2.0f * z * (1.0f + z2 * (1.0f / 3 + z2 * (1.0f / 5 + z2 * (1.0f / 7 + z2 * (1.0f / 9 + z2 * (1.0f / 11))))));
+  const float small = 2.0f * z * (1.0f + z2 * (1.0f / 3 + z2 * (1.0f / 5 + z2 * (1.0f / 7 + z2 * (1.0f / 9 + z2 * (1.0f / 11))))));
+  const float r = e > 0.5f ? large : small;
+  return x > 20.f ? x : r;
 }
 inline hipStream_t as_stream(chatts_stream_t s) { return reinterpret_cast<hipStream_t>(s); }
 

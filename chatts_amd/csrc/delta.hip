@@ -62,7 +62,7 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
       if (!ok) cw[u][g] = 0.f;
     }
   }
-  const float beta_in = pr[p.off_b + h], na = p.neg_a[h];
+  const float beta_in = pr[p.off_b + h];
   constexpr int kW = 8;      // 8-value pieces of this thread's low-rank row requested ahead
   const bool dec = tid < dim;
   const int lr = tid < dim + vdim ? tid : dim + vdim - 1, lrow = dec ? h * dim + tid : h * vdim + (lr - dim < 0 ? 0 : lr - dim);
@@ -71,7 +71,7 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
   u32x4 wv[kW];
 #pragma unroll
   for (int c = 0; c < kW; ++c) wv[c] = *reinterpret_cast<const u32x4*>(lw + (size_t)(c < lrank ? c : 0) * lrows * 8);
-  const float lbias = dec ? p.dt_bias[lrow] : 0.f;
+  const float lbias = dec ? p.dt_bias[lrow] : 0.f, lneg = dec ? p.neg_a[lrow] : 0.f;
   const float a_in = pr[p.off_a + (tid < p.rank_a ? tid : 0)], g_in = pr[p.off_g + (tid < p.rank_g ? tid : 0)];
   f32x4 s[NR];
 #pragma unroll
@@ -129,7 +129,7 @@ __global__ __launch_bounds__(NT) void delta_decode_kernel(ChattsDeltaArgs p, int
       c = kW;
     }
     for (; c < rank8; ++c) acc = dot8(*reinterpret_cast<const u32x4*>(w + (size_t)c * rows * 8), x + c * 8, acc);
-    if (de) sg[i] = exp_hw(na * softplus_f(acc + (i == tid ? lbias : p.dt_bias[o])));
+    if (de) sg[i] = exp_hw((i == tid ? lneg : p.neg_a[o]) * softplus_f(acc + (i == tid ? lbias : p.dt_bias[o])));
     else sgate[i - dim] = sigmoid_f(acc);
   }
 #pragma unroll
@@ -300,7 +300,7 @@ __global__ __launch_bounds__(256) void delta_prep_v_kernel(ChattsDeltaArgs p) {
       if (live[i]) p.beta[(size_t)(row0 + i) * p.heads + h] = sigmoid_f(p.proj[(size_t)(row0 + i) * p.ld_proj + p.off_b + h]);
 }
 
-// The low-rank products with what follows them:  g = exp(neg_a[h] * softplus(A2 a + dt_bias)),  gate = sigmoid(G2 gin).  grid (row tiles of 16, blocks of
+// The low-rank products with what follows them:  g = exp(neg_a * softplus(A2 a + dt_bias)),  gate = sigmoid(G2 gin).  grid (row tiles of 16, blocks of
 // 512 outputs): a wave keeps its 16 rows of a (or gin) in registers, split into bf16 planes (three of them in 32-bit runs: exact), and walks 8
 // tiles of 16 outputs, the weights requested two tiles ahead.
 constexpr int kLrTiles = 8;
@@ -357,29 +357,35 @@ __global__ __launch_bounds__(256) void delta_lowrank_kernel(ChattsDeltaArgs p, i
     }
   }
   // a lane: 4 consecutive outputs of row m0 + fr per tile
-  const float inv_dim = 1.0f / (float)p.dim;
+  const bool quads = (n & 3) == 0;
+  f32x4 na[kLrTiles], bias[kLrTiles];
+  if (dec)
+#pragma unroll
+    for (int t = 0; t < kLrTiles; ++t) {
+      const int o0 = n0 + t * 16 + fg * 4;
+      if (quads) {
+        const int o = o0 < n ? o0 : 0;
+        na[t] = *reinterpret_cast<const f32x4*>(p.neg_a + o);
+        bias[t] = *reinterpret_cast<const f32x4*>(p.dt_bias + o);
+      } else {
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const int o = o0 + q < n ? o0 + q : n - 1;
+          na[t][q] = p.neg_a[o];
+          bias[t][q] = p.dt_bias[o];
+        }
+      }
+    }
   if (m0 + fr >= p.n_rows) return;
   float* dst = (dec ? p.g : p.gate) + (size_t)(m0 + fr) * n;
-  const bool quads = (n & 3) == 0;
 #pragma unroll
   for (int t = 0; t < kLrTiles; ++t) {
     const int o0 = n0 + t * 16 + fg * 4;
-    if (o0 >= n) continue;
-    f32x4 v = acc[t];
-    if (dec) {
+    f32x4 v;
 #pragma unroll
-      for (int q = 0; q < 4; ++q) {
-        const int o = o0 + q < n ? o0 + q : n - 1;
-        int h = (int)((float)o * inv_dim);      // o / dim: off by one at most (o < 2^24), set right below
-        h += (o - h * p.dim >= p.dim) - (o < h * p.dim);
-        v[q] = exp_hw(p.neg_a[h] * softplus_f(v[q] + p.dt_bias[o]));
-      }
-    } else {
-#pragma unroll
-      for (int q = 0; q < 4; ++q) v[q] = sigmoid_f(v[q]);
-    }
+    for (int q = 0; q < 4; ++q) v[q] = dec ? exp_hw(na[t][q] * softplus_f(acc[t][q] + bias[t][q])) : sigmoid_f(acc[t][q]);
     if (quads) {
-      *reinterpret_cast<f32x4*>(dst + o0) = v;
+      if (o0 < n) *reinterpret_cast<f32x4*>(dst + o0) = v;
     } else {
 #pragma unroll
       for (int q = 0; q < 4; ++q)
@@ -780,8 +786,8 @@ extern "C" int chatts_delta_prep(const ChattsDeltaArgs* a, chatts_stream_t strea
   if (const int rc = check_delta(a, "delta_prep")) return rc;
   CHATTS_REQUIRE(a->q && a->k && a->v && a->g && a->gate && a->beta && a->a2 && a->g2, CHATTS_E_BADARG, "delta_prep: null scratch");
   if (a->n_rows == 0) return CHATTS_OK;
-  CHATTS_REQUIRE(a->rank_a % 32 == 0 && a->rank_g % 32 == 0 && ((uintptr_t)a->a2 % 16) == 0 && ((uintptr_t)a->g2 % 16) == 0 && a->off_a % 4 == 0 && a->off_g % 4 == 0,
-                 CHATTS_E_SHAPE, "delta_prep: ranks %d / %d must be padded to multiples of 32", a->rank_a, a->rank_g);
+  CHATTS_REQUIRE(a->rank_a % 32 == 0 && a->rank_g % 32 == 0 && ((uintptr_t)a->a2 % 16) == 0 && ((uintptr_t)a->g2 % 16) == 0 && a->off_a % 4 == 0 && a->off_g % 4 == 0 &&
+                     ((uintptr_t)a->neg_a % 16) == 0 && ((uintptr_t)a->dt_bias % 16) == 0, CHATTS_E_SHAPE, "delta_prep: ranks %d / %d must be padded to multiples of 32", a->rank_a, a->rank_g);
   const int ablocks = (a->heads * a->dim + 64 * kLrTiles - 1) / (64 * kLrTiles), gblocks = (a->heads * a->vdim + 64 * kLrTiles - 1) / (64 * kLrTiles);
   const dim3 g((a->n_rows + 15) / 16, ablocks + gblocks), b(256);
   if (a->exact) hipLaunchKernelGGL((delta_lowrank_kernel<3, 4>), g, b, 0, as_stream(stream), *a, ablocks);

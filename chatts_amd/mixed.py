@@ -266,7 +266,7 @@ class MixedDecoder(SlotModel):
                                  heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, taps=m.taps, rank_a=ra_p, rank_g=rg_p,
                                  conv_w=self._dev(conv), a2=self._mat(m.a2, None, ra_p)[0], g2=self._mat(m.g2, None, rg_p)[0],
                                  a2d=self._pieces(m.a2, ra_p), g2d=self._pieces(m.g2, rg_p), ld_a2=ra_p, ld_g2=rg_p,
-                                 dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32))), norm_w=self._f32(m.norm))
+                                 dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32)).repeat_interleave(m.dim)), norm_w=self._f32(m.norm))
 
     def _build(self, sd):
         cfg, lib, dev = self.config, self.lib, self.device

@@ -804,7 +804,7 @@ typedef struct ChattsDeltaArgs {
   const chatts_bf16 *a2d, *g2d;   /* chatts_delta_decode: the same, as [rank / 8, rows, 8] (neighbouring rows side by side) */
   int ld_a2, ld_g2;
   const float* dt_bias;      /* [heads * dim] */
-  const float* neg_a;        /* [heads] = -exp(A_log) */
+  const float* neg_a;        /* [heads * dim] = -exp(A_log), a head's value for each of its channels */
   const float* norm_w;       /* [vdim] */
   float eps;
   float* state;

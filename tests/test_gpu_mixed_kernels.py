@@ -129,7 +129,7 @@ class Delta:
         for n, t in self.conv.items():
             cw[:, self.off[n]:self.off[n] + t.shape[0]] = t.T
         pad = lambda t, c: torch.cat([t, torch.zeros(t.shape[0], c - t.shape[1], dtype=t.dtype)], 1)
-        self.t = dict(cw=cw, a2=pad(self.a2, self.rap), g2=pad(self.g2, self.rgp), dt=self.dt_bias, na=-torch.exp(self.a_log), nw=self.norm)
+        self.t = dict(cw=cw, a2=pad(self.a2, self.rap), g2=pad(self.g2, self.rgp), dt=self.dt_bias, na=-torch.exp(self.a_log).repeat_interleave(dim), nw=self.norm)
         for n in ("a2", "g2"):
             self.t[n + "d"] = self.t[n].view(self.t[n].shape[0], -1, 8).transpose(0, 1)
         self.t = {k: v.contiguous().to(DEV) for k, v in self.t.items()}
@@ -253,7 +253,7 @@ def test_delta_extreme_decays_and_repeated_keys(a_log, dt, what):
     """decay products that vanish within a few tokens or stay at 1, and one key written over and over at full strength"""
     m = Delta(2, 1, 48, 32, 2, 8, 8)
     m.a_log, m.dt_bias = torch.tensor([a_log, a_log - 1]), m.dt_bias * 0.5 + 1.5 + dt
-    m.t["na"], m.t["dt"] = (-torch.exp(m.a_log)).to(DEV), m.dt_bias.to(DEV)
+    m.t["na"], m.t["dt"] = (-torch.exp(m.a_log).repeat_interleave(m.dim)).to(DEV), m.dt_bias.to(DEV)
     T = 70
     x = m.inputs(T, 3)
     k0, nk = m.off["k"], m.KH * m.dim
