@@ -376,20 +376,31 @@ __global__ __launch_bounds__(256) void delta_lowrank_kernel(ChattsDeltaArgs p, i
         }
       }
     }
-  if (m0 + fr >= p.n_rows) return;
-  float* dst = (dec ? p.g : p.gate) + (size_t)(m0 + fr) * n;
+  // ... turned round in LDS (a wave's own part), so that a row's outputs leave as whole cache lines
+  constexpr int kCols = 16 * kLrTiles, kLd = kCols + 4;
+  __shared__ __attribute__((aligned(16))) float turn[4][16][kLd];
 #pragma unroll
   for (int t = 0; t < kLrTiles; ++t) {
-    const int o0 = n0 + t * 16 + fg * 4;
     f32x4 v;
 #pragma unroll
     for (int q = 0; q < 4; ++q) v[q] = dec ? exp_hw(na[t][q] * softplus_f(acc[t][q] + bias[t][q])) : sigmoid_f(acc[t][q]);
+    *reinterpret_cast<f32x4*>(&turn[wave][fr][t * 16 + fg * 4]) = v;
+  }
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  constexpr int kLanes = kCols / 4, kRows = 64 / kLanes;      // lanes of a row, rows at a time
+  float* dst = dec ? p.g : p.gate;
+  const int o0 = n0 + (lane % kLanes) * 4;
+#pragma unroll
+  for (int i = 0; i < 16 / kRows; ++i) {
+    const int rl = i * kRows + lane / kLanes, row = m0 + rl;
+    const f32x4 v = *reinterpret_cast<const f32x4*>(&turn[wave][rl][(lane % kLanes) * 4]);
+    if (row >= p.n_rows) continue;
     if (quads) {
-      if (o0 < n) *reinterpret_cast<f32x4*>(dst + o0) = v;
+      if (o0 < n) *reinterpret_cast<f32x4*>(dst + (size_t)row * n + o0) = v;
     } else {
 #pragma unroll
       for (int q = 0; q < 4; ++q)
-        if (o0 + q < n) dst[o0 + q] = v[q];
+        if (o0 + q < n) dst[(size_t)row * n + o0 + q] = v[q];
     }
   }
 }
