@@ -10,7 +10,7 @@ from . import build as _build
 _LIB = None
 
 OK, E_BADARG, E_SHAPE, E_COUNT_MISMATCH, E_LAUNCH, E_WORKSPACE = 0, -1, -2, -3, -4, -5
-EPI_NONE, EPI_GELU, EPI_RESID, EPI_SWIGLU, EPI_RELU2 = 0, 1, 2, 3, 4
+EPI_NONE, EPI_GELU, EPI_RESID, EPI_SWIGLU, EPI_RELU2, EPI_CLAMPGLU = 0, 1, 2, 3, 4, 5
 
 c_void_p, c_int, c_int32, c_int64, c_float, c_size_t, c_uint32 = (
     C.c_void_p, C.c_int, C.c_int32, C.c_int64, C.c_float, C.c_size_t, C.c_uint32)
@@ -29,7 +29,7 @@ class TsWeights(C.Structure):
                 ("b", c_void_p * 8)]
 
 
-ABI_VERSION = 10           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
+ABI_VERSION = 11           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
 W8_FP8, W8_INT8 = 0, 1     # ChattsLinearArgs.w8_format
 
 
@@ -42,7 +42,8 @@ class LinearArgs(C.Structure):
                 ("c_hi", c_void_p), ("c_lo", c_void_p), ("ld_cplanes", c_int),
                 ("post_norm_w", c_void_p), ("post_norm_eps", c_float), ("post_hi", c_void_p), ("post_lo", c_void_p), ("ld_post", c_int),
                 ("w4", c_void_p), ("w4_sz", c_void_p), ("ldw4", c_int), ("w4_group", c_int),
-                ("w8_format", c_int), ("tp_reduce", c_void_p), ("w_tiled", c_void_p), ("planes_tiled", c_int), ("exact_f32", c_int)]
+                ("w8_format", c_int), ("tp_reduce", c_void_p), ("w_tiled", c_void_p), ("planes_tiled", c_int), ("exact_f32", c_int),
+                ("glu_limit", c_float), ("glu_alpha", c_float)]
 
 
 class LinearFp8Args(C.Structure):
@@ -155,7 +156,56 @@ class LatentExpandArgs(C.Structure):
                 [("out", Operand), ("workspace", c_void_p), ("workspace_bytes", c_size_t)])
 
 
-MIX_LATENT, MIX_DELTA = 1, 2
+class EmbedPairArgs(C.Structure):
+    _fields_ = [("tokens", c_void_p), ("rows", c_void_p), ("t", c_int), ("single", c_int), ("width_p", c_int), ("vocab", c_int), ("embed", c_void_p),
+                ("scale", c_float), ("bigram", c_void_p), ("buckets", c_int64), ("mul_prev", c_int64), ("mul_cur", c_int64), ("prev", c_void_p),
+                ("x", c_void_p), ("x0", c_void_p)]
+
+
+class PairNormArgs(C.Structure):
+    _fields_ = [("x", c_void_p), ("t", c_int), ("width", c_int), ("ldx", c_int), ("groups", c_int), ("eps", c_float), ("y", c_void_p), ("place", c_void_p),
+                ("weight", c_void_p), ("kept", c_void_p), ("h", Operand), ("top", c_int), ("x0", c_void_p), ("w1", c_void_p), ("w2", c_void_p),
+                ("out1", Operand), ("out2", Operand), ("n_mix", c_int), ("mu", c_void_p), ("mix", Operand), ("mix_stride", c_int64), ("prev", c_void_p),
+                ("rows", c_void_p)]
+
+
+class TokenShiftArgs(C.Structure):
+    _fields_ = [("h", c_void_p), ("t", c_int), ("ldx", c_int), ("n_mix", c_int), ("mu", c_void_p), ("mix", Operand), ("mix_stride", c_int64),
+                ("prev", c_void_p), ("rows", c_void_p)]
+
+
+RECUR_WKV, RECUR_MLSTM = 1, 2
+
+
+class RecurArgs(C.Structure):
+    """ChattsRecurArgs: gated linear recurrences (csrc/recur.hip)"""
+    _fields_ = ([("kind", c_int), ("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_gate", "off_a", "off_i", "off_f", "heads",
+                                                                            "dim", "vdim", "rank")] +
+                [(n, c_void_p) for n in ("w2d", "w0", "u", "bias_i", "bias_f")] + [("cap", c_float), ("eps", c_float)] +
+                [(n, c_void_p) for n in ("norm_w", "state", "n_state", "m_state", "rows")] + [("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int),
+                 ("decay", c_void_p), ("ld_decay", c_int)] + [(n, c_void_p) for n in ("gates", "chunks", "o", "den")] +
+                [("out", Operand), ("h", c_void_p), ("prev", c_void_p), ("ld_h", c_int)])
+
+
+class WindowArgs(C.Structure):
+    """ChattsWindowArgs: grouped-head attention over paged keys and values (csrc/window.hip)"""
+    _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_gate", "heads", "kv_heads", "dim", "vdim", "dim_p", "vdim_p")] +
+                [("scale", c_float), ("eps", c_float), ("q_norm", c_void_p), ("k_norm", c_void_p), ("window", c_int), ("keep_first", c_int), ("sink", c_int),
+                 ("kcache", c_void_p), ("vcache", c_void_p), ("cache_f32", c_int), ("table", c_void_p), ("table_stride", c_int), ("log_block", c_int),
+                 ("rows", c_void_p), ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int), ("longest", c_int), ("q", Operand), ("n_splits", c_int),
+                 ("partial", c_void_p), ("out", Operand)])
+
+
+class MoeArgs(C.Structure):
+    """ChattsMoeArgs: mixture of experts (csrc/moe.hip)"""
+    _fields_ = ([(n, c_int) for n in ("experts", "identity", "top", "groups", "keep", "width_p", "ff_p")] +
+                [("gate_up", c_void_p), ("down", c_void_p), ("correction", c_void_p), ("logits", c_void_p), ("ld_logits", c_int), ("h", Operand), ("rows", c_void_p),
+                 ("n_rows", c_int), ("exact", c_int)] + [(n, c_void_p) for n in ("ids", "place", "order", "offsets", "tiles", "weight", "kept")] +
+                [("act", Operand), ("y", c_void_p)])
+
+
+MIX_LATENT, MIX_DELTA, MIX_RECUR, MIX_WINDOW = 1, 2, 3, 4
+FF_NONE, FF_RELU2, FF_CLAMPGLU, FF_MOE = 0, 1, 2, 3
 EXPAND_PAD = 128           # CHATTS_LATENT_EXPAND_PAD
 
 
@@ -163,23 +213,30 @@ class MixLayer(C.Structure):
     _fields_ = ([("kind", c_int)] + [(n, c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "in_t", "out", "out_t", "up", "up_t", "down",
                                                              "down_t")] +
                 [(n, c_int) for n in ("in_n", "out_k", "ff")] + [("uk", c_void_p), ("uv", c_void_p), ("ukx", c_void_p), ("uvx", c_void_p)] +
-                [(n, c_int) for n in ("dim_p", "vdim_p", "out_head")] + [("latent", LatentArgs), ("delta", DeltaArgs)])
+                [(n, c_int) for n in ("dim_p", "vdim_p", "out_head")] + [("latent", LatentArgs), ("delta", DeltaArgs), ("parallel", c_int), ("ff_kind", c_int),
+                 ("glu_limit", c_float), ("glu_alpha", c_float), ("n_mix", c_int), ("mix_row", c_int * 8), ("mix_t", c_void_p * 8), ("mu", c_void_p), ("w2", c_void_p), ("w2_n", c_int),
+                 ("recur", RecurArgs), ("window", WindowArgs), ("router", c_void_p), ("router_t", c_void_p), ("router_n", c_int), ("moe", MoeArgs)])
 
 
 class MixRun(C.Structure):
-    _fields_ = [("layer", c_int), ("add", c_void_p), ("cache", c_void_p), ("state", c_void_p), ("ring", c_void_p)]
+    _fields_ = [("layer", c_int), ("add", c_void_p), ("cache", c_void_p), ("state", c_void_p), ("ring", c_void_p), ("n_state", c_void_p), ("m_state", c_void_p),
+                ("vcache", c_void_p), ("join", c_void_p), ("join_t", c_void_p)]
 
 
 class MixConfig(C.Structure):
     _fields_ = ([(n, c_int) for n in ("width", "width_p", "n_layers", "n_runs", "exact", "t_max", "max_slots", "max_ctx", "expand_rows")] +
-                [("vocab", c_int64), ("vocab_p", c_int64), ("eps", c_float), ("block_size", c_int), ("table_stride", c_int)])
+                [("vocab", c_int64), ("vocab_p", c_int64), ("eps", c_float), ("block_size", c_int), ("table_stride", c_int), ("norm_groups", c_int),
+                 ("embed_scale", c_float), ("bigram_buckets", c_int64), ("bigram_prev", c_int64), ("bigram_cur", c_int64)])
 
 
 class MixBuffers(C.Structure):
     _fields_ = ([(n, c_void_p) for n in ("embed", "head", "head_t", "final_norm", "x", "y", "proj", "a_f32", "b_f32", "a_hi", "a_lo", "b_hi", "b_lo",
                                          "q_f32", "o_lat", "partial", "q_hi", "q_lo")] + [("partial_elems", c_size_t)] +
                 [(n, c_void_p) for n in ("qx", "cbuf", "krbuf", "kx_hi", "kx_lo", "vx_hi", "vx_lo", "zero")] +
-                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout", "rows", "spans", "table", "logits", "workspace")] +
+                [(n, c_void_p) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout", "bigram", "prev_token", "x0", "h", "m_f32", "m_hi", "m_lo")] +
+                [("mix_stride", c_int64)] +
+                [(n, c_void_p) for n in ("n_f32", "n_hi", "n_lo", "gates", "den", "moe_ids", "moe_place", "moe_order", "moe_offsets", "moe_tiles", "moe_weight",
+                                         "moe_kept", "moe_logits", "moe_y", "act_f32", "act_hi", "act_lo", "rows", "spans", "table", "logits", "workspace")] +
                 [("workspace_bytes", c_size_t)])
 
 
@@ -273,6 +330,21 @@ SIGNATURES = {
     "chatts_delta_out": (c_int, [C.POINTER(DeltaArgs), c_void_p]),
     "chatts_latent_prep": (c_int, [C.POINTER(LatentArgs), c_void_p]),
     "chatts_latent_attend": (c_int, [C.POINTER(LatentArgs), c_void_p]),
+    "chatts_embed_pair": (c_int, [C.POINTER(EmbedPairArgs), c_void_p]),
+    "chatts_pair_norm": (c_int, [C.POINTER(PairNormArgs), c_void_p]),
+    "chatts_token_shift": (c_int, [C.POINTER(TokenShiftArgs), c_void_p]),
+    "chatts_recur_decode": (c_int, [C.POINTER(RecurArgs), c_void_p]),
+    "chatts_recur_tanh": (c_int, [C.POINTER(RecurArgs), C.POINTER(Operand), c_void_p]),
+    "chatts_recur_scan": (c_int, [C.POINTER(RecurArgs), c_void_p]),
+    "chatts_recur_out": (c_int, [C.POINTER(RecurArgs), c_void_p]),
+    "chatts_recur_chunk_floats": (C.c_int64, [c_int, c_int, c_int, c_int]),
+    "chatts_window_prep": (c_int, [C.POINTER(WindowArgs), c_void_p]),
+    "chatts_window_attend": (c_int, [C.POINTER(WindowArgs), c_void_p]),
+    "chatts_window_prefill": (c_int, [C.POINTER(WindowArgs), c_void_p]),
+    "chatts_window_can_prefill": (c_int, [c_int, c_int]),
+    "chatts_moe_route": (c_int, [C.POINTER(MoeArgs), c_void_p]),
+    "chatts_moe_experts": (c_int, [C.POINTER(MoeArgs), c_void_p]),
+    "chatts_moe_tiles": (c_int, [c_int, c_int, c_int]),
     "chatts_mixdec_create": (c_void_p, [C.POINTER(MixConfig), C.POINTER(MixLayer), C.POINTER(MixRun), C.POINTER(MixBuffers)]),
     "chatts_mixdec_destroy": (None, [c_void_p]),
     "chatts_mixdec_workspace": (c_size_t, [C.POINTER(MixConfig), C.POINTER(MixLayer)]),

@@ -193,6 +193,14 @@ __device__ __forceinline__ float softplus_f(float x) {      // (both forms are c
   const float r = e > 0.5f ? large : small;
   return x > 20.f ? x : r;
 }
+// the gated feed-forward of a (gate, up) pair: silu(g) * u (CHATTS_EPI_SWIGLU, silu passed in by the caller), or with both clamped
+// (CHATTS_EPI_CLAMPGLU): g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1)
+__device__ __forceinline__ float clamp_glu(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * sigmoid_f(alpha * g) * (u + 1.0f);
+}
+__host__ __device__ constexpr bool epi_is_glu(int epilogue) { return epilogue == CHATTS_EPI_SWIGLU || epilogue == CHATTS_EPI_CLAMPGLU; }
 inline hipStream_t as_stream(chatts_stream_t s) { return reinterpret_cast<hipStream_t>(s); }
 
 // ---- stage ranges for traces (api.hip): roctx push / pop around the host-side enqueue of a stage, resolved with dlopen at first use

@@ -64,21 +64,21 @@ static int linear_impl(const ChattsLinearArgs* a, chatts_stream_t stream, const 
   const bool cplanes = a->c_hi || a->c_lo;
   CHATTS_REQUIRE((a->a || planes) && a->w && (a->c || cplanes), CHATTS_E_BADARG, "linear: null pointer");
   if (cplanes)
-    CHATTS_REQUIRE(a->c_hi && a->c_lo && a->m > 1 && a->ld_cplanes >= (a->epilogue == CHATTS_EPI_SWIGLU ? a->n / 2 : a->n),
+    CHATTS_REQUIRE(a->c_hi && a->c_lo && a->m > 1 && a->ld_cplanes >= (epi_is_glu(a->epilogue) ? a->n / 2 : a->n),
                    CHATTS_E_SHAPE, "linear: plane output needs both planes, M > 1 and ld_cplanes >= the output width");
   if (planes)
     CHATTS_REQUIRE(a->a_hi && a->a_lo && a->ld_planes >= a->k && a->ld_planes % 8 == 0 && ((uintptr_t)a->a_hi % 16) == 0 &&
                        ((uintptr_t)a->a_lo % 16) == 0 && a->m > 1 && !a->norm_w,
                    CHATTS_E_SHAPE, "linear: pre-split A needs both planes, ld_planes >= K and %% 8, 16-byte alignment, M > 1");
-  CHATTS_REQUIRE(a->epilogue >= CHATTS_EPI_NONE && a->epilogue <= CHATTS_EPI_RELU2, CHATTS_E_BADARG,
+  CHATTS_REQUIRE(a->epilogue >= CHATTS_EPI_NONE && a->epilogue <= CHATTS_EPI_CLAMPGLU, CHATTS_E_BADARG,
                  "linear: epilogue %d", a->epilogue);
   CHATTS_REQUIRE(a->epilogue != CHATTS_EPI_RESID || a->resid, CHATTS_E_BADARG, "linear: EPI_RESID without resid");
   CHATTS_REQUIRE(a->k % 32 == 0, CHATTS_E_SHAPE, "linear: K=%d must be a multiple of 32 (pad the weight)", a->k);
-  CHATTS_REQUIRE(a->n % 16 == 0 && (a->epilogue != CHATTS_EPI_SWIGLU || a->n % 32 == 0), CHATTS_E_SHAPE,
+  CHATTS_REQUIRE(a->n % 16 == 0 && (!epi_is_glu(a->epilogue) || a->n % 32 == 0), CHATTS_E_SHAPE,
                  "linear: N=%d must be a multiple of 16 (32 for SwiGLU)", a->n);
   CHATTS_REQUIRE((!a->a || (a->lda >= a->k && a->lda % 4 == 0)) && a->ldw >= a->k && a->ldw % 8 == 0, CHATTS_E_SHAPE,
                  "linear: leading dimensions lda=%d ldw=%d", a->lda, a->ldw);
-  const int ncols = a->epilogue == CHATTS_EPI_SWIGLU ? a->n / 2 : a->n;
+  const int ncols = epi_is_glu(a->epilogue) ? a->n / 2 : a->n;
   CHATTS_REQUIRE(a->ldc >= ncols || (cplanes && a->epilogue != CHATTS_EPI_RESID), CHATTS_E_SHAPE, "linear: ldc=%d < %d", a->ldc, ncols);
   CHATTS_REQUIRE(((uintptr_t)a->a % 16) == 0 && ((uintptr_t)a->w % 16) == 0 && ((uintptr_t)a->c % 16) == 0,
                  CHATTS_E_SHAPE, "linear: pointers must be 16-byte aligned");

@@ -53,7 +53,7 @@ __device__ __forceinline__ void gemm_store(const GemmParams& p, const f32x4 (&ac
       }
     return;
   }
-  if (p.epilogue == CHATTS_EPI_SWIGLU) {
+  if (epi_is_glu(p.epilogue)) {
 #pragma unroll
     for (int i = 0; i < FM; ++i)
 #pragma unroll
@@ -67,7 +67,7 @@ __device__ __forceinline__ void gemm_store(const GemmParams& p, const f32x4 (&ac
           for (int r = 0; r < 4; ++r) {
             const int row = m0 + wm * TM + i * 16 + crow0 + r;
             if (row < p.m) {
-              const float v = silu_g(acc[i][j][r] * sg + bg) * (acc[i][j + 1][r] * su + bu);
+              const float v = glu_value(p.epilogue, acc[i][j][r] * sg + bg, acc[i][j + 1][r] * su + bu, p.glu_limit, p.glu_alpha);
               if (p.c_hi) store_planes(p.c_hi, p.c_lo, (size_t)row * p.ldcp + ocol, v);
               else p.c[(size_t)row * p.ldc + ocol] = v;
             }
@@ -419,7 +419,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_stream_kernel(GemmParams p, cons
     }
   }
   if constexpr (FN == 1) {
-    if (p.direct && p.epilogue == CHATTS_EPI_SWIGLU) {
+    if (p.direct && epi_is_glu(p.epilogue)) {
       // a (gate, up) pair of 16-column fragments sits in waves (2 q, 2 q + 1): the odd wave hands its accumulator over through LDS
       // and the even one runs the two-fragment epilogue
       __syncthreads();                           // every wave is done reading the last stage
@@ -471,13 +471,13 @@ __global__ __launch_bounds__(256) void splitk_epilogue_kernel(const float* __res
                                                              const float* __restrict__ bias,
                                                              const float* __restrict__ resid, float* __restrict__ c,
                                                              int ldc, int epilogue, const float* __restrict__ scale,
-                                                             uint16_t* __restrict__ c_hi, uint16_t* __restrict__ c_lo, int ldcp) {
-  const int ncols = epilogue == CHATTS_EPI_SWIGLU ? n / 2 : n;
+                                                             uint16_t* __restrict__ c_hi, uint16_t* __restrict__ c_lo, int ldcp, float glu_limit, float glu_alpha) {
+  const int ncols = epi_is_glu(epilogue) ? n / 2 : n;
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= (size_t)m * ncols) return;
   const int row = (int)(idx / ncols), col = (int)(idx % ncols);
   const size_t plane = (size_t)m * n;
-  if (epilogue == CHATTS_EPI_SWIGLU) {
+  if (epi_is_glu(epilogue)) {
     const int prow = (col >> 4) * 32 + (col & 15);
     float g = 0.f, u = 0.f;
     for (int s = 0; s < sk; ++s) {
@@ -486,8 +486,9 @@ __global__ __launch_bounds__(256) void splitk_epilogue_kernel(const float* __res
     }
     if (scale) { g *= scale[prow]; u *= scale[prow + 16]; }
     if (bias) { g += bias[prow]; u += bias[prow + 16]; }
-    if (c_hi) store_planes(c_hi, c_lo, (size_t)row * ldcp + col, silu_g(g) * u);
-    else c[(size_t)row * ldc + col] = silu_g(g) * u;
+    const float v = glu_value(epilogue, g, u, glu_limit, glu_alpha);
+    if (c_hi) store_planes(c_hi, c_lo, (size_t)row * ldcp + col, v);
+    else c[(size_t)row * ldc + col] = v;
     return;
   }
   float v = 0.f;
@@ -965,6 +966,7 @@ int launch_gemm(const ChattsLinearArgs* a_in, hipStream_t s, const RopeFuse* rop
   p.w8 = a->w8; p.w8_scale = a->w8_scale; p.ldw8 = a->ldw8; p.w8_format = a->w8_format;
   p.c_hi = a->c_hi; p.c_lo = a->c_lo; p.ldcp = a->ld_cplanes;
   p.wt = ring ? a->w_tiled : nullptr; p.planes_tiled = a->planes_tiled;
+  p.glu_limit = a->glu_limit; p.glu_alpha = a->glu_alpha;
   if (sk > 1) {
     const size_t need = (size_t)sk * a->m * a->n * sizeof(float);
     CHATTS_REQUIRE(a->workspace && a->workspace_bytes >= need, CHATTS_E_WORKSPACE,
@@ -1068,7 +1070,7 @@ int launch_gemm(const ChattsLinearArgs* a_in, hipStream_t s, const RopeFuse* rop
     *rope_done = true;
     return CHATTS_OK;
   }
-  if (sk > 1 && sk <= 8 && a->epilogue != CHATTS_EPI_SWIGLU && a->n % 4 == 0 && a->ldc % 4 == 0 &&
+  if (sk > 1 && sk <= 8 && !epi_is_glu(a->epilogue) && a->n % 4 == 0 && a->ldc % 4 == 0 &&
       ((uintptr_t)a->c % 16) == 0 && ((uintptr_t)a->resid % 16) == 0 && ((uintptr_t)a->bias % 16) == 0 &&
       (!a->w8 || ((uintptr_t)a->w8_scale % 16) == 0) && opt_get(OPT_EPI_V4, 1) != 0) {
     const size_t total = (size_t)a->m * (a->n / 4);
@@ -1077,11 +1079,11 @@ int launch_gemm(const ChattsLinearArgs* a_in, hipStream_t s, const RopeFuse* rop
                        a->w8 ? a->w8_scale : nullptr, a->c_hi, a->c_lo, a->ld_cplanes);
     CHATTS_CHECK_LAUNCH("splitk_epilogue_v4");
   } else if (sk > 1) {
-    const int ncols = a->epilogue == CHATTS_EPI_SWIGLU ? a->n / 2 : a->n;
+    const int ncols = epi_is_glu(a->epilogue) ? a->n / 2 : a->n;
     const size_t total = (size_t)a->m * ncols;
     hipLaunchKernelGGL(splitk_epilogue_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, s,
                        reinterpret_cast<const float*>(a->workspace), sk, a->m, a->n, a->bias, a->resid, a->c,
-                       a->ldc, a->epilogue, a->w8 ? a->w8_scale : nullptr, a->c_hi, a->c_lo, a->ld_cplanes);
+                       a->ldc, a->epilogue, a->w8 ? a->w8_scale : nullptr, a->c_hi, a->c_lo, a->ld_cplanes, a->glu_limit, a->glu_alpha);
     CHATTS_CHECK_LAUNCH("splitk_epilogue");
   }
   if (post_norm)                  // no split-K epilogue to fuse into: the contract still holds, as its own launch

@@ -24,6 +24,7 @@ struct GemmParams {
   int ldcp;
   const uint16_t* wt;    // optional (gemm_ring_kernel): W in the tiled layout of chatts_tile_bf16 - a 1 KB LDS-DMA piece is 1 KB of memory
   int planes_tiled;      // a_hi / a_lo are in that layout too
+  float glu_limit, glu_alpha;
 };
 
 __device__ __forceinline__ void store_planes(uint16_t* hi, uint16_t* lo, size_t off, float v) {
@@ -39,6 +40,10 @@ __device__ __forceinline__ void store_planes(uint16_t* hi, uint16_t* lo, size_t 
 __device__ __forceinline__ float gelu_erf_f(float x) { return 0.5f * x * (1.0f + erff(x * 0.70710678118654752440f)); }
 __device__ __forceinline__ float relu2_f(float x) { const float r = fmaxf(x, 0.f); return r * r; }      // the square of relu
 __device__ __forceinline__ float silu_g(float x) { return x / (1.0f + expf(-x)); }
+
+__device__ __forceinline__ float glu_value(int epilogue, float g, float u, float limit, float alpha) {
+  return epilogue == CHATTS_EPI_SWIGLU ? silu_g(g) * u : clamp_glu(g, u, limit, alpha);
+}
 
 constexpr int kRingPanel = 256;      // W rows per panel of the prefill kernel
 // gemm_ring.hip: the prefill kernel's decomposition (M-tiles per panel, K splits) and launcher

@@ -12,6 +12,7 @@ struct GemmF32Params {
   const float* resid;
   float* c;
   int m, n, k, lda, ldw, ldc, epilogue;
+  float glu_limit, glu_alpha;
   int64_t a_batch, w_batch, c_batch;
 };
 
@@ -55,6 +56,19 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Params p) {
     }
   }
   float* c = p.c + (int64_t)blockIdx.z * p.c_batch;
+  if (epi_is_glu(p.epilogue)) {      // the two 16-column halves of a wave: gate and up of the same outputs
+    const int col = n0 + wn + (lane & 15);
+    if (col + 16 >= p.n) return;
+    const float bg = p.bias ? p.bias[col] : 0.f, bu = p.bias ? p.bias[col + 16] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int row = m0 + wm + i * 16 + (lane >> 4) * 4 + q;
+        if (row < p.m) c[(size_t)row * p.ldc + ((n0 + wn) >> 1) + (lane & 15)] = glu_value(p.epilogue, acc[i][0][q] + bg, acc[i][1][q] + bu, p.glu_limit, p.glu_alpha);
+      }
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < 2; ++i)
 #pragma unroll
@@ -77,15 +91,14 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(GemmF32Params p) {
 
 int launch_gemm_f32_batched(const float* a, int64_t a_batch, int lda, const uint16_t* w, int64_t w_batch, int ldw, float* c, int64_t c_batch, int ldc,
                             int m, int n, int k, int batch, hipStream_t s) {
-  GemmF32Params p{a, w, nullptr, nullptr, c, m, n, k, lda, ldw, ldc, CHATTS_EPI_NONE, a_batch, w_batch, c_batch};
+  GemmF32Params p{a, w, nullptr, nullptr, c, m, n, k, lda, ldw, ldc, CHATTS_EPI_NONE, 0.f, 0.f, a_batch, w_batch, c_batch};
   hipLaunchKernelGGL(gemm_f32_kernel, dim3((n + 63) / 64, (m + 63) / 64, batch), dim3(256), 0, s, p);
   CHATTS_CHECK_LAUNCH("gemm_f32");
   return CHATTS_OK;
 }
 
 int launch_gemm_f32(const ChattsLinearArgs* a, hipStream_t s) {
-  CHATTS_REQUIRE(a->epilogue != CHATTS_EPI_SWIGLU, CHATTS_E_BADARG, "linear: exact_f32 has no SwiGLU epilogue");
-  GemmF32Params p{a->a, a->w, a->bias, a->resid, a->c, a->m, a->n, a->k, a->lda, a->ldw, a->ldc, a->epilogue, 0, 0, 0};
+  GemmF32Params p{a->a, a->w, a->bias, a->resid, a->c, a->m, a->n, a->k, a->lda, a->ldw, a->ldc, a->epilogue, a->glu_limit, a->glu_alpha, 0, 0, 0};
   hipLaunchKernelGGL(gemm_f32_kernel, dim3((a->n + 63) / 64, (a->m + 63) / 64, 1), dim3(256), 0, s, p);
   CHATTS_CHECK_LAUNCH("gemm_f32");
   return CHATTS_OK;

@@ -46,6 +46,7 @@ struct GemvParams {
   int ldw4, w4_group;
   TpParams tp;            // kEpiResidTp only
   int ks;                 // gemv_ksplit_kernel: waves per row group
+  float glu_limit, glu_alpha;   // CHATTS_EPI_CLAMPGLU
 };
 
 // ---- the exchange inside the launch (kEpiResidTp) ---------------------------------------------------------------------------
@@ -102,14 +103,14 @@ template <int ROWS, int EPI>
 __device__ __forceinline__ void gemv_epilogue(const GemvParams& p, int task, int lane, const float (&acc)[ROWS], uint32_t epoch = 0) {
   if (EPI == kEpiResidTp) {
     tp_push_task<ROWS>(p, epoch, task, lane, acc);
-  } else if (EPI == CHATTS_EPI_SWIGLU) {
+  } else if (epi_is_glu(EPI)) {
 #pragma unroll
     for (int u = 0; u < ROWS / 2; ++u) {
       const int rg = task_row<ROWS, EPI>(task, 2 * u);
       if (lane == u && rg + 16 < p.n) {
         float g = acc[2 * u], v = acc[2 * u + 1];
         if (p.bias) { g += p.bias[rg]; v += p.bias[rg + 16]; }
-        p.out[task * (ROWS / 2) + u] = silu_f(g) * v;
+        p.out[task * (ROWS / 2) + u] = EPI == CHATTS_EPI_CLAMPGLU ? clamp_glu(g, v, p.glu_limit, p.glu_alpha) : silu_f(g) * v;
       }
     }
   } else {
@@ -579,6 +580,7 @@ static void launch_ldsx(const GemvParams& p, int epi, bool norm, int blocks, int
     case kEpiResidTp: hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, kEpiResidTp, false>), dim3(blocks), dim3(threads), lds, s, p); break;
     case CHATTS_EPI_SWIGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_SWIGLU>(p, norm, blocks, threads, lds, s); break;
     case CHATTS_EPI_RELU2: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_RELU2>(p, norm, blocks, threads, lds, s); break;
+    case CHATTS_EPI_CLAMPGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_CLAMPGLU>(p, norm, blocks, threads, lds, s); break;
     default: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_NONE>(p, norm, blocks, threads, lds, s); break;
   }
 }
@@ -610,7 +612,7 @@ static void launch8_norm(const GemvParams& p, bool norm, int rows, int unr, int 
 // Waves per workgroup (and workgroups per CU, 0 = whatever fits) of the bf16 GEMV for a shape: the sweep results of
 // tools/gemv_sweep.py.  Also read by decode_mega.hip, whose fused RMSNorm reproduces this kernel's summation order.
 void gemv_default_geometry(int n, int k, int epilogue, int cus, int* nw_out, int* occ_out) {
-  const int swiglu = epilogue == CHATTS_EPI_SWIGLU;
+  const int swiglu = epi_is_glu(epilogue);
   const int units = swiglu ? n / 2 : n;
   int nw_auto, occ_auto = 0;
   if (k > 8192) nw_auto = 16;                       // down_proj: 55 KB of x per workgroup -> amortise over 16 waves
@@ -675,8 +677,8 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
                    (long long)tp_capacity(a->tp_reduce));
     epilogue = kEpiResidTp;
   }
-  CHATTS_REQUIRE(a->epilogue != CHATTS_EPI_RELU2 || (!a->w4 && !a->w8), CHATTS_E_BADARG, "gemv: EPI_RELU2 takes bf16 weights");
-  const int swiglu = a->epilogue == CHATTS_EPI_SWIGLU;
+  CHATTS_REQUIRE((a->epilogue != CHATTS_EPI_RELU2 && a->epilogue != CHATTS_EPI_CLAMPGLU) || (!a->w4 && !a->w8), CHATTS_E_BADARG, "gemv: EPI_RELU2 / CLAMPGLU take bf16 weights");
+  const int swiglu = epi_is_glu(a->epilogue);
   const int units = swiglu ? a->n / 2 : a->n;
   const int nchunks = (a->k + 511) / 512;
   const size_t lds = (size_t)nchunks * 512 * 4 + 64 * 4;
@@ -769,6 +771,7 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
   // K-split form (see gemv_ksplit_kernel): when the row groups alone leave the chip nearly empty - fewer than ~6 waves per CU - and a
   // row is long enough to split.  Every TP = 1 shape of the supported models has >= 10 waves per CU and keeps the whole-K kernel.
   p.ks = 1;
+  p.glu_limit = a->glu_limit; p.glu_alpha = a->glu_alpha;
   if (!a->tp_reduce && rows == 2 && unr == 2 && nchunks >= 4) {
     int ks = gemv_pick_ksplit(p.tasks, nchunks, norm, (double)a->n * a->k * 2.0, cus);
     ks = opt_get(OPT_GEMV_KS, ks);
@@ -790,6 +793,10 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
         case CHATTS_EPI_SWIGLU:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_SWIGLU, true>), g, b, lds, s, p);
           else hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_SWIGLU, false>), g, b, lds, s, p);
+          break;
+        case CHATTS_EPI_CLAMPGLU:
+          if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_CLAMPGLU, true>), g, b, lds, s, p);
+          else hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_CLAMPGLU, false>), g, b, lds, s, p);
           break;
         case CHATTS_EPI_RELU2:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_RELU2, true>), g, b, lds, s, p);
@@ -818,7 +825,7 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
 // host-only query (no device touched): the K-split factor the bf16 decode GEMV picks for a shape on this device - see gemv_pick_ksplit
 extern "C" int chatts_gemv_ksplit(int n, int k, int epilogue, int has_norm) {
   if (n <= 0 || k <= 0) return -1;
-  const int swiglu = epilogue == CHATTS_EPI_SWIGLU;
+  const int swiglu = chatts::epi_is_glu(epilogue);
   const int units = swiglu ? n / 2 : n, upt = swiglu ? 1 : 2;
   const int cus = chatts::device_cus() > 0 ? chatts::device_cus() : 256;
   return chatts::gemv_pick_ksplit((units + upt - 1) / upt, (k + 511) / 512, has_norm != 0, (double)n * k * 2.0, cus);

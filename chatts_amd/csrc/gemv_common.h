@@ -27,7 +27,7 @@ __device__ __forceinline__ float silu_f(float x) { return x / (1.0f + expf(-x));
 
 template <int ROWS, int EPI>
 __device__ __forceinline__ int task_row(int task, int r) {
-  if (EPI == CHATTS_EPI_SWIGLU) {   // gate/up interleaved in blocks of 16 rows: unit u -> rows g(u), g(u)+16
+  if (epi_is_glu(EPI)) {   // gate/up interleaved in blocks of 16 rows: unit u -> rows g(u), g(u)+16
     const int unit = task * (ROWS / 2) + (r >> 1);
     return (unit >> 4) * 32 + (unit & 15) + (r & 1) * 16;
   }

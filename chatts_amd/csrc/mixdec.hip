@@ -1,8 +1,12 @@
-// mixdec.hip - host-side composition of decoders with mixed layers (latent attention / gated delta rule, norms before and after each
-// sublayer, looped layer ranges).  Like decoder.hip: nothing here allocates or synchronises, a decode step is capturable.
+// mixdec.hip - host-side composition of decoders with mixed layers (latent attention, gated delta rule, gated linear recurrences, windowed attention;
+// feed-forwards or experts; looped layer ranges).  Like decoder.hip: nothing here allocates or synchronises, a decode step is capturable.
 //
-// A layer:   norm1 (in the previous residual_norm launch) -> stacked input projection -> mixer kernels -> out projection
-//            -> residual_norm (x += norm1b(y); norm2(x)) -> up (squared relu in the epilogue) -> down -> residual_norm (..., next norm1)
+// Sequential layer (norms before and after each sublayer):
+//   norm1 (in the previous residual_norm launch) -> stacked input projection -> mixer kernels -> out projection
+//   -> residual_norm (x += norm1b(y); norm2(x)) -> up (squared relu in the epilogue) -> down -> residual_norm (..., next norm1)
+// Parallel layer (two norms of the same x):
+//   pair_norm (norm1(x), norm2(x), with the experts' sum of the layer before, the token shift of a decoded token) -> input projections -> mixer kernels
+//   -> out projection, added to x -> gate_up (gated unit in the epilogue) -> down, added to x;  or router -> experts, added by the next pair_norm
 // Operands between the launches travel in the format the next projection's kernel takes for this row count: bf16 hi / lo planes
 // (2 .. 16 rows: weight-streaming kernel; >= 96 rows: the prefill kernel) or float32.
 #include <new>
@@ -45,10 +49,14 @@ extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const Chatts
   };
   for (int i = 0; i < c->n_layers; ++i) {
     const ChattsMixLayer& l = layers[i];
-    add(l.in_n, c->width_p);
+    for (int j = 0; j < l.n_mix; ++j) add(l.mix_row[j + 1] - l.mix_row[j], c->width_p);
+    if (!l.n_mix) add(l.in_n, c->width_p);
     add(c->width_p, l.out_k);
-    if (l.up) { add(l.ff, c->width_p); add(c->width_p, l.ff); }
+    if (l.w2) add(l.w2_n, l.recur.rank);
+    if (l.up) { add(l.ff_kind == CHATTS_FF_CLAMPGLU ? 2 * l.ff : l.ff, c->width_p); add(c->width_p, l.ff); }
+    if (l.router) add(l.router_n, c->width_p);
   }
+  add(c->width_p, 2 * c->width_p);
   add((int)c->vocab_p, c->width_p);
   // keys and values written out from the latents: rows in whole tiles of 64
   size_t ws = 0;
@@ -82,8 +90,14 @@ extern "C" ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, cons
     if (runs[i].layer < 0 || runs[i].layer >= c->n_layers) { set_error("mixdec_create: run %d names layer %d", i, runs[i].layer); return nullptr; }
   for (int i = 0; i < c->n_layers; ++i) {
     const ChattsMixLayer& l = layers[i];
-    if ((l.kind != CHATTS_MIX_LATENT && l.kind != CHATTS_MIX_DELTA) || !l.in || !l.out || !l.norm1 || (l.up && !(l.down && l.norm2))) {
+    const bool pair = l.kind == CHATTS_MIX_RECUR || l.kind == CHATTS_MIX_WINDOW;
+    if ((l.kind != CHATTS_MIX_LATENT && l.kind != CHATTS_MIX_DELTA && !pair) || !l.in || !l.out || !l.norm1 || (l.up && !(l.down && l.norm2)) ||
+        (l.ff_kind == CHATTS_FF_MOE && !(l.router && l.norm2 && l.moe.gate_up && l.moe.down)) || l.n_mix < 0 || l.n_mix > 7 || (l.n_mix && !l.mu)) {
       set_error("mixdec_create: layer %d is incomplete", i);
+      return nullptr;
+    }
+    if (l.parallel != layers[0].parallel || (pair && !l.parallel) || (l.ff_kind > CHATTS_FF_RELU2 && !l.parallel) || (l.ff_kind == CHATTS_FF_RELU2 && l.parallel)) {
+      set_error("mixdec_create: layer %d: sequential and parallel layers do not mix", i);
       return nullptr;
     }
   }
@@ -112,8 +126,10 @@ static ChattsOperand operand(const ChattsMixDecoder* d, bool second, int m, int 
 }
 
 static int mix_linear(const ChattsMixDecoder* d, const ChattsOperand& in, const chatts_bf16* w, const chatts_bf16* w_t, int m, int n, int k, int epilogue,
-                      const ChattsOperand& out, chatts_stream_t s) {
+                      const ChattsOperand& out, chatts_stream_t s, float limit = 0.f, float alpha = 0.f) {
   ChattsLinearArgs a{};
+  a.glu_limit = limit; a.glu_alpha = alpha;
+  a.resid = epilogue == CHATTS_EPI_RESID ? out.f32 : nullptr;
   a.a = in.f32;
   a.lda = in.ld;
   if (!in.f32) { a.a_hi = in.hi; a.a_lo = in.lo; a.ld_planes = in.ld; }
@@ -245,6 +261,175 @@ static int mix_delta(const ChattsMixDecoder* d, const ChattsMixLayer& l, const C
   return chatts_delta_out(&a, s);
 }
 
+
+static ChattsOperand second_norm(const ChattsMixDecoder* d, const ChattsMixLayer& l, int m) {
+  ChattsOperand o{};
+  o.ld = d->c.width_p;
+  const bool planes = mix_planes(d->c, m, o.ld);
+  if (planes || (l.ff_kind == CHATTS_FF_MOE && !d->c.exact)) { o.hi = d->b.n_hi; o.lo = d->b.n_lo; }      // (experts take planes, the router what its kernel wants)
+  if (!planes) o.f32 = d->b.n_f32;
+  return o;
+}
+static ChattsOperand linear_form(const ChattsOperand& o) {      // one of the two forms
+  ChattsOperand r = o;
+  if (r.f32) r.hi = r.lo = nullptr;
+  return r;
+}
+static ChattsOperand shift_operand(const ChattsMixDecoder* d, int m, int block) {
+  ChattsOperand o{};
+  o.ld = d->c.width_p;
+  const int64_t at = block * d->b.mix_stride;
+  if (mix_planes(d->c, m, o.ld)) { o.hi = d->b.m_hi + at; o.lo = d->b.m_lo + at; }
+  else o.f32 = d->b.m_f32 + at;
+  return o;
+}
+
+static int mix_recur(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, int n_spans, bool single, const ChattsOperand& out,
+                     chatts_stream_t s) {
+  StageRange stage("chatts.mix.recur");
+  ChattsRecurArgs a = l.recur;
+  a.proj = d->b.proj; a.ld_proj = l.in_n; a.eps = d->c.eps;
+  a.state = run.state; a.n_state = run.n_state; a.m_state = run.m_state;
+  a.rows = d->b.rows; a.n_rows = t; a.spans = d->b.spans; a.n_spans = n_spans;
+  a.out = out;
+  if (single) return chatts_recur_decode(&a, s);
+  a.gates = d->b.gates; a.chunks = d->b.dchunks; a.o = d->b.dout; a.den = d->b.den;
+  int rc;
+  if (a.kind == CHATTS_RECUR_WKV) {
+    const ChattsOperand low = operand(d, true, t, a.rank);
+    if ((rc = chatts_recur_tanh(&a, &low, s)) != 0) return rc;
+    if ((rc = mix_linear(d, low, l.w2, nullptr, t, l.w2_n, a.rank, CHATTS_EPI_NONE, f32_out(d->b.dg, l.w2_n), s)) != 0) return rc;
+    a.decay = d->b.dg; a.ld_decay = l.w2_n;
+    a.h = d->b.h; a.prev = run.ring; a.ld_h = d->c.width_p;
+  }
+  if ((rc = chatts_recur_scan(&a, s)) != 0) return rc;
+  return chatts_recur_out(&a, s);
+}
+
+static int mix_window(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, const ChattsSpan* spans, int n_spans, bool single,
+                      const ChattsOperand& out, chatts_stream_t s) {
+  StageRange stage("chatts.mix.window");
+  ChattsWindowArgs a = l.window;
+  a.proj = d->b.proj; a.ld_proj = l.in_n; a.eps = d->c.eps;
+  a.kcache = run.cache; a.vcache = run.vcache; a.cache_f32 = d->c.exact;
+  a.table = d->b.table; a.table_stride = d->c.table_stride; a.log_block = kv_log_block(d->c.block_size);
+  a.rows = d->b.rows; a.n_rows = t; a.spans = d->b.spans; a.n_spans = single ? 0 : n_spans;
+  a.q.ld = a.heads * a.dim_p;
+  if (d->c.exact) a.q.f32 = d->b.q_f32;
+  else a.q.hi = d->b.q_hi;
+  a.out = out; a.n_splits = 1; a.longest = 0;
+  for (int i = 0; !single && i < n_spans; ++i)
+    if (spans[i].t > a.longest) a.longest = spans[i].t;
+  if (const int rc = chatts_window_prep(&a, s)) return rc;
+  if (a.longest >= 8 && !d->c.exact && chatts_window_can_prefill(a.dim_p, a.vdim_p)) return chatts_window_prefill(&a, s);
+  if (!d->c.exact) {      // few rows: a row's tiles (32 keys a wave, 4 waves) are spread over workgroups until there are about two per CU
+    const int group = a.heads / a.kv_heads, wgs = a.kv_heads * ((group + 15) / 16) * t;
+    const int keys = a.window > 0 && a.window + a.keep_first < d->c.max_ctx ? a.window + a.keep_first : d->c.max_ctx, most = (keys / 32 + 3) / 4;
+    int splits = (2 * device_cus() + wgs - 1) / wgs;
+    if (splits > most) splits = most;
+    if (splits > 64) splits = 64;
+    while (splits > 1 && (size_t)t * a.heads * splits * (a.vdim_p + 4) > d->b.partial_elems) --splits;
+    a.n_splits = splits < 1 ? 1 : splits;
+    a.partial = d->b.partial;
+  }
+  return chatts_window_attend(&a, s);
+}
+
+static ChattsMoeArgs mix_moe_args(const ChattsMixDecoder* d, const ChattsMixLayer& l, int t) {
+  const ChattsMixBuffers& b = d->b;
+  ChattsMoeArgs a = l.moe;
+  a.logits = b.moe_logits; a.ld_logits = l.router_n;
+  a.h = second_norm(d, l, t);
+  if (!d->c.exact) a.h.f32 = nullptr;
+  a.rows = b.rows; a.n_rows = t; a.exact = d->c.exact;
+  a.ids = b.moe_ids; a.place = b.moe_place; a.order = b.moe_order; a.offsets = b.moe_offsets; a.tiles = b.moe_tiles;
+  a.weight = b.moe_weight; a.kept = b.moe_kept; a.y = b.moe_y;
+  a.act = ChattsOperand{};
+  a.act.ld = a.ff_p;
+  if (d->c.exact) a.act.f32 = b.act_f32;
+  else { a.act.hi = b.act_hi; a.act.lo = b.act_lo; }
+  return a;
+}
+
+// x += what the experts of `moe` owe it; then the norms of `next` (or its joined input)
+static int mix_pair_norm(const ChattsMixDecoder* d, int t, const ChattsMixLayer* moe, const float* w1, const float* w2, const ChattsOperand& out1, const ChattsOperand& out2,
+                         bool join, const ChattsMixLayer* shift, float* prev, chatts_stream_t s) {
+  ChattsPairNormArgs a{};
+  a.x = d->b.x; a.t = t; a.width = d->c.width; a.ldx = d->c.width_p; a.groups = d->c.norm_groups; a.eps = d->c.eps;
+  if (moe) {
+    a.y = d->b.moe_y; a.place = d->b.moe_place; a.weight = d->b.moe_weight; a.kept = d->b.moe_kept; a.top = moe->moe.top;
+    a.h = linear_form(second_norm(d, *moe, t));
+  }
+  if (join) a.x0 = d->b.x0;
+  a.w1 = w1; a.w2 = w2; a.out1 = out1; a.out2 = out2;
+  if (shift) {
+    a.n_mix = shift->n_mix; a.mu = shift->mu; a.mix = shift_operand(d, t, 0); a.mix_stride = d->b.mix_stride; a.prev = prev; a.rows = d->b.rows;
+  }
+  return chatts_pair_norm(&a, s);
+}
+
+static int mix_parallel_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, const ChattsSpan* spans, int n_spans, bool single, chatts_stream_t s) {
+  const ChattsMixConfig& c = d->c;
+  const int wp = c.width_p;
+  const ChattsOperand none{}, X = f32_out(d->b.x, wp);
+  int rc;
+  {
+    ChattsEmbedPairArgs e{};
+    e.tokens = tokens; e.rows = d->b.rows; e.t = t; e.single = single; e.width_p = wp; e.vocab = (int)c.vocab;
+    e.embed = d->b.embed; e.scale = c.embed_scale; e.bigram = d->b.bigram; e.buckets = c.bigram_buckets; e.mul_prev = c.bigram_prev; e.mul_cur = c.bigram_cur;
+    e.prev = d->b.prev_token; e.x = d->b.x; e.x0 = d->b.x0;
+    if ((rc = chatts_embed_pair(&e, s)) != 0) return rc;
+  }
+  const ChattsMixLayer* owed = nullptr;      // the layer whose experts' outputs x still misses
+  for (int r = 0; r < c.n_runs; ++r) {
+    const ChattsMixRun& run = d->runs[r];
+    const ChattsMixLayer& l = d->layers[run.layer];
+    if (run.join) {
+      const ChattsOperand J = operand(d, true, t, 2 * wp);
+      if ((rc = mix_pair_norm(d, t, owed, nullptr, nullptr, J, none, true, nullptr, nullptr, s)) != 0) return rc;
+      owed = nullptr;
+      if ((rc = mix_linear(d, J, run.join, run.join_t, t, wp, 2 * wp, CHATTS_EPI_NONE, X, s)) != 0) return rc;
+    }
+    const bool shift = l.n_mix > 0, ff = l.ff_kind != CHATTS_FF_NONE;
+    const ChattsOperand A = shift && !single ? f32_out(d->b.h, wp) : operand(d, false, t, wp), N = second_norm(d, l, t);
+    if ((rc = mix_pair_norm(d, t, owed, l.norm1, ff ? l.norm2 : nullptr, A, N, false, shift && single ? &l : nullptr, run.ring, s)) != 0) return rc;
+    owed = nullptr;
+    if (shift) {
+      if (!single) {
+        ChattsTokenShiftArgs a{};
+        a.h = d->b.h; a.t = t; a.ldx = wp; a.n_mix = l.n_mix; a.mu = l.mu; a.mix = shift_operand(d, t, 0); a.mix_stride = d->b.mix_stride; a.prev = run.ring;
+        a.rows = d->b.rows;
+        if ((rc = chatts_token_shift(&a, s)) != 0) return rc;
+      }
+      for (int i = 0; i < l.n_mix; ++i) {
+        const size_t at = (size_t)l.mix_row[i] * wp;
+        if ((rc = mix_linear(d, shift_operand(d, t, i), l.in + at, l.mix_t[i], t, l.mix_row[i + 1] - l.mix_row[i], wp, CHATTS_EPI_NONE,
+                             f32_out(d->b.proj + l.mix_row[i], l.in_n), s)) != 0) return rc;
+      }
+    } else if ((rc = mix_linear(d, A, l.in, l.in_t, t, l.in_n, wp, CHATTS_EPI_NONE, f32_out(d->b.proj, l.in_n), s)) != 0) {
+      return rc;
+    }
+    const ChattsOperand B = operand(d, true, t, l.out_k);
+    rc = l.kind == CHATTS_MIX_WINDOW ? mix_window(d, l, run, t, spans, n_spans, single, B, s) : mix_recur(d, l, run, t, n_spans, single, B, s);
+    if (rc) return rc;
+    if ((rc = mix_linear(d, B, l.out, l.out_t, t, wp, l.out_k, CHATTS_EPI_RESID, X, s)) != 0) return rc;
+    if (l.ff_kind == CHATTS_FF_CLAMPGLU) {
+      const ChattsOperand F = operand(d, true, t, l.ff);
+      if ((rc = mix_linear(d, linear_form(N), l.up, l.up_t, t, 2 * l.ff, wp, CHATTS_EPI_CLAMPGLU, F, s, l.glu_limit, l.glu_alpha)) != 0) return rc;
+      if ((rc = mix_linear(d, F, l.down, l.down_t, t, wp, l.ff, CHATTS_EPI_RESID, X, s)) != 0) return rc;
+    } else if (l.ff_kind == CHATTS_FF_MOE) {
+      StageRange stage("chatts.mix.experts");
+      if ((rc = mix_linear(d, linear_form(N), l.router, l.router_t, t, l.router_n, wp, CHATTS_EPI_NONE, f32_out(d->b.moe_logits, l.router_n), s)) != 0) return rc;
+      const ChattsMoeArgs m = mix_moe_args(d, l, t);
+      if ((rc = chatts_moe_route(&m, s)) != 0) return rc;
+      if ((rc = chatts_moe_experts(&m, s)) != 0) return rc;
+      owed = &l;
+    }
+  }
+  if (owed) return mix_pair_norm(d, t, owed, nullptr, nullptr, none, none, false, nullptr, nullptr, s);
+  return CHATTS_OK;
+}
+
 static int mix_norm(const ChattsMixDecoder* d, int t, const float* y, const float* post, const float* add, const float* pre, const ChattsOperand& out,
                     chatts_stream_t s) {
   ChattsResidualNormArgs a{};
@@ -266,6 +451,7 @@ extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens,
     CHATTS_REQUIRE(rows == t, CHATTS_E_SHAPE, "mixdec_forward: segments hold %d of %d rows", rows, t);
   }
   StageRange stage(single ? "chatts.mix.decode" : "chatts.mix.prefill");
+  if (d->layers[0].parallel) return mix_parallel_forward(d, tokens, t, spans, n_spans, single != 0, s);
   int rc;
   if ((rc = chatts_embed_token_batched(tokens, t, d->b.embed, 0, c.vocab, c.width_p, d->b.x, s)) != 0) return rc;
   const ChattsOperand A = operand(d, false, t, c.width_p), Y = f32_out(d->b.y, c.width_p);
@@ -300,18 +486,27 @@ extern "C" int chatts_mixdec_logits(ChattsMixDecoder* d, const int32_t* index, i
   CHATTS_REQUIRE(n >= 0 && n <= c.t_max, CHATTS_E_SHAPE, "mixdec_logits: %d rows", n);
   if (n == 0) return CHATTS_OK;
   StageRange stage("chatts.mix.logits");
-  ChattsResidualNormArgs a{};
-  a.x = d->b.x;
+  const float* x = d->b.x;
   if (index) {
     hipLaunchKernelGGL(gather_rows_kernel, dim3(n), dim3(256), 0, as_stream(s), d->b.x, index, d->b.y, c.width_p);
     CHATTS_CHECK_LAUNCH("gather_rows");
-    a.x = d->b.y;
+    x = d->b.y;
   }
-  a.pre_w = d->b.final_norm;
-  a.out = operand(d, false, n, c.width_p);
-  a.t = n; a.width = c.width; a.ldx = a.ldy = c.width_p; a.eps = c.eps;
-  if (const int rc = chatts_residual_norm(&a, s)) return rc;
-  return mix_linear(d, a.out, d->b.head, d->b.head_t, n, (int)c.vocab_p, c.width_p, CHATTS_EPI_NONE, f32_out(logits, (int)c.vocab_p), s);
+  const ChattsOperand A = operand(d, false, n, c.width_p);
+  int rc;
+  if (d->layers[0].parallel) {
+    ChattsPairNormArgs a{};
+    a.x = const_cast<float*>(x); a.t = n; a.width = c.width; a.ldx = c.width_p; a.groups = c.norm_groups; a.eps = c.eps;
+    a.w1 = d->b.final_norm; a.out1 = A;
+    rc = chatts_pair_norm(&a, s);
+  } else {
+    ChattsResidualNormArgs a{};
+    a.x = const_cast<float*>(x); a.pre_w = d->b.final_norm; a.out = A;
+    a.t = n; a.width = c.width; a.ldx = a.ldy = c.width_p; a.eps = c.eps;
+    rc = chatts_residual_norm(&a, s);
+  }
+  if (rc) return rc;
+  return mix_linear(d, A, d->b.head, d->b.head_t, n, (int)c.vocab_p, c.width_p, CHATTS_EPI_NONE, f32_out(logits, (int)c.vocab_p), s);
 }
 
 extern "C" int chatts_mixdec_decode(ChattsMixDecoder* d, int batch, const int64_t* token, const int32_t* pos, float* logits, chatts_stream_t s) {

@@ -1,0 +1,574 @@
+// window.hip - attention over paged keys and values with grouped heads: per-head RMS norms of queries and keys, an optional sliding window that keeps
+// a sequence's first tokens, an optional sink (one more term exp(0) in the denominator), an optional output gate.
+//   window_prep_kernel      norms; queries as an operand, keys and values into their pages
+//   window_attend_kernel    one row and query head per workgroup, vector units: 32-bit runs, head sizes beyond the matrix kernels
+//   window_decode_kernel    one row: the query heads of a key head share its tiles on the matrix pipe; tiles spread over waves and workgroups
+//   window_prefill_kernel   flash attention for segments of many rows
+// Pages: keys [page][kv head][token][dim_p], values [page][kv head][token][vdim_p]; a page holds a multiple of 64 tokens, so a tile of up to 64
+// keys of a head is contiguous memory.
+#include "gemm_common.h"
+
+namespace chatts {
+
+typedef short w16x4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) w16x4* lds_w16x4;
+
+__device__ __forceinline__ size_t window_tile(const ChattsWindowArgs& p, int slot, int hk, int key) {      // row number of a key in its pool
+  const int blk = p.table[(size_t)slot * p.table_stride + (key >> p.log_block)];
+  return (((size_t)blk * p.kv_heads + hk) << p.log_block) + (key & ((1 << p.log_block) - 1));
+}
+// tiles of K keys that a row at `pos` (or rows pos_lo .. pos) sees: the first `kept`, then from `from` to the tile of pos
+struct WindowTiles {
+  int kept, from, last;
+  __device__ __forceinline__ WindowTiles(const ChattsWindowArgs& p, int pos_lo, int pos, int log_tile) {
+    last = pos >> log_tile;
+    if (p.window <= 0) { kept = 0; from = 0; return; }
+    const int w = pos_lo - p.window + 1;
+    from = (w > 0 ? w : 0) >> log_tile;
+    kept = (p.keep_first + (1 << log_tile) - 1) >> log_tile;
+    if (kept > last + 1) kept = last + 1;
+    if (from < kept) from = kept;
+  }
+  __device__ __forceinline__ int count() const { return kept + last + 1 - from; }
+  __device__ __forceinline__ int tile(int i) const { return i < kept ? i : from + i - kept; }
+};
+__device__ __forceinline__ bool window_sees(const ChattsWindowArgs& p, int pos, int key) {
+  return key <= pos && (p.window <= 0 || pos - key < p.window || key < p.keep_first);
+}
+__device__ __forceinline__ float window_gate(const ChattsWindowArgs& p, size_t row, int at) {
+  return p.off_gate < 0 ? 1.f : sigmoid_f(p.proj[row * p.ld_proj + p.off_gate + at]);
+}
+
+template <typename CT>
+__device__ __forceinline__ CT to_page(float v) {
+  if constexpr (sizeof(CT) == 4) return v;
+  else return __builtin_bit_cast(uint16_t, (__bf16)v);
+}
+
+// grid (rows): a wave takes heads [q | k | v] in turn
+template <typename CT>
+__global__ __launch_bounds__(256) void window_prep_kernel(ChattsWindowArgs p) {
+  const int row = blockIdx.x, lane = threadIdx.x & 63;
+  const ChattsRow R = p.rows[row];
+  if (R.pos < 0) return;
+  const int H = p.heads, G = p.kv_heads;
+  const float* pr = p.proj + (size_t)row * p.ld_proj;
+  for (int e = threadIdx.x >> 6; e < H + 2 * G; e += 4) {
+    const bool value = e >= H + G;
+    const int hk = e < H ? 0 : (value ? e - H - G : e - H), n = value ? p.vdim : p.dim, np = value ? p.vdim_p : p.dim_p;
+    const float* x = pr + (e < H ? p.off_q + e * p.dim : (value ? p.off_v + hk * p.vdim : p.off_k + hk * p.dim));
+    float v[4], f = 1.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = j * 64 + lane < n ? x[j * 64 + lane] : 0.f;
+    const float* w = value ? nullptr : (e < H ? p.q_norm : p.k_norm);
+    if (w) f = 1.0f / sqrtf(wave_sum((v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3])) / (float)n + p.eps);
+    CT* dst = nullptr;
+    if (e >= H) dst = reinterpret_cast<CT*>(value ? p.vcache : p.kcache) + window_tile(p, R.slot, hk, R.pos) * np;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int c = j * 64 + lane;
+      if (c >= np) break;
+      const float y = w && c < n ? v[j] * f * w[c] : v[j];
+      if (dst) dst[c] = to_page<CT>(y);
+      else store_operand(p.q, row, e * p.dim_p + c, y);
+    }
+  }
+}
+
+// ---- vector units: grid (heads, rows) ----
+template <typename CT>
+__global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, hk = h / (p.heads / p.kv_heads);
+  const ChattsRow R = p.rows[row];
+  if (R.pos < 0) return;
+  float* sq = sm;              // [dim_p]
+  float* sc = sq + p.dim_p;    // [64] scores, then weights
+  for (int i = tid; i < p.dim_p; i += 256) {
+    const size_t at = (size_t)row * p.q.ld + h * p.dim_p + i;
+    sq[i] = p.q.f32 ? p.q.f32[at] : bf16_to_f32(p.q.hi[at]) + (p.q.lo ? bf16_to_f32(p.q.lo[at]) : 0.f);
+  }
+  float m = p.sink ? 0.f : -INFINITY, l = p.sink ? 1.f : 0.f, o = 0.f;      // column tid
+  const WindowTiles T(p, R.pos, R.pos, 6);
+  const int n = T.count();
+  for (int i = 0; i < n; ++i) {
+    __syncthreads();
+    const int k0 = T.tile(i) * 64;
+    const size_t at = window_tile(p, R.slot, hk, k0);
+    const CT* kt = reinterpret_cast<const CT*>(p.kcache) + at * p.dim_p;
+    const CT* vt = reinterpret_cast<const CT*>(p.vcache) + at * p.vdim_p;
+    const int key = tid >> 2, part = tid & 3;
+    const bool sees = window_sees(p, R.pos, k0 + key);
+    float d = 0.f;
+    if (sees)
+      for (int c = part; c < p.dim_p; c += 4) {
+        float kv;
+        if constexpr (sizeof(CT) == 4) kv = kt[(size_t)key * p.dim_p + c];
+        else kv = bf16_to_f32(kt[(size_t)key * p.dim_p + c]);
+        d += kv * sq[c];
+      }
+    d += lane_xor1(d);
+    d += lane_xor2(d);
+    if (part == 0) sc[key] = sees ? d * p.scale : -INFINITY;
+    __syncthreads();
+    const float s = sc[tid & 63];
+    const float mn = fmaxf(m, wave_max(s)), safe = mn == -INFINITY ? 0.f : mn;
+    const float e = expf(s - safe), alpha = expf(m - safe);
+    l = l * alpha + wave_sum(e);
+    m = mn;
+    __syncthreads();
+    if (tid < 64) sc[tid] = e;
+    __syncthreads();
+    if (tid < p.vdim) {
+      const int lim = R.pos + 1 - k0 < 64 ? R.pos + 1 - k0 : 64;
+      o *= alpha;
+      for (int k = 0; k < lim; ++k) {
+        const float w = sc[k];
+        if (w == 0.f) continue;      // (uniform)
+        if constexpr (sizeof(CT) == 4) o += w * vt[(size_t)k * p.vdim_p + tid];
+        else o += w * bf16_to_f32(vt[(size_t)k * p.vdim_p + tid]);
+      }
+    }
+  }
+  if (tid < p.vdim) store_operand(p.out, row, h * p.vdim + tid, o / l * window_gate(p, row, h * p.vdim + tid));
+}
+
+// ---- one row on the matrix pipe: grid (splits, kv heads * head tiles, rows), 4 waves ----
+// A wave walks tiles of 32 keys on its own (tiles 4 split + wave, ...): S^T = K Q^T with the key rows straight from memory as A fragments, so that a
+// lane ends up with 8 scores of one head (column = lane & 15); O^T = V^T P^T with V through a private piece of LDS and transposing reads - its B
+// fragment IS the 8 probabilities of the lane (K slot 8 g + j = key 4 g + j, j < 4, or 16 + 4 g + j - 4, on both sides).  The waves' softmaxes meet once.
+template <int NK, int NV>      // dim_p <= 32 NK, vdim_p <= 16 NV
+__global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const int split = blockIdx.x, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const ChattsRow R = p.rows[row];
+  if (R.pos < 0) return;
+  const int group = p.heads / p.kv_heads, htiles = (group + 15) / 16, hk = blockIdx.y / htiles, h0 = (blockIdx.y - hk * htiles) * 16;
+  const int nk = p.dim_p >> 5, nv = p.vdim_p >> 4, ldv = p.vdim_p + 16;
+  const int hl = h0 + fr < group ? h0 + fr : group - 1, head = hk * group + hl;
+  uint16_t* vs = reinterpret_cast<uint16_t*>(smem) + wave * 32 * ldv;
+  bf16x8_t q[NK];
+#pragma unroll
+  for (int k = 0; k < NK; ++k)
+    if (k < nk) q[k] = *reinterpret_cast<const bf16x8_t*>(p.q.hi + (size_t)row * p.q.ld + head * p.dim_p + k * 32 + fg * 8);
+  const WindowTiles T(p, R.pos, R.pos, 5);
+  const int n = T.count(), stride = 4 * p.n_splits;
+  float m = -INFINITY, l = 0.f;
+  f32x4 o[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) o[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const float scale2 = p.scale * 1.44269504088896341f;
+  constexpr int VP = (NV * 32 * 16 + 511) / 512;      // 16-byte pieces of a value tile per lane
+  const int vc = p.vdim_p >> 3, pieces = 32 * vc;
+  for (int i = split * 4 + wave; i < n; i += stride) {
+    const int k0 = T.tile(i) * 32;
+    const size_t at = window_tile(p, R.slot, hk, k0);
+    const uint16_t* kt = reinterpret_cast<const uint16_t*>(p.kcache) + at * p.dim_p;
+    const uint16_t* vt = reinterpret_cast<const uint16_t*>(p.vcache) + at * p.vdim_p;
+    bf16x8_t kf[2][NK];
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      if (k < nk) {
+        kf[0][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)fr * p.dim_p + k * 32 + fg * 8);
+        kf[1][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)(16 + fr) * p.dim_p + k * 32 + fg * 8);
+      }
+    u32x4 rv[VP];
+#pragma unroll
+    for (int e = 0; e < VP; ++e) {
+      const int x = e * 64 + lane;
+      const int key = x / vc;
+      rv[e] = (u32x4){0u, 0u, 0u, 0u};
+      if (x < pieces && k0 + key <= R.pos) rv[e] = *reinterpret_cast<const u32x4*>(vt + (size_t)x * 8);      // (a row never written may hold anything)
+    }
+    f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      if (k < nk) {
+        s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0][k], q[k], s[0], 0, 0, 0);
+        s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][k], q[k], s[1], 0, 0, 0);
+      }
+    float v[8], mx = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int key = k0 + (j >> 2) * 16 + fg * 4 + (j & 3);
+      v[j] = window_sees(p, R.pos, key) ? s[j >> 2][j & 3] * scale2 : -INFINITY;
+      mx = fmaxf(mx, v[j]);
+    }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx), safe = mn == -INFINITY ? 0.f : mn, alpha = __builtin_amdgcn_exp2f(m - safe);
+    m = mn;
+    bf16x8_t pf;
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float e = __builtin_amdgcn_exp2f(v[j] - safe);
+      sum += e;
+      pf[j] = (__bf16)e;
+    }
+    l = l * alpha + sum;
+#pragma unroll
+    for (int e = 0; e < VP; ++e) {
+      const int x = e * 64 + lane, key = x / vc;
+      if (x < pieces) *reinterpret_cast<u32x4*>(vs + key * ldv + (x - key * vc) * 8) = rv[e];
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    const uint16_t* t0 = vs + (fg * 4 + (fr >> 2)) * ldv + (fr & 3) * 4;
+#pragma unroll
+    for (int f = 0; f < NV; ++f)
+      if (f < nv) {
+        union { w16x4 h[2]; bf16x8_t v; } a;
+        a.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + f * 16));
+        a.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + 16 * ldv + f * 16));
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[f][r] *= alpha;
+        o[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pf, o[f], 0, 0, 0);
+      }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // this tile has been read before the next one is written
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  // the four waves meet: [wave][16 heads][vdim_p + 4]
+  __syncthreads();
+  float* part = reinterpret_cast<float*>(smem);
+  const int ldp = p.vdim_p + 4;
+#pragma unroll
+  for (int f = 0; f < NV; ++f)
+    if (f < nv) *reinterpret_cast<f32x4*>(part + (wave * 16 + fr) * ldp + f * 16 + fg * 4) = o[f];
+  if (fg == 0) {
+    part[(wave * 16 + fr) * ldp + p.vdim_p] = m;
+    part[(wave * 16 + fr) * ldp + p.vdim_p + 1] = l;
+  }
+  __syncthreads();
+  const bool whole = p.n_splits == 1;
+  const int hn = group - h0 < 16 ? group - h0 : 16;
+  for (int x = tid; x < hn * p.vdim_p; x += 256) {
+    const int hh = x / p.vdim_p, c = x - hh * p.vdim_p;
+    const int hd = hk * group + h0 + hh;
+    float mw[4], M = whole && p.sink ? 0.f : -INFINITY;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) { mw[w] = part[(w * 16 + hh) * ldp + p.vdim_p]; M = fmaxf(M, mw[w]); }
+    const float safe = M == -INFINITY ? 0.f : M;
+    float L = whole && p.sink ? __builtin_amdgcn_exp2f(-safe) : 0.f, acc = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float f = __builtin_amdgcn_exp2f(mw[w] - safe);
+      L += f * part[(w * 16 + hh) * ldp + p.vdim_p + 1];
+      acc += f * part[(w * 16 + hh) * ldp + c];
+    }
+    if (whole) {
+      if (c < p.vdim) store_operand(p.out, row, hd * p.vdim + c, acc / L * window_gate(p, row, hd * p.vdim + c));
+    } else {
+      float* dst = p.partial + (((size_t)row * p.heads + hd) * p.n_splits + split) * ldp;
+      dst[c] = acc;
+      if (c == 0) { dst[p.vdim_p] = M; dst[p.vdim_p + 1] = L; }
+    }
+  }
+}
+
+// merge of the splits: grid (heads, rows)
+__global__ __launch_bounds__(128) void window_merge_kernel(ChattsWindowArgs p) {
+  __shared__ float w[64];
+  const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, ld = p.vdim_p + 4;
+  if (p.rows[row].pos < 0) return;
+  const float* part = p.partial + ((size_t)row * p.heads + h) * p.n_splits * ld;
+  if (tid < 64) {
+    const float m = tid < p.n_splits ? part[(size_t)tid * ld + p.vdim_p] : -INFINITY, l = tid < p.n_splits ? part[(size_t)tid * ld + p.vdim_p + 1] : 0.f;
+    float M = wave_max(m);
+    if (p.sink) M = fmaxf(M, 0.f);
+    const float f = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - M);
+    const float L = wave_sum(f * l) + (p.sink ? __builtin_amdgcn_exp2f(-M) : 0.f);
+    w[tid] = f / L;
+  }
+  __syncthreads();
+  for (int c = tid; c < p.vdim; c += 128) {
+    float o = 0.f;
+#pragma unroll 4
+    for (int s = 0; s < p.n_splits; ++s) o += w[s] * part[(size_t)s * ld + c];
+    store_operand(p.out, row, h * p.vdim + c, o * window_gate(p, row, h * p.vdim + c));
+  }
+}
+
+// ---- many rows: grid (heads, query tiles of 128, spans); a wave owns 32 queries of one head, 64 keys per step ----
+// S^T = K Q^T, O^T = V^T P^T as above; keys and values of a tile are staged by all waves, the next tile's requested while this one is multiplied.
+template <int NK, int NV, int OCC>      // dim_p <= 32 NK, vdim_p <= 16 NV
+__global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowArgs p) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const ChattsSpan sp = p.spans[blockIdx.z];
+  const int qt0 = (gridDim.y - 1 - blockIdx.y) * 128, h = blockIdx.x, hk = h / (p.heads / p.kv_heads);
+  if (qt0 >= sp.t) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const int dq = p.dim_p, ldk = dq + 8, ldv = p.vdim_p + 16, nk = dq >> 5, nv = p.vdim_p >> 4;
+  uint16_t* ks = reinterpret_cast<uint16_t*>(smem);      // [64][ldk]
+  uint16_t* vs = ks + 64 * ldk;                          // [64][ldv]
+  const int qlast = qt0 + 127 < sp.t ? qt0 + 127 : sp.t - 1;
+  const WindowTiles T(p, sp.pos0 + qt0, sp.pos0 + qlast, 6);
+  const int n = T.count(), plast = sp.pos0 + qlast;
+  const int q0 = qt0 + wave * 32, w0 = sp.pos0 + q0, w1 = w0 + 31 < plast ? w0 + 31 : plast;      // this wave's positions
+  bf16x8_t q[2][NK];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    int r = q0 + u * 16 + fr;
+    if (r > sp.t - 1) r = sp.t - 1;
+    const uint16_t* src = p.q.hi + (size_t)(sp.row0 + r) * p.q.ld + h * dq + fg * 8;
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      if (k < nk) q[u][k] = *reinterpret_cast<const bf16x8_t*>(src + k * 32);
+  }
+  f32x4 o[NV][2];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) o[i][0] = o[i][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const float m0 = p.sink ? 0.f : -INFINITY, l0 = p.sink && fg == 0 ? 1.f : 0.f;
+  float m[2] = {m0, m0}, l[2] = {l0, l0};
+  const float scale2 = p.scale * 1.44269504088896341f;      // scores in base 2
+  constexpr int KP = NK, VP = (NV + 1) / 2;
+  u32x4 rk[KP], rv[VP];
+  const int kc = dq >> 3, vc = p.vdim_p >> 3;
+  auto fetch = [&](int i) __attribute__((always_inline)) {
+    const int k0 = T.tile(i) * 64;
+    const size_t at = window_tile(p, sp.slot, hk, k0);
+    const uint16_t* kt = reinterpret_cast<const uint16_t*>(p.kcache) + at * dq;
+    const uint16_t* vt = reinterpret_cast<const uint16_t*>(p.vcache) + at * p.vdim_p;
+#pragma unroll
+    for (int e = 0; e < KP; ++e) {
+      const int x = e * 256 + tid;
+      if (x < 64 * kc) rk[e] = *reinterpret_cast<const u32x4*>(kt + (size_t)x * 8);
+    }
+#pragma unroll
+    for (int e = 0; e < VP; ++e) {
+      const int x = e * 256 + tid;
+      rv[e] = (u32x4){0u, 0u, 0u, 0u};
+      if (x < 64 * vc && k0 + x / vc <= plast) rv[e] = *reinterpret_cast<const u32x4*>(vt + (size_t)x * 8);      // (a row never written may hold anything)
+    }
+  };
+  fetch(0);
+  for (int i = 0; i < n; ++i) {
+    __syncthreads();
+#pragma unroll
+    for (int e = 0; e < KP; ++e) {
+      const int x = e * 256 + tid, r = x / kc;
+      if (x < 64 * kc) *reinterpret_cast<u32x4*>(ks + r * ldk + (x - r * kc) * 8) = rk[e];
+    }
+#pragma unroll
+    for (int e = 0; e < VP; ++e) {
+      const int x = e * 256 + tid, r = x / vc;
+      if (x < 64 * vc) *reinterpret_cast<u32x4*>(vs + r * ldv + (x - r * vc) * 8) = rv[e];
+    }
+    __syncthreads();
+    if (i + 1 < n) fetch(i + 1);
+    const int k0 = T.tile(i) * 64;
+    // (uniform per wave) nothing of the tile is visible to this wave's queries
+    if (k0 > w1 || w0 > w1 || (p.window > 0 && w0 - (k0 + 63) >= p.window && k0 >= p.keep_first)) continue;
+    const bool edge = k0 + 63 > w0 || (p.window > 0 && w1 - k0 >= p.window && k0 + 63 >= p.keep_first);      // some key is hidden from some query
+    f32x4 s[4][2];      // [16-key block][query block]
+#pragma unroll
+    for (int a = 0; a < 4; ++a) s[a][0] = s[a][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const uint16_t* kb = ks + fr * ldk + fg * 8;
+    {
+      bf16x8_t kf[2][4];
+      auto request = [&](int k, bf16x8_t (&dst)[4]) __attribute__((always_inline)) {
+#pragma unroll
+        for (int a = 0; a < 4; ++a) dst[a] = *reinterpret_cast<const bf16x8_t*>(kb + a * 16 * ldk + k * 32);
+      };
+      request(0, kf[0]);
+#pragma unroll
+      for (int k = 0; k < NK; ++k)
+        if (k < nk) {
+          if (k + 1 < NK && k + 1 < nk) request(k + 1, kf[(k + 1) & 1]);
+          __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+          for (int a = 0; a < 4; ++a) {
+            s[a][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k & 1][a], q[0][k], s[a][0], 0, 0, 0);
+            s[a][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[k & 1][a], q[1][k], s[a][1], 0, 0, 0);
+          }
+          __builtin_amdgcn_sched_barrier(0);
+        }
+    }
+    bf16x8_t pf[2][2];      // [32-key group][query block]
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int qpos = w0 + u * 16 + fr;
+      float mx = -INFINITY;
+#pragma unroll
+      for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          float v = s[a][u][r] * scale2;
+          if (edge && !window_sees(p, qpos, k0 + a * 16 + fg * 4 + r)) v = -INFINITY;
+          s[a][u][r] = v;
+          mx = fmaxf(mx, v);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m[u], mx), safe = mn == -INFINITY ? 0.f : mn, alpha = __builtin_amdgcn_exp2f(m[u] - safe);
+      m[u] = mn;
+      float sum = 0.f;
+#pragma unroll
+      for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = __builtin_amdgcn_exp2f(s[a][u][r] - safe);
+          sum += e;
+          pf[a >> 1][u][(a & 1) * 4 + r] = (__bf16)e;
+        }
+      l[u] = l[u] * alpha + sum;
+      if (__any(alpha != 1.0f)) {
+#pragma unroll
+        for (int f = 0; f < NV; ++f)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o[f][u][r] *= alpha;
+      }
+    }
+    {
+      // transposing reads: lane -> rows 4 g + (fr >> 2) (and + 16) of a 32-key group, 4 columns of the fragment's 16
+      const uint16_t* t0 = vs + (fg * 4 + (fr >> 2)) * ldv + (fr & 3) * 4;
+      union Tr { w16x4 h[2]; bf16x8_t v; };
+      Tr vf[2][2];
+      auto request = [&](int f, Tr (&dst)[2]) __attribute__((always_inline)) {
+#pragma unroll
+        for (int g = 0; g < 2; ++g) {
+          dst[g].h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + g * 32 * ldv + f * 16));
+          dst[g].h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + (g * 32 + 16) * ldv + f * 16));
+        }
+      };
+      request(0, vf[0]);
+#pragma unroll
+      for (int f = 0; f < NV; ++f)
+        if (f < nv) {
+          if (f + 1 < NV && f + 1 < nv) request(f + 1, vf[(f + 1) & 1]);
+          __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+          for (int g = 0; g < 2; ++g) {
+            o[f][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[f & 1][g].v, pf[g][0], o[f][0], 0, 0, 0);
+            o[f][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[f & 1][g].v, pf[g][1], o[f][1], 0, 0, 0);
+          }
+          __builtin_amdgcn_sched_barrier(0);
+        }
+    }
+  }
+  const bool quads = p.vdim % 4 == 0 && (p.off_gate < 0 || p.off_gate % 4 == 0) && p.out.ld % 4 == 0;
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int r = q0 + u * 16 + fr;
+    float L = l[u];
+    L += __shfl_xor(L, 16, 64);
+    L += __shfl_xor(L, 32, 64);
+    if (r >= sp.t) continue;
+    const float inv = 1.0f / L;
+    const size_t row = sp.row0 + r;
+#pragma unroll
+    for (int f = 0; f < NV; ++f) {
+      const int c = f * 16 + fg * 4, at = h * p.vdim + c;
+      if (f >= nv || c >= p.vdim) continue;
+      if (quads) {
+        f32x4 g = {1.f, 1.f, 1.f, 1.f};
+        if (p.off_gate >= 0) {
+          g = *reinterpret_cast<const f32x4*>(p.proj + row * p.ld_proj + p.off_gate + at);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) g[k] = sigmoid_f(g[k]);
+        }
+        const float v[4] = {o[f][u][0] * inv * g[0], o[f][u][1] * inv * g[1], o[f][u][2] * inv * g[2], o[f][u][3] * inv * g[3]};
+        store_operand4(p.out, row, at, v);
+      } else {
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+          if (c + k < p.vdim) store_operand(p.out, row, at + k, o[f][u][k] * inv * window_gate(p, row, at + k));
+      }
+    }
+  }
+}
+
+static int check_window(const ChattsWindowArgs* a, const char* who) {
+  CHATTS_REQUIRE(a && a->proj && a->kcache && a->vcache && a->table && a->rows && a->q_norm && a->k_norm && (a->q.f32 || a->q.hi), CHATTS_E_BADARG, "%s: null pointer", who);
+  CHATTS_REQUIRE(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim >= 1 && a->dim <= a->dim_p && a->dim_p <= 256 && a->dim_p % 32 == 0 &&
+                     a->vdim >= 1 && a->vdim <= a->vdim_p && a->vdim_p <= 256 && a->vdim_p % 16 == 0, CHATTS_E_SHAPE, "%s: heads %d / %d of %d, %d (at most 256)", who,
+                 a->heads, a->kv_heads, a->dim, a->vdim);
+  CHATTS_REQUIRE(a->off_q >= 0 && a->off_k >= 0 && a->off_v >= 0 && a->off_q + a->heads * a->dim <= a->ld_proj && a->off_k + a->kv_heads * a->dim <= a->ld_proj &&
+                     a->off_v + a->kv_heads * a->vdim <= a->ld_proj && a->off_gate + a->heads * a->vdim <= a->ld_proj && a->ld_proj % 4 == 0, CHATTS_E_SHAPE,
+                 "%s: column blocks", who);
+  CHATTS_REQUIRE(a->n_rows >= 0 && a->n_rows <= 65535, CHATTS_E_SHAPE, "%s: %d rows", who, a->n_rows);
+  CHATTS_REQUIRE(a->log_block >= 6 && a->log_block <= 15 && a->window >= 0 && a->keep_first >= 0, CHATTS_E_SHAPE, "%s: pages of 2^%d tokens, window %d, kept %d", who,
+                 a->log_block, a->window, a->keep_first);
+  CHATTS_REQUIRE((((uintptr_t)a->kcache | (uintptr_t)a->vcache | (uintptr_t)a->proj) % 16) == 0 && a->q.ld >= a->heads * a->dim_p && a->q.ld % 8 == 0 &&
+                     (a->cache_f32 ? a->q.f32 != nullptr : a->q.hi != nullptr), CHATTS_E_SHAPE, "%s: alignment / queries", who);
+  return CHATTS_OK;
+}
+static bool window_out_ok(const ChattsWindowArgs* a) { return (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim; }
+
+template <typename K>
+static int window_lds(K kernel, size_t bytes, bool& done) {
+  if (!done) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+    CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "window attention: cannot reserve LDS: %s", hipGetErrorString(e));
+    done = true;
+  }
+  return CHATTS_OK;
+}
+
+template <int NK, int NV>
+static int launch_window_decode(const ChattsWindowArgs* a, hipStream_t s) {
+  static bool done = false;
+  const size_t most = 4 * 16 * (NV * 16 + 4) * 4 > 4 * 32 * (NV * 16 + 16) * 2 ? 4 * 16 * (NV * 16 + 4) * 4 : 4 * 32 * (NV * 16 + 16) * 2;
+  if (const int rc = window_lds(&window_decode_kernel<NK, NV>, most, done)) return rc;
+  const size_t tiles = (size_t)4 * 32 * (a->vdim_p + 16) * 2, meet = (size_t)4 * 16 * (a->vdim_p + 4) * 4;
+  const int group = a->heads / a->kv_heads;
+  hipLaunchKernelGGL((window_decode_kernel<NK, NV>), dim3(a->n_splits, a->kv_heads * ((group + 15) / 16), a->n_rows), dim3(256), tiles > meet ? tiles : meet, s, *a);
+  CHATTS_CHECK_LAUNCH("window_decode");
+  return CHATTS_OK;
+}
+template <int NK, int NV, int OCC>
+static int launch_window_prefill(const ChattsWindowArgs* a, hipStream_t s) {
+  static bool done = false;
+  if (const int rc = window_lds(&window_prefill_kernel<NK, NV, OCC>, (size_t)64 * (NK * 32 + 8 + NV * 16 + 16) * 2, done)) return rc;
+  hipLaunchKernelGGL((window_prefill_kernel<NK, NV, OCC>), dim3(a->heads, (a->longest + 127) / 128, a->n_spans), dim3(256),
+                     (size_t)64 * (a->dim_p + 8 + a->vdim_p + 16) * 2, s, *a);
+  CHATTS_CHECK_LAUNCH("window_prefill");
+  return CHATTS_OK;
+}
+
+}  // namespace chatts
+
+using namespace chatts;
+
+extern "C" int chatts_window_prep(const ChattsWindowArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_window(a, "window_prep")) return rc;
+  if (a->n_rows == 0) return CHATTS_OK;
+  if (a->cache_f32) hipLaunchKernelGGL(window_prep_kernel<float>, dim3(a->n_rows), dim3(256), 0, as_stream(stream), *a);
+  else hipLaunchKernelGGL(window_prep_kernel<uint16_t>, dim3(a->n_rows), dim3(256), 0, as_stream(stream), *a);
+  CHATTS_CHECK_LAUNCH("window_prep");
+  return CHATTS_OK;
+}
+
+extern "C" int chatts_window_can_prefill(int dim_p, int vdim_p) { return dim_p <= 256 && vdim_p <= 256; }
+
+extern "C" int chatts_window_attend(const ChattsWindowArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_window(a, "window_attend")) return rc;
+  CHATTS_REQUIRE(window_out_ok(a), CHATTS_E_BADARG, "window_attend: no output");
+  if (a->n_rows == 0) return CHATTS_OK;
+  hipStream_t s = as_stream(stream);
+  if (a->cache_f32) {
+    hipLaunchKernelGGL(window_attend_kernel<float>, dim3(a->heads, a->n_rows), dim3(256), (size_t)(a->dim_p + 64) * sizeof(float), s, *a);
+    CHATTS_CHECK_LAUNCH("window_attend");
+    return CHATTS_OK;
+  }
+  CHATTS_REQUIRE(a->n_splits >= 1 && a->n_splits <= 64 && (a->n_splits == 1 || a->partial), CHATTS_E_BADARG, "window_attend: %d splits", a->n_splits);
+  int rc;
+  if (a->dim_p <= 64 && a->vdim_p <= 64) rc = launch_window_decode<2, 4>(a, s);
+  else if (a->dim_p <= 128 && a->vdim_p <= 128) rc = launch_window_decode<4, 8>(a, s);
+  else rc = launch_window_decode<8, 16>(a, s);
+  if (rc) return rc;
+  if (a->n_splits > 1) {
+    hipLaunchKernelGGL(window_merge_kernel, dim3(a->heads, a->n_rows), dim3(128), 0, s, *a);
+    CHATTS_CHECK_LAUNCH("window_merge");
+  }
+  return CHATTS_OK;
+}
+
+extern "C" int chatts_window_prefill(const ChattsWindowArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_window(a, "window_prefill")) return rc;
+  CHATTS_REQUIRE(window_out_ok(a) && a->spans && !a->cache_f32, CHATTS_E_BADARG, "window_prefill: bad arguments");
+  if (a->n_rows == 0 || a->n_spans == 0 || a->longest == 0) return CHATTS_OK;
+  if (a->dim_p <= 64 && a->vdim_p <= 64) return launch_window_prefill<2, 4, 2>(a, as_stream(stream));
+  if (a->dim_p <= 128 && a->vdim_p <= 128) return launch_window_prefill<4, 8, 2>(a, as_stream(stream));
+  return launch_window_prefill<8, 16, 1>(a, as_stream(stream));
+}

@@ -1,10 +1,14 @@
 """MixedDecoder - a served model whose layers each name their mixer, run by csrc/mixdec.hip.
 
-A layer is norm1 -> mixer -> norm1b -> residual, then optionally norm2 -> squared-relu feed-forward -> norm2b -> residual.  Mixers:
+A sequential layer is norm1 -> mixer -> norm1b -> residual, then optionally norm2 -> squared-relu feed-forward -> norm2b -> residual; a parallel one adds
+mixer(norm1(x)) + feed-forward(norm2(x)) to x, both norms of the same x in groups (csrc/pair.hip).  Mixers:
   LatentMixer   attention over a paged cache of one latent + one rotated key part per token (csrc/latent.hip)
   DeltaMixer    gated delta rule: a float32 state and a ring of convolution inputs per slot (csrc/delta.hip)
-A design (chatts_amd/fobolix.py) says in which order layers run (config.runs(): a layer may run several times, every run has its own pages or
-state) and maps its tensor names onto LayerWeights.
+  WindowMixer   grouped-head attention over paged keys and values: per-head norms, window, kept first tokens, sink, gate (csrc/window.hip)
+  WkvMixer, MlstmMixer   gated linear recurrences: a float32 state per slot (csrc/recur.hip)
+Feed-forwards of parallel layers: ClampGlu, Experts (csrc/moe.hip).
+A design (chatts_amd/fobolix.py, chatts_amd/medilix.py) says in which order layers run (config.runs(): a layer may run several times, every run has
+its own pages or state) and maps its tensor names onto LayerWeights.
 
 Everything is padded once, at load: widths and feed-forwards to multiples of 64, the stacked input projections block by block, heads to
 what the kernels tile by.  Padding is zero weights, so activations never need clearing.
@@ -71,14 +75,90 @@ class DeltaMixer:
 
 
 @dataclass
+class WindowMixer:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int     # 0: every earlier position
+    keep_first: int
+    sink: bool
+    q: Any
+    k: Any
+    v: Any
+    g: Any          # output gate [heads * vdim, width] or None
+    q_norm: Any
+    k_norm: Any
+    o: Any
+
+
+@dataclass
+class WkvMixer:
+    heads: int
+    dim: int
+    mu: Any         # of r, k, v, g, w
+    r: Any
+    k: Any
+    v: Any
+    g: Any
+    w1: Any
+    w2: Any
+    w0: Any
+    u: Any
+    norm: Any
+    o: Any
+
+
+@dataclass
+class MlstmMixer:
+    heads: int
+    dim: int
+    vdim: int
+    cap: float
+    q: Any
+    k: Any
+    v: Any
+    g: Any
+    i: Any
+    f: Any
+    bias_i: Any
+    bias_f: Any
+    norm: Any
+    o: Any
+
+
+@dataclass
+class ClampGlu:
+    gate: Any
+    up: Any
+    down: Any
+    limit: float
+    alpha: float
+
+
+@dataclass
+class Experts:
+    router: Any         # [experts + identity, width]
+    correction: Any
+    experts: Any        # (gate, up, down) each
+    identity: int
+    top: int
+    groups: int
+    keep: int
+
+
+@dataclass
 class LayerWeights:
     mixer: Any
     norm1: Any
-    norm1b: Any
+    norm1b: Any = None
     norm2: Any = None
     norm2b: Any = None
-    up: Any = None
+    up: Any = None      # squared-relu feed-forward of a sequential layer
     down: Any = None
+    ff: Any = None      # ClampGlu or Experts of a parallel layer
+    parallel: bool = False
 
 
 def _up(n, m):
@@ -160,12 +240,16 @@ class MixedDecoder(SlotModel):
         sd = {}
         for name, shape in config.tensor_shapes(rank_a or big, rank_g or big).items():
             t = torch.randn(shape, generator=gen, device=m.device)
-            if len(shape) == 2 and not name.endswith(".conv") and name != "embed":
+            if len(shape) == 2 and not name.endswith((".conv", ".u")) and name not in ("embed", "bigram"):
                 t *= shape[1] ** -0.5
             if name.endswith(("norm", "norm1", "norm2", "norm1b", "norm2b")):
                 t = 1.0 + 0.1 * t
             if name.endswith("dt_bias"):
                 t = 0.5 * t - 3.0
+            if name.endswith(("mix.w0", "mix.f.b")):
+                t = t + (-4.0 if name.endswith("w0") else 4.0)
+            if ".mu." in name:
+                t = 0.5 + 0.1 * t
             sd[name] = t.to(torch.bfloat16)
         m.load_weights(sd.items())
         return m
@@ -268,6 +352,75 @@ class MixedDecoder(SlotModel):
                                  a2d=self._pieces(m.a2, ra_p), g2d=self._pieces(m.g2, rg_p), ld_a2=ra_p, ld_g2=rg_p,
                                  dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32)).repeat_interleave(m.dim)), norm_w=self._f32(m.norm))
 
+    def _blocks(self, L, blocks, split=False):
+        """stacked input projection of a layer -> {name: first row}; split: every block has an operand of its own"""
+        w, off = self._stack([(n, t, _up(t.shape[0], 64)) for n, t in blocks])
+        L.in_n = w.shape[0]
+        L.w_in, L.in_t = self._mat(w, tile=not split)
+        if split:
+            L.n_mix = len(blocks)
+            for j, (n, _) in enumerate(blocks):
+                L.mix_row[j] = off[n]
+            L.mix_row[len(blocks)] = L.in_n
+            for j in range(len(blocks)):
+                L.mix_t[j] = self._mat(w[L.mix_row[j]:L.mix_row[j + 1]], tile=True)[1] if self.tiled else None
+        return off
+
+    def _window_layer(self, L, m):
+        L.kind = _lib.MIX_WINDOW
+        off = self._blocks(L, [("q", m.q), ("k", m.k), ("v", m.v)] + ([("g", m.g)] if m.g is not None else []))
+        n, dim_p, vdim_p = m.heads * m.vdim, _up(m.dim, 32), _up(m.vdim, 16)
+        L.out_k = _up(n, 64)
+        L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
+        L.window = _lib.WindowArgs(off_q=off["q"], off_k=off["k"], off_v=off["v"], off_gate=off.get("g", -1), heads=m.heads, kv_heads=m.kv_heads, dim=m.dim,
+                                   vdim=m.vdim, dim_p=dim_p, vdim_p=vdim_p, scale=m.scale, q_norm=self._f32(m.q_norm), k_norm=self._f32(m.k_norm),
+                                   window=m.window, keep_first=m.keep_first if m.window else 0, sink=int(m.sink))
+        self._lat_q, self._lat_o = max(self._lat_q, m.heads * dim_p), max(self._lat_o, m.heads * (vdim_p + 4))
+
+    def _wkv_layer(self, L, m):
+        n, rank = m.heads * m.dim, _up(m.w1.shape[0], 64)
+        L.kind = _lib.MIX_RECUR
+        off = self._blocks(L, [("r", m.r), ("k", m.k), ("v", m.v), ("g", m.g), ("w", m.w1)], split=True)
+        mu = torch.zeros((len(m.mu), self._wp), dtype=torch.float32, device=self.device)
+        for j, t in enumerate(m.mu):
+            mu[j, :t.shape[0]] = t.to(torch.float32)
+        L.mu, L.out_k, L.w2_n = self._dev(mu), _up(n, 64), _up(n, 64)
+        L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
+        L.w2 = self._mat(m.w2, L.w2_n, rank)[0]
+        L.recur = _lib.RecurArgs(kind=_lib.RECUR_WKV, off_q=off["r"], off_k=off["k"], off_v=off["v"], off_gate=off["g"], off_a=off["w"], heads=m.heads, dim=m.dim,
+                                 vdim=m.dim, rank=rank, w2d=self._pieces(m.w2, rank), w0=self._f32(m.w0), u=self._f32(m.u), norm_w=self._f32(m.norm))
+
+    def _mlstm_layer(self, L, m):
+        L.kind = _lib.MIX_RECUR
+        off = self._blocks(L, [("q", m.q), ("k", m.k), ("v", m.v), ("g", m.g), ("i", m.i), ("f", m.f)])
+        L.out_k = _up(m.heads * m.vdim, 64)
+        L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
+        L.recur = _lib.RecurArgs(kind=_lib.RECUR_MLSTM, off_q=off["q"], off_k=off["k"], off_v=off["v"], off_gate=off["g"], off_i=off["i"], off_f=off["f"],
+                                 heads=m.heads, dim=m.dim, vdim=m.vdim, bias_i=self._f32(m.bias_i), bias_f=self._f32(m.bias_f), cap=m.cap, norm_w=self._f32(m.norm))
+
+    def _gate_up(self, gate, up, ff):
+        """[2 ff, width_p]: gate and up rows in turn, 16 of each"""
+        w = torch.zeros((ff // 16, 2, 16, self._wp), dtype=torch.bfloat16, device=self.device)
+        for j, t in enumerate((gate, up)):
+            w[:, j] = _pad(t.to(torch.bfloat16), ff, self._wp).view(ff // 16, 16, self._wp)
+        return w.view(2 * ff, self._wp)
+
+    def _glu(self, L, m):
+        L.ff_kind, L.ff, L.glu_limit, L.glu_alpha = _lib.FF_CLAMPGLU, _up(m.gate.shape[0], 64), m.limit, m.alpha
+        L.up, L.up_t = self._mat(self._gate_up(m.gate, m.up, L.ff), tile=True)
+        L.down, L.down_t = self._mat(m.down, self._wp, L.ff, tile=True)
+
+    def _experts(self, L, m):
+        n, ff = len(m.experts), _up(m.experts[0][0].shape[0], 64)
+        gu = torch.empty((n, 2 * ff, self._wp), dtype=torch.bfloat16, device=self.device)
+        dn = torch.empty((n, self._wp, ff), dtype=torch.bfloat16, device=self.device)
+        for e, (gate, up, down) in enumerate(m.experts):
+            gu[e], dn[e] = self._gate_up(gate, up, ff), _pad(down.to(torch.bfloat16), self._wp, ff)
+        L.ff_kind, L.router_n = _lib.FF_MOE, _up(n + m.identity, 64)
+        L.router, L.router_t = self._mat(m.router, L.router_n, self._wp, tile=True)
+        L.moe = _lib.MoeArgs(experts=n, identity=m.identity, top=m.top, groups=m.groups, keep=m.keep, width_p=self._wp, ff_p=ff, gate_up=self._dev(gu),
+                             down=self._dev(dn), correction=self._f32(m.correction))
+
     def _build(self, sd):
         cfg, lib, dev = self.config, self.lib, self.device
         W, self._wp = cfg.hidden_size, _up(cfg.hidden_size, 64)
@@ -277,11 +430,19 @@ class MixedDecoder(SlotModel):
         self.expand_rows = 0 if self.exact else _up(min(self.max_ctx, max(8192, 2 * T)), 64) + 64 * MB
         self._exp = [0] * 5                              # latent, rotated part, keys, values, queries of the expanded form: widest layer
         mixers, arr = [], (_lib.MixLayer * len(cfg.layers))()
+        build = {LatentMixer: self._latent_layer, DeltaMixer: self._delta_layer, WindowMixer: self._window_layer, WkvMixer: self._wkv_layer,
+                 MlstmMixer: self._mlstm_layer}
         for i in range(len(cfg.layers)):
             lw, L = self.layer_weights(sd, i), arr[i]
-            L.norm1, L.norm1b = self._f32(lw.norm1, Wp), self._f32(lw.norm1b, Wp)
-            (self._latent_layer if isinstance(lw.mixer, LatentMixer) else self._delta_layer)(L, lw.mixer)
+            L.norm1, L.parallel = self._f32(lw.norm1, Wp), int(lw.parallel)
+            if lw.norm1b is not None:
+                L.norm1b = self._f32(lw.norm1b, Wp)
+            build[type(lw.mixer)](L, lw.mixer)
+            if lw.ff is not None:
+                L.norm2 = self._f32(lw.norm2, Wp)
+                (self._glu if isinstance(lw.ff, ClampGlu) else self._experts)(L, lw.ff)
             if lw.up is not None:
+                L.ff_kind = _lib.FF_RELU2
                 L.norm2, L.norm2b, L.ff = self._f32(lw.norm2, Wp), self._f32(lw.norm2b, Wp), _up(lw.up.shape[0], 64)
                 L.up, L.up_t = self._mat(lw.up, L.ff, Wp, tile=True)
                 L.down, L.down_t = self._mat(lw.down, Wp, L.ff, tile=True)
@@ -299,15 +460,33 @@ class MixedDecoder(SlotModel):
         order = cfg.runs()
         runs = (_lib.MixRun * len(order))()
         self.cache_bytes = self.state_bytes = 0
+        join = None
+        if mw.get("join") is not None:                   # [x | x0], each half padded
+            w = torch.zeros((Wp, 2, Wp), dtype=torch.bfloat16, device=dev)
+            w[:W, :, :W] = mw["join"].view(W, 2, W).to(torch.bfloat16)
+            join = self._mat(w.view(Wp, 2 * Wp), tile=True)
         for r, (i, opens) in enumerate(order):
             runs[r].layer = i
-            if opens is not None:
+            if opens is not None and mw.get("steps") is not None:
                 runs[r].add = self._f32(mw["steps"][opens], Wp)
+            if opens is not None and mw.get("join") is not None:
+                runs[r].join, runs[r].join_t = join
             if isinstance(mixers[i], LatentMixer):
                 a = arr[i].latent
                 t = torch.zeros((nblk, self.kv_block_size, a.rank_p + a.rot_p), dtype=cache_dtype, device=dev)
                 runs[r].cache = self._dev(t)
                 self.cache_bytes += t.numel() * t.element_size()
+            elif isinstance(mixers[i], WindowMixer):
+                a = arr[i].window
+                k, v = (torch.zeros((nblk, a.kv_heads, self.kv_block_size, d), dtype=cache_dtype, device=dev) for d in (a.dim_p, a.vdim_p))
+                runs[r].cache, runs[r].vcache = self._dev(k), self._dev(v)
+                self.cache_bytes += (k.numel() + v.numel()) * k.element_size()
+            elif arr[i].kind == _lib.MIX_RECUR:
+                a = arr[i].recur
+                mem = [torch.zeros((MB, a.heads, a.dim, _up(a.vdim, 4)), **f32), torch.zeros((MB, Wp), **f32) if arr[i].n_mix else None]
+                mem += [torch.zeros((MB, a.heads, a.dim), **f32), torch.zeros((MB, a.heads), **f32)] if a.kind == _lib.RECUR_MLSTM else [None, None]
+                runs[r].state, runs[r].ring, runs[r].n_state, runs[r].m_state = [None if t is None else self._dev(t) for t in mem]
+                self.state_bytes += sum(4 * t.numel() for t in mem if t is not None)
             else:
                 a = arr[i].delta
                 s = torch.zeros((MB, a.heads, a.dim, _up(a.vdim, 4)), **f32)
@@ -316,12 +495,19 @@ class MixedDecoder(SlotModel):
                 self.state_bytes += 4 * (s.numel() + ring.numel())
         head, head_t = self._mat(mw["head"], Vp, Wp, tile=True)
         embed = self._mat(mw["embed"], V, Wp)[0]
-        kmax = max([Wp] + [max(L.out_k, L.ff) for L in arr])
-        deltas = [L for L in arr if L.kind == _lib.MIX_DELTA]
+        kmax = max([2 * Wp if join else Wp] + [max(L.out_k, L.ff, L.recur.rank) for L in arr])
+        deltas, recurs, moes = ([L for L in arr if c(L)] for c in (lambda L: L.kind == _lib.MIX_DELTA, lambda L: L.kind == _lib.MIX_RECUR,
+                                                                lambda L: L.ff_kind == _lib.FF_MOE))
         most = lambda f: max([f(L) for L in deltas], default=1)
+        over = lambda layers, f: max([f(L) for L in layers], default=1)
+        shifts, pairs, n_mix = bool(over(recurs, lambda L: L.n_mix) > 1), T * over(moes, lambda L: L.moe.top), over(arr, lambda L: L.n_mix)
+        bigram = mw.get("bigram")
         mc = _lib.MixConfig(width=W, width_p=Wp, n_layers=len(arr), n_runs=len(order), exact=int(self.exact), t_max=T, max_slots=MB, max_ctx=self.max_ctx,
                             expand_rows=self.expand_rows if self._exp[0] else 0,
-                            vocab=V, vocab_p=Vp, eps=cfg.rms_norm_eps, block_size=self.kv_block_size, table_stride=bps)
+                            vocab=V, vocab_p=Vp, eps=cfg.rms_norm_eps, block_size=self.kv_block_size, table_stride=bps,
+                            norm_groups=getattr(cfg, "norm_groups", 1), embed_scale=mw.get("embed_scale", 1.0))
+        if bigram:
+            mc.bigram_buckets, mc.bigram_prev, mc.bigram_cur = bigram[1:]
         ws = int(lib.chatts_mixdec_workspace(C.byref(mc), arr))
         rows = T + 1                                     # (kernels may read one row past the last)
         bf = dict(dtype=torch.bfloat16, device=dev)
@@ -340,10 +526,24 @@ class MixedDecoder(SlotModel):
             "dq": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
             "dk": torch.zeros((rows, most(lambda L: L.delta.kv_heads * L.delta.dim)), **f32),
             "dv": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
-            "dg": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.dim)), **f32),
+            "dg": torch.zeros((rows, max(most(lambda L: L.delta.heads * L.delta.dim), over(recurs, lambda L: L.w2_n))), **f32),
             "dgate": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32), "dbeta": torch.zeros((rows, most(lambda L: L.delta.heads)), **f32),
-            "dchunks": torch.zeros(most(lambda L: int(lib.chatts_delta_chunk_floats(L.delta.heads, L.delta.dim, T, MB))), **f32),
-            "dout": torch.zeros((rows, most(lambda L: L.delta.heads * L.delta.vdim)), **f32),
+            "dchunks": torch.zeros(max(most(lambda L: int(lib.chatts_delta_chunk_floats(L.delta.heads, L.delta.dim, T, MB))),
+                                       over(recurs, lambda L: int(lib.chatts_recur_chunk_floats(L.recur.heads, L.recur.dim, T, MB)))), **f32),
+            "dout": torch.zeros((rows, max(most(lambda L: L.delta.heads * L.delta.vdim), over(recurs, lambda L: L.recur.heads * L.recur.vdim))), **f32),
+            "prev_token": torch.zeros(MB, dtype=torch.int64, device=dev), "x0": torch.zeros((rows, Wp) if join else (1, 1), **f32),
+            "h": torch.zeros((rows, Wp) if shifts else (1, 1), **f32), "m_f32": torch.zeros((n_mix, rows, Wp) if shifts else (1, 1), **f32),
+            "m_planes": torch.zeros((2, n_mix, rows, Wp) if shifts and not self.exact else (2, 1, 1), **bf),
+            "n_f32": torch.zeros((rows, Wp), **f32), "n_planes": torch.zeros((2, rows, Wp) if not self.exact else (2, 1, 1), **bf),
+            "gates": torch.zeros((rows, 4 * over(recurs, lambda L: L.recur.heads)), **f32), "den": torch.zeros((rows, over(recurs, lambda L: L.recur.heads)), **f32),
+            "moe_ids": torch.zeros(pairs, dtype=torch.int32, device=dev), "moe_place": torch.zeros(pairs, dtype=torch.int32, device=dev),
+            "moe_order": torch.zeros(pairs, dtype=torch.int32, device=dev),
+            "moe_offsets": torch.zeros(over(moes, lambda L: L.moe.experts) + 1, dtype=torch.int32, device=dev),
+            "moe_tiles": torch.zeros(4 * over(moes, lambda L: int(lib.chatts_moe_tiles(T, L.moe.top, L.moe.experts))), dtype=torch.int32, device=dev),
+            "moe_weight": torch.zeros(pairs, **f32), "moe_kept": torch.zeros(rows, **f32), "moe_logits": torch.zeros((rows, over(moes, lambda L: L.router_n)), **f32),
+            "moe_y": torch.zeros((pairs, Wp) if moes else (1, 1), **f32),
+            "act_f32": torch.zeros((pairs, over(moes, lambda L: L.moe.ff_p)) if self.exact else (1, 1), **f32),
+            "act_planes": torch.zeros((2, pairs, over(moes, lambda L: L.moe.ff_p)) if not self.exact else (2, 1, 1), **bf),
             "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
             "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),
@@ -359,7 +559,11 @@ class MixedDecoder(SlotModel):
                              q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), qx=P(B["x_q"]), cbuf=P(B["x_c"]), krbuf=P(B["x_kr"]),
                              kx_hi=P(B["x_k"][0]), kx_lo=P(B["x_k"][1]), vx_hi=P(B["x_v"][0]), vx_lo=P(B["x_v"][1]), zero=P(B["x_zero"]), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
                              logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
-                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout")})
+                             bigram=self._mat(bigram[0], None, Wp)[0] if bigram else None, x0=P(B["x0"]) if join else None, mix_stride=rows * Wp,
+                             **{f"{n}_{h}": P(B[f"{n}_planes"][j]) for n in ("m", "n", "act") for j, h in enumerate(("hi", "lo"))},
+                             **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout", "prev_token", "h", "m_f32", "n_f32", "gates", "den",
+                                                     "moe_ids", "moe_place", "moe_order", "moe_offsets", "moe_tiles", "moe_weight", "moe_kept", "moe_logits", "moe_y",
+                                                     "act_f32")})
         h = lib.chatts_mixdec_create(C.byref(mc), arr, runs, C.byref(mb))
         if not h:
             raise _lib.ChattsError(-1, lib.chatts_last_error().decode())

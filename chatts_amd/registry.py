@@ -10,6 +10,7 @@ import os
 ARCHITECTURES = {
     None: ("chatts_amd", "ChatTSConfig", "ChatTSForCausalLM"),
     "Fobolix": ("chatts_amd.fobolix", "FobolixConfig", "FobolixForCausalLM"),
+    "Medilix": ("chatts_amd.medilix", "MedilixConfig", "MedilixForCausalLM"),
 }
 
 

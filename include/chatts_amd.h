@@ -51,8 +51,10 @@ const char* chatts_last_error(void);
  *     chatts_tp_set_bulk_release / chatts_tp_bulk_release); tiled prefill weights (chatts_tile_bf16, ChattsLinearArgs.w_tiled /
  *     planes_tiled, ChattsLayerWeights.*_t);
  * 10: decoders of mixed layers chatts_mixdec_* with their kernels (chatts_residual_norm, chatts_delta_*, chatts_latent_*, chatts_head_linear),
- *     CHATTS_EPI_RELU2, ChattsLinearArgs.exact_f32. */
-#define CHATTS_ABI_VERSION 10
+ *     CHATTS_EPI_RELU2, ChattsLinearArgs.exact_f32;
+ * 11: chatts_recur_*, chatts_window_*, chatts_moe_*, chatts_pair_norm, chatts_token_shift, chatts_embed_pair; parallel layers and joined passes of
+ *     chatts_mixdec_*; CHATTS_EPI_CLAMPGLU, ChattsLinearArgs.glu_limit / glu_alpha. */
+#define CHATTS_ABI_VERSION 11
 int chatts_abi_version(void);
 /* Number of CUs of the current device (grid sizing), or <0. */
 int chatts_device_cus(void);
@@ -152,6 +154,8 @@ int chatts_ts_encode(const float* series, const int32_t* row_off, const int32_t*
 #define CHATTS_EPI_SWIGLU 3   /* W rows are gate/up interleaved in blocks of 16 rows;               */
                               /* C[M,N/2] = silu(gate) * up            (Qwen2MLP.forward)           */
 #define CHATTS_EPI_RELU2 4    /* C = max(acc + bias, 0)^2              (bf16 weights)               */
+#define CHATTS_EPI_CLAMPGLU 5 /* rows as for SWIGLU; g = min(gate, glu_limit), u = clamp(up, +-glu_limit): */
+                              /* C[M,N/2] = g sigmoid(glu_alpha g) (u + 1)   (bf16 weights)         */
 
 typedef struct ChattsLinearArgs {
   const float* a;          /* [M, lda] */
@@ -224,6 +228,7 @@ typedef struct ChattsLinearArgs {
   /* optional: every product and sum in float32 (M > 1: the float32 matrix pipe on the widened weights, gemm_f32.hip; M == 1: the GEMV as
    * always).  Needs float32 `a` and `c`, bf16 `w`; no planes, no fused norm.  For 32-bit runs of a model, not a fast path. */
   int exact_f32;
+  float glu_limit, glu_alpha;      /* EPI_CLAMPGLU */
 } ChattsLinearArgs;
 #define CHATTS_W8_FP8 0
 #define CHATTS_W8_INT8 1
@@ -871,9 +876,162 @@ typedef struct ChattsLatentExpandArgs {
 int chatts_latent_can_expand(int dim_p, int rot_p, int vdim_p, int rank_p);
 int chatts_latent_expanded(const ChattsLatentExpandArgs* args, chatts_stream_t stream);
 
+/* ---- layers whose mixer and feed-forward read two norms of the same x (pair.hip) ----
+ * chatts_embed_pair: x = scale * embed[token] + bigram[(prev * mul_prev + token * mul_cur) mod buckets], the table's last row (number `buckets`)
+ * for a sequence's first token; prev: the last token of every slot, kept current (device). */
+typedef struct ChattsEmbedPairArgs {
+  const int64_t* tokens;     /* [T] */
+  const ChattsRow* rows;
+  int t, single, width_p, vocab;
+  const chatts_bf16* embed;  /* [vocab, width_p] */
+  float scale;
+  const chatts_bf16* bigram; /* [buckets + 1, width_p] or NULL */
+  int64_t buckets, mul_prev, mul_cur;
+  int64_t* prev;             /* [slots] */
+  float *x, *x0;             /* [T, width_p]; x0: a copy, or NULL */
+} ChattsEmbedPairArgs;
+int chatts_embed_pair(const ChattsEmbedPairArgs* args, chatts_stream_t stream);
+
+/* One launch per row of the stream:
+ *   x += sum_j weight[j] y[place[j]] + kept h            experts of the layer before (y != NULL); h: the input they had
+ *   join:  out1 = [x | x0]                                (x0 != NULL: the input of a projection that joins a pass to the embedding), nothing else
+ *   n = x, each of `groups` equal consecutive parts divided by its root mean square;  out1 = n w1,  out2 = n w2  (w2 NULL: none)
+ *   mix != 0 (rows of one-token segments): out1's values h enter operand block s as h + (h' - h) mu[s], h' = the slot's previous h (zero at
+ *   position 0), which becomes h; out1 itself is then not written */
+typedef struct ChattsPairNormArgs {
+  float* x;                  /* [T, ldx] */
+  int t, width, ldx, groups;
+  float eps;
+  const float* y;            /* [places, ldx] or NULL */
+  const int32_t* place;      /* [T, top], < 0: none */
+  const float* weight;       /* [T, top] */
+  const float* kept;         /* [T] */
+  ChattsOperand h;
+  int top;
+  const float* x0;
+  const float *w1, *w2;      /* padded with zeros to ldx */
+  ChattsOperand out1, out2;
+  int n_mix;
+  const float* mu;           /* [n_mix, ldx] */
+  ChattsOperand mix;         /* block s: mix_stride elements further */
+  int64_t mix_stride;
+  float* prev;               /* [slots, ldx] */
+  const ChattsRow* rows;
+} ChattsPairNormArgs;
+int chatts_pair_norm(const ChattsPairNormArgs* args, chatts_stream_t stream);
+/* the same mixes for segments of several tokens: h [T, ldx] float32; `prev` is read, not written (chatts_recur_out does that) */
+typedef struct ChattsTokenShiftArgs {
+  const float* h;
+  int t, ldx, n_mix;
+  const float* mu;
+  ChattsOperand mix;
+  int64_t mix_stride;
+  const float* prev;
+  const ChattsRow* rows;
+} ChattsTokenShiftArgs;
+int chatts_token_shift(const ChattsTokenShiftArgs* args, chatts_stream_t stream);
+
+/* ---- gated linear recurrences (recur.hip): S <- diag(g_t) S + k_t v_t^T per head, float32 ----
+ * CHATTS_RECUR_WKV    g = exp(-exp(W2 tanh(a) + w0)) per key channel;  o = S^T q + (q . (u k)) v with S before the token's own write;
+ *                     out = o / rms(o) * norm_w * silu(gate)
+ * CHATTS_RECUR_MLSTM  logarithms i = cap tanh((i + bi) / cap), f = logsigmoid(cap tanh((f + bf) / cap)), running maximum m' = max(f + m, i):
+ *                     g = exp(f + m - m'), k scaled by exp(i - m');  n like S with v = 1;  q scaled by dim^-1/2;
+ *                     o = S^T q / (max(|n . q|, exp(-m')) + 1e-6);  out = o / rms(o) * norm_w * sigmoid(gate)
+ * Input: rows of one projection with the blocks q, k [heads * dim], v, gate [heads * vdim], and a [rank] / i, f [heads].
+ * State per slot: S [heads, dim, vdim4] (vdim4 = vdim rounded up to 4), n [heads, dim], m [heads].  A row at position 0 starts from zero whatever
+ * the slot holds. */
+#define CHATTS_RECUR_WKV 1
+#define CHATTS_RECUR_MLSTM 2
+typedef struct ChattsRecurArgs {
+  int kind;
+  const float* proj;
+  int ld_proj, off_q, off_k, off_v, off_gate, off_a, off_i, off_f;
+  int heads, dim, vdim, rank;      /* rank padded to a multiple of 8 (zero weights) */
+  const chatts_bf16* w2d;          /* [rank / 8, heads * dim, 8] */
+  const float *w0, *u;             /* [heads * dim] */
+  const float *bias_i, *bias_f;    /* [heads] */
+  float cap, eps;
+  const float* norm_w;             /* [heads * vdim] */
+  float *state, *n_state, *m_state;
+  const ChattsRow* rows;
+  int n_rows;
+  const ChattsSpan* spans;         /* device; they cover rows 0 .. n_rows - 1 in order, without gaps */
+  int n_spans;
+  /* scratch of the several-token form: decay [T, ld_decay] = W2 tanh(a) (wkv), gates [T, heads, 4] (mlstm), chunks: chatts_recur_chunk_floats(),
+   * o [T, heads * vdim], den [T, heads] (mlstm) */
+  const float* decay;
+  int ld_decay;
+  float *gates, *chunks, *o, *den;
+  ChattsOperand out;
+  const float* h;                  /* chatts_recur_out: the mixer's input [T, ld_h], whose last row per segment becomes prev[slot] (or NULL) */
+  float* prev;
+  int ld_h;
+} ChattsRecurArgs;
+int chatts_recur_decode(const ChattsRecurArgs* args, chatts_stream_t stream);      /* every row is a segment of one token: one launch */
+int chatts_recur_tanh(const ChattsRecurArgs* args, const ChattsOperand* out, chatts_stream_t stream);   /* wkv: tanh(a) as an operand over `rank` columns */
+int chatts_recur_scan(const ChattsRecurArgs* args, chatts_stream_t stream);        /* gates, chunks of 16 tokens, the state passed along ... */
+int chatts_recur_out(const ChattsRecurArgs* args, chatts_stream_t stream);         /* ... norm and gate of the read-outs */
+int64_t chatts_recur_chunk_floats(int heads, int dim, int n_rows, int n_spans);
+
+/* ---- attention over paged keys and values, grouped heads, per-head norms, optional window / kept first tokens / sink / gate (window.hip) ----
+ * Pages of 2^log_block tokens: keys [page][kv head][token][dim_p], values [page][kv head][token][vdim_p], bf16 or float32.
+ * Position i sees j <= i with i - j < window or j < keep_first (window 0: all).  sink: one more term exp(0) in the softmax's denominator. */
+typedef struct ChattsWindowArgs {
+  const float* proj;
+  int ld_proj, off_q, off_k, off_v, off_gate;        /* off_gate < 0: no gate */
+  int heads, kv_heads, dim, vdim, dim_p, vdim_p;     /* dim_p % 32 == 0, vdim_p % 16 == 0 */
+  float scale, eps;
+  const float *q_norm, *k_norm;                      /* [dim] */
+  int window, keep_first, sink;
+  void *kcache, *vcache;
+  int cache_f32;
+  const int32_t* table;
+  int table_stride, log_block;
+  const ChattsRow* rows;
+  int n_rows;
+  const ChattsSpan* spans;                           /* device */
+  int n_spans, longest;                              /* longest: rows of the longest span */
+  ChattsOperand q;                                   /* normed queries [T, heads * dim_p]: hi plane, or float32 with float32 pages */
+  int n_splits;
+  float* partial;                                    /* [T, heads, n_splits, vdim_p + 4] when n_splits > 1 */
+  ChattsOperand out;                                 /* [T, heads * vdim] */
+} ChattsWindowArgs;
+int chatts_window_prep(const ChattsWindowArgs* args, chatts_stream_t stream);      /* norms, cache write */
+int chatts_window_attend(const ChattsWindowArgs* args, chatts_stream_t stream);    /* row by row: decoding, short segments, 32-bit runs */
+int chatts_window_prefill(const ChattsWindowArgs* args, chatts_stream_t stream);   /* segments of many rows (bf16 pages) */
+int chatts_window_can_prefill(int dim_p, int vdim_p);
+
+/* ---- mixture of experts (moe.hip): softmax router with a correction of the choice, groups, identity experts ----
+ * Outputs of the router: `experts` feed-forwards W_down (silu(W_gate h) * W_up h), then `identity` outputs that return h. */
+typedef struct ChattsMoeArgs {
+  int experts, identity, top, groups, keep;
+  int width_p, ff_p;                    /* both % 64 == 0 */
+  const chatts_bf16* gate_up;           /* [experts][2 ff_p][width_p], gate / up rows interleaved in blocks of 16 */
+  const chatts_bf16* down;              /* [experts][width_p][ff_p] */
+  const float* correction;              /* [experts + identity] */
+  const float* logits;                  /* [T, ld_logits] */
+  int ld_logits;
+  ChattsOperand h;                      /* planes, or float32 when exact */
+  const ChattsRow* rows;
+  int n_rows, exact;
+  int32_t *ids, *place, *order, *offsets, *tiles;   /* [T, top], [T, top], [T * top], [experts + 1], chatts_moe_tiles() * 4 */
+  float *weight, *kept;                 /* [T, top], [T] (weight of the identity outputs) */
+  ChattsOperand act;                    /* [T * top, ff_p] */
+  float* y;                             /* [T * top, width_p] */
+} ChattsMoeArgs;
+int chatts_moe_route(const ChattsMoeArgs* args, chatts_stream_t stream);
+int chatts_moe_experts(const ChattsMoeArgs* args, chatts_stream_t stream);
+int chatts_moe_tiles(int rows, int top, int experts);
+
 /* ---- the composed decoder (mixdec.hip) ---- */
 #define CHATTS_MIX_LATENT 1
 #define CHATTS_MIX_DELTA 2
+#define CHATTS_MIX_RECUR 3
+#define CHATTS_MIX_WINDOW 4
+#define CHATTS_FF_NONE 0
+#define CHATTS_FF_RELU2 1
+#define CHATTS_FF_CLAMPGLU 2
+#define CHATTS_FF_MOE 3
 typedef struct ChattsMixLayer {
   int kind;                                          /* CHATTS_MIX_* */
   const float *norm1, *norm1b, *norm2, *norm2b;      /* before / after the mixer, before / after the feed-forward; padded with zeros to width_p */
@@ -886,13 +1044,30 @@ typedef struct ChattsMixLayer {
   int dim_p, vdim_p, out_head;                       /* out_head: columns between heads in the input of `out` */
   ChattsLatentArgs latent;                           /* sizes, offsets and weights; the rest is filled in per step */
   ChattsDeltaArgs delta;
+  int parallel;                                      /* x += mixer(norm1(x)) + ff(norm2(x)), norms in groups; no norm1b / norm2b */
+  int ff_kind;                                       /* CHATTS_FF_*; CLAMPGLU: up = [2 ff, width_p] interleaved, parallel layers only (MOE too) */
+  float glu_limit, glu_alpha;
+  int n_mix;                                         /* recur: operands of the stacked projection (token shift), 0: one operand */
+  int mix_row[8];                                    /* ... first row of every operand's block; mix_row[n_mix] = in_n */
+  const chatts_bf16* mix_t[8];                       /* ... chatts_tile_bf16 copy of every block, or NULL */
+  const float* mu;                                   /* [n_mix, width_p] */
+  const chatts_bf16* w2;                             /* recur, wkv: [up64(heads * dim), rank], rank % 64 == 0 */
+  int w2_n;
+  ChattsRecurArgs recur;
+  ChattsWindowArgs window;
+  const chatts_bf16 *router, *router_t;              /* [router_n, width_p] */
+  int router_n;
+  ChattsMoeArgs moe;
 } ChattsMixLayer;
 typedef struct ChattsMixRun {      /* one pass through a layer */
   int layer;
   const float* add;                /* vector added to the residual stream before it, or NULL */
   void* cache;                     /* latent: this run's pages */
-  float* state;                    /* delta: this run's states and convolution rings */
-  float* ring;
+  float* state;                    /* delta, recur: this run's states */
+  float* ring;                     /* delta: convolution rings; recur: the previous token's mixer input [slots, width_p] */
+  float *n_state, *m_state;        /* recur, mlstm */
+  void* vcache;                    /* window: value pages (cache: key pages) */
+  const chatts_bf16 *join, *join_t;   /* x <- join [x | x0] before it, [width_p, 2 width_p], or NULL */
 } ChattsMixRun;
 typedef struct ChattsMixConfig {
   int width, width_p, n_layers, n_runs, exact, t_max, max_slots, max_ctx;
@@ -900,6 +1075,9 @@ typedef struct ChattsMixConfig {
   int64_t vocab, vocab_p;
   float eps;
   int block_size, table_stride;
+  int norm_groups;
+  float embed_scale;
+  int64_t bigram_buckets, bigram_prev, bigram_cur;
 } ChattsMixConfig;
 typedef struct ChattsMixBuffers {
   const chatts_bf16 *embed, *head, *head_t;          /* [vocab, width_p], [vocab_p, width_p] */
@@ -913,6 +1091,20 @@ typedef struct ChattsMixBuffers {
   chatts_bf16 *qx, *cbuf, *krbuf, *kx_hi, *kx_lo, *vx_hi, *vx_lo;   /* latent, expanded form (ChattsLatentExpandArgs) */
   const chatts_bf16* zero;
   float *dq, *dk, *dv, *dg, *dgate, *dbeta, *dchunks, *dout;
+  const chatts_bf16* bigram;                         /* [buckets + 1, width_p] or NULL */
+  int64_t* prev_token;                               /* [max_slots] */
+  float* x0;                                         /* [t_max, width_p] or NULL */
+  float* h;                                          /* recur: the mixer's input [t_max, width_p] */
+  float* m_f32;                                      /* operands of the token shift [n_mix][t_max + 1, width_p] */
+  chatts_bf16 *m_hi, *m_lo;
+  int64_t mix_stride;
+  float* n_f32;                                      /* second norm's operand [t_max, width_p] */
+  chatts_bf16 *n_hi, *n_lo;
+  float *gates, *den;
+  int32_t *moe_ids, *moe_place, *moe_order, *moe_offsets, *moe_tiles;
+  float *moe_weight, *moe_kept, *moe_logits, *moe_y;
+  float* act_f32;                                    /* experts' activations [t_max * top, widest ff] */
+  chatts_bf16 *act_hi, *act_lo;
   ChattsRow* rows;                                   /* device, [t_max] */
   ChattsSpan* spans;                                 /* device, [max_slots] */
   int32_t* table;                                    /* device, [max_slots, table_stride] */

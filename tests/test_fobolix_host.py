@@ -95,6 +95,9 @@ def test_struct_layouts_match_the_header(tmp_path):
     from chatts_amd import _lib
     names = {"ChattsRow": 16, "ChattsSpan": C.sizeof(_lib.Span), "ChattsLatentExpandArgs": C.sizeof(_lib.LatentExpandArgs), "ChattsOperand": C.sizeof(_lib.Operand), "ChattsResidualNormArgs": C.sizeof(_lib.ResidualNormArgs),
              "ChattsHeadLinearArgs": C.sizeof(_lib.HeadLinearArgs), "ChattsDeltaArgs": C.sizeof(_lib.DeltaArgs), "ChattsLatentArgs": C.sizeof(_lib.LatentArgs),
+             "ChattsEmbedPairArgs": C.sizeof(_lib.EmbedPairArgs), "ChattsPairNormArgs": C.sizeof(_lib.PairNormArgs),
+             "ChattsTokenShiftArgs": C.sizeof(_lib.TokenShiftArgs), "ChattsRecurArgs": C.sizeof(_lib.RecurArgs),
+             "ChattsWindowArgs": C.sizeof(_lib.WindowArgs), "ChattsMoeArgs": C.sizeof(_lib.MoeArgs),
              "ChattsMixLayer": C.sizeof(_lib.MixLayer), "ChattsMixRun": C.sizeof(_lib.MixRun), "ChattsMixConfig": C.sizeof(_lib.MixConfig),
              "ChattsMixBuffers": C.sizeof(_lib.MixBuffers), "ChattsLinearArgs": C.sizeof(_lib.LinearArgs)}
     src = tmp_path / "s.c"
