@@ -139,9 +139,24 @@ def route(z, correction, r):
     return idx, w / (w.sum(-1, keepdim=True) + 1e-20)
 
 
-def experts(h, sd, p, spec):
+def choice_margin(z, correction, r):
+    """how much a router's logits z [T, N] prefer what is chosen to the next best, groups and outputs: a much smaller rounding changes nothing"""
+    choice, groups, T = torch.softmax(z, -1) + correction, r.get("groups") or {"count": 1, "keep": 1}, z.shape[0]
+
+    def gap(v, n):
+        v = v.sort(-1, descending=True).values
+        return v[:, n - 1] - v[:, n] if n < v.shape[1] else torch.full((T,), math.inf, dtype=z.dtype)
+    best = choice.view(T, groups["count"], -1).max(-1).values
+    out = best < best.sort(-1, descending=True).values[:, groups["keep"] - 1:groups["keep"]]
+    return torch.minimum(gap(best, groups["keep"]), gap(choice.masked_fill(out.repeat_interleave(z.shape[1] // groups["count"], 1), -1e9), r["top"]))
+
+
+def experts(h, sd, p, spec, margins=None):
     r = spec["router"]
-    idx, w = route(h @ sd[p + "router"].T, sd[p + "correction"], r)
+    z = h @ sd[p + "router"].T
+    idx, w = route(z, sd[p + "correction"], r)
+    if margins is not None:
+        margins.append(choice_margin(z, sd[p + "correction"], r))
     y = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for e, a in zip(idx[t].tolist(), w[t]):
@@ -154,12 +169,12 @@ def experts(h, sd, p, spec):
     return y
 
 
-def layer(x, sd, i, spec, norm):
+def layer(x, sd, i, spec, norm, margins=None):
     p = f"l{i}."
     y = MIXERS[spec["type"]](group_norm(x, sd[p + "norm1"], norm["groups"], norm["eps"]), sd, p + "mix.", spec["mixer"], norm["eps"])
     if spec.get("mlp"):
         h = group_norm(x, sd[p + "norm2"], norm["groups"], norm["eps"])
-        y = y + (experts if spec["mlp"]["kind"] == "moe" else dense)(h, sd, p + "mlp.", spec["mlp"])
+        y = y + (experts(h, sd, p + "mlp.", spec["mlp"], margins) if spec["mlp"]["kind"] == "moe" else dense(h, sd, p + "mlp.", spec["mlp"]))
     return x + y
 
 
@@ -175,15 +190,15 @@ def runs(cfg):
     return out + [(i, None) for i in range(b, n)]
 
 
-def forward(cfg, sd, tokens, dtype=torch.float64, want_layers=False):
-    """-> logits [T, vocab] (and the residual stream after every layer run)"""
+def forward(cfg, sd, tokens, dtype=torch.float64, want_layers=False, margins=None):
+    """-> logits [T, vocab] (and the residual stream after every layer run); margins: a list that gets choice_margin of every router run"""
     sd = {k: v.to(dtype) for k, v in sd.items()}
     x = x0 = embedding(cfg, sd, tokens)
     streams = []
     for i, t in runs(cfg):
         if t is not None:
             x = torch.cat([x, x0], -1) @ sd["loop.in"].T
-        x = layer(x, sd, i, cfg["layers"][i], cfg["norm"])
+        x = layer(x, sd, i, cfg["layers"][i], cfg["norm"], margins)
         streams.append(x)
     logits = group_norm(x, sd["final.norm"], cfg["norm"]["groups"], cfg["norm"]["eps"]) @ sd["head"].T
     return (logits, streams) if want_layers else logits
