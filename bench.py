@@ -518,38 +518,56 @@ def bench_batched(args, model, cfg, comm, world, device):
 DESIGN_SIZES = {"s": (2048, 9216, 6144, 16), "m": (4096, 18432, 12288, 32), "l": (5120, 20736, 13824, 40)}      # width, ff, SwiGLU ff, heads
 
 
-def design_configs(size, layers=8, vocab=32000):
-    """-> (Fobolix configuration: three delta layers, then one latent attention layer, repeated; Qwen configuration of the same size)"""
-    from chatts_amd.config import preset
+def fobolix_config(size, layers, vocab):
+    """three delta layers, then one latent attention layer, repeated"""
     from chatts_amd.fobolix import FobolixConfig
-    W, ff, inter, heads = DESIGN_SIZES[size]
+    W, ff, _, heads = DESIGN_SIZES[size]
     mlp = {"kind": "dense", "ff": ff}
     delta = {"type": "channel_delta", "mixer": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}, "mlp": mlp}
     latent = {"type": "latent_attention", "mlp": mlp,
               "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
                         "rot": {"base": 1e6, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
-    fob = FobolixConfig(vocab=vocab, width=W, layers=[latent if i % 4 == 3 else delta for i in range(layers)], norm={"eps": 1e-5}, name=f"fobolix-{size}")
-    qwen = preset("chatts-8b", vocab_size=vocab, hidden_size=W, intermediate_size=inter, num_hidden_layers=layers, num_attention_heads=heads,
+    return FobolixConfig(vocab=vocab, width=W, layers=[latent if i % 4 == 3 else delta for i in range(layers)], norm={"eps": 1e-5}, name=f"fobolix-{size}")
+
+
+def medilix_config(size, layers, vocab):
+    """wkv, mlstm, windowed attention, wkv, repeated; every second feed-forward has experts (four chosen ones weigh as much as a dense one)"""
+    from chatts_amd.medilix import MedilixConfig
+    W, _, inter, heads = DESIGN_SIZES[size]
+    dense = {"kind": "dense", "ff": inter, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": inter // 4}, "router": {"experts": 28, "identity": 4, "top": 4, "groups": {"count": 4, "keep": 3}}}
+    wkv = {"type": "wkv", "mixer": {"heads": heads, "dim": 128}}
+    mlstm = {"type": "mlstm", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "gate_cap": 15.0}}
+    window = {"type": "attention", "mixer": {"heads": heads, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024, "keep_first": 64}}}
+    kinds = [dict(wkv, mlp=dense), dict(mlstm, mlp=moe), dict(window, mlp=dense), dict(wkv, mlp=moe)]
+    return MedilixConfig(vocab=vocab, width=W, layers=[kinds[i % 4] for i in range(layers)], norm={"eps": 1e-5, "groups": 4}, name=f"medilix-{size}",
+                         embedding={"scale": 1.0, "bigram": {"buckets": 32003, "mul_prev": 31, "mul_cur": 7}})
+
+
+def qwen_config(size, layers, vocab):
+    from chatts_amd.config import preset
+    W, _, inter, heads = DESIGN_SIZES[size]
+    return preset("chatts-8b", vocab_size=vocab, hidden_size=W, intermediate_size=inter, num_hidden_layers=layers, num_attention_heads=heads,
                   num_key_value_heads=8, ts_token_start_index=vocab - 20, eos_token_id=[vocab - 18, vocab - 17], im_start_token_id=vocab - 16)
-    return fob, qwen
 
 
 def bench_design(args):
     """one JSON line per size and model: prefill tokens/s (one prompt of --design-prompt tokens, and four of a quarter each) and decode tokens/s
     (1 and 16 sequences behind --design-prompt tokens)"""
     import torch
-    from chatts_amd.fobolix import FobolixForCausalLM
-    from chatts_amd.modeling import ChatTSForCausalLM
+    from chatts_amd.registry import model_class
     T, dev = args.design_prompt, "cuda:0"
     torch.cuda.set_device(0)
     g = torch.Generator().manual_seed(0)
     for size in args.design_sizes.split(","):
-        for name, cfg, cls in zip(("fobolix", "qwen"), design_configs(size, args.layers or 8), (FobolixForCausalLM, ChatTSForCausalLM)):
+        for name, make in ((args.design, {"fobolix": fobolix_config, "medilix": medilix_config}[args.design]), ("qwen", qwen_config)):
             if args.design_only and name != args.design_only:
                 continue
+            cfg = make(size, args.layers or 8, 32000)
+            cls = model_class(cfg)
             r = {"design": name, "size": size, "width": cfg.hidden_size, "layers": cfg.num_hidden_layers, "prompt": T, "dtype": "bf16", "data": "synthetic"}
             for batch in (1, 16):
-                kw = {} if name == "fobolix" else {"kv_block_size": 64}
+                kw = {"kv_block_size": 64} if name == "qwen" else {}
                 model = cls.from_synthetic(cfg, seed=0, device=dev, max_ctx=T + 256, max_prefill_tokens=T, max_batch=batch, **kw)
                 ids = torch.randint(0, 31000, (T,), generator=g).tolist()
 
@@ -582,6 +600,7 @@ def bench_design(args):
                     model.reserve_kv(s, T + 200)
                 model.buf["pos_all"].fill_(T)
                 model.buf["step_all"].zero_()
+                model.buf["token_all"].copy_(torch.tensor(ids[:batch]))
                 step = model.decode_step if batch == 1 else model.batched_step
                 if batch == 1 and name == "qwen":
                     model.buf["x"].zero_()
@@ -667,10 +686,10 @@ def main():
     ap.add_argument("--weights", default="bf16", choices=["bf16", "fp8", "int8", "int4"],
                     help="fp8 = BASELINE.json config 5 weight format, int4 = the GPTQ-Int4 checkpoint's (NOT the headline: separate workloads)")
     ap.add_argument("--launch-check", action="store_true", help="only prove the N-rank launch path (no model): rank 0 prints the world it saw")
-    ap.add_argument("--design", default=None, choices=["fobolix"], help="another workload: layers of this design beside the Qwen decoder at equal size, random weights")
+    ap.add_argument("--design", default=None, choices=["fobolix", "medilix"], help="another workload: layers of this design beside the Qwen decoder at equal size, random weights")
     ap.add_argument("--design-sizes", default="s,m,l", help=f"of {sorted(DESIGN_SIZES)}")
     ap.add_argument("--design-prompt", type=int, default=2048)
-    ap.add_argument("--design-only", default=None, choices=["fobolix", "qwen"], help="one of the two models (profiling)")
+    ap.add_argument("--design-only", default=None, choices=["fobolix", "medilix", "qwen"], help="one of the two models (profiling)")
     args = ap.parse_args()
 
     if args.design:

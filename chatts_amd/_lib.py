@@ -43,7 +43,8 @@ class LinearArgs(C.Structure):
                 ("post_norm_w", c_void_p), ("post_norm_eps", c_float), ("post_hi", c_void_p), ("post_lo", c_void_p), ("ld_post", c_int),
                 ("w4", c_void_p), ("w4_sz", c_void_p), ("ldw4", c_int), ("w4_group", c_int),
                 ("w8_format", c_int), ("tp_reduce", c_void_p), ("w_tiled", c_void_p), ("planes_tiled", c_int), ("exact_f32", c_int),
-                ("glu_limit", c_float), ("glu_alpha", c_float)]
+                ("glu_limit", c_float), ("glu_alpha", c_float),
+                ("batch", c_int), ("a_stride", c_int64), ("w_stride", c_int64), ("c_stride", c_int64), ("w_tiled_batch", c_void_p)]
 
 
 class LinearFp8Args(C.Structure):
@@ -199,7 +200,7 @@ class WindowArgs(C.Structure):
 class MoeArgs(C.Structure):
     """ChattsMoeArgs: mixture of experts (csrc/moe.hip)"""
     _fields_ = ([(n, c_int) for n in ("experts", "identity", "top", "groups", "keep", "width_p", "ff_p")] +
-                [("gate_up", c_void_p), ("down", c_void_p), ("correction", c_void_p), ("logits", c_void_p), ("ld_logits", c_int), ("h", Operand), ("rows", c_void_p),
+                [("gate_up", c_void_p), ("down", c_void_p), ("gate_up_t", c_void_p), ("down_t", c_void_p), ("correction", c_void_p), ("logits", c_void_p), ("ld_logits", c_int), ("h", Operand), ("rows", c_void_p),
                  ("n_rows", c_int), ("exact", c_int)] + [(n, c_void_p) for n in ("ids", "place", "order", "offsets", "tiles", "weight", "kept")] +
                 [("act", Operand), ("y", c_void_p)])
 
@@ -257,6 +258,7 @@ SIGNATURES = {
     "chatts_ts_encode": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, C.POINTER(TsWeights), c_void_p,
                                  c_void_p, c_void_p, c_void_p, c_void_p, c_size_t, c_void_p]),
     "chatts_linear_workspace": (c_size_t, [c_int, c_int, c_int]),
+    "chatts_linear_workspace_batch": (c_size_t, [c_int, c_int, c_int, c_int]),
     "chatts_gemv_ksplit": (c_int, [c_int, c_int, c_int, c_int]),
     "chatts_linear": (c_int, [C.POINTER(LinearArgs), c_void_p]),
     "chatts_quantize_rows_fp8": (c_int, [c_void_p, c_int, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p, c_void_p]),

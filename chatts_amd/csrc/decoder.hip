@@ -12,6 +12,8 @@
 namespace chatts {
 int launch_gemv(const ChattsLinearArgs* a, hipStream_t s);
 int launch_gemm_f32(const ChattsLinearArgs* a, hipStream_t s);
+bool gemm_batched_stream(const ChattsLinearArgs* a);
+size_t gemm_workspace_batch(int m, int n, int k, int batch);
 int launch_gemm(const ChattsLinearArgs* a, hipStream_t s, const RopeFuse* rope = nullptr, bool* rope_done = nullptr);
 int attention_decode_batched_impl(const float* qkv_raw, int batch, int n_q, int n_kv, const float* q_norm_w, const float* k_norm_w,
                                   float norm_eps, const float* cos_tab, const float* sin_tab, int pos, const int32_t* pos_dev,
@@ -50,6 +52,10 @@ static int64_t embed_rows(const ChattsDecoder* d) { return d->cfg.embed_rows > 0
 static int64_t embed_offset(const ChattsDecoder* d) { return d->cfg.embed_rows > 0 ? d->cfg.embed_offset : d->cfg.vocab_offset; }
 
 extern "C" size_t chatts_linear_workspace(int m, int n, int k) { return gemm_workspace(m, n, k); }
+extern "C" size_t chatts_linear_workspace_batch(int m, int n, int k, int batch) {
+  const size_t one = gemm_workspace(m, n, k), all = gemm_workspace_batch(m, n, k, batch);
+  return all > one ? all : one;
+}
 
 static int linear_impl(const ChattsLinearArgs* a, chatts_stream_t stream, const RopeFuse* rope, bool* rope_done);
 extern "C" int chatts_linear(const ChattsLinearArgs* a, chatts_stream_t stream) { return linear_impl(a, stream, nullptr, nullptr); }
@@ -94,6 +100,24 @@ static int linear_impl(const ChattsLinearArgs* a, chatts_stream_t stream, const 
                        (a->epilogue == CHATTS_EPI_NONE || a->epilogue == CHATTS_EPI_RESID) && !cplanes,
                    CHATTS_E_BADARG, "linear: post-norm planes need M > 1, float32 c, EPI_NONE / EPI_RESID, both planes, ld_post >= N");
   if (a->tp_reduce) CHATTS_REQUIRE(a->m == 1, CHATTS_E_BADARG, "linear: tp_reduce is available for M == 1 (the decode GEMV) only");
+  if (a->batch > 1) {
+    CHATTS_REQUIRE(a->epilogue == CHATTS_EPI_NONE && !a->bias && !a->w8 && !a->w4 && !a->norm_w && !a->post_norm_w && !a->tp_reduce && a->a_stride % 8 == 0 &&
+                       a->w_stride % 8 == 0 && a->c_stride % 4 == 0, CHATTS_E_BADARG, "linear: a batch of %d takes plain products of one shape", a->batch);
+    if (!(a->m == 1 || (!a->exact_f32 && gemm_batched_stream(a)))) {
+      for (int i = 0; i < a->batch; ++i) {
+        ChattsLinearArgs b = *a;
+        b.batch = 0;
+        if (b.a) b.a += i * a->a_stride;
+        if (b.a_hi) { b.a_hi += i * a->a_stride; b.a_lo += i * a->a_stride; }
+        b.w += i * a->w_stride;
+        b.w_tiled = a->w_tiled_batch ? a->w_tiled_batch[i] : nullptr;
+        if (b.c) b.c += i * a->c_stride;
+        if (b.c_hi) { b.c_hi += i * a->c_stride; b.c_lo += i * a->c_stride; }
+        if (const int rc = linear_impl(&b, stream, nullptr, nullptr)) return rc;
+      }
+      return CHATTS_OK;
+    }
+  }
   if (a->m == 1 && a->epilogue != CHATTS_EPI_GELU) return launch_gemv(a, as_stream(stream));      // (products and sums in float32 already)
   if (a->exact_f32) {
     CHATTS_REQUIRE(a->a && a->c && !cplanes && !a->post_norm_w && !a->norm_w && !a->w8, CHATTS_E_BADARG,

@@ -291,6 +291,12 @@ __device__ __forceinline__ void wait_stages(int later) {
 template <int NSTAGE, bool W8, int MB, int NW = 4, bool I8 = false>
 __global__ __launch_bounds__(64 * NW) void gemm_stream_kernel(GemmParams p, const uint16_t* __restrict__ a_hi,
                                                               const uint16_t* __restrict__ a_lo, int ldp) {
+  if (gridDim.y > 1) {      // (uniform) one of several products of the same shape
+    p.w += blockIdx.y * p.w_stride;
+    a_hi += blockIdx.y * p.a_stride;
+    a_lo += blockIdx.y * p.a_stride;
+    p.c += blockIdx.y * p.c_stride;
+  }
   static_assert(!W8 || MB == 1, "the fp8 weight stream is a batched-decode format (M <= 16)");
   static_assert(NW == 4 || (NW == 8 && (W8 || MB % 2 == 0)), "8 waves: fp8 W (one A piece per wave), or bf16 W with an even block count");
   // wave grid inside the 16 MB x 128 tile: WM x WN.  4 waves: 1 x 4 (32 columns each).  8 waves, fp8 W (M <= 16): 1 x 8 (16 columns).
@@ -508,7 +514,8 @@ __global__ __launch_bounds__(256) void splitk_epilogue_v4_kernel(const float* __
                                                                 const float* __restrict__ bias, const float* __restrict__ resid,
                                                                 float* __restrict__ c, int ldc, int epilogue,
                                                                 const float* __restrict__ scale, uint16_t* __restrict__ c_hi,
-                                                                uint16_t* __restrict__ c_lo, int ldcp) {
+                                                                uint16_t* __restrict__ c_lo, int ldcp, int64_t c_stride) {
+  if (gridDim.y > 1) { ws += blockIdx.y * (size_t)sk * m * n; c += blockIdx.y * c_stride; }
   const int n4 = n >> 2;
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= (size_t)m * n4) return;
@@ -906,9 +913,20 @@ static int launch_stream_t(const GemmParams& p, const ChattsLinearArgs* a, int s
     CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "gemm_stream: cannot reserve %d bytes of LDS: %s", LDS, hipGetErrorString(e));
     configured = true;
   }
-  dim3 grid((a->n + kStreamBN - 1) / kStreamBN, 1, sk), block(64 * NW);
+  dim3 grid((a->n + kStreamBN - 1) / kStreamBN, a->batch > 1 ? a->batch : 1, sk), block(64 * NW);
   hipLaunchKernelGGL((gemm_stream_kernel<NSTAGE, W8, MB, NW, I8>), grid, block, LDS, s, p, a->a_hi, a->a_lo, a->ld_planes);
   return CHATTS_OK;
+}
+
+// can the weight-streaming kernel run all members of ChattsLinearArgs.batch at once (and the plain split-K epilogue finish them)?
+bool gemm_batched_stream(const ChattsLinearArgs* a) {
+  return a->m >= 2 && a->m <= 16 && use_stream(a) && !a->w8 && a->c && !a->c_hi && a->epilogue == CHATTS_EPI_NONE && a->n % 4 == 0 && a->ldc % 4 == 0 && a->c_stride % 4 == 0 &&
+         a->a_stride % 8 == 0 && a->w_stride % 8 == 0 && ((uintptr_t)a->c % 16) == 0 && opt_get(OPT_EPI_V4, 1) != 0 && pick_stream_sk(a->n * a->batch, a->k, false) <= 8;
+}
+size_t gemm_workspace_batch(int m, int n, int k, int batch) {
+  if (batch <= 1 || m < 2 || m > 16 || k % 64) return 0;
+  const int sk = pick_stream_sk(n * batch, k, false);
+  return sk > 1 ? (size_t)batch * sk * m * n * sizeof(float) : 0;
 }
 
 size_t gemm_workspace(int m, int n, int k) {
@@ -937,11 +955,12 @@ int launch_gemm(const ChattsLinearArgs* a_in, hipStream_t s, const RopeFuse* rop
   }
   const bool stream = use_stream(a);
   const bool ring = !stream && use_ring(a);
+  const int batch = a->batch > 1 ? a->batch : 1;      // > 1: gemm_batched_stream(a) holds
   RingGeom rg{};
   CHATTS_REQUIRE(!a->planes_tiled || ring, CHATTS_E_SHAPE, "linear: tiled planes are the prefill kernel's operand format (M=%d K=%d take another kernel)", a->m, a->k);
   CHATTS_REQUIRE(!ring || !a->w_tiled || (((uintptr_t)a->w_tiled % 16) == 0 && a->ldw == a->k), CHATTS_E_SHAPE, "linear: w_tiled needs 16-byte alignment and ldw == K");
   if (stream) {
-    sk = pick_stream_sk(a->n, a->k, a->w8 != nullptr);
+    sk = pick_stream_sk(a->n * batch, a->k, a->w8 != nullptr);
     bm = 16;
   } else if (ring) {
     if (const int rc = check_ring_operands(a)) return rc;
@@ -968,13 +987,16 @@ int launch_gemm(const ChattsLinearArgs* a_in, hipStream_t s, const RopeFuse* rop
   p.wt = ring ? a->w_tiled : nullptr; p.planes_tiled = a->planes_tiled;
   p.glu_limit = a->glu_limit; p.glu_alpha = a->glu_alpha;
   if (sk > 1) {
-    const size_t need = (size_t)sk * a->m * a->n * sizeof(float);
+    const size_t need = (size_t)batch * sk * a->m * a->n * sizeof(float);
     CHATTS_REQUIRE(a->workspace && a->workspace_bytes >= need, CHATTS_E_WORKSPACE,
                    "linear: split-K needs %zu workspace bytes, got %zu", need, a->workspace_bytes);
     p.c = reinterpret_cast<float*>(a->workspace);
+    p.c_stride = (int64_t)sk * a->m * a->n;
   } else {
     p.c = a->c;
+    p.c_stride = a->c_stride;
   }
+  p.a_stride = a->a_stride; p.w_stride = a->w_stride;
   const int nt_count = (a->n + 127) / 128, mt_count = (a->m + bm - 1) / bm;
   dim3 grid(8 * ((nt_count + 7) / 8) * mt_count, 1, sk), block(256);
   if (stream) {
@@ -1074,9 +1096,9 @@ int launch_gemm(const ChattsLinearArgs* a_in, hipStream_t s, const RopeFuse* rop
       ((uintptr_t)a->c % 16) == 0 && ((uintptr_t)a->resid % 16) == 0 && ((uintptr_t)a->bias % 16) == 0 &&
       (!a->w8 || ((uintptr_t)a->w8_scale % 16) == 0) && opt_get(OPT_EPI_V4, 1) != 0) {
     const size_t total = (size_t)a->m * (a->n / 4);
-    hipLaunchKernelGGL(splitk_epilogue_v4_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, s,
+    hipLaunchKernelGGL(splitk_epilogue_v4_kernel, dim3((unsigned)((total + 255) / 256), batch), dim3(256), 0, s,
                        reinterpret_cast<const float*>(a->workspace), sk, a->m, a->n, a->bias, a->resid, a->c, a->ldc, a->epilogue,
-                       a->w8 ? a->w8_scale : nullptr, a->c_hi, a->c_lo, a->ld_cplanes);
+                       a->w8 ? a->w8_scale : nullptr, a->c_hi, a->c_lo, a->ld_cplanes, a->c_stride);
     CHATTS_CHECK_LAUNCH("splitk_epilogue_v4");
   } else if (sk > 1) {
     const int ncols = epi_is_glu(a->epilogue) ? a->n / 2 : a->n;

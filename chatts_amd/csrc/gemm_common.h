@@ -25,6 +25,7 @@ struct GemmParams {
   const uint16_t* wt;    // optional (gemm_ring_kernel): W in the tiled layout of chatts_tile_bf16 - a 1 KB LDS-DMA piece is 1 KB of memory
   int planes_tiled;      // a_hi / a_lo are in that layout too
   float glu_limit, glu_alpha;
+  int64_t a_stride, w_stride, c_stride;   // several products of one shape (gemm_stream_kernel, grid y)
 };
 
 __device__ __forceinline__ void store_planes(uint16_t* hi, uint16_t* lo, size_t off, float v) {
@@ -54,6 +55,17 @@ struct RingGeom {
   int wpx;            // workgroups per XCD (grid = 8 * wpx)
 };
 void ring_pick(int m, int n, int k, int cus, int force_t, int force_sk, RingGeom& g);
+// the same kernel over lists of rows with weights of their own (experts): tiles [count][4] = {matrix, first place, places, -}, places of a tile
+// at most kRingTile; order != nullptr: place -> row of A = order[place] / top, else A is packed by place.  C is packed by place; p.m: rows of A - 1 at most
+struct RingGroup {
+  const int32_t* tiles;
+  const int32_t* count;      // device: number of tiles
+  const int32_t* order;
+  int top;
+  int64_t w_stride;          // elements between matrices (p.w and p.wt)
+};
+constexpr int kRingTile = 160;
+int launch_ring_group(const GemmParams& p, const uint16_t* a_hi, const uint16_t* a_lo, int ldp, const RingGroup& g, int most_tiles, hipStream_t s);
 int launch_ring(const GemmParams& p, const uint16_t* a_hi, const uint16_t* a_lo, int ldp, const RingGeom& g, bool single, hipStream_t s);
 
 typedef const __attribute__((address_space(1))) void* gptr_t;

@@ -39,10 +39,27 @@ constexpr int kRingLds = kRingSlots * kRingHalf;             // 144 KB
 constexpr int kRingThreads = 768, kRingCompute = 8, kRingLoaders = 4;
 
 
+// GROUPED (launch_ring_group): unit = (W panel, tile of a list), the tiles' number is only known on the device
+__device__ __forceinline__ RingUnit ring_group_unit(const GemmParams& p, const RingGroup& gr, int T, int u, int& matrix, int& places) {
+  RingUnit r;
+  const int mt = u % T;
+  const int32_t* t = gr.tiles + (size_t)mt * 4;
+  matrix = t[0];
+  r.m0 = t[1];
+  places = t[2];
+  r.panel = u / T;
+  r.split = 0;
+  r.f = (places + 15) >> 4;
+  r.f0 = (r.f + 1) >> 1;
+  r.kbeg = 0;
+  r.nh = p.k >> 5;
+  return r;
+}
+
 // SINGLE: the "bf16" speed mode - the lo plane is neither staged nor multiplied (activations rounded to bf16: NOT parity grade)
-template <bool SINGLE>
+template <bool SINGLE, bool GROUPED = false>
 __global__ __launch_bounds__(kRingThreads) void gemm_ring_kernel(GemmParams p, const uint16_t* __restrict__ a_hi,
-                                                                 const uint16_t* __restrict__ a_lo, int ldp, RingGeom g) {
+                                                                 const uint16_t* __restrict__ a_lo, int ldp, RingGeom g, RingGroup gr) {
   extern __shared__ __attribute__((aligned(1024))) char smem[];
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -50,12 +67,22 @@ __global__ __launch_bounds__(kRingThreads) void gemm_ring_kernel(GemmParams p, c
   // workgroups take every wpx-th unit of it, so that at any time an XCD works on ~wpx consecutive units: the M-tiles of a few W panels
   // at the same K offset - each K-slice of a panel is fetched into that L2 once for all of them
   const int xcd = blockIdx.x & 7, local = blockIdx.x >> 3;
+  if constexpr (GROUPED) {
+    g.T = *gr.count;
+    g.units = g.T * g.P;
+  }
+  auto unit = [&](int u, int& matrix, int& places) __attribute__((always_inline)) {
+    if constexpr (GROUPED) return ring_group_unit(p, gr, g.T, u, matrix, places);
+    else return ring_unit(p, g, u);
+  };
   const int share = g.units >> 3, rem = g.units & 7;
   const int ubeg = xcd * share + (xcd < rem ? xcd : rem), ucnt = share + (xcd < rem);
   if (local >= ucnt) return;                                   // padding workgroup (fewer units than workgroups): uniform exit
   const int uend = ubeg + ucnt, u0 = ubeg + local, ustep = g.wpx;
   int G = 0;                                                   // half-steps of this workgroup = barriers after the first
-  for (int u = u0; u < uend; u += ustep) G += ring_unit(p, g, u).nh;
+  if constexpr (GROUPED) G = (uend - u0 + ustep - 1) / ustep * (p.k >> 5);
+  else
+    for (int u = u0; u < uend; u += ustep) G += ring_unit(p, g, u).nh;
 
   if (wave >= kRingCompute) {
     // ---- loader wave L: pieces of 16 rows x 64 bytes (1 KB per wave instruction).  W pieces {L, L + 4, L + 8, L + 12}; of the unit's
@@ -70,21 +97,23 @@ __global__ __launch_bounds__(kRingThreads) void gemm_ring_kernel(GemmParams p, c
     int dst[9];
     int np = 0, nh_cur = 0, hh = 0, ucur = u0;
     auto setup = [&](int u) {
-      const RingUnit r = ring_unit(p, g, u);
+      int matrix = 0, places = 0;
+      const RingUnit r = unit(u, matrix, places);
       nh_cur = r.nh;
       np = 0;
       const int n0 = r.panel * kRingBN;
+      const size_t skip = GROUPED ? (size_t)matrix * gr.w_stride : 0;
 #pragma unroll
       for (int h = 0; h < 4; ++h) {
         if (wtiled) {
           int rb = (n0 >> 4) + L + 4 * h;
           const int rbmax = ((p.n + 15) >> 4) - 1;
           if (rb > rbmax) rb = rbmax;
-          src[h] = reinterpret_cast<const char*>(p.wt + ((size_t)rb * nkt + (r.kbeg >> 5)) * 512) + lane * 16;
+          src[h] = reinterpret_cast<const char*>(p.wt + skip + ((size_t)rb * nkt + (r.kbeg >> 5)) * 512) + lane * 16;
         } else {
           int wr = n0 + (L + 4 * h) * 16 + prow;
           if (wr > p.n - 1) wr = p.n - 1;
-          src[h] = reinterpret_cast<const char*>(p.w + (size_t)wr * p.ldw + r.kbeg + gchunk * 8);
+          src[h] = reinterpret_cast<const char*>(p.w + skip + (size_t)wr * p.ldw + r.kbeg + gchunk * 8);
         }
         dst[h] = kRingWOff + (L + 4 * h) * 1024;
       }
@@ -99,7 +128,12 @@ __global__ __launch_bounds__(kRingThreads) void gemm_ring_kernel(GemmParams p, c
             src[4 + h] = reinterpret_cast<const char*>((plane ? a_lo : a_hi) + ((size_t)((r.m0 >> 4) + frag) * nkt + (r.kbeg >> 5)) * 512) + lane * 16;
           } else {
             int am = r.m0 + frag * 16 + prow;
-            if (am > p.m - 1) am = p.m - 1;
+            if constexpr (GROUPED) {
+              if (am > r.m0 + places - 1) am = r.m0 + places - 1;
+              if (gr.order) am = gr.order[am] / gr.top;
+            } else if (am > p.m - 1) {
+              am = p.m - 1;
+            }
             src[4 + h] = reinterpret_cast<const char*>((plane ? a_lo : a_hi) + (size_t)am * ldp + r.kbeg + gchunk * 8);
           }
           dst[4 + h] = plane * kRingAPlane + frag * 1024;
@@ -146,7 +180,9 @@ __global__ __launch_bounds__(kRingThreads) void gemm_ring_kernel(GemmParams p, c
   __builtin_amdgcn_s_barrier();                                // half-stage 0 published
   int gh = 0;
   for (int u = u0; u < uend; u += ustep) {
-    const RingUnit r = ring_unit(p, g, u);
+    int matrix = 0, places = 0;
+    const RingUnit r = unit(u, matrix, places);
+    if constexpr (GROUPED) p.m = r.m0 + places;
     const int fml = wm ? r.f - r.f0 : r.f0;
     const int rowblk = wm ? r.f0 : 0;                          // first fragment of this wave within the tile
     if (fml == 0) {
@@ -293,7 +329,24 @@ static int launch_ring_t(const GemmParams& p, const uint16_t* a_hi, const uint16
     CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "gemm_ring: cannot reserve %d bytes of LDS: %s", kRingLds, hipGetErrorString(e));
     configured = true;
   }
-  hipLaunchKernelGGL(gemm_ring_kernel<SINGLE>, dim3(8 * g.wpx), dim3(kRingThreads), kRingLds, s, p, a_hi, a_lo, ldp, g);
+  hipLaunchKernelGGL(gemm_ring_kernel<SINGLE>, dim3(8 * g.wpx), dim3(kRingThreads), kRingLds, s, p, a_hi, a_lo, ldp, g, RingGroup{});
+  return CHATTS_OK;
+}
+int launch_ring_group(const GemmParams& p, const uint16_t* a_hi, const uint16_t* a_lo, int ldp, const RingGroup& gr, int most_tiles, hipStream_t s) {
+  static_assert(kRingTile == kRingMaxF * 16, "a tile's places");
+  static bool configured = false;
+  if (!configured) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm_ring_kernel<false, true>), hipFuncAttributeMaxDynamicSharedMemorySize, kRingLds);
+    CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "gemm_ring: cannot reserve %d bytes of LDS: %s", kRingLds, hipGetErrorString(e));
+    configured = true;
+  }
+  RingGeom g{};
+  g.P = (p.n + kRingBN - 1) / kRingBN;
+  const int cus = device_cus(), most = (most_tiles * g.P + 7) / 8;
+  g.wpx = cus / 8 < most ? cus / 8 : most;
+  if (g.wpx < 1) g.wpx = 1;
+  hipLaunchKernelGGL((gemm_ring_kernel<false, true>), dim3(8 * g.wpx), dim3(kRingThreads), kRingLds, s, p, a_hi, a_lo, ldp, g, gr);
+  CHATTS_CHECK_LAUNCH("gemm_ring_group");
   return CHATTS_OK;
 }
 int launch_ring(const GemmParams& p, const uint16_t* a_hi, const uint16_t* a_lo, int ldp, const RingGeom& g, bool single, hipStream_t s) {

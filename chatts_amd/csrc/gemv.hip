@@ -47,6 +47,7 @@ struct GemvParams {
   TpParams tp;            // kEpiResidTp only
   int ks;                 // gemv_ksplit_kernel: waves per row group
   float glu_limit, glu_alpha;   // CHATTS_EPI_CLAMPGLU
+  int64_t x_stride, w_stride, out_stride;   // grid y: further products of the same shape
 };
 
 // ---- the exchange inside the launch (kEpiResidTp) ---------------------------------------------------------------------------
@@ -135,6 +136,7 @@ __device__ __forceinline__ void gemv_epilogue(const GemvParams& p, int task, int
 template <int ROWS, int UNR, int EPI, bool NORM>
 __global__ __launch_bounds__(1024) void gemv_ldsx_kernel(GemvParams p) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
+  if (gridDim.y > 1) { p.x += blockIdx.y * p.x_stride; p.w += blockIdx.y * p.w_stride; p.out += blockIdx.y * p.out_stride; }
   f32x4* xs4 = reinterpret_cast<f32x4*>(smem);            // permuted x: [chunk][half][lane] float4
   float* red = reinterpret_cast<float*>(smem) + (size_t)((p.k + 511) / 512) * 512;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -225,6 +227,7 @@ template <int EPI, bool NORM>
 __global__ __launch_bounds__(1024) void gemv_ksplit_kernel(GemvParams p) {
   constexpr int ROWS = 2, UNR = 2;
   extern __shared__ __attribute__((aligned(16))) char smem[];
+  if (gridDim.y > 1) { p.x += blockIdx.y * p.x_stride; p.w += blockIdx.y * p.w_stride; p.out += blockIdx.y * p.out_stride; }
   f32x4* xs4 = reinterpret_cast<f32x4*>(smem);            // permuted x: [chunk][half][lane] float4
   float* red = reinterpret_cast<float*>(smem) + (size_t)((p.k + 511) / 512) * 512;
   float* part = red + 16;                                 // [nw][ROWS] partial sums of the K-slices
@@ -569,15 +572,15 @@ __global__ __launch_bounds__(1024) void gemv4_ldsx_kernel(GemvParams p) {
 
 // ---- dispatch ------------------------------------------------------------------------------------
 template <int ROWS, int UNR, int EPI>
-static void launch_ldsx_norm(const GemvParams& p, bool norm, int blocks, int threads, size_t lds, hipStream_t s) {
-  if (norm) hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, EPI, true>), dim3(blocks), dim3(threads), lds, s, p);
-  else hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, EPI, false>), dim3(blocks), dim3(threads), lds, s, p);
+static void launch_ldsx_norm(const GemvParams& p, bool norm, dim3 blocks, int threads, size_t lds, hipStream_t s) {
+  if (norm) hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, EPI, true>), blocks, dim3(threads), lds, s, p);
+  else hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, EPI, false>), blocks, dim3(threads), lds, s, p);
 }
 template <int ROWS, int UNR>
-static void launch_ldsx(const GemvParams& p, int epi, bool norm, int blocks, int threads, size_t lds, hipStream_t s) {
+static void launch_ldsx(const GemvParams& p, int epi, bool norm, dim3 blocks, int threads, size_t lds, hipStream_t s) {
   switch (epi) {
     case CHATTS_EPI_RESID: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_RESID>(p, norm, blocks, threads, lds, s); break;
-    case kEpiResidTp: hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, kEpiResidTp, false>), dim3(blocks), dim3(threads), lds, s, p); break;
+    case kEpiResidTp: hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, kEpiResidTp, false>), blocks, dim3(threads), lds, s, p); break;
     case CHATTS_EPI_SWIGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_SWIGLU>(p, norm, blocks, threads, lds, s); break;
     case CHATTS_EPI_RELU2: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_RELU2>(p, norm, blocks, threads, lds, s); break;
     case CHATTS_EPI_CLAMPGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_CLAMPGLU>(p, norm, blocks, threads, lds, s); break;
@@ -772,8 +775,10 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
   // row is long enough to split.  Every TP = 1 shape of the supported models has >= 10 waves per CU and keeps the whole-K kernel.
   p.ks = 1;
   p.glu_limit = a->glu_limit; p.glu_alpha = a->glu_alpha;
+  p.x_stride = a->a_stride; p.w_stride = a->w_stride; p.out_stride = a->c_stride;
+  const int batch = a->batch > 1 ? a->batch : 1;
   if (!a->tp_reduce && rows == 2 && unr == 2 && nchunks >= 4) {
-    int ks = gemv_pick_ksplit(p.tasks, nchunks, norm, (double)a->n * a->k * 2.0, cus);
+    int ks = gemv_pick_ksplit(p.tasks * batch, nchunks, norm, (double)a->n * a->k * 2.0 * batch, cus);
     ks = opt_get(OPT_GEMV_KS, ks);
     if (ks > 16) ks = 16;
     if (ks > 1) {
@@ -784,7 +789,7 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
       const int occk = (int)((150 * 1024) / lds) < 32 / nwk ? (int)((150 * 1024) / lds) : 32 / nwk;
       if (blocksk > cus * (occk < 1 ? 1 : occk)) blocksk = cus * (occk < 1 ? 1 : occk);
       p.ks = ks;
-      const dim3 g(blocksk), b(nwk * 64);
+      const dim3 g(blocksk, batch), b(nwk * 64);
       switch (epilogue) {
         case CHATTS_EPI_RESID:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_RESID, true>), g, b, lds, s, p);
@@ -812,10 +817,10 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
     }
   }
   if (a->tp_reduce) p.tp = tp_issue(a->tp_reduce, false);
-  if (rows == 4 && unr == 2) launch_ldsx<4, 2>(p, epilogue, norm, blocks, threads, lds_launch, s);
-  else if (rows == 4) launch_ldsx<4, 4>(p, epilogue, norm, blocks, threads, lds_launch, s);
-  else if (unr == 2) launch_ldsx<2, 2>(p, epilogue, norm, blocks, threads, lds_launch, s);
-  else launch_ldsx<2, 4>(p, epilogue, norm, blocks, threads, lds_launch, s);
+  if (rows == 4 && unr == 2) launch_ldsx<4, 2>(p, epilogue, norm, dim3(blocks, batch), threads, lds_launch, s);
+  else if (rows == 4) launch_ldsx<4, 4>(p, epilogue, norm, dim3(blocks, batch), threads, lds_launch, s);
+  else if (unr == 2) launch_ldsx<2, 2>(p, epilogue, norm, dim3(blocks, batch), threads, lds_launch, s);
+  else launch_ldsx<2, 4>(p, epilogue, norm, dim3(blocks, batch), threads, lds_launch, s);
   CHATTS_CHECK_LAUNCH("gemv_ldsx");
   return CHATTS_OK;
 }

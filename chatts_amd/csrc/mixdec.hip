@@ -40,6 +40,13 @@ struct ChattsMixDecoder {
 
 static bool mix_planes(const ChattsMixConfig& c, int m, int k) { return !c.exact && k % 64 == 0 && ((m >= 2 && m <= 16) || m >= 96); }
 
+static int mix_equal_blocks(const ChattsMixLayer& l, int i) {      // how many operand blocks from i on have the size of block i
+  const int rows = l.mix_row[i + 1] - l.mix_row[i];
+  int n = 1;
+  while (i + n < l.n_mix && l.mix_row[i + n + 1] - l.mix_row[i + n] == rows) ++n;
+  return n;
+}
+
 extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const ChattsMixLayer* layers) {
   if (!c || !layers) return 0;
   std::vector<std::pair<int, int>> shapes;
@@ -72,6 +79,14 @@ extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const Chatts
       if (b > ws) ws = b;
     }
   }
+  for (int i = 0; i < c->n_layers; ++i)
+    for (int j = 0, n; j < layers[i].n_mix; j += n) {
+      n = mix_equal_blocks(layers[i], j);
+      for (int t = 2; t <= 16 && t <= c->t_max; ++t) {
+        const size_t w = chatts_linear_workspace_batch(t, layers[i].mix_row[j + 1] - layers[i].mix_row[j], c->width_p, n);
+        if (w > ws) ws = w;
+      }
+    }
   const size_t am = argmax_scratch_bytes(c->max_slots > 1 ? c->max_slots : 1);
   if (am > ws) ws = am;
   for (int t = 2; t <= c->t_max; ++t)
@@ -401,10 +416,18 @@ static int mix_parallel_forward(ChattsMixDecoder* d, const int64_t* tokens, int 
         a.rows = d->b.rows;
         if ((rc = chatts_token_shift(&a, s)) != 0) return rc;
       }
-      for (int i = 0; i < l.n_mix; ++i) {
-        const size_t at = (size_t)l.mix_row[i] * wp;
-        if ((rc = mix_linear(d, shift_operand(d, t, i), l.in + at, l.mix_t[i], t, l.mix_row[i + 1] - l.mix_row[i], wp, CHATTS_EPI_NONE,
-                             f32_out(d->b.proj + l.mix_row[i], l.in_n), s)) != 0) return rc;
+      for (int i = 0, n; i < l.n_mix; i += n) {      // blocks of equal size are one batch
+        n = mix_equal_blocks(l, i);
+        const ChattsOperand in = shift_operand(d, t, i);
+        const int rows = l.mix_row[i + 1] - l.mix_row[i];
+        ChattsLinearArgs a{};
+        a.a = in.f32; a.lda = wp;
+        if (!in.f32) { a.a_hi = in.hi; a.a_lo = in.lo; a.ld_planes = wp; }
+        a.w = l.in + (size_t)l.mix_row[i] * wp; a.ldw = wp; a.w_tiled = l.mix_t[i]; a.w_tiled_batch = l.mix_t + i;
+        a.m = t; a.n = rows; a.k = wp; a.epilogue = CHATTS_EPI_NONE; a.c = d->b.proj + l.mix_row[i]; a.ldc = l.in_n;
+        a.batch = n; a.a_stride = d->b.mix_stride; a.w_stride = (int64_t)rows * wp; a.c_stride = rows;
+        a.exact_f32 = c.exact; a.workspace = d->b.workspace; a.workspace_bytes = d->b.workspace_bytes;
+        if ((rc = chatts_linear(&a, s)) != 0) return rc;
       }
     } else if ((rc = mix_linear(d, A, l.in, l.in_t, t, l.in_n, wp, CHATTS_EPI_NONE, f32_out(d->b.proj, l.in_n), s)) != 0) {
       return rc;

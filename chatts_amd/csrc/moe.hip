@@ -4,7 +4,8 @@
 //   moe_list_kernel       a workgroup per expert: its (token, choice) pairs as a list, in order; tiles of the lists for the tiled products
 //   moe_route_small_kernel  both in one workgroup, for up to 16 rows; the tiles are then the experts in use
 //   moe_stream_kernel     up to 16 rows: an expert's weights stream once for all of its tokens
-//   moe_gemm_kernel       many rows: tiles of BM tokens x 128 weight rows, A gathered through the list
+//   moe_gemm_kernel       some more rows: tiles of 32 tokens x 128 weight rows, A gathered through the list
+//   gemm_ring_kernel (gemm_ring.hip), grouped: many rows
 //   moe_gemm_f32_kernel   32-bit runs
 // Places: the pairs of expert e are places offsets[e] .. offsets[e + 1) of the packed buffers act and y; order[place] = token * top + choice.
 // The weighted sum over a token's places is part of the norm that follows (chatts_pair_norm).
@@ -14,6 +15,8 @@ namespace chatts {
 
 constexpr int kMoeSmall = 16;       // rows of the streaming form
 constexpr int kMoeMaxOut = 1024;    // router outputs
+constexpr int kMoeListThreads = 1024;
+static_assert(kMoeListThreads == 1024 && kMoeMaxOut <= 1024, "moe_list_kernel: 16 waves, one expert per thread");
 
 __device__ __forceinline__ void wave_best(float& v, int& i) {      // largest value, lowest index
 #pragma unroll
@@ -93,55 +96,59 @@ __global__ __launch_bounds__(256) void moe_route_kernel(ChattsMoeArgs p) {
   if (row < p.n_rows) moe_route_row(p, row, threadIdx.x & 63, sm + wave * (2 * (p.experts + p.identity) + p.groups));
 }
 
-// grid (experts); tiles: {expert, first place, places, 0} per BM places of an expert, in order; the rest {-1, ..}
-__global__ __launch_bounds__(256) void moe_list_kernel(ChattsMoeArgs p, int bm, int n_tiles) {
+// grid (experts); tiles: {expert, first place, places, 0}, at most bm places each, an expert's 16-place fragments dealt evenly; the rest {-1, ..}
+__global__ __launch_bounds__(kMoeListThreads) void moe_list_kernel(ChattsMoeArgs p, int bm, int n_tiles) {
   __shared__ int hist[kMoeMaxOut];
-  __shared__ int wsum[4];
+  __shared__ int wsum[2][16], sums[16][4];
   const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n = p.n_rows * p.top;
-  for (int i = tid; i < p.experts; i += 256) hist[i] = 0;
+  for (int i = tid; i < p.experts; i += 1024) hist[i] = 0;
   __syncthreads();
-  for (int i = tid; i < n; i += 256) {
+  for (int i = tid; i < n; i += 1024) {
     const int id = p.ids[i];
     if (id >= 0) atomicAdd(&hist[id], 1);
   }
   __syncthreads();
-  int before = 0, tile0 = 0, all = 0, all_tiles = 0;      // (every thread adds up the same short table)
-  for (int i = 0; i < p.experts; ++i) {
-    const int c = hist[i], t = (c + bm - 1) / bm;
-    if (i < e) { before += c; tile0 += t; }
-    all += c;
-    all_tiles += t;
+  {
+    const int c = tid < p.experts ? hist[tid] : 0, t = (c + bm - 1) / bm;      // (experts <= 1024: one per thread)
+    const int v[4] = {wave_sum_i(tid < e ? c : 0), wave_sum_i(tid < e ? t : 0), wave_sum_i(c), wave_sum_i(t)};
+    if (lane == 0)
+      for (int k = 0; k < 4; ++k) sums[wave][k] = v[k];
   }
-  const int mine = hist[e];
+  __syncthreads();
+  int before = 0, tile0 = 0, all = 0, all_tiles = 0;
+  for (int w = 0; w < 16; ++w) { before += sums[w][0]; tile0 += sums[w][1]; all += sums[w][2]; all_tiles += sums[w][3]; }
+  const int mine = hist[e], tiles = (mine + bm - 1) / bm, frags = (mine + 15) >> 4;
   if (tid == 0) {
     p.offsets[e] = before;
-    if (e == p.experts - 1) p.offsets[p.experts] = all;
+    if (e == p.experts - 1) { p.offsets[p.experts] = all; p.offsets[p.experts + 1] = all_tiles; }
   }
-  for (int t = tid; t * bm < mine; t += 256) {
+  for (int t = tid; t < tiles; t += 1024) {
+    const int base = frags / tiles, rem = frags % tiles, at = (t * base + (t < rem ? t : rem)) * 16, len = (base + (t < rem)) * 16;
     int32_t* o = p.tiles + (size_t)(tile0 + t) * 4;
     o[0] = e;
-    o[1] = before + t * bm;
-    o[2] = mine - t * bm < bm ? mine - t * bm : bm;
+    o[1] = before + at;
+    o[2] = mine - at < len ? mine - at : len;
     o[3] = 0;
   }
   if (e == 0)
-    for (int t = all_tiles + tid; t < n_tiles; t += 256) p.tiles[(size_t)t * 4] = -1;
-  int at = before;
-  for (int i0 = 0; i0 < n; i0 += 256) {
+    for (int t = all_tiles + tid; t < n_tiles; t += 1024) p.tiles[(size_t)t * 4] = -1;
+  int at = before, b = 0;
+  int next = tid < n ? p.ids[tid] : -1;
+  for (int i0 = 0; i0 < n; i0 += 1024, b ^= 1) {
     const int i = i0 + tid;
-    const bool hit = i < n && p.ids[i] == e;
+    const bool hit = i < n && next == e;
+    next = i + 1024 < n ? p.ids[i + 1024] : -1;
     const unsigned long long mask = __ballot(hit);
-    if (lane == 0) wsum[wave] = __popcll(mask);
+    if (lane == 0) wsum[b][wave] = __popcll(mask);
     __syncthreads();
     int w0 = 0, total = 0;
-    for (int w = 0; w < 4; ++w) { if (w < wave) w0 += wsum[w]; total += wsum[w]; }
+    for (int w = 0; w < 16; ++w) { if (w < wave) w0 += wsum[b][w]; total += wsum[b][w]; }
     if (hit) {
       const int pl = at + w0 + __popcll(mask & ((1ull << lane) - 1));
       p.order[pl] = i;
       p.place[i] = pl;
     }
     at += total;
-    __syncthreads();
   }
 }
 
@@ -190,7 +197,7 @@ __global__ __launch_bounds__(1024) void moe_route_small_kernel(ChattsMoeArgs p, 
         o[3] = 0;
       }
     }
-    if (tid == 0) p.offsets[p.experts] = all;
+    if (tid == 0) { p.offsets[p.experts] = all; p.offsets[p.experts + 1] = all_used; }
     for (int t = all_used + tid; t < n_tiles; t += 1024) p.tiles[(size_t)t * 4] = -1;
   }
   __syncthreads();
@@ -268,7 +275,7 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
   }
 }
 
-// ---- many rows: grid (tiles, blocks of 128 weight rows), 4 waves; K in steps of 64 through LDS, the next step requested while this one is multiplied.
+// ---- more rows: grid (tiles, blocks of 128 weight rows), 4 waves; K in steps of 64 through LDS, the next step requested while this one is multiplied.
 // D = W . A^T, wave = 128 / WN weight rows x BM / WM tokens ----
 constexpr int kMoeLd = 72;      // LDS row of 64 K-values: 144 bytes, sixteen rows meet sixteen different groups of banks
 template <bool GLU, int BM, int WM, int WN>
@@ -436,7 +443,7 @@ static bool moe_small(const ChattsMoeArgs* a) { return a->n_rows <= kMoeSmall &&
 static int moe_bm(const ChattsMoeArgs* a) {      // tokens of a tile
   if (a->exact) return 64;
   if (moe_small(a)) return kMoeSmall;
-  return (int64_t)a->n_rows * a->top >= 48 * (int64_t)(a->experts + a->identity) ? 128 : 32;
+  return (int64_t)a->n_rows * a->top >= 48 * (int64_t)(a->experts + a->identity) ? kRingTile : 32;
 }
 static int moe_tile_bound(int rows, int top, int experts, int bm) {      // sum of ceil(count / bm) over at most min(experts, rows * top) lists
   const int64_t pairs = (int64_t)rows * top, lists = experts < pairs ? experts : pairs;
@@ -477,7 +484,7 @@ extern "C" int chatts_moe_route(const ChattsMoeArgs* a, chatts_stream_t stream) 
     return CHATTS_OK;
   }
   hipLaunchKernelGGL(moe_route_kernel, dim3((a->n_rows + 3) / 4), dim3(256), per * 4, s, *a);
-  hipLaunchKernelGGL(moe_list_kernel, dim3(a->experts), dim3(256), 0, s, *a, bm, tiles);
+  hipLaunchKernelGGL(moe_list_kernel, dim3(a->experts), dim3(kMoeListThreads), 0, s, *a, bm, tiles);
   CHATTS_CHECK_LAUNCH("moe_route");
   return CHATTS_OK;
 }
@@ -502,9 +509,17 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
     return CHATTS_OK;
   }
   int rc;
-  if (bm == 128) {
-    if ((rc = launch_moe_gemm<true, 128, 2, 2>(a, tiles, s)) != 0) return rc;
-    return launch_moe_gemm<false, 128, 2, 2>(a, tiles, s);
+  if (bm == kRingTile) {
+    RingGroup g{a->tiles, a->offsets + a->experts + 1, a->order, a->top, (int64_t)2 * a->ff_p * a->width_p};
+    GemmParams p{};
+    p.w = a->gate_up; p.wt = a->gate_up_t; p.m = a->n_rows; p.n = 2 * a->ff_p; p.k = p.ldw = a->width_p; p.epilogue = CHATTS_EPI_SWIGLU;
+    p.k_per_split = p.k; p.direct = 1; p.c_hi = a->act.hi; p.c_lo = a->act.lo; p.ldcp = a->act.ld; p.ldc = a->act.ld;
+    if ((rc = launch_ring_group(p, a->h.hi, a->h.lo, a->h.ld, g, tiles, s)) != 0) return rc;
+    g.order = nullptr;
+    g.w_stride = (int64_t)a->width_p * a->ff_p;
+    p.w = a->down; p.wt = a->down_t; p.n = a->width_p; p.k = p.ldw = a->ff_p; p.k_per_split = p.k; p.epilogue = CHATTS_EPI_NONE;
+    p.c_hi = p.c_lo = nullptr; p.c = a->y; p.ldc = a->width_p;
+    return launch_ring_group(p, a->act.hi, a->act.lo, a->act.ld, g, tiles, s);
   }
   if ((rc = launch_moe_gemm<true, 32, 1, 4>(a, tiles, s)) != 0) return rc;
   return launch_moe_gemm<false, 32, 1, 4>(a, tiles, s);

@@ -64,38 +64,56 @@ __device__ __forceinline__ void store_row4(const ChattsOperand& o, size_t row, i
   store_operand4(o, row, c, v);
 }
 
-// a workgroup per row; a thread keeps its columns in registers.  QUADS: the groups are made of whole quads of columns.
-template <int NV, bool QUADS>
-__global__ __launch_bounds__(256) void pair_norm_kernel(ChattsPairNormArgs p, int padded) {
+// a workgroup per row; a thread keeps its columns in registers.  QUADS: the groups are made of whole quads of columns.  NT: threads (more of them
+// for a few rows: then every load of a row is in flight at once)
+template <int NT, int NV, bool QUADS>
+__global__ __launch_bounds__(NT) void pair_norm_kernel(ChattsPairNormArgs p, int padded) {
   extern __shared__ float sm[];
   const size_t row = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, part = p.width / p.groups;
   const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-  f32x4 x[NV];
+  ChattsRow R{0, -1, 0, 0};
+  if (p.n_mix) R = p.rows[row];
+  f32x4 x[NV], wa[NV], wb[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (i * 256 + tid) * 4;
+    const int c = (i * NT + tid) * 4;
     x[i] = c < padded ? *reinterpret_cast<const f32x4*>(p.x + row * p.ldx + c) : zero;
   }
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {      // (the weights travel while the row is reduced)
+    const int c = (i * NT + tid) * 4;
+    wa[i] = p.w1 && c < padded ? *reinterpret_cast<const f32x4*>(p.w1 + c) : zero;
+    wb[i] = p.w2 && c < padded ? *reinterpret_cast<const f32x4*>(p.w2 + c) : zero;
+  }
   if (p.y) {
-    for (int j = 0; j < p.top; ++j) {
-      const int at = p.place[row * p.top + j];      // (uniform)
-      if (at < 0) continue;
-      const float w = p.weight[row * p.top + j];
+    constexpr int U = 4;      // experts' rows requested at once
+    for (int j0 = 0; j0 < p.top; j0 += U) {
+      int at[U];
+      float w[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int j = j0 + u < p.top ? j0 + u : j0;
+        at[u] = j0 + u < p.top ? p.place[row * p.top + j] : -1;      // (uniform)
+        w[u] = p.weight[row * p.top + j];
+      }
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
-        const int c = (i * 256 + tid) * 4;
-        if (c < padded) {
-          const f32x4 y = *reinterpret_cast<const f32x4*>(p.y + (size_t)at * p.ldx + c);
+        const int c = (i * NT + tid) * 4;
+        if (c >= padded) continue;
+        f32x4 y[U];
 #pragma unroll
-          for (int k = 0; k < 4; ++k) x[i][k] += w * y[k];
-        }
+        for (int u = 0; u < U; ++u) y[u] = at[u] >= 0 ? *reinterpret_cast<const f32x4*>(p.y + (size_t)at[u] * p.ldx + c) : zero;
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+          for (int k = 0; k < 4; ++k) x[i][k] += at[u] >= 0 ? w[u] * y[u][k] : 0.f;
       }
     }
     const float kept = p.kept[row];
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int c = (i * 256 + tid) * 4;
+      const int c = (i * NT + tid) * 4;
       if (c < padded) {
         if (kept != 0.f) {
           const f32x4 h = load_operand4(p.h, row, c);
@@ -109,7 +127,7 @@ __global__ __launch_bounds__(256) void pair_norm_kernel(ChattsPairNormArgs p, in
   if (p.x0) {
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int c = (i * 256 + tid) * 4;
+      const int c = (i * NT + tid) * 4;
       if (c >= padded) continue;
       store_row4(p.out1, row, c, x[i]);
       store_row4(p.out1, row, p.ldx + c, *reinterpret_cast<const f32x4*>(p.x0 + row * p.ldx + c));
@@ -122,7 +140,7 @@ __global__ __launch_bounds__(256) void pair_norm_kernel(ChattsPairNormArgs p, in
   float* inv = sm + units;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (i * 256 + tid) * 4;
+    const int c = (i * NT + tid) * 4;
     if (QUADS) {
       if (c < p.width) sm[c >> 2] = (x[i][0] * x[i][0] + x[i][1] * x[i][1]) + (x[i][2] * x[i][2] + x[i][3] * x[i][3]);
     } else {
@@ -131,48 +149,53 @@ __global__ __launch_bounds__(256) void pair_norm_kernel(ChattsPairNormArgs p, in
         if (c + k < p.width) sm[c + k] = x[i][k] * x[i][k];
     }
   }
+  f32x4 before[NV];      // the token shift: h of the slot's previous token
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * NT + tid) * 4;
+    before[i] = R.pos > 0 && c < padded ? *reinterpret_cast<const f32x4*>(p.prev + (size_t)R.slot * p.ldx + c) : zero;
+  }
   __syncthreads();
-  for (int g = wave; g < p.groups; g += 4) {
+  for (int g = wave; g < p.groups; g += NT / 64) {
     float ss = 0.f;
     for (int u = lane; u < per; u += 64) ss += sm[g * per + u];
     ss = wave_sum(ss);
     if (lane == 0) inv[g] = 1.0f / sqrtf(ss / (float)part + p.eps);
   }
   __syncthreads();
-  ChattsRow R{0, -1, 0, 0};
-  if (p.n_mix) R = p.rows[row];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (i * 256 + tid) * 4;
+    const int c = (i * NT + tid) * 4;
     if (c >= padded) continue;
-    f32x4 n;
+    f32x4 n, h, d;
 #pragma unroll
-    for (int k = 0; k < 4; ++k) n[k] = c + k < p.width ? x[i][k] * inv[(c + (QUADS ? 0 : k)) / part] : 0.f;
-    const f32x4 w1 = *reinterpret_cast<const f32x4*>(p.w1 + c);
-    f32x4 h;
-#pragma unroll
-    for (int k = 0; k < 4; ++k) h[k] = n[k] * w1[k];
+    for (int k = 0; k < 4; ++k) {
+      n[k] = c + k < p.width ? x[i][k] * inv[(c + (QUADS ? 0 : k)) / part] : 0.f;
+      h[k] = n[k] * wa[i][k];
+      d[k] = before[i][k] - h[k];
+    }
     if (p.n_mix) {
-      float* prev = p.prev + (size_t)R.slot * p.ldx + c;
-      f32x4 d = zero;
-      if (R.pos > 0) d = *reinterpret_cast<const f32x4*>(prev);
+      constexpr int U = 5;
+      for (int s0 = 0; s0 < p.n_mix; s0 += U) {
+        f32x4 mu[U];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) d[k] -= h[k];
-      for (int s = 0; s < p.n_mix; ++s) {
-        const f32x4 mu = *reinterpret_cast<const f32x4*>(p.mu + (size_t)s * p.ldx + c);
-        f32x4 m;
+        for (int u = 0; u < U; ++u) mu[u] = *reinterpret_cast<const f32x4*>(p.mu + (size_t)(s0 + u < p.n_mix ? s0 + u : s0) * p.ldx + c);
 #pragma unroll
-        for (int k = 0; k < 4; ++k) m[k] = h[k] + d[k] * mu[k];
-        store_row4(operand_block(p.mix, s * p.mix_stride), row, c, m);
+        for (int u = 0; u < U; ++u) {
+          if (s0 + u >= p.n_mix) break;
+          f32x4 m;
+#pragma unroll
+          for (int k = 0; k < 4; ++k) m[k] = h[k] + d[k] * mu[u][k];
+          store_row4(operand_block(p.mix, (s0 + u) * p.mix_stride), row, c, m);
+        }
       }
-      if (R.pos >= 0) *reinterpret_cast<f32x4*>(prev) = h;
+      if (R.pos >= 0) *reinterpret_cast<f32x4*>(p.prev + (size_t)R.slot * p.ldx + c) = h;
     } else {
       store_row4(p.out1, row, c, h);
     }
     if (p.w2) {
-      const f32x4 w2 = *reinterpret_cast<const f32x4*>(p.w2 + c);
 #pragma unroll
-      for (int k = 0; k < 4; ++k) h[k] = n[k] * w2[k];
+      for (int k = 0; k < 4; ++k) h[k] = n[k] * wb[i][k];
       store_row4(p.out2, row, c, h);
     }
   }
@@ -216,12 +239,12 @@ extern "C" int chatts_embed_pair(const ChattsEmbedPairArgs* a, chatts_stream_t s
   return CHATTS_OK;
 }
 
-template <int NV>
+template <int NT, int NV>
 static void launch_pair_norm(const ChattsPairNormArgs* a, hipStream_t s) {
   const bool quads = a->width % (4 * a->groups) == 0;
   const size_t lds = (size_t)((quads ? a->width / 4 : a->width) + a->groups) * sizeof(float);
-  if (quads) hipLaunchKernelGGL((pair_norm_kernel<NV, true>), dim3(a->t), dim3(256), lds, s, *a, a->ldx);
-  else hipLaunchKernelGGL((pair_norm_kernel<NV, false>), dim3(a->t), dim3(256), lds, s, *a, a->ldx);
+  if (quads) hipLaunchKernelGGL((pair_norm_kernel<NT, NV, true>), dim3(a->t), dim3(NT), lds, s, *a, a->ldx);
+  else hipLaunchKernelGGL((pair_norm_kernel<NT, NV, false>), dim3(a->t), dim3(NT), lds, s, *a, a->ldx);
 }
 
 extern "C" int chatts_pair_norm(const ChattsPairNormArgs* a, chatts_stream_t stream) {
@@ -236,11 +259,13 @@ extern "C" int chatts_pair_norm(const ChattsPairNormArgs* a, chatts_stream_t str
   CHATTS_REQUIRE(!a->n_mix || (a->mu && a->prev && a->rows && ok(a->mix, a->ldx) && a->mix_stride % 4 == 0), CHATTS_E_BADARG, "pair_norm: token shift");
   if (a->t == 0) return CHATTS_OK;
   hipStream_t s = as_stream(stream);
-  if (a->ldx <= 1024) launch_pair_norm<1>(a, s);
-  else if (a->ldx <= 2048) launch_pair_norm<2>(a, s);
-  else if (a->ldx <= 4096) launch_pair_norm<4>(a, s);
-  else if (a->ldx <= 8192) launch_pair_norm<8>(a, s);
-  else launch_pair_norm<16>(a, s);
+  if (a->ldx <= 1024) launch_pair_norm<256, 1>(a, s);
+  else if (a->t <= 64 && a->ldx <= 4096) launch_pair_norm<1024, 1>(a, s);
+  else if (a->t <= 64 && a->ldx <= 8192) launch_pair_norm<1024, 2>(a, s);
+  else if (a->ldx <= 2048) launch_pair_norm<256, 2>(a, s);
+  else if (a->ldx <= 4096) launch_pair_norm<256, 4>(a, s);
+  else if (a->ldx <= 8192) launch_pair_norm<256, 8>(a, s);
+  else launch_pair_norm<1024, 4>(a, s);
   CHATTS_CHECK_LAUNCH("pair_norm");
   return CHATTS_OK;
 }

@@ -142,42 +142,44 @@ __global__ __launch_bounds__(256) void recur_tanh_kernel(ChattsRecurArgs p, Chat
   store_operand4(out, row, c, v);
 }
 
-// mlstm: a wave = one head of one span, 64 tokens at a time.  (sum of f, running maximum) pairs combine associatively:
+// mlstm: a workgroup = one head of one span, 1024 tokens at a time.  (sum of f, running maximum) pairs combine associatively:
 // m_t = max(m_0 + F_t, M_t) with (F, M) o (F', M') = (F + F', max(M + F', M')).
-__global__ __launch_bounds__(64) void recur_gates_kernel(ChattsRecurArgs p) {
+__global__ __launch_bounds__(1024) void recur_gates_kernel(ChattsRecurArgs p) {
+  __shared__ float wf[16], wm[16];
   const ChattsSpan sp = p.spans[blockIdx.y];
-  const int h = blockIdx.x, lane = threadIdx.x;
+  const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   if (sp.t < 1) return;
   float m0 = sp.pos0 > 0 ? p.m_state[(size_t)sp.slot * p.heads + h] : 0.f;
   const float bi = p.bias_i[h], bf = p.bias_f[h];
-  float ni = 0.f, nf = 0.f;
-  auto request = [&](int t0) {
-    const int t = t0 + lane < sp.t ? t0 + lane : sp.t - 1;
-    const float* pr = p.proj + (size_t)(sp.row0 + t) * p.ld_proj;
-    ni = pr[p.off_i + h];
-    nf = pr[p.off_f + h];
-  };
-  request(0);
-  for (int t0 = 0; t0 < sp.t; t0 += 64) {
-    const bool ok = t0 + lane < sp.t;
-    const float i = ok ? p.cap * tanhf((ni + bi) / p.cap) : -INFINITY, f = ok ? -softplus_f(-p.cap * tanhf((nf + bf) / p.cap)) : 0.f;
-    if (t0 + 64 < sp.t) request(t0 + 64);
+  for (int t0 = 0; t0 < sp.t; t0 += 1024) {
+    const int t = t0 + tid;
+    const bool ok = t < sp.t;
+    const float* pr = p.proj + (size_t)(sp.row0 + (ok ? t : sp.t - 1)) * p.ld_proj;
+    const float i = ok ? p.cap * tanhf((pr[p.off_i + h] + bi) / p.cap) : -INFINITY, f = ok ? -softplus_f(-p.cap * tanhf((pr[p.off_f + h] + bf) / p.cap)) : 0.f;
     float F = f, M = i;
 #pragma unroll
     for (int d = 1; d < 64; d <<= 1) {
       const float F1 = __shfl_up(F, d, 64), M1 = __shfl_up(M, d, 64);
       if (lane >= d) { M = fmaxf(M1 + F, M); F += F1; }
     }
-    const float m = fmaxf(m0 + F, M);
+    __syncthreads();
+    if (lane == 63) { wf[wave] = F; wm[wave] = M; }
+    __syncthreads();
+    float mw = m0, end = m0;      // the running maximum before this wave's tokens, after all of them
+    for (int w = 0; w < 16; ++w) {
+      if (w == wave) mw = end;
+      end = fmaxf(end + wf[w], wm[w]);
+    }
+    const float m = fmaxf(mw + F, M);
     float before = __shfl_up(m, 1, 64);
-    if (lane == 0) before = m0;
+    if (lane == 0) before = mw;
     if (ok) {
       const f32x4 g = {exp_hw(f + before - m), exp_hw(i - m), exp_hw(-m), 0.f};
-      *reinterpret_cast<f32x4*>(p.gates + ((size_t)(sp.row0 + t0 + lane) * p.heads + h) * 4) = g;
+      *reinterpret_cast<f32x4*>(p.gates + ((size_t)(sp.row0 + t) * p.heads + h) * 4) = g;
     }
-    m0 = __shfl(m, 63, 64);
+    m0 = end;
   }
-  if (lane == 0) p.m_state[(size_t)sp.slot * p.heads + h] = m0;
+  if (tid == 0) p.m_state[(size_t)sp.slot * p.heads + h] = m0;
 }
 
 // With G_t = g_0 .. g_t from the chunk's start and D(s, t) = g_{s+1} .. g_t (every product runs forward: factors <= 1, nothing is divided), a chunk
@@ -575,7 +577,7 @@ extern "C" int chatts_recur_scan(const ChattsRecurArgs* a, chatts_stream_t strea
   if (wkv) {
     launch_recur_scan<CHATTS_RECUR_WKV>(a, as_stream(stream));
   } else {
-    hipLaunchKernelGGL(recur_gates_kernel, dim3(a->heads, a->n_spans), dim3(64), 0, as_stream(stream), *a);
+    hipLaunchKernelGGL(recur_gates_kernel, dim3(a->heads, a->n_spans), dim3(1024), 0, as_stream(stream), *a);
     CHATTS_CHECK_LAUNCH("recur_gates");
     launch_recur_scan<CHATTS_RECUR_MLSTM>(a, as_stream(stream));
   }

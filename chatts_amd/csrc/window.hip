@@ -45,7 +45,7 @@ __device__ __forceinline__ CT to_page(float v) {
   else return __builtin_bit_cast(uint16_t, (__bf16)v);
 }
 
-// grid (rows): a wave takes heads [q | k | v] in turn
+// grid (rows, n): the 4 n waves of a row take heads [q | k | v] in turn
 template <typename CT>
 __global__ __launch_bounds__(256) void window_prep_kernel(ChattsWindowArgs p) {
   const int row = blockIdx.x, lane = threadIdx.x & 63;
@@ -53,7 +53,7 @@ __global__ __launch_bounds__(256) void window_prep_kernel(ChattsWindowArgs p) {
   if (R.pos < 0) return;
   const int H = p.heads, G = p.kv_heads;
   const float* pr = p.proj + (size_t)row * p.ld_proj;
-  for (int e = threadIdx.x >> 6; e < H + 2 * G; e += 4) {
+  for (int e = blockIdx.y * 4 + (threadIdx.x >> 6); e < H + 2 * G; e += 4 * gridDim.y) {
     const bool value = e >= H + G;
     const int hk = e < H ? 0 : (value ? e - H - G : e - H), n = value ? p.vdim : p.dim, np = value ? p.vdim_p : p.dim_p;
     const float* x = pr + (e < H ? p.off_q + e * p.dim : (value ? p.off_v + hk * p.vdim : p.off_k + hk * p.dim));
@@ -160,32 +160,33 @@ __global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) 
   const float scale2 = p.scale * 1.44269504088896341f;
   constexpr int VP = (NV * 32 * 16 + 511) / 512;      // 16-byte pieces of a value tile per lane
   const int vc = p.vdim_p >> 3, pieces = 32 * vc;
-  for (int i = split * 4 + wave; i < n; i += stride) {
+  struct Tile { bf16x8_t k[2][NK]; u32x4 v[VP]; };
+  auto request = [&](int i, Tile& t) __attribute__((always_inline)) {
     const int k0 = T.tile(i) * 32;
     const size_t at = window_tile(p, R.slot, hk, k0);
     const uint16_t* kt = reinterpret_cast<const uint16_t*>(p.kcache) + at * p.dim_p;
     const uint16_t* vt = reinterpret_cast<const uint16_t*>(p.vcache) + at * p.vdim_p;
-    bf16x8_t kf[2][NK];
 #pragma unroll
     for (int k = 0; k < NK; ++k)
       if (k < nk) {
-        kf[0][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)fr * p.dim_p + k * 32 + fg * 8);
-        kf[1][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)(16 + fr) * p.dim_p + k * 32 + fg * 8);
+        t.k[0][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)fr * p.dim_p + k * 32 + fg * 8);
+        t.k[1][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)(16 + fr) * p.dim_p + k * 32 + fg * 8);
       }
-    u32x4 rv[VP];
 #pragma unroll
     for (int e = 0; e < VP; ++e) {
       const int x = e * 64 + lane;
-      const int key = x / vc;
-      rv[e] = (u32x4){0u, 0u, 0u, 0u};
-      if (x < pieces && k0 + key <= R.pos) rv[e] = *reinterpret_cast<const u32x4*>(vt + (size_t)x * 8);      // (a row never written may hold anything)
+      t.v[e] = (u32x4){0u, 0u, 0u, 0u};
+      if (x < pieces && k0 + x / vc <= R.pos) t.v[e] = *reinterpret_cast<const u32x4*>(vt + (size_t)x * 8);      // (a row never written may hold anything)
     }
+  };
+  auto use = [&](int i, const Tile& t) __attribute__((always_inline)) {
+    const int k0 = T.tile(i) * 32;
     f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int k = 0; k < NK; ++k)
       if (k < nk) {
-        s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0][k], q[k], s[0], 0, 0, 0);
-        s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][k], q[k], s[1], 0, 0, 0);
+        s[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(t.k[0][k], q[k], s[0], 0, 0, 0);
+        s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(t.k[1][k], q[k], s[1], 0, 0, 0);
       }
     float v[8], mx = -INFINITY;
 #pragma unroll
@@ -210,7 +211,7 @@ __global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) 
 #pragma unroll
     for (int e = 0; e < VP; ++e) {
       const int x = e * 64 + lane, key = x / vc;
-      if (x < pieces) *reinterpret_cast<u32x4*>(vs + key * ldv + (x - key * vc) * 8) = rv[e];
+      if (x < pieces) *reinterpret_cast<u32x4*>(vs + key * ldv + (x - key * vc) * 8) = t.v[e];
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     const uint16_t* t0 = vs + (fg * 4 + (fr >> 2)) * ldv + (fr & 3) * 4;
@@ -225,6 +226,26 @@ __global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) 
         o[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pf, o[f], 0, 0, 0);
       }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // this tile has been read before the next one is written
+  };
+  const int first = split * 4 + wave;
+  if constexpr (NK <= 4) {      // the next tile travels while this one is multiplied
+    Tile t[2];
+    if (first < n) request(first, t[0]);
+    for (int i = first; i < n; i += 2 * stride) {
+      if (i + stride < n) request(i + stride, t[1]);
+      __builtin_amdgcn_sched_barrier(0);
+      use(i, t[0]);
+      if (i + stride >= n) break;
+      if (i + 2 * stride < n) request(i + 2 * stride, t[0]);
+      __builtin_amdgcn_sched_barrier(0);
+      use(i + stride, t[1]);
+    }
+  } else {
+    Tile t;
+    for (int i = first; i < n; i += stride) {
+      request(i, t);
+      use(i, t);
+    }
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
@@ -533,8 +554,10 @@ using namespace chatts;
 extern "C" int chatts_window_prep(const ChattsWindowArgs* a, chatts_stream_t stream) {
   if (const int rc = check_window(a, "window_prep")) return rc;
   if (a->n_rows == 0) return CHATTS_OK;
-  if (a->cache_f32) hipLaunchKernelGGL(window_prep_kernel<float>, dim3(a->n_rows), dim3(256), 0, as_stream(stream), *a);
-  else hipLaunchKernelGGL(window_prep_kernel<uint16_t>, dim3(a->n_rows), dim3(256), 0, as_stream(stream), *a);
+  int per_row = (a->heads + 2 * a->kv_heads + 3) / 4;
+  if (per_row > 8192 / a->n_rows) per_row = 8192 / a->n_rows > 1 ? 8192 / a->n_rows : 1;
+  if (a->cache_f32) hipLaunchKernelGGL(window_prep_kernel<float>, dim3(a->n_rows, per_row), dim3(256), 0, as_stream(stream), *a);
+  else hipLaunchKernelGGL(window_prep_kernel<uint16_t>, dim3(a->n_rows, per_row), dim3(256), 0, as_stream(stream), *a);
   CHATTS_CHECK_LAUNCH("window_prep");
   return CHATTS_OK;
 }

@@ -405,6 +405,13 @@ class MixedDecoder(SlotModel):
             w[:, j] = _pad(t.to(torch.bfloat16), ff, self._wp).view(ff // 16, 16, self._wp)
         return w.view(2 * ff, self._wp)
 
+    def _tiles(self, t):
+        """chatts_tile_bf16 copies of [n, rows, cols], one after the other"""
+        out = torch.empty_like(t)
+        for e in range(t.shape[0]):
+            _lib.check(self.lib.chatts_tile_bf16(t[e].data_ptr(), t.shape[1], t.shape[2], t.shape[2], out[e].data_ptr(), _lib.stream_ptr()))
+        return self._dev(out)
+
     def _glu(self, L, m):
         L.ff_kind, L.ff, L.glu_limit, L.glu_alpha = _lib.FF_CLAMPGLU, _up(m.gate.shape[0], 64), m.limit, m.alpha
         L.up, L.up_t = self._mat(self._gate_up(m.gate, m.up, L.ff), tile=True)
@@ -416,10 +423,11 @@ class MixedDecoder(SlotModel):
         dn = torch.empty((n, self._wp, ff), dtype=torch.bfloat16, device=self.device)
         for e, (gate, up, down) in enumerate(m.experts):
             gu[e], dn[e] = self._gate_up(gate, up, ff), _pad(down.to(torch.bfloat16), self._wp, ff)
+        gut, dnt = (self._tiles(t) if self.tiled else None for t in (gu, dn))
         L.ff_kind, L.router_n = _lib.FF_MOE, _up(n + m.identity, 64)
         L.router, L.router_t = self._mat(m.router, L.router_n, self._wp, tile=True)
         L.moe = _lib.MoeArgs(experts=n, identity=m.identity, top=m.top, groups=m.groups, keep=m.keep, width_p=self._wp, ff_p=ff, gate_up=self._dev(gu),
-                             down=self._dev(dn), correction=self._f32(m.correction))
+                             down=self._dev(dn), gate_up_t=gut, down_t=dnt, correction=self._f32(m.correction))
 
     def _build(self, sd):
         cfg, lib, dev = self.config, self.lib, self.device
@@ -538,7 +546,7 @@ class MixedDecoder(SlotModel):
             "gates": torch.zeros((rows, 4 * over(recurs, lambda L: L.recur.heads)), **f32), "den": torch.zeros((rows, over(recurs, lambda L: L.recur.heads)), **f32),
             "moe_ids": torch.zeros(pairs, dtype=torch.int32, device=dev), "moe_place": torch.zeros(pairs, dtype=torch.int32, device=dev),
             "moe_order": torch.zeros(pairs, dtype=torch.int32, device=dev),
-            "moe_offsets": torch.zeros(over(moes, lambda L: L.moe.experts) + 1, dtype=torch.int32, device=dev),
+            "moe_offsets": torch.zeros(over(moes, lambda L: L.moe.experts) + 2, dtype=torch.int32, device=dev),
             "moe_tiles": torch.zeros(4 * over(moes, lambda L: int(lib.chatts_moe_tiles(T, L.moe.top, L.moe.experts))), dtype=torch.int32, device=dev),
             "moe_weight": torch.zeros(pairs, **f32), "moe_kept": torch.zeros(rows, **f32), "moe_logits": torch.zeros((rows, over(moes, lambda L: L.router_n)), **f32),
             "moe_y": torch.zeros((pairs, Wp) if moes else (1, 1), **f32),

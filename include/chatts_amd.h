@@ -229,10 +229,17 @@ typedef struct ChattsLinearArgs {
    * always).  Needs float32 `a` and `c`, bf16 `w`; no planes, no fused norm.  For 32-bit runs of a model, not a fast path. */
   int exact_f32;
   float glu_limit, glu_alpha;      /* EPI_CLAMPGLU */
+  /* optional: `batch` products of one shape, member i with a / a_hi / a_lo + i * a_stride, w + i * w_stride, c / c_hi / c_lo + i * c_stride (elements;
+   * EPI_NONE, no bias, no further options).  One launch for few rows (M == 1, 2 <= M <= 16 with planes), one per member otherwise.
+   * 0 or 1: one product. */
+  int batch;
+  int64_t a_stride, w_stride, c_stride;
+  const chatts_bf16* const* w_tiled_batch;   /* host: w_tiled of every member, or NULL */
 } ChattsLinearArgs;
 #define CHATTS_W8_FP8 0
 #define CHATTS_W8_INT8 1
 size_t chatts_linear_workspace(int m, int n, int k);
+size_t chatts_linear_workspace_batch(int m, int n, int k, int batch);
 /* Host-only query (no device work): how many waves share a row group of the M == 1 bf16 GEMV for this shape on the current device
  * (1 = the whole-K kernel every TP = 1 projection of the supported models runs; > 1 = the K-split form of shard-sized column-parallel
  * projections, which sums a row in another order).  Lets a host-side test pin which shapes take which kernel. */
@@ -1008,13 +1015,14 @@ typedef struct ChattsMoeArgs {
   int width_p, ff_p;                    /* both % 64 == 0 */
   const chatts_bf16* gate_up;           /* [experts][2 ff_p][width_p], gate / up rows interleaved in blocks of 16 */
   const chatts_bf16* down;              /* [experts][width_p][ff_p] */
+  const chatts_bf16 *gate_up_t, *down_t;   /* chatts_tile_bf16 copy of every matrix, one after the other, or NULL */
   const float* correction;              /* [experts + identity] */
   const float* logits;                  /* [T, ld_logits] */
   int ld_logits;
   ChattsOperand h;                      /* planes, or float32 when exact */
   const ChattsRow* rows;
   int n_rows, exact;
-  int32_t *ids, *place, *order, *offsets, *tiles;   /* [T, top], [T, top], [T * top], [experts + 1], chatts_moe_tiles() * 4 */
+  int32_t *ids, *place, *order, *offsets, *tiles;   /* [T, top], [T, top], [T * top], [experts + 2] (.., places in use, tiles), chatts_moe_tiles() * 4 */
   float *weight, *kept;                 /* [T, top], [T] (weight of the identity outputs) */
   ChattsOperand act;                    /* [T * top, ff_p] */
   float* y;                             /* [T * top, width_p] */

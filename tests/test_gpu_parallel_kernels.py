@@ -451,7 +451,7 @@ def test_experts(case, T, exact):
     parked = T == 7
     rows = torch.tensor([[i, -1 if parked and i == 2 else 5, i, 0] for i in range(T)], dtype=torch.int32, device=DEV)
     I = lambda n: torch.full((n,), -7, dtype=torch.int32, device=DEV)
-    ids, place, order, offsets, tiles = I(T * top), I(T * top), I(T * top), I(E + 1), I(4 * int(_lib.load().chatts_moe_tiles(T, top, E)))
+    ids, place, order, offsets, tiles = I(T * top), I(T * top), I(T * top), I(E + 2), I(4 * int(_lib.load().chatts_moe_tiles(T, top, E)))
     weight, kept, y = torch.zeros(T, top, device=DEV), torch.zeros(T, device=DEV), torch.zeros(T * top, Wp, device=DEV)
     act = torch.zeros(T * top, fp, device=DEV) if exact else torch.zeros(2, T * top, fp, dtype=torch.bfloat16, device=DEV)
     gud, dnd, cd = gu.to(DEV), dn.to(DEV), sd["correction"].to(DEV)
@@ -497,3 +497,26 @@ def test_linear_clamp_glu(m, exact, n, k):
         hp, out = planes_of(ad), torch.zeros(2, m, n, dtype=torch.bfloat16, device=DEV)
         call("chatts_linear", _lib.LinearArgs(a_hi=hp[0].data_ptr(), a_lo=hp[1].data_ptr(), ld_planes=k, c_hi=out[0].data_ptr(), c_lo=out[1].data_ptr(), ld_cplanes=n, **kw))
         assert rel(out[0].float() + out[1].float(), want) < 4e-5
+
+
+# ---- several projections of one shape ---------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("m", [1, 2, 16, 40, 130])
+@pytest.mark.parametrize("exact", [0, 1])
+@pytest.mark.parametrize("n,k", [(64, 128), (192, 2048)])
+def test_linear_batch(m, exact, n, k):
+    g, B = gen(m), 3
+    a, w = torch.randn(B, m + 1, k, generator=g), (torch.randn(B, n, k, generator=g) / math.sqrt(k)).to(torch.bfloat16)
+    want = torch.stack([a[i, :m].double() @ w[i].double().T for i in range(B)], 1)
+    ad, wd = a.to(DEV), w.to(DEV)
+    ws = torch.zeros(max(16, int(_lib.load().chatts_linear_workspace_batch(m, n, k, B))), dtype=torch.uint8, device=DEV)
+    kw = dict(w=wd.data_ptr(), m=m, n=n, k=k, ldw=k, ldc=B * n + 64, epilogue=_lib.EPI_NONE, exact_f32=exact, workspace=ws.data_ptr(), workspace_bytes=ws.numel(), batch=B,
+              a_stride=(m + 1) * k, w_stride=n * k, c_stride=n)
+    forms = [dict(a=ad.data_ptr(), lda=k)]
+    if m > 1 and not exact:
+        hp = planes_of(ad)
+        forms.append(dict(a_hi=hp[0].data_ptr(), a_lo=hp[1].data_ptr(), ld_planes=k))
+    for f in forms:
+        c = torch.zeros(m, B * n + 64, device=DEV)
+        call("chatts_linear", _lib.LinearArgs(c=c.data_ptr(), **f, **kw))
+        assert rel(c[:, :B * n].reshape(m, B, n), want) < (1e-6 if exact or m == 1 else 2e-5)
+        assert float(c[:, B * n:].abs().sum()) == 0
