@@ -337,11 +337,13 @@ static int mix_window(const ChattsMixDecoder* d, const ChattsMixLayer& l, const 
     if (spans[i].t > a.longest) a.longest = spans[i].t;
   if (const int rc = chatts_window_prep(&a, s)) return rc;
   if (a.longest >= 8 && !d->c.exact && chatts_window_can_prefill(a.dim_p, a.vdim_p)) return chatts_window_prefill(&a, s);
-  if (!d->c.exact) {      // few rows: a row's tiles (32 keys a wave, 4 waves) are spread over workgroups until there are about two per CU
+  if (!d->c.exact) {      // few rows: a row's tiles (32 keys a wave, 4 waves) are spread over workgroups, about three per CU, the same number to every wave
     const int group = a.heads / a.kv_heads, wgs = a.kv_heads * ((group + 15) / 16) * t;
-    const int keys = a.window > 0 && a.window + a.keep_first < d->c.max_ctx ? a.window + a.keep_first : d->c.max_ctx, most = (keys / 32 + 3) / 4;
-    int splits = (2 * device_cus() + wgs - 1) / wgs;
-    if (splits > most) splits = most;
+    const int tiles = (a.window > 0 && a.window + a.keep_first + 64 < d->c.max_ctx ? a.window + a.keep_first + 64 : d->c.max_ctx) / 32;
+    int splits = 3 * device_cus() / wgs;
+    if (splits < 1) splits = 1;
+    const int each = (tiles + 4 * splits - 1) / (4 * splits);
+    splits = (tiles + 4 * each - 1) / (4 * each);
     if (splits > 64) splits = 64;
     while (splits > 1 && (size_t)t * a.heads * splits * (a.vdim_p + 4) > d->b.partial_elems) --splits;
     a.n_splits = splits < 1 ? 1 : splits;

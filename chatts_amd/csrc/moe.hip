@@ -214,7 +214,8 @@ __device__ __forceinline__ float moe_glu(float g, float u) { return g * sigmoid_
 
 // ---- up to 16 rows: grid (blocks of 32 weight rows, tiles), 4 waves split K; D = W . A^T: a lane holds 4 consecutive outputs of one token.
 // GLU: the two 16-row halves of a block are gate and up rows of the same outputs ----
-template <bool GLU>
+// TILED: weights from the chatts_tile_bf16 copy: a fragment's 64 pieces are 1 KB of consecutive memory
+template <bool GLU, bool TILED>
 __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
   __shared__ f32x4 red[4][2][64];
   const int32_t* tile = p.tiles + (size_t)blockIdx.y * 4;
@@ -222,7 +223,9 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
   if (e < 0) return;
   const int place0 = tile[1], count = tile[2], lane = threadIdx.x & 63, wave = threadIdx.x >> 6, fr = lane & 15, fg = lane >> 4;
   const int K = GLU ? p.width_p : p.ff_p, N = GLU ? 2 * p.ff_p : p.width_p, n0 = blockIdx.x * 32;
-  const uint16_t* w = (GLU ? p.gate_up : p.down) + ((size_t)e * N + n0 + fr) * K + fg * 8;
+  const uint16_t* w = TILED ? (GLU ? p.gate_up_t : p.down_t) + ((size_t)e * N + n0) * K + (fr * 4 + (fg ^ ((fr >> 3) << 1))) * 8
+                            : (GLU ? p.gate_up : p.down) + ((size_t)e * N + n0 + fr) * K + fg * 8;
+  constexpr int kStep = TILED ? 16 : 1;      // elements of w per K-value
   const int pl = place0 + (fr < count ? fr : 0);
   const size_t arow = GLU ? (size_t)(p.order[pl] / p.top) * p.h.ld : (size_t)pl * p.act.ld;
   const uint16_t* ah = (GLU ? p.h.hi : p.act.hi) + arow + fg * 8;
@@ -235,7 +238,7 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
 #pragma unroll
     for (int u = 0; u < U; ++u) {
       const int k = k0 + 4 * u < steps ? (k0 + 4 * u) * 32 : 0;
-      const u32x4 a = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + k)), b = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + (size_t)16 * K + k));
+      const u32x4 a = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + k * kStep)), b = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + (size_t)16 * K + k * kStep));
       wv[u][0] = __builtin_bit_cast(bf16x8_t, a);
       wv[u][1] = __builtin_bit_cast(bf16x8_t, b);
     }
@@ -503,8 +506,11 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
     return CHATTS_OK;
   }
   if (moe_small(a)) {
-    hipLaunchKernelGGL(moe_stream_kernel<true>, dim3(2 * a->ff_p / 32, tiles), dim3(256), 0, s, *a);
-    hipLaunchKernelGGL(moe_stream_kernel<false>, dim3(a->width_p / 32, tiles), dim3(256), 0, s, *a);
+    const dim3 g1(2 * a->ff_p / 32, tiles), g2(a->width_p / 32, tiles), b(256);
+    if (a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<true, true>), g1, b, 0, s, *a);
+    else hipLaunchKernelGGL((moe_stream_kernel<true, false>), g1, b, 0, s, *a);
+    if (a->down_t) hipLaunchKernelGGL((moe_stream_kernel<false, true>), g2, b, 0, s, *a);
+    else hipLaunchKernelGGL((moe_stream_kernel<false, false>), g2, b, 0, s, *a);
     CHATTS_CHECK_LAUNCH("moe_stream");
     return CHATTS_OK;
   }

@@ -233,9 +233,12 @@ __global__ __launch_bounds__(256) void recur_chunk_kernel(ChattsRecurArgs p) {
   {
     // P: thread = (token s, 1 / 16 of the channels), w = D(s, t) k_s walks forward in t
     const int s = tid >> 4, l16 = tid & 15;
-    f32x4 w[NC];
+    f32x4 w[NC], own[NC];
 #pragma unroll
-    for (int c = 0; c < NC; ++c) w[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int c = 0; c < NC; ++c) {
+      w[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      own[c] = *reinterpret_cast<const f32x4*>(&sk[s][c * 64 + l16 * 4]);
+    }
     float kp = 0.f;      // of token t = l16
 #pragma unroll 4
     for (int t = 0; t < kRcChunk; ++t) {
@@ -244,16 +247,16 @@ __global__ __launch_bounds__(256) void recur_chunk_kernel(ChattsRecurArgs p) {
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
         const int ch = c * 64 + l16 * 4;
-        const f32x4 k = *reinterpret_cast<const f32x4*>(&sk[t][ch]), q = *reinterpret_cast<const f32x4*>(&sq[t][ch]);
+        const f32x4 q = *reinterpret_cast<const f32x4*>(&sq[t][ch]);
         f32x4 g = {a, a, a, a};
         if constexpr (WKV) g = *reinterpret_cast<const f32x4*>(&sg[t][ch]);
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           if constexpr (WKV) {
             b += q[j] * w[c][j];
-            w[c][j] = t == s ? k[j] : w[c][j] * g[j];
+            w[c][j] = t == s ? own[c][j] : w[c][j] * g[j];
           } else {
-            w[c][j] = t == s ? k[j] : w[c][j] * g[j];
+            w[c][j] = t == s ? own[c][j] : w[c][j] * g[j];
             b += q[j] * w[c][j];
           }
         }

@@ -135,16 +135,17 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
 
 // ---- one row on the matrix pipe: grid (splits, kv heads * head tiles, rows), 4 waves ----
 // A wave walks tiles of 32 keys on its own (tiles 4 split + wave, ...): S^T = K Q^T with the key rows straight from memory as A fragments, so that a
-// lane ends up with 8 scores of one head (column = lane & 15); O^T = V^T P^T with V through a private piece of LDS and transposing reads - its B
+// lane ends up with 8 scores of one head (column = lane & 15); O^T = V^T P^T with V through a private piece of LDS (LDS-DMA) and transposing reads - its B
 // fragment IS the 8 probabilities of the lane (K slot 8 g + j = key 4 g + j, j < 4, or 16 + 4 g + j - 4, on both sides).  The waves' softmaxes meet once.
 template <int NK, int NV>      // dim_p <= 32 NK, vdim_p <= 16 NV
-__global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) {
+__global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_decode_kernel(ChattsWindowArgs p) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int split = blockIdx.x, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const int split = blockIdx.x, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, fr = lane & 15, fg = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const ChattsRow R = p.rows[row];
   if (R.pos < 0) return;
   const int group = p.heads / p.kv_heads, htiles = (group + 15) / 16, hk = blockIdx.y / htiles, h0 = (blockIdx.y - hk * htiles) * 16;
-  const int nk = p.dim_p >> 5, nv = p.vdim_p >> 4, ldv = p.vdim_p + 16;
+  const int nk = p.dim_p >> 5, nv = p.vdim_p >> 4, ldv = p.vdim_p;
   const int hl = h0 + fr < group ? h0 + fr : group - 1, head = hk * group + hl;
   uint16_t* vs = reinterpret_cast<uint16_t*>(smem) + wave * 32 * ldv;
   bf16x8_t q[NK];
@@ -158,9 +159,10 @@ __global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) 
 #pragma unroll
   for (int i = 0; i < NV; ++i) o[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
   const float scale2 = p.scale * 1.44269504088896341f;
-  constexpr int VP = (NV * 32 * 16 + 511) / 512;      // 16-byte pieces of a value tile per lane
-  const int vc = p.vdim_p >> 3, pieces = 32 * vc;
-  struct Tile { bf16x8_t k[2][NK]; u32x4 v[VP]; };
+  constexpr int VP = NV;      // LDS-DMA requests of a value tile: 64 pieces of 16 bytes each
+  // 16-byte piece c of row r lies at position c ^ (r & sw): the transposing reads of neighbouring rows meet different banks
+  const int vc = p.vdim_p >> 3, sw = (vc & 7) == 0 ? 7 : ((vc & 3) == 0 ? 3 : 1);
+  struct Tile { bf16x8_t k[2][NK]; };
   auto request = [&](int i, Tile& t) __attribute__((always_inline)) {
     const int k0 = T.tile(i) * 32;
     const size_t at = window_tile(p, R.slot, hk, k0);
@@ -169,15 +171,15 @@ __global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) 
 #pragma unroll
     for (int k = 0; k < NK; ++k)
       if (k < nk) {
-        t.k[0][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)fr * p.dim_p + k * 32 + fg * 8);
-        t.k[1][k] = *reinterpret_cast<const bf16x8_t*>(kt + (size_t)(16 + fr) * p.dim_p + k * 32 + fg * 8);
+        t.k[0][k] = *reinterpret_cast<const bf16x8_t*>(kt + (uint32_t)(fr * p.dim_p + k * 32 + fg * 8));
+        t.k[1][k] = *reinterpret_cast<const bf16x8_t*>(kt + (uint32_t)((16 + fr) * p.dim_p + k * 32 + fg * 8));
       }
 #pragma unroll
-    for (int e = 0; e < VP; ++e) {
-      const int x = e * 64 + lane;
-      t.v[e] = (u32x4){0u, 0u, 0u, 0u};
-      if (x < pieces && k0 + x / vc <= R.pos) t.v[e] = *reinterpret_cast<const u32x4*>(vt + (size_t)x * 8);      // (a row never written may hold anything)
-    }
+    for (int e = 0; e < VP; ++e)
+      if (e * 64 < 32 * vc) {      // (uniform: a tile is a whole number of requests)
+        const int x = e * 64 + lane, r = x / vc, c = x - r * vc;
+        __builtin_amdgcn_global_load_lds((gptr_t)(vt + (uint32_t)(r * p.vdim_p + ((c ^ (r & sw)) << 3))), (lptr_t)(vs + e * 512), 16, 0, 0);
+      }
   };
   auto use = [&](int i, const Tile& t) __attribute__((always_inline)) {
     const int k0 = T.tile(i) * 32;
@@ -208,44 +210,30 @@ __global__ __launch_bounds__(256) void window_decode_kernel(ChattsWindowArgs p) 
       pf[j] = (__bf16)e;
     }
     l = l * alpha + sum;
-#pragma unroll
-    for (int e = 0; e < VP; ++e) {
-      const int x = e * 64 + lane, key = x / vc;
-      if (x < pieces) *reinterpret_cast<u32x4*>(vs + key * ldv + (x - key * vc) * 8) = t.v[e];
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // the values have landed
+    const int lim = R.pos + 1 - k0;
+    if (lim < 32) {      // rows never written may hold anything: zeros
+      for (int x = lim * vc + lane; x < 32 * vc; x += 64) *reinterpret_cast<u32x4*>(vs + x * 8) = (u32x4){0u, 0u, 0u, 0u};
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     }
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    const uint16_t* t0 = vs + (fg * 4 + (fr >> 2)) * ldv + (fr & 3) * 4;
+    const int tr = fg * 4 + (fr >> 2), swz = tr & sw, cb = (fr >> 1) & 1;
+    const uint16_t* t0 = vs + tr * ldv + (fr & 1) * 4;
 #pragma unroll
     for (int f = 0; f < NV; ++f)
       if (f < nv) {
         union { w16x4 h[2]; bf16x8_t v; } a;
-        a.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + f * 16));
-        a.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + 16 * ldv + f * 16));
+        a.h[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + (((2 * f + cb) ^ swz) << 3)));
+        a.h[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_w16x4)(t0 + 16 * ldv + (((2 * f + cb) ^ swz) << 3)));
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[f][r] *= alpha;
         o[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pf, o[f], 0, 0, 0);
       }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // this tile has been read before the next one is written
   };
-  const int first = split * 4 + wave;
-  if constexpr (NK <= 4) {      // the next tile travels while this one is multiplied
-    Tile t[2];
-    if (first < n) request(first, t[0]);
-    for (int i = first; i < n; i += 2 * stride) {
-      if (i + stride < n) request(i + stride, t[1]);
-      __builtin_amdgcn_sched_barrier(0);
-      use(i, t[0]);
-      if (i + stride >= n) break;
-      if (i + 2 * stride < n) request(i + 2 * stride, t[0]);
-      __builtin_amdgcn_sched_barrier(0);
-      use(i + stride, t[1]);
-    }
-  } else {
-    Tile t;
-    for (int i = first; i < n; i += stride) {
-      request(i, t);
-      use(i, t);
-    }
+  Tile t;
+  for (int i = split * 4 + wave; i < n; i += stride) {
+    request(i, t);
+    use(i, t);
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
@@ -529,11 +517,11 @@ static int window_lds(K kernel, size_t bytes, bool& done) {
 template <int NK, int NV>
 static int launch_window_decode(const ChattsWindowArgs* a, hipStream_t s) {
   static bool done = false;
-  const size_t most = 4 * 16 * (NV * 16 + 4) * 4 > 4 * 32 * (NV * 16 + 16) * 2 ? 4 * 16 * (NV * 16 + 4) * 4 : 4 * 32 * (NV * 16 + 16) * 2;
+  const size_t most = (size_t)4 * 16 * (NV * 16 + 4) * 4;      // the waves' meeting; their value tiles (4 x 32 x vdim_p bf16) are smaller
   if (const int rc = window_lds(&window_decode_kernel<NK, NV>, most, done)) return rc;
-  const size_t tiles = (size_t)4 * 32 * (a->vdim_p + 16) * 2, meet = (size_t)4 * 16 * (a->vdim_p + 4) * 4;
   const int group = a->heads / a->kv_heads;
-  hipLaunchKernelGGL((window_decode_kernel<NK, NV>), dim3(a->n_splits, a->kv_heads * ((group + 15) / 16), a->n_rows), dim3(256), tiles > meet ? tiles : meet, s, *a);
+  hipLaunchKernelGGL((window_decode_kernel<NK, NV>), dim3(a->n_splits, a->kv_heads * ((group + 15) / 16), a->n_rows), dim3(256),
+                     (size_t)4 * 16 * (a->vdim_p + 4) * 4, s, *a);
   CHATTS_CHECK_LAUNCH("window_decode");
   return CHATTS_OK;
 }

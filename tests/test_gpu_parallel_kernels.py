@@ -460,18 +460,29 @@ def test_experts(case, T, exact):
                      exact=exact, ids=ids.data_ptr(), place=place.data_ptr(), order=order.data_ptr(), offsets=offsets.data_ptr(), tiles=tiles.data_ptr(),
                      weight=weight.data_ptr(), kept=kept.data_ptr(), act=operand(act if exact else None, None if exact else act, fp), y=y.data_ptr())
     call("chatts_moe_route", a)
-    ids, place = ids.view(T, top).cpu(), place.view(T, top).cpu()
+    chosen, at = ids.view(T, top).cpu(), place.view(T, top).cpu()
     live = [t for t in range(T) if not (parked and t == 2)]
     for t in live:
-        assert sorted(i for i in ids[t].tolist() if i >= 0) == sorted(i for i in idx[t].tolist() if i < E)
+        assert sorted(i for i in chosen[t].tolist() if i >= 0) == sorted(i for i in idx[t].tolist() if i < E)
     if parked:
-        assert (ids[2] == -1).all() and (place[2] == -1).all() and float(kept[2]) == 0
-    used = place[place >= 0].tolist()
+        assert (chosen[2] == -1).all() and (at[2] == -1).all() and float(kept[2]) == 0
+    used = at[at >= 0].tolist()
     assert sorted(used) == list(range(len(used)))                    # the places are packed, experts in order
-    assert torch.equal(ids.view(-1)[order.cpu()[:len(used)].long()], ids.view(-1)[ids.view(-1) >= 0].sort().values)
-    call("chatts_moe_experts", a)
+    assert torch.equal(chosen.view(-1)[order.cpu()[:len(used)].long()], chosen[chosen >= 0].sort().values)
     x = torch.zeros(T, Wp, device=DEV)
-    call("chatts_pair_norm", _lib.PairNormArgs(x=x.data_ptr(), t=T, width=W, ldx=Wp, groups=1, eps=1e-5, y=y.data_ptr(), place=a.place, weight=weight.data_ptr(),
+    tiled = [torch.empty_like(t) for t in (gud, dnd)]
+    for src, dst, n, k in ((gud, tiled[0], 2 * fp, Wp), (dnd, tiled[1], Wp, fp)):
+        for e in range(E):
+            _lib.check(_lib.load().chatts_tile_bf16(src[e].data_ptr(), n, k, k, dst[e].data_ptr(), _lib.stream_ptr()))
+    if not exact:                                                    # the weights' tiled copies: the same products
+        a.gate_up_t, a.down_t = (t.data_ptr() for t in tiled)
+        call("chatts_moe_experts", a)
+        from_tiles = y.clone()
+        y.zero_()
+        a.gate_up_t = a.down_t = None
+    call("chatts_moe_experts", a)
+    assert exact or torch.equal(y, from_tiles)
+    call("chatts_pair_norm", _lib.PairNormArgs(x=x.data_ptr(), t=T, width=W, ldx=Wp, groups=1, eps=1e-5, y=y.data_ptr(), place=place.data_ptr(), weight=weight.data_ptr(),
                                                kept=kept.data_ptr(), h=a.h, top=top))
     assert rel(x.cpu()[live][:, :W], want[live]) < (2e-6 if exact else 5e-5)
     assert float(x[:, W:].abs().sum()) == 0
