@@ -41,11 +41,11 @@ def _digest():
     return h.hexdigest()
 
 
-# AddressSanitizer on the HOST half of the library only ("ASan host build of the shim"): argument validation, the
+# AddressSanitizer on the HOST half of the library only: argument validation, the
 # options table, error strings, geometry choices, handle bookkeeping - everything the C-ABI does before a kernel is enqueued.  GPU ASan
-# needs xnack+ code objects, which this pool refuses; -fno-gpu-sanitize keeps the device code as shipped.
-ASAN_FLAGS = ["--offload-arch=gfx950", "-O1", "-g", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-fsanitize=address",
-              "-fno-gpu-sanitize", "-shared-libsan", "-fno-omit-frame-pointer", *NO_PACKED_FP32]
+# needs xnack+ code objects; -fno-gpu-sanitize keeps the device code as shipped.
+ASAN = ["-fsanitize=address", "-fno-gpu-sanitize", "-shared-libsan"]
+ASAN_FLAGS = ["--offload-arch=gfx950", "-O1", "-g", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", *ASAN, "-fno-omit-frame-pointer", *NO_PACKED_FP32]
 ASAN_LIBDIR = os.path.join(HERE, "lib_asan")
 ASAN_LIB = os.path.join(ASAN_LIBDIR, "libchatts_amd_asan.so")
 
@@ -85,7 +85,7 @@ def build(force=False, verbose=False, asan=False):
         objs = list(ex.map(compile_one, SOURCES))
     cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", lib, *objs, "-ldl"]
     if asan:
-        cmd += ["-fsanitize=address", "-fno-gpu-sanitize", "-shared-libsan"]
+        cmd += ASAN
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
