@@ -10,7 +10,7 @@ from . import build as _build
 _LIB = None
 
 OK, E_BADARG, E_SHAPE, E_COUNT_MISMATCH, E_LAUNCH, E_WORKSPACE = 0, -1, -2, -3, -4, -5
-EPI_NONE, EPI_GELU, EPI_RESID, EPI_SWIGLU, EPI_RELU2, EPI_CLAMPGLU = 0, 1, 2, 3, 4, 5
+EPI_NONE, EPI_GELU, EPI_RESID, EPI_SWIGLU, EPI_RELU2, EPI_CLAMPGLU, EPI_GEGLU = 0, 1, 2, 3, 4, 5, 6
 
 c_void_p, c_int, c_int32, c_int64, c_float, c_size_t, c_uint32 = (
     C.c_void_p, C.c_int, C.c_int32, C.c_int64, C.c_float, C.c_size_t, C.c_uint32)
@@ -29,7 +29,7 @@ class TsWeights(C.Structure):
                 ("b", c_void_p * 8)]
 
 
-ABI_VERSION = 11           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
+ABI_VERSION = 12           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
 W8_FP8, W8_INT8 = 0, 1     # ChattsLinearArgs.w8_format
 
 
@@ -178,6 +178,12 @@ class TokenShiftArgs(C.Structure):
 RECUR_WKV, RECUR_MLSTM = 1, 2
 
 
+class PostNormArgs(C.Structure):
+    """ChattsPostNormArgs: the norm of a sum, in place (csrc/postnorm.hip)"""
+    _fields_ = [("x", c_void_p), ("t", c_int), ("width", c_int), ("ldx", c_int), ("alpha", c_float), ("eps", c_float), ("y", c_void_p), ("ey", c_void_p),
+                ("place", c_void_p), ("weight", c_void_p), ("top", c_int), ("w", c_void_p), ("out", Operand)]
+
+
 class RecurArgs(C.Structure):
     """ChattsRecurArgs: gated linear recurrences (csrc/recur.hip)"""
     _fields_ = ([("kind", c_int), ("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_gate", "off_a", "off_i", "off_f", "heads",
@@ -192,21 +198,25 @@ class WindowArgs(C.Structure):
     """ChattsWindowArgs: grouped-head attention over paged keys and values (csrc/window.hip)"""
     _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_gate", "heads", "kv_heads", "dim", "vdim", "dim_p", "vdim_p")] +
                 [("scale", c_float), ("eps", c_float), ("q_norm", c_void_p), ("k_norm", c_void_p), ("window", c_int), ("keep_first", c_int), ("sink", c_int),
-                 ("kcache", c_void_p), ("vcache", c_void_p), ("cache_f32", c_int), ("table", c_void_p), ("table_stride", c_int), ("log_block", c_int),
+                 ("chunk", c_int), ("softcap", c_float), ("slopes", c_void_p)] + [(n, c_int) for n in ("gate_heads", "norm_whole", "rot", "unit")] +
+                [("cos_tab", c_void_p), ("sin_tab", c_void_p), ("taps", c_int), ("conv_ch", c_int), ("conv_w", c_void_p), ("ring", c_void_p), ("vmix", c_float),
+                 ("vfirst", c_void_p), ("ld_vfirst", c_int), ("vfirst_write", c_int), ("kcache", c_void_p), ("vcache", c_void_p), ("cache_f32", c_int), ("table", c_void_p), ("table_stride", c_int), ("log_block", c_int),
                  ("rows", c_void_p), ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int), ("longest", c_int), ("q", Operand), ("n_splits", c_int),
                  ("partial", c_void_p), ("out", Operand)])
 
 
 class MoeArgs(C.Structure):
     """ChattsMoeArgs: mixture of experts (csrc/moe.hip)"""
-    _fields_ = ([(n, c_int) for n in ("experts", "identity", "top", "groups", "keep", "width_p", "ff_p")] +
+    _fields_ = ([(n, c_int) for n in ("experts", "identity", "top", "groups", "keep", "choose", "act_kind", "width_p", "ff_p")] +
                 [("gate_up", c_void_p), ("down", c_void_p), ("gate_up_t", c_void_p), ("down_t", c_void_p), ("correction", c_void_p), ("logits", c_void_p), ("ld_logits", c_int), ("h", Operand), ("rows", c_void_p),
                  ("n_rows", c_int), ("exact", c_int)] + [(n, c_void_p) for n in ("ids", "place", "order", "offsets", "tiles", "weight", "kept")] +
                 [("act", Operand), ("y", c_void_p)])
 
 
 MIX_LATENT, MIX_DELTA, MIX_RECUR, MIX_WINDOW = 1, 2, 3, 4
-FF_NONE, FF_RELU2, FF_CLAMPGLU, FF_MOE = 0, 1, 2, 3
+FF_NONE, FF_RELU2, FF_CLAMPGLU, FF_MOE, FF_GEGLU = 0, 1, 2, 3, 4
+CHOOSE_SOFTMAX, CHOOSE_LOGITS = 0, 1
+EXPERT_SWIGLU, EXPERT_RELU2 = 0, 1
 EXPAND_PAD = 128           # CHATTS_LATENT_EXPAND_PAD
 
 
@@ -216,7 +226,8 @@ class MixLayer(C.Structure):
                 [(n, c_int) for n in ("in_n", "out_k", "ff")] + [("uk", c_void_p), ("uv", c_void_p), ("ukx", c_void_p), ("uvx", c_void_p)] +
                 [(n, c_int) for n in ("dim_p", "vdim_p", "out_head")] + [("latent", LatentArgs), ("delta", DeltaArgs), ("parallel", c_int), ("ff_kind", c_int),
                  ("glu_limit", c_float), ("glu_alpha", c_float), ("n_mix", c_int), ("mix_row", c_int * 8), ("mix_t", c_void_p * 8), ("mu", c_void_p), ("w2", c_void_p), ("w2_n", c_int),
-                 ("recur", RecurArgs), ("window", WindowArgs), ("router", c_void_p), ("router_t", c_void_p), ("router_n", c_int), ("moe", MoeArgs)])
+                 ("recur", RecurArgs), ("window", WindowArgs), ("router", c_void_p), ("router_t", c_void_p), ("router_n", c_int), ("moe", MoeArgs),
+                 ("post", c_int), ("in_bias", c_void_p)])
 
 
 class MixRun(C.Structure):
@@ -227,7 +238,7 @@ class MixRun(C.Structure):
 class MixConfig(C.Structure):
     _fields_ = ([(n, c_int) for n in ("width", "width_p", "n_layers", "n_runs", "exact", "t_max", "max_slots", "max_ctx", "expand_rows")] +
                 [("vocab", c_int64), ("vocab_p", c_int64), ("eps", c_float), ("block_size", c_int), ("table_stride", c_int), ("norm_groups", c_int),
-                 ("embed_scale", c_float), ("bigram_buckets", c_int64), ("bigram_prev", c_int64), ("bigram_cur", c_int64)])
+                 ("embed_scale", c_float), ("bigram_buckets", c_int64), ("bigram_prev", c_int64), ("bigram_cur", c_int64), ("alpha", c_float)])
 
 
 class MixBuffers(C.Structure):
@@ -238,7 +249,7 @@ class MixBuffers(C.Structure):
                 [("mix_stride", c_int64)] +
                 [(n, c_void_p) for n in ("n_f32", "n_hi", "n_lo", "gates", "den", "moe_ids", "moe_place", "moe_order", "moe_offsets", "moe_tiles", "moe_weight",
                                          "moe_kept", "moe_logits", "moe_y", "act_f32", "act_hi", "act_lo", "rows", "spans", "table", "logits", "workspace")] +
-                [("workspace_bytes", c_size_t)])
+                [("workspace_bytes", c_size_t), ("vfirst", c_void_p), ("ld_vfirst", c_int)])
 
 
 # name -> (restype, argtypes); this table IS the list of symbols include/chatts_amd.h declares
@@ -334,6 +345,7 @@ SIGNATURES = {
     "chatts_latent_attend": (c_int, [C.POINTER(LatentArgs), c_void_p]),
     "chatts_embed_pair": (c_int, [C.POINTER(EmbedPairArgs), c_void_p]),
     "chatts_pair_norm": (c_int, [C.POINTER(PairNormArgs), c_void_p]),
+    "chatts_post_norm": (c_int, [C.POINTER(PostNormArgs), c_void_p]),
     "chatts_token_shift": (c_int, [C.POINTER(TokenShiftArgs), c_void_p]),
     "chatts_recur_decode": (c_int, [C.POINTER(RecurArgs), c_void_p]),
     "chatts_recur_tanh": (c_int, [C.POINTER(RecurArgs), C.POINTER(Operand), c_void_p]),

@@ -193,14 +193,18 @@ __device__ __forceinline__ float softplus_f(float x) {      // (both forms are c
   const float r = e > 0.5f ? large : small;
   return x > 20.f ? x : r;
 }
-// the gated feed-forward of a (gate, up) pair: silu(g) * u (CHATTS_EPI_SWIGLU, silu passed in by the caller), or with both clamped
+// the gated feed-forward of a (gate, up) pair: silu(g) * u (CHATTS_EPI_SWIGLU, by the caller), with both clamped
 // (CHATTS_EPI_CLAMPGLU): g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1)
 __device__ __forceinline__ float clamp_glu(float g, float u, float limit, float alpha) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
   return g * sigmoid_f(alpha * g) * (u + 1.0f);
 }
-__host__ __device__ constexpr bool epi_is_glu(int epilogue) { return epilogue == CHATTS_EPI_SWIGLU || epilogue == CHATTS_EPI_CLAMPGLU; }
+// gelu(g) * u, gelu(g) = g (1 + tanh(t)) / 2 = g sigmoid(2 t) with t = sqrt(2 / pi) (g + 0.044715 g^3)  (CHATTS_EPI_GEGLU)
+__device__ __forceinline__ float gelu_tanh_glu(float g, float u) { return g * sigmoid_f(1.5957691216057308f * (g + 0.044715f * g * g * g)) * u; }
+__host__ __device__ constexpr bool epi_is_glu(int epilogue) {
+  return epilogue == CHATTS_EPI_SWIGLU || epilogue == CHATTS_EPI_CLAMPGLU || epilogue == CHATTS_EPI_GEGLU;
+}
 inline hipStream_t as_stream(chatts_stream_t s) { return reinterpret_cast<hipStream_t>(s); }
 
 // ---- stage ranges for traces (api.hip): roctx push / pop around the host-side enqueue of a stage, resolved with dlopen at first use

@@ -76,7 +76,7 @@ static int linear_impl(const ChattsLinearArgs* a, chatts_stream_t stream, const 
     CHATTS_REQUIRE(a->a_hi && a->a_lo && a->ld_planes >= a->k && a->ld_planes % 8 == 0 && ((uintptr_t)a->a_hi % 16) == 0 &&
                        ((uintptr_t)a->a_lo % 16) == 0 && a->m > 1 && !a->norm_w,
                    CHATTS_E_SHAPE, "linear: pre-split A needs both planes, ld_planes >= K and %% 8, 16-byte alignment, M > 1");
-  CHATTS_REQUIRE(a->epilogue >= CHATTS_EPI_NONE && a->epilogue <= CHATTS_EPI_CLAMPGLU, CHATTS_E_BADARG,
+  CHATTS_REQUIRE(a->epilogue >= CHATTS_EPI_NONE && a->epilogue <= CHATTS_EPI_GEGLU, CHATTS_E_BADARG,
                  "linear: epilogue %d", a->epilogue);
   CHATTS_REQUIRE(a->epilogue != CHATTS_EPI_RESID || a->resid, CHATTS_E_BADARG, "linear: EPI_RESID without resid");
   CHATTS_REQUIRE(a->k % 32 == 0, CHATTS_E_SHAPE, "linear: K=%d must be a multiple of 32 (pad the weight)", a->k);

@@ -43,7 +43,7 @@ __device__ __forceinline__ float relu2_f(float x) { const float r = fmaxf(x, 0.f
 __device__ __forceinline__ float silu_g(float x) { return x / (1.0f + expf(-x)); }
 
 __device__ __forceinline__ float glu_value(int epilogue, float g, float u, float limit, float alpha) {
-  return epilogue == CHATTS_EPI_SWIGLU ? silu_g(g) * u : clamp_glu(g, u, limit, alpha);
+  return epilogue == CHATTS_EPI_SWIGLU ? silu_g(g) * u : (epilogue == CHATTS_EPI_GEGLU ? gelu_tanh_glu(g, u) : clamp_glu(g, u, limit, alpha));
 }
 
 constexpr int kRingPanel = 256;      // W rows per panel of the prefill kernel

@@ -271,6 +271,9 @@ __global__ __launch_bounds__(kRingThreads) void gemm_ring_kernel(GemmParams p, c
     } else if (p.epilogue == CHATTS_EPI_CLAMPGLU) {
       if (planes) ring_store<kStClampGlu, true>(p, acc, fml, tok0, fb0, lane, 0);
       else ring_store<kStClampGlu, false>(p, acc, fml, tok0, fb0, lane, 0);
+    } else if (p.epilogue == CHATTS_EPI_GEGLU) {
+      if (planes) ring_store<kStGeglu, true>(p, acc, fml, tok0, fb0, lane, 0);
+      else ring_store<kStGeglu, false>(p, acc, fml, tok0, fb0, lane, 0);
     } else if (p.epilogue == CHATTS_EPI_RELU2) {
       if (planes) ring_store<kStRelu2, true>(p, acc, fml, tok0, fb0, lane, 0);
       else ring_store<kStRelu2, false>(p, acc, fml, tok0, fb0, lane, 0);

@@ -111,7 +111,8 @@ __device__ __forceinline__ void gemv_epilogue(const GemvParams& p, int task, int
       if (lane == u && rg + 16 < p.n) {
         float g = acc[2 * u], v = acc[2 * u + 1];
         if (p.bias) { g += p.bias[rg]; v += p.bias[rg + 16]; }
-        p.out[task * (ROWS / 2) + u] = EPI == CHATTS_EPI_CLAMPGLU ? clamp_glu(g, v, p.glu_limit, p.glu_alpha) : silu_f(g) * v;
+        p.out[task * (ROWS / 2) + u] = EPI == CHATTS_EPI_CLAMPGLU ? clamp_glu(g, v, p.glu_limit, p.glu_alpha)
+                                        : (EPI == CHATTS_EPI_GEGLU ? gelu_tanh_glu(g, v) : silu_f(g) * v);
       }
     }
   } else {
@@ -583,6 +584,7 @@ static void launch_ldsx(const GemvParams& p, int epi, bool norm, dim3 blocks, in
     case kEpiResidTp: hipLaunchKernelGGL((gemv_ldsx_kernel<ROWS, UNR, kEpiResidTp, false>), blocks, dim3(threads), lds, s, p); break;
     case CHATTS_EPI_SWIGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_SWIGLU>(p, norm, blocks, threads, lds, s); break;
     case CHATTS_EPI_RELU2: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_RELU2>(p, norm, blocks, threads, lds, s); break;
+    case CHATTS_EPI_GEGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_GEGLU>(p, norm, blocks, threads, lds, s); break;
     case CHATTS_EPI_CLAMPGLU: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_CLAMPGLU>(p, norm, blocks, threads, lds, s); break;
     default: launch_ldsx_norm<ROWS, UNR, CHATTS_EPI_NONE>(p, norm, blocks, threads, lds, s); break;
   }
@@ -680,7 +682,7 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
                    (long long)tp_capacity(a->tp_reduce));
     epilogue = kEpiResidTp;
   }
-  CHATTS_REQUIRE((a->epilogue != CHATTS_EPI_RELU2 && a->epilogue != CHATTS_EPI_CLAMPGLU) || (!a->w4 && !a->w8), CHATTS_E_BADARG, "gemv: EPI_RELU2 / CLAMPGLU take bf16 weights");
+  CHATTS_REQUIRE((a->epilogue != CHATTS_EPI_RELU2 && a->epilogue != CHATTS_EPI_CLAMPGLU && a->epilogue != CHATTS_EPI_GEGLU) || (!a->w4 && !a->w8), CHATTS_E_BADARG, "gemv: EPI_RELU2 / CLAMPGLU / GEGLU take bf16 weights");
   const int swiglu = epi_is_glu(a->epilogue);
   const int units = swiglu ? a->n / 2 : a->n;
   const int nchunks = (a->k + 511) / 512;
@@ -802,6 +804,10 @@ int launch_gemv(const ChattsLinearArgs* a, hipStream_t s) {
         case CHATTS_EPI_CLAMPGLU:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_CLAMPGLU, true>), g, b, lds, s, p);
           else hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_CLAMPGLU, false>), g, b, lds, s, p);
+          break;
+        case CHATTS_EPI_GEGLU:
+          if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_GEGLU, true>), g, b, lds, s, p);
+          else hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_GEGLU, false>), g, b, lds, s, p);
           break;
         case CHATTS_EPI_RELU2:
           if (norm) hipLaunchKernelGGL((gemv_ksplit_kernel<CHATTS_EPI_RELU2, true>), g, b, lds, s, p);

@@ -7,6 +7,9 @@
 // Parallel layer (two norms of the same x):
 //   pair_norm (norm1(x), norm2(x), with the experts' sum of the layer before, the token shift of a decoded token) -> input projections -> mixer kernels
 //   -> out projection, added to x -> gate_up (gated unit in the epilogue) -> down, added to x;  or router -> experts, added by the next pair_norm
+// Layer with its norms after the sums (sublayers read x itself):
+//   input projections -> mixer kernels -> out projection -> post_norm (x = norm1(alpha x + y), as the next operand too)
+//   -> gate_up (gated unit in the epilogue) -> down;  or router -> experts, beside a shared one: up -> down -> post_norm (x = norm2(alpha x + y + experts))
 // Operands between the launches travel in the format the next projection's kernel takes for this row count: bf16 hi / lo planes
 // (2 .. 16 rows: weight-streaming kernel; >= 96 rows: the prefill kernel) or float32.
 #include <new>
@@ -60,7 +63,7 @@ extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const Chatts
     if (!l.n_mix) add(l.in_n, c->width_p);
     add(c->width_p, l.out_k);
     if (l.w2) add(l.w2_n, l.recur.rank);
-    if (l.up) { add(l.ff_kind == CHATTS_FF_CLAMPGLU ? 2 * l.ff : l.ff, c->width_p); add(c->width_p, l.ff); }
+    if (l.up) { add(l.ff_kind == CHATTS_FF_CLAMPGLU || l.ff_kind == CHATTS_FF_GEGLU ? 2 * l.ff : l.ff, c->width_p); add(c->width_p, l.ff); }
     if (l.router) add(l.router_n, c->width_p);
   }
   add(c->width_p, 2 * c->width_p);
@@ -111,6 +114,14 @@ extern "C" ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, cons
       set_error("mixdec_create: layer %d is incomplete", i);
       return nullptr;
     }
+    if (l.post || layers[0].post) {
+      if (!l.post || !layers[0].post || l.parallel || l.kind != CHATTS_MIX_WINDOW || (l.ff_kind != CHATTS_FF_NONE && !l.norm2) ||
+          (l.ff_kind == CHATTS_FF_GEGLU ? !l.up : (l.ff_kind != CHATTS_FF_NONE && l.ff_kind != CHATTS_FF_MOE)) || (l.window.vfirst_write && !b->vfirst)) {
+        set_error("mixdec_create: layer %d: a layer with norms after the sums has windowed attention and a gated unit, experts or nothing", i);
+        return nullptr;
+      }
+      continue;
+    }
     if (l.parallel != layers[0].parallel || (pair && !l.parallel) || (l.ff_kind > CHATTS_FF_RELU2 && !l.parallel) || (l.ff_kind == CHATTS_FF_RELU2 && l.parallel)) {
       set_error("mixdec_create: layer %d: sequential and parallel layers do not mix", i);
       return nullptr;
@@ -141,8 +152,9 @@ static ChattsOperand operand(const ChattsMixDecoder* d, bool second, int m, int 
 }
 
 static int mix_linear(const ChattsMixDecoder* d, const ChattsOperand& in, const chatts_bf16* w, const chatts_bf16* w_t, int m, int n, int k, int epilogue,
-                      const ChattsOperand& out, chatts_stream_t s, float limit = 0.f, float alpha = 0.f) {
+                      const ChattsOperand& out, chatts_stream_t s, float limit = 0.f, float alpha = 0.f, const float* bias = nullptr) {
   ChattsLinearArgs a{};
+  a.bias = bias;
   a.glu_limit = limit; a.glu_alpha = alpha;
   a.resid = epilogue == CHATTS_EPI_RESID ? out.f32 : nullptr;
   a.a = in.f32;
@@ -327,6 +339,8 @@ static int mix_window(const ChattsMixDecoder* d, const ChattsMixLayer& l, const 
   ChattsWindowArgs a = l.window;
   a.proj = d->b.proj; a.ld_proj = l.in_n; a.eps = d->c.eps;
   a.kcache = run.cache; a.vcache = run.vcache; a.cache_f32 = d->c.exact;
+  a.ring = run.ring;
+  if (a.ld_vfirst) { a.vfirst = d->b.vfirst; a.ld_vfirst = d->b.ld_vfirst; }
   a.table = d->b.table; a.table_stride = d->c.table_stride; a.log_block = kv_log_block(d->c.block_size);
   a.rows = d->b.rows; a.n_rows = t; a.spans = d->b.spans; a.n_spans = single ? 0 : n_spans;
   a.q.ld = a.heads * a.dim_p;
@@ -339,7 +353,8 @@ static int mix_window(const ChattsMixDecoder* d, const ChattsMixLayer& l, const 
   if (a.longest >= 8 && !d->c.exact && chatts_window_can_prefill(a.dim_p, a.vdim_p)) return chatts_window_prefill(&a, s);
   if (!d->c.exact) {      // few rows: a row's tiles (32 keys a wave, 4 waves) are spread over workgroups, about three per CU, the same number to every wave
     const int group = a.heads / a.kv_heads, wgs = a.kv_heads * ((group + 15) / 16) * t;
-    const int tiles = (a.window > 0 && a.window + a.keep_first + 64 < d->c.max_ctx ? a.window + a.keep_first + 64 : d->c.max_ctx) / 32;
+    const int most = a.window > 0 ? a.window + a.keep_first + 64 : (a.chunk > 0 ? a.chunk + a.keep_first + 64 : d->c.max_ctx);
+    const int tiles = (most < d->c.max_ctx ? most : d->c.max_ctx) / 32;
     int splits = 3 * device_cus() / wgs;
     if (splits < 1) splits = 1;
     const int each = (tiles + 4 * splits - 1) / (4 * splits);
@@ -352,11 +367,11 @@ static int mix_window(const ChattsMixDecoder* d, const ChattsMixLayer& l, const 
   return chatts_window_attend(&a, s);
 }
 
-static ChattsMoeArgs mix_moe_args(const ChattsMixDecoder* d, const ChattsMixLayer& l, int t) {
+static ChattsMoeArgs mix_moe_args(const ChattsMixDecoder* d, const ChattsMixLayer& l, int t, const ChattsOperand& h) {
   const ChattsMixBuffers& b = d->b;
   ChattsMoeArgs a = l.moe;
   a.logits = b.moe_logits; a.ld_logits = l.router_n;
-  a.h = second_norm(d, l, t);
+  a.h = h;
   if (!d->c.exact) a.h.f32 = nullptr;
   a.rows = b.rows; a.n_rows = t; a.exact = d->c.exact;
   a.ids = b.moe_ids; a.place = b.moe_place; a.order = b.moe_order; a.offsets = b.moe_offsets; a.tiles = b.moe_tiles;
@@ -445,13 +460,69 @@ static int mix_parallel_forward(ChattsMixDecoder* d, const int64_t* tokens, int 
     } else if (l.ff_kind == CHATTS_FF_MOE) {
       StageRange stage("chatts.mix.experts");
       if ((rc = mix_linear(d, linear_form(N), l.router, l.router_t, t, l.router_n, wp, CHATTS_EPI_NONE, f32_out(d->b.moe_logits, l.router_n), s)) != 0) return rc;
-      const ChattsMoeArgs m = mix_moe_args(d, l, t);
+      const ChattsMoeArgs m = mix_moe_args(d, l, t, N);
       if ((rc = chatts_moe_route(&m, s)) != 0) return rc;
       if ((rc = chatts_moe_experts(&m, s)) != 0) return rc;
       owed = &l;
     }
   }
   if (owed) return mix_pair_norm(d, t, owed, nullptr, nullptr, none, none, false, nullptr, nullptr, s);
+  return CHATTS_OK;
+}
+
+// ---- norms after the sums ----
+// x as the operand of what reads it next: x itself where float32 is taken, planes beside it for wide steps and for experts
+static ChattsOperand stream_operand(const ChattsMixDecoder* d, int m, bool experts) {
+  ChattsOperand o{};
+  o.ld = d->c.width_p;
+  const bool planes = mix_planes(d->c, m, o.ld);
+  if (planes || (experts && !d->c.exact)) { o.hi = d->b.a_hi; o.lo = d->b.a_lo; }
+  if (!planes) o.f32 = d->b.x;
+  return o;
+}
+static int mix_post_norm(const ChattsMixDecoder* d, int t, const float* y, const ChattsMixLayer* moe, const float* w, ChattsOperand out, chatts_stream_t s) {
+  ChattsPostNormArgs a{};
+  a.x = d->b.x; a.t = t; a.width = d->c.width; a.ldx = d->c.width_p; a.alpha = d->c.alpha; a.eps = d->c.eps; a.y = y; a.w = w;
+  if (moe) { a.ey = d->b.moe_y; a.place = d->b.moe_place; a.weight = d->b.moe_weight; a.top = moe->moe.top; }
+  out.f32 = nullptr;      // (x itself)
+  a.out = out;
+  return chatts_post_norm(&a, s);
+}
+
+static int mix_post_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, const ChattsSpan* spans, int n_spans, bool single, chatts_stream_t s) {
+  const ChattsMixConfig& c = d->c;
+  const int wp = c.width_p;
+  const ChattsOperand Y = f32_out(d->b.y, wp);
+  int rc;
+  if ((rc = chatts_embed_token_batched(tokens, t, d->b.embed, 0, c.vocab, wp, d->b.x, s)) != 0) return rc;
+  ChattsOperand X = stream_operand(d, t, false);
+  if (X.hi && (rc = chatts_split_bf16x2(d->b.x, t, wp, wp, X.hi, X.lo, wp, s)) != 0) return rc;
+  for (int r = 0; r < c.n_runs; ++r) {
+    const ChattsMixRun& run = d->runs[r];
+    const ChattsMixLayer& l = d->layers[run.layer];
+    if ((rc = mix_linear(d, linear_form(X), l.in, l.in_t, t, l.in_n, wp, CHATTS_EPI_NONE, f32_out(d->b.proj, l.in_n), s, 0.f, 0.f, l.in_bias)) != 0) return rc;
+    const ChattsOperand B = operand(d, true, t, l.out_k);
+    if ((rc = mix_window(d, l, run, t, spans, n_spans, single, B, s)) != 0) return rc;
+    if ((rc = mix_linear(d, B, l.out, l.out_t, t, wp, l.out_k, CHATTS_EPI_NONE, Y, s)) != 0) return rc;
+    const bool moe = l.ff_kind == CHATTS_FF_MOE;
+    X = stream_operand(d, t, moe);
+    if ((rc = mix_post_norm(d, t, d->b.y, nullptr, l.norm1, X, s)) != 0) return rc;
+    if (l.ff_kind == CHATTS_FF_NONE) continue;
+    if (l.up) {
+      const ChattsOperand F = operand(d, true, t, l.ff);
+      if ((rc = mix_linear(d, linear_form(X), l.up, l.up_t, t, moe ? l.ff : 2 * l.ff, wp, moe ? CHATTS_EPI_RELU2 : CHATTS_EPI_GEGLU, F, s)) != 0) return rc;
+      if ((rc = mix_linear(d, F, l.down, l.down_t, t, wp, l.ff, CHATTS_EPI_NONE, Y, s)) != 0) return rc;
+    }
+    if (moe) {
+      StageRange stage("chatts.mix.experts");
+      if ((rc = mix_linear(d, linear_form(X), l.router, l.router_t, t, l.router_n, wp, CHATTS_EPI_NONE, f32_out(d->b.moe_logits, l.router_n), s)) != 0) return rc;
+      const ChattsMoeArgs m = mix_moe_args(d, l, t, X);
+      if ((rc = chatts_moe_route(&m, s)) != 0) return rc;
+      if ((rc = chatts_moe_experts(&m, s)) != 0) return rc;
+    }
+    X = stream_operand(d, t, false);
+    if ((rc = mix_post_norm(d, t, l.up ? d->b.y : nullptr, moe ? &l : nullptr, l.norm2, X, s)) != 0) return rc;
+  }
   return CHATTS_OK;
 }
 
@@ -476,6 +547,7 @@ extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens,
     CHATTS_REQUIRE(rows == t, CHATTS_E_SHAPE, "mixdec_forward: segments hold %d of %d rows", rows, t);
   }
   StageRange stage(single ? "chatts.mix.decode" : "chatts.mix.prefill");
+  if (d->layers[0].post) return mix_post_forward(d, tokens, t, spans, n_spans, single != 0, s);
   if (d->layers[0].parallel) return mix_parallel_forward(d, tokens, t, spans, n_spans, single != 0, s);
   int rc;
   if ((rc = chatts_embed_token_batched(tokens, t, d->b.embed, 0, c.vocab, c.width_p, d->b.x, s)) != 0) return rc;

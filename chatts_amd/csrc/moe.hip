@@ -1,5 +1,5 @@
-// moe.hip - mixture of experts: a softmax router with a correction of the choice and choice groups, experts W_down (silu(W_gate h) * W_up h), identity
-// outputs.
+// moe.hip - mixture of experts: choice by softmax values or logits, with a correction of the choice and choice groups; experts
+// W_down (silu(W_gate h) * W_up h) or W_down max(W_up h, 0)^2, identity outputs.
 //   moe_route_kernel      a wave per token: scores, the best groups, the best `top` outputs, their weights
 //   moe_list_kernel       a workgroup per expert: its (token, choice) pairs as a list, in order; tiles of the lists for the tiled products
 //   moe_route_small_kernel  both in one workgroup, for up to 16 rows; the tiles are then the experts in use
@@ -33,21 +33,29 @@ __device__ __forceinline__ void moe_route_row(const ChattsMoeArgs& p, int row, i
   float* ch = sc + N;
   float* gr = ch + N;
   const bool parked = p.rows[row].pos < 0;
+  const bool logits = p.choose == CHATTS_CHOOSE_LOGITS;
   const float* z = p.logits + (size_t)row * p.ld_logits;
-  float mx = -INFINITY;
-  for (int i = lane; i < N; i += 64) mx = fmaxf(mx, z[i]);
-  mx = wave_max(mx);
-  float sum = 0.f;
-  for (int i = lane; i < N; i += 64) {
-    const float e = expf(z[i] - mx);
-    sc[i] = e;
-    sum += e;
-  }
-  sum = wave_sum(sum);
-  for (int i = lane; i < N; i += 64) {
-    const float s = sc[i] / sum;
-    sc[i] = s;
-    ch[i] = s + p.correction[i];
+  if (logits) {
+    for (int i = lane; i < N; i += 64) {
+      sc[i] = z[i];
+      ch[i] = z[i] + (p.correction ? p.correction[i] : 0.f);
+    }
+  } else {
+    float mx = -INFINITY;
+    for (int i = lane; i < N; i += 64) mx = fmaxf(mx, z[i]);
+    mx = wave_max(mx);
+    float sum = 0.f;
+    for (int i = lane; i < N; i += 64) {
+      const float e = expf(z[i] - mx);
+      sc[i] = e;
+      sum += e;
+    }
+    sum = wave_sum(sum);
+    for (int i = lane; i < N; i += 64) {
+      const float s = sc[i] / sum;
+      sc[i] = s;
+      ch[i] = s + (p.correction ? p.correction[i] : 0.f);
+    }
   }
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");      // (the wave's own LDS: no barrier)
   if (p.keep < p.groups) {
@@ -66,8 +74,8 @@ __device__ __forceinline__ void moe_route_row(const ChattsMoeArgs& p, int row, i
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
   }
-  float total = 0.f, kept = 0.f, mine = 0.f;
-  int id = -1;      // lane j: choice j
+  float total = 0.f, kept = 0.f, mine = logits ? -INFINITY : 0.f;
+  int id = -1, own = -1;      // lane j: choice j
   for (int j = 0; j < p.top; ++j) {
     float v = -INFINITY;
     int b = 1 << 30;
@@ -79,7 +87,13 @@ __device__ __forceinline__ void moe_route_row(const ChattsMoeArgs& p, int row, i
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     total += s;
     if (b < N && b >= p.experts) kept += s;
-    if (lane == j) { id = b < p.experts ? b : -1; mine = s; }
+    if (lane == j && b < N) { own = b; id = b < p.experts ? b : -1; mine = s; }
+  }
+  if (logits) {      // softmax over the chosen logits
+    const float mx = wave_max(mine);
+    mine = lane < p.top ? expf(mine - mx) : 0.f;
+    total = wave_sum(mine);
+    kept = wave_sum(own >= p.experts ? mine : 0.f);
   }
   const float inv = 1.0f / (total + 1e-20f);
   if (lane < p.top) {
@@ -212,24 +226,35 @@ __global__ __launch_bounds__(1024) void moe_route_small_kernel(ChattsMoeArgs p, 
 
 __device__ __forceinline__ float moe_glu(float g, float u) { return g * sigmoid_f(g) * u; }
 
+// the products of an expert: its input projection (kGated: gate and up rows interleaved in blocks of 16, kRelu2: up rows alone), the output projection
+enum { kDown = 0, kGated, kRelu2 };
+__device__ __host__ __forceinline__ int moe_in_rows(const ChattsMoeArgs& p) { return p.act_kind == CHATTS_EXPERT_RELU2 ? p.ff_p : 2 * p.ff_p; }
+__device__ __forceinline__ void moe_relu2_4(const ChattsOperand& o, size_t row, int col, const f32x4& s) {
+  float v[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) v[r] = relu2_f(s[r]);
+  store_operand4(o, row, col, v);
+}
+
 // ---- up to 16 rows: grid (blocks of 32 weight rows, tiles), 4 waves split K; D = W . A^T: a lane holds 4 consecutive outputs of one token.
-// GLU: the two 16-row halves of a block are gate and up rows of the same outputs ----
+// kGated: the two 16-row halves of a block are gate and up rows of the same outputs ----
 // TILED: weights from the chatts_tile_bf16 copy: a fragment's 64 pieces are 1 KB of consecutive memory
-template <bool GLU, bool TILED>
+template <int STEP, bool TILED>
 __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
   __shared__ f32x4 red[4][2][64];
+  constexpr bool IN = STEP != kDown;
   const int32_t* tile = p.tiles + (size_t)blockIdx.y * 4;
   const int e = tile[0];
   if (e < 0) return;
   const int place0 = tile[1], count = tile[2], lane = threadIdx.x & 63, wave = threadIdx.x >> 6, fr = lane & 15, fg = lane >> 4;
-  const int K = GLU ? p.width_p : p.ff_p, N = GLU ? 2 * p.ff_p : p.width_p, n0 = blockIdx.x * 32;
-  const uint16_t* w = TILED ? (GLU ? p.gate_up_t : p.down_t) + ((size_t)e * N + n0) * K + (fr * 4 + (fg ^ ((fr >> 3) << 1))) * 8
-                            : (GLU ? p.gate_up : p.down) + ((size_t)e * N + n0 + fr) * K + fg * 8;
+  const int K = IN ? p.width_p : p.ff_p, N = IN ? moe_in_rows(p) : p.width_p, n0 = blockIdx.x * 32;
+  const uint16_t* w = TILED ? (IN ? p.gate_up_t : p.down_t) + ((size_t)e * N + n0) * K + (fr * 4 + (fg ^ ((fr >> 3) << 1))) * 8
+                            : (IN ? p.gate_up : p.down) + ((size_t)e * N + n0 + fr) * K + fg * 8;
   constexpr int kStep = TILED ? 16 : 1;      // elements of w per K-value
   const int pl = place0 + (fr < count ? fr : 0);
-  const size_t arow = GLU ? (size_t)(p.order[pl] / p.top) * p.h.ld : (size_t)pl * p.act.ld;
-  const uint16_t* ah = (GLU ? p.h.hi : p.act.hi) + arow + fg * 8;
-  const uint16_t* al = (GLU ? p.h.lo : p.act.lo) + arow + fg * 8;
+  const size_t arow = IN ? (size_t)(p.order[pl] / p.top) * p.h.ld : (size_t)pl * p.act.ld;
+  const uint16_t* ah = (IN ? p.h.hi : p.act.hi) + arow + fg * 8;
+  const uint16_t* al = (IN ? p.h.lo : p.act.lo) + arow + fg * 8;
   f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
   constexpr int U = 4;
   const int steps = K >> 5;      // K-steps of 32: wave, wave + 4, ...
@@ -261,14 +286,16 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
   red[wave][0][lane] = acc[0];
   red[wave][1][lane] = acc[1];
   __syncthreads();
-  if (wave >= (GLU ? 1 : 2)) return;
+  if (wave >= (STEP == kGated ? 1 : 2)) return;
   f32x4 s[2];
 #pragma unroll
   for (int f = 0; f < 2; ++f)
 #pragma unroll
     for (int r = 0; r < 4; ++r) s[f][r] = (red[0][f][lane][r] + red[1][f][lane][r]) + (red[2][f][lane][r] + red[3][f][lane][r]);
   if (fr >= count) return;
-  if (GLU) {
+  if (STEP == kRelu2) {
+    moe_relu2_4(p.act, place0 + fr, n0 + wave * 16 + fg * 4, wave ? s[1] : s[0]);
+  } else if (STEP == kGated) {
     float v[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = moe_glu(s[0][r], s[1][r]);
@@ -281,15 +308,16 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
 // ---- more rows: grid (tiles, blocks of 128 weight rows), 4 waves; K in steps of 64 through LDS, the next step requested while this one is multiplied.
 // D = W . A^T, wave = 128 / WN weight rows x BM / WM tokens ----
 constexpr int kMoeLd = 72;      // LDS row of 64 K-values: 144 bytes, sixteen rows meet sixteen different groups of banks
-template <bool GLU, int BM, int WM, int WN>
+template <int STEP, int BM, int WM, int WN>
 __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(ChattsMoeArgs p) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
+  constexpr bool IN = STEP != kDown;
   constexpr int FN = 8 / WN, FM = BM / 16 / WM;      // fragments of a wave: weight rows, tokens
   const int32_t* tile = p.tiles + (size_t)blockIdx.x * 4;
   const int e = tile[0];
   if (e < 0) return;
   const int place0 = tile[1], count = tile[2], tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, fr = lane & 15, fg = lane >> 4;
-  const int wm = wave / WN, wn = wave % WN, K = GLU ? p.width_p : p.ff_p, N = GLU ? 2 * p.ff_p : p.width_p, n0 = blockIdx.y * 128;
+  const int wm = wave / WN, wn = wave % WN, K = IN ? p.width_p : p.ff_p, N = IN ? moe_in_rows(p) : p.width_p, n0 = blockIdx.y * 128;
   uint16_t* sw = reinterpret_cast<uint16_t*>(smem);      // [128][kMoeLd]
   uint16_t* sh = sw + 128 * kMoeLd;                      // [BM][kMoeLd]
   uint16_t* sl = sh + BM * kMoeLd;
@@ -301,14 +329,14 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(ChattsMoeArgs p) {
 #pragma unroll
   for (int i = 0; i < PW; ++i) {
     const int r = n0 + r0 + i * 32;
-    wsrc[i] = (GLU ? p.gate_up : p.down) + ((size_t)e * N + (r < N ? r : N - 1)) * K + c;
+    wsrc[i] = (IN ? p.gate_up : p.down) + ((size_t)e * N + (r < N ? r : N - 1)) * K + c;
   }
 #pragma unroll
   for (int i = 0; i < PA; ++i) {
     const int r = r0 + i * 32, pl = place0 + (r < count ? r : count - 1);
-    const size_t at = (GLU ? (size_t)(p.order[pl] / p.top) * p.h.ld : (size_t)pl * p.act.ld) + c;
-    hsrc[i] = (GLU ? p.h.hi : p.act.hi) + at;
-    lsrc[i] = (GLU ? p.h.lo : p.act.lo) + at;
+    const size_t at = (IN ? (size_t)(p.order[pl] / p.top) * p.h.ld : (size_t)pl * p.act.ld) + c;
+    hsrc[i] = (IN ? p.h.hi : p.act.hi) + at;
+    lsrc[i] = (IN ? p.h.lo : p.act.lo) + at;
   }
   u32x4 rw[PW], rh[PA], rl[PA];
   auto fetch = [&](int k) __attribute__((always_inline)) {
@@ -357,7 +385,13 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(ChattsMoeArgs p) {
   for (int i = 0; i < FM; ++i) {
     const int m = (wm * FM + i) * 16 + fr;
     if (m >= count) continue;
-    if constexpr (GLU) {
+    if constexpr (STEP == kRelu2) {
+#pragma unroll
+      for (int j = 0; j < FN; ++j) {
+        const int n = n0 + (wn * FN + j) * 16;
+        if (n < N) moe_relu2_4(p.act, place0 + m, n + fg * 4, acc[i][j]);
+      }
+    } else if constexpr (STEP == kGated) {
 #pragma unroll
       for (int j = 0; j < FN; j += 2) {
         const int n = n0 + (wn * FN + j) * 16;
@@ -379,17 +413,18 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(ChattsMoeArgs p) {
 
 // ---- 32-bit runs: grid (tiles of 64, N / 64), float32 products and sums; wave = 32 tokens x 32 weight rows ----
 constexpr int kMoeF32Ld = 36;
-template <bool GLU>
+template <int STEP>
 __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(ChattsMoeArgs p) {
   __shared__ __attribute__((aligned(16))) float sa[64 * kMoeF32Ld], sw[64 * kMoeF32Ld];
+  constexpr bool IN = STEP != kDown;
   const int32_t* tile = p.tiles + (size_t)blockIdx.x * 4;
   const int e = tile[0];
   if (e < 0) return;
   const int place0 = tile[1], count = tile[2], tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int K = GLU ? p.width_p : p.ff_p, N = GLU ? 2 * p.ff_p : p.width_p, n0 = blockIdx.y * 64, wm = (wave >> 1) * 32, wn = (wave & 1) * 32;
+  const int K = IN ? p.width_p : p.ff_p, N = IN ? moe_in_rows(p) : p.width_p, n0 = blockIdx.y * 64, wm = (wave >> 1) * 32, wn = (wave & 1) * 32;
   const int r = tid >> 2, kc = (tid & 3) * 8, pl = place0 + (r < count ? r : count - 1);
-  const float* a = GLU ? p.h.f32 + (size_t)(p.order[pl] / p.top) * p.h.ld : p.act.f32 + (size_t)pl * p.act.ld;
-  const uint16_t* w = (GLU ? p.gate_up : p.down) + ((size_t)e * N + n0 + r) * K;
+  const float* a = IN ? p.h.f32 + (size_t)(p.order[pl] / p.top) * p.h.ld : p.act.f32 + (size_t)pl * p.act.ld;
+  const uint16_t* w = (IN ? p.gate_up : p.down) + ((size_t)e * N + n0 + r) * K;
   f32x4 acc[2][2] = {};
   for (int k0 = 0; k0 < K; k0 += 32) {
     const f32x4 a0 = *reinterpret_cast<const f32x4*>(a + k0 + kc), a1 = *reinterpret_cast<const f32x4*>(a + k0 + kc + 4);
@@ -424,7 +459,10 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(ChattsMoeArgs p) {
     for (int q = 0; q < 4; ++q) {
       const int m = wm + i * 16 + (lane >> 4) * 4 + q;
       if (m >= count) continue;
-      if (GLU) {
+      if (STEP == kRelu2) {
+#pragma unroll
+        for (int j = 0; j < 2; ++j) p.act.f32[(size_t)(place0 + m) * p.act.ld + n0 + wn + j * 16 + (lane & 15)] = relu2_f(acc[i][j][q]);
+      } else if (STEP == kGated) {
         p.act.f32[(size_t)(place0 + m) * p.act.ld + ((n0 + wn) >> 1) + (lane & 15)] = moe_glu(acc[i][0][q], acc[i][1][q]);
       } else {
 #pragma unroll
@@ -439,6 +477,8 @@ static int check_moe(const ChattsMoeArgs* a, const char* who) {
   CHATTS_REQUIRE(a->experts >= 1 && a->identity >= 0 && n <= kMoeMaxOut && a->top >= 1 && a->top <= 64 && a->groups >= 1 && n % a->groups == 0 && a->keep >= 1 &&
                      a->keep <= a->groups && a->top <= n / a->groups * a->keep, CHATTS_E_SHAPE, "%s: %d experts + %d, top %d, %d of %d groups", who, a->experts,
                  a->identity, a->top, a->keep, a->groups);
+  CHATTS_REQUIRE((a->choose == CHATTS_CHOOSE_SOFTMAX || a->choose == CHATTS_CHOOSE_LOGITS) && (a->act_kind == CHATTS_EXPERT_SWIGLU || a->act_kind == CHATTS_EXPERT_RELU2),
+                 CHATTS_E_BADARG, "%s: choice %d, experts of kind %d", who, a->choose, a->act_kind);
   CHATTS_REQUIRE(a->width_p > 0 && a->width_p % 64 == 0 && a->ff_p > 0 && a->ff_p % 64 == 0, CHATTS_E_SHAPE, "%s: widths %d, %d", who, a->width_p, a->ff_p);
   return CHATTS_OK;
 }
@@ -453,17 +493,17 @@ static int moe_tile_bound(int rows, int top, int experts, int bm) {      // sum 
   return (int)(pairs / bm + lists);
 }
 
-template <bool GLU, int BM, int WM, int WN>
+template <int STEP, int BM, int WM, int WN>
 static int launch_moe_gemm(const ChattsMoeArgs* a, int tiles, hipStream_t s) {
   constexpr int LDS = (128 + 2 * BM) * kMoeLd * 2;
   static bool done = false;
   if (!done) {
-    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_gemm_kernel<GLU, BM, WM, WN>), hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_gemm_kernel<STEP, BM, WM, WN>), hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
     CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "moe_gemm: cannot reserve LDS: %s", hipGetErrorString(e));
     done = true;
   }
-  const int N = GLU ? 2 * a->ff_p : a->width_p;
-  hipLaunchKernelGGL((moe_gemm_kernel<GLU, BM, WM, WN>), dim3(tiles, (N + 127) / 128), dim3(256), LDS, s, *a);
+  const int N = STEP ? moe_in_rows(*a) : a->width_p;
+  hipLaunchKernelGGL((moe_gemm_kernel<STEP, BM, WM, WN>), dim3(tiles, (N + 127) / 128), dim3(256), LDS, s, *a);
   CHATTS_CHECK_LAUNCH("moe_gemm");
   return CHATTS_OK;
 }
@@ -476,7 +516,7 @@ extern "C" int chatts_moe_tiles(int rows, int top, int experts) { return moe_til
 
 extern "C" int chatts_moe_route(const ChattsMoeArgs* a, chatts_stream_t stream) {
   if (const int rc = check_moe(a, "moe_route")) return rc;
-  CHATTS_REQUIRE(a->logits && a->correction && a->ld_logits >= a->experts + a->identity, CHATTS_E_BADARG, "moe_route: null pointer");
+  CHATTS_REQUIRE(a->logits && a->ld_logits >= a->experts + a->identity, CHATTS_E_BADARG, "moe_route: null pointer");
   if (a->n_rows == 0) return CHATTS_OK;
   hipStream_t s = as_stream(stream);
   const int bm = moe_bm(a), tiles = moe_tile_bound(a->n_rows, a->top, a->experts, bm);
@@ -498,27 +538,32 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
                      a->act.ld >= a->ff_p && a->h.ld % 8 == 0 && a->act.ld % 8 == 0, CHATTS_E_BADARG, "moe_experts: operands");
   if (a->n_rows == 0) return CHATTS_OK;
   hipStream_t s = as_stream(stream);
-  const int bm = moe_bm(a), tiles = moe_tile_bound(a->n_rows, a->top, a->experts, bm);
+  const int bm = moe_bm(a), tiles = moe_tile_bound(a->n_rows, a->top, a->experts, bm), in_rows = moe_in_rows(*a);
+  const bool relu2 = a->act_kind == CHATTS_EXPERT_RELU2;
   if (a->exact) {
-    hipLaunchKernelGGL(moe_gemm_f32_kernel<true>, dim3(tiles, 2 * a->ff_p / 64), dim3(256), 0, s, *a);
-    hipLaunchKernelGGL(moe_gemm_f32_kernel<false>, dim3(tiles, a->width_p / 64), dim3(256), 0, s, *a);
+    if (relu2) hipLaunchKernelGGL(moe_gemm_f32_kernel<kRelu2>, dim3(tiles, in_rows / 64), dim3(256), 0, s, *a);
+    else hipLaunchKernelGGL(moe_gemm_f32_kernel<kGated>, dim3(tiles, in_rows / 64), dim3(256), 0, s, *a);
+    hipLaunchKernelGGL(moe_gemm_f32_kernel<kDown>, dim3(tiles, a->width_p / 64), dim3(256), 0, s, *a);
     CHATTS_CHECK_LAUNCH("moe_gemm_f32");
     return CHATTS_OK;
   }
   if (moe_small(a)) {
-    const dim3 g1(2 * a->ff_p / 32, tiles), g2(a->width_p / 32, tiles), b(256);
-    if (a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<true, true>), g1, b, 0, s, *a);
-    else hipLaunchKernelGGL((moe_stream_kernel<true, false>), g1, b, 0, s, *a);
-    if (a->down_t) hipLaunchKernelGGL((moe_stream_kernel<false, true>), g2, b, 0, s, *a);
-    else hipLaunchKernelGGL((moe_stream_kernel<false, false>), g2, b, 0, s, *a);
+    const dim3 g1(in_rows / 32, tiles), g2(a->width_p / 32, tiles), b(256);
+    if (relu2 && a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<kRelu2, true>), g1, b, 0, s, *a);
+    else if (relu2) hipLaunchKernelGGL((moe_stream_kernel<kRelu2, false>), g1, b, 0, s, *a);
+    else if (a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<kGated, true>), g1, b, 0, s, *a);
+    else hipLaunchKernelGGL((moe_stream_kernel<kGated, false>), g1, b, 0, s, *a);
+    if (a->down_t) hipLaunchKernelGGL((moe_stream_kernel<kDown, true>), g2, b, 0, s, *a);
+    else hipLaunchKernelGGL((moe_stream_kernel<kDown, false>), g2, b, 0, s, *a);
     CHATTS_CHECK_LAUNCH("moe_stream");
     return CHATTS_OK;
   }
   int rc;
   if (bm == kRingTile) {
-    RingGroup g{a->tiles, a->offsets + a->experts + 1, a->order, a->top, (int64_t)2 * a->ff_p * a->width_p};
+    RingGroup g{a->tiles, a->offsets + a->experts + 1, a->order, a->top, (int64_t)in_rows * a->width_p};
     GemmParams p{};
-    p.w = a->gate_up; p.wt = a->gate_up_t; p.m = a->n_rows; p.n = 2 * a->ff_p; p.k = p.ldw = a->width_p; p.epilogue = CHATTS_EPI_SWIGLU;
+    p.w = a->gate_up; p.wt = a->gate_up_t; p.m = a->n_rows; p.n = in_rows; p.k = p.ldw = a->width_p;
+    p.epilogue = relu2 ? CHATTS_EPI_RELU2 : CHATTS_EPI_SWIGLU;
     p.k_per_split = p.k; p.direct = 1; p.c_hi = a->act.hi; p.c_lo = a->act.lo; p.ldcp = a->act.ld; p.ldc = a->act.ld;
     if ((rc = launch_ring_group(p, a->h.hi, a->h.lo, a->h.ld, g, tiles, s)) != 0) return rc;
     g.order = nullptr;
@@ -527,6 +572,6 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
     p.c_hi = p.c_lo = nullptr; p.c = a->y; p.ldc = a->width_p;
     return launch_ring_group(p, a->act.hi, a->act.lo, a->act.ld, g, tiles, s);
   }
-  if ((rc = launch_moe_gemm<true, 32, 1, 4>(a, tiles, s)) != 0) return rc;
-  return launch_moe_gemm<false, 32, 1, 4>(a, tiles, s);
+  if ((rc = relu2 ? launch_moe_gemm<kRelu2, 32, 1, 4>(a, tiles, s) : launch_moe_gemm<kGated, 32, 1, 4>(a, tiles, s)) != 0) return rc;
+  return launch_moe_gemm<kDown, 32, 1, 4>(a, tiles, s);
 }

@@ -6,7 +6,7 @@
 namespace chatts {
 
 // modes of the branch-free epilogue (selected once per unit)
-enum { kStRaw = 0, kStNone, kStGelu, kStResid, kStSwiglu, kStRelu2, kStClampGlu };
+enum { kStRaw = 0, kStNone, kStGelu, kStResid, kStSwiglu, kStRelu2, kStClampGlu, kStGeglu };
 
 __device__ __forceinline__ void ring_wait_vmcnt(int n) {      // wave-uniform n: at most n of this wave's loads outstanding
 #define CHATTS_VM(N) case N: asm volatile("s_waitcnt vmcnt(" #N ")" ::: "memory"); break;
@@ -72,7 +72,8 @@ __device__ __forceinline__ void ring_store(const GemmParams& p, const f32x4 (&ac
         }
       }
     }
-  } else if constexpr (MODE == kStSwiglu || MODE == kStClampGlu) {
+  } else if constexpr (MODE == kStSwiglu || MODE == kStClampGlu || MODE == kStGeglu) {
+    constexpr int kEpi = MODE == kStSwiglu ? CHATTS_EPI_SWIGLU : (MODE == kStGeglu ? CHATTS_EPI_GEGLU : CHATTS_EPI_CLAMPGLU);
     f32x4 bg[2], bu[2];
 #pragma unroll
     for (int q = 0; q < 2; ++q) {
@@ -92,8 +93,7 @@ __device__ __forceinline__ void ring_store(const GemmParams& p, const f32x4 (&ac
           float v[4];
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            v[r] = glu_value(MODE == kStSwiglu ? CHATTS_EPI_SWIGLU : CHATTS_EPI_CLAMPGLU, acc[i][2 * q][r] + bg[q][r], acc[i][2 * q + 1][r] + bu[q][r],
-                             p.glu_limit, p.glu_alpha);
+            v[r] = glu_value(kEpi, acc[i][2 * q][r] + bg[q][r], acc[i][2 * q + 1][r] + bu[q][r], p.glu_limit, p.glu_alpha);
           if (tok < p.m && fb + 19 < p.n) put((size_t)tok * p.ldc, (size_t)tok * p.ldcp, ocol, v);
         }
       }

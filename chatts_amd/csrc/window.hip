@@ -1,6 +1,9 @@
-// window.hip - attention over paged keys and values with grouped heads: per-head RMS norms of queries and keys, an optional sliding window that keeps
-// a sequence's first tokens, an optional sink (one more term exp(0) in the denominator), an optional output gate.
-//   window_prep_kernel      norms; queries as an operand, keys and values into their pages
+// window.hip - attention over paged keys and values with grouped heads.  Optional, each by its own parameter: short convolutions, norms of queries and
+// keys (per head, over all heads, unit after a rotation of pairs), mixed values; capped scores, a distance bias per head, a sliding window that keeps
+// a sequence's first tokens, chunks, a sink (one more term exp(0) in the denominator); an output gate per value or per head.
+//   window_prep_kernel      per-head work: norms, rotation, values; queries as an operand, keys and values into their pages
+//   window_prep_rows_kernel the same for layers with convolutions or norms over all heads: a workgroup owns whole rows
+//   window_ring_kernel      the last convolution inputs of every segment
 //   window_attend_kernel    one row and query head per workgroup, vector units: 32-bit runs, head sizes beyond the matrix kernels
 //   window_decode_kernel    one row: the query heads of a key head share its tiles on the matrix pipe; tiles spread over waves and workgroups
 //   window_prefill_kernel   flash attention for segments of many rows
@@ -17,13 +20,18 @@ __device__ __forceinline__ size_t window_tile(const ChattsWindowArgs& p, int slo
   const int blk = p.table[(size_t)slot * p.table_stride + (key >> p.log_block)];
   return (((size_t)blk * p.kv_heads + hk) << p.log_block) + (key & ((1 << p.log_block) - 1));
 }
+__device__ __forceinline__ bool window_masked(const ChattsWindowArgs& p) { return p.window > 0 || p.chunk > 0; }
+__device__ __forceinline__ int window_low(const ChattsWindowArgs& p, int pos) {      // first position that `pos` sees beside the kept ones
+  if (p.window > 0) return pos - p.window + 1;
+  return p.chunk > 0 ? pos - pos % p.chunk : 0;
+}
 // tiles of K keys that a row at `pos` (or rows pos_lo .. pos) sees: the first `kept`, then from `from` to the tile of pos
 struct WindowTiles {
   int kept, from, last;
   __device__ __forceinline__ WindowTiles(const ChattsWindowArgs& p, int pos_lo, int pos, int log_tile) {
     last = pos >> log_tile;
-    if (p.window <= 0) { kept = 0; from = 0; return; }
-    const int w = pos_lo - p.window + 1;
+    if (!window_masked(p)) { kept = 0; from = 0; return; }
+    const int w = window_low(p, pos_lo);
     from = (w > 0 ? w : 0) >> log_tile;
     kept = (p.keep_first + (1 << log_tile) - 1) >> log_tile;
     if (kept > last + 1) kept = last + 1;
@@ -32,12 +40,24 @@ struct WindowTiles {
   __device__ __forceinline__ int count() const { return kept + last + 1 - from; }
   __device__ __forceinline__ int tile(int i) const { return i < kept ? i : from + i - kept; }
 };
-__device__ __forceinline__ bool window_sees(const ChattsWindowArgs& p, int pos, int key) {
-  return key <= pos && (p.window <= 0 || pos - key < p.window || key < p.keep_first);
+__device__ __forceinline__ bool window_sees(const ChattsWindowArgs& p, int pos, int low, int key) { return key <= pos && (key >= low || key < p.keep_first); }
+__device__ __forceinline__ float window_gate(const ChattsWindowArgs& p, size_t row, int h, int c) {
+  return p.off_gate < 0 ? 1.f : sigmoid_f(p.proj[row * p.ld_proj + p.off_gate + (p.gate_heads ? h : h * p.vdim + c)]);
 }
-__device__ __forceinline__ float window_gate(const ChattsWindowArgs& p, size_t row, int at) {
-  return p.off_gate < 0 ? 1.f : sigmoid_f(p.proj[row * p.ld_proj + p.off_gate + at]);
+constexpr float kLog2e = 1.44269504088896341f;
+// what the matrix kernels are compiled for (registers are scarce there): plain scores, a distance bias, capped scores (with chunks), or whatever is set
+enum { kPlain = 0, kSlope, kCap, kAny };
+template <int SCORE>
+__device__ __forceinline__ bool window_capped(const ChattsWindowArgs& p) { return SCORE == kCap || (SCORE == kAny && p.softcap > 0.f); }
+template <int SCORE>
+__device__ __forceinline__ bool window_sloped(const ChattsWindowArgs& p) { return SCORE == kSlope || (SCORE == kAny && p.slopes != nullptr); }
+template <int SCORE>
+__device__ __forceinline__ int window_low_of(const ChattsWindowArgs& p, int pos) {
+  if (SCORE == kPlain || SCORE == kSlope) return p.window > 0 ? pos - p.window + 1 : 0;      // (no chunks there)
+  return window_low(p, pos);
 }
+// cap tanh(x / cap), in units of cap: tanh(y) = 1 - 2 / (1 + exp(2 y));  k = 2 log2(e) / cap
+__device__ __forceinline__ float window_cap(float x, float k, float cap) { return cap - 2.f * cap * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * k)); }
 
 template <typename CT>
 __device__ __forceinline__ CT to_page(float v) {
@@ -61,18 +81,218 @@ __global__ __launch_bounds__(256) void window_prep_kernel(ChattsWindowArgs p) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) v[j] = j * 64 + lane < n ? x[j * 64 + lane] : 0.f;
     const float* w = value ? nullptr : (e < H ? p.q_norm : p.k_norm);
-    if (w) f = 1.0f / sqrtf(wave_sum((v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3])) / (float)n + p.eps);
+    auto inv_rms = [&]() { return 1.0f / sqrtf(wave_sum((v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3])) / (float)n + p.eps); };
+    if (w) f = inv_rms();
+    if (!value && (p.rot || p.unit)) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int c = j * 64 + lane;
+        if (w) v[j] = c < n ? v[j] * f * w[c] : 0.f;
+        if (j * 64 < p.rot) {      // (uniform; the other dimension of a pair is in the neighbouring lane)
+          const float other = lane_xor1(v[j]);
+          if (c < p.rot) {
+            const size_t at = (size_t)R.pos * (p.rot >> 1) + (c >> 1);
+            const float s = p.sin_tab[at];
+            v[j] = v[j] * p.cos_tab[at] + (c & 1 ? other * s : -other * s);
+          }
+        }
+      }
+      f = p.unit ? inv_rms() : 1.f;
+      w = nullptr;
+    }
+    if (value && p.vfirst) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int c = j * 64 + lane;
+        if (c >= n) break;
+        float* first = p.vfirst + (size_t)row * p.ld_vfirst + hk * n + c;
+        if (p.vfirst_write) *first = v[j];
+        else v[j] = (1.f - p.vmix) * v[j] + p.vmix * *first;
+      }
+    }
     CT* dst = nullptr;
     if (e >= H) dst = reinterpret_cast<CT*>(value ? p.vcache : p.kcache) + window_tile(p, R.slot, hk, R.pos) * np;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int c = j * 64 + lane;
       if (c >= np) break;
-      const float y = w && c < n ? v[j] * f * w[c] : v[j];
+      const float y = v[j] * f * (w && c < n ? w[c] : 1.f);
       if (dst) dst[c] = to_page<CT>(y);
       else store_operand(p.q, row, e * p.dim_p + c, y);
     }
   }
+}
+
+// A workgroup owns ROWS rows, a thread quads of channels of [q | k | v]: convolutions over a window of rows in registers (inputs before a segment come from
+// the ring), norms over all heads, mixed values.
+constexpr int kConvRegs = 4;      // taps whose weights stay in registers
+template <typename CT, int NT, int NV, int ROWS>
+__global__ __launch_bounds__(NT) void window_prep_rows_kernel(ChattsWindowArgs p) {
+  __shared__ float red[NT / 64][2 * ROWS];
+  const int row0 = blockIdx.x * ROWS, tid = threadIdx.x, H = p.heads, G = p.kv_heads;
+  const int n[3] = {H * p.dim, G * p.dim, G * p.vdim}, quads[3] = {(n[0] + 3) >> 2, (n[1] + 3) >> 2, (n[2] + 3) >> 2}, total = quads[0] + quads[1] + quads[2];
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  ChattsRow R[ROWS];
+  bool one = true;      // the rows are consecutive rows of one segment
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    R[r] = row0 + r < p.n_rows ? p.rows[row0 + r] : ChattsRow{0, -1, 0, 0};
+    if (row0 + r < p.n_rows) one = one && R[r].pos >= 0 && R[r].first == R[0].first;
+  }
+  if (ROWS == 1 && R[0].pos < 0) return;
+  auto place = [&](int u, int& block, int& c) __attribute__((always_inline)) {      // quad -> its block and first channel there
+    block = u < quads[0] ? 0 : (u < quads[0] + quads[1] ? 1 : 2);
+    c = 4 * (u - (block > 0 ? quads[0] : 0) - (block > 1 ? quads[1] : 0));
+    return (block == 0 ? p.off_q : (block == 1 ? p.off_k : p.off_v)) + c;
+  };
+  auto input = [&](int r, int row, int back, int col) __attribute__((always_inline)) {      // the projected value `back` tokens before row r's
+    if (row - back >= R[r].first) return *reinterpret_cast<const f32x4*>(p.proj + (size_t)(row - back) * p.ld_proj + col);
+    const int q = R[r].pos - back;
+    return q >= 0 ? *reinterpret_cast<const f32x4*>(p.ring + ((size_t)R[r].slot * p.taps + q % p.taps) * p.conv_ch + col) : zero;
+  };
+  f32x4 y[NV][ROWS];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int u = i * NT + tid;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) y[i][r] = zero;
+    if (u >= total) continue;
+    int block, c;
+    const int col = place(u, block, c);
+    if (!p.taps) {
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r)
+        if (R[r].pos >= 0) y[i][r] = *reinterpret_cast<const f32x4*>(p.proj + (size_t)(row0 + r) * p.ld_proj + col);
+      continue;
+    }
+    const float* cw = p.conv_w + col;
+    if (one && p.taps <= kConvRegs) {
+      f32x4 w[kConvRegs];      // [tokens back]
+#pragma unroll
+      for (int g = 0; g < kConvRegs; ++g) w[g] = g < p.taps ? *reinterpret_cast<const f32x4*>(cw + (size_t)(p.taps - 1 - g) * p.conv_ch) : zero;
+#pragma unroll
+      for (int j = 1 - kConvRegs; j < ROWS; ++j) {      // input j: row row0 + j
+        if (j <= -p.taps || row0 + j >= p.n_rows) continue;
+        const f32x4 v = input(0, row0, -j, col);
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+          if (r - j >= 0 && r - j < kConvRegs) y[i][r] += w[r - j] * v;
+      }
+    } else {
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r)
+        if (R[r].pos >= 0)
+          for (int g = p.taps - 1; g >= 0; --g) y[i][r] += *reinterpret_cast<const f32x4*>(cw + (size_t)(p.taps - 1 - g) * p.conv_ch) * input(r, row0 + r, g, col);
+    }
+    if (p.n_spans == 0) {      // segments of one token: nobody else reads this entry of the ring
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r)
+        if (R[r].pos >= 0) *reinterpret_cast<f32x4*>(p.ring + ((size_t)R[r].slot * p.taps + R[r].pos % p.taps) * p.conv_ch + col) = input(r, row0 + r, 0, col);
+    }
+  }
+  float inv[2][ROWS];
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) inv[0][r] = inv[1][r] = 1.f;
+  if (p.norm_whole) {
+    const int wave = tid >> 6, lane = tid & 63;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) {
+      float ss[2] = {0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int u = i * NT + tid;
+        const float s = (y[i][r][0] * y[i][r][0] + y[i][r][1] * y[i][r][1]) + (y[i][r][2] * y[i][r][2] + y[i][r][3] * y[i][r][3]);
+        if (u < quads[0]) ss[0] += s;
+        else if (u < quads[0] + quads[1]) ss[1] += s;
+      }
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        const float s = wave_sum(ss[b]);
+        if (lane == 0) red[wave][2 * r + b] = s;
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        float s = 0.f;
+#pragma unroll
+        for (int w = 0; w < NT / 64; ++w) s += red[w][2 * r + b];
+        inv[b][r] = 1.0f / sqrtf(s / (float)n[b] + p.eps);
+      }
+  }
+  const bool whole = p.dim % 4 == 0 && p.vdim % 4 == 0;      // a quad stays in one head
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int u = i * NT + tid;
+    if (u >= total) continue;
+    int block, c;
+    place(u, block, c);
+    const float* nw = block == 0 ? p.q_norm : (block == 1 ? p.k_norm : nullptr);
+    f32x4 w = {1.f, 1.f, 1.f, 1.f};
+    if (nw) w = *reinterpret_cast<const f32x4*>(nw + c);
+    const int d = block == 2 ? p.vdim : p.dim, dp = block == 2 ? p.vdim_p : p.dim_p, e0 = c / d, c0 = c - e0 * d;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) {
+      if (R[r].pos < 0) continue;
+      const int row = row0 + r;
+      f32x4 v;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) v[k] = block == 2 ? y[i][r][k] : y[i][r][k] * inv[block & 1][r] * w[k];
+      if (block == 2 && p.vfirst) {
+        float* first = p.vfirst + (size_t)row * p.ld_vfirst + c;
+        if (p.vfirst_write) *reinterpret_cast<f32x4*>(first) = v;
+        else v = (1.f - p.vmix) * v + p.vmix * *reinterpret_cast<const f32x4*>(first);
+      }
+      const float out[4] = {v[0], v[1], v[2], v[3]};
+      CT* pages = reinterpret_cast<CT*>(block == 2 ? p.vcache : p.kcache);
+      if (whole) {
+        if (block == 0) {
+          store_operand4(p.q, row, e0 * p.dim_p + c0, out);
+        } else {
+          CT* dst = pages + window_tile(p, R[r].slot, e0, R[r].pos) * dp + c0;
+          if constexpr (sizeof(CT) == 4) *reinterpret_cast<f32x4*>(dst) = v;
+          else *reinterpret_cast<w16x4*>(dst) = (w16x4){(short)to_page<CT>(v[0]), (short)to_page<CT>(v[1]), (short)to_page<CT>(v[2]), (short)to_page<CT>(v[3])};
+        }
+      } else {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+          if (c + k >= n[block]) break;
+          const int e = (c + k) / d, cc = c + k - e * d;
+          if (block == 0) store_operand(p.q, row, e * p.dim_p + cc, out[k]);
+          else pages[window_tile(p, R[r].slot, e, R[r].pos) * dp + cc] = to_page<CT>(out[k]);
+        }
+      }
+    }
+  }
+  // padding between heads: queries multiply it, so it must not hold another layer's numbers
+  const int pad = p.dim_p - p.dim;
+  for (int x = tid; x < ROWS * (H + G) * pad; x += NT) {
+    const int r = x / ((H + G) * pad), z = x - r * (H + G) * pad, e = z / pad, c = p.dim + z - e * pad;
+    if (row0 + r >= p.n_rows) break;
+    const ChattsRow Z = p.rows[row0 + r];
+    if (Z.pos < 0) continue;
+    if (e < H) store_operand(p.q, row0 + r, e * p.dim_p + c, 0.f);
+    else reinterpret_cast<CT*>(p.kcache)[window_tile(p, Z.slot, e - H, Z.pos) * p.dim_p + c] = 0;
+  }
+  const int vpad = p.vdim_p - p.vdim;
+  for (int x = tid; x < ROWS * G * vpad; x += NT) {
+    const int r = x / (G * vpad), z = x - r * G * vpad, e = z / vpad;
+    if (row0 + r >= p.n_rows) break;
+    const ChattsRow Z = p.rows[row0 + r];
+    if (Z.pos >= 0) reinterpret_cast<CT*>(p.vcache)[window_tile(p, Z.slot, e, Z.pos) * p.vdim_p + p.vdim + z - e * vpad] = 0;
+  }
+}
+
+// grid (taps - 1, spans, columns / 1024): the inputs that the next step's convolutions read
+__global__ __launch_bounds__(256) void window_ring_kernel(ChattsWindowArgs p) {
+  const ChattsSpan sp = p.spans[blockIdx.y];
+  const int i = blockIdx.x, c = (blockIdx.z * 256 + threadIdx.x) * 4;
+  if (i >= sp.t || c >= p.conv_ch) return;
+  const int last = sp.t - 1 - i;
+  *reinterpret_cast<f32x4*>(p.ring + ((size_t)sp.slot * p.taps + (sp.pos0 + last) % p.taps) * p.conv_ch + c) =
+      *reinterpret_cast<const f32x4*>(p.proj + (size_t)(sp.row0 + last) * p.ld_proj + c);
 }
 
 // ---- vector units: grid (heads, rows) ----
@@ -90,7 +310,8 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
   }
   float m = p.sink ? 0.f : -INFINITY, l = p.sink ? 1.f : 0.f, o = 0.f;      // column tid
   const WindowTiles T(p, R.pos, R.pos, 6);
-  const int n = T.count();
+  const int n = T.count(), low = window_low(p, R.pos);
+  const float slope = p.slopes ? p.slopes[h] : 0.f;
   for (int i = 0; i < n; ++i) {
     __syncthreads();
     const int k0 = T.tile(i) * 64;
@@ -98,7 +319,7 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
     const CT* kt = reinterpret_cast<const CT*>(p.kcache) + at * p.dim_p;
     const CT* vt = reinterpret_cast<const CT*>(p.vcache) + at * p.vdim_p;
     const int key = tid >> 2, part = tid & 3;
-    const bool sees = window_sees(p, R.pos, k0 + key);
+    const bool sees = window_sees(p, R.pos, low, k0 + key);
     float d = 0.f;
     if (sees)
       for (int c = part; c < p.dim_p; c += 4) {
@@ -109,7 +330,9 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
       }
     d += lane_xor1(d);
     d += lane_xor2(d);
-    if (part == 0) sc[key] = sees ? d * p.scale : -INFINITY;
+    d *= p.scale;
+    if (p.softcap > 0.f) d = p.softcap * tanhf(d / p.softcap);
+    if (part == 0) sc[key] = sees ? d - slope * (float)(R.pos - k0 - key) : -INFINITY;
     __syncthreads();
     const float s = sc[tid & 63];
     const float mn = fmaxf(m, wave_max(s)), safe = mn == -INFINITY ? 0.f : mn;
@@ -130,14 +353,14 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
       }
     }
   }
-  if (tid < p.vdim) store_operand(p.out, row, h * p.vdim + tid, o / l * window_gate(p, row, h * p.vdim + tid));
+  if (tid < p.vdim) store_operand(p.out, row, h * p.vdim + tid, o / l * window_gate(p, row, h, tid));
 }
 
 // ---- one row on the matrix pipe: grid (splits, kv heads * head tiles, rows), 4 waves ----
 // A wave walks tiles of 32 keys on its own (tiles 4 split + wave, ...): S^T = K Q^T with the key rows straight from memory as A fragments, so that a
 // lane ends up with 8 scores of one head (column = lane & 15); O^T = V^T P^T with V through a private piece of LDS (LDS-DMA) and transposing reads - its B
 // fragment IS the 8 probabilities of the lane (K slot 8 g + j = key 4 g + j, j < 4, or 16 + 4 g + j - 4, on both sides).  The waves' softmaxes meet once.
-template <int NK, int NV>      // dim_p <= 32 NK, vdim_p <= 16 NV
+template <int NK, int NV, int SCORE>      // dim_p <= 32 NK, vdim_p <= 16 NV
 __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_decode_kernel(ChattsWindowArgs p) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int split = blockIdx.x, row = blockIdx.z, tid = threadIdx.x, lane = tid & 63, fr = lane & 15, fg = lane >> 4;
@@ -153,12 +376,13 @@ __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_d
   for (int k = 0; k < NK; ++k)
     if (k < nk) q[k] = *reinterpret_cast<const bf16x8_t*>(p.q.hi + (size_t)row * p.q.ld + head * p.dim_p + k * 32 + fg * 8);
   const WindowTiles T(p, R.pos, R.pos, 5);
-  const int n = T.count(), stride = 4 * p.n_splits;
+  const int n = T.count(), stride = 4 * p.n_splits, low = window_low_of<SCORE>(p, R.pos);
+  const float slope2 = window_sloped<SCORE>(p) ? p.slopes[head] * kLog2e : 0.f;
   float m = -INFINITY, l = 0.f;
   f32x4 o[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) o[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  const float scale2 = p.scale * 1.44269504088896341f;
+  const float scale2 = p.scale * kLog2e, cap2 = p.softcap * kLog2e, capk = window_capped<SCORE>(p) ? 2.f * kLog2e * p.scale / p.softcap : 0.f;
   constexpr int VP = NV;      // LDS-DMA requests of a value tile: 64 pieces of 16 bytes each
   // 16-byte piece c of row r lies at position c ^ (r & sw): the transposing reads of neighbouring rows meet different banks
   const int vc = p.vdim_p >> 3, sw = (vc & 7) == 0 ? 7 : ((vc & 3) == 0 ? 3 : 1);
@@ -191,10 +415,19 @@ __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_d
         s[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(t.k[1][k], q[k], s[1], 0, 0, 0);
       }
     float v[8], mx = -INFINITY;
+    if (window_capped<SCORE>(p)) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = window_cap(s[j >> 2][j & 3], capk, cap2);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = s[j >> 2][j & 3] * scale2;
+    }
+    const float d0 = (float)(k0 + fg * 4 - R.pos);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int key = k0 + (j >> 2) * 16 + fg * 4 + (j & 3);
-      v[j] = window_sees(p, R.pos, key) ? s[j >> 2][j & 3] * scale2 : -INFINITY;
+      if (SCORE == kSlope || SCORE == kAny) v[j] += slope2 * (d0 + (float)((j >> 2) * 16 + (j & 3)));
+      if (!window_sees(p, R.pos, low, key)) v[j] = -INFINITY;
       mx = fmaxf(mx, v[j]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -266,7 +499,7 @@ __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_d
       acc += f * part[(w * 16 + hh) * ldp + c];
     }
     if (whole) {
-      if (c < p.vdim) store_operand(p.out, row, hd * p.vdim + c, acc / L * window_gate(p, row, hd * p.vdim + c));
+      if (c < p.vdim) store_operand(p.out, row, hd * p.vdim + c, acc / L * window_gate(p, row, hd, c));
     } else {
       float* dst = p.partial + (((size_t)row * p.heads + hd) * p.n_splits + split) * ldp;
       dst[c] = acc;
@@ -294,13 +527,13 @@ __global__ __launch_bounds__(128) void window_merge_kernel(ChattsWindowArgs p) {
     float o = 0.f;
 #pragma unroll 4
     for (int s = 0; s < p.n_splits; ++s) o += w[s] * part[(size_t)s * ld + c];
-    store_operand(p.out, row, h * p.vdim + c, o * window_gate(p, row, h * p.vdim + c));
+    store_operand(p.out, row, h * p.vdim + c, o * window_gate(p, row, h, c));
   }
 }
 
 // ---- many rows: grid (heads, query tiles of 128, spans); a wave owns 32 queries of one head, 64 keys per step ----
 // S^T = K Q^T, O^T = V^T P^T as above; keys and values of a tile are staged by all waves, the next tile's requested while this one is multiplied.
-template <int NK, int NV, int OCC>      // dim_p <= 32 NK, vdim_p <= 16 NV
+template <int NK, int NV, int OCC, int SCORE>      // dim_p <= 32 NK, vdim_p <= 16 NV
 __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowArgs p) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const ChattsSpan sp = p.spans[blockIdx.z];
@@ -329,7 +562,13 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
   for (int i = 0; i < NV; ++i) o[i][0] = o[i][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
   const float m0 = p.sink ? 0.f : -INFINITY, l0 = p.sink && fg == 0 ? 1.f : 0.f;
   float m[2] = {m0, m0}, l[2] = {l0, l0};
-  const float scale2 = p.scale * 1.44269504088896341f;      // scores in base 2
+  const float scale2 = p.scale * kLog2e;      // scores in base 2
+  const float cap2 = p.softcap * kLog2e, capk = window_capped<SCORE>(p) ? 2.f * kLog2e * p.scale / p.softcap : 0.f;
+  const float slope2 = window_sloped<SCORE>(p) ? p.slopes[h] * kLog2e : 0.f;
+  const int low_first = window_low_of<SCORE>(p, w0), low_last = window_low_of<SCORE>(p, w1);
+  int lows[2] = {0, 0};
+  if (SCORE == kCap || SCORE == kAny) { lows[0] = window_low(p, w0 + fr); lows[1] = window_low(p, w0 + 16 + fr); }
+  const bool masked = window_masked(p);
   constexpr int KP = NK, VP = (NV + 1) / 2;
   u32x4 rk[KP], rv[VP];
   const int kc = dq >> 3, vc = p.vdim_p >> 3;
@@ -367,8 +606,8 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
     if (i + 1 < n) fetch(i + 1);
     const int k0 = T.tile(i) * 64;
     // (uniform per wave) nothing of the tile is visible to this wave's queries
-    if (k0 > w1 || w0 > w1 || (p.window > 0 && w0 - (k0 + 63) >= p.window && k0 >= p.keep_first)) continue;
-    const bool edge = k0 + 63 > w0 || (p.window > 0 && w1 - k0 >= p.window && k0 + 63 >= p.keep_first);      // some key is hidden from some query
+    if (k0 > w1 || w0 > w1 || (masked && k0 + 63 < low_first && k0 >= p.keep_first)) continue;
+    const bool edge = k0 + 63 > w0 || (masked && k0 < low_last && k0 + 63 >= p.keep_first);      // some key is hidden from some query
     f32x4 s[4][2];      // [16-key block][query block]
 #pragma unroll
     for (int a = 0; a < 4; ++a) s[a][0] = s[a][1] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -396,14 +635,32 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
     bf16x8_t pf[2][2];      // [32-key group][query block]
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      const int qpos = w0 + u * 16 + fr;
+      const int qpos = w0 + u * 16 + fr, low = SCORE == kCap || SCORE == kAny ? lows[u] : window_low_of<SCORE>(p, qpos);
+      if (window_capped<SCORE>(p)) {
+#pragma unroll
+        for (int a = 0; a < 4; ++a)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[a][u][r] = window_cap(s[a][u][r], capk, cap2);
+      } else {
+#pragma unroll
+        for (int a = 0; a < 4; ++a)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[a][u][r] *= scale2;
+      }
+      if (window_sloped<SCORE>(p)) {
+        const float d0 = (float)(k0 + fg * 4 - qpos);
+#pragma unroll
+        for (int a = 0; a < 4; ++a)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[a][u][r] += slope2 * (d0 + (float)(a * 16 + r));
+      }
       float mx = -INFINITY;
 #pragma unroll
       for (int a = 0; a < 4; ++a)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          float v = s[a][u][r] * scale2;
-          if (edge && !window_sees(p, qpos, k0 + a * 16 + fg * 4 + r)) v = -INFINITY;
+          float v = s[a][u][r];
+          if (edge && !window_sees(p, qpos, low, k0 + a * 16 + fg * 4 + r)) v = -INFINITY;
           s[a][u][r] = v;
           mx = fmaxf(mx, v);
         }
@@ -455,7 +712,7 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
         }
     }
   }
-  const bool quads = p.vdim % 4 == 0 && (p.off_gate < 0 || p.off_gate % 4 == 0) && p.out.ld % 4 == 0;
+  const bool quads = p.vdim % 4 == 0 && (p.off_gate < 0 || p.gate_heads || p.off_gate % 4 == 0) && p.out.ld % 4 == 0;
 #pragma unroll
   for (int u = 0; u < 2; ++u) {
     const int r = q0 + u * 16 + fr;
@@ -463,15 +720,15 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
     L += __shfl_xor(L, 16, 64);
     L += __shfl_xor(L, 32, 64);
     if (r >= sp.t) continue;
-    const float inv = 1.0f / L;
     const size_t row = sp.row0 + r;
+    const float inv = 1.0f / L * (p.gate_heads ? window_gate(p, row, h, 0) : 1.f);
 #pragma unroll
     for (int f = 0; f < NV; ++f) {
       const int c = f * 16 + fg * 4, at = h * p.vdim + c;
       if (f >= nv || c >= p.vdim) continue;
       if (quads) {
         f32x4 g = {1.f, 1.f, 1.f, 1.f};
-        if (p.off_gate >= 0) {
+        if (p.off_gate >= 0 && !p.gate_heads) {
           g = *reinterpret_cast<const f32x4*>(p.proj + row * p.ld_proj + p.off_gate + at);
 #pragma unroll
           for (int k = 0; k < 4; ++k) g[k] = sigmoid_f(g[k]);
@@ -481,28 +738,56 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
       } else {
 #pragma unroll
         for (int k = 0; k < 4; ++k)
-          if (c + k < p.vdim) store_operand(p.out, row, at + k, o[f][u][k] * inv * window_gate(p, row, at + k));
+          if (c + k < p.vdim) store_operand(p.out, row, at + k, o[f][u][k] * inv * (p.gate_heads ? 1.f : window_gate(p, row, h, c + k)));
       }
     }
   }
 }
 
 static int check_window(const ChattsWindowArgs* a, const char* who) {
-  CHATTS_REQUIRE(a && a->proj && a->kcache && a->vcache && a->table && a->rows && a->q_norm && a->k_norm && (a->q.f32 || a->q.hi), CHATTS_E_BADARG, "%s: null pointer", who);
+  CHATTS_REQUIRE(a && a->proj && a->kcache && a->vcache && a->table && a->rows && (a->q_norm != nullptr) == (a->k_norm != nullptr) && (a->q.f32 || a->q.hi), CHATTS_E_BADARG, "%s: null pointer", who);
   CHATTS_REQUIRE(a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim >= 1 && a->dim <= a->dim_p && a->dim_p <= 256 && a->dim_p % 32 == 0 &&
                      a->vdim >= 1 && a->vdim <= a->vdim_p && a->vdim_p <= 256 && a->vdim_p % 16 == 0, CHATTS_E_SHAPE, "%s: heads %d / %d of %d, %d (at most 256)", who,
                  a->heads, a->kv_heads, a->dim, a->vdim);
   CHATTS_REQUIRE(a->off_q >= 0 && a->off_k >= 0 && a->off_v >= 0 && a->off_q + a->heads * a->dim <= a->ld_proj && a->off_k + a->kv_heads * a->dim <= a->ld_proj &&
-                     a->off_v + a->kv_heads * a->vdim <= a->ld_proj && a->off_gate + a->heads * a->vdim <= a->ld_proj && a->ld_proj % 4 == 0, CHATTS_E_SHAPE,
-                 "%s: column blocks", who);
+                     a->off_v + a->kv_heads * a->vdim <= a->ld_proj && a->off_gate + (a->gate_heads ? a->heads : a->heads * a->vdim) <= a->ld_proj &&
+                     a->ld_proj % 4 == 0, CHATTS_E_SHAPE, "%s: column blocks", who);
   CHATTS_REQUIRE(a->n_rows >= 0 && a->n_rows <= 65535, CHATTS_E_SHAPE, "%s: %d rows", who, a->n_rows);
   CHATTS_REQUIRE(a->log_block >= 6 && a->log_block <= 15 && a->window >= 0 && a->keep_first >= 0, CHATTS_E_SHAPE, "%s: pages of 2^%d tokens, window %d, kept %d", who,
                  a->log_block, a->window, a->keep_first);
+  CHATTS_REQUIRE(a->chunk >= 0 && (a->chunk == 0 || a->window == 0) && a->softcap >= 0.f && (!a->gate_heads || a->off_gate >= 0), CHATTS_E_SHAPE,
+                 "%s: window %d and chunks of %d, scores capped at %g", who, a->window, a->chunk, (double)a->softcap);
+  CHATTS_REQUIRE(a->rot >= 0 && a->rot % 2 == 0 && a->rot <= a->dim && (a->rot == 0 || (a->cos_tab && a->sin_tab)), CHATTS_E_SHAPE, "%s: %d of %d dimensions rotated", who,
+                 a->rot, a->dim);
+  CHATTS_REQUIRE(a->taps >= 0 && (a->taps == 0 || (a->conv_w && a->ring && a->conv_ch % 4 == 0 && a->conv_ch <= a->ld_proj && a->off_q + a->heads * a->dim <= a->conv_ch &&
+                                                   a->off_k + a->kv_heads * a->dim <= a->conv_ch && a->off_v + a->kv_heads * a->vdim <= a->conv_ch)),
+                 CHATTS_E_SHAPE, "%s: convolutions over %d tokens of %d columns", who, a->taps, a->conv_ch);
+  CHATTS_REQUIRE(!a->vfirst || (a->ld_vfirst >= a->kv_heads * a->vdim && a->ld_vfirst % 4 == 0 && ((uintptr_t)a->vfirst % 16) == 0), CHATTS_E_SHAPE,
+                 "%s: rows of %d first values", who, a->ld_vfirst);
+  const bool rows = a->taps > 0 || a->norm_whole;
+  CHATTS_REQUIRE(!rows || (!a->rot && !a->unit && (!a->q_norm || a->norm_whole)), CHATTS_E_SHAPE, "%s: convolutions and norms over all heads do not combine with per-head steps", who);
+  CHATTS_REQUIRE(!rows || (a->off_q % 4 == 0 && a->off_k % 4 == 0 && a->off_v % 4 == 0 && (!a->norm_whole || (a->q_norm && ((uintptr_t)a->q_norm % 16) == 0 &&
+                           ((uintptr_t)a->k_norm % 16) == 0)) && (((uintptr_t)a->conv_w | (uintptr_t)a->ring) % 16) == 0 &&
+                           a->heads * a->dim + a->kv_heads * (a->dim + a->vdim) + 12 <= 32768 && a->off_q + (a->heads * a->dim + 3) / 4 * 4 <= a->ld_proj &&
+                           a->off_k + (a->kv_heads * a->dim + 3) / 4 * 4 <= a->ld_proj && a->off_v + (a->kv_heads * a->vdim + 3) / 4 * 4 <= a->ld_proj), CHATTS_E_SHAPE,
+                 "%s: %d + %d heads by whole rows", who, a->heads, a->kv_heads);
   CHATTS_REQUIRE((((uintptr_t)a->kcache | (uintptr_t)a->vcache | (uintptr_t)a->proj) % 16) == 0 && a->q.ld >= a->heads * a->dim_p && a->q.ld % 8 == 0 &&
                      (a->cache_f32 ? a->q.f32 != nullptr : a->q.hi != nullptr), CHATTS_E_SHAPE, "%s: alignment / queries", who);
   return CHATTS_OK;
 }
 static bool window_out_ok(const ChattsWindowArgs* a) { return (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim; }
+
+template <typename CT>
+static int launch_window_rows(const ChattsWindowArgs* a, hipStream_t s) {
+  const int quads = (a->heads * a->dim + 3) / 4 + (a->kv_heads * a->dim + 3) / 4 + (a->kv_heads * a->vdim + 3) / 4;
+  if (a->n_rows > 64 && quads <= 8 * 256) hipLaunchKernelGGL((window_prep_rows_kernel<CT, 256, 8, 4>), dim3((a->n_rows + 3) / 4), dim3(256), 0, s, *a);
+  else if (quads <= 2 * 1024) hipLaunchKernelGGL((window_prep_rows_kernel<CT, 1024, 2, 1>), dim3(a->n_rows), dim3(1024), 0, s, *a);
+  else hipLaunchKernelGGL((window_prep_rows_kernel<CT, 1024, 8, 1>), dim3(a->n_rows), dim3(1024), 0, s, *a);
+  if (a->n_spans > 0 && a->taps > 1)
+    hipLaunchKernelGGL(window_ring_kernel, dim3(a->taps - 1, a->n_spans, (a->conv_ch + 1023) / 1024), dim3(256), 0, s, *a);
+  CHATTS_CHECK_LAUNCH("window_prep_rows");
+  return CHATTS_OK;
+}
 
 template <typename K>
 static int window_lds(K kernel, size_t bytes, bool& done) {
@@ -514,25 +799,49 @@ static int window_lds(K kernel, size_t bytes, bool& done) {
   return CHATTS_OK;
 }
 
-template <int NK, int NV>
-static int launch_window_decode(const ChattsWindowArgs* a, hipStream_t s) {
+static int window_score(const ChattsWindowArgs* a) {
+  if (a->softcap > 0.f && !a->slopes) return kCap;
+  if (a->softcap > 0.f || a->chunk > 0) return kAny;
+  return a->slopes ? kSlope : kPlain;
+}
+
+template <int NK, int NV, int SCORE>
+static int launch_window_decode_as(const ChattsWindowArgs* a, hipStream_t s) {
   static bool done = false;
   const size_t most = (size_t)4 * 16 * (NV * 16 + 4) * 4;      // the waves' meeting; their value tiles (4 x 32 x vdim_p bf16) are smaller
-  if (const int rc = window_lds(&window_decode_kernel<NK, NV>, most, done)) return rc;
+  if (const int rc = window_lds(&window_decode_kernel<NK, NV, SCORE>, most, done)) return rc;
   const int group = a->heads / a->kv_heads;
-  hipLaunchKernelGGL((window_decode_kernel<NK, NV>), dim3(a->n_splits, a->kv_heads * ((group + 15) / 16), a->n_rows), dim3(256),
+  hipLaunchKernelGGL((window_decode_kernel<NK, NV, SCORE>), dim3(a->n_splits, a->kv_heads * ((group + 15) / 16), a->n_rows), dim3(256),
                      (size_t)4 * 16 * (a->vdim_p + 4) * 4, s, *a);
   CHATTS_CHECK_LAUNCH("window_decode");
   return CHATTS_OK;
 }
-template <int NK, int NV, int OCC>
-static int launch_window_prefill(const ChattsWindowArgs* a, hipStream_t s) {
+template <int NK, int NV>
+static int launch_window_decode(const ChattsWindowArgs* a, hipStream_t s) {
+  switch (window_score(a)) {
+    case kPlain: return launch_window_decode_as<NK, NV, kPlain>(a, s);
+    case kSlope: return launch_window_decode_as<NK, NV, kSlope>(a, s);
+    case kCap: return launch_window_decode_as<NK, NV, kCap>(a, s);
+    default: return launch_window_decode_as<NK, NV, kAny>(a, s);
+  }
+}
+template <int NK, int NV, int OCC, int SCORE>
+static int launch_window_prefill_as(const ChattsWindowArgs* a, hipStream_t s) {
   static bool done = false;
-  if (const int rc = window_lds(&window_prefill_kernel<NK, NV, OCC>, (size_t)64 * (NK * 32 + 8 + NV * 16 + 16) * 2, done)) return rc;
-  hipLaunchKernelGGL((window_prefill_kernel<NK, NV, OCC>), dim3(a->heads, (a->longest + 127) / 128, a->n_spans), dim3(256),
+  if (const int rc = window_lds(&window_prefill_kernel<NK, NV, OCC, SCORE>, (size_t)64 * (NK * 32 + 8 + NV * 16 + 16) * 2, done)) return rc;
+  hipLaunchKernelGGL((window_prefill_kernel<NK, NV, OCC, SCORE>), dim3(a->heads, (a->longest + 127) / 128, a->n_spans), dim3(256),
                      (size_t)64 * (a->dim_p + 8 + a->vdim_p + 16) * 2, s, *a);
   CHATTS_CHECK_LAUNCH("window_prefill");
   return CHATTS_OK;
+}
+template <int NK, int NV, int OCC>
+static int launch_window_prefill(const ChattsWindowArgs* a, hipStream_t s) {
+  switch (window_score(a)) {
+    case kPlain: return launch_window_prefill_as<NK, NV, OCC, kPlain>(a, s);
+    case kSlope: return launch_window_prefill_as<NK, NV, OCC, kSlope>(a, s);
+    case kCap: return launch_window_prefill_as<NK, NV, OCC, kCap>(a, s);
+    default: return launch_window_prefill_as<NK, NV, OCC, kAny>(a, s);
+  }
 }
 
 }  // namespace chatts
@@ -542,6 +851,7 @@ using namespace chatts;
 extern "C" int chatts_window_prep(const ChattsWindowArgs* a, chatts_stream_t stream) {
   if (const int rc = check_window(a, "window_prep")) return rc;
   if (a->n_rows == 0) return CHATTS_OK;
+  if (a->taps > 0 || a->norm_whole) return a->cache_f32 ? launch_window_rows<float>(a, as_stream(stream)) : launch_window_rows<uint16_t>(a, as_stream(stream));
   int per_row = (a->heads + 2 * a->kv_heads + 3) / 4;
   if (per_row > 8192 / a->n_rows) per_row = 8192 / a->n_rows > 1 ? 8192 / a->n_rows : 1;
   if (a->cache_f32) hipLaunchKernelGGL(window_prep_kernel<float>, dim3(a->n_rows, per_row), dim3(256), 0, as_stream(stream), *a);

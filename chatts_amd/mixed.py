@@ -1,13 +1,16 @@
 """MixedDecoder - a served model whose layers each name their mixer, run by csrc/mixdec.hip.
 
 A sequential layer is norm1 -> mixer -> norm1b -> residual, then optionally norm2 -> squared-relu feed-forward -> norm2b -> residual; a parallel one adds
-mixer(norm1(x)) + feed-forward(norm2(x)) to x, both norms of the same x in groups (csrc/pair.hip).  Mixers:
+mixer(norm1(x)) + feed-forward(norm2(x)) to x, both norms of the same x in groups (csrc/pair.hip); a post-norm one is x <- norm1(alpha x + mixer(x)), then
+x <- norm2(alpha x + feed-forward(x)) (csrc/postnorm.hip).  Mixers:
   LatentMixer   attention over a paged cache of one latent + one rotated key part per token (csrc/latent.hip)
   DeltaMixer    gated delta rule: a float32 state and a ring of convolution inputs per slot (csrc/delta.hip)
-  WindowMixer   grouped-head attention over paged keys and values: per-head norms, window, kept first tokens, sink, gate (csrc/window.hip)
+  WindowMixer   grouped-head attention over paged keys and values (csrc/window.hip); by its fields: short convolutions with a ring of inputs per slot, norms
+                per head / over all heads / after a rotation, values mixed with an earlier layer's, window or chunks, kept first tokens, sink, capped
+                scores, a distance bias, a gate per value or per head
   WkvMixer, MlstmMixer   gated linear recurrences: a float32 state per slot (csrc/recur.hip)
-Feed-forwards of parallel layers: ClampGlu, Experts (csrc/moe.hip).
-A design (chatts_amd/fobolix.py, chatts_amd/medilix.py) says in which order layers run (config.runs(): a layer may run several times, every run has
+Feed-forwards of parallel and post-norm layers: ClampGlu, GeluGlu, Experts (csrc/moe.hip).
+A design (chatts_amd/fobolix.py, chatts_amd/medilix.py, chatts_amd/mefurax.py) says in which order layers run (config.runs(): a layer may run several times, every run has
 its own pages or state) and maps its tensor names onto LayerWeights.
 
 Everything is padded once, at load: widths and feed-forwards to multiples of 64, the stacked input projections block by block, heads to
@@ -88,9 +91,20 @@ class WindowMixer:
     k: Any
     v: Any
     g: Any          # output gate [heads * vdim, width] or None
-    q_norm: Any
+    q_norm: Any     # [dim] (norm_whole: [heads * dim], [kv_heads * dim]) or None
     k_norm: Any
     o: Any
+    bias: Any = None            # of q, k, v: (3 vectors) or None
+    conv: Any = None            # of q, k, v: ([channels, taps] each) or None
+    norm_whole: bool = False    # the norms run over all heads at once
+    rot: int = 0                # rotated dimensions, paired (2 i, 2 i + 1)
+    rot_base: float = 0.0
+    unit: bool = False          # queries and keys divided by their root mean square, after the rotation
+    chunk: int = 0              # 0: none
+    softcap: float = 0.0        # 0: none
+    slopes: Any = None          # [heads] or None
+    gate_heads: bool = False    # g is [heads, width]: one gate per head
+    vmix: Optional[float] = None    # values become (1 - vmix) v + vmix v_first, v_first those of the first layer that has a vmix
 
 
 @dataclass
@@ -138,14 +152,23 @@ class ClampGlu:
 
 
 @dataclass
+class GeluGlu:
+    gate: Any
+    up: Any
+    down: Any
+
+
+@dataclass
 class Experts:
     router: Any         # [experts + identity, width]
-    correction: Any
-    experts: Any        # (gate, up, down) each
+    correction: Any     # or None
+    experts: Any        # (gate, up, down) each; (up, down): squared relu
     identity: int
     top: int
     groups: int
     keep: int
+    by_logits: bool = False     # chosen by logits, weights: softmax over the chosen ones
+    shared: Any = None          # (up, down) of a squared-relu expert that every token uses (post-norm layers)
 
 
 @dataclass
@@ -157,8 +180,9 @@ class LayerWeights:
     norm2b: Any = None
     up: Any = None      # squared-relu feed-forward of a sequential layer
     down: Any = None
-    ff: Any = None      # ClampGlu or Experts of a parallel layer
+    ff: Any = None      # ClampGlu, GeluGlu or Experts of a parallel or post-norm layer
     parallel: bool = False
+    post: bool = False  # norms after the sums; norm1 / norm2 as they multiply
 
 
 def _up(n, m):
@@ -354,10 +378,15 @@ class MixedDecoder(SlotModel):
                                  a2d=self._pieces(m.a2, ra_p), g2d=self._pieces(m.g2, rg_p), ld_a2=ra_p, ld_g2=rg_p,
                                  dt_bias=self._f32(m.dt_bias), neg_a=self._f32(-torch.exp(m.a_log.to(torch.float32)).repeat_interleave(m.dim)), norm_w=self._f32(m.norm))
 
-    def _blocks(self, L, blocks, split=False):
-        """stacked input projection of a layer -> {name: first row}; split: every block has an operand of its own"""
+    def _blocks(self, L, blocks, split=False, bias=None):
+        """stacked input projection of a layer -> {name: first row}; split: every block has an operand of its own; bias: {name: vector}"""
         w, off = self._stack([(n, t, _up(t.shape[0], 64)) for n, t in blocks])
         L.in_n = w.shape[0]
+        if bias:
+            b = torch.zeros(L.in_n, dtype=torch.float32, device=self.device)
+            for n, t in bias.items():
+                b[off[n]:off[n] + t.shape[0]] = t.to(torch.float32)
+            L.in_bias = self._dev(b)
         L.w_in, L.in_t = self._mat(w, tile=not split)
         if split:
             L.n_mix = len(blocks)
@@ -370,13 +399,29 @@ class MixedDecoder(SlotModel):
 
     def _window_layer(self, L, m):
         L.kind = _lib.MIX_WINDOW
-        off = self._blocks(L, [("q", m.q), ("k", m.k), ("v", m.v)] + ([("g", m.g)] if m.g is not None else []))
+        off = self._blocks(L, [("q", m.q), ("k", m.k), ("v", m.v)] + ([("g", m.g)] if m.g is not None else []), bias=dict(zip("qkv", m.bias)) if m.bias else None)
         n, dim_p, vdim_p = m.heads * m.vdim, _up(m.dim, 32), _up(m.vdim, 16)
         L.out_k = _up(n, 64)
         L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
         L.window = _lib.WindowArgs(off_q=off["q"], off_k=off["k"], off_v=off["v"], off_gate=off.get("g", -1), heads=m.heads, kv_heads=m.kv_heads, dim=m.dim,
-                                   vdim=m.vdim, dim_p=dim_p, vdim_p=vdim_p, scale=m.scale, q_norm=self._f32(m.q_norm), k_norm=self._f32(m.k_norm),
-                                   window=m.window, keep_first=m.keep_first if m.window else 0, sink=int(m.sink))
+                                   vdim=m.vdim, dim_p=dim_p, vdim_p=vdim_p, scale=m.scale, window=m.window, keep_first=m.keep_first if m.window or m.chunk else 0, sink=int(m.sink),
+                                   chunk=m.chunk, softcap=m.softcap, gate_heads=int(m.gate_heads), norm_whole=int(m.norm_whole), rot=m.rot, unit=int(m.unit))
+        a = L.window
+        if m.q_norm is not None:
+            a.q_norm, a.k_norm = (self._f32(t, _up(t.shape[0], 4)) for t in (m.q_norm, m.k_norm))
+        if m.slopes is not None:
+            a.slopes = self._f32(torch.tensor(m.slopes, device=self.device))
+        if m.rot:
+            cos, sin = rotary_tables(m.rot, m.rot_base, self.max_ctx, None, self.device)
+            a.cos_tab, a.sin_tab = self._dev(cos), self._dev(sin)
+        if m.conv:
+            a.taps, a.conv_ch = m.conv[0].shape[1], off["v"] + _up(m.v.shape[0], 64)
+            conv = torch.zeros((a.taps, a.conv_ch), dtype=torch.float32, device=self.device)
+            for n_, t in zip("qkv", m.conv):
+                conv[:, off[n_]:off[n_] + t.shape[0]] = t.to(torch.float32).t()
+            a.conv_w = self._dev(conv)
+        if m.vmix is not None:
+            a.vmix, a.ld_vfirst = m.vmix, _up(m.kv_heads * m.vdim, 4)
         self._lat_q, self._lat_o = max(self._lat_q, m.heads * dim_p), max(self._lat_o, m.heads * (vdim_p + 4))
 
     def _wkv_layer(self, L, m):
@@ -419,17 +464,28 @@ class MixedDecoder(SlotModel):
         L.up, L.up_t = self._mat(self._gate_up(m.gate, m.up, L.ff), tile=True)
         L.down, L.down_t = self._mat(m.down, self._wp, L.ff, tile=True)
 
+    def _gelu_glu(self, L, m):
+        L.ff_kind, L.ff = _lib.FF_GEGLU, _up(m.gate.shape[0], 64)
+        L.up, L.up_t = self._mat(self._gate_up(m.gate, m.up, L.ff), tile=True)
+        L.down, L.down_t = self._mat(m.down, self._wp, L.ff, tile=True)
+
     def _experts(self, L, m):
-        n, ff = len(m.experts), _up(m.experts[0][0].shape[0], 64)
-        gu = torch.empty((n, 2 * ff, self._wp), dtype=torch.bfloat16, device=self.device)
+        n, ff, gated = len(m.experts), _up(m.experts[0][0].shape[0], 64), len(m.experts[0]) == 3
+        gu = torch.empty((n, 2 * ff if gated else ff, self._wp), dtype=torch.bfloat16, device=self.device)
         dn = torch.empty((n, self._wp, ff), dtype=torch.bfloat16, device=self.device)
-        for e, (gate, up, down) in enumerate(m.experts):
-            gu[e], dn[e] = self._gate_up(gate, up, ff), _pad(down.to(torch.bfloat16), self._wp, ff)
+        for e, x in enumerate(m.experts):
+            gu[e], dn[e] = self._gate_up(x[0], x[1], ff) if gated else _pad(x[0].to(torch.bfloat16), ff, self._wp), _pad(x[-1].to(torch.bfloat16), self._wp, ff)
         gut, dnt = (self._tiles(t) if self.tiled else None for t in (gu, dn))
         L.ff_kind, L.router_n = _lib.FF_MOE, _up(n + m.identity, 64)
         L.router, L.router_t = self._mat(m.router, L.router_n, self._wp, tile=True)
-        L.moe = _lib.MoeArgs(experts=n, identity=m.identity, top=m.top, groups=m.groups, keep=m.keep, width_p=self._wp, ff_p=ff, gate_up=self._dev(gu),
-                             down=self._dev(dn), gate_up_t=gut, down_t=dnt, correction=self._f32(m.correction))
+        L.moe = _lib.MoeArgs(experts=n, identity=m.identity, top=m.top, groups=m.groups, keep=m.keep,
+                             choose=_lib.CHOOSE_LOGITS if m.by_logits else _lib.CHOOSE_SOFTMAX, act_kind=_lib.EXPERT_SWIGLU if gated else _lib.EXPERT_RELU2,
+                             width_p=self._wp, ff_p=ff, gate_up=self._dev(gu), down=self._dev(dn), gate_up_t=gut, down_t=dnt,
+                             correction=None if m.correction is None else self._f32(m.correction))
+        if m.shared is not None:
+            L.ff = _up(m.shared[0].shape[0], 64)
+            L.up, L.up_t = self._mat(m.shared[0], L.ff, self._wp, tile=True)
+            L.down, L.down_t = self._mat(m.shared[1], self._wp, L.ff, tile=True)
 
     def _build(self, sd):
         cfg, lib, dev = self.config, self.lib, self.device
@@ -444,13 +500,13 @@ class MixedDecoder(SlotModel):
                  MlstmMixer: self._mlstm_layer}
         for i in range(len(cfg.layers)):
             lw, L = self.layer_weights(sd, i), arr[i]
-            L.norm1, L.parallel = self._f32(lw.norm1, Wp), int(lw.parallel)
+            L.norm1, L.parallel, L.post = self._f32(lw.norm1, Wp), int(lw.parallel), int(lw.post)
             if lw.norm1b is not None:
                 L.norm1b = self._f32(lw.norm1b, Wp)
             build[type(lw.mixer)](L, lw.mixer)
             if lw.ff is not None:
                 L.norm2 = self._f32(lw.norm2, Wp)
-                (self._glu if isinstance(lw.ff, ClampGlu) else self._experts)(L, lw.ff)
+                {ClampGlu: self._glu, GeluGlu: self._gelu_glu, Experts: self._experts}[type(lw.ff)](L, lw.ff)
             if lw.up is not None:
                 L.ff_kind = _lib.FF_RELU2
                 L.norm2, L.norm2b, L.ff = self._f32(lw.norm2, Wp), self._f32(lw.norm2b, Wp), _up(lw.up.shape[0], 64)
@@ -491,6 +547,10 @@ class MixedDecoder(SlotModel):
                 k, v = (torch.zeros((nblk, a.kv_heads, self.kv_block_size, d), dtype=cache_dtype, device=dev) for d in (a.dim_p, a.vdim_p))
                 runs[r].cache, runs[r].vcache = self._dev(k), self._dev(v)
                 self.cache_bytes += (k.numel() + v.numel()) * k.element_size()
+                if a.taps:
+                    ring = torch.zeros((MB, a.taps, a.conv_ch), **f32)
+                    runs[r].ring = self._dev(ring)
+                    self.state_bytes += 4 * ring.numel()
             elif arr[i].kind == _lib.MIX_RECUR:
                 a = arr[i].recur
                 mem = [torch.zeros((MB, a.heads, a.dim, _up(a.vdim, 4)), **f32), torch.zeros((MB, Wp), **f32) if arr[i].n_mix else None]
@@ -511,11 +571,18 @@ class MixedDecoder(SlotModel):
         most = lambda f: max([f(L) for L in deltas], default=1)
         over = lambda layers, f: max([f(L) for L in layers], default=1)
         shifts, pairs, n_mix = bool(over(recurs, lambda L: L.n_mix) > 1), T * over(moes, lambda L: L.moe.top), over(arr, lambda L: L.n_mix)
+        mixing = [i for i, _ in order if isinstance(mixers[i], WindowMixer) and mixers[i].vmix is not None]      # value mixing: the first leaves its values
+        if mixing:
+            if len({mixers[i].kv_heads * mixers[i].vdim for i in mixing}) > 1:
+                raise ValueError("layers that mix their values with the first one's must have as many")
+            arr[mixing[0]].window.vfirst_write = 1
+        ldv = arr[mixing[0]].window.ld_vfirst if mixing else 4
         bigram = mw.get("bigram")
         mc = _lib.MixConfig(width=W, width_p=Wp, n_layers=len(arr), n_runs=len(order), exact=int(self.exact), t_max=T, max_slots=MB, max_ctx=self.max_ctx,
                             expand_rows=self.expand_rows if self._exp[0] else 0,
                             vocab=V, vocab_p=Vp, eps=cfg.rms_norm_eps, block_size=self.kv_block_size, table_stride=bps,
-                            norm_groups=getattr(cfg, "norm_groups", 1), embed_scale=mw.get("embed_scale", 1.0))
+                            norm_groups=getattr(cfg, "norm_groups", 1), embed_scale=mw.get("embed_scale", 1.0),
+                            alpha=mw.get("alpha", 1.0))
         if bigram:
             mc.bigram_buckets, mc.bigram_prev, mc.bigram_cur = bigram[1:]
         ws = int(lib.chatts_mixdec_workspace(C.byref(mc), arr))
@@ -554,6 +621,7 @@ class MixedDecoder(SlotModel):
             "moe_y": torch.zeros((pairs, Wp) if moes else (1, 1), **f32),
             "act_f32": torch.zeros((pairs, over(moes, lambda L: L.moe.ff_p)) if self.exact else (1, 1), **f32),
             "act_planes": torch.zeros((2, pairs, over(moes, lambda L: L.moe.ff_p)) if not self.exact else (2, 1, 1), **bf),
+            "vfirst": torch.zeros((rows, ldv) if mixing else (1, 4), **f32),
             "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
             "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),
@@ -569,7 +637,7 @@ class MixedDecoder(SlotModel):
                              q_lo=P(B["q_planes"][1]), partial_elems=B["partial"].numel(), qx=P(B["x_q"]), cbuf=P(B["x_c"]), krbuf=P(B["x_kr"]),
                              kx_hi=P(B["x_k"][0]), kx_lo=P(B["x_k"][1]), vx_hi=P(B["x_v"][0]), vx_lo=P(B["x_v"][1]), zero=P(B["x_zero"]), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
                              logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
-                             bigram=self._mat(bigram[0], None, Wp)[0] if bigram else None, x0=P(B["x0"]) if join else None, mix_stride=rows * Wp,
+                             bigram=self._mat(bigram[0], None, Wp)[0] if bigram else None, x0=P(B["x0"]) if join else None, mix_stride=rows * Wp, vfirst=P(B["vfirst"]), ld_vfirst=ldv,
                              **{f"{n}_{h}": P(B[f"{n}_planes"][j]) for n in ("m", "n", "act") for j, h in enumerate(("hi", "lo"))},
                              **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout", "prev_token", "h", "m_f32", "n_f32", "gates", "den",
                                                      "moe_ids", "moe_place", "moe_order", "moe_offsets", "moe_tiles", "moe_weight", "moe_kept", "moe_logits", "moe_y",

@@ -53,8 +53,11 @@ const char* chatts_last_error(void);
  * 10: decoders of mixed layers chatts_mixdec_* with their kernels (chatts_residual_norm, chatts_delta_*, chatts_latent_*, chatts_head_linear),
  *     CHATTS_EPI_RELU2, ChattsLinearArgs.exact_f32;
  * 11: chatts_recur_*, chatts_window_*, chatts_moe_*, chatts_pair_norm, chatts_token_shift, chatts_embed_pair; parallel layers and joined passes of
- *     chatts_mixdec_*; CHATTS_EPI_CLAMPGLU, ChattsLinearArgs.glu_limit / glu_alpha. */
-#define CHATTS_ABI_VERSION 11
+ *     chatts_mixdec_*; CHATTS_EPI_CLAMPGLU, ChattsLinearArgs.glu_limit / glu_alpha;
+ * 12: chatts_post_norm and layers with their norms after the sums; windowed attention with chunks, capped scores, distance slopes, gates per head,
+ *     rotation, unit queries and keys, norms over all heads, short convolutions and mixed values; experts without a gate, choice by logits;
+ *     CHATTS_EPI_GEGLU. */
+#define CHATTS_ABI_VERSION 12
 int chatts_abi_version(void);
 /* Number of CUs of the current device (grid sizing), or <0. */
 int chatts_device_cus(void);
@@ -156,6 +159,7 @@ int chatts_ts_encode(const float* series, const int32_t* row_off, const int32_t*
 #define CHATTS_EPI_RELU2 4    /* C = max(acc + bias, 0)^2              (bf16 weights)               */
 #define CHATTS_EPI_CLAMPGLU 5 /* rows as for SWIGLU; g = min(gate, glu_limit), u = clamp(up, +-glu_limit): */
                               /* C[M,N/2] = g sigmoid(glu_alpha g) (u + 1)   (bf16 weights)         */
+#define CHATTS_EPI_GEGLU 6    /* rows as for SWIGLU; C[M,N/2] = gelu(gate) * up, gelu in its tanh form (bf16 weights) */
 
 typedef struct ChattsLinearArgs {
   const float* a;          /* [M, lda] */
@@ -938,6 +942,23 @@ typedef struct ChattsTokenShiftArgs {
 } ChattsTokenShiftArgs;
 int chatts_token_shift(const ChattsTokenShiftArgs* args, chatts_stream_t stream);
 
+/* ---- layers whose norm stands after the sum (postnorm.hip): one launch per row of the stream ----
+ *   x <- n w,  n = s / rms(s),  s = alpha x + y + sum_j weight[j] ey[place[j]]        (y NULL: none; ey NULL: no experts)
+ * `w` is the weight as it multiplies, padded with zeros to ldx.  out: the new x once more as an operand (NULL pointers: not wanted). */
+typedef struct ChattsPostNormArgs {
+  float* x;                  /* [T, ldx], updated in place */
+  int t, width, ldx;
+  float alpha, eps;
+  const float* y;            /* [T, ldx] */
+  const float* ey;           /* [places, ldx] */
+  const int32_t* place;      /* [T, top], < 0: none */
+  const float* weight;       /* [T, top] */
+  int top;
+  const float* w;
+  ChattsOperand out;
+} ChattsPostNormArgs;
+int chatts_post_norm(const ChattsPostNormArgs* args, chatts_stream_t stream);
+
 /* ---- gated linear recurrences (recur.hip): S <- diag(g_t) S + k_t v_t^T per head, float32 ----
  * CHATTS_RECUR_WKV    g = exp(-exp(W2 tanh(a) + w0)) per key channel;  o = S^T q + (q . (u k)) v with S before the token's own write;
  *                     out = o / rms(o) * norm_w * silu(gate)
@@ -980,16 +1001,36 @@ int chatts_recur_scan(const ChattsRecurArgs* args, chatts_stream_t stream);     
 int chatts_recur_out(const ChattsRecurArgs* args, chatts_stream_t stream);         /* ... norm and gate of the read-outs */
 int64_t chatts_recur_chunk_floats(int heads, int dim, int n_rows, int n_spans);
 
-/* ---- attention over paged keys and values, grouped heads, per-head norms, optional window / kept first tokens / sink / gate (window.hip) ----
+/* ---- attention over paged keys and values, grouped heads (window.hip); everything that follows is optional ----
  * Pages of 2^log_block tokens: keys [page][kv head][token][dim_p], values [page][kv head][token][vdim_p], bf16 or float32.
- * Position i sees j <= i with i - j < window or j < keep_first (window 0: all).  sink: one more term exp(0) in the softmax's denominator. */
+ * On the way in (chatts_window_prep), in this order:
+ *   taps          q, k, v: y_t = sum_j conv_w[j] u_(t - taps + 1 + j) per channel, zeros before the sequence; the last inputs stay in `ring`
+ *   q_norm        RMS norm of every head with a weight [dim]; norm_whole: of all heads at once with a weight [heads * dim]
+ *   rot           dimensions 2 i and 2 i + 1 < rot of a head turned by the angle whose cos / sin are in row `pos` of the tables
+ *   unit          queries and keys divided by their root mean square, per head
+ *   vfirst        values become (1 - vmix) v + vmix vfirst of the same row; vfirst_write: they are left there as they are instead
+ * (taps and norm_whole work on whole rows; they do not combine with per-head norms, rot or unit.)
+ * Scores: q . k * scale, then softcap tanh(score / softcap), then minus slopes[h] * distance.
+ * Position i sees j <= i with i - j < window or j < keep_first (window 0: all); chunk: with i / chunk == j / chunk.
+ * sink: one more term exp(0) in the softmax's denominator.  Gate: sigmoid, one per output; gate_heads: one per head. */
 typedef struct ChattsWindowArgs {
   const float* proj;
   int ld_proj, off_q, off_k, off_v, off_gate;        /* off_gate < 0: no gate */
   int heads, kv_heads, dim, vdim, dim_p, vdim_p;     /* dim_p % 32 == 0, vdim_p % 16 == 0 */
   float scale, eps;
-  const float *q_norm, *k_norm;                      /* [dim] */
+  const float *q_norm, *k_norm;                      /* [dim] (norm_whole: [heads * dim], [kv_heads * dim], padded to fours), both or neither */
   int window, keep_first, sink;
+  int chunk;                                         /* not beside a window */
+  float softcap;                                     /* 0: none */
+  const float* slopes;                               /* [heads] or NULL */
+  int gate_heads, norm_whole, rot, unit;             /* rot even */
+  const float *cos_tab, *sin_tab;                    /* [positions, rot / 2] */
+  int taps, conv_ch;                                 /* 0: no convolution; q, k, v lie in the first conv_ch columns */
+  const float* conv_w;                               /* [taps, conv_ch] */
+  float* ring;                                       /* [slots, taps, conv_ch]: inputs by position modulo taps */
+  float vmix;
+  float* vfirst;                                     /* [T, ld_vfirst] or NULL */
+  int ld_vfirst, vfirst_write;
   void *kcache, *vcache;
   int cache_f32;
   const int32_t* table;
@@ -1008,12 +1049,20 @@ int chatts_window_attend(const ChattsWindowArgs* args, chatts_stream_t stream); 
 int chatts_window_prefill(const ChattsWindowArgs* args, chatts_stream_t stream);   /* segments of many rows (bf16 pages) */
 int chatts_window_can_prefill(int dim_p, int vdim_p);
 
-/* ---- mixture of experts (moe.hip): softmax router with a correction of the choice, groups, identity experts ----
- * Outputs of the router: `experts` feed-forwards W_down (silu(W_gate h) * W_up h), then `identity` outputs that return h. */
+/* ---- mixture of experts (moe.hip): choice groups, identity experts ----
+ * Outputs of the router: `experts` feed-forwards, then `identity` outputs that return h.
+ * CHATTS_CHOOSE_SOFTMAX  the best softmax + correction; weights: the chosen softmax values over their sum
+ * CHATTS_CHOOSE_LOGITS   the best logit + correction (NULL: none); weights: softmax over the chosen logits
+ * CHATTS_EXPERT_SWIGLU   W_down (silu(W_gate h) * W_up h);   CHATTS_EXPERT_RELU2   W_down max(W_up h, 0)^2 */
+#define CHATTS_CHOOSE_SOFTMAX 0
+#define CHATTS_CHOOSE_LOGITS 1
+#define CHATTS_EXPERT_SWIGLU 0
+#define CHATTS_EXPERT_RELU2 1
 typedef struct ChattsMoeArgs {
   int experts, identity, top, groups, keep;
+  int choose, act_kind;                 /* CHATTS_CHOOSE_*, CHATTS_EXPERT_* */
   int width_p, ff_p;                    /* both % 64 == 0 */
-  const chatts_bf16* gate_up;           /* [experts][2 ff_p][width_p], gate / up rows interleaved in blocks of 16 */
+  const chatts_bf16* gate_up;           /* SWIGLU: [experts][2 ff_p][width_p], gate / up rows interleaved in blocks of 16; RELU2: up [experts][ff_p][width_p] */
   const chatts_bf16* down;              /* [experts][width_p][ff_p] */
   const chatts_bf16 *gate_up_t, *down_t;   /* chatts_tile_bf16 copy of every matrix, one after the other, or NULL */
   const float* correction;              /* [experts + identity] */
@@ -1040,6 +1089,7 @@ int chatts_moe_tiles(int rows, int top, int experts);
 #define CHATTS_FF_RELU2 1
 #define CHATTS_FF_CLAMPGLU 2
 #define CHATTS_FF_MOE 3
+#define CHATTS_FF_GEGLU 4
 typedef struct ChattsMixLayer {
   int kind;                                          /* CHATTS_MIX_* */
   const float *norm1, *norm1b, *norm2, *norm2b;      /* before / after the mixer, before / after the feed-forward; padded with zeros to width_p */
@@ -1066,13 +1116,16 @@ typedef struct ChattsMixLayer {
   const chatts_bf16 *router, *router_t;              /* [router_n, width_p] */
   int router_n;
   ChattsMoeArgs moe;
+  int post;                                          /* norms after the sums: x <- norm1(alpha x + mixer(x)), x <- norm2(alpha x + ff(x)); MIX_WINDOW;
+                                                      * FF_GEGLU: up = [2 ff, width_p] interleaved; FF_MOE: up / down: a shared squared-relu expert */
+  const float* in_bias;                              /* [in_n] or NULL (post) */
 } ChattsMixLayer;
 typedef struct ChattsMixRun {      /* one pass through a layer */
   int layer;
   const float* add;                /* vector added to the residual stream before it, or NULL */
   void* cache;                     /* latent: this run's pages */
   float* state;                    /* delta, recur: this run's states */
-  float* ring;                     /* delta: convolution rings; recur: the previous token's mixer input [slots, width_p] */
+  float* ring;                     /* delta, window: convolution rings; recur: the previous token's mixer input [slots, width_p] */
   float *n_state, *m_state;        /* recur, mlstm */
   void* vcache;                    /* window: value pages (cache: key pages) */
   const chatts_bf16 *join, *join_t;   /* x <- join [x | x0] before it, [width_p, 2 width_p], or NULL */
@@ -1086,6 +1139,7 @@ typedef struct ChattsMixConfig {
   int norm_groups;
   float embed_scale;
   int64_t bigram_buckets, bigram_prev, bigram_cur;
+  float alpha;                     /* layers with norms after the sums: factor of x in them */
 } ChattsMixConfig;
 typedef struct ChattsMixBuffers {
   const chatts_bf16 *embed, *head, *head_t;          /* [vocab, width_p], [vocab_p, width_p] */
@@ -1119,6 +1173,8 @@ typedef struct ChattsMixBuffers {
   float* logits;                                     /* [>= rows asked for, vocab_p] */
   void* workspace;
   size_t workspace_bytes;
+  float* vfirst;                                     /* window, mixed values: [t_max, ld_vfirst] */
+  int ld_vfirst;
 } ChattsMixBuffers;
 typedef struct ChattsMixDecoder ChattsMixDecoder;
 ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, const ChattsMixLayer* layers, const ChattsMixRun* runs, const ChattsMixBuffers* b);
