@@ -544,6 +544,23 @@ def medilix_config(size, layers, vocab):
                          embedding={"scale": 1.0, "bigram": {"buckets": 32003, "mul_prev": 31, "mul_cur": 7}})
 
 
+def mefurax_config(size, layers, vocab):
+    """chunked and windowed attention in turn, both with mixed values; every second feed-forward has experts (the chosen ones and the shared one weigh
+    as much as a dense one)"""
+    from chatts_amd.mefurax import MefuraxConfig
+    W, _, inter, heads = DESIGN_SIZES[size]
+    dense = {"kind": "dense", "ff": inter}
+    moe = {"kind": "moe", "expert": {"ff": inter * 3 // 16}, "router": {"experts": 32, "top": 4}, "shared": {"ff": inter * 3 // 4}}
+    common = {"heads": heads, "kv_heads": 8, "dim": 128, "vdim": 128, "v_mix": True, "mask": {"size": 1024}}
+    window = {"type": "attention", "mixer": dict(common, scale=128 ** -0.5, conv=4)}
+    chunk = {"type": "attention_2", "mixer": dict(common, mask={"size": 1536}, scale=0.125, softcap=30.0, rot={"base": 500000.0, "dims": 64})}
+    kinds = [dict(chunk, mlp=dense), dict(window, mlp=moe), dict(chunk, mlp=moe), dict(window, mlp=dense)]
+    return MefuraxConfig(vocab=vocab, width=W, layers=[kinds[i % 4] for i in range(layers)], norm={"eps": 1e-5}, postln_alpha=2.0, name=f"mefurax-{size}")
+
+
+DESIGNS = {"fobolix": fobolix_config, "medilix": medilix_config, "mefurax": mefurax_config}
+
+
 def qwen_config(size, layers, vocab):
     from chatts_amd.config import preset
     W, _, inter, heads = DESIGN_SIZES[size]
@@ -560,7 +577,7 @@ def bench_design(args):
     torch.cuda.set_device(0)
     g = torch.Generator().manual_seed(0)
     for size in args.design_sizes.split(","):
-        for name, make in ((args.design, {"fobolix": fobolix_config, "medilix": medilix_config}[args.design]), ("qwen", qwen_config)):
+        for name, make in ((args.design, DESIGNS[args.design]), ("qwen", qwen_config)):
             if args.design_only and name != args.design_only:
                 continue
             cfg = make(size, args.layers or 8, 32000)
@@ -686,10 +703,10 @@ def main():
     ap.add_argument("--weights", default="bf16", choices=["bf16", "fp8", "int8", "int4"],
                     help="fp8 = BASELINE.json config 5 weight format, int4 = the GPTQ-Int4 checkpoint's (NOT the headline: separate workloads)")
     ap.add_argument("--launch-check", action="store_true", help="only prove the N-rank launch path (no model): rank 0 prints the world it saw")
-    ap.add_argument("--design", default=None, choices=["fobolix", "medilix"], help="another workload: layers of this design beside the Qwen decoder at equal size, random weights")
+    ap.add_argument("--design", default=None, choices=sorted(DESIGNS), help="another workload: layers of this design beside the Qwen decoder at equal size, random weights")
     ap.add_argument("--design-sizes", default="s,m,l", help=f"of {sorted(DESIGN_SIZES)}")
     ap.add_argument("--design-prompt", type=int, default=2048)
-    ap.add_argument("--design-only", default=None, choices=["fobolix", "medilix", "qwen"], help="one of the two models (profiling)")
+    ap.add_argument("--design-only", default=None, choices=sorted(DESIGNS) + ["qwen"], help="one of the two models (profiling)")
     args = ap.parse_args()
 
     if args.design:

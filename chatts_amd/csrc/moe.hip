@@ -9,6 +9,8 @@
 //   moe_gemm_f32_kernel   32-bit runs
 // Places: the pairs of expert e are places offsets[e] .. offsets[e + 1) of the packed buffers act and y; order[place] = token * top + choice.
 // The weighted sum over a token's places is part of the norm that follows (chatts_pair_norm).
+#include <type_traits>
+
 #include "gemm_common.h"
 
 namespace chatts {
@@ -236,18 +238,19 @@ __device__ __forceinline__ void moe_relu2_4(const ChattsOperand& o, size_t row, 
   store_operand4(o, row, col, v);
 }
 
-// ---- up to 16 rows: grid (blocks of 32 weight rows, tiles), 4 waves split K; D = W . A^T: a lane holds 4 consecutive outputs of one token.
-// kGated: the two 16-row halves of a block are gate and up rows of the same outputs ----
+// ---- up to 16 rows: grid (blocks of 16 RF weight rows, tiles), NW waves split K; D = W . A^T: a lane holds 4 consecutive outputs of one token.
+// kGated (RF = 2): the two 16-row halves of a block are gate and up rows of the same outputs ----
 // TILED: weights from the chatts_tile_bf16 copy: a fragment's 64 pieces are 1 KB of consecutive memory
-template <int STEP, bool TILED>
-__global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
-  __shared__ f32x4 red[4][2][64];
+template <int STEP, bool TILED, int NW, int RF>
+__global__ __launch_bounds__(64 * NW) void moe_stream_kernel(ChattsMoeArgs p) {
+  __shared__ f32x4 red[NW][RF][64];
+  static_assert(STEP != kGated || RF == 2, "a pair of fragments");
   constexpr bool IN = STEP != kDown;
   const int32_t* tile = p.tiles + (size_t)blockIdx.y * 4;
   const int e = tile[0];
   if (e < 0) return;
-  const int place0 = tile[1], count = tile[2], lane = threadIdx.x & 63, wave = threadIdx.x >> 6, fr = lane & 15, fg = lane >> 4;
-  const int K = IN ? p.width_p : p.ff_p, N = IN ? moe_in_rows(p) : p.width_p, n0 = blockIdx.x * 32;
+  const int place0 = tile[1], count = tile[2], lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), fr = lane & 15, fg = lane >> 4;
+  const int K = IN ? p.width_p : p.ff_p, N = IN ? moe_in_rows(p) : p.width_p, n0 = blockIdx.x * 16 * RF;
   const uint16_t* w = TILED ? (IN ? p.gate_up_t : p.down_t) + ((size_t)e * N + n0) * K + (fr * 4 + (fg ^ ((fr >> 3) << 1))) * 8
                             : (IN ? p.gate_up : p.down) + ((size_t)e * N + n0 + fr) * K + fg * 8;
   constexpr int kStep = TILED ? 16 : 1;      // elements of w per K-value
@@ -255,53 +258,59 @@ __global__ __launch_bounds__(256) void moe_stream_kernel(ChattsMoeArgs p) {
   const size_t arow = IN ? (size_t)(p.order[pl] / p.top) * p.h.ld : (size_t)pl * p.act.ld;
   const uint16_t* ah = (IN ? p.h.hi : p.act.hi) + arow + fg * 8;
   const uint16_t* al = (IN ? p.h.lo : p.act.lo) + arow + fg * 8;
-  f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-  constexpr int U = 4;
-  const int steps = K >> 5;      // K-steps of 32: wave, wave + 4, ...
-  for (int k0 = wave; k0 < steps; k0 += 4 * U) {
-    bf16x8_t wv[U][2], hv[U], lv[U];
+  f32x4 acc[RF];
+#pragma unroll
+  for (int f = 0; f < RF; ++f) acc[f] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  // K-steps of 32: wave, wave + NW, ...; U of them requested at once
+  auto run = [&](auto u_c, int k0) __attribute__((always_inline)) {
+    constexpr int U = decltype(u_c)::value;
+    bf16x8_t wv[U][RF], hv[U], lv[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int f = 0; f < RF; ++f)
+        wv[u][f] = __builtin_bit_cast(bf16x8_t, __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + (size_t)16 * f * K + (k0 + NW * u) * 32 * kStep)));
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const int k = k0 + 4 * u < steps ? (k0 + 4 * u) * 32 : 0;
-      const u32x4 a = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + k * kStep)), b = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w + (size_t)16 * K + k * kStep));
-      wv[u][0] = __builtin_bit_cast(bf16x8_t, a);
-      wv[u][1] = __builtin_bit_cast(bf16x8_t, b);
-    }
-#pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const int k = k0 + 4 * u < steps ? (k0 + 4 * u) * 32 : 0;
-      hv[u] = *reinterpret_cast<const bf16x8_t*>(ah + k);
-      lv[u] = *reinterpret_cast<const bf16x8_t*>(al + k);
+      hv[u] = *reinterpret_cast<const bf16x8_t*>(ah + (k0 + NW * u) * 32);
+      lv[u] = *reinterpret_cast<const bf16x8_t*>(al + (k0 + NW * u) * 32);
     }
 #pragma unroll
     for (int u = 0; u < U; ++u)
-      if (k0 + 4 * u < steps) {
 #pragma unroll
-        for (int f = 0; f < 2; ++f) {
-          acc[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][f], lv[u], acc[f], 0, 0, 0);
-          acc[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][f], hv[u], acc[f], 0, 0, 0);
-        }
+      for (int f = 0; f < RF; ++f) {
+        acc[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][f], lv[u], acc[f], 0, 0, 0);
+        acc[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u][f], hv[u], acc[f], 0, 0, 0);
       }
-  }
-  red[wave][0][lane] = acc[0];
-  red[wave][1][lane] = acc[1];
+  };
+  const int steps = K >> 5;
+  int mine = wave < steps ? (steps - wave + NW - 1) / NW : 0, k0 = wave;
+  for (; mine >= 4; mine -= 4, k0 += 4 * NW) run(std::integral_constant<int, 4>{}, k0);
+  if (mine == 3) run(std::integral_constant<int, 3>{}, k0);
+  else if (mine == 2) run(std::integral_constant<int, 2>{}, k0);
+  else if (mine == 1) run(std::integral_constant<int, 1>{}, k0);
+#pragma unroll
+  for (int f = 0; f < RF; ++f) red[wave][f][lane] = acc[f];
   __syncthreads();
-  if (wave >= (STEP == kGated ? 1 : 2)) return;
-  f32x4 s[2];
+  if (wave >= (STEP == kGated ? 1 : RF)) return;
+  f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};      // (kGated: gate and up; otherwise s[0] = this wave's fragment)
 #pragma unroll
-  for (int f = 0; f < 2; ++f)
+  for (int f = 0; f < (STEP == kGated ? 2 : 1); ++f)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) s[f][r] = (red[0][f][lane][r] + red[1][f][lane][r]) + (red[2][f][lane][r] + red[3][f][lane][r]);
+    for (int x = 0; x < NW; x += 4) {
+      const int g = STEP == kGated ? f : wave;
+      s[f] += (red[x][g][lane] + red[x + 1][g][lane]) + (red[x + 2][g][lane] + red[x + 3][g][lane]);
+    }
   if (fr >= count) return;
   if (STEP == kRelu2) {
-    moe_relu2_4(p.act, place0 + fr, n0 + wave * 16 + fg * 4, wave ? s[1] : s[0]);
+    moe_relu2_4(p.act, place0 + fr, n0 + wave * 16 + fg * 4, s[0]);
   } else if (STEP == kGated) {
     float v[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = moe_glu(s[0][r], s[1][r]);
     store_operand4(p.act, place0 + fr, (n0 >> 1) + fg * 4, v);
   } else {
-    *reinterpret_cast<f32x4*>(p.y + (size_t)(place0 + fr) * p.width_p + n0 + wave * 16 + fg * 4) = wave ? s[1] : s[0];
+    *reinterpret_cast<f32x4*>(p.y + (size_t)(place0 + fr) * p.width_p + n0 + wave * 16 + fg * 4) = s[0];
   }
 }
 
@@ -493,6 +502,20 @@ static int moe_tile_bound(int rows, int top, int experts, int bm) {      // sum 
   return (int)(pairs / bm + lists);
 }
 
+template <int STEP, int RF>
+static void launch_moe_stream_as(const ChattsMoeArgs* a, int n, int tiles, hipStream_t s) {
+  constexpr int NW = STEP == kGated ? 4 : 16;
+  const dim3 g(n / (16 * RF), tiles), b(64 * NW);
+  if (STEP == kDown ? a->down_t : a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<STEP, true, NW, RF>), g, b, 0, s, *a);
+  else hipLaunchKernelGGL((moe_stream_kernel<STEP, false, NW, RF>), g, b, 0, s, *a);
+}
+template <int STEP>
+static void launch_moe_stream(const ChattsMoeArgs* a, int n, int tiles, hipStream_t s) {      // few workgroups: smaller ones, so that the CUs get as much each
+  if constexpr (STEP != kGated)
+    if (n / 32 * tiles < 2 * device_cus()) return launch_moe_stream_as<STEP, 1>(a, n, tiles, s);
+  launch_moe_stream_as<STEP, 2>(a, n, tiles, s);
+}
+
 template <int STEP, int BM, int WM, int WN>
 static int launch_moe_gemm(const ChattsMoeArgs* a, int tiles, hipStream_t s) {
   constexpr int LDS = (128 + 2 * BM) * kMoeLd * 2;
@@ -548,13 +571,9 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
     return CHATTS_OK;
   }
   if (moe_small(a)) {
-    const dim3 g1(in_rows / 32, tiles), g2(a->width_p / 32, tiles), b(256);
-    if (relu2 && a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<kRelu2, true>), g1, b, 0, s, *a);
-    else if (relu2) hipLaunchKernelGGL((moe_stream_kernel<kRelu2, false>), g1, b, 0, s, *a);
-    else if (a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<kGated, true>), g1, b, 0, s, *a);
-    else hipLaunchKernelGGL((moe_stream_kernel<kGated, false>), g1, b, 0, s, *a);
-    if (a->down_t) hipLaunchKernelGGL((moe_stream_kernel<kDown, true>), g2, b, 0, s, *a);
-    else hipLaunchKernelGGL((moe_stream_kernel<kDown, false>), g2, b, 0, s, *a);
+    if (relu2) launch_moe_stream<kRelu2>(a, in_rows, tiles, s);
+    else launch_moe_stream<kGated>(a, in_rows, tiles, s);
+    launch_moe_stream<kDown>(a, a->width_p, tiles, s);
     CHATTS_CHECK_LAUNCH("moe_stream");
     return CHATTS_OK;
   }

@@ -2,6 +2,7 @@
 // keys (per head, over all heads, unit after a rotation of pairs), mixed values; capped scores, a distance bias per head, a sliding window that keeps
 // a sequence's first tokens, chunks, a sink (one more term exp(0) in the denominator); an output gate per value or per head.
 //   window_prep_kernel      per-head work: norms, rotation, values; queries as an operand, keys and values into their pages
+//   window_prep_quads_kernel  the same, four channels a lane
 //   window_prep_rows_kernel the same for layers with convolutions or norms over all heads: a workgroup owns whole rows
 //   window_ring_kernel      the last convolution inputs of every segment
 //   window_attend_kernel    one row and query head per workgroup, vector units: 32-bit runs, head sizes beyond the matrix kernels
@@ -123,21 +124,101 @@ __global__ __launch_bounds__(256) void window_prep_kernel(ChattsWindowArgs p) {
   }
 }
 
+// The same with quads of neighbouring channels per lane, LPH lanes to a head (dim, vdim <= 4 LPH, all sizes % 4 == 0): grid (rows, n), the 4 n waves of a row
+// take 64 / LPH heads at a time, two such groups requested at once
+template <int LPH>
+__device__ __forceinline__ float head_sum(float v) {
+  v = row16_sum(v);
+  if (LPH >= 32) v += __shfl_xor(v, 16, 64);
+  if (LPH >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+__device__ __forceinline__ float quad_squares(const f32x4& v) { return (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+template <typename CT>
+__device__ __forceinline__ void store_page4(CT* dst, const f32x4& v) {
+  if constexpr (sizeof(CT) == 4) *reinterpret_cast<f32x4*>(dst) = v;
+  else *reinterpret_cast<w16x4*>(dst) = (w16x4){(short)to_page<CT>(v[0]), (short)to_page<CT>(v[1]), (short)to_page<CT>(v[2]), (short)to_page<CT>(v[3])};
+}
+template <typename CT, int LPH>
+__global__ __launch_bounds__(256) void window_prep_quads_kernel(ChattsWindowArgs p) {
+  constexpr int PER = 64 / LPH;
+  const int row = blockIdx.x, lane = threadIdx.x & 63, H = p.heads, G = p.kv_heads, c = (lane & (LPH - 1)) * 4;
+  const ChattsRow R = p.rows[row];
+  if (R.pos < 0) return;
+  const float* pr = p.proj + (size_t)row * p.ld_proj;
+  const size_t page = window_tile(p, R.slot, 0, R.pos);      // head e of the page: e << log_block rows further
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  const int stride = 4 * PER * gridDim.y;
+  for (int e0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * PER + lane / LPH; e0 - lane / LPH < H + 2 * G; e0 += 2 * stride) {      // (uniform)
+    f32x4 x[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int e = e0 + u * stride;
+      const bool value = e >= H + G;
+      const int n = value ? p.vdim : p.dim;
+      x[u] = zero;
+      if (e < H + 2 * G && c < n) x[u] = *reinterpret_cast<const f32x4*>(pr + (e < H ? p.off_q + e * n : (value ? p.off_v + (e - H - G) * n : p.off_k + (e - H) * n)) + c);
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int e = e0 + u * stride;
+      const bool value = e >= H + G, live = e < H + 2 * G;
+      const int n = value ? p.vdim : p.dim, np = value ? p.vdim_p : p.dim_p, hk = value ? e - H - G : e - H;
+      f32x4 v = x[u];
+      if (p.q_norm && !value) {
+        const float* w = e < H ? p.q_norm : p.k_norm;
+        const float f = 1.0f / sqrtf(head_sum<LPH>(quad_squares(v)) / (float)n + p.eps);
+        if (c < n) v = v * f * *reinterpret_cast<const f32x4*>(w + c);
+      }
+      if (!value && c < p.rot) {
+        const size_t at = (size_t)R.pos * (p.rot >> 1) + (c >> 1);
+        const float c0 = p.cos_tab[at], s0 = p.sin_tab[at];
+        v = (f32x4){v[0] * c0 - v[1] * s0, v[1] * c0 + v[0] * s0, v[2], v[3]};
+        if (c + 2 < p.rot) {
+          const float c1 = p.cos_tab[at + 1], s1 = p.sin_tab[at + 1];
+          v = (f32x4){v[0], v[1], v[2] * c1 - v[3] * s1, v[3] * c1 + v[2] * s1};
+        }
+      }
+      if (p.unit && !value) v = v * (1.0f / sqrtf(head_sum<LPH>(quad_squares(v)) / (float)n + p.eps));
+      if (value && p.vfirst && live && c < n) {
+        float* first = p.vfirst + (size_t)row * p.ld_vfirst + hk * n + c;
+        if (p.vfirst_write) *reinterpret_cast<f32x4*>(first) = v;
+        else v = (1.f - p.vmix) * v + p.vmix * *reinterpret_cast<const f32x4*>(first);
+      }
+      if (!live) continue;
+      for (int cc = c; cc < np; cc += 4 * LPH) {      // (a second pass only over padding)
+        const f32x4 y = cc == c ? v : zero;
+        if (e < H) {
+          const float o[4] = {y[0], y[1], y[2], y[3]};
+          store_operand4(p.q, row, e * p.dim_p + cc, o);
+        } else {
+          store_page4(reinterpret_cast<CT*>(value ? p.vcache : p.kcache) + (page + ((size_t)hk << p.log_block)) * np + cc, y);
+        }
+      }
+    }
+  }
+}
+
 // A workgroup owns ROWS rows, a thread quads of channels of [q | k | v]: convolutions over a window of rows in registers (inputs before a segment come from
 // the ring), norms over all heads, mixed values.
 constexpr int kConvRegs = 4;      // taps whose weights stay in registers
 template <typename CT, int NT, int NV, int ROWS>
-__global__ __launch_bounds__(NT) void window_prep_rows_kernel(ChattsWindowArgs p) {
+__global__ __launch_bounds__(NT, 4) void window_prep_rows_kernel(ChattsWindowArgs p) {
   __shared__ float red[NT / 64][2 * ROWS];
-  const int row0 = blockIdx.x * ROWS, tid = threadIdx.x, H = p.heads, G = p.kv_heads;
+  // neighbouring groups share rows: XCD x (= blockIdx % 8; speed only) takes a contiguous eighth of them
+  const int share = gridDim.x >> 3, rem = gridDim.x & 7, xcd = blockIdx.x & 7;
+  const int group = ROWS == 1 ? blockIdx.x : xcd * share + (xcd < rem ? xcd : rem) + (blockIdx.x >> 3);
+  const int row0 = group * ROWS, tid = threadIdx.x, H = p.heads, G = p.kv_heads;
   const int n[3] = {H * p.dim, G * p.dim, G * p.vdim}, quads[3] = {(n[0] + 3) >> 2, (n[1] + 3) >> 2, (n[2] + 3) >> 2}, total = quads[0] + quads[1] + quads[2];
   const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
   ChattsRow R[ROWS];
+  size_t page[ROWS];
   bool one = true;      // the rows are consecutive rows of one segment
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) {
     R[r] = row0 + r < p.n_rows ? p.rows[row0 + r] : ChattsRow{0, -1, 0, 0};
-    if (row0 + r < p.n_rows) one = one && R[r].pos >= 0 && R[r].first == R[0].first;
+    page[r] = R[r].pos >= 0 ? window_tile(p, R[r].slot, 0, R[r].pos) : 0;
+    one = one && R[r].pos >= 0 && R[r].first == R[0].first;
   }
   if (ROWS == 1 && R[0].pos < 0) return;
   auto place = [&](int u, int& block, int& c) __attribute__((always_inline)) {      // quad -> its block and first channel there
@@ -152,42 +233,58 @@ __global__ __launch_bounds__(NT) void window_prep_rows_kernel(ChattsWindowArgs p
   };
   f32x4 y[NV][ROWS];
 #pragma unroll
-  for (int i = 0; i < NV; ++i) {
-    const int u = i * NT + tid;
+  for (int i = 0; i < NV; ++i)
 #pragma unroll
     for (int r = 0; r < ROWS; ++r) y[i][r] = zero;
-    if (u >= total) continue;
-    int block, c;
-    const int col = place(u, block, c);
-    if (!p.taps) {
+  if (one && p.taps && p.taps <= kConvRegs && row0 - R[0].first >= p.taps - 1) {      // every input is a row of this step
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int u = i * NT + tid;
+      if (u >= total) continue;
+      int block, c;
+      const int col = place(u, block, c);
+      f32x4 w[kConvRegs], in[kConvRegs - 1 + ROWS];
+#pragma unroll
+      for (int j = 0; j < kConvRegs - 1 + ROWS; ++j)      // input j: row row0 + j - (kConvRegs - 1)
+        in[j] = j > kConvRegs - 1 - p.taps ? *reinterpret_cast<const f32x4*>(p.proj + (size_t)(row0 + j - (kConvRegs - 1)) * p.ld_proj + col) : zero;
+#pragma unroll
+      for (int g = 0; g < kConvRegs; ++g)      // [tokens back]
+        w[g] = g < p.taps ? *reinterpret_cast<const f32x4*>(p.conv_w + (size_t)(p.taps - 1 - g) * p.conv_ch + col) : zero;
 #pragma unroll
       for (int r = 0; r < ROWS; ++r)
-        if (R[r].pos >= 0) y[i][r] = *reinterpret_cast<const f32x4*>(p.proj + (size_t)(row0 + r) * p.ld_proj + col);
-      continue;
+#pragma unroll
+        for (int g = kConvRegs - 1; g >= 0; --g) y[i][r] += w[g] * in[r + kConvRegs - 1 - g];
     }
-    const float* cw = p.conv_w + col;
-    if (one && p.taps <= kConvRegs) {
-      f32x4 w[kConvRegs];      // [tokens back]
+  } else {
 #pragma unroll
-      for (int g = 0; g < kConvRegs; ++g) w[g] = g < p.taps ? *reinterpret_cast<const f32x4*>(cw + (size_t)(p.taps - 1 - g) * p.conv_ch) : zero;
+    for (int i = 0; i < NV; ++i) {
+      const int u = i * NT + tid;
+      if (u >= total) continue;
+      int block, c;
+      const int col = place(u, block, c);
 #pragma unroll
-      for (int j = 1 - kConvRegs; j < ROWS; ++j) {      // input j: row row0 + j
-        if (j <= -p.taps || row0 + j >= p.n_rows) continue;
-        const f32x4 v = input(0, row0, -j, col);
+      for (int r = 0; r < ROWS; ++r) {
+        if (R[r].pos < 0) continue;
+        const f32x4 now = input(r, row0 + r, 0, col);
+        if (!p.taps) {
+          y[i][r] = now;
+          continue;
+        }
+        const float* cw = p.conv_w + (size_t)(p.taps - 1) * p.conv_ch + col;      // (the newest token's)
+        for (int g0 = p.taps - 1; g0 >= 0; g0 -= kConvRegs) {      // the oldest first, kConvRegs requested at once
+          f32x4 w[kConvRegs], in[kConvRegs];
 #pragma unroll
-        for (int r = 0; r < ROWS; ++r)
-          if (r - j >= 0 && r - j < kConvRegs) y[i][r] += w[r - j] * v;
+          for (int j = 0; j < kConvRegs; ++j) {
+            const int g = g0 - j;
+            in[j] = g > 0 ? input(r, row0 + r, g, col) : now;
+            w[j] = g >= 0 ? *reinterpret_cast<const f32x4*>(cw - (size_t)(g >= 0 ? g : 0) * p.conv_ch) : zero;
+          }
+#pragma unroll
+          for (int j = 0; j < kConvRegs; ++j) y[i][r] += w[j] * in[j];
+        }
+        if (p.n_spans == 0)      // segments of one token: nobody else reads this entry of the ring
+          *reinterpret_cast<f32x4*>(p.ring + ((size_t)R[r].slot * p.taps + R[r].pos % p.taps) * p.conv_ch + col) = now;
       }
-    } else {
-#pragma unroll
-      for (int r = 0; r < ROWS; ++r)
-        if (R[r].pos >= 0)
-          for (int g = p.taps - 1; g >= 0; --g) y[i][r] += *reinterpret_cast<const f32x4*>(cw + (size_t)(p.taps - 1 - g) * p.conv_ch) * input(r, row0 + r, g, col);
-    }
-    if (p.n_spans == 0) {      // segments of one token: nobody else reads this entry of the ring
-#pragma unroll
-      for (int r = 0; r < ROWS; ++r)
-        if (R[r].pos >= 0) *reinterpret_cast<f32x4*>(p.ring + ((size_t)R[r].slot * p.taps + R[r].pos % p.taps) * p.conv_ch + col) = input(r, row0 + r, 0, col);
     }
   }
   float inv[2][ROWS];
@@ -201,7 +298,7 @@ __global__ __launch_bounds__(NT) void window_prep_rows_kernel(ChattsWindowArgs p
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
         const int u = i * NT + tid;
-        const float s = (y[i][r][0] * y[i][r][0] + y[i][r][1] * y[i][r][1]) + (y[i][r][2] * y[i][r][2] + y[i][r][3] * y[i][r][3]);
+        const float s = quad_squares(y[i][r]);
         if (u < quads[0]) ss[0] += s;
         else if (u < quads[0] + quads[1]) ss[1] += s;
       }
@@ -233,55 +330,52 @@ __global__ __launch_bounds__(NT) void window_prep_rows_kernel(ChattsWindowArgs p
     f32x4 w = {1.f, 1.f, 1.f, 1.f};
     if (nw) w = *reinterpret_cast<const f32x4*>(nw + c);
     const int d = block == 2 ? p.vdim : p.dim, dp = block == 2 ? p.vdim_p : p.dim_p, e0 = c / d, c0 = c - e0 * d;
+    CT* pages = reinterpret_cast<CT*>(block == 2 ? p.vcache : p.kcache);
+    f32x4 first[ROWS];
+    const bool mix = block == 2 && p.vfirst;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) first[r] = mix && !p.vfirst_write && R[r].pos >= 0 ? *reinterpret_cast<const f32x4*>(p.vfirst + (size_t)(row0 + r) * p.ld_vfirst + c) : zero;
 #pragma unroll
     for (int r = 0; r < ROWS; ++r) {
       if (R[r].pos < 0) continue;
       const int row = row0 + r;
-      f32x4 v;
-#pragma unroll
-      for (int k = 0; k < 4; ++k) v[k] = block == 2 ? y[i][r][k] : y[i][r][k] * inv[block & 1][r] * w[k];
-      if (block == 2 && p.vfirst) {
-        float* first = p.vfirst + (size_t)row * p.ld_vfirst + c;
-        if (p.vfirst_write) *reinterpret_cast<f32x4*>(first) = v;
-        else v = (1.f - p.vmix) * v + p.vmix * *reinterpret_cast<const f32x4*>(first);
+      f32x4 v = block == 2 ? y[i][r] : y[i][r] * inv[block & 1][r] * w;
+      if (mix) {
+        if (p.vfirst_write) *reinterpret_cast<f32x4*>(p.vfirst + (size_t)row * p.ld_vfirst + c) = v;
+        else v = (1.f - p.vmix) * v + p.vmix * first[r];
       }
-      const float out[4] = {v[0], v[1], v[2], v[3]};
-      CT* pages = reinterpret_cast<CT*>(block == 2 ? p.vcache : p.kcache);
       if (whole) {
         if (block == 0) {
+          const float out[4] = {v[0], v[1], v[2], v[3]};
           store_operand4(p.q, row, e0 * p.dim_p + c0, out);
         } else {
-          CT* dst = pages + window_tile(p, R[r].slot, e0, R[r].pos) * dp + c0;
-          if constexpr (sizeof(CT) == 4) *reinterpret_cast<f32x4*>(dst) = v;
-          else *reinterpret_cast<w16x4*>(dst) = (w16x4){(short)to_page<CT>(v[0]), (short)to_page<CT>(v[1]), (short)to_page<CT>(v[2]), (short)to_page<CT>(v[3])};
+          store_page4(pages + (page[r] + ((size_t)e0 << p.log_block)) * dp + c0, v);
         }
       } else {
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
           if (c + k >= n[block]) break;
           const int e = (c + k) / d, cc = c + k - e * d;
-          if (block == 0) store_operand(p.q, row, e * p.dim_p + cc, out[k]);
-          else pages[window_tile(p, R[r].slot, e, R[r].pos) * dp + cc] = to_page<CT>(out[k]);
+          if (block == 0) store_operand(p.q, row, e * p.dim_p + cc, v[k]);
+          else pages[(page[r] + ((size_t)e << p.log_block)) * dp + cc] = to_page<CT>(v[k]);
         }
       }
     }
   }
   // padding between heads: queries multiply it, so it must not hold another layer's numbers
-  const int pad = p.dim_p - p.dim;
-  for (int x = tid; x < ROWS * (H + G) * pad; x += NT) {
-    const int r = x / ((H + G) * pad), z = x - r * (H + G) * pad, e = z / pad, c = p.dim + z - e * pad;
-    if (row0 + r >= p.n_rows) break;
-    const ChattsRow Z = p.rows[row0 + r];
-    if (Z.pos < 0) continue;
-    if (e < H) store_operand(p.q, row0 + r, e * p.dim_p + c, 0.f);
-    else reinterpret_cast<CT*>(p.kcache)[window_tile(p, Z.slot, e - H, Z.pos) * p.dim_p + c] = 0;
-  }
-  const int vpad = p.vdim_p - p.vdim;
-  for (int x = tid; x < ROWS * G * vpad; x += NT) {
-    const int r = x / (G * vpad), z = x - r * G * vpad, e = z / vpad;
-    if (row0 + r >= p.n_rows) break;
-    const ChattsRow Z = p.rows[row0 + r];
-    if (Z.pos >= 0) reinterpret_cast<CT*>(p.vcache)[window_tile(p, Z.slot, e, Z.pos) * p.vdim_p + p.vdim + z - e * vpad] = 0;
+  const int pad = p.dim_p - p.dim, vpad = p.vdim_p - p.vdim;
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    if (R[r].pos < 0) continue;
+    for (int x = tid; x < (H + G) * pad; x += NT) {
+      const int e = x / pad, c = p.dim + x - e * pad;
+      if (e < H) store_operand(p.q, row0 + r, e * p.dim_p + c, 0.f);
+      else reinterpret_cast<CT*>(p.kcache)[(page[r] + ((size_t)(e - H) << p.log_block)) * p.dim_p + c] = 0;
+    }
+    for (int x = tid; x < G * vpad; x += NT) {
+      const int e = x / vpad;
+      reinterpret_cast<CT*>(p.vcache)[(page[r] + ((size_t)e << p.log_block)) * p.vdim_p + p.vdim + x - e * vpad] = 0;
+    }
   }
 }
 
@@ -778,9 +872,18 @@ static int check_window(const ChattsWindowArgs* a, const char* who) {
 static bool window_out_ok(const ChattsWindowArgs* a) { return (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim; }
 
 template <typename CT>
+static void launch_window_quads(const ChattsWindowArgs* a, int heads, int widest, hipStream_t s) {
+  const int lph = widest <= 64 ? 16 : (widest <= 128 ? 32 : 64), groups = (heads * lph + 255) / 256;      // workgroups that would take one group of heads per wave
+  const dim3 g(a->n_rows, a->n_rows <= 64 ? groups : (groups + 1) / 2), b(256);
+  if (lph == 16) hipLaunchKernelGGL((window_prep_quads_kernel<CT, 16>), g, b, 0, s, *a);
+  else if (lph == 32) hipLaunchKernelGGL((window_prep_quads_kernel<CT, 32>), g, b, 0, s, *a);
+  else hipLaunchKernelGGL((window_prep_quads_kernel<CT, 64>), g, b, 0, s, *a);
+}
+
+template <typename CT>
 static int launch_window_rows(const ChattsWindowArgs* a, hipStream_t s) {
   const int quads = (a->heads * a->dim + 3) / 4 + (a->kv_heads * a->dim + 3) / 4 + (a->kv_heads * a->vdim + 3) / 4;
-  if (a->n_rows > 64 && quads <= 8 * 256) hipLaunchKernelGGL((window_prep_rows_kernel<CT, 256, 8, 4>), dim3((a->n_rows + 3) / 4), dim3(256), 0, s, *a);
+  if (a->n_rows > 64 && quads <= 4 * 512) hipLaunchKernelGGL((window_prep_rows_kernel<CT, 512, 4, 4>), dim3((a->n_rows + 3) / 4), dim3(512), 0, s, *a);
   else if (quads <= 2 * 1024) hipLaunchKernelGGL((window_prep_rows_kernel<CT, 1024, 2, 1>), dim3(a->n_rows), dim3(1024), 0, s, *a);
   else hipLaunchKernelGGL((window_prep_rows_kernel<CT, 1024, 8, 1>), dim3(a->n_rows), dim3(1024), 0, s, *a);
   if (a->n_spans > 0 && a->taps > 1)
@@ -852,7 +955,14 @@ extern "C" int chatts_window_prep(const ChattsWindowArgs* a, chatts_stream_t str
   if (const int rc = check_window(a, "window_prep")) return rc;
   if (a->n_rows == 0) return CHATTS_OK;
   if (a->taps > 0 || a->norm_whole) return a->cache_f32 ? launch_window_rows<float>(a, as_stream(stream)) : launch_window_rows<uint16_t>(a, as_stream(stream));
-  int per_row = (a->heads + 2 * a->kv_heads + 3) / 4;
+  const int heads = a->heads + 2 * a->kv_heads, widest = a->dim > a->vdim ? a->dim : a->vdim;
+  if ((a->dim | a->vdim | a->off_q | a->off_k | a->off_v) % 4 == 0 && ((uintptr_t)a->q_norm | (uintptr_t)a->k_norm) % 16 == 0) {
+    if (a->cache_f32) launch_window_quads<float>(a, heads, widest, as_stream(stream));
+    else launch_window_quads<uint16_t>(a, heads, widest, as_stream(stream));
+    CHATTS_CHECK_LAUNCH("window_prep_quads");
+    return CHATTS_OK;
+  }
+  int per_row = (heads + 3) / 4;
   if (per_row > 8192 / a->n_rows) per_row = 8192 / a->n_rows > 1 ? 8192 / a->n_rows : 1;
   if (a->cache_f32) hipLaunchKernelGGL(window_prep_kernel<float>, dim3(a->n_rows, per_row), dim3(256), 0, as_stream(stream), *a);
   else hipLaunchKernelGGL(window_prep_kernel<uint16_t>, dim3(a->n_rows, per_row), dim3(256), 0, as_stream(stream), *a);
