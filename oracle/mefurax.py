@@ -179,3 +179,50 @@ def generate(cfg, sd, tokens, n, dtype=torch.float64):
     for _ in range(n):
         seq.append(int(forward(cfg, sd, seq, dtype)[-1].argmax()))
     return seq[len(tokens):]
+
+
+def random_model(cfg, seed=0):
+    """bf16-representable random weights -> name -> bfloat16 tensor.  Queries and keys share directions, so that single scores stand out; router logits
+    lie apart."""
+    gen = torch.Generator().manual_seed(seed)
+    W, V = cfg["width"], cfg["vocab"]
+
+    def lin(o, i, gain=1.0):
+        return torch.randn(o, i, generator=gen) * gain / math.sqrt(i)
+
+    def vec(n, mean, spread):
+        return mean + spread * torch.randn(n, generator=gen)
+
+    sd = {"embed": torch.randn(V, W, generator=gen), "final.norm": vec(W, 0, 0.2), "head": lin(V, W)}
+    for i, spec in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", spec["mixer"]
+        q, H, G, D, E = p + "mix.", m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        sd[p + "norm1"] = vec(W, 0, 0.2)
+        k = lin(G * D, W)
+        sd[q + "k"] = k
+        sd[q + "q"] = 0.6 * k.view(G, 1, D, W).expand(G, H // G, D, W).reshape(H * D, W) + lin(H * D, W, 0.8)
+        sd[q + "v"], sd[q + "o"] = lin(G * E, W, 1.5), lin(W, H * E, 2.0)
+        if m.get("v_mix"):
+            sd[q + "vmix"] = 0.2 + 0.6 * torch.rand((), generator=gen)
+        if spec["type"] == "attention":
+            for n, r in (("q", H * D), ("k", G * D), ("v", G * E)):
+                sd[f"{q}{n}.b"] = vec(r, 0, 0.5)
+                w = 0.4 * torch.randn(r, m["conv"], generator=gen)
+                w[:, -1] += 1.0
+                sd[f"{q}{n}.conv"] = w
+            sd[q + "q.norm"], sd[q + "k.norm"] = vec(H * D, 1.3, 0.3), vec(G * D, 1.3, 0.3)
+        else:
+            sd[q + "g"] = lin(H, W, 2.0)
+        mlp, q = spec.get("mlp"), p + "mlp."
+        if not mlp:
+            continue
+        sd[p + "norm2"] = vec(W, 0, 0.2)
+        if mlp.get("kind", "dense") == "dense":
+            sd[q + "gate"], sd[q + "up"], sd[q + "down"] = lin(mlp["ff"], W, 1.5), lin(mlp["ff"], W), lin(W, mlp["ff"])
+            continue
+        sd[q + "router"] = lin(mlp["router"]["experts"], W, 2.0)
+        for e in range(mlp["router"]["experts"]):
+            sd[f"{q}e{e}.up"], sd[f"{q}e{e}.down"] = lin(mlp["expert"]["ff"], W), lin(W, mlp["expert"]["ff"])
+        if mlp.get("shared"):
+            sd[q + "shared.up"], sd[q + "shared.down"] = lin(mlp["shared"]["ff"], W), lin(W, mlp["shared"]["ff"])
+    return {k: v.to(torch.bfloat16) for k, v in sd.items()}
