@@ -55,7 +55,7 @@ def in_window(i, j, size):
 
 
 def in_chunk(i, j, size):
-    """earlier positions of the same chunk (chunks counted from position 0)"""
+    """earlier positions of the same chunk; position 0 opens the first one"""
     return j <= i and (not size or i // size == j // size)
 
 
