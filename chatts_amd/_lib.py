@@ -29,7 +29,7 @@ class TsWeights(C.Structure):
                 ("b", c_void_p * 8)]
 
 
-ABI_VERSION = 12           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
+ABI_VERSION = 13           # CHATTS_ABI_VERSION of include/chatts_amd.h this binding was written against (checked by load())
 W8_FP8, W8_INT8 = 0, 1     # ChattsLinearArgs.w8_format
 
 
@@ -160,7 +160,7 @@ class LatentExpandArgs(C.Structure):
 class EmbedPairArgs(C.Structure):
     _fields_ = [("tokens", c_void_p), ("rows", c_void_p), ("t", c_int), ("single", c_int), ("width_p", c_int), ("vocab", c_int), ("embed", c_void_p),
                 ("scale", c_float), ("bigram", c_void_p), ("buckets", c_int64), ("mul_prev", c_int64), ("mul_cur", c_int64), ("prev", c_void_p),
-                ("x", c_void_p), ("x0", c_void_p)]
+                ("x", c_void_p), ("x0", c_void_p), ("width", c_int), ("pos_fine", c_void_p), ("pos_coarse", c_void_p)]
 
 
 class PairNormArgs(C.Structure):
@@ -184,6 +184,28 @@ class PostNormArgs(C.Structure):
                 ("place", c_void_p), ("weight", c_void_p), ("top", c_int), ("w", c_void_p), ("out", Operand)]
 
 
+class DepthNormArgs(C.Structure):
+    """ChattsDepthNormArgs: a sublayer's share, averages over depth, the next norm (csrc/depth.hip)"""
+    _fields_ = [("x", c_void_p), ("t", c_int), ("width", c_int), ("ldx", c_int), ("mult", c_float), ("eps", c_float), ("y", c_void_p), ("ey", c_void_p),
+                ("place", c_void_p), ("weight", c_void_p), ("top", c_int), ("depth", c_void_p), ("streams", c_void_p), ("stream_stride", c_int64),
+                ("n_streams", c_int), ("keep", c_int), ("w", c_void_p), ("out", Operand)]
+
+
+class GruArgs(C.Structure):
+    """ChattsGruArgs: minimal gated recurrence (csrc/gru.hip)"""
+    _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_z", "off_x", "off_g", "width")] + [("out_scale", c_float), ("state", c_void_p),
+                 ("rows", c_void_p), ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int), ("out", Operand)])
+
+
+class SelectArgs(C.Structure):
+    """ChattsSelectArgs: selective scan (csrc/select.hip)"""
+    _fields_ = ([("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_x", "off_z", "inner", "state", "taps", "conv_ch")] +
+                [("conv_w", c_void_p), ("conv_b", c_void_p), ("low", c_void_p)] + [(n, c_int) for n in ("ld_low", "off_dt", "off_b", "off_c", "rank")] +
+                [("w_dt", c_void_p), ("dt_bias", c_void_p), ("a", c_void_p), ("d", c_void_p), ("out_scale", c_float), ("s", c_void_p), ("ring", c_void_p),
+                 ("rows", c_void_p), ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int), ("u", Operand), ("delta", c_void_p), ("ld_delta", c_int),
+                 ("out", Operand)])
+
+
 class RecurArgs(C.Structure):
     """ChattsRecurArgs: gated linear recurrences (csrc/recur.hip)"""
     _fields_ = ([("kind", c_int), ("proj", c_void_p)] + [(n, c_int) for n in ("ld_proj", "off_q", "off_k", "off_v", "off_gate", "off_a", "off_i", "off_f", "heads",
@@ -202,7 +224,7 @@ class WindowArgs(C.Structure):
                 [("cos_tab", c_void_p), ("sin_tab", c_void_p), ("taps", c_int), ("conv_ch", c_int), ("conv_w", c_void_p), ("ring", c_void_p), ("vmix", c_float),
                  ("vfirst", c_void_p), ("ld_vfirst", c_int), ("vfirst_write", c_int), ("kcache", c_void_p), ("vcache", c_void_p), ("cache_f32", c_int), ("table", c_void_p), ("table_stride", c_int), ("log_block", c_int),
                  ("rows", c_void_p), ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int), ("longest", c_int), ("q", Operand), ("n_splits", c_int),
-                 ("partial", c_void_p), ("out", Operand)])
+                 ("partial", c_void_p), ("out", Operand), ("log_r1", c_void_p), ("log_r2", c_void_p), ("out_scale", c_float)])
 
 
 class MoeArgs(C.Structure):
@@ -210,13 +232,13 @@ class MoeArgs(C.Structure):
     _fields_ = ([(n, c_int) for n in ("experts", "identity", "top", "groups", "keep", "choose", "act_kind", "width_p", "ff_p")] +
                 [("gate_up", c_void_p), ("down", c_void_p), ("gate_up_t", c_void_p), ("down_t", c_void_p), ("correction", c_void_p), ("logits", c_void_p), ("ld_logits", c_int), ("h", Operand), ("rows", c_void_p),
                  ("n_rows", c_int), ("exact", c_int)] + [(n, c_void_p) for n in ("ids", "place", "order", "offsets", "tiles", "weight", "kept")] +
-                [("act", Operand), ("y", c_void_p)])
+                [("act", Operand), ("y", c_void_p), ("weight_scale", c_float), ("glu_limit", c_float), ("glu_alpha", c_float)])
 
 
-MIX_LATENT, MIX_DELTA, MIX_RECUR, MIX_WINDOW = 1, 2, 3, 4
+MIX_LATENT, MIX_DELTA, MIX_RECUR, MIX_WINDOW, MIX_GRU, MIX_SELECT = 1, 2, 3, 4, 5, 6
 FF_NONE, FF_RELU2, FF_CLAMPGLU, FF_MOE, FF_GEGLU = 0, 1, 2, 3, 4
-CHOOSE_SOFTMAX, CHOOSE_LOGITS = 0, 1
-EXPERT_SWIGLU, EXPERT_RELU2 = 0, 1
+CHOOSE_SOFTMAX, CHOOSE_LOGITS, CHOOSE_SCORES = 0, 1, 2
+EXPERT_SWIGLU, EXPERT_RELU2, EXPERT_CLAMPGLU = 0, 1, 2
 EXPAND_PAD = 128           # CHATTS_LATENT_EXPAND_PAD
 
 
@@ -227,18 +249,20 @@ class MixLayer(C.Structure):
                 [(n, c_int) for n in ("dim_p", "vdim_p", "out_head")] + [("latent", LatentArgs), ("delta", DeltaArgs), ("parallel", c_int), ("ff_kind", c_int),
                  ("glu_limit", c_float), ("glu_alpha", c_float), ("n_mix", c_int), ("mix_row", c_int * 8), ("mix_t", c_void_p * 8), ("mu", c_void_p), ("w2", c_void_p), ("w2_n", c_int),
                  ("recur", RecurArgs), ("window", WindowArgs), ("router", c_void_p), ("router_t", c_void_p), ("router_n", c_int), ("moe", MoeArgs),
-                 ("post", c_int), ("in_bias", c_void_p)])
+                 ("post", c_int), ("in_bias", c_void_p), ("pre", c_int), ("beside", c_int), ("beside_col", c_int), ("depth", c_void_p), ("gru", GruArgs),
+                 ("select", SelectArgs), ("sel_low", c_void_p), ("sel_low_t", c_void_p), ("sel_dt", c_void_p), ("sel_k", c_int), ("sel_dt_n", c_int)])
 
 
 class MixRun(C.Structure):
     _fields_ = [("layer", c_int), ("add", c_void_p), ("cache", c_void_p), ("state", c_void_p), ("ring", c_void_p), ("n_state", c_void_p), ("m_state", c_void_p),
-                ("vcache", c_void_p), ("join", c_void_p), ("join_t", c_void_p)]
+                ("vcache", c_void_p), ("join", c_void_p), ("join_t", c_void_p), ("gru_state", c_void_p), ("sel_state", c_void_p), ("sel_ring", c_void_p)]
 
 
 class MixConfig(C.Structure):
     _fields_ = ([(n, c_int) for n in ("width", "width_p", "n_layers", "n_runs", "exact", "t_max", "max_slots", "max_ctx", "expand_rows")] +
                 [("vocab", c_int64), ("vocab_p", c_int64), ("eps", c_float), ("block_size", c_int), ("table_stride", c_int), ("norm_groups", c_int),
-                 ("embed_scale", c_float), ("bigram_buckets", c_int64), ("bigram_prev", c_int64), ("bigram_cur", c_int64), ("alpha", c_float)])
+                 ("embed_scale", c_float), ("bigram_buckets", c_int64), ("bigram_prev", c_int64), ("bigram_cur", c_int64), ("alpha", c_float),
+                 ("mult", c_float), ("logit_cap", c_float)])
 
 
 class MixBuffers(C.Structure):
@@ -249,7 +273,8 @@ class MixBuffers(C.Structure):
                 [("mix_stride", c_int64)] +
                 [(n, c_void_p) for n in ("n_f32", "n_hi", "n_lo", "gates", "den", "moe_ids", "moe_place", "moe_order", "moe_offsets", "moe_tiles", "moe_weight",
                                          "moe_kept", "moe_logits", "moe_y", "act_f32", "act_hi", "act_lo", "rows", "spans", "table", "logits", "workspace")] +
-                [("workspace_bytes", c_size_t), ("vfirst", c_void_p), ("ld_vfirst", c_int)])
+                [("workspace_bytes", c_size_t), ("vfirst", c_void_p), ("ld_vfirst", c_int), ("pos_fine", c_void_p), ("pos_coarse", c_void_p), ("streams", c_void_p),
+                 ("stream_stride", c_int64)] + [(n, c_void_p) for n in ("sel_u", "sel_low", "sel_delta", "sel_u_hi", "sel_u_lo", "sel_dt_hi", "sel_dt_lo")])
 
 
 # name -> (restype, argtypes); this table IS the list of symbols include/chatts_amd.h declares
@@ -346,6 +371,13 @@ SIGNATURES = {
     "chatts_embed_pair": (c_int, [C.POINTER(EmbedPairArgs), c_void_p]),
     "chatts_pair_norm": (c_int, [C.POINTER(PairNormArgs), c_void_p]),
     "chatts_post_norm": (c_int, [C.POINTER(PostNormArgs), c_void_p]),
+    "chatts_depth_norm": (c_int, [C.POINTER(DepthNormArgs), c_void_p]),
+    "chatts_soft_cap": (c_int, [c_void_p, c_int64, c_float, c_void_p]),
+    "chatts_gru_decode": (c_int, [C.POINTER(GruArgs), c_void_p]),
+    "chatts_gru_scan": (c_int, [C.POINTER(GruArgs), c_void_p]),
+    "chatts_select_conv": (c_int, [C.POINTER(SelectArgs), c_void_p]),
+    "chatts_select_decode": (c_int, [C.POINTER(SelectArgs), c_void_p]),
+    "chatts_select_scan": (c_int, [C.POINTER(SelectArgs), c_void_p]),
     "chatts_token_shift": (c_int, [C.POINTER(TokenShiftArgs), c_void_p]),
     "chatts_recur_decode": (c_int, [C.POINTER(RecurArgs), c_void_p]),
     "chatts_recur_tanh": (c_int, [C.POINTER(RecurArgs), C.POINTER(Operand), c_void_p]),

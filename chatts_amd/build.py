@@ -13,7 +13,7 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIBDIR = os.path.join(HERE, "lib")
 LIB = os.path.join(LIBDIR, "libchatts_amd.so")
-SOURCES = ["api.hip", "ts_frontend.hip", "gemv.hip", "gemm.hip", "gemm_ring.hip", "gemm_f16q.hip", "gemm_fp8.hip", "gemm_f32.hip", "elementwise.hip", "sampler.hip", "attention.hip", "tp.hip", "decoder.hip", "delta.hip", "latent.hip", "pair.hip", "postnorm.hip", "recur.hip", "window.hip", "moe.hip", "mixdec.hip"]
+SOURCES = ["api.hip", "ts_frontend.hip", "gemv.hip", "gemm.hip", "gemm_ring.hip", "gemm_f16q.hip", "gemm_fp8.hip", "gemm_f32.hip", "elementwise.hip", "sampler.hip", "attention.hip", "tp.hip", "decoder.hip", "delta.hip", "depth.hip", "gru.hip", "latent.hip", "pair.hip", "postnorm.hip", "recur.hip", "select.hip", "window.hip", "moe.hip", "mixdec.hip"]
 # no packed float32 instructions (v_pk_add / mul / fma_f32): the compiler forms them from ordinary float code and some of their forms
 # have given wrong results on this hardware
 NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]

@@ -1,5 +1,5 @@
-// mixdec.hip - host-side composition of decoders with mixed layers (latent attention, gated delta rule, gated linear recurrences, windowed attention;
-// feed-forwards or experts; looped layer ranges).  Like decoder.hip: nothing here allocates or synchronises, a decode step is capturable.
+// mixdec.hip - host-side composition of decoders with mixed layers (latent attention, gated delta rule, gated linear recurrences, windowed attention, minimal
+// gated recurrence, selective scan; feed-forwards or experts; looped layer ranges).  Like decoder.hip: nothing here allocates or synchronises, a decode step is capturable.
 //
 // Sequential layer (norms before and after each sublayer):
 //   norm1 (in the previous residual_norm launch) -> stacked input projection -> mixer kernels -> out projection
@@ -10,6 +10,10 @@
 // Layer with its norms after the sums (sublayers read x itself):
 //   input projections -> mixer kernels -> out projection -> post_norm (x = norm1(alpha x + y), as the next operand too)
 //   -> gate_up (gated unit in the epilogue) -> down;  or router -> experts, beside a shared one: up -> down -> post_norm (x = norm2(alpha x + y + experts))
+// Layer with norms before its sublayers only (a factor of what is added; the streams of all layers averaged after each):
+//   input projections -> mixer kernels, two mixers side by side writing neighbouring columns of one operand -> out projection
+//   -> depth_norm (x += mult y; norm2(x)) -> router -> experts, beside a shared one: gate_up -> down
+//   -> depth_norm (x += mult (y + experts); average over depth; the next layer's norm1)
 // Operands between the launches travel in the format the next projection's kernel takes for this row count: bf16 hi / lo planes
 // (2 .. 16 rows: weight-streaming kernel; >= 96 rows: the prefill kernel) or float32.
 #include <new>
@@ -50,6 +54,11 @@ static int mix_equal_blocks(const ChattsMixLayer& l, int i) {      // how many o
   return n;
 }
 
+static bool mix_pairs(const ChattsMixLayer& l) {      // `up` holds gate and up rows
+  return l.ff_kind == CHATTS_FF_CLAMPGLU || l.ff_kind == CHATTS_FF_GEGLU || (l.ff_kind == CHATTS_FF_MOE && l.pre);
+}
+static bool mix_has(const ChattsMixLayer& l, int kind) { return l.kind == kind || l.beside == kind; }
+
 extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const ChattsMixLayer* layers) {
   if (!c || !layers) return 0;
   std::vector<std::pair<int, int>> shapes;
@@ -63,8 +72,9 @@ extern "C" size_t chatts_mixdec_workspace(const ChattsMixConfig* c, const Chatts
     if (!l.n_mix) add(l.in_n, c->width_p);
     add(c->width_p, l.out_k);
     if (l.w2) add(l.w2_n, l.recur.rank);
-    if (l.up) { add(l.ff_kind == CHATTS_FF_CLAMPGLU || l.ff_kind == CHATTS_FF_GEGLU ? 2 * l.ff : l.ff, c->width_p); add(c->width_p, l.ff); }
+    if (l.up) { add(mix_pairs(l) ? 2 * l.ff : l.ff, c->width_p); add(c->width_p, l.ff); }
     if (l.router) add(l.router_n, c->width_p);
+    if (l.sel_low) { add(l.select.ld_low, l.sel_k); add(l.sel_dt_n, l.select.rank); }
   }
   add(c->width_p, 2 * c->width_p);
   add((int)c->vocab_p, c->width_p);
@@ -106,14 +116,29 @@ extern "C" ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, cons
   if (kv_log_block(c->block_size) < 0) { set_error("mixdec_create: pages of %d tokens (power of two, 64 .. 32768)", c->block_size); return nullptr; }
   for (int i = 0; i < c->n_runs; ++i)
     if (runs[i].layer < 0 || runs[i].layer >= c->n_layers) { set_error("mixdec_create: run %d names layer %d", i, runs[i].layer); return nullptr; }
+  for (int i = 0; i < c->n_runs; ++i)
+    if (layers[runs[i].layer].depth && b->stream_stride < (int64_t)c->t_max * c->width_p) { set_error("mixdec_create: streams of %lld values", (long long)b->stream_stride); return nullptr; }
   for (int i = 0; i < c->n_layers; ++i) {
     const ChattsMixLayer& l = layers[i];
     const bool pair = l.kind == CHATTS_MIX_RECUR || l.kind == CHATTS_MIX_WINDOW;
-    if ((l.kind != CHATTS_MIX_LATENT && l.kind != CHATTS_MIX_DELTA && !pair) || !l.in || !l.out || !l.norm1 || (l.up && !(l.down && l.norm2)) ||
+    if (l.kind < CHATTS_MIX_LATENT || l.kind > CHATTS_MIX_SELECT || !l.in || !l.out || !l.norm1 || (l.up && !(l.down && l.norm2)) ||
         (l.ff_kind == CHATTS_FF_MOE && !(l.router && l.norm2 && l.moe.gate_up && l.moe.down)) || l.n_mix < 0 || l.n_mix > 7 || (l.n_mix && !l.mu)) {
       set_error("mixdec_create: layer %d is incomplete", i);
       return nullptr;
     }
+    if (l.pre || layers[0].pre) {
+      auto fits = [&](int kind) { return kind == CHATTS_MIX_WINDOW || kind == CHATTS_MIX_GRU || kind == CHATTS_MIX_SELECT; };
+      if (!l.pre || !layers[0].pre || l.parallel || l.post || !fits(l.kind) || (l.beside && (!fits(l.beside) || l.beside == l.kind || l.beside_col < 0 || l.beside_col >= l.out_k)) ||
+          (l.ff_kind != CHATTS_FF_NONE && l.ff_kind != CHATTS_FF_CLAMPGLU && l.ff_kind != CHATTS_FF_MOE) || (l.ff_kind != CHATTS_FF_NONE && !l.norm2) ||
+          (l.ff_kind == CHATTS_FF_CLAMPGLU && !l.up) || (l.depth && !b->streams) || (mix_has(l, CHATTS_MIX_WINDOW) && l.window.ld_vfirst && !b->vfirst) ||
+          (mix_has(l, CHATTS_MIX_SELECT) && !(l.sel_low && l.sel_dt && b->sel_u && b->sel_low && b->sel_delta && (c->exact || (b->sel_u_hi && b->sel_dt_hi))))) {
+        set_error("mixdec_create: layer %d: a layer with norms before its sublayers has attention, minimal recurrence or selective scan (one or two of them) and a clamped "
+                  "gated unit, experts or nothing", i);
+        return nullptr;
+      }
+      continue;
+    }
+    if (l.kind > CHATTS_MIX_WINDOW || l.beside) { set_error("mixdec_create: layer %d: this mixer needs norms before its sublayers only", i); return nullptr; }
     if (l.post || layers[0].post) {
       if (!l.post || !layers[0].post || l.parallel || l.kind != CHATTS_MIX_WINDOW || (l.ff_kind != CHATTS_FF_NONE && !l.norm2) ||
           (l.ff_kind == CHATTS_FF_GEGLU ? !l.up : (l.ff_kind != CHATTS_FF_NONE && l.ff_kind != CHATTS_FF_MOE)) || (l.window.vfirst_write && !b->vfirst)) {
@@ -526,6 +551,112 @@ static int mix_post_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, c
   return CHATTS_OK;
 }
 
+// ---- norms before the sublayers only ----
+static int mix_gru(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, int n_spans, bool single, const ChattsOperand& out, chatts_stream_t s) {
+  StageRange stage("chatts.mix.gru");
+  ChattsGruArgs a = l.gru;
+  a.proj = d->b.proj; a.ld_proj = l.in_n;
+  a.state = run.gru_state;
+  a.rows = d->b.rows; a.n_rows = t; a.spans = d->b.spans; a.n_spans = n_spans;
+  a.out = out;
+  return single ? chatts_gru_decode(&a, s) : chatts_gru_scan(&a, s);
+}
+
+static int mix_select(const ChattsMixDecoder* d, const ChattsMixLayer& l, const ChattsMixRun& run, int t, int n_spans, bool single, const ChattsOperand& out, chatts_stream_t s) {
+  StageRange stage("chatts.mix.select");
+  const ChattsMixBuffers& b = d->b;
+  ChattsSelectArgs a = l.select;
+  a.proj = b.proj; a.ld_proj = l.in_n;
+  a.s = run.sel_state; a.ring = run.sel_ring;
+  a.rows = b.rows; a.n_rows = t; a.spans = b.spans; a.n_spans = single ? 0 : n_spans;
+  a.u.f32 = b.sel_u; a.u.ld = l.sel_k;
+  ChattsOperand in = f32_out(b.sel_u, l.sel_k);
+  if (mix_planes(d->c, t, l.sel_k)) {
+    a.u.hi = b.sel_u_hi; a.u.lo = b.sel_u_lo;
+    in.f32 = nullptr; in.hi = b.sel_u_hi; in.lo = b.sel_u_lo;
+  }
+  a.low = b.sel_low; a.out = out;
+  int rc;
+  if ((rc = chatts_select_conv(&a, s)) != 0) return rc;
+  if ((rc = mix_linear(d, in, l.sel_low, l.sel_low_t, t, a.ld_low, l.sel_k, CHATTS_EPI_NONE, f32_out(b.sel_low, a.ld_low), s)) != 0) return rc;
+  if (single) return chatts_select_decode(&a, s);
+  ChattsOperand dt = f32_out(b.sel_low + a.off_dt, a.ld_low);
+  if (mix_planes(d->c, t, a.rank)) {
+    if ((rc = chatts_split_bf16x2(dt.f32, t, a.rank, a.ld_low, b.sel_dt_hi, b.sel_dt_lo, a.rank, s)) != 0) return rc;
+    dt.f32 = nullptr; dt.hi = b.sel_dt_hi; dt.lo = b.sel_dt_lo; dt.ld = a.rank;
+  }
+  if ((rc = mix_linear(d, dt, l.sel_dt, nullptr, t, l.sel_dt_n, a.rank, CHATTS_EPI_NONE, f32_out(b.sel_delta, l.sel_dt_n), s)) != 0) return rc;
+  a.delta = b.sel_delta; a.ld_delta = l.sel_dt_n;
+  return chatts_select_scan(&a, s);
+}
+
+static int mix_one(const ChattsMixDecoder* d, const ChattsMixLayer& l, int kind, const ChattsMixRun& run, int t, const ChattsSpan* spans, int n_spans, bool single,
+                   const ChattsOperand& out, chatts_stream_t s) {
+  if (kind == CHATTS_MIX_WINDOW) return mix_window(d, l, run, t, spans, n_spans, single, out, s);
+  return kind == CHATTS_MIX_GRU ? mix_gru(d, l, run, t, n_spans, single, out, s) : mix_select(d, l, run, t, n_spans, single, out, s);
+}
+
+// x += mult (y + what the experts of `moe` owe it), averaged over depth after the run number `stream` of a layer with such weights; then the next norm
+static int mix_depth_norm(const ChattsMixDecoder* d, int t, const float* y, const ChattsMixLayer* moe, const float* depth, int stream, const float* w, const ChattsOperand& out,
+                          chatts_stream_t s) {
+  ChattsDepthNormArgs a{};
+  a.x = d->b.x; a.t = t; a.width = d->c.width; a.ldx = d->c.width_p; a.mult = d->c.mult; a.eps = d->c.eps; a.y = y;
+  if (moe) { a.ey = d->b.moe_y; a.place = d->b.moe_place; a.weight = d->b.moe_weight; a.top = moe->moe.top; }
+  a.depth = depth; a.streams = d->b.streams; a.stream_stride = d->b.stream_stride; a.n_streams = stream + 1; a.keep = depth && stream + 1 < d->c.n_runs;
+  a.w = w; a.out = out;
+  return chatts_depth_norm(&a, s);
+}
+
+static int mix_pre_forward(ChattsMixDecoder* d, const int64_t* tokens, int t, const ChattsSpan* spans, int n_spans, bool single, chatts_stream_t s) {
+  const ChattsMixConfig& c = d->c;
+  const int wp = c.width_p;
+  const ChattsOperand none{}, A = operand(d, false, t, wp), Y = f32_out(d->b.y, wp);
+  int rc;
+  {
+    ChattsEmbedPairArgs e{};
+    e.tokens = tokens; e.rows = d->b.rows; e.t = t; e.single = single; e.width_p = wp; e.vocab = (int)c.vocab; e.embed = d->b.embed; e.scale = c.embed_scale;
+    e.x = d->b.x; e.x0 = d->b.streams; e.width = c.width; e.pos_fine = d->b.pos_fine; e.pos_coarse = d->b.pos_coarse;
+    if ((rc = chatts_embed_pair(&e, s)) != 0) return rc;
+  }
+  if ((rc = mix_depth_norm(d, t, nullptr, nullptr, nullptr, 0, d->layers[d->runs[0].layer].norm1, A, s)) != 0) return rc;
+  for (int r = 0; r < c.n_runs; ++r) {
+    const ChattsMixRun& run = d->runs[r];
+    const ChattsMixLayer& l = d->layers[run.layer];
+    const float* next = r + 1 < c.n_runs ? d->layers[d->runs[r + 1].layer].norm1 : nullptr;
+    if ((rc = mix_linear(d, A, l.in, l.in_t, t, l.in_n, wp, CHATTS_EPI_NONE, f32_out(d->b.proj, l.in_n), s, 0.f, 0.f, l.in_bias)) != 0) return rc;
+    const ChattsOperand B = operand(d, true, t, l.out_k);
+    if ((rc = mix_one(d, l, l.kind, run, t, spans, n_spans, single, B, s)) != 0) return rc;
+    if (l.beside) {
+      ChattsOperand C = B;
+      if (C.f32) C.f32 += l.beside_col;
+      else { C.hi += l.beside_col; C.lo += l.beside_col; }
+      if ((rc = mix_one(d, l, l.beside, run, t, spans, n_spans, single, C, s)) != 0) return rc;
+    }
+    if ((rc = mix_linear(d, B, l.out, l.out_t, t, wp, l.out_k, CHATTS_EPI_NONE, Y, s)) != 0) return rc;
+    const bool moe = l.ff_kind == CHATTS_FF_MOE;
+    if (l.ff_kind == CHATTS_FF_NONE) {
+      if ((rc = mix_depth_norm(d, t, d->b.y, nullptr, l.depth, r, next, next ? A : none, s)) != 0) return rc;
+      continue;
+    }
+    const ChattsOperand N = second_norm(d, l, t);
+    if ((rc = mix_depth_norm(d, t, d->b.y, nullptr, nullptr, 0, l.norm2, N, s)) != 0) return rc;
+    if (moe) {
+      StageRange stage("chatts.mix.experts");
+      if ((rc = mix_linear(d, linear_form(N), l.router, l.router_t, t, l.router_n, wp, CHATTS_EPI_NONE, f32_out(d->b.moe_logits, l.router_n), s)) != 0) return rc;
+      const ChattsMoeArgs m = mix_moe_args(d, l, t, N);
+      if ((rc = chatts_moe_route(&m, s)) != 0) return rc;
+      if ((rc = chatts_moe_experts(&m, s)) != 0) return rc;
+    }
+    if (l.up) {
+      const ChattsOperand F = operand(d, true, t, l.ff);
+      if ((rc = mix_linear(d, linear_form(N), l.up, l.up_t, t, 2 * l.ff, wp, CHATTS_EPI_CLAMPGLU, F, s, l.glu_limit, l.glu_alpha)) != 0) return rc;
+      if ((rc = mix_linear(d, F, l.down, l.down_t, t, wp, l.ff, CHATTS_EPI_NONE, Y, s)) != 0) return rc;
+    }
+    if ((rc = mix_depth_norm(d, t, l.up ? d->b.y : nullptr, moe ? &l : nullptr, l.depth, r, next, next ? A : none, s)) != 0) return rc;
+  }
+  return CHATTS_OK;
+}
+
 static int mix_norm(const ChattsMixDecoder* d, int t, const float* y, const float* post, const float* add, const float* pre, const ChattsOperand& out,
                     chatts_stream_t s) {
   ChattsResidualNormArgs a{};
@@ -547,6 +678,7 @@ extern "C" int chatts_mixdec_forward(ChattsMixDecoder* d, const int64_t* tokens,
     CHATTS_REQUIRE(rows == t, CHATTS_E_SHAPE, "mixdec_forward: segments hold %d of %d rows", rows, t);
   }
   StageRange stage(single ? "chatts.mix.decode" : "chatts.mix.prefill");
+  if (d->layers[0].pre) return mix_pre_forward(d, tokens, t, spans, n_spans, single != 0, s);
   if (d->layers[0].post) return mix_post_forward(d, tokens, t, spans, n_spans, single != 0, s);
   if (d->layers[0].parallel) return mix_parallel_forward(d, tokens, t, spans, n_spans, single != 0, s);
   int rc;
@@ -603,7 +735,8 @@ extern "C" int chatts_mixdec_logits(ChattsMixDecoder* d, const int32_t* index, i
     rc = chatts_residual_norm(&a, s);
   }
   if (rc) return rc;
-  return mix_linear(d, A, d->b.head, d->b.head_t, n, (int)c.vocab_p, c.width_p, CHATTS_EPI_NONE, f32_out(logits, (int)c.vocab_p), s);
+  if ((rc = mix_linear(d, A, d->b.head, d->b.head_t, n, (int)c.vocab_p, c.width_p, CHATTS_EPI_NONE, f32_out(logits, (int)c.vocab_p), s)) != 0) return rc;
+  return c.logit_cap > 0.f ? chatts_soft_cap(logits, n * c.vocab_p, c.logit_cap, s) : CHATTS_OK;
 }
 
 extern "C" int chatts_mixdec_decode(ChattsMixDecoder* d, int batch, const int64_t* token, const int32_t* pos, float* logits, chatts_stream_t s) {

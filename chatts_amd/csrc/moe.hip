@@ -1,5 +1,5 @@
-// moe.hip - mixture of experts: choice by softmax values or logits, with a correction of the choice and choice groups; experts
-// W_down (silu(W_gate h) * W_up h) or W_down max(W_up h, 0)^2, identity outputs.
+// moe.hip - mixture of experts: choice by softmax values or logits, with a correction of the choice and choice groups; weights over the chosen ones, or the
+// softmax values as they are times a factor; experts W_down (silu(W_gate h) * W_up h), the clamped gated unit or W_down max(W_up h, 0)^2, identity outputs.
 //   moe_route_kernel      a wave per token: scores, the best groups, the best `top` outputs, their weights
 //   moe_list_kernel       a workgroup per expert: its (token, choice) pairs as a list, in order; tiles of the lists for the tiled products
 //   moe_route_small_kernel  both in one workgroup, for up to 16 rows; the tiles are then the experts in use
@@ -97,7 +97,7 @@ __device__ __forceinline__ void moe_route_row(const ChattsMoeArgs& p, int row, i
     total = wave_sum(mine);
     kept = wave_sum(own >= p.experts ? mine : 0.f);
   }
-  const float inv = 1.0f / (total + 1e-20f);
+  const float inv = p.choose == CHATTS_CHOOSE_SCORES ? p.weight_scale : 1.0f / (total + 1e-20f);
   if (lane < p.top) {
     p.ids[(size_t)row * p.top + lane] = parked ? -1 : id;
     p.weight[(size_t)row * p.top + lane] = mine * inv;
@@ -228,8 +228,13 @@ __global__ __launch_bounds__(1024) void moe_route_small_kernel(ChattsMoeArgs p, 
 
 __device__ __forceinline__ float moe_glu(float g, float u) { return g * sigmoid_f(g) * u; }
 
-// the products of an expert: its input projection (kGated: gate and up rows interleaved in blocks of 16, kRelu2: up rows alone), the output projection
-enum { kDown = 0, kGated, kRelu2 };
+// the products of an expert: its input projection (kGated, kClamped: gate and up rows interleaved in blocks of 16, kRelu2: up rows alone), the output projection
+enum { kDown = 0, kGated, kRelu2, kClamped };
+__host__ __device__ constexpr bool moe_pairs(int step) { return step == kGated || step == kClamped; }
+template <int STEP>
+__device__ __forceinline__ float moe_unit(const ChattsMoeArgs& p, float g, float u) {
+  return STEP == kClamped ? clamp_glu(g, u, p.glu_limit, p.glu_alpha) : moe_glu(g, u);
+}
 __device__ __host__ __forceinline__ int moe_in_rows(const ChattsMoeArgs& p) { return p.act_kind == CHATTS_EXPERT_RELU2 ? p.ff_p : 2 * p.ff_p; }
 __device__ __forceinline__ void moe_relu2_4(const ChattsOperand& o, size_t row, int col, const f32x4& s) {
   float v[4];
@@ -239,12 +244,12 @@ __device__ __forceinline__ void moe_relu2_4(const ChattsOperand& o, size_t row, 
 }
 
 // ---- up to 16 rows: grid (blocks of 16 RF weight rows, tiles), NW waves split K; D = W . A^T: a lane holds 4 consecutive outputs of one token.
-// kGated (RF = 2): the two 16-row halves of a block are gate and up rows of the same outputs ----
+// pairs (RF = 2): the two 16-row halves of a block are gate and up rows of the same outputs ----
 // TILED: weights from the chatts_tile_bf16 copy: a fragment's 64 pieces are 1 KB of consecutive memory
 template <int STEP, bool TILED, int NW, int RF>
 __global__ __launch_bounds__(64 * NW) void moe_stream_kernel(ChattsMoeArgs p) {
   __shared__ f32x4 red[NW][RF][64];
-  static_assert(STEP != kGated || RF == 2, "a pair of fragments");
+  static_assert(!moe_pairs(STEP) || RF == 2, "a pair of fragments");
   constexpr bool IN = STEP != kDown;
   const int32_t* tile = p.tiles + (size_t)blockIdx.y * 4;
   const int e = tile[0];
@@ -292,22 +297,22 @@ __global__ __launch_bounds__(64 * NW) void moe_stream_kernel(ChattsMoeArgs p) {
 #pragma unroll
   for (int f = 0; f < RF; ++f) red[wave][f][lane] = acc[f];
   __syncthreads();
-  if (wave >= (STEP == kGated ? 1 : RF)) return;
-  f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};      // (kGated: gate and up; otherwise s[0] = this wave's fragment)
+  if (wave >= (moe_pairs(STEP) ? 1 : RF)) return;
+  f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};      // (a pair: gate and up; otherwise s[0] = this wave's fragment)
 #pragma unroll
-  for (int f = 0; f < (STEP == kGated ? 2 : 1); ++f)
+  for (int f = 0; f < (moe_pairs(STEP) ? 2 : 1); ++f)
 #pragma unroll
     for (int x = 0; x < NW; x += 4) {
-      const int g = STEP == kGated ? f : wave;
+      const int g = moe_pairs(STEP) ? f : wave;
       s[f] += (red[x][g][lane] + red[x + 1][g][lane]) + (red[x + 2][g][lane] + red[x + 3][g][lane]);
     }
   if (fr >= count) return;
   if (STEP == kRelu2) {
     moe_relu2_4(p.act, place0 + fr, n0 + wave * 16 + fg * 4, s[0]);
-  } else if (STEP == kGated) {
+  } else if (moe_pairs(STEP)) {
     float v[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = moe_glu(s[0][r], s[1][r]);
+    for (int r = 0; r < 4; ++r) v[r] = moe_unit<STEP>(p, s[0][r], s[1][r]);
     store_operand4(p.act, place0 + fr, (n0 >> 1) + fg * 4, v);
   } else {
     *reinterpret_cast<f32x4*>(p.y + (size_t)(place0 + fr) * p.width_p + n0 + wave * 16 + fg * 4) = s[0];
@@ -400,14 +405,14 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(ChattsMoeArgs p) {
         const int n = n0 + (wn * FN + j) * 16;
         if (n < N) moe_relu2_4(p.act, place0 + m, n + fg * 4, acc[i][j]);
       }
-    } else if constexpr (STEP == kGated) {
+    } else if constexpr (moe_pairs(STEP)) {
 #pragma unroll
       for (int j = 0; j < FN; j += 2) {
         const int n = n0 + (wn * FN + j) * 16;
         if (n >= N) continue;
         float v[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = moe_glu(acc[i][j][r], acc[i][j + 1][r]);
+        for (int r = 0; r < 4; ++r) v[r] = moe_unit<STEP>(p, acc[i][j][r], acc[i][j + 1][r]);
         store_operand4(p.act, place0 + m, (n >> 1) + fg * 4, v);
       }
     } else {
@@ -471,8 +476,8 @@ __global__ __launch_bounds__(256) void moe_gemm_f32_kernel(ChattsMoeArgs p) {
       if (STEP == kRelu2) {
 #pragma unroll
         for (int j = 0; j < 2; ++j) p.act.f32[(size_t)(place0 + m) * p.act.ld + n0 + wn + j * 16 + (lane & 15)] = relu2_f(acc[i][j][q]);
-      } else if (STEP == kGated) {
-        p.act.f32[(size_t)(place0 + m) * p.act.ld + ((n0 + wn) >> 1) + (lane & 15)] = moe_glu(acc[i][0][q], acc[i][1][q]);
+      } else if (moe_pairs(STEP)) {
+        p.act.f32[(size_t)(place0 + m) * p.act.ld + ((n0 + wn) >> 1) + (lane & 15)] = moe_unit<STEP>(p, acc[i][0][q], acc[i][1][q]);
       } else {
 #pragma unroll
         for (int j = 0; j < 2; ++j) p.y[(size_t)(place0 + m) * p.width_p + n0 + wn + j * 16 + (lane & 15)] = acc[i][j][q];
@@ -486,7 +491,7 @@ static int check_moe(const ChattsMoeArgs* a, const char* who) {
   CHATTS_REQUIRE(a->experts >= 1 && a->identity >= 0 && n <= kMoeMaxOut && a->top >= 1 && a->top <= 64 && a->groups >= 1 && n % a->groups == 0 && a->keep >= 1 &&
                      a->keep <= a->groups && a->top <= n / a->groups * a->keep, CHATTS_E_SHAPE, "%s: %d experts + %d, top %d, %d of %d groups", who, a->experts,
                  a->identity, a->top, a->keep, a->groups);
-  CHATTS_REQUIRE((a->choose == CHATTS_CHOOSE_SOFTMAX || a->choose == CHATTS_CHOOSE_LOGITS) && (a->act_kind == CHATTS_EXPERT_SWIGLU || a->act_kind == CHATTS_EXPERT_RELU2),
+  CHATTS_REQUIRE(a->choose >= CHATTS_CHOOSE_SOFTMAX && a->choose <= CHATTS_CHOOSE_SCORES && a->act_kind >= CHATTS_EXPERT_SWIGLU && a->act_kind <= CHATTS_EXPERT_CLAMPGLU,
                  CHATTS_E_BADARG, "%s: choice %d, experts of kind %d", who, a->choose, a->act_kind);
   CHATTS_REQUIRE(a->width_p > 0 && a->width_p % 64 == 0 && a->ff_p > 0 && a->ff_p % 64 == 0, CHATTS_E_SHAPE, "%s: widths %d, %d", who, a->width_p, a->ff_p);
   return CHATTS_OK;
@@ -504,14 +509,14 @@ static int moe_tile_bound(int rows, int top, int experts, int bm) {      // sum 
 
 template <int STEP, int RF>
 static void launch_moe_stream_as(const ChattsMoeArgs* a, int n, int tiles, hipStream_t s) {
-  constexpr int NW = STEP == kGated ? 4 : 16;
+  constexpr int NW = moe_pairs(STEP) ? 4 : 16;
   const dim3 g(n / (16 * RF), tiles), b(64 * NW);
   if (STEP == kDown ? a->down_t : a->gate_up_t) hipLaunchKernelGGL((moe_stream_kernel<STEP, true, NW, RF>), g, b, 0, s, *a);
   else hipLaunchKernelGGL((moe_stream_kernel<STEP, false, NW, RF>), g, b, 0, s, *a);
 }
 template <int STEP>
 static void launch_moe_stream(const ChattsMoeArgs* a, int n, int tiles, hipStream_t s) {      // few workgroups: smaller ones, so that the CUs get as much each
-  if constexpr (STEP != kGated)
+  if constexpr (!moe_pairs(STEP))
     if (n / 32 * tiles < 2 * device_cus()) return launch_moe_stream_as<STEP, 1>(a, n, tiles, s);
   launch_moe_stream_as<STEP, 2>(a, n, tiles, s);
 }
@@ -562,9 +567,10 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
   if (a->n_rows == 0) return CHATTS_OK;
   hipStream_t s = as_stream(stream);
   const int bm = moe_bm(a), tiles = moe_tile_bound(a->n_rows, a->top, a->experts, bm), in_rows = moe_in_rows(*a);
-  const bool relu2 = a->act_kind == CHATTS_EXPERT_RELU2;
+  const bool relu2 = a->act_kind == CHATTS_EXPERT_RELU2, clamped = a->act_kind == CHATTS_EXPERT_CLAMPGLU;
   if (a->exact) {
     if (relu2) hipLaunchKernelGGL(moe_gemm_f32_kernel<kRelu2>, dim3(tiles, in_rows / 64), dim3(256), 0, s, *a);
+    else if (clamped) hipLaunchKernelGGL(moe_gemm_f32_kernel<kClamped>, dim3(tiles, in_rows / 64), dim3(256), 0, s, *a);
     else hipLaunchKernelGGL(moe_gemm_f32_kernel<kGated>, dim3(tiles, in_rows / 64), dim3(256), 0, s, *a);
     hipLaunchKernelGGL(moe_gemm_f32_kernel<kDown>, dim3(tiles, a->width_p / 64), dim3(256), 0, s, *a);
     CHATTS_CHECK_LAUNCH("moe_gemm_f32");
@@ -572,6 +578,7 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
   }
   if (moe_small(a)) {
     if (relu2) launch_moe_stream<kRelu2>(a, in_rows, tiles, s);
+    else if (clamped) launch_moe_stream<kClamped>(a, in_rows, tiles, s);
     else launch_moe_stream<kGated>(a, in_rows, tiles, s);
     launch_moe_stream<kDown>(a, a->width_p, tiles, s);
     CHATTS_CHECK_LAUNCH("moe_stream");
@@ -582,7 +589,8 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
     RingGroup g{a->tiles, a->offsets + a->experts + 1, a->order, a->top, (int64_t)in_rows * a->width_p};
     GemmParams p{};
     p.w = a->gate_up; p.wt = a->gate_up_t; p.m = a->n_rows; p.n = in_rows; p.k = p.ldw = a->width_p;
-    p.epilogue = relu2 ? CHATTS_EPI_RELU2 : CHATTS_EPI_SWIGLU;
+    p.epilogue = relu2 ? CHATTS_EPI_RELU2 : (clamped ? CHATTS_EPI_CLAMPGLU : CHATTS_EPI_SWIGLU);
+    p.glu_limit = a->glu_limit; p.glu_alpha = a->glu_alpha;
     p.k_per_split = p.k; p.direct = 1; p.c_hi = a->act.hi; p.c_lo = a->act.lo; p.ldcp = a->act.ld; p.ldc = a->act.ld;
     if ((rc = launch_ring_group(p, a->h.hi, a->h.lo, a->h.ld, g, tiles, s)) != 0) return rc;
     g.order = nullptr;
@@ -591,6 +599,7 @@ extern "C" int chatts_moe_experts(const ChattsMoeArgs* a, chatts_stream_t stream
     p.c_hi = p.c_lo = nullptr; p.c = a->y; p.ldc = a->width_p;
     return launch_ring_group(p, a->act.hi, a->act.lo, a->act.ld, g, tiles, s);
   }
-  if ((rc = relu2 ? launch_moe_gemm<kRelu2, 32, 1, 4>(a, tiles, s) : launch_moe_gemm<kGated, 32, 1, 4>(a, tiles, s)) != 0) return rc;
+  rc = relu2 ? launch_moe_gemm<kRelu2, 32, 1, 4>(a, tiles, s) : (clamped ? launch_moe_gemm<kClamped, 32, 1, 4>(a, tiles, s) : launch_moe_gemm<kGated, 32, 1, 4>(a, tiles, s));
+  if (rc) return rc;
   return launch_moe_gemm<kDown, 32, 1, 4>(a, tiles, s);
 }

@@ -1,6 +1,6 @@
-// pair.hip - the residual stream of layers whose mixer and feed-forward read two norms of the same x: embedding with a row per token pair, the two
-// norms (in groups) in one launch together with what else touches the row - the experts' weighted sum, the input of a joining projection, the
-// operands of a token shift.
+// pair.hip - the residual stream of layers whose mixer and feed-forward read two norms of the same x: embedding (optionally with a row per token pair, or
+// with sinusoidal positions), the two norms (in groups) in one launch together with what else touches the row - the experts' weighted sum, the input of
+// a joining projection, the operands of a token shift.
 #include "common.h"
 
 namespace chatts {
@@ -31,6 +31,16 @@ __global__ __launch_bounds__(256) void embed_pair_kernel(ChattsEmbedPairArgs p) 
       x[1] += bf16_hi(gv[0]);
       x[2] += bf16_lo(gv[1]);
       x[3] += bf16_hi(gv[1]);
+    }
+    if (p.pos_fine) {
+      const int pos = R.pos > 0 ? R.pos : 0;
+      const f32x4 a = *reinterpret_cast<const f32x4*>(p.pos_fine + (size_t)(pos & 63) * p.width_p + c);
+      const f32x4 b = *reinterpret_cast<const f32x4*>(p.pos_coarse + (size_t)(pos >> 6) * p.width_p + c);
+#pragma unroll
+      for (int k = 0; k < 4; k += 2) {
+        x[k] += c + k < p.width ? a[k] * b[k + 1] + a[k + 1] * b[k] : 0.f;
+        x[k + 1] += c + k + 1 < p.width ? a[k + 1] * b[k + 1] - a[k] * b[k] : 0.f;
+      }
     }
     *reinterpret_cast<f32x4*>(p.x + (size_t)row * p.width_p + c) = x;
     if (p.x0) *reinterpret_cast<f32x4*>(p.x0 + (size_t)row * p.width_p + c) = x;
@@ -229,6 +239,8 @@ extern "C" int chatts_embed_pair(const ChattsEmbedPairArgs* a, chatts_stream_t s
   CHATTS_REQUIRE(a && a->tokens && a->rows && a->embed && a->x && a->t >= 0 && a->width_p > 0 && a->width_p % 4 == 0 && a->vocab > 0, CHATTS_E_BADARG,
                  "embed_pair: bad arguments");
   CHATTS_REQUIRE(!a->bigram || (a->buckets > 0 && a->prev), CHATTS_E_BADARG, "embed_pair: %lld buckets", (long long)a->buckets);
+  CHATTS_REQUIRE(!a->pos_fine || (a->pos_coarse && a->width > 0 && a->width <= a->width_p && (((uintptr_t)a->pos_fine | (uintptr_t)a->pos_coarse) % 16) == 0),
+                 CHATTS_E_BADARG, "embed_pair: positions");
   if (a->t == 0) return CHATTS_OK;
   hipLaunchKernelGGL(embed_pair_kernel, dim3(a->t), dim3(256), 0, as_stream(stream), *a);
   CHATTS_CHECK_LAUNCH("embed_pair");

@@ -1,6 +1,6 @@
 // window.hip - attention over paged keys and values with grouped heads.  Optional, each by its own parameter: short convolutions, norms of queries and
-// keys (per head, over all heads, unit after a rotation of pairs), mixed values; capped scores, a distance bias per head, a sliding window that keeps
-// a sequence's first tokens, chunks, a sink (one more term exp(0) in the denominator); an output gate per value or per head.
+// keys (per head, over all heads, unit after a rotation of pairs), mixed values; capped scores, a distance bias per head (linear or logarithmic), a sliding window that
+// keeps a sequence's first tokens, chunks, a sink (one more term exp(0) in the denominator); an output gate per value or per head.
 //   window_prep_kernel      per-head work: norms, rotation, values; queries as an operand, keys and values into their pages
 //   window_prep_quads_kernel  the same, four channels a lane
 //   window_prep_rows_kernel the same for layers with convolutions or norms over all heads: a workgroup owns whole rows
@@ -46,15 +46,20 @@ __device__ __forceinline__ float window_gate(const ChattsWindowArgs& p, size_t r
   return p.off_gate < 0 ? 1.f : sigmoid_f(p.proj[row * p.ld_proj + p.off_gate + (p.gate_heads ? h : h * p.vdim + c)]);
 }
 constexpr float kLog2e = 1.44269504088896341f;
-// what the matrix kernels are compiled for (registers are scarce there): plain scores, a distance bias, capped scores (with chunks), or whatever is set
-enum { kPlain = 0, kSlope, kCap, kAny };
+// what the matrix kernels are compiled for (registers are scarce there): plain scores, a distance bias, capped scores (with chunks), a logarithmic bias, or
+// whatever is set
+enum { kPlain = 0, kSlope, kCap, kLog, kAny };
 template <int SCORE>
 __device__ __forceinline__ bool window_capped(const ChattsWindowArgs& p) { return SCORE == kCap || (SCORE == kAny && p.softcap > 0.f); }
 template <int SCORE>
 __device__ __forceinline__ bool window_sloped(const ChattsWindowArgs& p) { return SCORE == kSlope || (SCORE == kAny && p.slopes != nullptr); }
 template <int SCORE>
+__device__ __forceinline__ bool window_logged(const ChattsWindowArgs& p) { return SCORE == kLog || (SCORE == kAny && p.log_r1 != nullptr); }
+// r1 log2(1 + r2 d)
+__device__ __forceinline__ float window_log(float r1, float r2, float d) { return r1 * __builtin_amdgcn_logf(1.f + r2 * d); }
+template <int SCORE>
 __device__ __forceinline__ int window_low_of(const ChattsWindowArgs& p, int pos) {
-  if (SCORE == kPlain || SCORE == kSlope) return p.window > 0 ? pos - p.window + 1 : 0;      // (no chunks there)
+  if (SCORE == kPlain || SCORE == kSlope || SCORE == kLog) return p.window > 0 ? pos - p.window + 1 : 0;      // (no chunks there)
   return window_low(p, pos);
 }
 // cap tanh(x / cap), in units of cap: tanh(y) = 1 - 2 / (1 + exp(2 y));  k = 2 log2(e) / cap
@@ -405,7 +410,7 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
   float m = p.sink ? 0.f : -INFINITY, l = p.sink ? 1.f : 0.f, o = 0.f;      // column tid
   const WindowTiles T(p, R.pos, R.pos, 6);
   const int n = T.count(), low = window_low(p, R.pos);
-  const float slope = p.slopes ? p.slopes[h] : 0.f;
+  const float slope = p.slopes ? p.slopes[h] : 0.f, r1 = p.log_r1 ? p.log_r1[h] : 0.f, r2 = p.log_r1 ? p.log_r2[h] : 0.f;
   for (int i = 0; i < n; ++i) {
     __syncthreads();
     const int k0 = T.tile(i) * 64;
@@ -426,7 +431,8 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
     d += lane_xor2(d);
     d *= p.scale;
     if (p.softcap > 0.f) d = p.softcap * tanhf(d / p.softcap);
-    if (part == 0) sc[key] = sees ? d - slope * (float)(R.pos - k0 - key) : -INFINITY;
+    const float far = (float)(R.pos - k0 - key);
+    if (part == 0) sc[key] = sees ? d - slope * far - (p.log_r1 ? r1 * log1pf(r2 * far) : 0.f) : -INFINITY;
     __syncthreads();
     const float s = sc[tid & 63];
     const float mn = fmaxf(m, wave_max(s)), safe = mn == -INFINITY ? 0.f : mn;
@@ -447,7 +453,7 @@ __global__ __launch_bounds__(256) void window_attend_kernel(ChattsWindowArgs p) 
       }
     }
   }
-  if (tid < p.vdim) store_operand(p.out, row, h * p.vdim + tid, o / l * window_gate(p, row, h, tid));
+  if (tid < p.vdim) store_operand(p.out, row, h * p.vdim + tid, o / l * window_gate(p, row, h, tid) * p.out_scale);
 }
 
 // ---- one row on the matrix pipe: grid (splits, kv heads * head tiles, rows), 4 waves ----
@@ -472,6 +478,7 @@ __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_d
   const WindowTiles T(p, R.pos, R.pos, 5);
   const int n = T.count(), stride = 4 * p.n_splits, low = window_low_of<SCORE>(p, R.pos);
   const float slope2 = window_sloped<SCORE>(p) ? p.slopes[head] * kLog2e : 0.f;
+  const float r1 = window_logged<SCORE>(p) ? p.log_r1[head] : 0.f, r2 = window_logged<SCORE>(p) ? p.log_r2[head] : 0.f;
   float m = -INFINITY, l = 0.f;
   f32x4 o[NV];
 #pragma unroll
@@ -521,6 +528,7 @@ __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_d
     for (int j = 0; j < 8; ++j) {
       const int key = k0 + (j >> 2) * 16 + fg * 4 + (j & 3);
       if (SCORE == kSlope || SCORE == kAny) v[j] += slope2 * (d0 + (float)((j >> 2) * 16 + (j & 3)));
+      if (window_logged<SCORE>(p)) v[j] -= window_log(r1, r2, -d0 - (float)((j >> 2) * 16 + (j & 3)));      // (NaN only for keys ahead, which are masked)
       if (!window_sees(p, R.pos, low, key)) v[j] = -INFINITY;
       mx = fmaxf(mx, v[j]);
     }
@@ -593,7 +601,7 @@ __global__ __launch_bounds__(256, NV <= 4 ? 4 : (NV <= 8 ? 3 : 1)) void window_d
       acc += f * part[(w * 16 + hh) * ldp + c];
     }
     if (whole) {
-      if (c < p.vdim) store_operand(p.out, row, hd * p.vdim + c, acc / L * window_gate(p, row, hd, c));
+      if (c < p.vdim) store_operand(p.out, row, hd * p.vdim + c, acc / L * window_gate(p, row, hd, c) * p.out_scale);
     } else {
       float* dst = p.partial + (((size_t)row * p.heads + hd) * p.n_splits + split) * ldp;
       dst[c] = acc;
@@ -621,7 +629,7 @@ __global__ __launch_bounds__(128) void window_merge_kernel(ChattsWindowArgs p) {
     float o = 0.f;
 #pragma unroll 4
     for (int s = 0; s < p.n_splits; ++s) o += w[s] * part[(size_t)s * ld + c];
-    store_operand(p.out, row, h * p.vdim + c, o * window_gate(p, row, h, c));
+    store_operand(p.out, row, h * p.vdim + c, o * window_gate(p, row, h, c) * p.out_scale);
   }
 }
 
@@ -659,6 +667,7 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
   const float scale2 = p.scale * kLog2e;      // scores in base 2
   const float cap2 = p.softcap * kLog2e, capk = window_capped<SCORE>(p) ? 2.f * kLog2e * p.scale / p.softcap : 0.f;
   const float slope2 = window_sloped<SCORE>(p) ? p.slopes[h] * kLog2e : 0.f;
+  const float r1 = window_logged<SCORE>(p) ? p.log_r1[h] : 0.f, r2 = window_logged<SCORE>(p) ? p.log_r2[h] : 0.f;
   const int low_first = window_low_of<SCORE>(p, w0), low_last = window_low_of<SCORE>(p, w1);
   int lows[2] = {0, 0};
   if (SCORE == kCap || SCORE == kAny) { lows[0] = window_low(p, w0 + fr); lows[1] = window_low(p, w0 + 16 + fr); }
@@ -748,6 +757,13 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
 #pragma unroll
           for (int r = 0; r < 4; ++r) s[a][u][r] += slope2 * (d0 + (float)(a * 16 + r));
       }
+      if (window_logged<SCORE>(p)) {
+        const float d0 = (float)(qpos - k0 - fg * 4);
+#pragma unroll
+        for (int a = 0; a < 4; ++a)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[a][u][r] -= window_log(r1, r2, d0 - (float)(a * 16 + r));      // (NaN only for keys ahead, which are masked)
+      }
       float mx = -INFINITY;
 #pragma unroll
       for (int a = 0; a < 4; ++a)
@@ -815,7 +831,7 @@ __global__ __launch_bounds__(256, OCC) void window_prefill_kernel(ChattsWindowAr
     L += __shfl_xor(L, 32, 64);
     if (r >= sp.t) continue;
     const size_t row = sp.row0 + r;
-    const float inv = 1.0f / L * (p.gate_heads ? window_gate(p, row, h, 0) : 1.f);
+    const float inv = 1.0f / L * p.out_scale * (p.gate_heads ? window_gate(p, row, h, 0) : 1.f);
 #pragma unroll
     for (int f = 0; f < NV; ++f) {
       const int c = f * 16 + fg * 4, at = h * p.vdim + c;
@@ -851,6 +867,7 @@ static int check_window(const ChattsWindowArgs* a, const char* who) {
                  a->log_block, a->window, a->keep_first);
   CHATTS_REQUIRE(a->chunk >= 0 && (a->chunk == 0 || a->window == 0) && a->softcap >= 0.f && (!a->gate_heads || a->off_gate >= 0), CHATTS_E_SHAPE,
                  "%s: window %d and chunks of %d, scores capped at %g", who, a->window, a->chunk, (double)a->softcap);
+  CHATTS_REQUIRE((a->log_r1 != nullptr) == (a->log_r2 != nullptr), CHATTS_E_BADARG, "%s: half of a logarithmic bias", who);
   CHATTS_REQUIRE(a->rot >= 0 && a->rot % 2 == 0 && a->rot <= a->dim && (a->rot == 0 || (a->cos_tab && a->sin_tab)), CHATTS_E_SHAPE, "%s: %d of %d dimensions rotated", who,
                  a->rot, a->dim);
   CHATTS_REQUIRE(a->taps >= 0 && (a->taps == 0 || (a->conv_w && a->ring && a->conv_ch % 4 == 0 && a->conv_ch <= a->ld_proj && a->off_q + a->heads * a->dim <= a->conv_ch &&
@@ -868,6 +885,11 @@ static int check_window(const ChattsWindowArgs* a, const char* who) {
   CHATTS_REQUIRE((((uintptr_t)a->kcache | (uintptr_t)a->vcache | (uintptr_t)a->proj) % 16) == 0 && a->q.ld >= a->heads * a->dim_p && a->q.ld % 8 == 0 &&
                      (a->cache_f32 ? a->q.f32 != nullptr : a->q.hi != nullptr), CHATTS_E_SHAPE, "%s: alignment / queries", who);
   return CHATTS_OK;
+}
+static ChattsWindowArgs window_scaled(const ChattsWindowArgs* args) {      // out_scale 0: 1
+  ChattsWindowArgs a = *args;
+  if (a.out_scale == 0.f) a.out_scale = 1.f;
+  return a;
 }
 static bool window_out_ok(const ChattsWindowArgs* a) { return (a->out.f32 || a->out.hi) && a->out.ld >= a->heads * a->vdim; }
 
@@ -903,9 +925,9 @@ static int window_lds(K kernel, size_t bytes, bool& done) {
 }
 
 static int window_score(const ChattsWindowArgs* a) {
-  if (a->softcap > 0.f && !a->slopes) return kCap;
-  if (a->softcap > 0.f || a->chunk > 0) return kAny;
-  return a->slopes ? kSlope : kPlain;
+  if (a->softcap > 0.f && !a->slopes && !a->log_r1) return kCap;
+  if (a->softcap > 0.f || a->chunk > 0 || (a->slopes && a->log_r1)) return kAny;
+  return a->log_r1 ? kLog : (a->slopes ? kSlope : kPlain);
 }
 
 template <int NK, int NV, int SCORE>
@@ -925,6 +947,7 @@ static int launch_window_decode(const ChattsWindowArgs* a, hipStream_t s) {
     case kPlain: return launch_window_decode_as<NK, NV, kPlain>(a, s);
     case kSlope: return launch_window_decode_as<NK, NV, kSlope>(a, s);
     case kCap: return launch_window_decode_as<NK, NV, kCap>(a, s);
+    case kLog: return launch_window_decode_as<NK, NV, kLog>(a, s);
     default: return launch_window_decode_as<NK, NV, kAny>(a, s);
   }
 }
@@ -943,6 +966,7 @@ static int launch_window_prefill(const ChattsWindowArgs* a, hipStream_t s) {
     case kPlain: return launch_window_prefill_as<NK, NV, OCC, kPlain>(a, s);
     case kSlope: return launch_window_prefill_as<NK, NV, OCC, kSlope>(a, s);
     case kCap: return launch_window_prefill_as<NK, NV, OCC, kCap>(a, s);
+    case kLog: return launch_window_prefill_as<NK, NV, OCC, kLog>(a, s);
     default: return launch_window_prefill_as<NK, NV, OCC, kAny>(a, s);
   }
 }
@@ -972,8 +996,9 @@ extern "C" int chatts_window_prep(const ChattsWindowArgs* a, chatts_stream_t str
 
 extern "C" int chatts_window_can_prefill(int dim_p, int vdim_p) { return dim_p <= 256 && vdim_p <= 256; }
 
-extern "C" int chatts_window_attend(const ChattsWindowArgs* a, chatts_stream_t stream) {
-  if (const int rc = check_window(a, "window_attend")) return rc;
+extern "C" int chatts_window_attend(const ChattsWindowArgs* args, chatts_stream_t stream) {
+  if (const int rc = check_window(args, "window_attend")) return rc;
+  const ChattsWindowArgs scaled = window_scaled(args), *a = &scaled;
   CHATTS_REQUIRE(window_out_ok(a), CHATTS_E_BADARG, "window_attend: no output");
   if (a->n_rows == 0) return CHATTS_OK;
   hipStream_t s = as_stream(stream);
@@ -995,8 +1020,9 @@ extern "C" int chatts_window_attend(const ChattsWindowArgs* a, chatts_stream_t s
   return CHATTS_OK;
 }
 
-extern "C" int chatts_window_prefill(const ChattsWindowArgs* a, chatts_stream_t stream) {
-  if (const int rc = check_window(a, "window_prefill")) return rc;
+extern "C" int chatts_window_prefill(const ChattsWindowArgs* args, chatts_stream_t stream) {
+  if (const int rc = check_window(args, "window_prefill")) return rc;
+  const ChattsWindowArgs scaled = window_scaled(args), *a = &scaled;
   CHATTS_REQUIRE(window_out_ok(a) && a->spans && !a->cache_f32, CHATTS_E_BADARG, "window_prefill: bad arguments");
   if (a->n_rows == 0 || a->n_spans == 0 || a->longest == 0) return CHATTS_OK;
   if (a->dim_p <= 64 && a->vdim_p <= 64) return launch_window_prefill<2, 4, 2>(a, as_stream(stream));

@@ -2,15 +2,19 @@
 
 A sequential layer is norm1 -> mixer -> norm1b -> residual, then optionally norm2 -> squared-relu feed-forward -> norm2b -> residual; a parallel one adds
 mixer(norm1(x)) + feed-forward(norm2(x)) to x, both norms of the same x in groups (csrc/pair.hip); a post-norm one is x <- norm1(alpha x + mixer(x)), then
-x <- norm2(alpha x + feed-forward(x)) (csrc/postnorm.hip).  Mixers:
+x <- norm2(alpha x + feed-forward(x)) (csrc/postnorm.hip); a pre-norm one adds factors of mixer(norm1(x)) and feed-forward(norm2(x)) in turn and may average the
+streams of all layers so far (csrc/depth.hip).  Mixers:
   LatentMixer   attention over a paged cache of one latent + one rotated key part per token (csrc/latent.hip)
   DeltaMixer    gated delta rule: a float32 state and a ring of convolution inputs per slot (csrc/delta.hip)
   WindowMixer   grouped-head attention over paged keys and values (csrc/window.hip); by its fields: short convolutions with a ring of inputs per slot, norms
                 per head / over all heads / after a rotation, values mixed with an earlier layer's, window or chunks, kept first tokens, sink, capped
-                scores, a distance bias, a gate per value or per head
+                scores, a distance bias (linear or logarithmic), a gate per value or per head
   WkvMixer, MlstmMixer   gated linear recurrences: a float32 state per slot (csrc/recur.hip)
-Feed-forwards of parallel and post-norm layers: ClampGlu, GeluGlu, Experts (csrc/moe.hip).
-A design (chatts_amd/fobolix.py, chatts_amd/medilix.py, chatts_amd/mefurax.py) says in which order layers run (config.runs(): a layer may run several times, every run has
+  MinGruMixer   a gated recurrence per channel whose gates read the current token alone: a float32 state per slot (csrc/gru.hip)
+  SelectMixer   selective scan: a float32 state and a ring of convolution inputs per slot (csrc/select.hip)
+  SideBySide    two of WindowMixer, MinGruMixer, SelectMixer reading the same rows, their outputs added with a factor each
+Feed-forwards of parallel, post-norm and pre-norm layers: ClampGlu, GeluGlu, Experts (csrc/moe.hip).
+A design (chatts_amd/fobolix.py, medilix.py, mefurax.py, muvetar.py) says in which order layers run (config.runs(): a layer may run several times, every run has
 its own pages or state) and maps its tensor names onto LayerWeights.
 
 Everything is padded once, at load: widths and feed-forwards to multiples of 64, the stacked input projections block by block, heads to
@@ -21,6 +25,7 @@ position, so prefixes are not reused between requests.
 """
 import ctypes as C
 import glob
+import math
 import os
 from dataclasses import dataclass
 from types import SimpleNamespace
@@ -30,7 +35,7 @@ import torch
 
 from . import _lib
 from .kv_blocks import BlockPool
-from .rotary import rotary_tables
+from .rotary import rotary_tables, sinusoid_tables
 from .slot_model import SlotModel
 from .tp import LocalComm
 
@@ -104,6 +109,7 @@ class WindowMixer:
     softcap: float = 0.0        # 0: none
     slopes: Any = None          # [heads] or None
     gate_heads: bool = False    # g is [heads, width]: one gate per head
+    log_bias: Any = None        # (r1, r2), [heads] each: r1 ln(1 + r2 distance) is taken off the scores; or None
     vmix: Optional[float] = None    # values become (1 - vmix) v + vmix v_first, v_first those of the first layer that has a vmix
 
 
@@ -143,6 +149,39 @@ class MlstmMixer:
 
 
 @dataclass
+class MinGruMixer:
+    z: Any          # [channels, width]: gate, candidate, output gate
+    x: Any
+    g: Any
+    bias_z: Any
+    bias_x: Any
+    o: Any
+
+
+@dataclass
+class SelectMixer:
+    state: int      # states per channel
+    rank: int       # of the step sizes
+    w_in: Any       # [x: channels | z: channels, width]
+    conv: Any       # [channels, taps]
+    conv_bias: Any
+    x: Any          # [dt: rank | B: state | C: state, channels]
+    dt: Any         # [channels, rank]
+    dt_bias: Any
+    a_log: Any      # [channels, state]
+    d: Any
+    o: Any
+
+
+@dataclass
+class SideBySide:
+    left: Any
+    right: Any      # of another kind than left
+    left_scale: float
+    right_scale: float
+
+
+@dataclass
 class ClampGlu:
     gate: Any
     up: Any
@@ -168,7 +207,10 @@ class Experts:
     groups: int
     keep: int
     by_logits: bool = False     # chosen by logits, weights: softmax over the chosen ones
-    shared: Any = None          # (up, down) of a squared-relu expert that every token uses (post-norm layers)
+    shared: Any = None          # an expert that every token uses: (up, down), squared relu, in post-norm layers; (gate, up, down), clamped, in pre-norm ones
+    weight_scale: Optional[float] = None    # weights: the chosen softmax values as they are, times this
+    clamp: Optional[tuple] = None           # (limit, alpha): experts are clamped gated units
+    shared_clamp: Optional[tuple] = None
 
 
 @dataclass
@@ -180,9 +222,11 @@ class LayerWeights:
     norm2b: Any = None
     up: Any = None      # squared-relu feed-forward of a sequential layer
     down: Any = None
-    ff: Any = None      # ClampGlu, GeluGlu or Experts of a parallel or post-norm layer
+    ff: Any = None      # ClampGlu, GeluGlu or Experts of a parallel, post-norm or pre-norm layer
     parallel: bool = False
     post: bool = False  # norms after the sums; norm1 / norm2 as they multiply
+    pre: bool = False   # norms before the sublayers only
+    depth: Any = None   # pre: weights of the embedding output and of every layer's result so far, whose sum goes on
 
 
 def _up(n, m):
@@ -276,6 +320,12 @@ class MixedDecoder(SlotModel):
                 t = 0.5 + 0.1 * t
             if name.endswith(".correction"):
                 t = 0.01 * t        # (larger ones would send every token to the same few experts)
+            if name.endswith(".dt.b"):
+                t = 0.5 * t - 3.0
+            if name.endswith((".r1", ".r2")):
+                t = 0.5 * t.abs()
+            if name.endswith(".dwa"):
+                t = t / shape[0]
             sd[name] = t.to(torch.bfloat16)
         m.load_weights(sd.items())
         return m
@@ -321,16 +371,21 @@ class MixedDecoder(SlotModel):
         t = _pad(t.to(torch.bfloat16), t.shape[0], cols)
         return self._dev(t.view(t.shape[0], cols // 8, 8).transpose(0, 1).contiguous())
 
-    def _stack(self, blocks):
-        """stacked input projection: (name, [rows, width], padded rows) -> (matrix, {name: first row})"""
+    def _stack(self, blocks, cols=None):
+        """stacked projection: (name, [rows, width], padded rows) -> (matrix, {name: first row}); cols: padded width of its input"""
         off, at = {}, 0
         for name, t, rows in blocks:
             off[name] = at
             at += rows
-        out = torch.zeros((_up(at, 64), self._wp), dtype=torch.bfloat16, device=self.device)
+        out = torch.zeros((_up(at, 64), cols or self._wp), dtype=torch.bfloat16, device=self.device)
         for name, t, rows in blocks:
             out[off[name]:off[name] + t.shape[0], :t.shape[1]] = t.to(torch.bfloat16)
         return out, off
+
+    def _state(self, shape):
+        t = torch.zeros(shape, dtype=torch.float32, device=self.device)
+        self.state_bytes += 4 * t.numel()
+        return self._dev(t)
 
     def _latent_layer(self, L, m):
         H, W = m.heads, self.config.hidden_size
@@ -397,16 +452,18 @@ class MixedDecoder(SlotModel):
                 L.mix_t[j] = self._mat(w[L.mix_row[j]:L.mix_row[j + 1]], tile=True)[1] if self.tiled else None
         return off
 
-    def _window_layer(self, L, m):
-        L.kind = _lib.MIX_WINDOW
-        off = self._blocks(L, [("q", m.q), ("k", m.k), ("v", m.v)] + ([("g", m.g)] if m.g is not None else []), bias=dict(zip("qkv", m.bias)) if m.bias else None)
-        n, dim_p, vdim_p = m.heads * m.vdim, _up(m.dim, 32), _up(m.vdim, 16)
-        L.out_k = _up(n, 64)
-        L.out, L.out_t = self._mat(m.o, self._wp, L.out_k, tile=True)
+    # a mixer that may stand beside another: its blocks of the stacked input projection and their biases, and what its kernels need (off: first rows of its blocks)
+    def _window_blocks(self, m):
+        return [("q", m.q), ("k", m.k), ("v", m.v)] + ([("g", m.g)] if m.g is not None else []), dict(zip("qkv", m.bias)) if m.bias else {}
+
+    def _window_args(self, L, m, off, scale):
+        dim_p, vdim_p = _up(m.dim, 32), _up(m.vdim, 16)
         L.window = _lib.WindowArgs(off_q=off["q"], off_k=off["k"], off_v=off["v"], off_gate=off.get("g", -1), heads=m.heads, kv_heads=m.kv_heads, dim=m.dim,
                                    vdim=m.vdim, dim_p=dim_p, vdim_p=vdim_p, scale=m.scale, window=m.window, keep_first=m.keep_first if m.window or m.chunk else 0, sink=int(m.sink),
-                                   chunk=m.chunk, softcap=m.softcap, gate_heads=int(m.gate_heads), norm_whole=int(m.norm_whole), rot=m.rot, unit=int(m.unit))
+                                   chunk=m.chunk, softcap=m.softcap, gate_heads=int(m.gate_heads), norm_whole=int(m.norm_whole), rot=m.rot, unit=int(m.unit), out_scale=scale)
         a = L.window
+        if m.log_bias is not None:
+            a.log_r1, a.log_r2 = (self._f32(t) for t in m.log_bias)
         if m.q_norm is not None:
             a.q_norm, a.k_norm = (self._f32(t, _up(t.shape[0], 4)) for t in (m.q_norm, m.k_norm))
         if m.slopes is not None:
@@ -423,6 +480,58 @@ class MixedDecoder(SlotModel):
         if m.vmix is not None:
             a.vmix, a.ld_vfirst = m.vmix, _up(m.kv_heads * m.vdim, 4)
         self._lat_q, self._lat_o = max(self._lat_q, m.heads * dim_p), max(self._lat_o, m.heads * (vdim_p + 4))
+
+    def _gru_blocks(self, m):
+        return [("z", m.z), ("x", m.x), ("g", m.g)], {"z": m.bias_z, "x": m.bias_x}
+
+    def _gru_args(self, L, m, off, scale):
+        L.gru = _lib.GruArgs(off_z=off["z"], off_x=off["x"], off_g=off["g"], width=m.z.shape[0], out_scale=scale)
+
+    def _select_blocks(self, m):
+        n = m.conv.shape[0]
+        return [("x", m.w_in[:n]), ("z", m.w_in[n:])], {}
+
+    def _select_args(self, L, m, off, scale):
+        (n, taps), N, rank = m.conv.shape, m.state, _up(m.rank, 64)
+        n4, N4, L.sel_k = _up(n, 4), _up(N, 4), _up(n, 64)
+        low, at = self._stack([("dt", m.x[:m.rank], rank), ("b", m.x[m.rank:m.rank + N], _up(N, 16)), ("c", m.x[m.rank + N:], _up(N, 16))], L.sel_k)
+        L.sel_low, L.sel_low_t = self._mat(low, tile=True)
+        L.sel_dt_n = L.sel_k
+        L.sel_dt = self._mat(m.dt, L.sel_dt_n, rank)[0]
+        conv, a = torch.zeros((taps, n4), dtype=torch.float32, device=self.device), torch.zeros((n, N4), dtype=torch.float32, device=self.device)
+        conv[:, :n] = m.conv.to(torch.float32).t()
+        a[:, :N] = (-torch.exp(m.a_log.to(torch.float64)) * math.log2(math.e)).float()
+        L.select = _lib.SelectArgs(off_x=off["x"], off_z=off["z"], inner=n, state=N, taps=taps, conv_ch=n4, conv_w=self._dev(conv), conv_b=self._f32(m.conv_bias, n4),
+                                   ld_low=low.shape[0], off_dt=at["dt"], off_b=at["b"], off_c=at["c"], rank=rank, w_dt=L.sel_dt, dt_bias=self._f32(m.dt_bias, n4),
+                                   a=self._dev(a), d=self._f32(m.d, n4), out_scale=scale)
+
+    def _mixers(self, L, parts):
+        """one mixer, or two side by side: (mixer, factor of its output) each"""
+        about = {WindowMixer: (_lib.MIX_WINDOW, self._window_blocks, self._window_args), MinGruMixer: (_lib.MIX_GRU, self._gru_blocks, self._gru_args),
+                 SelectMixer: (_lib.MIX_SELECT, self._select_blocks, self._select_args)}
+        blocks, bias = [], {}
+        for j, (m, _) in enumerate(parts):
+            rows, b = about[type(m)][1](m)
+            blocks += [((j, n), t) for n, t in rows]
+            bias.update({(j, n): t for n, t in b.items()})
+        off = self._blocks(L, blocks, bias=bias)
+        cols = [_up(m.o.shape[1], 64) for m, _ in parts]
+        L.kind, L.out_k = about[type(parts[0][0])][0], sum(cols)
+        out = torch.zeros((self._wp, L.out_k), dtype=torch.bfloat16, device=self.device)
+        for j, (m, scale) in enumerate(parts):
+            at = sum(cols[:j])
+            if scale:      # (the kernels take a factor of zero for none)
+                out[:m.o.shape[0], at:at + m.o.shape[1]] = m.o.to(torch.bfloat16)
+            about[type(m)][2](L, m, {n: r for (i, n), r in off.items() if i == j}, scale)
+        L.out, L.out_t = self._mat(out, tile=True)
+        if len(parts) > 1:
+            L.beside, L.beside_col = about[type(parts[1][0])][0], cols[0]
+
+    def _single_layer(self, L, m):
+        self._mixers(L, [(m, 1.0)])
+
+    def _side_by_side(self, L, m):
+        self._mixers(L, [(m.left, m.left_scale), (m.right, m.right_scale)])
 
     def _wkv_layer(self, L, m):
         n, rank = m.heads * m.dim, _up(m.w1.shape[0], 64)
@@ -479,13 +588,17 @@ class MixedDecoder(SlotModel):
         L.ff_kind, L.router_n = _lib.FF_MOE, _up(n + m.identity, 64)
         L.router, L.router_t = self._mat(m.router, L.router_n, self._wp, tile=True)
         L.moe = _lib.MoeArgs(experts=n, identity=m.identity, top=m.top, groups=m.groups, keep=m.keep,
-                             choose=_lib.CHOOSE_LOGITS if m.by_logits else _lib.CHOOSE_SOFTMAX, act_kind=_lib.EXPERT_SWIGLU if gated else _lib.EXPERT_RELU2,
+                             choose=_lib.CHOOSE_LOGITS if m.by_logits else (_lib.CHOOSE_SOFTMAX if m.weight_scale is None else _lib.CHOOSE_SCORES),
+                             act_kind=_lib.EXPERT_CLAMPGLU if m.clamp else (_lib.EXPERT_SWIGLU if gated else _lib.EXPERT_RELU2), weight_scale=m.weight_scale or 0.0,
+                             glu_limit=m.clamp[0] if m.clamp else 0.0, glu_alpha=m.clamp[1] if m.clamp else 0.0,
                              width_p=self._wp, ff_p=ff, gate_up=self._dev(gu), down=self._dev(dn), gate_up_t=gut, down_t=dnt,
                              correction=None if m.correction is None else self._f32(m.correction))
         if m.shared is not None:
             L.ff = _up(m.shared[0].shape[0], 64)
-            L.up, L.up_t = self._mat(m.shared[0], L.ff, self._wp, tile=True)
-            L.down, L.down_t = self._mat(m.shared[1], self._wp, L.ff, tile=True)
+            if m.shared_clamp:
+                L.glu_limit, L.glu_alpha = m.shared_clamp
+            L.up, L.up_t = self._mat(self._gate_up(m.shared[0], m.shared[1], L.ff) if m.shared_clamp else m.shared[0], None if m.shared_clamp else L.ff, self._wp, tile=True)
+            L.down, L.down_t = self._mat(m.shared[-1], self._wp, L.ff, tile=True)
 
     def _build(self, sd):
         cfg, lib, dev = self.config, self.lib, self.device
@@ -496,11 +609,13 @@ class MixedDecoder(SlotModel):
         self.expand_rows = 0 if self.exact else _up(min(self.max_ctx, max(8192, 2 * T)), 64) + 64 * MB
         self._exp = [0] * 5                              # latent, rotated part, keys, values, queries of the expanded form: widest layer
         mixers, arr = [], (_lib.MixLayer * len(cfg.layers))()
-        build = {LatentMixer: self._latent_layer, DeltaMixer: self._delta_layer, WindowMixer: self._window_layer, WkvMixer: self._wkv_layer,
-                 MlstmMixer: self._mlstm_layer}
+        build = {LatentMixer: self._latent_layer, DeltaMixer: self._delta_layer, WindowMixer: self._single_layer, WkvMixer: self._wkv_layer,
+                 MlstmMixer: self._mlstm_layer, MinGruMixer: self._single_layer, SelectMixer: self._single_layer, SideBySide: self._side_by_side}
         for i in range(len(cfg.layers)):
             lw, L = self.layer_weights(sd, i), arr[i]
-            L.norm1, L.parallel, L.post = self._f32(lw.norm1, Wp), int(lw.parallel), int(lw.post)
+            L.norm1, L.parallel, L.post, L.pre = self._f32(lw.norm1, Wp), int(lw.parallel), int(lw.post), int(lw.pre)
+            if lw.depth is not None:
+                L.depth = self._f32(lw.depth)
             if lw.norm1b is not None:
                 L.norm1b = self._f32(lw.norm1b, Wp)
             build[type(lw.mixer)](L, lw.mixer)
@@ -542,15 +657,20 @@ class MixedDecoder(SlotModel):
                 t = torch.zeros((nblk, self.kv_block_size, a.rank_p + a.rot_p), dtype=cache_dtype, device=dev)
                 runs[r].cache = self._dev(t)
                 self.cache_bytes += t.numel() * t.element_size()
-            elif isinstance(mixers[i], WindowMixer):
-                a = arr[i].window
-                k, v = (torch.zeros((nblk, a.kv_heads, self.kv_block_size, d), dtype=cache_dtype, device=dev) for d in (a.dim_p, a.vdim_p))
-                runs[r].cache, runs[r].vcache = self._dev(k), self._dev(v)
-                self.cache_bytes += (k.numel() + v.numel()) * k.element_size()
-                if a.taps:
-                    ring = torch.zeros((MB, a.taps, a.conv_ch), **f32)
-                    runs[r].ring = self._dev(ring)
-                    self.state_bytes += 4 * ring.numel()
+            elif arr[i].kind in (_lib.MIX_WINDOW, _lib.MIX_GRU, _lib.MIX_SELECT):
+                kinds = (arr[i].kind, arr[i].beside)
+                if _lib.MIX_WINDOW in kinds:
+                    a = arr[i].window
+                    k, v = (torch.zeros((nblk, a.kv_heads, self.kv_block_size, d), dtype=cache_dtype, device=dev) for d in (a.dim_p, a.vdim_p))
+                    runs[r].cache, runs[r].vcache = self._dev(k), self._dev(v)
+                    self.cache_bytes += (k.numel() + v.numel()) * k.element_size()
+                    if a.taps:
+                        runs[r].ring = self._state((MB, a.taps, a.conv_ch))
+                if _lib.MIX_GRU in kinds:
+                    runs[r].gru_state = self._state((MB, _up(arr[i].gru.width, 4)))
+                if _lib.MIX_SELECT in kinds:
+                    a = arr[i].select
+                    runs[r].sel_state, runs[r].sel_ring = self._state((MB, a.inner, _up(a.state, 4))), self._state((MB, a.taps, a.conv_ch))
             elif arr[i].kind == _lib.MIX_RECUR:
                 a = arr[i].recur
                 mem = [torch.zeros((MB, a.heads, a.dim, _up(a.vdim, 4)), **f32), torch.zeros((MB, Wp), **f32) if arr[i].n_mix else None]
@@ -571,6 +691,8 @@ class MixedDecoder(SlotModel):
         most = lambda f: max([f(L) for L in deltas], default=1)
         over = lambda layers, f: max([f(L) for L in layers], default=1)
         shifts, pairs, n_mix = bool(over(recurs, lambda L: L.n_mix) > 1), T * over(moes, lambda L: L.moe.top), over(arr, lambda L: L.n_mix)
+        selects = [L for L in arr if _lib.MIX_SELECT in (L.kind, L.beside)]
+        depth = any(L.depth for L in arr)
         mixing = [i for i, _ in order if isinstance(mixers[i], WindowMixer) and mixers[i].vmix is not None]      # value mixing: the first leaves its values
         if mixing:
             if len({mixers[i].kv_heads * mixers[i].vdim for i in mixing}) > 1:
@@ -582,7 +704,7 @@ class MixedDecoder(SlotModel):
                             expand_rows=self.expand_rows if self._exp[0] else 0,
                             vocab=V, vocab_p=Vp, eps=cfg.rms_norm_eps, block_size=self.kv_block_size, table_stride=bps,
                             norm_groups=getattr(cfg, "norm_groups", 1), embed_scale=mw.get("embed_scale", 1.0),
-                            alpha=mw.get("alpha", 1.0))
+                            alpha=mw.get("alpha", 1.0), mult=mw.get("mult", 1.0), logit_cap=mw.get("logit_cap", 0.0))
         if bigram:
             mc.bigram_buckets, mc.bigram_prev, mc.bigram_cur = bigram[1:]
         ws = int(lib.chatts_mixdec_workspace(C.byref(mc), arr))
@@ -622,6 +744,11 @@ class MixedDecoder(SlotModel):
             "act_f32": torch.zeros((pairs, over(moes, lambda L: L.moe.ff_p)) if self.exact else (1, 1), **f32),
             "act_planes": torch.zeros((2, pairs, over(moes, lambda L: L.moe.ff_p)) if not self.exact else (2, 1, 1), **bf),
             "vfirst": torch.zeros((rows, ldv) if mixing else (1, 4), **f32),
+            "streams": torch.zeros((len(order), rows, Wp) if depth else (1, 1, 4), **f32),
+            "sel_u": torch.zeros((rows, over(selects, lambda L: L.sel_k)), **f32), "sel_low": torch.zeros((rows, over(selects, lambda L: L.select.ld_low)), **f32),
+            "sel_delta": torch.zeros((rows, over(selects, lambda L: L.sel_dt_n)), **f32),
+            "sel_u_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, over(selects, lambda L: L.sel_k)), **bf),
+            "sel_dt_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, over(selects, lambda L: L.select.rank)), **bf),
             "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
             "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),
@@ -631,6 +758,7 @@ class MixedDecoder(SlotModel):
         }
         B["pos"], B["step"], B["token"], B["out_tokens"] = B["pos_all"][:1], B["step_all"][:1], B["token_all"][:1], B["out_tokens_all"][0]
         P = _lib.ptr
+        fine, coarse = (self._dev(t) for t in sinusoid_tables(W, Wp, self.max_ctx, mw["sinusoid"], dev)) if mw.get("sinusoid") else (None, None)
         mb = _lib.MixBuffers(embed=embed, head=head, head_t=head_t, final_norm=self._f32(mw["final_norm"], Wp), x=P(B["x"]), y=P(B["y"]), proj=P(B["proj"]),
                              a_f32=P(B["a_f32"]), b_f32=P(B["b_f32"]), a_hi=P(B["a_planes"][0]), a_lo=P(B["a_planes"][1]), b_hi=P(B["b_planes"][0]),
                              b_lo=P(B["b_planes"][1]), q_f32=P(B["q_f32"]), o_lat=P(B["o_lat"]), partial=P(B["partial"]), q_hi=P(B["q_planes"][0]),
@@ -638,10 +766,11 @@ class MixedDecoder(SlotModel):
                              kx_hi=P(B["x_k"][0]), kx_lo=P(B["x_k"][1]), vx_hi=P(B["x_v"][0]), vx_lo=P(B["x_v"][1]), zero=P(B["x_zero"]), rows=P(B["rows"]), spans=P(B["spans"]), table=P(B["kv_table"]),
                              logits=P(B["logits_all"]), workspace=P(B["ws"]), workspace_bytes=ws,
                              bigram=self._mat(bigram[0], None, Wp)[0] if bigram else None, x0=P(B["x0"]) if join else None, mix_stride=rows * Wp, vfirst=P(B["vfirst"]), ld_vfirst=ldv,
-                             **{f"{n}_{h}": P(B[f"{n}_planes"][j]) for n in ("m", "n", "act") for j, h in enumerate(("hi", "lo"))},
+                             pos_fine=fine, pos_coarse=coarse, streams=P(B["streams"]) if depth else None, stream_stride=rows * Wp,
+                             **{f"{n}_{h}": P(B[f"{n}_planes"][j]) for n in ("m", "n", "act", "sel_u", "sel_dt") for j, h in enumerate(("hi", "lo"))},
                              **{n: P(B[n]) for n in ("dq", "dk", "dv", "dg", "dgate", "dbeta", "dchunks", "dout", "prev_token", "h", "m_f32", "n_f32", "gates", "den",
                                                      "moe_ids", "moe_place", "moe_order", "moe_offsets", "moe_tiles", "moe_weight", "moe_kept", "moe_logits", "moe_y",
-                                                     "act_f32")})
+                                                     "act_f32", "sel_u", "sel_low", "sel_delta")})
         h = lib.chatts_mixdec_create(C.byref(mc), arr, runs, C.byref(mb))
         if not h:
             raise _lib.ChattsError(-1, lib.chatts_last_error().decode())

@@ -11,6 +11,7 @@ ARCHITECTURES = {
     None: ("chatts_amd", "ChatTSConfig", "ChatTSForCausalLM"),
     "Fobolix": ("chatts_amd.fobolix", "FobolixConfig", "FobolixForCausalLM"),
     "Medilix": ("chatts_amd.medilix", "MedilixConfig", "MedilixForCausalLM"),
+    "Muvetar": ("chatts_amd.muvetar", "MuvetarConfig", "MuvetarForCausalLM"),
     "Mefurax": ("chatts_amd.mefurax", "MefuraxConfig", "MefuraxForCausalLM"),
 }
 

@@ -1,4 +1,4 @@
-"""Rotary position tables with optional YaRN scaling (constants as parameters)."""
+"""Rotary position tables with optional YaRN scaling, and sinusoidal position vectors (constants as parameters)."""
 import math
 
 import torch
@@ -26,3 +26,17 @@ def rotary_tables(dims, base, n, scaling=None, device=None):
         f, mag = torch.exp(torch.arange(dims // 2, dtype=torch.float64) * (-2.0 / dims * math.log(base))), 1.0
     a = torch.arange(n, dtype=torch.float64)[:, None] * f[None, :]
     return (a.cos() * mag).float().contiguous().to(device), (a.sin() * mag).float().contiguous().to(device)
+
+
+def sinusoid_tables(width, width_p, n, base, device=None):
+    """float32 tables [64, width_p] of positions 0 .. 63 and [n / 64, width_p] of positions 0, 64, 128, ...: columns 2 i and 2 i + 1 hold sine and cosine of
+    position * base^(-2 i / width).  A position's vector is the sum of the angles of one row of each."""
+    f = torch.exp(torch.arange((width + 1) // 2, dtype=torch.float64) * (-2.0 / width * math.log(base)))
+
+    def table(pos):
+        a = torch.tensor(pos, dtype=torch.float64)[:, None] * f[None, :]
+        t = torch.zeros((len(pos), width_p), dtype=torch.float32)
+        pairs = torch.stack([a.sin(), a.cos()], -1).view(len(pos), -1).float()
+        t[:, :pairs.shape[1]] = pairs
+        return t.to(device)
+    return table(list(range(64))), table(list(range(0, max(n, 1), 64)))

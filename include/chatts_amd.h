@@ -56,8 +56,11 @@ const char* chatts_last_error(void);
  *     chatts_mixdec_*; CHATTS_EPI_CLAMPGLU, ChattsLinearArgs.glu_limit / glu_alpha;
  * 12: chatts_post_norm and layers with their norms after the sums; windowed attention with chunks, capped scores, distance slopes, gates per head,
  *     rotation, unit queries and keys, norms over all heads, short convolutions and mixed values; experts without a gate, choice by logits;
- *     CHATTS_EPI_GEGLU. */
-#define CHATTS_ABI_VERSION 12
+ *     CHATTS_EPI_GEGLU;
+ * 13: layers of chatts_mixdec_* with norms before the sublayers only, a factor of what is added and averages over depth (chatts_depth_norm), two mixers side by
+ *     side, chatts_gru_*, chatts_select_*; attention with a logarithmic distance bias; clamped gated experts, choice by scores that stay as they are;
+ *     sinusoidal positions in chatts_embed_pair; chatts_soft_cap. */
+#define CHATTS_ABI_VERSION 13
 int chatts_abi_version(void);
 /* Number of CUs of the current device (grid sizing), or <0. */
 int chatts_device_cus(void);
@@ -889,7 +892,9 @@ int chatts_latent_expanded(const ChattsLatentExpandArgs* args, chatts_stream_t s
 
 /* ---- layers whose mixer and feed-forward read two norms of the same x (pair.hip) ----
  * chatts_embed_pair: x = scale * embed[token] + bigram[(prev * mul_prev + token * mul_cur) mod buckets], the table's last row (number `buckets`)
- * for a sequence's first token; prev: the last token of every slot, kept current (device). */
+ * for a sequence's first token; prev: the last token of every slot, kept current (device).
+ * pos_fine, pos_coarse: columns 2 i and 2 i + 1 (below `width`) get sine and cosine of the position's angle i added, by the addition theorem from rows
+ * position % 64 and position / 64 of the two tables. */
 typedef struct ChattsEmbedPairArgs {
   const int64_t* tokens;     /* [T] */
   const ChattsRow* rows;
@@ -900,6 +905,9 @@ typedef struct ChattsEmbedPairArgs {
   int64_t buckets, mul_prev, mul_cur;
   int64_t* prev;             /* [slots] */
   float *x, *x0;             /* [T, width_p]; x0: a copy, or NULL */
+  int width;                 /* with positions */
+  const float* pos_fine;     /* [64, width_p]: (sin, cos) pairs of positions 0 .. 63, or NULL */
+  const float* pos_coarse;   /* [positions / 64, width_p]: of positions 0, 64, 128, ... */
 } ChattsEmbedPairArgs;
 int chatts_embed_pair(const ChattsEmbedPairArgs* args, chatts_stream_t stream);
 
@@ -959,6 +967,79 @@ typedef struct ChattsPostNormArgs {
 } ChattsPostNormArgs;
 int chatts_post_norm(const ChattsPostNormArgs* args, chatts_stream_t stream);
 
+/* ---- layers with norms before their sublayers only (depth.hip): one launch per row of the stream ----
+ *   s = x + mult (y + sum_j weight[j] ey[place[j]])                          (y NULL: none; ey NULL: no experts)
+ *   depth NULL: x <- s;  otherwise x <- sum_{j < n} depth[j] streams[j] + depth[n] s,  n = n_streams, and s is left in streams[n] (keep)
+ *   out = x / rms(x) * w                                                     (w NULL: no output) */
+typedef struct ChattsDepthNormArgs {
+  float* x;                  /* [T, ldx], updated in place */
+  int t, width, ldx;
+  float mult, eps;
+  const float* y;            /* [T, ldx] */
+  const float* ey;           /* [places, ldx] */
+  const int32_t* place;      /* [T, top], < 0: none */
+  const float* weight;       /* [T, top] */
+  int top;
+  const float* depth;        /* [n_streams + 1] */
+  float* streams;            /* stream j: stream_stride floats further, rows like x */
+  int64_t stream_stride;
+  int n_streams, keep;
+  const float* w;            /* padded with zeros to ldx */
+  ChattsOperand out;
+} ChattsDepthNormArgs;
+int chatts_depth_norm(const ChattsDepthNormArgs* args, chatts_stream_t stream);
+/* x <- cap tanh(x / cap), n values */
+int chatts_soft_cap(float* x, int64_t n, float cap, chatts_stream_t stream);
+
+/* ---- minimal gated recurrence (gru.hip), gates from the current token alone, float32 ----
+ * Blocks z, x, g [width] of a projection (biases included):  s = sigmoid(z),  c = x + 1/2 (x >= 0) or sigmoid(x) (x < 0)
+ *   S <- (1 - s) S + s c;   out = out_scale S silu(g)
+ * State per slot: S [ld_state] (width rounded up to 4).  A row at position 0 starts from zero whatever the slot holds. */
+typedef struct ChattsGruArgs {
+  const float* proj;
+  int ld_proj, off_z, off_x, off_g, width;
+  float out_scale;
+  float* state;              /* [slots, width rounded up to 4] */
+  const ChattsRow* rows;
+  int n_rows;
+  const ChattsSpan* spans;   /* device */
+  int n_spans;
+  ChattsOperand out;
+} ChattsGruArgs;
+int chatts_gru_decode(const ChattsGruArgs* args, chatts_stream_t stream);      /* every row is a segment of one token */
+int chatts_gru_scan(const ChattsGruArgs* args, chatts_stream_t stream);        /* segments of several tokens */
+
+/* ---- selective scan (select.hip), float32 ----
+ * Blocks x, z [inner] of a projection.  u = silu(conv(x) + conv_b), the convolution causal over `taps` tokens per channel;  a second projection of u gives `low` =
+ * [dt: rank | B: state | C: state];  d = softplus(W_dt dt + dt_bias) per channel
+ *   S[c, n] <- exp(d_c A[c, n]) S[c, n] + d_c u_c B_n;   y_c = sum_n S[c, n] C_n + D_c u_c;   out = out_scale y silu(z)
+ * State per slot: S [inner, state4] (state4 = state rounded up to 4) and the convolution's inputs as a ring over positions [taps, conv_ch].  A row at position 0
+ * starts from zero whatever the slot holds. */
+typedef struct ChattsSelectArgs {
+  const float* proj;
+  int ld_proj, off_x, off_z, inner, state, taps, conv_ch;      /* conv_ch: inner rounded up to 4 or more, columns of conv_w, conv_b and the ring */
+  const float *conv_w, *conv_b;      /* [taps, conv_ch], [conv_ch] */
+  const float* low;                  /* [T, ld_low] */
+  int ld_low, off_dt, off_b, off_c, rank;      /* rank padded to a multiple of 8 (zero weights) */
+  const chatts_bf16* w_dt;           /* [inner, rank] */
+  const float* dt_bias;              /* [conv_ch] */
+  const float* a;                    /* [inner, state4]: log2(e) A, zeros beyond `state` */
+  const float* d;                    /* [conv_ch] */
+  float out_scale;
+  float *s, *ring;
+  const ChattsRow* rows;
+  int n_rows;
+  const ChattsSpan* spans;           /* device */
+  int n_spans;                       /* chatts_select_conv: 0 = every row is a segment of one token */
+  ChattsOperand u;                   /* [T, inner]: float32 always, planes for the second projection if it takes them */
+  const float* delta;                /* [T, ld_delta] = W_dt dt: chatts_select_scan */
+  int ld_delta;
+  ChattsOperand out;
+} ChattsSelectArgs;
+int chatts_select_conv(const ChattsSelectArgs* args, chatts_stream_t stream);      /* u, and the ring */
+int chatts_select_decode(const ChattsSelectArgs* args, chatts_stream_t stream);    /* every row is a segment of one token; W_dt dt in the same launch */
+int chatts_select_scan(const ChattsSelectArgs* args, chatts_stream_t stream);      /* segments of several tokens */
+
 /* ---- gated linear recurrences (recur.hip): S <- diag(g_t) S + k_t v_t^T per head, float32 ----
  * CHATTS_RECUR_WKV    g = exp(-exp(W2 tanh(a) + w0)) per key channel;  o = S^T q + (q . (u k)) v with S before the token's own write;
  *                     out = o / rms(o) * norm_w * silu(gate)
@@ -1010,9 +1091,9 @@ int64_t chatts_recur_chunk_floats(int heads, int dim, int n_rows, int n_spans);
  *   unit          queries and keys divided by their root mean square, per head
  *   vfirst        values become (1 - vmix) v + vmix vfirst of the same row; vfirst_write: they are left there as they are instead
  * (taps and norm_whole work on whole rows; they do not combine with per-head norms, rot or unit.)
- * Scores: q . k * scale, then softcap tanh(score / softcap), then minus slopes[h] * distance.
+ * Scores: q . k * scale, then softcap tanh(score / softcap), then minus slopes[h] * distance, minus log_r1[h] ln(1 + log_r2[h] * distance).
  * Position i sees j <= i with i - j < window or j < keep_first (window 0: all); chunk: with i / chunk == j / chunk.
- * sink: one more term exp(0) in the softmax's denominator.  Gate: sigmoid, one per output; gate_heads: one per head. */
+ * sink: one more term exp(0) in the softmax's denominator.  Gate: sigmoid, one per output; gate_heads: one per head.  out_scale: factor of the outputs (0: 1). */
 typedef struct ChattsWindowArgs {
   const float* proj;
   int ld_proj, off_q, off_k, off_v, off_gate;        /* off_gate < 0: no gate */
@@ -1043,6 +1124,8 @@ typedef struct ChattsWindowArgs {
   int n_splits;
   float* partial;                                    /* [T, heads, n_splits, vdim_p + 4] when n_splits > 1 */
   ChattsOperand out;                                 /* [T, heads * vdim] */
+  const float *log_r1, *log_r2;                      /* [heads], both or neither */
+  float out_scale;
 } ChattsWindowArgs;
 int chatts_window_prep(const ChattsWindowArgs* args, chatts_stream_t stream);      /* norms, cache write */
 int chatts_window_attend(const ChattsWindowArgs* args, chatts_stream_t stream);    /* row by row: decoding, short segments, 32-bit runs */
@@ -1053,16 +1136,19 @@ int chatts_window_can_prefill(int dim_p, int vdim_p);
  * Outputs of the router: `experts` feed-forwards, then `identity` outputs that return h.
  * CHATTS_CHOOSE_SOFTMAX  the best softmax + correction; weights: the chosen softmax values over their sum
  * CHATTS_CHOOSE_LOGITS   the best logit + correction (NULL: none); weights: softmax over the chosen logits
- * CHATTS_EXPERT_SWIGLU   W_down (silu(W_gate h) * W_up h);   CHATTS_EXPERT_RELU2   W_down max(W_up h, 0)^2 */
+ * CHATTS_CHOOSE_SCORES   as SOFTMAX; weights: the chosen softmax values as they are, times weight_scale
+ * CHATTS_EXPERT_SWIGLU   W_down (silu(W_gate h) * W_up h);   CHATTS_EXPERT_RELU2   W_down max(W_up h, 0)^2;   CHATTS_EXPERT_CLAMPGLU   the unit of CHATTS_EPI_CLAMPGLU */
 #define CHATTS_CHOOSE_SOFTMAX 0
 #define CHATTS_CHOOSE_LOGITS 1
+#define CHATTS_CHOOSE_SCORES 2
 #define CHATTS_EXPERT_SWIGLU 0
 #define CHATTS_EXPERT_RELU2 1
+#define CHATTS_EXPERT_CLAMPGLU 2
 typedef struct ChattsMoeArgs {
   int experts, identity, top, groups, keep;
   int choose, act_kind;                 /* CHATTS_CHOOSE_*, CHATTS_EXPERT_* */
   int width_p, ff_p;                    /* both % 64 == 0 */
-  const chatts_bf16* gate_up;           /* SWIGLU: [experts][2 ff_p][width_p], gate / up rows interleaved in blocks of 16; RELU2: up [experts][ff_p][width_p] */
+  const chatts_bf16* gate_up;           /* SWIGLU, CLAMPGLU: [experts][2 ff_p][width_p], gate / up rows interleaved in blocks of 16; RELU2: up [experts][ff_p][width_p] */
   const chatts_bf16* down;              /* [experts][width_p][ff_p] */
   const chatts_bf16 *gate_up_t, *down_t;   /* chatts_tile_bf16 copy of every matrix, one after the other, or NULL */
   const float* correction;              /* [experts + identity] */
@@ -1075,6 +1161,8 @@ typedef struct ChattsMoeArgs {
   float *weight, *kept;                 /* [T, top], [T] (weight of the identity outputs) */
   ChattsOperand act;                    /* [T * top, ff_p] */
   float* y;                             /* [T * top, width_p] */
+  float weight_scale;                   /* CHOOSE_SCORES */
+  float glu_limit, glu_alpha;           /* EXPERT_CLAMPGLU */
 } ChattsMoeArgs;
 int chatts_moe_route(const ChattsMoeArgs* args, chatts_stream_t stream);
 int chatts_moe_experts(const ChattsMoeArgs* args, chatts_stream_t stream);
@@ -1085,6 +1173,8 @@ int chatts_moe_tiles(int rows, int top, int experts);
 #define CHATTS_MIX_DELTA 2
 #define CHATTS_MIX_RECUR 3
 #define CHATTS_MIX_WINDOW 4
+#define CHATTS_MIX_GRU 5
+#define CHATTS_MIX_SELECT 6
 #define CHATTS_FF_NONE 0
 #define CHATTS_FF_RELU2 1
 #define CHATTS_FF_CLAMPGLU 2
@@ -1118,7 +1208,16 @@ typedef struct ChattsMixLayer {
   ChattsMoeArgs moe;
   int post;                                          /* norms after the sums: x <- norm1(alpha x + mixer(x)), x <- norm2(alpha x + ff(x)); MIX_WINDOW;
                                                       * FF_GEGLU: up = [2 ff, width_p] interleaved; FF_MOE: up / down: a shared squared-relu expert */
-  const float* in_bias;                              /* [in_n] or NULL (post) */
+  const float* in_bias;                              /* [in_n] or NULL (post, pre) */
+  int pre;                                           /* x += mult mixer(norm1(x)), x += mult ff(norm2(x)); MIX_WINDOW, MIX_GRU, MIX_SELECT; FF_CLAMPGLU, FF_MOE (up /
+                                                      * down: a shared expert with the layer's glu_limit / glu_alpha, up = [2 ff, width_p] interleaved) or nothing */
+  int beside, beside_col;                            /* pre: a second mixer (CHATTS_MIX_*, another kind) of the same input, or 0; its outputs' first column in the input of `out` */
+  const float* depth;                                /* pre: weights of the streams after this layer, [run number + 2], or NULL */
+  ChattsGruArgs gru;
+  ChattsSelectArgs select;
+  const chatts_bf16 *sel_low, *sel_low_t;            /* select: second projection [ld_low, inner padded to 64], W_dt [sel_dt_n, rank] padded to 64 */
+  const chatts_bf16* sel_dt;
+  int sel_k, sel_dt_n;
 } ChattsMixLayer;
 typedef struct ChattsMixRun {      /* one pass through a layer */
   int layer;
@@ -1129,6 +1228,7 @@ typedef struct ChattsMixRun {      /* one pass through a layer */
   float *n_state, *m_state;        /* recur, mlstm */
   void* vcache;                    /* window: value pages (cache: key pages) */
   const chatts_bf16 *join, *join_t;   /* x <- join [x | x0] before it, [width_p, 2 width_p], or NULL */
+  float *gru_state, *sel_state, *sel_ring;   /* gru, select */
 } ChattsMixRun;
 typedef struct ChattsMixConfig {
   int width, width_p, n_layers, n_runs, exact, t_max, max_slots, max_ctx;
@@ -1140,6 +1240,8 @@ typedef struct ChattsMixConfig {
   float embed_scale;
   int64_t bigram_buckets, bigram_prev, bigram_cur;
   float alpha;                     /* layers with norms after the sums: factor of x in them */
+  float mult;                      /* layers with norms before their sublayers only: factor of what they add */
+  float logit_cap;                 /* logits <- cap tanh(logits / cap); 0: none */
 } ChattsMixConfig;
 typedef struct ChattsMixBuffers {
   const chatts_bf16 *embed, *head, *head_t;          /* [vocab, width_p], [vocab_p, width_p] */
@@ -1175,6 +1277,11 @@ typedef struct ChattsMixBuffers {
   size_t workspace_bytes;
   float* vfirst;                                     /* window, mixed values: [t_max, ld_vfirst] */
   int ld_vfirst;
+  const float *pos_fine, *pos_coarse;                /* sinusoidal positions (ChattsEmbedPairArgs) or NULL */
+  float* streams;                                    /* averages over depth: [n_runs][stream_stride], stream 0 the embedding output */
+  int64_t stream_stride;
+  float *sel_u, *sel_low, *sel_delta;                /* select: [t_max, widest sel_k], [t_max, widest ld_low], [t_max, widest sel_dt_n] */
+  chatts_bf16 *sel_u_hi, *sel_u_lo, *sel_dt_hi, *sel_dt_lo;      /* ... planes of u, of dt [t_max, widest rank] */
 } ChattsMixBuffers;
 typedef struct ChattsMixDecoder ChattsMixDecoder;
 ChattsMixDecoder* chatts_mixdec_create(const ChattsMixConfig* c, const ChattsMixLayer* layers, const ChattsMixRun* runs, const ChattsMixBuffers* b);

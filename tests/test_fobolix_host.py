@@ -97,6 +97,8 @@ def test_struct_layouts_match_the_header(tmp_path):
              "ChattsHeadLinearArgs": C.sizeof(_lib.HeadLinearArgs), "ChattsDeltaArgs": C.sizeof(_lib.DeltaArgs), "ChattsLatentArgs": C.sizeof(_lib.LatentArgs),
              "ChattsEmbedPairArgs": C.sizeof(_lib.EmbedPairArgs), "ChattsPairNormArgs": C.sizeof(_lib.PairNormArgs),
              "ChattsTokenShiftArgs": C.sizeof(_lib.TokenShiftArgs), "ChattsRecurArgs": C.sizeof(_lib.RecurArgs),
+             "ChattsPostNormArgs": C.sizeof(_lib.PostNormArgs), "ChattsDepthNormArgs": C.sizeof(_lib.DepthNormArgs), "ChattsGruArgs": C.sizeof(_lib.GruArgs),
+             "ChattsSelectArgs": C.sizeof(_lib.SelectArgs),
              "ChattsWindowArgs": C.sizeof(_lib.WindowArgs), "ChattsMoeArgs": C.sizeof(_lib.MoeArgs),
              "ChattsMixLayer": C.sizeof(_lib.MixLayer), "ChattsMixRun": C.sizeof(_lib.MixRun), "ChattsMixConfig": C.sizeof(_lib.MixConfig),
              "ChattsMixBuffers": C.sizeof(_lib.MixBuffers), "ChattsLinearArgs": C.sizeof(_lib.LinearArgs)}
