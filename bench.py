@@ -558,7 +558,21 @@ def mefurax_config(size, layers, vocab):
     return MefuraxConfig(vocab=vocab, width=W, layers=[kinds[i % 4] for i in range(layers)], norm={"eps": 1e-5}, postln_alpha=2.0, name=f"mefurax-{size}")
 
 
-DESIGNS = {"fobolix": fobolix_config, "medilix": medilix_config, "mefurax": mefurax_config}
+def muvetar_config(size, layers, vocab):
+    """attention beside a selective scan and minimal recurrences in turn; every feed-forward has experts (the chosen ones and the shared one weigh as much
+    as a dense one)"""
+    from chatts_amd.muvetar import MuvetarConfig
+    W, _, inter, heads = DESIGN_SIZES[size]
+    moe = {"kind": "moe", "expert": {"ff": inter // 8, "limit": 7.0}, "router": {"experts": 32, "top": 4, "scale": 1.0}, "shared": {"ff": inter // 2, "limit": 7.0}}
+    both = {"type": "parallel", "mlp": moe,
+            "mixer": {"left": {"heads": heads, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5},
+                      "right": {"inner": 2 * W, "state": 16, "dt_rank": W // 16, "conv": 4}, "left_scale": 0.7, "right_scale": 0.7}}
+    gru = {"type": "mingru", "mixer": {"width": W}, "mlp": moe}
+    return MuvetarConfig(vocab=vocab, width=W, layers=[both if i % 2 == 0 else gru for i in range(layers)], norm={"eps": 1e-5}, residual_mult=0.5, logit_softcap=30.0,
+                         name=f"muvetar-{size}")
+
+
+DESIGNS = {"fobolix": fobolix_config, "medilix": medilix_config, "mefurax": mefurax_config, "muvetar": muvetar_config}
 
 
 def qwen_config(size, layers, vocab):

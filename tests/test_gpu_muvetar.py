@@ -1,0 +1,249 @@
+"""Muvetar through the framework: whole prompts, portions, batches, decoding, reused pages and slots, generation - against the plain reference."""
+import json
+import os
+import subprocess
+
+import numpy as np
+import pytest
+import torch
+
+from chatts_amd.engine import Engine
+from chatts_amd.muvetar import MuvetarConfig, MuvetarForCausalLM
+from chatts_amd.llm import LLM, SamplingParams
+from oracle import muvetar as F
+from tests.muvetar_models import CONFIGS, model
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+DTYPES = ["bfloat16", "float32"]
+# bfloat16: rounding queries, keys, values and probabilities in the reference alone moves a row by up to 3e-3 (odd, plain), 6e-3 (wide); float32: the reference itself
+# run in float32 moves rows of "wide" by 8e-6
+TOL = {("odd", "bfloat16"): 8e-3, ("plain", "bfloat16"): 8e-3, ("wide", "bfloat16"): 1.5e-2, ("wide", "float32"): 3e-5}
+CACHE = {}
+
+
+def load(name, dtype, **kw):
+    cfg, public, sd = model(name, all_experts=dtype == "bfloat16")
+    m = MuvetarForCausalLM(MuvetarConfig.from_dict(public), dtype=dtype, **kw)
+    m.load_weights(sd.items())
+    return m
+
+
+def tokens(name, n, seed=0):
+    return np.random.default_rng(seed).integers(0, CONFIGS[name]["vocab"], n).tolist()
+
+
+def want(name, toks, dtype="float32"):
+    """(a router's close call may go either way in bfloat16: there every expert is chosen)"""
+    key = (name, tuple(toks), dtype)
+    if key not in CACHE:
+        cfg, _, sd = model(name, all_experts=dtype == "bfloat16")
+        CACHE[key] = F.forward(cfg, sd, toks)
+    return CACHE[key]
+
+
+def worst(got, ref):
+    """largest error of a row, relative to the rows' typical spread"""
+    got, ref = got.double().cpu(), ref.double()
+    d = got - ref
+    d = d - d.mean(-1, keepdim=True)
+    return float((d.pow(2).mean(-1).sqrt() / ref.std(-1).mean()).max())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_whole_prompts(name, dtype):
+    m = load(name, dtype, max_ctx=256, max_batch=2)
+    for n in (1, 2, 3, 17, 65, 130):
+        toks = tokens(name, n, n)
+        got = m.step_tokens([(n % 2, toks, list(range(n)))])
+        assert worst(got, want(name, toks, dtype)) < TOL.get((name, dtype), 1e-5), n
+        m.release_slot(n % 2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_token_by_token_and_portions(name, dtype):
+    m = load(name, dtype, max_ctx=256, max_batch=3)
+    toks = tokens(name, 140, 1)
+    ref = want(name, toks, dtype)
+    got = torch.cat([m.step_tokens([(0, [t], [0])]) for t in toks])
+    assert worst(got, ref) < TOL.get((name, dtype), 1e-5)
+    for slot, sizes in ((1, [2]), (2, [64, 2, 24, 2, 3, 1, 5])):
+        out, at, i = [], 0, 0
+        while at < len(toks):
+            n = min(sizes[i % len(sizes)], len(toks) - at)
+            out.append(m.step_tokens([(slot, toks[at:at + n], list(range(n)))]))
+            at, i = at + n, i + 1
+        assert worst(torch.cat(out), ref) < TOL.get((name, dtype), 1e-5), sizes
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_unequal_batches_with_reused_slots_and_pages(name, dtype):
+    """portions of some requests beside single tokens of others; the pool is smaller than the slots, so pages and slots come around again"""
+    lens = [97, 23, 66, 1, 128, 40, 2, 75]
+    reqs = [tokens(name, n, 50 + i) for i, n in enumerate(lens)]
+    m = load(name, dtype, max_ctx=192, max_batch=3, kv_pool_blocks=6, max_prefill_tokens=70)
+    rng = np.random.default_rng(3)
+    free, live, waiting, got = [0, 1, 2], {}, list(range(len(reqs))), {i: [] for i in range(len(reqs))}
+    held = lambda: sum(-(-len(reqs[i]) // 64) for i in live)
+    while waiting or live:
+        while waiting and free and held() + -(-lens[waiting[0]] // 64) <= 6:
+            live[waiting.pop(0)] = [free.pop(), 0]
+        entries, who = [], []
+        for i, (slot, at) in live.items():
+            n = int(min(rng.choice([1, 1, 2, 3, 16, 33, 64]), lens[i] - at))
+            if rng.random() < 0.2 and len(live) > 1:
+                continue                                   # left out of this step
+            entries.append((slot, reqs[i][at:at + n], list(range(n))))
+            who.append((i, n))
+        if not entries:
+            continue
+        out, row = m.step_tokens(entries), 0
+        for i, n in who:
+            got[i].append(out[row:row + n])
+            row += n
+            live[i][1] += n
+            if live[i][1] == lens[i]:
+                slot = live.pop(i)[0]
+                m.release_slot(slot)
+                free.append(slot)
+    for i, r in enumerate(reqs):
+        assert worst(torch.cat(got[i]), want(name, r, dtype)) < TOL.get((name, dtype), 1e-5), i
+    assert m._kv.check()
+
+
+def test_order_of_wanted_places_and_empty_wants():
+    m = load("plain", "float32", max_ctx=128, max_batch=2)
+    toks = tokens("plain", 20)
+    ref = want("plain", toks)
+    assert m.step_tokens([(0, toks[:5], [])]).shape == (0, 96)
+    got = m.step_tokens([(0, toks[5:12], [6, 0, 3])])
+    assert worst(got, ref[[11, 5, 8]]) < 3e-5
+    with pytest.raises(ValueError):
+        m.step_tokens([(0, toks * 10, [])])
+    with pytest.raises(ValueError):
+        m.step_tokens([(1, [96], [])])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_long_decoding(name, dtype):
+    """a short prompt, then many single tokens over several pages"""
+    m = load(name, dtype, max_ctx=448, max_batch=1)
+    toks = tokens(name, 400, 9)
+    out = torch.cat([m.step_tokens([(0, toks[:3], [0, 1, 2])])] + [m.step_tokens([(0, [t], [0])]) for t in toks[3:]])
+    assert worst(out, want(name, toks, dtype)) < TOL.get((name, dtype), 1e-5)
+
+
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_chosen_experts_in_bfloat16(name):
+    """with fewer experts chosen than there are: almost every row agrees, those with a close call of a router (at them or before them) aside"""
+    cfg, public, sd = model(name)
+    m = MuvetarForCausalLM(MuvetarConfig.from_dict(public), dtype="bfloat16", max_ctx=256, max_batch=2)
+    m.load_weights(sd.items())
+    toks = tokens(name, 200, 4)
+    margins = []
+    ref = F.forward(cfg, sd, toks, margins=margins)
+    clear = torch.stack(margins).min(0).values > 0.05
+    for sizes in ([200], [120, 16, 2, 1, 33, 28]):
+        out, at = [], 0
+        for n in sizes:
+            out.append(m.step_tokens([(0, toks[at:at + n], list(range(n)))]))
+            at += n
+        m.release_slot(0)
+        d = torch.cat(out).double().cpu() - ref
+        err = (d - d.mean(-1, keepdim=True)).pow(2).mean(-1).sqrt() / ref.std(-1).mean()
+        assert int(clear.sum()) > 100 and float(err[clear].median()) < 1e-2 and float((err[clear] < 5e-2).double().mean()) > 0.9
+
+
+@pytest.mark.parametrize("max_batch", [1, 3])
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_greedy_generation_llm(name, max_batch, tmp_path):
+    """through the public entry point, from a checkpoint directory; captured decode graphs, more requests than slots"""
+    from safetensors.torch import save_file
+    cfg, public, sd = model(name)
+    (tmp_path / "config.json").write_text(json.dumps(public))
+    save_file(sd, str(tmp_path / "model.safetensors"))
+    llm = LLM(str(tmp_path), max_model_len=256, max_num_seqs=max_batch, dtype="float32")
+    prompts = [tokens(name, n, 70 + n) for n in (5, 40, 1, 66)]
+    outs = llm.generate([{"prompt_token_ids": p} for p in prompts], SamplingParams(max_tokens=12))
+    for p, o in zip(prompts, outs):
+        assert o.outputs[0].token_ids == F.generate(cfg, sd, p, 12)
+    text = " ".join(str(t) for t in prompts[0])
+    assert llm.generate(text, SamplingParams(max_tokens=3))[0].outputs[0].text == " ".join(str(t) for t in outs[0].outputs[0].token_ids[:3])
+
+
+@pytest.mark.parametrize("graph", [True, False])
+def test_engine_scheduler(graph):
+    """requests that arrive while others decode; chunked prefill; a pool smaller than the slots; sampling beside greedy requests"""
+    cfg, public, sd = model("odd")
+    m = load("odd", "float32", max_ctx=192, max_batch=3, kv_pool_blocks=6, use_graph=graph)
+    from chatts_amd.processing import TextProcessor
+    from chatts_amd.tokenizer import TokenIdTokenizer
+    eng = Engine(m, TextProcessor(TokenIdTokenizer()), prefill_chunk_tokens=16)
+    prompts = [tokens("odd", n, 200 + n) for n in (7, 90, 33, 12, 64)]
+    reqs = [eng.add_request(prompts[i], max_tokens=10) for i in range(2)]
+    for _ in range(4):
+        eng.step()
+    reqs += [eng.add_request(prompts[i], max_tokens=10) for i in range(2, 5)]
+    hot = eng.add_request(tokens("odd", 9, 5), max_tokens=10, temperature=1.0, top_k=20, seed=11)
+    eng.run_until_done()
+    for p, r in zip(prompts, reqs):
+        assert r.error is None and r.tokens == F.generate(cfg, sd, p, 10)
+    assert hot.error is None and len(hot.tokens) == 10
+    again = eng.add_request(tokens("odd", 9, 5), max_tokens=10, temperature=1.0, top_k=20, seed=11)
+    bad = eng.add_request([1, 2, 999], max_tokens=4)
+    eng.run_until_done()
+    assert bad.error is not None and again.error is None
+    assert m._kv.check()
+
+
+def test_graph_replays_match_eager_steps():
+    """several replays with eager work in between"""
+    out = []
+    for graph in (True, False):
+        m = load("wide", "bfloat16", max_ctx=128, max_batch=2, use_graph=graph)
+        m._admit(0, tokens("wide", 20, 1), None, None, 30)
+        logits = []
+        for i in range(12):
+            m.batched_step()
+            if i % 4 == 1:
+                torch.cuda.synchronize()
+                logits.append(m.buf["logits_all"][0].clone())
+            if i == 5:
+                m._admit(1, tokens("wide", 9, 2), None, None, 30)
+        out.append((m.buf["out_tokens_all"][:, :7].cpu(), torch.stack(logits).cpu()))
+    assert torch.equal(out[0][0][0], out[1][0][0]) and torch.equal(out[0][1], out[1][1])
+
+
+def test_generate_surface():
+    cfg, public, sd = model("plain")
+    m = load("plain", "float32", max_ctx=128, max_batch=2)
+    ids = torch.tensor([tokens("plain", 6, 1), tokens("plain", 6, 2)])
+    out = m.generate(input_ids=ids, max_new_tokens=5)
+    for b in range(2):
+        assert out[b].tolist() == ids[b].tolist() + F.generate(cfg, sd, ids[b].tolist(), 5)
+
+
+def test_trace_run_program(tmp_path):
+    """bin/trace_run as a child process: steps in, files and `done` lines out"""
+    from safetensors.torch import save_file
+    cfg, public, sd = model("plain")
+    mdir, odir = tmp_path / "m", tmp_path / "o"
+    mdir.mkdir(); odir.mkdir()
+    (mdir / "config.json").write_text(json.dumps(public))
+    save_file(sd, str(mdir / "model.safetensors"))
+    a, b = tokens("plain", 12, 1), tokens("plain", 5, 2)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:7], "want": [6, 1]}, {"id": "b", "tokens": b, "want": []}], "end": ["b"]},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[7:8], "want": []}], "end": []},
+             {"step": 2, "entries": [{"id": "c", "tokens": b, "want": [4]}, {"id": "a", "tokens": a[8:], "want": [3]}], "end": ["a", "c"]}]
+    r = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", str(mdir), "--dtype", "float32", "--out", str(odir), "--max-tokens", "128"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=100)
+    assert r.returncode == 0, r.stderr
+    assert [l for l in r.stdout.splitlines() if l.startswith("done")] == ["done 0", "done 1", "done 2"]
+    get = lambda n: torch.from_numpy(np.fromfile(odir / f"{n}.f32", "<f4").reshape(-1, 96))
+    ra, rb = want("plain", a), want("plain", b)
+    assert not (odir / "1.f32").exists()
+    assert worst(get(0), ra[[6, 1]]) < 3e-5 and worst(get(2), torch.stack([rb[4], ra[11]])) < 3e-5

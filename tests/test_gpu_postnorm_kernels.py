@@ -8,6 +8,7 @@ import torch
 from chatts_amd import _lib
 from chatts_amd.rotary import rotary_tables
 from oracle import mefurax as F
+from oracle import muvetar as M
 from tests.test_gpu_mixed_kernels import DEV, call, gen, operand, rel
 from tests.test_gpu_parallel_kernels import planes_of, rows_of, up
 
@@ -48,7 +49,7 @@ class Attn:
     """paged keys and values and convolution rings of a few slots; the plain formula over whole sequences"""
 
     def __init__(self, H, G, D, E, window=0, chunk=0, keep=0, sink=0, gate=None, f32=False, scale=0.25, softcap=0.0, slopes=False, taps=0, whole=False, heads_norm=False, rot=0,
-                 base=1000.0, unit=False, mix=None, seed=0, slots=3, pages=5):
+                 base=1000.0, unit=False, mix=None, log=False, out_scale=0.0, seed=0, slots=3, pages=5):
         g = gen(seed)
         self.__dict__.update({k: v for k, v in locals().items() if k not in ("self", "g")}, eps=1e-4, Dp=up(D, 32), Ep=up(E, 16))
         self.off, at = {}, 0
@@ -67,9 +68,10 @@ class Attn:
         conv = torch.zeros(max(taps, 1), self.conv_ch)
         for n, t in self.w.items():
             conv[:, self.off[n]:self.off[n] + t.shape[0]] = t.t()
+        self.r1, self.r2 = 2.5 * torch.rand(H, generator=g), 0.02 + 0.6 * torch.rand(H, generator=g)
         padded = lambda t: torch.cat([t, torch.zeros(-t.numel() % 4)]).to(DEV)
         cos, sin = rotary_tables(max(rot, 2), base, pages * 64)
-        self.t = dict(qn=padded(self.qn), kn=padded(self.kn), conv=conv.to(DEV), cos=cos.to(DEV), sin=sin.to(DEV), slopes=torch.tensor(F.slopes(H), device=DEV))
+        self.t = dict(qn=padded(self.qn), kn=padded(self.kn), conv=conv.to(DEV), cos=cos.to(DEV), sin=sin.to(DEV), slopes=torch.tensor(F.slopes(H), device=DEV), r1=self.r1.to(DEV), r2=self.r2.to(DEV))
 
     def inputs(self, T, seed):
         x = torch.zeros(T, self.ld)
@@ -106,11 +108,13 @@ class Attn:
         dist = (torch.arange(T)[:, None] - torch.arange(T)[None, :]).double()
         if self.slopes:
             s = s - torch.tensor(F.slopes(H), dtype=torch.float64)[:, None, None] * dist
+        if self.log:
+            s = s - M.distance_bias(self.r1.double(), self.r2.double(), dist.clamp(min=0))
         if self.sink:
             s = torch.cat([torch.zeros(H, T, 1, dtype=torch.float64), s], -1)
         see = self.sees(T)
         a = torch.softmax(s.masked_fill(~torch.cat([torch.ones(T, self.sink, dtype=torch.bool), see], 1), -math.inf), -1)[:, :, self.sink:]
-        o = torch.einsum("hij,jhe->ihe", a, v[:, head])
+        o = torch.einsum("hij,jhe->ihe", a, v[:, head]) * (self.out_scale or 1.0)
         gate = x[:, self.off["g"]:].double()
         if self.gate == "heads":
             o = o * torch.sigmoid(gate[:, :H])[:, :, None]
@@ -142,7 +146,7 @@ class Attn:
                             vcache=self.vc.data_ptr(), cache_f32=int(self.f32), table=self.table.data_ptr(), table_stride=self.table.shape[1], log_block=6, rows=rows.data_ptr(),
                             n_rows=T, spans=spans.data_ptr(), n_spans=0 if single else len(segs), longest=max(s[1] for s in segs), n_splits=splits, partial=part.data_ptr(),
                             q=_lib.Operand(f32=q.data_ptr() if self.f32 else None, hi=None if self.f32 else q.data_ptr(), lo=None, ld=self.H * self.Dp),
-                            out=operand(out, None, n))
+                            out=operand(out, None, n), log_r1=P["r1"] if self.log else None, log_r2=P["r2"] if self.log else None, out_scale=self.out_scale)
         call("chatts_window_prep", a)
         call("chatts_window_" + form, a)
         if write:
