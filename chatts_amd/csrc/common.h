@@ -185,13 +185,11 @@ __device__ __forceinline__ void store_operand4(const ChattsOperand& o, size_t ro
 // float32 transcendentals on the hardware's exp2 / log2 / rcp (each within ~1 ulp of its own result)
 __device__ __forceinline__ float exp_hw(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896341f); }
 __device__ __forceinline__ float sigmoid_f(float x) { return __builtin_amdgcn_rcpf(1.0f + exp_hw(-x)); }
-// log(1 + e^x): for a small e = e^x through log(1 + e) = 2 atanh(e / (2 + e)), which keeps the relative precision log(1 + e) would lose
-__device__ __forceinline__ float softplus_f(float x) {      // (both forms are computed and selected: no branches in unrolled loops)
-  const float e = exp_hw(fminf(x, 20.f)), large = __builtin_amdgcn_logf(1.0f + e) * 0.69314718055994531f;
-  const float z = e * __builtin_amdgcn_rcpf(2.0f + e), z2 = z * z;
-  const float small = 2.0f * z * (1.0f + z2 * (1.0f / 3 + z2 * (1.0f / 5 + z2 * (1.0f / 7 + z2 * (1.0f / 9 + z2 * (1.0f / 11))))));
-  const float r = e > 0.5f ? large : small;
-  return x > 20.f ? x : r;
+// log(1 + e^x) = max(x, 0) + log(1 + e), e = e^-|x|, through log(1 + e) = 2 atanh(e / (2 + e)), which keeps the relative precision of a small e
+__device__ __forceinline__ float softplus_f(float x) {
+  const float e = exp_hw(-fabsf(x)), z = e * __builtin_amdgcn_rcpf(2.0f + e), z2 = z * z;      // z <= 1 / 3
+  const float q = 1.0f + z2 * (1.0f / 3 + z2 * (1.0f / 5 + z2 * (1.0f / 7 + z2 * (1.0f / 9 + z2 * (1.0f / 11 + z2 * (1.0f / 13))))));
+  return fmaxf(x, 0.0f) + 2.0f * z * q;
 }
 // the gated feed-forward of a (gate, up) pair: silu(g) * u (CHATTS_EPI_SWIGLU, by the caller), with both clamped
 // (CHATTS_EPI_CLAMPGLU): g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1)

@@ -3,7 +3,8 @@
 //   select_conv_kernel    u = silu(short convolution), with the inputs before a segment from a ring per slot
 //   select_ring_kernel    the last convolution inputs of every segment
 //   select_decode_kernel  one token per sequence: the step sizes' projection, the state's update and the read-out in one launch
-//   select_scan_kernel    segments of several tokens: a channel's states lie in LPC neighbouring lanes, SPL in each; tokens in tiles through LDS
+//   select_scan_kernel    segments of several tokens, in tiles through LDS
+// A channel's states lie in LPC neighbouring lanes, SPL in each.
 #include "common.h"
 
 namespace chatts {
@@ -96,6 +97,8 @@ __device__ __forceinline__ void states_load(const float* src, int l, int n4, flo
       const f32x4 x = *reinterpret_cast<const f32x4*>(src + l * SPL + i);
 #pragma unroll
       for (int k = 0; k < 4; ++k) s[i + k] = x[k];
+    } else if constexpr (V == 1) {
+      s[i] = src[l + i];
     } else {
       const float2 x = *reinterpret_cast<const float2*>(src + l * SPL + i);
       s[i] = x.x;
@@ -110,144 +113,307 @@ __device__ __forceinline__ void states_store(float* dst, int l, int n4, const fl
   for (int i = 0; i < SPL; i += V) {
     if (l * SPL + i >= n4) continue;
     if constexpr (V == 4) *reinterpret_cast<f32x4*>(dst + l * SPL + i) = (f32x4){s[i], s[i + 1], s[i + 2], s[i + 3]};
+    else if constexpr (V == 1) dst[l + i] = s[i];
     else *reinterpret_cast<float2*>(dst + l * SPL + i) = make_float2(s[i], s[i + 1]);
   }
 }
 
-// grid (channels / (256 / LPC), rows)
-template <int SPL, int LPC>
+// grid (channels / (256 / LPC), rows / NR): NR sequences share what a workgroup reads of W_dt
+template <int SPL, int LPC, int NR>
 __global__ __launch_bounds__(256) void select_decode_kernel(ChattsSelectArgs p) {
   constexpr int CH = 256 / LPC;
-  const int row = blockIdx.y, l = threadIdx.x & (LPC - 1), c = blockIdx.x * CH + threadIdx.x / LPC, n4 = (p.state + 3) & ~3;
-  const ChattsRow R = p.rows[row];
-  if (R.pos < 0) return;
+  const int row0 = blockIdx.y * NR, l = threadIdx.x & (LPC - 1), c = blockIdx.x * CH + threadIdx.x / LPC, n4 = (p.state + 3) & ~3;
   const bool live = c < p.inner;
   const int cc = live ? c : 0;
-  const float* low = p.low + (size_t)row * p.ld_low;
-  const float u = p.u.f32[(size_t)row * p.u.ld + cc], z = p.proj[(size_t)row * p.ld_proj + p.off_z + cc], bias = p.dt_bias[cc], d = p.d[cc];
-  float a[SPL], B[SPL], Cn[SPL], s[SPL];
+  int pos[NR], row[NR];
+  float* S[NR];
+  float s[NR][SPL], u[NR], z[NR], acc[NR], a[SPL];
+  bool any = false;
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    row[r] = row0 + r < p.n_rows ? row0 + r : p.n_rows - 1;
+    const ChattsRow R = p.rows[row[r]];
+    pos[r] = row0 + r < p.n_rows ? R.pos : -1;
+    any = any || pos[r] >= 0;
+    S[r] = p.s + ((size_t)(pos[r] >= 0 ? R.slot : 0) * p.inner + cc) * n4;
+    acc[r] = 0.f;
+  }
+  if (!any) return;
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    states_load<SPL>(S[r], l, n4, s[r]);
+    u[r] = p.u.f32[(size_t)row[r] * p.u.ld + cc];
+    z[r] = p.proj[(size_t)row[r] * p.ld_proj + p.off_z + cc];
+  }
   states_load<SPL>(p.a + (size_t)cc * n4, l, n4, a);
-  states_load<SPL>(low + p.off_b, l, n4, B);
-  states_load<SPL>(low + p.off_c, l, n4, Cn);
-  float* S = p.s + ((size_t)R.slot * p.inner + cc) * n4;
-  states_load<SPL>(S, l, n4, s);
-  // the step size: the channel's lanes share its row of W_dt
-  float acc = 0.f;
+  const float bias = p.dt_bias[cc], d = p.d[cc];
+  // the step sizes: a channel's lanes share its row of W_dt
   const uint16_t* w = p.w_dt + (size_t)cc * p.rank;
   for (int i = l * 8; i < p.rank; i += LPC * 8) {
     const u32x4 wv = *reinterpret_cast<const u32x4*>(w + i);
-    const f32x4 x0 = *reinterpret_cast<const f32x4*>(low + p.off_dt + i), x1 = *reinterpret_cast<const f32x4*>(low + p.off_dt + i + 4);
-    acc += (bf16_lo(wv[0]) * x0[0] + bf16_hi(wv[0]) * x0[1]) + (bf16_lo(wv[1]) * x0[2] + bf16_hi(wv[1]) * x0[3]);
-    acc += (bf16_lo(wv[2]) * x1[0] + bf16_hi(wv[2]) * x1[1]) + (bf16_lo(wv[3]) * x1[2] + bf16_hi(wv[3]) * x1[3]);
-  }
-  const float dt = softplus_f(lanes_sum<LPC>(acc) + bias), du = dt * u;
-  float y = 0.f;
 #pragma unroll
-  for (int i = 0; i < SPL; ++i) {
-    s[i] = __builtin_amdgcn_exp2f(dt * a[i]) * (R.pos > 0 ? s[i] : 0.f) + du * B[i];
-    y += s[i] * Cn[i];
+    for (int r = 0; r < NR; ++r) {
+      const float* x = p.low + (size_t)row[r] * p.ld_low + p.off_dt + i;
+      const f32x4 x0 = *reinterpret_cast<const f32x4*>(x), x1 = *reinterpret_cast<const f32x4*>(x + 4);
+      acc[r] += (bf16_lo(wv[0]) * x0[0] + bf16_hi(wv[0]) * x0[1]) + (bf16_lo(wv[1]) * x0[2] + bf16_hi(wv[1]) * x0[3]);
+      acc[r] += (bf16_lo(wv[2]) * x1[0] + bf16_hi(wv[2]) * x1[1]) + (bf16_lo(wv[3]) * x1[2] + bf16_hi(wv[3]) * x1[3]);
+    }
   }
-  y = lanes_sum<LPC>(y);
-  if (!live) return;
-  states_store<SPL>(S, l, n4, s);
-  if (l == 0) store_operand(p.out, row, c, (y + d * u) * z * sigmoid_f(z) * p.out_scale);
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    const float* low = p.low + (size_t)row[r] * p.ld_low;
+    float B[SPL], Cn[SPL], y = 0.f;
+    states_load<SPL>(low + p.off_b, l, n4, B);
+    states_load<SPL>(low + p.off_c, l, n4, Cn);
+    const float dt = softplus_f(lanes_sum<LPC>(acc[r]) + bias), du = dt * u[r];
+#pragma unroll
+    for (int i = 0; i < SPL; ++i) {
+      s[r][i] = __builtin_amdgcn_exp2f(dt * a[i]) * (pos[r] > 0 ? s[r][i] : 0.f) + du * B[i];
+      y += s[r][i] * Cn[i];
+    }
+    y = lanes_sum<LPC>(y);
+    if (!live || pos[r] < 0) continue;
+    states_store<SPL>(S[r], l, n4, s[r]);
+    if (l == 0) store_operand(p.out, row[r], c, (y + d * u[r]) * z[r] * sigmoid_f(z[r]) * p.out_scale);
+  }
 }
 
-// grid (channels / (256 / LPC), spans)
-template <int SPL, int LPC>
-__global__ __launch_bounds__(256) void select_scan_kernel(ChattsSelectArgs p) {
-  constexpr int CH = 256 / LPC, TT = 4 * LPC < 32 ? 4 * LPC : 32, NP = SPL * LPC, CQ = CH / 4, KB = TT * NP / 4 > 256 ? TT * NP / 1024 : 1;
-  __shared__ __attribute__((aligned(16))) float sdt[TT][CH], sdu[TT][CH], sy[TT][CH], sb[TT][NP], sc[TT][NP];
+// grid (channels / (256 / LPC), spans), 8 waves.  Waves 0 .. 3 run the recurrence of 64 / LPC channels each and do nothing else; wave 4 + w prepares the next
+// tile for wave w (step sizes as quads of tokens, B and C for everyone) and finishes the previous one (adds the lanes' shares of the read-outs, gates and
+// stores them).  Everything between them lies in LDS twice; one barrier per tile.
+template <int SPL, int LPC, int TT>
+constexpr int select_lds() {      // floats, each twice: step sizes, step sizes times u [channels][TT + 4], shares [4][TT / 4][64][4], B, C [states][TT + 4]
+  return 2 * (2 * (256 / LPC) * (TT + 4) + 256 * TT + 2 * SPL * LPC * (TT + 4));
+}
+template <int SPL, int LPC, int TT>
+__global__ __launch_bounds__(512, TT == 16 ? 4 : 2) void select_scan_kernel(ChattsSelectArgs p) {
+  constexpr int LD = TT + 4, T4 = TT / 4, CW = 64 / LPC, NP = SPL * LPC, NQ = NP / 4, KB = (TT * NQ + 255) / 256, NT = TT * CW > 64 ? TT * CW / 64 : 1;
+  constexpr bool kRows = NQ <= 4;      // B and C: neighbouring lanes take a row's quads (whole lines), or - many states - neighbouring rows (no bank met twice)
+  extern __shared__ __attribute__((aligned(16))) float sm[];
   const ChattsSpan sp = p.spans[blockIdx.y];
   if (sp.t < 1) return;
-  const int tid = threadIdx.x, l = tid & (LPC - 1), ch = tid / LPC, c0 = blockIdx.x * CH, c = c0 + ch, n4 = (p.state + 3) & ~3;
-  const bool live = c < p.inner;
-  const int cc = live ? c : 0;
-  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-  float a[SPL], s[SPL];
-  float* S = p.s + ((size_t)sp.slot * p.inner + cc) * n4;
-  states_load<SPL>(p.a + (size_t)cc * n4, l, n4, a);
+  const int tid = threadIdx.x & 255, lane = tid & 63, role = __builtin_amdgcn_readfirstlane(threadIdx.x >> 8), wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int n4 = (p.state + 3) & ~3, c0 = (blockIdx.x * 4 + wave) * CW, t_all = __builtin_amdgcn_readfirstlane(sp.t), tiles = (t_all + 2 * TT - 1) / (2 * TT) * 2;      // (an empty one at the end of some)
+  constexpr int kStep = 4 * CW * LD, kShare = 256 * TT;      // floats of a buffer
+  float* sdt = sm + wave * CW * LD;                          // + buffer * kStep; step sizes times u: 2 kStep further
+  float* sy = sm + 4 * kStep + wave * 64 * TT;               // + buffer * kShare
+  float* sbc = sm + 4 * kStep + 2 * kShare;                  // [buffer][B, C][NP][LD]
+  auto meet = [&]() __attribute__((always_inline)) {         // (LDS alone: what goes to and from memory stays on its way)
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+  };
+  if (role == 0) {
+    const int l = lane & (LPC - 1), c = c0 + lane / LPC, cc = c < p.inner ? c : 0;
+    float a[SPL], s[SPL];
+    float* S = p.s + ((size_t)sp.slot * p.inner + cc) * n4;
+    states_load<SPL>(p.a + (size_t)cc * n4, l, n4, a);
 #pragma unroll
-  for (int i = 0; i < SPL; ++i) s[i] = 0.f;
-  if (sp.pos0 > 0 && live) states_load<SPL>(S, l, n4, s);
-  // staging: thread = (token, four channels)
-  const int lt = tid / CQ, lc = c0 + (tid - lt * CQ) * 4;
-  const bool stage = tid < TT * CQ && lc < ((p.inner + 3) & ~3);
-  f32x4 bias = zero, dw = zero;
-  if (stage) {
-    bias = *reinterpret_cast<const f32x4*>(p.dt_bias + lc);
-    dw = *reinterpret_cast<const f32x4*>(p.d + lc);
+    for (int i = 0; i < SPL; ++i) s[i] = 0.f;
+    if (sp.pos0 > 0 && c < p.inner) states_load<SPL>(S, l, n4, s);
+    meet();
+    for (int k = 0; k < tiles; ++k) {
+      const int buf = k & 1;
+      const float* rdt = sdt + buf * kStep + (lane / LPC) * LD;
+      const float* rdu = rdt + 2 * kStep;
+      const float* b = sbc + (buf * 2 * NP + l * SPL) * LD;
+      float* y0 = sy + buf * kShare + lane * 4;
+      struct Quad { f32x4 dt, du, B[SPL], C[SPL]; };      // four tokens
+      auto request = [&](int g, Quad& q) __attribute__((always_inline)) {
+        q.dt = *reinterpret_cast<const f32x4*>(rdt + g * 4);
+        q.du = *reinterpret_cast<const f32x4*>(rdu + g * 4);
+#pragma unroll
+        for (int i = 0; i < SPL; ++i) {
+          q.B[i] = *reinterpret_cast<const f32x4*>(b + i * LD + g * 4);
+          q.C[i] = *reinterpret_cast<const f32x4*>(b + (NP + i) * LD + g * 4);
+        }
+      };
+      auto run = [&](int g, const Quad& q) __attribute__((always_inline)) {
+        f32x4 y = {0.f, 0.f, 0.f, 0.f};
+        float e[SPL][4];
+#pragma unroll
+        for (int i = 0; i < SPL; ++i)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) e[i][j] = __builtin_amdgcn_exp2f(q.dt[j] * a[i]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int i = 0; i < SPL; ++i) {
+            s[i] = e[i][j] * s[i] + q.du[j] * q.B[i][j];
+            y[j] += s[i] * q.C[i][j];
+          }
+        *reinterpret_cast<f32x4*>(y0 + g * 256) = y;
+      };
+      if constexpr (SPL <= 4) {      // the next quad travels while one is worked on
+        Quad quad[2];
+        request(0, quad[0]);
+#pragma unroll
+        for (int g = 0; g < T4; ++g) {
+          if (g + 1 < T4) request(g + 1, quad[(g + 1) & 1]);
+          __builtin_amdgcn_sched_barrier(0);
+          run(g, quad[g & 1]);
+          __builtin_amdgcn_sched_barrier(0);
+        }
+      } else {
+#pragma unroll 1
+        for (int g = 0; g < T4; ++g) {
+          Quad quad;
+          request(g, quad);
+          run(g, quad);
+        }
+      }
+      meet();
+    }
+    if (c < p.inner) states_store<SPL>(S, l, n4, s);
+    return;
   }
-  f32x4 dl = zero, un = zero, zn = zero, rb[KB], rc[KB];
-  auto fetch = [&](int t0) __attribute__((always_inline)) {
-    if (stage) {
-      const size_t row = sp.row0 + (t0 + lt < sp.t ? t0 + lt : sp.t - 1);
-      dl = *reinterpret_cast<const f32x4*>(p.delta + row * p.ld_delta + lc);
-      un = *reinterpret_cast<const f32x4*>(p.u.f32 + row * p.u.ld + lc);
-      zn = *reinterpret_cast<const f32x4*>(p.proj + row * p.ld_proj + p.off_z + lc);
+  // lane = (channel oc, tokens NT og ..)
+  const bool mine = TT * CW >= 64 || lane / CW < TT;      // (few channels: not every lane has a token)
+  const int oc = lane & (CW - 1), og = mine ? lane / CW : 0, och = c0 + oc;
+  const bool stage = mine && och < p.inner;
+  const int at = stage ? och : 0;
+  const float bias = p.dt_bias[at], dw = p.d[at];
+  struct Inputs { float d[NT], u[NT], z[NT]; f32x4 b[KB], c[KB]; };      // of a tile; two tiles are on their way
+  Inputs in[2];
+  float out[NT], u[3][NT], z[3][NT];      // u, z: of the tile prepared last, the one before, ...
+#pragma unroll
+  for (int j = 0; j < NT; ++j) {
+    out[j] = 0.f;
+    u[0][j] = u[1][j] = u[2][j] = z[0][j] = z[1][j] = z[2][j] = 0.f;
+  }
+  auto at1 = [](const float* base, uint32_t off) __attribute__((always_inline)) { return *reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + off); };
+  // (no branches: requests stay in flight across them only if no two paths meet.  Beyond the end: the last row)
+  auto fetch = [&](int k, Inputs& x) __attribute__((always_inline)) {
+    const int t0 = k * TT < t_all ? k * TT : t_all - 1, last = t_all - 1 - t0;
+    const size_t row = sp.row0 + t0;
+    const float* d0 = p.delta + row * p.ld_delta;
+    const float* u0 = p.u.f32 + row * p.u.ld;
+    const float* z0 = p.proj + row * p.ld_proj + p.off_z;
+    const float* low = p.low + row * p.ld_low;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      const int own = og * NT + j, t = own < last ? own : last;
+      x.d[j] = at1(d0, (uint32_t)(__mul24(t, p.ld_delta) + at) * 4u);
+      x.u[j] = at1(u0, (uint32_t)(__mul24(t, p.u.ld) + at) * 4u);
+      x.z[j] = at1(z0, (uint32_t)(__mul24(t, p.ld_proj) + at) * 4u);
     }
 #pragma unroll
     for (int e = 0; e < KB; ++e) {
-      const int i = e * 256 + tid, t = i / (NP / 4), n = (i - t * (NP / 4)) * 4;
-      rb[e] = rc[e] = zero;
-      if (i < TT * NP / 4 && n < n4) {
-        const float* low = p.low + (size_t)(sp.row0 + (t0 + t < sp.t ? t0 + t : sp.t - 1)) * p.ld_low;
-        rb[e] = *reinterpret_cast<const f32x4*>(low + p.off_b + n);
-        rc[e] = *reinterpret_cast<const f32x4*>(low + p.off_c + n);
+      const int i = e * 256 + tid, own = kRows ? i / NQ : i % TT, t = own < last ? own : last, n = (kRows ? i % NQ : i / TT) * 4;
+      const float* src = low + (uint32_t)(__mul24(t, p.ld_low) + (n < n4 ? n : 0));
+      x.b[e] = *reinterpret_cast<const f32x4*>(src + p.off_b);
+      x.c[e] = *reinterpret_cast<const f32x4*>(src + p.off_c);
+    }
+  };
+  auto prepare = [&](int k, Inputs& x) __attribute__((always_inline)) {      // tile k from registers to LDS
+    const int buf = k & 1;
+    float dt[NT], du[NT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      u[2][j] = u[1][j];
+      z[2][j] = z[1][j];
+      u[1][j] = u[0][j];
+      z[1][j] = z[0][j];
+      u[0][j] = x.u[j];
+      z[0][j] = x.z[j];
+      const uint32_t keep = stage && k * TT + og * NT + j < t_all ? 0xffffffffu : 0u;      // (beyond the end: the state stays)
+      dt[j] = __uint_as_float(__float_as_uint(softplus_f(x.d[j] + bias)) & keep);
+      du[j] = dt[j] * x.u[j];
+    }
+    float* d = sdt + buf * kStep + oc * LD + og * NT;
+    if (mine) {
+      if constexpr (NT == 4) {
+        *reinterpret_cast<f32x4*>(d) = (f32x4){dt[0], dt[1], dt[2], dt[3]};
+        *reinterpret_cast<f32x4*>(d + 2 * kStep) = (f32x4){du[0], du[1], du[2], du[3]};
+      } else {
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+          d[j] = dt[j];
+          d[2 * kStep + j] = du[j];
+        }
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < KB; ++e) {
+      const int i = e * 256 + tid, t = kRows ? i / NQ : i % TT, n = (kRows ? i % NQ : i / TT) * 4;
+      if (i < TT * NQ) {
+        float* dst = sbc + (buf * 2 * NP + n) * LD + t;
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          dst[q * LD] = n < n4 ? x.b[e][q] : 0.f;
+          dst[(NP + q) * LD] = n < n4 ? x.c[e][q] : 0.f;
+        }
       }
     }
   };
-  fetch(0);
-  for (int t0 = 0; t0 < sp.t; t0 += TT) {
-    const f32x4 u = un, z = zn;
-    if (tid < TT * CQ) {
-      f32x4 dt, du;
+  auto finish = [&](int k, const float (&uk)[NT], const float (&zk)[NT]) __attribute__((always_inline)) {      // shares -> read-outs
+    const float* part = sy + (k & 1) * kShare + ((og * NT >> 2) * 64 + oc * LPC) * 4 + (og * NT & 3);
+    float y[NT];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) {
-        dt[k] = stage && t0 + lt < sp.t ? softplus_f(dl[k] + bias[k]) : 0.f;      // (beyond the end: the state stays)
-        du[k] = dt[k] * u[k];
-      }
-      *reinterpret_cast<f32x4*>(&sdt[lt][lc - c0]) = dt;
-      *reinterpret_cast<f32x4*>(&sdu[lt][lc - c0]) = du;
-    }
+    for (int j = 0; j < NT; ++j) y[j] = 0.f;
+    constexpr int G = LPC < 8 ? LPC : 8;      // shares requested at once
 #pragma unroll
-    for (int e = 0; e < KB; ++e) {
-      const int i = e * 256 + tid, t = i / (NP / 4), n = (i - t * (NP / 4)) * 4;
-      if (i < TT * NP / 4) {
-        *reinterpret_cast<f32x4*>(&sb[t][n]) = rb[e];
-        *reinterpret_cast<f32x4*>(&sc[t][n]) = rc[e];
-      }
-    }
-    __syncthreads();
-    if (t0 + TT < sp.t) fetch(t0 + TT);
-    for (int tb = 0; tb < TT; tb += LPC) {
-      float mine = 0.f;
-#pragma unroll LPC < 16 ? LPC : 16
-      for (int j = 0; j < LPC; ++j) {
-        const float dt = sdt[tb + j][ch], du = sdu[tb + j][ch];
-        float B[SPL], Cn[SPL], y = 0.f;
-        states_load<SPL>(sb[tb + j], l, NP, B);
-        states_load<SPL>(sc[tb + j], l, NP, Cn);
+    for (int i0 = 0; i0 < LPC; i0 += G) {
+      float v[G][NT];
 #pragma unroll
-        for (int i = 0; i < SPL; ++i) {
-          s[i] = __builtin_amdgcn_exp2f(dt * a[i]) * s[i] + du * B[i];
-          y += s[i] * Cn[i];
+      for (int i = 0; i < G; ++i) {      // (in turn, so that neighbouring channels meet different banks)
+        const float* q = part + ((i0 + i + oc) & (LPC - 1)) * 4;
+        if constexpr (NT == 4) {
+          const f32x4 x = *reinterpret_cast<const f32x4*>(q);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[i][j] = x[j];
+        } else {
+#pragma unroll
+          for (int j = 0; j < NT; ++j) v[i][j] = q[j];
         }
-        y = lanes_sum<LPC>(y);
-        mine = l == j ? y : mine;
       }
-      sy[tb + l][ch] = mine;
-    }
-    __syncthreads();
-    if (stage && t0 + lt < sp.t) {
-      const f32x4 y = *reinterpret_cast<const f32x4*>(&sy[lt][lc - c0]);
-      float v[4];
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int k = 0; k < 4; ++k) v[k] = (y[k] + dw[k] * u[k]) * z[k] * sigmoid_f(z[k]) * p.out_scale;
-      store_operand4(p.out, sp.row0 + t0 + lt, lc, v);
+      for (int j = 0; j < NT; ++j) {
+        float t[G];
+#pragma unroll
+        for (int i = 0; i < G; ++i) t[i] = v[i][j];
+#pragma unroll
+        for (int d = G / 2; d > 0; d >>= 1)
+#pragma unroll
+          for (int i = 0; i < d; ++i) t[i] += t[i + d];
+        y[j] += t[0];
+      }
     }
+#pragma unroll
+    for (int j = 0; j < NT; ++j) out[j] = (y[j] + dw * uk[j]) * zk[j] * sigmoid_f(zk[j]) * p.out_scale;
+  };
+  auto emit = [&](int k) __attribute__((always_inline)) {
+    const int left = t_all - k * TT;
+    const size_t row = (size_t)(sp.row0 + k * TT) * p.out.ld;
+    ChattsOperand o = p.out;
+    if (o.f32) o.f32 += row;
+    if (o.hi) o.hi += row;
+    if (o.lo) o.lo += row;
+    if (stage)
+#pragma unroll
+      for (int j = 0; j < NT; ++j)
+        if (left >= TT || og * NT + j < left) store_operand(o, 0, __mul24(og * NT + j, o.ld) + och, out[j]);
+  };
+  fetch(0, in[0]);
+  prepare(0, in[0]);
+  fetch(1, in[1]);
+  fetch(2, in[0]);
+  meet();
+  auto tile = [&](int k, Inputs& x) __attribute__((always_inline)) {      // (read-outs are stored a tile late, ahead of the requests that are waited for next)
+    prepare(k + 1, x);
+    if (k > 1) emit(k - 2);
+    fetch(k + 3, x);
+    if (k > 0) finish(k - 1, u[2], z[2]);
+    meet();
+  };
+  for (int k = 0; k < tiles; k += 2) {
+    tile(k, in[1]);
+    tile(k + 1, in[0]);
   }
-  if (live) states_store<SPL>(S, l, n4, s);
+  emit(tiles - 2);
+  finish(tiles - 1, u[1], z[1]);
+  emit(tiles - 1);
 }
 
 static int check_select(const ChattsSelectArgs* a, const char* who) {
@@ -272,18 +438,43 @@ static int check_select_state(const ChattsSelectArgs* a, const char* who) {
 }
 
 template <int SPL, int LPC>
-static void launch_select(const ChattsSelectArgs* a, bool decode, hipStream_t s) {
+static int launch_select_decode(const ChattsSelectArgs* a, hipStream_t s) {
   const int blocks = (a->inner + 256 / LPC - 1) / (256 / LPC);
-  if (decode) hipLaunchKernelGGL((select_decode_kernel<SPL, LPC>), dim3(blocks, a->n_rows), dim3(256), 0, s, *a);
-  else hipLaunchKernelGGL((select_scan_kernel<SPL, LPC>), dim3(blocks, a->n_spans), dim3(256), 0, s, *a);
+  if (a->n_rows < 4) hipLaunchKernelGGL((select_decode_kernel<SPL, LPC, 1>), dim3(blocks, a->n_rows), dim3(256), 0, s, *a);
+  else hipLaunchKernelGGL((select_decode_kernel<SPL, LPC, 4>), dim3(blocks, (a->n_rows + 3) / 4), dim3(256), 0, s, *a);
+  CHATTS_CHECK_LAUNCH("select_decode");
+  return CHATTS_OK;
 }
-static void launch_select_for(const ChattsSelectArgs* a, bool decode, hipStream_t s) {
-  if (a->state <= 8) launch_select<2, 4>(a, decode, s);
-  else if (a->state <= 16) launch_select<2, 8>(a, decode, s);
-  else if (a->state <= 32) launch_select<2, 16>(a, decode, s);
-  else if (a->state <= 64) launch_select<4, 16>(a, decode, s);
-  else if (a->state <= 128) launch_select<4, 32>(a, decode, s);
-  else launch_select<8, 32>(a, decode, s);
+template <int SPL, int LPC, int TT>
+static int launch_select_scan(const ChattsSelectArgs* a, hipStream_t s) {
+  constexpr size_t lds = select_lds<SPL, LPC, TT>() * sizeof(float);
+  static_assert(lds <= 160 * 1024, "LDS");
+  static bool done = false;
+  if (!done) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&select_scan_kernel<SPL, LPC, TT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    CHATTS_REQUIRE(e == hipSuccess, CHATTS_E_LAUNCH, "select_scan: cannot reserve LDS: %s", hipGetErrorString(e));
+    done = true;
+  }
+  hipLaunchKernelGGL((select_scan_kernel<SPL, LPC, TT>), dim3((a->inner + 256 / LPC - 1) / (256 / LPC), a->n_spans), dim3(512), lds, s, *a);
+  CHATTS_CHECK_LAUNCH("select_scan");
+  return CHATTS_OK;
+}
+static int launch_select_decode_for(const ChattsSelectArgs* a, hipStream_t s) {
+  if (a->state <= 8) return launch_select_decode<2, 4>(a, s);
+  if (a->state <= 16) return launch_select_decode<2, 8>(a, s);
+  if (a->state <= 32) return launch_select_decode<4, 8>(a, s);
+  if (a->state <= 64) return launch_select_decode<8, 8>(a, s);
+  return a->state <= 128 ? launch_select_decode<8, 16>(a, s) : launch_select_decode<8, 32>(a, s);
+}
+// tiles of 32 tokens: one workgroup per CU; of 16: two.  More states a lane where the lanes do not run out
+static int launch_select_scan_for(const ChattsSelectArgs* a, hipStream_t s) {
+  const int64_t wide = (int64_t)((a->inner + 63) / 64) * a->n_spans, groups = (int64_t)((a->inner + 31) / 32) * a->n_spans;
+  const bool many = wide >= device_cus(), alone = groups <= device_cus();
+  if (a->state <= 8) return many ? launch_select_scan<2, 4, 16>(a, s) : (alone ? launch_select_scan<1, 8, 32>(a, s) : launch_select_scan<1, 8, 16>(a, s));
+  if (a->state <= 16) return many ? launch_select_scan<4, 4, 16>(a, s) : (alone ? launch_select_scan<2, 8, 32>(a, s) : launch_select_scan<2, 8, 16>(a, s));
+  if (a->state <= 32) return alone ? launch_select_scan<4, 8, 32>(a, s) : launch_select_scan<4, 8, 16>(a, s);
+  if (a->state <= 64) return launch_select_scan<8, 8, 16>(a, s);
+  return a->state <= 128 ? launch_select_scan<8, 16, 16>(a, s) : launch_select_scan<8, 32, 16>(a, s);
 }
 
 template <int TAPS>
@@ -322,9 +513,7 @@ extern "C" int chatts_select_decode(const ChattsSelectArgs* a, chatts_stream_t s
   if (const int rc = check_select_state(a, "select_decode")) return rc;
   CHATTS_REQUIRE(a->w_dt, CHATTS_E_BADARG, "select_decode: null pointer");
   if (a->n_rows == 0) return CHATTS_OK;
-  launch_select_for(a, true, as_stream(stream));
-  CHATTS_CHECK_LAUNCH("select_decode");
-  return CHATTS_OK;
+  return launch_select_decode_for(a, as_stream(stream));
 }
 
 extern "C" int chatts_select_scan(const ChattsSelectArgs* a, chatts_stream_t stream) {
@@ -332,7 +521,5 @@ extern "C" int chatts_select_scan(const ChattsSelectArgs* a, chatts_stream_t str
   if (const int rc = check_select_state(a, "select_scan")) return rc;
   CHATTS_REQUIRE(a->delta && a->ld_delta >= ((a->inner + 3) & ~3) && a->ld_delta % 4 == 0 && a->spans && a->n_spans >= 0, CHATTS_E_BADARG, "select_scan: step sizes");
   if (a->n_rows == 0 || a->n_spans == 0) return CHATTS_OK;
-  launch_select_for(a, false, as_stream(stream));
-  CHATTS_CHECK_LAUNCH("select_scan");
-  return CHATTS_OK;
+  return launch_select_scan_for(a, as_stream(stream));
 }

@@ -251,6 +251,38 @@ def test_selective_scan_of_unequal_segments(case):
     assert torch.equal(w.s[:2], before[0][:2]) and torch.equal(w.ring[:2], before[1][:2]) and not torch.equal(w.s[2], before[0][2])
 
 
+@pytest.mark.parametrize("case", [dict(C_=8200, N=7, R=8, taps=2), dict(C_=8200, N=13, R=8, taps=3), dict(C_=8300, N=25, R=8, taps=4), dict(C_=4100, N=16, R=16, taps=4)],
+                         ids=lambda c: f"C{c['C_']}-N{c['N']}")
+def test_selective_scan_of_many_channels(case):
+    """the forms for more workgroups than there are CUs, with three sequences"""
+    w = Select(**case)
+    xs = [w.inputs(n, n) for n in (70, 33, 47)]
+    want, cut = [w.plain(x) for x in xs], (40, 1, 16)
+    a = w.run(torch.cat([x[:c] for x, c in zip(xs, cut)]), [(0, 40, 0, 2), (40, 1, 0, 0), (41, 16, 0, 1)])
+    b = w.run(torch.cat([x[c:] for x, c in zip(xs, cut)]), [(0, 30, 40, 2), (30, 32, 1, 0), (62, 31, 16, 1)])
+    assert rel(a, torch.cat([t[:c] for t, c in zip(want, cut)])) < STOL and rel(b, torch.cat([t[c:] for t, c in zip(want, cut)])) < STOL
+    assert rel(w.run(xs[0], [(0, 70, 0, 1)]), want[0]) < STOL
+
+
+@pytest.mark.parametrize("case", SELECTS[:6], ids=lambda c: f"N{c['N']}")
+def test_selective_decoding_of_many_sequences(case):
+    """sequences at different positions in one step (groups of rows share weights), a parked one among them, some from their first token"""
+    w = Select(**case, slots=7)
+    xs = [w.inputs(30, 20 + i) for i in range(7)]
+    want, start = [w.plain(x) for x in xs], [0, 3, 17, 1, 0, 9, 5]
+    for i, n in enumerate(start):
+        if n:
+            w.run(xs[i][:n], [(0, n, 0, i)])
+    for step in range(8):
+        parked = step % 7 if step < 4 else -1
+        rows = [(i, 1, -1 if i == parked else start[i], i) for i in range(7)]
+        got = w.run(torch.cat([xs[i][start[i]:start[i] + 1] for i in range(7)]), rows, single=True)
+        for i in range(7):
+            if i != parked:
+                assert rel(got[i], want[i][start[i]]) < STOL, (step, i)
+                start[i] += 1
+
+
 @pytest.mark.parametrize("kw", [dict(a_mean=-9.0, a_spread=1.0), dict(a_mean=6.0, a_spread=1.0), dict(dt_mean=-12.0), dict(dt_mean=30.0)], ids=lambda k: str(k))
 def test_selective_scan_with_extreme_decays(kw):
     """states that keep everything, states that forget at once, step sizes from 1e-5 to 30"""

@@ -17,8 +17,8 @@ pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 DTYPES = ["bfloat16", "float32"]
 # bfloat16: rounding queries, keys, values and probabilities in the reference alone moves a row by up to 3e-3 (odd, plain), 6e-3 (wide); float32: the reference itself
-# run in float32 moves rows of "wide" by 8e-6
-TOL = {("odd", "bfloat16"): 8e-3, ("plain", "bfloat16"): 8e-3, ("wide", "bfloat16"): 1.5e-2, ("wide", "float32"): 3e-5}
+# run in float32 moves rows by up to 8e-6
+TOL = {("odd", "bfloat16"): 8e-3, ("plain", "bfloat16"): 8e-3, ("wide", "bfloat16"): 1.5e-2}
 CACHE = {}
 
 
@@ -57,7 +57,7 @@ def test_whole_prompts(name, dtype):
     for n in (1, 2, 3, 17, 65, 130):
         toks = tokens(name, n, n)
         got = m.step_tokens([(n % 2, toks, list(range(n)))])
-        assert worst(got, want(name, toks, dtype)) < TOL.get((name, dtype), 1e-5), n
+        assert worst(got, want(name, toks, dtype)) < TOL.get((name, dtype), 3e-5), n
         m.release_slot(n % 2)
 
 
@@ -68,14 +68,14 @@ def test_token_by_token_and_portions(name, dtype):
     toks = tokens(name, 140, 1)
     ref = want(name, toks, dtype)
     got = torch.cat([m.step_tokens([(0, [t], [0])]) for t in toks])
-    assert worst(got, ref) < TOL.get((name, dtype), 1e-5)
+    assert worst(got, ref) < TOL.get((name, dtype), 3e-5)
     for slot, sizes in ((1, [2]), (2, [64, 2, 24, 2, 3, 1, 5])):
         out, at, i = [], 0, 0
         while at < len(toks):
             n = min(sizes[i % len(sizes)], len(toks) - at)
             out.append(m.step_tokens([(slot, toks[at:at + n], list(range(n)))]))
             at, i = at + n, i + 1
-        assert worst(torch.cat(out), ref) < TOL.get((name, dtype), 1e-5), sizes
+        assert worst(torch.cat(out), ref) < TOL.get((name, dtype), 3e-5), sizes
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -110,7 +110,7 @@ def test_unequal_batches_with_reused_slots_and_pages(name, dtype):
                 m.release_slot(slot)
                 free.append(slot)
     for i, r in enumerate(reqs):
-        assert worst(torch.cat(got[i]), want(name, r, dtype)) < TOL.get((name, dtype), 1e-5), i
+        assert worst(torch.cat(got[i]), want(name, r, dtype)) < TOL.get((name, dtype), 3e-5), i
     assert m._kv.check()
 
 
@@ -134,7 +134,7 @@ def test_long_decoding(name, dtype):
     m = load(name, dtype, max_ctx=448, max_batch=1)
     toks = tokens(name, 400, 9)
     out = torch.cat([m.step_tokens([(0, toks[:3], [0, 1, 2])])] + [m.step_tokens([(0, [t], [0])]) for t in toks[3:]])
-    assert worst(out, want(name, toks, dtype)) < TOL.get((name, dtype), 1e-5)
+    assert worst(out, want(name, toks, dtype)) < TOL.get((name, dtype), 3e-5)
 
 
 @pytest.mark.parametrize("name", ["odd", "wide"])
