@@ -203,7 +203,7 @@ class SelectArgs(C.Structure):
                 [("conv_w", c_void_p), ("conv_b", c_void_p), ("low", c_void_p)] + [(n, c_int) for n in ("ld_low", "off_dt", "off_b", "off_c", "rank")] +
                 [("w_dt", c_void_p), ("dt_bias", c_void_p), ("a", c_void_p), ("d", c_void_p), ("out_scale", c_float), ("s", c_void_p), ("ring", c_void_p),
                  ("rows", c_void_p), ("n_rows", c_int), ("spans", c_void_p), ("n_spans", c_int), ("u", Operand), ("delta", c_void_p), ("ld_delta", c_int),
-                 ("out", Operand)])
+                 ("delta_steps", c_int), ("w_dt_f", c_void_p), ("dt_hi", c_void_p), ("dt_lo", c_void_p), ("out", Operand)])
 
 
 class RecurArgs(C.Structure):
@@ -377,6 +377,8 @@ SIGNATURES = {
     "chatts_gru_scan": (c_int, [C.POINTER(GruArgs), c_void_p]),
     "chatts_select_conv": (c_int, [C.POINTER(SelectArgs), c_void_p]),
     "chatts_select_decode": (c_int, [C.POINTER(SelectArgs), c_void_p]),
+    "chatts_select_can_steps": (c_int, [c_int]),
+    "chatts_select_steps": (c_int, [C.POINTER(SelectArgs), c_void_p]),
     "chatts_select_scan": (c_int, [C.POINTER(SelectArgs), c_void_p]),
     "chatts_token_shift": (c_int, [C.POINTER(TokenShiftArgs), c_void_p]),
     "chatts_recur_decode": (c_int, [C.POINTER(RecurArgs), c_void_p]),

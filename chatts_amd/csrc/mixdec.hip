@@ -581,12 +581,17 @@ static int mix_select(const ChattsMixDecoder* d, const ChattsMixLayer& l, const 
   if ((rc = mix_linear(d, in, l.sel_low, l.sel_low_t, t, a.ld_low, l.sel_k, CHATTS_EPI_NONE, f32_out(b.sel_low, a.ld_low), s)) != 0) return rc;
   if (single) return chatts_select_decode(&a, s);
   ChattsOperand dt = f32_out(b.sel_low + a.off_dt, a.ld_low);
+  a.delta = b.sel_delta; a.ld_delta = l.sel_dt_n;
+  if (t >= 96 && a.w_dt_f) {
+    a.delta_steps = 1; a.dt_hi = b.sel_dt_hi; a.dt_lo = b.sel_dt_lo;
+    if ((rc = chatts_select_steps(&a, s)) != 0) return rc;
+    return chatts_select_scan(&a, s);
+  }
   if (mix_planes(d->c, t, a.rank)) {
     if ((rc = chatts_split_bf16x2(dt.f32, t, a.rank, a.ld_low, b.sel_dt_hi, b.sel_dt_lo, a.rank, s)) != 0) return rc;
     dt.f32 = nullptr; dt.hi = b.sel_dt_hi; dt.lo = b.sel_dt_lo; dt.ld = a.rank;
   }
   if ((rc = mix_linear(d, dt, l.sel_dt, nullptr, t, l.sel_dt_n, a.rank, CHATTS_EPI_NONE, f32_out(b.sel_delta, l.sel_dt_n), s)) != 0) return rc;
-  a.delta = b.sel_delta; a.ld_delta = l.sel_dt_n;
   return chatts_select_scan(&a, s);
 }
 

@@ -3,9 +3,12 @@
 //   select_conv_kernel    u = silu(short convolution), with the inputs before a segment from a ring per slot
 //   select_ring_kernel    the last convolution inputs of every segment
 //   select_decode_kernel  one token per sequence: the step sizes' projection, the state's update and the read-out in one launch
+//   select_split_kernel   dt of many rows as bf16 hi + lo matrix fragments (a fragment is 1 KB of consecutive memory: sixteen cache lines a load would cost four
+//                         times as much)
+//   select_steps_kernel   their step sizes: W_dt in registers, the fragments streamed past it, softplus in the epilogue
 //   select_scan_kernel    segments of several tokens, in tiles through LDS
 // A channel's states lie in LPC neighbouring lanes, SPL in each.
-#include "common.h"
+#include "gemm_common.h"
 
 namespace chatts {
 
@@ -178,6 +181,87 @@ __global__ __launch_bounds__(256) void select_decode_kernel(ChattsSelectArgs p) 
   }
 }
 
+// grid (channels / 128, rows / kStepRows), 4 waves of 32 channels each.  rank = 32 KS; a wave keeps its rows of W_dt, the fragments of 16 rows of dt pass through LDS
+// (LDS-DMA, the next ones while these are multiplied); D = W . A^T: a lane holds four neighbouring channels of one row
+constexpr int kStepRows = 128;
+// grid (rows / 16, rank / 128): a thread = 8 K-values of a row
+__global__ __launch_bounds__(256) void select_split_kernel(ChattsSelectArgs p) {
+  const int l = threadIdx.x & 63, kt = blockIdx.y * 4 + (threadIdx.x >> 6), row = blockIdx.x * 16 + (l & 15), nk = p.rank >> 5;
+  if (kt >= nk) return;
+  const float* src = p.low + (size_t)(row < p.n_rows ? row : p.n_rows - 1) * p.ld_low + p.off_dt + kt * 32 + (l >> 4) * 8;
+  const f32x4 a = *reinterpret_cast<const f32x4*>(src), b = *reinterpret_cast<const f32x4*>(src + 4);
+  const float v0[4] = {a[0], a[1], a[2], a[3]}, v1[4] = {b[0], b[1], b[2], b[3]};
+  ChattsOperand o{};
+  o.hi = p.dt_hi; o.lo = p.dt_lo;
+  const int at = l * 8;
+  const size_t block = ((size_t)blockIdx.x * nk + kt) * 512;
+  o.hi += block; o.lo += block;
+  store_operand4(o, 0, at, v0);
+  store_operand4(o, 0, at + 4, v1);
+}
+template <int KS>
+__global__ __launch_bounds__(256, 2) void select_steps_kernel(ChattsSelectArgs p) {
+  constexpr int CT = 2;
+  __shared__ __attribute__((aligned(16))) uint16_t sa[2][2 * KS * 512];      // hi fragments, lo fragments
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), fr = lane & 15, fg = lane >> 4;
+  const int c0 = (blockIdx.x * 4 + wave) * 16 * CT, r0 = blockIdx.y * kStepRows, c4 = (p.inner + 3) & ~3, last = ((p.inner + 63) >> 4 & ~3) - 1;      // (W_dt's last fragment)
+  bf16x8_t w[CT][KS];
+  f32x4 bias[CT], d[CT];
+#pragma unroll
+  for (int t = 0; t < CT; ++t) {
+    const int c = c0 + t * 16 + fg * 4, f = (c0 >> 4) + t < last ? (c0 >> 4) + t : last;
+#pragma unroll
+    for (int k = 0; k < KS; ++k) w[t][k] = *reinterpret_cast<const bf16x8_t*>(p.w_dt_f + ((size_t)f * KS + k) * 512 + lane * 8);
+    d[t] = bias[t] = *reinterpret_cast<const f32x4*>(p.dt_bias + (c < c4 ? c : 0));
+  }
+  const int end = r0 + kStepRows < p.n_rows ? r0 + kStepRows : p.n_rows;
+  auto request = [&](int r, int buf) __attribute__((always_inline)) {      // a wave takes every fourth fragment
+    const size_t at = (size_t)(r >> 4) * KS * 512 + lane * 8;
+#pragma unroll
+    for (int i = 0; i < KS / 2; ++i) {
+      const int f = i * 4 + wave;      // (uniform)
+      const uint16_t* src = (f < KS ? p.dt_hi + f * 512 : p.dt_lo + (f - KS) * 512) + at;
+      __builtin_amdgcn_global_load_lds((gptr_t)src, (lptr_t)(&sa[buf][f * 512]), 16, 0, 0);
+    }
+  };
+  auto store = [&](int r) __attribute__((always_inline)) {
+#pragma unroll
+    for (int t = 0; t < CT; ++t) {
+      const int c = c0 + t * 16 + fg * 4;
+      if (r + fr < end && c < c4) *reinterpret_cast<f32x4*>(p.delta + (size_t)(r + fr) * p.ld_delta + c) = d[t];
+    }
+  };
+  auto meet = []() __attribute__((always_inline)) {
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+  };
+  request(r0, 0);
+  meet();
+  int buf = 0;
+  for (int r = r0; r < end; r += 16, buf ^= 1) {
+    if (r > r0) store(r - 16);      // (behind the barrier that follows they have had a tile's time)
+    if (r + 16 < end) request(r + 16, buf ^ 1);
+#pragma unroll
+    for (int t = 0; t < CT; ++t) d[t] = bias[t];
+    const uint16_t* a = &sa[buf][lane * 8];
+#pragma unroll
+    for (int k = 0; k < KS; ++k) {
+      const bf16x8_t h = *reinterpret_cast<const bf16x8_t*>(a + k * 512), l = *reinterpret_cast<const bf16x8_t*>(a + (KS + k) * 512);
+#pragma unroll
+      for (int t = 0; t < CT; ++t) d[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[t][k], l, d[t], 0, 0, 0);
+#pragma unroll
+      for (int t = 0; t < CT; ++t) d[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[t][k], h, d[t], 0, 0, 0);
+    }
+#pragma unroll
+    for (int t = 0; t < CT; ++t)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) d[t][j] = softplus_f(d[t][j]);
+    meet();
+  }
+  store(r0 + (end - r0 - 1) / 16 * 16);
+}
+
 // grid (channels / (256 / LPC), spans), 8 waves.  Waves 0 .. 3 run the recurrence of 64 / LPC channels each and do nothing else; wave 4 + w prepares the next
 // tile for wave w (step sizes as quads of tokens, B and C for everyone) and finishes the previous one (adds the lanes' shares of the read-outs, gates and
 // stores them).  Everything between them lies in LDS twice; one barrier per tile.
@@ -317,7 +401,7 @@ __global__ __launch_bounds__(512, TT == 16 ? 4 : 2) void select_scan_kernel(Chat
       u[0][j] = x.u[j];
       z[0][j] = x.z[j];
       const uint32_t keep = stage && k * TT + og * NT + j < t_all ? 0xffffffffu : 0u;      // (beyond the end: the state stays)
-      dt[j] = __uint_as_float(__float_as_uint(softplus_f(x.d[j] + bias)) & keep);
+      dt[j] = __uint_as_float(__float_as_uint(p.delta_steps ? x.d[j] : softplus_f(x.d[j] + bias)) & keep);
       du[j] = dt[j] * x.u[j];
     }
     float* d = sdt + buf * kStep + oc * LD + og * NT;
@@ -514,6 +598,31 @@ extern "C" int chatts_select_decode(const ChattsSelectArgs* a, chatts_stream_t s
   CHATTS_REQUIRE(a->w_dt, CHATTS_E_BADARG, "select_decode: null pointer");
   if (a->n_rows == 0) return CHATTS_OK;
   return launch_select_decode_for(a, as_stream(stream));
+}
+
+extern "C" int chatts_select_can_steps(int rank) { return rank > 0 && rank % 64 == 0 && rank <= 384; }
+
+extern "C" int chatts_select_steps(const ChattsSelectArgs* a, chatts_stream_t stream) {
+  if (const int rc = check_select(a, "select_steps")) return rc;
+  CHATTS_REQUIRE(a->low && a->w_dt_f && a->dt_hi && a->dt_lo && a->dt_bias && a->delta && (a->ld_low | a->off_dt) % 4 == 0 && a->off_dt >= 0 && a->off_dt + a->rank <= a->ld_low && chatts_select_can_steps(a->rank) && a->ld_delta >= ((a->inner + 3) & ~3) && a->ld_delta % 4 == 0,
+                 CHATTS_E_SHAPE, "select_steps: step sizes of rank %d (multiples of 64, at most 384)", a->rank);
+  CHATTS_REQUIRE((((uintptr_t)a->low | (uintptr_t)a->w_dt_f | (uintptr_t)a->dt_hi | (uintptr_t)a->dt_lo | (uintptr_t)a->dt_bias | (uintptr_t)a->delta) % 16) == 0, CHATTS_E_SHAPE,
+                 "select_steps: alignment");
+  if (a->n_rows == 0) return CHATTS_OK;
+  hipStream_t s = as_stream(stream);
+  const unsigned rows = (a->n_rows + kStepRows - 1) / kStepRows;
+  const dim3 g((a->inner + 127) / 128, rows), b(256);
+  hipLaunchKernelGGL(select_split_kernel, dim3((a->n_rows + 15) / 16, (a->rank + 127) / 128), b, 0, s, *a);
+  switch (a->rank / 64) {
+    case 1: hipLaunchKernelGGL(select_steps_kernel<2>, g, b, 0, s, *a); break;
+    case 2: hipLaunchKernelGGL(select_steps_kernel<4>, g, b, 0, s, *a); break;
+    case 3: hipLaunchKernelGGL(select_steps_kernel<6>, g, b, 0, s, *a); break;
+    case 4: hipLaunchKernelGGL(select_steps_kernel<8>, g, b, 0, s, *a); break;
+    case 5: hipLaunchKernelGGL(select_steps_kernel<10>, g, b, 0, s, *a); break;
+    default: hipLaunchKernelGGL(select_steps_kernel<12>, g, b, 0, s, *a); break;
+  }
+  CHATTS_CHECK_LAUNCH("select_steps");
+  return CHATTS_OK;
 }
 
 extern "C" int chatts_select_scan(const ChattsSelectArgs* a, chatts_stream_t stream) {

@@ -498,11 +498,14 @@ class MixedDecoder(SlotModel):
         L.sel_low, L.sel_low_t = self._mat(low, tile=True)
         L.sel_dt_n = L.sel_k
         L.sel_dt = self._mat(m.dt, L.sel_dt_n, rank)[0]
+        frags = None
+        if not self.exact and self.lib.chatts_select_can_steps(rank):
+            frags = self._dev(_pad(m.dt.to(torch.bfloat16), L.sel_k, rank).view(L.sel_k // 16, 16, rank // 32, 4, 8).permute(0, 2, 3, 1, 4).contiguous())
         conv, a = torch.zeros((taps, n4), dtype=torch.float32, device=self.device), torch.zeros((n, N4), dtype=torch.float32, device=self.device)
         conv[:, :n] = m.conv.to(torch.float32).t()
         a[:, :N] = (-torch.exp(m.a_log.to(torch.float64)) * math.log2(math.e)).float()
         L.select = _lib.SelectArgs(off_x=off["x"], off_z=off["z"], inner=n, state=N, taps=taps, conv_ch=n4, conv_w=self._dev(conv), conv_b=self._f32(m.conv_bias, n4),
-                                   ld_low=low.shape[0], off_dt=at["dt"], off_b=at["b"], off_c=at["c"], rank=rank, w_dt=L.sel_dt, dt_bias=self._f32(m.dt_bias, n4),
+                                   ld_low=low.shape[0], off_dt=at["dt"], off_b=at["b"], off_c=at["c"], rank=rank, w_dt=L.sel_dt, w_dt_f=frags, dt_bias=self._f32(m.dt_bias, n4),
                                    a=self._dev(a), d=self._f32(m.d, n4), out_scale=scale)
 
     def _mixers(self, L, parts):
@@ -748,7 +751,7 @@ class MixedDecoder(SlotModel):
             "sel_u": torch.zeros((rows, over(selects, lambda L: L.sel_k)), **f32), "sel_low": torch.zeros((rows, over(selects, lambda L: L.select.ld_low)), **f32),
             "sel_delta": torch.zeros((rows, over(selects, lambda L: L.sel_dt_n)), **f32),
             "sel_u_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, over(selects, lambda L: L.sel_k)), **bf),
-            "sel_dt_planes": torch.zeros((2, 1, 1) if self.exact else (2, rows, over(selects, lambda L: L.select.rank)), **bf),
+            "sel_dt_planes": torch.zeros((2, 1, 1) if self.exact else (2, _up(rows, 16), over(selects, lambda L: L.select.rank)), **bf),
             "rows": torch.zeros((rows, 4), dtype=torch.int32, device=dev), "spans": torch.zeros((MB, 5), dtype=torch.int32, device=dev),
             "kv_table": torch.zeros((MB, bps), dtype=torch.int32, device=dev), "ids": torch.zeros(rows, dtype=torch.int64, device=dev),
             "logits_all": torch.zeros((MB, Vp), **f32), "ws": torch.zeros(ws, dtype=torch.uint8, device=dev),

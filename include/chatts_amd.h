@@ -1032,12 +1032,18 @@ typedef struct ChattsSelectArgs {
   const ChattsSpan* spans;           /* device */
   int n_spans;                       /* chatts_select_conv: 0 = every row is a segment of one token */
   ChattsOperand u;                   /* [T, inner]: float32 always, planes for the second projection if it takes them */
-  const float* delta;                /* [T, ld_delta] = W_dt dt: chatts_select_scan */
-  int ld_delta;
+  float* delta;                      /* [T, ld_delta] = W_dt dt (delta_steps: d itself): chatts_select_scan */
+  int ld_delta, delta_steps;
+  /* chatts_select_steps: W_dt and (scratch, rows rounded up to 16) hi and lo planes of dt in matrix fragments: [rows / 16][rank / 32][64][8], place l of a
+   * fragment holds row l % 16, K-values 8 (l / 16) .. + 7; W_dt's rows (inner) rounded up to 64 with zeros */
+  const chatts_bf16* w_dt_f;
+  chatts_bf16 *dt_hi, *dt_lo;
   ChattsOperand out;
 } ChattsSelectArgs;
 int chatts_select_conv(const ChattsSelectArgs* args, chatts_stream_t stream);      /* u, and the ring */
 int chatts_select_decode(const ChattsSelectArgs* args, chatts_stream_t stream);    /* every row is a segment of one token; W_dt dt in the same launch */
+int chatts_select_can_steps(int rank);
+int chatts_select_steps(const ChattsSelectArgs* args, chatts_stream_t stream);     /* many rows: delta = softplus(W_dt dt + dt_bias) on the matrix pipe */
 int chatts_select_scan(const ChattsSelectArgs* args, chatts_stream_t stream);      /* segments of several tokens */
 
 /* ---- gated linear recurrences (recur.hip): S <- diag(g_t) S + k_t v_t^T per head, float32 ----

@@ -210,12 +210,20 @@ class Select:
         low = u @ self.low.t()                       # (a projection of the framework's in the product)
         delta = low[:, :self.rank].contiguous() @ self.wdt.t()
         a.low, a.delta, a.ld_delta = low.data_ptr(), delta.data_ptr(), self.k
+        if planes and not single and self.rank <= 384:                    # the step sizes by the kernel for many rows
+            steps, hp = torch.zeros(T, self.k, device=DEV), torch.zeros(2, up(T, 16), self.rank, dtype=torch.bfloat16, device=DEV)
+            frags = self.wdt.to(torch.bfloat16).view(self.k // 16, 16, self.rank // 32, 4, 8).permute(0, 2, 3, 1, 4).contiguous()
+            a.delta, a.delta_steps, a.w_dt_f, a.dt_hi, a.dt_lo = steps.data_ptr(), 1, frags.data_ptr(), hp[0].data_ptr(), hp[1].data_ptr()
+            call("chatts_select_steps", a)
+            want = F.softplus(delta.double().cpu()[:, :self.C] + self.w["dt.b"].double())
+            assert float((steps.cpu().double()[:, :self.C] / want - 1).abs().max()) < 1e-4
         call("chatts_select_decode" if single else "chatts_select_scan", a)
         return (out[0].float() + out[1].float() if planes else out)[:, :self.C].cpu()
 
 
 SELECTS = [dict(C_=50, N=5, R=7, taps=5), dict(C_=91, N=19, R=70, taps=1), dict(C_=128, N=1, R=8, taps=2), dict(C_=64, N=16, R=16, taps=4), dict(C_=200, N=32, R=130, taps=3),
-           dict(C_=70, N=40, R=30, taps=4), dict(C_=33, N=128, R=3, taps=9), dict(C_=20, N=200, R=12, taps=4), dict(C_=1100, N=8, R=64, taps=4, scale=0.3)]
+           dict(C_=70, N=40, R=30, taps=4), dict(C_=33, N=128, R=3, taps=9), dict(C_=20, N=200, R=12, taps=4), dict(C_=1100, N=8, R=64, taps=4, scale=0.3),
+           dict(C_=300, N=12, R=256, taps=4), dict(C_=130, N=16, R=320, taps=4), dict(C_=70, N=4, R=500, taps=4)]
 STOL = 1e-5
 
 
